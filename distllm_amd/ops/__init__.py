@@ -2,7 +2,7 @@
 reference on CPU.
 
 Policy (required by the build rules): on a GPU tensor the HIP extension
-is the ONLY path — if `_hip_ops` failed to import, GPU calls raise
+is the ONLY path — if its module failed to import, GPU calls raise
 immediately instead of silently falling back to eager PyTorch. CPU
 tensors use distllm_amd.ops.torch_ref (fp32), which also serves as the
 numerics ground truth in tests.
@@ -15,26 +15,16 @@ import math
 import torch
 
 from . import torch_ref
+from .native import Native
 
-_HIP_ERR: Exception | None = None
-try:
-    from . import _hip_ops  # type: ignore
-
-    HAVE_HIP = True
-except Exception as e:  # pragma: no cover - import-time environment issue
-    _hip_ops = None  # type: ignore
-    HAVE_HIP = False
-    _HIP_ERR = e
+# One namespace over the built extension modules (native.py).
+_hip_ops = Native()
+HAVE_HIP = not _hip_ops.errors
+_HIP_ERR: Exception | None = next(iter(_hip_ops.errors.values()), None)
 
 
-def _require_hip():
-    if not HAVE_HIP:
-        raise RuntimeError(
-            "distllm_amd HIP extension (_hip_ops) is not built but a GPU "
-            "tensor reached the ops layer. Build with "
-            "`python setup.py build_ext --inplace` (PYTORCH_ROCM_ARCH="
-            f"gfx950). Import error: {_HIP_ERR!r}"
-        )
+def _require_hip(name: str = "_hip_ops"):
+    _hip_ops.require(name)
 
 
 # Activation codes shared with csrc/gemm.hip
@@ -124,7 +114,7 @@ def gemm(A, B, bias=None, act=ACT_NONE):
     """C = A @ B^T via the hand-written MFMA kernel (GPU, padded shapes)
     or fp32 reference (CPU)."""
     if A.is_cuda:
-        _require_hip()
+        _require_hip("_hip_gemm")
         return _hip_ops.gemm_bf16(A, B, bias, act)
     return torch_ref.gemm(A, B, bias, act)
 
@@ -206,8 +196,10 @@ def linear(x, weight, bias=None, act=ACT_NONE):
     M, K = x2.shape
     N = weight.shape[0]
     if x.is_cuda:
-        _require_hip()
+        _require_hip("_hip_gemm")
         mode = os.environ.get("DISTLLM_GEMM", "auto")
+        if x2.dtype == torch.float32:  # true 32-bit products
+            mode = "blaslt"
         if (mode != "blaslt" and act == ACT_NONE and M <= 256
                 and N % 64 == 0 and K % 64 == 0 and x2.is_contiguous()):
             if mode == "decode":  # forced in-chain A/B (profiling)
@@ -404,7 +396,7 @@ def gateup_swiglu(x, wgup, bias=None):
     M, K = x2.shape
     I = wgup.shape[0] // 2
     if x.is_cuda:
-        _require_hip()
+        _require_hip("_hip_gemm")
         if M <= 256 and wgup.shape[0] % 128 == 0 and x2.is_contiguous():
             sk = _decode_splitk(M, wgup.shape[0], K)
             if sk > 1:
@@ -416,6 +408,25 @@ def gateup_swiglu(x, wgup, bias=None):
     else:
         out = swiglu(gu[:, :I], gu[:, I:])
     return out.reshape(*orig_shape[:-1], I)
+
+
+def gateup_clamped_glu(x, wgup, limit, alpha, shift):
+    """Clamped gated unit of x @ Wg^T and x @ Wu^T, Wg|Wu packed as wgup
+    [2I, K]: min(g, limit) * sigmoid(alpha * g) * (clamp(u) + shift), all
+    with the clamped g. Decode-sized inputs fuse it into the split-K
+    reduce of ONE GEMM, as gateup_swiglu does."""
+    M, K = x.shape
+    if x.is_cuda:
+        _require_hip("_hip_gemm")
+        _require_hip("_hip_latent")
+        if (M <= 256 and x.dtype == torch.bfloat16 and K % 64 == 0
+                and wgup.shape[0] % 128 == 0):
+            sk = _decode_splitk(M, wgup.shape[0], K)
+            if sk > 1:
+                return _hip_ops.decode_gemm(x, wgup, None, sk, 2, limit,
+                                            alpha, shift)
+        return _hip_ops.clamped_glu(linear(x, wgup), limit, alpha, shift)
+    return torch_ref.clamped_glu(linear(x, wgup), limit, alpha, shift)
 
 
 def quantize_fp8_rows(w: torch.Tensor):
@@ -510,3 +521,89 @@ def cache_put(knew, vnew, kcache, vcache, block_table, slot):
         blk = int(block_table[b, pos // BLK])
         kcache[blk, :, pos % BLK] = knew[b]
         vcache[blk, :, pos % BLK] = vnew[b]
+
+
+# ---- sandwich-norm / latent-attention decoder -----------------------------
+
+def embed_norm(tokens, table, w_next, n, eps):
+    """Start of the residual stream: x = table[token] in fp32 and h =
+    rms(x) * w_next, statistics over the first n columns. -> (h, x)"""
+    if table.is_cuda:
+        _require_hip("_hip_latent")
+        x = torch.empty(tokens.shape[0], table.shape[1],
+                        dtype=torch.float32, device=table.device)
+        h = _hip_ops.sandwich_norm(table, tokens, x, None, w_next, n, eps)
+        return h, x
+    return torch_ref.embed_norm(tokens, table, w_next, n, eps)
+
+
+def post_norm_add(y, x, w_post, w_next, n, eps):
+    """End of a sandwich-normed sublayer: x += rms(y) * w_post (x fp32,
+    in place), returns the next sublayer's input rms(x) * w_next."""
+    if y.is_cuda:
+        _require_hip("_hip_latent")
+        return _hip_ops.sandwich_norm(y, None, x, w_post, w_next, n, eps)
+    return torch_ref.post_norm_add(y, x, w_post, w_next, n, eps)
+
+
+def latent_prep(ab, q_cols, q_rank, rank, wq, wc, eps, cache, block_table,
+                row_seq, ctx):
+    """Norm both down-projections of a latent-attention layer in one
+    launch: the query latent (first q_cols columns of ab) is returned,
+    the key/value latent goes straight to its cache slot (position
+    ctx - 1 of block-table row row_seq; ctx 0 writes nothing). cache
+    None: the layer has no latent of its own."""
+    if ab.is_cuda:
+        _require_hip("_hip_latent")
+        return _hip_ops.latent_prep(ab, q_cols, q_rank, rank, wq, wc, eps,
+                                    cache, block_table, row_seq, ctx)
+    return torch_ref.latent_prep(ab, q_cols, q_rank, rank, wq, wc, eps,
+                                 cache, block_table, row_seq, ctx)
+
+
+def latent_gather(cache, block_table, key_seq, key_pos):
+    """Cached latents of (sequence, position) pairs, packed."""
+    if cache.is_cuda:
+        _require_hip("_hip_latent")
+        return _hip_ops.latent_gather(cache, block_table, key_seq, key_pos)
+    return torch_ref.latent_gather(cache, block_table, key_seq, key_pos)
+
+
+def head_gemm(x, w, out=None):
+    """One product per head: x [M, H, K], w [H, N, K] -> [M, H, N]."""
+    if x.is_cuda and x.dtype == torch.bfloat16:
+        _require_hip("_hip_latent")
+        if out is None:
+            out = x.new_empty(x.shape[0], x.shape[1], w.shape[1])
+        _hip_ops.head_gemm(x.contiguous(), w, out)
+        return out
+    res = torch_ref.head_gemm(x, w)
+    if out is None:
+        return res
+    return out.copy_(res)
+
+
+def latent_attn(q, cache, block_table, row_seq, ctx, window, scale):
+    """Attention of single-token rows over paged latents, queries folded
+    into the latent space: q [M, H, R] -> [M, H, R]. A row sees the last
+    `window` positions of its sequence up to its own (ctx - 1)."""
+    if q.is_cuda:
+        _require_hip("_hip_latent")
+        return _hip_ops.latent_attn(q, cache, block_table, row_seq, ctx,
+                                    window, scale)
+    return torch_ref.latent_attn(q, cache, block_table, row_seq, ctx,
+                                 window, scale)
+
+
+def attn_window(q, kv, out, cu_q, cu_k, block_map, window, scale):
+    """Sliding-window causal attention of packed queries that are the
+    last ones of their packed keys (a prompt portion after its cached
+    part). q [Tq, H, DK], kv [Tk, H*DK + H*DV], out [Tq, H, DV]."""
+    if q.is_cuda:
+        _require_hip("_hip_latent")
+        blk_seq, blk_qb = block_map
+        _hip_ops.attn_window(q, kv, out, cu_q, cu_k, blk_seq, blk_qb,
+                             window, scale)
+        return out
+    return out.copy_(torch_ref.attn_window(q, kv, out.shape[2], cu_q, cu_k,
+                                           window, scale))

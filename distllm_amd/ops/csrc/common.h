@@ -115,3 +115,19 @@ __device__ __forceinline__ float gelu_erf(float x) {
 __device__ __forceinline__ float silu(float x) {
   return x * fast_rcp(1.f + fast_exp(-x));
 }
+// Clamped gated unit (see clamped_glu.hip): the fast form for 16-bit
+// outputs and the form on library functions for 32-bit ones.
+__device__ __forceinline__ float clamped_glu(float gate, float up,
+                                             float limit, float alpha,
+                                             float shift) {
+  const float g = fminf(gate, limit);
+  const float u = fminf(fmaxf(up, -limit), limit);
+  return g * fast_rcp(1.f + fast_exp(-alpha * g)) * (u + shift);
+}
+__device__ __forceinline__ float clamped_glu_exact(float gate, float up,
+                                                   float limit, float alpha,
+                                                   float shift) {
+  const float g = fminf(gate, limit);
+  const float u = fminf(fmaxf(up, -limit), limit);
+  return g / (1.f + expf(-alpha * g)) * (u + shift);
+}

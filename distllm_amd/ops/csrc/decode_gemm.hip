@@ -161,15 +161,16 @@ dg_reduce_kernel(const float* __restrict__ slabs,
   }
 }
 
-// reduce fp32 slabs [SPLITK, MP, 2I] -> bf16 [M, I] with the swiglu
-// fused: out = silu(gate + bg) * (up + bu). Kills the separate swiglu
-// launch and the [M, 2I] bf16 round-trip in the decode layer
-//
+// reduce fp32 slabs [SPLITK, MP, 2I] -> bf16 [M, I] with the gated unit
+// fused, which saves its launch and the [M, 2I] bf16 round-trip in the
+// decode layer. ACT 1: swiglu, silu(gate + bg) * (up + bu); ACT 2: the
+// clamped unit of clamped_glu.hip.
+template <int ACT>
 __global__ void __launch_bounds__(256)
-dg_reduce_swiglu_kernel(const float* __restrict__ slabs,
-                        const unsigned short* __restrict__ bias,
-                        unsigned short* __restrict__ out, int M, int MP,
-                        int N, int splitk) {
+dg_reduce_glu_kernel(const float* __restrict__ slabs,
+                     const unsigned short* __restrict__ bias,
+                     unsigned short* __restrict__ out, int M, int MP, int N,
+                     int splitk, float limit, float alpha, float shift) {
   const int I = N / 2;
   const long total = (long)M * I;
   const long stride = (long)gridDim.x * blockDim.x;
@@ -187,13 +188,15 @@ dg_reduce_swiglu_kernel(const float* __restrict__ slabs,
       g += bf2f(bias[col]);
       u += bf2f(bias[col + I]);
     }
-    out[i] = f2bf(silu(g) * u);
+    out[i] = f2bf(ACT == 1 ? silu(g) * u
+                           : clamped_glu(g, u, limit, alpha, shift));
   }
 }
 
 extern "C" void launch_decode_gemm(const void* X, const void* W,
                                    const void* bias, void* out, void* slabs,
                                    int M, int N, int K, int splitk, int act,
+                                   float limit, float alpha, float shift,
                                    hipStream_t stream) {
   const int MP = M <= 128 ? 128 : 256;
   const int ncb = N / DG_BN;
@@ -209,17 +212,20 @@ extern "C" void launch_decode_gemm(const void* X, const void* W,
   else { if (slab) DG(256, true); else DG(256, false); }
 #undef DG
   if (slab) {
-    const long total = (long)M * (act == 1 ? N / 2 : N);
+    const long total = (long)M * (act != 0 ? N / 2 : N);
     int blocks = (int)min((total / 256) + 1, (long)2048);
-    if (act == 1)
-      hipLaunchKernelGGL(dg_reduce_swiglu_kernel, dim3(blocks), dim3(256),
-                         0, stream, (const float*)slabs,
-                         (const unsigned short*)bias, (unsigned short*)out,
-                         M, MP, N, splitk);
+#define DGR(A)                                                                 \
+  hipLaunchKernelGGL((dg_reduce_glu_kernel<A>), dim3(blocks), dim3(256), 0,    \
+                     stream, (const float*)slabs,                              \
+                     (const unsigned short*)bias, (unsigned short*)out, M, MP, \
+                     N, splitk, limit, alpha, shift)
+    if (act == 1) DGR(1);
+    else if (act == 2) DGR(2);
     else
       hipLaunchKernelGGL(dg_reduce_kernel, dim3(blocks), dim3(256), 0,
                          stream, (const float*)slabs,
                          (const unsigned short*)bias, (unsigned short*)out,
                          M, MP, N, splitk);
+#undef DGR
   }
 }

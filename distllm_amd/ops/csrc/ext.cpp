@@ -4,22 +4,7 @@
 // on GPU if this extension is missing — no silent eager fallback.
 // All kernels are hand-written CDNA4 HIP (see *.hip in this directory);
 // this file only validates tensors and forwards device pointers.
-#include <torch/extension.h>
-
-#include <hip/hip_runtime.h>
-#include <c10/hip/HIPStream.h>
-
-#define CHECK_DEV(x) TORCH_CHECK(x.is_cuda(), #x " must be on GPU")
-#define CHECK_CONT(x) TORCH_CHECK(x.is_contiguous(), #x " must be contiguous")
-#define CHECK_BF16(x) \
-  TORCH_CHECK(x.scalar_type() == at::kBFloat16, #x " must be bf16")
-#define CHECK_F32(x) \
-  TORCH_CHECK(x.scalar_type() == at::kFloat, #x " must be f32")
-#define CHECK_I32(x) TORCH_CHECK(x.scalar_type() == at::kInt, #x " must be i32")
-
-static hipStream_t cur_stream() {
-  return c10::hip::getCurrentHIPStream().stream();
-}
+#include "ext_common.h"
 
 extern "C" {
 void launch_norm_fwd(const void*, const void*, const void*, const void*,
@@ -35,14 +20,6 @@ void launch_last_token_pool(const void*, const int*, float*, int, int, int,
                             bool, bool, hipStream_t);
 void launch_l2_normalize(const float*, float*, int, int, hipStream_t);
 void launch_adjacent_cosine(const float*, float*, int, int, hipStream_t);
-void launch_gemm_bf16(const void*, const void*, const void*, void*, int, int,
-                      int, int, hipStream_t);
-void launch_gemm8_bf16(const void*, const void*, const void*, void*, int, int,
-                       int, int, hipStream_t);
-void launch_gemm16_bf16(const void*, const void*, const void*, void*, int,
-                        int, int, int, hipStream_t);
-void launch_decode_gemm(const void*, const void*, const void*, void*, void*,
-                        int, int, int, int, int, hipStream_t);
 void launch_attn_fwd(const void*, const void*, const void*, const float*,
                      void*, int, int, int, int, int, int, bool, float, long,
                      long, long, long, hipStream_t);
@@ -168,81 +145,6 @@ torch::Tensor adjacent_cosine(torch::Tensor emb) {
   if (N >= 2)
     launch_adjacent_cosine(emb.data_ptr<float>(), out.data_ptr<float>(), N, H,
                            cur_stream());
-  return out;
-}
-
-// ---- GEMM ------------------------------------------------------------------
-torch::Tensor gemm_bf16(torch::Tensor A, torch::Tensor B,
-                        c10::optional<torch::Tensor> bias, int64_t act) {
-  CHECK_DEV(A); CHECK_CONT(A); CHECK_BF16(A);
-  CHECK_DEV(B); CHECK_CONT(B); CHECK_BF16(B);
-  const int M = A.size(0), K = A.size(1), N = B.size(0);
-  TORCH_CHECK(B.size(1) == K, "K mismatch");
-  TORCH_CHECK(M % 128 == 0 && N % 128 == 0 && K % 64 == 0,
-              "gemm_bf16 requires M,N % 128 == 0 and K % 64 == 0");
-  auto C = torch::empty({M, N}, A.options());
-  launch_gemm_bf16(A.data_ptr(), B.data_ptr(),
-                   bias ? bias->data_ptr() : nullptr, C.data_ptr(), M, N, K,
-                   (int)act, cur_stream());
-  return C;
-}
-
-torch::Tensor gemm8_bf16(torch::Tensor A, torch::Tensor B,
-                         c10::optional<torch::Tensor> bias, int64_t act) {
-  CHECK_DEV(A); CHECK_CONT(A); CHECK_BF16(A);
-  CHECK_DEV(B); CHECK_CONT(B); CHECK_BF16(B);
-  const int M = A.size(0), K = A.size(1), N = B.size(0);
-  TORCH_CHECK(B.size(1) == K, "K mismatch");
-  TORCH_CHECK(M % 256 == 0 && N % 256 == 0 && K % 64 == 0,
-              "gemm8 requires M,N % 256 == 0 and K % 64 == 0");
-  auto C = torch::empty({M, N}, A.options());
-  launch_gemm8_bf16(A.data_ptr(), B.data_ptr(),
-                    bias ? bias->data_ptr() : nullptr, C.data_ptr(), M, N, K,
-                    (int)act, cur_stream());
-  return C;
-}
-
-torch::Tensor gemm16_bf16(torch::Tensor A, torch::Tensor B,
-                          c10::optional<torch::Tensor> bias, int64_t act) {
-  CHECK_DEV(A); CHECK_CONT(A); CHECK_BF16(A);
-  CHECK_DEV(B); CHECK_CONT(B); CHECK_BF16(B);
-  const int M = A.size(0), K = A.size(1), N = B.size(0);
-  TORCH_CHECK(B.size(1) == K, "K mismatch");
-  TORCH_CHECK(M % 256 == 0 && N % 256 == 0 && K % 128 == 0,
-              "gemm16 requires M,N % 256 == 0 and K % 128 == 0");
-  auto C = torch::empty({M, N}, A.options());
-  launch_gemm16_bf16(A.data_ptr(), B.data_ptr(),
-                     bias ? bias->data_ptr() : nullptr, C.data_ptr(), M, N,
-                     K, (int)act, cur_stream());
-  return C;
-}
-
-torch::Tensor decode_gemm(torch::Tensor X, torch::Tensor W,
-                          c10::optional<torch::Tensor> bias,
-                          int64_t splitk, int64_t act = 0) {
-  // act 1 = packed swiglu in the reduce: W is [2I, K] (gate rows then
-  // up rows), output is [M, I]; requires splitk > 1.
-  CHECK_DEV(X); CHECK_CONT(X); CHECK_BF16(X);
-  CHECK_DEV(W); CHECK_CONT(W); CHECK_BF16(W);
-  const int M = X.size(0), K = X.size(1), N = W.size(0);
-  TORCH_CHECK(W.size(1) == K, "K mismatch");
-  TORCH_CHECK(M <= 256, "decode_gemm is for M <= 256");
-  TORCH_CHECK(N % 64 == 0, "N % 64");
-  TORCH_CHECK(K % (64 * splitk) == 0, "K % (64*splitk)");
-  TORCH_CHECK(act == 0 || (splitk > 1 && N % 128 == 0),
-              "swiglu fusion needs splitk > 1 and even I");
-  const int MP = M <= 128 ? 128 : 256;
-  auto out = torch::empty({M, act == 1 ? N / 2 : N}, X.options());
-  torch::Tensor slabs;
-  void* slabp = nullptr;
-  if (splitk > 1) {
-    slabs = torch::empty({splitk, (long)MP, (long)N},
-                         X.options().dtype(at::kFloat));
-    slabp = slabs.data_ptr();
-  }
-  launch_decode_gemm(X.data_ptr(), W.data_ptr(),
-                     bias ? bias->data_ptr() : nullptr, out.data_ptr(),
-                     slabp, M, N, K, (int)splitk, (int)act, cur_stream());
   return out;
 }
 
@@ -424,11 +326,6 @@ void cache_put(torch::Tensor knew, torch::Tensor vnew, torch::Tensor kcache,
                    fp8, cur_stream());
 }
 
-// blt_gemm.cpp: hipBLASLt GEMM with fused bias/GELU/swish epilogue.
-torch::Tensor blt_linear(torch::Tensor x, torch::Tensor w,
-                         c10::optional<torch::Tensor> bias, int64_t epi);
-
-
 torch::Tensor ivf_score(torch::Tensor slabs, torch::Tensor lens,
                         torch::Tensor probes, torch::Tensor q) {
   CHECK_DEV(slabs); CHECK_CONT(slabs); CHECK_F32(slabs);
@@ -476,8 +373,6 @@ torch::Tensor gemv_fp8(torch::Tensor x, torch::Tensor wq,
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
-  m.def("blt_linear", &blt_linear,
-        "hipBLASLt linear with fused bias/GELU/swish epilogue");
   m.def("norm_fwd", &norm_fwd, "fused residual+LayerNorm/RMSNorm");
   m.def("bias_gelu", &bias_gelu);
   m.def("swiglu", &swiglu);
@@ -487,11 +382,6 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("last_token_pool", &last_token_pool);
   m.def("l2_normalize", &l2_normalize);
   m.def("adjacent_cosine", &adjacent_cosine);
-  m.def("gemm_bf16", &gemm_bf16);
-  m.def("gemm8_bf16", &gemm8_bf16);
-  m.def("gemm16_bf16", &gemm16_bf16);
-  m.def("decode_gemm", &decode_gemm, py::arg("X"), py::arg("W"),
-        py::arg("bias"), py::arg("splitk"), py::arg("act") = 0);
   m.def("attn_fwd", &attn_fwd);
   m.def("attn_varlen", &attn_varlen);
   m.def("rope_apply", &rope_apply, py::arg("x"), py::arg("cs"),

@@ -1,0 +1,19 @@
+// Shared by the torch binding files: tensor checks and the current stream.
+#pragma once
+
+#include <torch/extension.h>
+
+#include <hip/hip_runtime.h>
+#include <c10/hip/HIPStream.h>
+
+#define CHECK_DEV(x) TORCH_CHECK(x.is_cuda(), #x " must be on GPU")
+#define CHECK_CONT(x) TORCH_CHECK(x.is_contiguous(), #x " must be contiguous")
+#define CHECK_BF16(x) \
+  TORCH_CHECK(x.scalar_type() == at::kBFloat16, #x " must be bf16")
+#define CHECK_F32(x) \
+  TORCH_CHECK(x.scalar_type() == at::kFloat, #x " must be f32")
+#define CHECK_I32(x) TORCH_CHECK(x.scalar_type() == at::kInt, #x " must be i32")
+
+static inline hipStream_t cur_stream() {
+  return c10::hip::getCurrentHIPStream().stream();
+}

@@ -1,0 +1,111 @@
+// Torch bindings of the matrix products: the hand-written MFMA GEMMs and
+// hipBLASLt with a fused epilogue. Every model family needs these, so
+// they form an extension of their own.
+#include "ext_common.h"
+
+extern "C" {
+void launch_gemm_bf16(const void*, const void*, const void*, void*, int, int,
+                      int, int, hipStream_t);
+void launch_gemm8_bf16(const void*, const void*, const void*, void*, int, int,
+                       int, int, hipStream_t);
+void launch_gemm16_bf16(const void*, const void*, const void*, void*, int,
+                        int, int, int, hipStream_t);
+void launch_decode_gemm(const void*, const void*, const void*, void*, void*,
+                        int, int, int, int, int, float, float, float,
+                        hipStream_t);
+}
+
+// ---- GEMM ------------------------------------------------------------------
+torch::Tensor gemm_bf16(torch::Tensor A, torch::Tensor B,
+                        c10::optional<torch::Tensor> bias, int64_t act) {
+  CHECK_DEV(A); CHECK_CONT(A); CHECK_BF16(A);
+  CHECK_DEV(B); CHECK_CONT(B); CHECK_BF16(B);
+  const int M = A.size(0), K = A.size(1), N = B.size(0);
+  TORCH_CHECK(B.size(1) == K, "K mismatch");
+  TORCH_CHECK(M % 128 == 0 && N % 128 == 0 && K % 64 == 0,
+              "gemm_bf16 requires M,N % 128 == 0 and K % 64 == 0");
+  auto C = torch::empty({M, N}, A.options());
+  launch_gemm_bf16(A.data_ptr(), B.data_ptr(),
+                   bias ? bias->data_ptr() : nullptr, C.data_ptr(), M, N, K,
+                   (int)act, cur_stream());
+  return C;
+}
+
+torch::Tensor gemm8_bf16(torch::Tensor A, torch::Tensor B,
+                         c10::optional<torch::Tensor> bias, int64_t act) {
+  CHECK_DEV(A); CHECK_CONT(A); CHECK_BF16(A);
+  CHECK_DEV(B); CHECK_CONT(B); CHECK_BF16(B);
+  const int M = A.size(0), K = A.size(1), N = B.size(0);
+  TORCH_CHECK(B.size(1) == K, "K mismatch");
+  TORCH_CHECK(M % 256 == 0 && N % 256 == 0 && K % 64 == 0,
+              "gemm8 requires M,N % 256 == 0 and K % 64 == 0");
+  auto C = torch::empty({M, N}, A.options());
+  launch_gemm8_bf16(A.data_ptr(), B.data_ptr(),
+                    bias ? bias->data_ptr() : nullptr, C.data_ptr(), M, N, K,
+                    (int)act, cur_stream());
+  return C;
+}
+
+torch::Tensor gemm16_bf16(torch::Tensor A, torch::Tensor B,
+                          c10::optional<torch::Tensor> bias, int64_t act) {
+  CHECK_DEV(A); CHECK_CONT(A); CHECK_BF16(A);
+  CHECK_DEV(B); CHECK_CONT(B); CHECK_BF16(B);
+  const int M = A.size(0), K = A.size(1), N = B.size(0);
+  TORCH_CHECK(B.size(1) == K, "K mismatch");
+  TORCH_CHECK(M % 256 == 0 && N % 256 == 0 && K % 128 == 0,
+              "gemm16 requires M,N % 256 == 0 and K % 128 == 0");
+  auto C = torch::empty({M, N}, A.options());
+  launch_gemm16_bf16(A.data_ptr(), B.data_ptr(),
+                     bias ? bias->data_ptr() : nullptr, C.data_ptr(), M, N,
+                     K, (int)act, cur_stream());
+  return C;
+}
+
+torch::Tensor decode_gemm(torch::Tensor X, torch::Tensor W,
+                          c10::optional<torch::Tensor> bias,
+                          int64_t splitk, int64_t act = 0,
+                          double limit = 0.0, double alpha = 0.0,
+                          double shift = 0.0) {
+  // act != 0 = packed gated unit in the reduce (1 swiglu, 2 clamped with
+  // the given constants): W is [2I, K] (gate rows then up rows), output
+  // is [M, I]; requires splitk > 1.
+  CHECK_DEV(X); CHECK_CONT(X); CHECK_BF16(X);
+  CHECK_DEV(W); CHECK_CONT(W); CHECK_BF16(W);
+  const int M = X.size(0), K = X.size(1), N = W.size(0);
+  TORCH_CHECK(W.size(1) == K, "K mismatch");
+  TORCH_CHECK(M <= 256, "decode_gemm is for M <= 256");
+  TORCH_CHECK(N % 64 == 0, "N % 64");
+  TORCH_CHECK(K % (64 * splitk) == 0, "K % (64*splitk)");
+  TORCH_CHECK(act == 0 || (splitk > 1 && N % 128 == 0),
+              "gated-unit fusion needs splitk > 1 and even I");
+  const int MP = M <= 128 ? 128 : 256;
+  auto out = torch::empty({M, act != 0 ? N / 2 : N}, X.options());
+  torch::Tensor slabs;
+  void* slabp = nullptr;
+  if (splitk > 1) {
+    slabs = torch::empty({splitk, (long)MP, (long)N},
+                         X.options().dtype(at::kFloat));
+    slabp = slabs.data_ptr();
+  }
+  launch_decode_gemm(X.data_ptr(), W.data_ptr(),
+                     bias ? bias->data_ptr() : nullptr, out.data_ptr(),
+                     slabp, M, N, K, (int)splitk, (int)act, (float)limit,
+                     (float)alpha, (float)shift, cur_stream());
+  return out;
+}
+
+// blt_gemm.cpp: hipBLASLt GEMM with fused bias/GELU/swish epilogue.
+torch::Tensor blt_linear(torch::Tensor x, torch::Tensor w,
+                         c10::optional<torch::Tensor> bias, int64_t epi);
+
+PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.def("blt_linear", &blt_linear,
+        "hipBLASLt linear with fused bias/GELU/swish epilogue");
+  m.def("gemm_bf16", &gemm_bf16);
+  m.def("gemm8_bf16", &gemm8_bf16);
+  m.def("gemm16_bf16", &gemm16_bf16);
+  m.def("decode_gemm", &decode_gemm, py::arg("X"), py::arg("W"),
+        py::arg("bias"), py::arg("splitk"), py::arg("act") = 0,
+        py::arg("limit") = 0.0, py::arg("alpha") = 0.0,
+        py::arg("shift") = 0.0);
+}

@@ -1,0 +1,289 @@
+// Attention over a paged cache of low-rank latents.
+//
+// A token's cache entry is one latent vector c of R numbers (rank n padded
+// with zeros to R); keys and values of every head are linear in it,
+// k_h = Uk_h c and v_h = Uv_h c. Folding Uk into the query (q'_h = Uk_h^T
+// q_h) and Uv into the output leaves one shared "head" whose key and value
+// are both c:
+//     s_hj = scale * q'_h . c_j      o'_h = sum_j softmax(s)_hj c_j
+// so a decode step reads R numbers per cached token for all heads.
+//
+// Cache layout: [num_blocks, PBLK, R], block_table [S, max_blocks] int32.
+// Every row of a batch is one token: row_seq[row] is its block-table row,
+// ctx[row] its position + 1 (0: padding row, nothing is read or written).
+// A row sees the last `window` positions up to its own.
+#include "common.h"
+
+#define PBLK 16  // tokens per cache block
+#define LOG2E 1.4426950408889634f
+
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+
+extern __shared__ __attribute__((aligned(16))) char smem[];
+
+__device__ __forceinline__ float to_f(unsigned short v) { return bf2f(v); }
+__device__ __forceinline__ float to_f(float v) { return v; }
+__device__ __forceinline__ void from_f(unsigned short* p, float v) {
+  *p = f2bf(v);
+}
+__device__ __forceinline__ void from_f(float* p, float v) { *p = v; }
+
+// ---- norm of the two down-projections + cache write ----------------------
+// ab [M, QP (+ R)]: wave 0 of a workgroup norms the query latent (first QP
+// columns, true size qn), wave 1 the cached latent (next R columns, true
+// size rn) and writes it to its cache slot. cache == nullptr: the layer
+// reads another layer's cache and has no latent of its own.
+template <typename T>
+__global__ void __launch_bounds__(128)
+latent_prep_kernel(const T* __restrict__ ab, int ld, int QP, int qn, int R,
+                   int rn, const float* __restrict__ wq,
+                   const float* __restrict__ wc, float eps,
+                   T* __restrict__ cq, T* __restrict__ cache,
+                   const int* __restrict__ block_table, int max_blocks,
+                   int num_blocks, const int* __restrict__ row_seq,
+                   const int* __restrict__ ctx) {
+  const int row = blockIdx.x;
+  const int lane = threadIdx.x & 63;
+  const bool latent = threadIdx.x >= 64;
+  const int n = latent ? rn : qn;
+  const int np = latent ? R : QP;
+  const T* src = ab + (long)row * ld + (latent ? QP : 0);
+  const float* w = latent ? wc : wq;
+  T* dst = cq + (long)row * QP;
+  if (latent) {
+    const int pos = ctx[row] - 1;
+    if (pos < 0 || pos / PBLK >= max_blocks) return;
+    const int blk = block_table[(long)row_seq[row] * max_blocks + pos / PBLK];
+    if (blk < 0 || blk >= num_blocks) return;
+    dst = cache + ((long)blk * PBLK + pos % PBLK) * R;
+  }
+  float ss = 0.f;
+  for (int c = lane; c < np; c += 64) {
+    const float v = to_f(src[c]);
+    ss += v * v;
+  }
+  ss = wave_reduce_sum(ss);
+  const float inv = 1.f / sqrtf(ss / n + eps);
+  for (int c = lane; c < np; c += 64)
+    from_f(dst + c, to_f(src[c]) * inv * w[c]);
+}
+
+extern "C" void launch_latent_prep(
+    const void* ab, int M, int ld, int QP, int qn, int R, int rn,
+    const float* wq, const float* wc, float eps, void* cq, void* cache,
+    const int* block_table, int max_blocks, int num_blocks,
+    const int* row_seq, const int* ctx, bool fp32, hipStream_t stream) {
+  const dim3 grid(M), block(cache != nullptr ? 128 : 64);
+#define LP(T)                                                               \
+  hipLaunchKernelGGL((latent_prep_kernel<T>), grid, block, 0, stream,       \
+                     (const T*)ab, ld, QP, qn, R, rn, wq, wc, eps, (T*)cq,  \
+                     (T*)cache, block_table, max_blocks, num_blocks,        \
+                     row_seq, ctx)
+  if (fp32) LP(float);
+  else LP(unsigned short);
+#undef LP
+}
+
+// ---- latents of chosen positions, packed ----------------------------------
+// out[i] = cache entry of position key_pos[i] of block-table row key_seq[i]
+__global__ void __launch_bounds__(256)
+latent_gather_kernel(const i32x4* __restrict__ cache,
+                     const int* __restrict__ block_table, int max_blocks,
+                     int num_blocks, const int* __restrict__ key_seq,
+                     const int* __restrict__ key_pos, i32x4* __restrict__ out,
+                     int T, int vec) {
+  const long total = (long)T * vec;
+  const long stride = (long)gridDim.x * blockDim.x;
+  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
+       i += stride) {
+    const int row = (int)(i / vec), c = (int)(i % vec);
+    const int pos = key_pos[row];
+    i32x4 v = {0, 0, 0, 0};
+    if (pos >= 0 && pos / PBLK < max_blocks) {
+      const int blk =
+          block_table[(long)key_seq[row] * max_blocks + pos / PBLK];
+      if (blk >= 0 && blk < num_blocks)
+        v = cache[((long)blk * PBLK + pos % PBLK) * vec + c];
+    }
+    out[i] = v;
+  }
+}
+
+extern "C" void launch_latent_gather(const void* cache,
+                                     const int* block_table, int max_blocks,
+                                     int num_blocks, const int* key_seq,
+                                     const int* key_pos, void* out, int T,
+                                     int row_bytes, hipStream_t stream) {
+  const int vec = row_bytes / 16;
+  const int blocks = (int)min(((long)T * vec + 255) / 256, (long)4096);
+  hipLaunchKernelGGL(latent_gather_kernel, dim3(blocks), dim3(256), 0, stream,
+                     (const i32x4*)cache, block_table, max_blocks, num_blocks,
+                     key_seq, key_pos, (i32x4*)out, T, vec);
+}
+
+// ---- per-head products -----------------------------------------------------
+// out[m, h, :] = W[h] x[m, h, :], W [H, N, K] bf16, for the few rows of a
+// decode step (weight-streaming bound). A wave owns 16 output columns; the
+// weight fragment is read once and used for MT tiles of 16 rows.
+template <int MT>
+__global__ void __launch_bounds__(256)
+head_gemm_kernel(const unsigned short* __restrict__ x,
+                 const unsigned short* __restrict__ W,
+                 unsigned short* __restrict__ out, int M, int H, int N,
+                 int K) {
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int nb = N / 64;
+  const int head = blockIdx.x / nb;
+  const int n0 = (blockIdx.x % nb) * 64 + wid * 16;
+  const int m0 = blockIdx.y * (16 * MT);
+  const int i16 = lane & 15, g = lane >> 4;
+  const unsigned short* wrow =
+      W + ((long)head * N + n0 + i16) * K + g * 8;
+  const unsigned short* xrow[MT];
+#pragma unroll
+  for (int t = 0; t < MT; ++t) {
+    const int m = min(m0 + t * 16 + i16, M - 1);
+    xrow[t] = x + ((long)m * H + head) * K + g * 8;
+  }
+  f32x4 acc[MT];
+#pragma unroll
+  for (int t = 0; t < MT; ++t) acc[t] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+  for (int k = 0; k < K; k += 32) {
+    const bf16x8 wf = *reinterpret_cast<const bf16x8*>(wrow + k);
+#pragma unroll
+    for (int t = 0; t < MT; ++t) {
+      const bf16x8 xf = *reinterpret_cast<const bf16x8*>(xrow[t] + k);
+      acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, xf, acc[t], 0, 0,
+                                                       0);
+    }
+  }
+#pragma unroll
+  for (int t = 0; t < MT; ++t) {
+    const int m = m0 + t * 16 + i16;
+    if (m < M) {
+      s16x4 o;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[r] = (short)f2bf(acc[t][r]);
+      *reinterpret_cast<s16x4*>(out + ((long)m * H + head) * N + n0 + g * 4) =
+          o;
+    }
+  }
+}
+
+extern "C" void launch_head_gemm(const void* x, const void* W, void* out,
+                                 int M, int H, int N, int K,
+                                 hipStream_t stream) {
+#define HG(MT)                                                            \
+  hipLaunchKernelGGL((head_gemm_kernel<MT>),                              \
+                     dim3(H*(N / 64), (M + 16 * MT - 1) / (16 * MT)),     \
+                     dim3(256), 0, stream, (const unsigned short*)x,      \
+                     (const unsigned short*)W, (unsigned short*)out, M, H, \
+                     N, K)
+  if (M <= 16) HG(1);
+  else if (M <= 32) HG(2);
+  else if (M <= 64) HG(4);
+  else HG(8);
+#undef HG
+}
+
+// ---- attention, one workgroup per (row, head), any rank and type ----------
+// NV: latent columns per thread (R <= 256 * NV).
+template <typename T, int NV>
+__global__ void __launch_bounds__(256)
+latent_attn_rows_kernel(const T* __restrict__ q, const T* __restrict__ cache,
+                        const int* __restrict__ block_table,
+                        const int* __restrict__ row_seq,
+                        const int* __restrict__ ctx, T* __restrict__ out,
+                        int H, int R, int max_blocks, int window,
+                        float scale) {
+  constexpr int V = 16 / sizeof(T);
+  typedef __attribute__((ext_vector_type(V))) T vec;
+  float* q_lds = reinterpret_cast<float*>(smem);  // R
+  float* p_lds = q_lds + R;                       // 256
+  int* off_lds = reinterpret_cast<int*>(p_lds + 256);  // 256 cache rows
+  float* red = reinterpret_cast<float*>(off_lds + 256);  // 8
+  const int row = blockIdx.x / H, head = blockIdx.x % H;
+  const int tid = threadIdx.x, wid = tid >> 6, lane = tid & 63;
+  const int L = min(ctx[row], max_blocks * PBLK);
+  const int lo = L > window ? L - window : 0;
+  const int* bt = block_table + (long)row_seq[row] * max_blocks;
+  const T* qr = q + ((long)row * H + head) * R;
+  for (int c = tid; c < R; c += 256) q_lds[c] = to_f(qr[c]) * scale;
+
+  float m = -INFINITY, l = 0.f, acc[NV];
+#pragma unroll
+  for (int i = 0; i < NV; ++i) acc[i] = 0.f;
+  for (int t0 = lo; t0 < L; t0 += 256) {
+    const int key = t0 + tid;
+    const bool live = key < L;
+    __syncthreads();  // q is staged; the previous tile is consumed
+    float s = -INFINITY;
+    if (live) {
+      const int off = bt[key / PBLK] * PBLK + key % PBLK;
+      off_lds[tid] = off;
+      const T* c = cache + (long)off * R;
+      float dot = 0.f;
+      for (int k = 0; k < R; k += V) {
+        const vec cv = *reinterpret_cast<const vec*>(c + k);
+#pragma unroll
+        for (int i = 0; i < V; ++i) dot += to_f((T)cv[i]) * q_lds[k + i];
+      }
+      s = dot;
+    }
+    const float wmax = wave_reduce_max(s);
+    if (lane == 0) red[wid] = wmax;
+    __syncthreads();
+    const float mn =
+        fmaxf(m, fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])));
+    const float p = live ? expf(s - mn) : 0.f;
+    p_lds[tid] = p;
+    const float wsum = wave_reduce_sum(p);
+    if (lane == 0) red[4 + wid] = wsum;
+    __syncthreads();
+    const float alpha = expf(m - mn);  // 0 on the first tile
+    l = l * alpha + (red[4] + red[5]) + (red[6] + red[7]);
+    m = mn;
+    const int nk = min(256, L - t0);
+#pragma unroll
+    for (int i = 0; i < NV; ++i) {
+      const int c = tid + i * 256;
+      if (c < R) {
+        float a = acc[i] * alpha;
+        for (int j = 0; j < nk; ++j)
+          a += p_lds[j] * to_f(cache[(long)off_lds[j] * R + c]);
+        acc[i] = a;
+      }
+    }
+  }
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+  T* o = out + ((long)row * H + head) * R;
+#pragma unroll
+  for (int i = 0; i < NV; ++i) {
+    const int c = tid + i * 256;
+    if (c < R) from_f(o + c, acc[i] * inv);
+  }
+}
+
+extern "C" void launch_latent_attn_rows(
+    const void* q, const void* cache, const int* block_table,
+    const int* row_seq, const int* ctx, void* out, int M, int H, int R,
+    int max_blocks, int window, float scale, bool fp32, hipStream_t stream) {
+  const int lds = (R + 256 + 256 + 8) * 4;
+#define LA(T, NV)                                                            \
+  hipLaunchKernelGGL((latent_attn_rows_kernel<T, NV>), dim3(M * H),          \
+                     dim3(256), lds, stream, (const T*)q, (const T*)cache,   \
+                     block_table, row_seq, ctx, (T*)out, H, R, max_blocks,   \
+                     window, scale)
+#define LA_N(T)                    \
+  do {                             \
+    if (R <= 256) LA(T, 1);        \
+    else if (R <= 512) LA(T, 2);   \
+    else if (R <= 1024) LA(T, 4);  \
+    else LA(T, 16);                \
+  } while (0)
+  if (fp32) LA_N(float);
+  else LA_N(unsigned short);
+#undef LA_N
+#undef LA
+}

@@ -269,3 +269,102 @@ def paged_attn(q, kcache, vcache, block_table, ctx_len, scale):
         p = torch.softmax(s, dim=-1)
         out[b] = (p.unsqueeze(-1) * v).sum(1).to(q.dtype)
     return out
+
+
+# ---- sandwich-norm / latent-attention decoder -----------------------------
+
+def embed_norm(tokens, table, w_next, n, eps):
+    """x = table[token] (fp32), h = rms(x) over the first n columns."""
+    x = table[tokens.long()].float()
+    ms = x.pow(2).sum(-1, keepdim=True) / n
+    return (x / torch.sqrt(ms + eps) * w_next).to(table.dtype), x
+
+
+def post_norm_add(y, x, w_post, w_next, n, eps):
+    """x += rms(y) * w_post in place; returns h = rms(x) * w_next."""
+    yf = y.float()
+    ms = yf.pow(2).sum(-1, keepdim=True) / n
+    x += yf / torch.sqrt(ms + eps) * w_post
+    ms = x.pow(2).sum(-1, keepdim=True) / n
+    return (x / torch.sqrt(ms + eps) * w_next).to(y.dtype)
+
+
+def _cache_rows(block_table, row_seq, pos, blk):
+    """Flat cache row of position pos[i] of sequence row_seq[i]."""
+    p = pos.long()
+    page = block_table.long()[row_seq.long(), p // blk]
+    return page * blk + p % blk
+
+
+def latent_prep(ab, q_cols, q_rank, rank, wq, wc, eps, cache, block_table,
+                row_seq, ctx):
+    """Norm of the query latent (returned) and of the cached latent
+    (written to the cache at position ctx - 1 of each live row)."""
+
+    def norm(v, n, w):
+        v = v.float()
+        ms = v.pow(2).sum(-1, keepdim=True) / n
+        return (v / torch.sqrt(ms + eps) * w).to(ab.dtype)
+
+    if cache is not None:
+        live = ctx > 0
+        rows = _cache_rows(block_table, row_seq[live], ctx[live] - 1,
+                           cache.shape[1])
+        cache.view(-1, cache.shape[2])[rows] = norm(
+            ab[live, q_cols:], rank, wc)
+    return norm(ab[:, :q_cols], q_rank, wq)
+
+
+def latent_gather(cache, block_table, key_seq, key_pos):
+    rows = _cache_rows(block_table, key_seq, key_pos, cache.shape[1])
+    return cache.view(-1, cache.shape[2])[rows]
+
+
+def head_gemm(x, w):
+    """[M, H, K] x [H, N, K] -> [M, H, N]."""
+    out = torch.bmm(x.float().transpose(0, 1),
+                    w.float().transpose(1, 2).contiguous())
+    return out.transpose(0, 1).to(x.dtype).contiguous()
+
+
+def latent_attn(q, cache, block_table, row_seq, ctx, window, scale):
+    """q [M, H, R] against the cached latents of each row's sequence; key
+    and value are both the latent."""
+    out = torch.zeros_like(q)
+    for r in range(q.shape[0]):
+        L = int(ctx[r])
+        if L <= 0:
+            continue
+        pos = torch.arange(max(0, L - window), L)
+        c = latent_gather(cache, block_table,
+                          row_seq[r].expand(len(pos)), pos).float()
+        p = torch.softmax(q[r].float() @ c.t() * scale, dim=-1)
+        out[r] = (p @ c).to(q.dtype)
+    return out
+
+
+def attn_window(q, kv, dv, cu_q, cu_k, window, scale):
+    """Packed continuation attention: the queries of a sequence are the
+    last ones of its keys. q [Tq, H, DK]; kv [Tk, H*DK + H*DV]."""
+    Tq, H, dk = q.shape
+    k = kv[:, : H * dk].view(-1, H, dk).float()
+    v = kv[:, H * dk:].view(-1, H, dv).float()
+    out = torch.zeros(Tq, H, dv, dtype=q.dtype)
+    for b in range(len(cu_q) - 1):
+        q0, q1 = int(cu_q[b]), int(cu_q[b + 1])
+        k0, k1 = int(cu_k[b]), int(cu_k[b + 1])
+        i = torch.arange(q1 - q0)[:, None] + (k1 - k0) - (q1 - q0)
+        j = torch.arange(k1 - k0)[None]
+        s = torch.einsum("qhd,khd->hqk", q[q0:q1].float(),
+                         k[k0:k1]) * scale
+        s = s.masked_fill((j > i) | (j <= i - window), float("-inf"))
+        out[q0:q1] = torch.einsum("hqk,khd->qhd", torch.softmax(s, -1),
+                                  v[k0:k1]).to(q.dtype)
+    return out
+
+
+def clamped_glu(gu, limit, alpha, shift):
+    F_ = gu.shape[-1] // 2
+    g = gu[..., :F_].float().clamp(max=limit)
+    u = gu[..., F_:].float().clamp(-limit, limit)
+    return (g * torch.sigmoid(alpha * g) * (u + shift)).to(gu.dtype)

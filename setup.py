@@ -1,9 +1,16 @@
-"""Build the distllm-amd HIP extension in-tree for gfx950 (MI355X).
+"""Build the distllm-amd HIP extensions in-tree for gfx950 (MI355X).
 
     python setup.py build_ext --inplace
 
-The resulting distllm_amd/ops/_hip_ops*.so travels with the repo
-snapshot to GPU boxes (it is git-ignored but NOT gpurun-ignored).
+The kernels are grouped into a few extensions, so that a process which
+needs one group does not have to compile the others:
+
+    _hip_gemm    matrix products (every model)
+    _hip_latent  latent attention, sandwich norms, clamped GLU
+    _hip_ops     everything else
+
+DISTLLM_EXT=_hip_gemm,_hip_latent restricts a build to the named ones.
+The resulting distllm_amd/ops/_hip_*.so are git-ignored.
 """
 
 import os
@@ -15,23 +22,39 @@ from setuptools import setup
 from torch.utils.cpp_extension import BuildExtension, CUDAExtension
 
 CSRC = Path(__file__).parent / "distllm_amd" / "ops" / "csrc"
+GROUPS = {
+    "_hip_gemm": ["ext_gemm.cpp", "blt_gemm.cpp", "gemm.hip", "gemm8.hip",
+                  "gemm16.hip", "decode_gemm.hip"],
+    "_hip_latent": ["ext_latent.cpp", "latent_attention.hip",
+                    "window_attention.hip", "sandwich_norm.hip",
+                    "clamped_glu.hip"],
+}
+_taken = {s for group in GROUPS.values() for s in group}
 # *_hip.hip files are torch-hipify build artifacts — exclude them.
-SOURCES = [str(CSRC / "ext.cpp"), str(CSRC / "blt_gemm.cpp")] + sorted(
-    str(p) for p in CSRC.glob("*.hip") if not p.name.endswith("_hip.hip")
+GROUPS["_hip_ops"] = ["ext.cpp"] + sorted(
+    p.name for p in CSRC.glob("*.hip")
+    if not p.name.endswith("_hip.hip") and p.name not in _taken
 )
+
+wanted = os.environ.get("DISTLLM_EXT", "")
+names = [n for n in wanted.split(",") if n] or list(GROUPS)
+
+# hipcc -O3 forms packed-FP32 instructions from ordinary float code; some
+# of their forms have given wrong results on this hardware, so the
+# feature is off for every kernel.
+HIPCC_FLAGS = ["-O3", "--offload-arch=gfx950", "-std=c++17",
+               "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 
 setup(
     name="distllm_amd_ops",
     ext_modules=[
         CUDAExtension(
-            name="distllm_amd.ops._hip_ops",
-            sources=SOURCES,
-            extra_compile_args={
-                "cxx": ["-O3"],
-                "nvcc": ["-O3", "--offload-arch=gfx950", "-std=c++17"],
-            },
-            libraries=["hipblaslt"],
+            name=f"distllm_amd.ops.{name}",
+            sources=[str(CSRC / s) for s in GROUPS[name]],
+            extra_compile_args={"cxx": ["-O3"], "nvcc": HIPCC_FLAGS},
+            libraries=["hipblaslt"] if name == "_hip_gemm" else [],
         )
+        for name in names
     ],
     cmdclass={"build_ext": BuildExtension},
 )
