@@ -3,10 +3,12 @@ fused HIP sampling. Replaces the reference's vLLM dependency
 (reference generate/generators/vllm_backend.py).
 
 Architecture (MI355X-first):
-  - per-layer paged KV caches [num_blocks, HKV, BLK=16, D] bf16 sized
-    for the 288 GB HBM budget;
+  - a paged cache sized for the 288 GB HBM budget, in the model's own
+    layout (per-layer K/V pages, or pages of latents);
   - prefill: batched padded forward through the flash-attention prefill
-    kernel, K/V scattered into the paged cache;
+    kernel, K/V scattered into the paged cache; models that run ragged
+    step batches (engine/step.py) take prompts in portions instead, in
+    the same step as the decoded tokens of other sequences;
   - decode: one fused paged-attention kernel call per layer for the
     whole running batch (batch grows/shrinks every step =
     token-granularity continuous batching);
@@ -23,6 +25,7 @@ import torch
 
 from .. import ops
 from ..models.mistral import DecoderModel
+from .step import StepBatch
 
 
 @dataclass
@@ -46,10 +49,20 @@ class _Seq:
     done: bool = False
     # per-sequence token budget; None -> the batch SamplingParams cap
     max_tokens: int | None = None
+    cached: int = 0  # leading tokens whose cache entries are written
 
     @property
     def length(self) -> int:
         return len(self.prompt_ids) + len(self.out_ids)
+
+    def pending(self, n: int | None = None) -> list[int]:
+        """The next n (default: all) tokens that are not cached yet."""
+        end = self.length if n is None else self.cached + n
+        p = len(self.prompt_ids)
+        if self.cached >= p:
+            return self.out_ids[self.cached - p: end - p]
+        return (self.prompt_ids[self.cached: end]
+                + self.out_ids[: max(0, end - p)])
 
 
 class BlockManager:
@@ -79,6 +92,8 @@ class BlockManager:
 
 class LLMEngine:
     BLK = 16
+    # prompt tokens that a ragged step takes on at most
+    STEP_TOKENS = 8192
 
     def __init__(self, model: DecoderModel, max_batch_size: int = 64,
                  max_model_len: int = 4096,
@@ -99,42 +114,36 @@ class LLMEngine:
         if weight_dtype == "fp8_e4m3":
             if not str(model.device).startswith("cuda"):
                 raise ValueError("fp8_e4m3 weights require a GPU")
+            if not hasattr(model, "enable_fp8_decode"):
+                raise ValueError(f"{type(model).__name__} has no "
+                                 "fp8_e4m3 weight path")
             model.enable_fp8_decode()
         self.device = model.device
         self.max_batch_size = max_batch_size
         self.max_model_len = min(max_model_len, d.max_position_embeddings)
         dev = self.device
-        hkv = getattr(model, 'local_kv_heads', d.kv_heads)
-        hd, L = d.head_dim, d.num_layers
         # optional OCP fp8-e4m3 KV cache (CDNA4-native): halves KV
         # bandwidth/footprint; off by default (bf16 = reference dtype)
         if kv_cache_dtype not in ("bf16", "fp8_e4m3"):
             raise ValueError(f"kv_cache_dtype {kv_cache_dtype!r}")
         self.kv_cache_dtype = kv_cache_dtype
-        kv_el = 1 if kv_cache_dtype == "fp8_e4m3" else 2
-        bytes_per_block_layer = hkv * self.BLK * hd * kv_el * 2  # k+v
         if num_blocks is None:
             if str(dev).startswith("cuda"):
                 free, _total = torch.cuda.mem_get_info(dev)
                 budget = int(free * kv_memory_fraction)
             else:
                 budget = 64 << 20  # CPU tests: 64 MiB
-            num_blocks = max(budget // (bytes_per_block_layer * L), 16)
+            num_blocks = max(budget // model.cache_bytes_per_block(
+                self.BLK, kv_cache_dtype), 16)
             # cap: enough for max_batch_size * max_model_len
             need = (self.max_model_len // self.BLK + 1) * max_batch_size
             num_blocks = min(num_blocks, need)
         num_blocks += 1  # block 0 is reserved (graph-padding dummy)
         self.num_blocks = num_blocks
-        cache_dt = (torch.uint8 if kv_cache_dtype == "fp8_e4m3"
-                    else model.dtype)
         if kv_cache_dtype == "fp8_e4m3" and not str(dev).startswith("cuda"):
             raise ValueError("fp8_e4m3 KV cache requires a GPU")
-        self.kcaches = [
-            torch.zeros(num_blocks, hkv, self.BLK, hd, dtype=cache_dt,
-                        device=dev)
-            for _ in range(L)
-        ]
-        self.vcaches = [torch.zeros_like(k) for k in self.kcaches]
+        self.cache = model.make_cache(num_blocks, self.BLK, kv_cache_dtype)
+        self.ragged = model.ragged
         self.blockman = BlockManager(num_blocks, self.BLK)
         self._next_id = 0
         # hipGraph-captured decode (one graph per pow2 batch bucket):
@@ -151,6 +160,14 @@ class LLMEngine:
         self._rng.manual_seed(0x5EED)
         self.max_blocks_per_seq = (self.max_model_len // self.BLK) + 1
         self._graphs: dict[int, "_GraphRunner"] = {}
+
+    @property
+    def kcaches(self):
+        return self.cache.k
+
+    @property
+    def vcaches(self):
+        return self.cache.v
 
     # ---- public --------------------------------------------------------
     @torch.no_grad()
@@ -181,7 +198,7 @@ class LLMEngine:
                 s.blocks = self.blockman.alloc(need)
                 admitted.append(waiting.pop(0))
             if admitted:
-                self._run_prefill(admitted, params, results)
+                self._start(admitted, params, results)
                 running.extend(s for s in admitted if not s.done)
             if not running:
                 if admitted or not waiting:
@@ -191,11 +208,107 @@ class LLMEngine:
                 raise RuntimeError(
                     "cannot admit any sequence: KV pool too small"
                 )
-            # one decode step for the whole running batch
-            self._run_decode(running, params, results)
+            # one step for the whole running batch
+            self._advance(running, params, results)
             running = [s for s in running if not s.done]
 
         return [results.get(i, []) for i in range(len(prompts_ids))]
+
+    def _start(self, seqs: list[_Seq], params: SamplingParams,
+               results: dict[int, list[int]]) -> None:
+        """Take up admitted sequences. Ragged models need nothing here:
+        the following steps bring the prompts in."""
+        if not self.ragged:
+            self._run_prefill(seqs, params, results)
+
+    def _advance(self, seqs: list[_Seq], params: SamplingParams,
+                 results: dict[int, list[int]]) -> None:
+        """One step of the running batch: every sequence that has been
+        sampled decodes its token; prompts advance by what is left of
+        the step's token budget."""
+        if not self.ragged or all(s.length - s.cached == 1 and s.cached
+                                  for s in seqs):
+            self._run_decode(seqs, params, results)
+            return
+        budget = self.STEP_TOKENS
+        work, ready = [], []
+        for s in sorted(seqs, key=lambda s: s.length - s.cached > 1):
+            left = s.length - s.cached
+            if left == 0:
+                raise ValueError("a sequence needs at least one token")
+            n = min(left, budget)
+            if n == 0:
+                continue
+            budget -= n
+            work.append((s, s.pending(n)))
+            if n == left:
+                ready.append((s, len(work) - 1, n - 1))
+        want: list[list[int]] = [[] for _ in work]
+        for _, w, last in ready:
+            want[w] = [last]
+        logits = self.step(work, want)
+        if ready:
+            self._sample_and_append([s for s, _, _ in ready], logits,
+                                    params, results)
+
+    @torch.no_grad()
+    def step(self, work: list[tuple[_Seq, list[int]]],
+             want: list[list[int]]) -> torch.Tensor | None:
+        """Run one ragged step: for each (sequence, its next tokens).
+        Returns the f32 logits [wanted, vocab] at the places `want` names
+        among each entry's tokens, in entry order; None if there are
+        none. Cache blocks are allotted as sequences grow."""
+        if not self.ragged:
+            raise RuntimeError("this model does not run ragged steps")
+        self._grow(work)
+        if (all(len(t) == 1 and s.cached for s, t in work)
+                and len(work) <= self.max_batch_size):
+            tokens = torch.tensor([t[0] for _, t in work],
+                                  device=self.device)
+            ctx = torch.tensor([s.cached + 1 for s, _ in work],
+                               dtype=torch.int32, device=self.device)
+            logits = self._decode_logits([s for s, _ in work], tokens, ctx)
+            pick = [i for i, w in enumerate(want) for _ in w]
+            out = None
+            if pick:
+                out = (logits if pick == list(range(len(work)))
+                       else logits[pick])
+        else:
+            batch = StepBatch.build(
+                [(t, s.cached, s.blocks) for s, t in work], self.BLK,
+                self.device, self.model.expand_min)
+            hidden = self.model.forward_step(batch, self.cache)
+            pick = [int(batch.rows[i][k]) for i, w in enumerate(want)
+                    for k in w]
+            out = None
+            if pick:
+                rows = torch.tensor(pick, device=self.device)
+                out = self.model.logits(hidden[rows])
+        for s, t in work:
+            s.cached += len(t)
+        return out
+
+    def _grow(self, work) -> None:
+        need = []
+        for s, t in work:
+            end = s.cached + len(t)
+            if end > self.max_model_len:
+                raise RuntimeError(
+                    f"sequence {s.seq_id} exceeds max_model_len "
+                    f"{self.max_model_len}")
+            need.append(max(0, self.blockman.blocks_for(end)
+                            - len(s.blocks)))
+        if not self.blockman.can_alloc(sum(need)):
+            raise RuntimeError("KV blocks exhausted")
+        for (s, _), n in zip(work, need):
+            if n:
+                s.blocks = s.blocks + self.blockman.alloc(n)
+
+    def release(self, s: _Seq) -> None:
+        """Give back everything a finished sequence holds."""
+        self.blockman.release(s.blocks)
+        s.blocks = []
+        s.cached = 0
 
     def _block_table(self, seqs: list[_Seq],
                      width: int | None = None) -> torch.Tensor:
@@ -211,6 +324,12 @@ class LLMEngine:
     @torch.no_grad()
     def _run_prefill(self, seqs: list[_Seq], params: SamplingParams,
                      results: dict[int, list[int]]) -> None:
+        if self.ragged:
+            todo = list(seqs)
+            while todo:
+                self._advance(todo, params, results)
+                todo = [s for s in todo if not s.out_ids]
+            return
         dev = self.device
         B = len(seqs)
         maxlen = max(s.length for s in seqs)
@@ -242,6 +361,8 @@ class LLMEngine:
                 vsel = vsel.to(torch.float8_e4m3fn).view(torch.uint8)
             self.kcaches[li][flat_blk, :, flat_slot] = ksel
             self.vcaches[li][flat_blk, :, flat_slot] = vsel
+        for s in seqs:
+            s.cached = s.length
         # last-token logits -> first sampled token
         last = (lens - 1).long()
         hlast = hidden[torch.arange(B, device=dev), last]
@@ -276,21 +397,28 @@ class LLMEngine:
     def _run_decode(self, seqs: list[_Seq], params: SamplingParams,
                     results: dict[int, list[int]]) -> None:
         dev = self.device
-        tokens = torch.tensor([s.out_ids[-1] for s in seqs], device=dev)
+        # (a prompt that a step's budget cut one short has no output yet)
+        tokens = torch.tensor([(s.out_ids or s.prompt_ids)[-1]
+                               for s in seqs], device=dev)
         ctx = torch.tensor([s.length for s in seqs], dtype=torch.int32,
                            device=dev)
+        logits = self._decode_logits(seqs, tokens, ctx)
+        for s in seqs:
+            s.cached = s.length
+        self._sample_and_append(seqs, logits, params, results)
+
+    def _decode_logits(self, seqs: list[_Seq], tokens: torch.Tensor,
+                       ctx: torch.Tensor) -> torch.Tensor:
+        """Logits of one token per sequence, from the captured graph of
+        the batch bucket where graphs are in use."""
         runner = None
         if self.use_graphs:
             runner = self._graph_for_or_eager(len(seqs))
         if runner is not None:
             bt = self._block_table(seqs, width=self.max_blocks_per_seq)
-            logits = runner.run(tokens, bt, ctx)
-            logits = logits[: len(seqs)]
-        else:
-            bt = self._block_table(seqs)
-            logits = self.model.decode_step(tokens, self.kcaches,
-                                            self.vcaches, bt, ctx)
-        self._sample_and_append(seqs, logits, params, results)
+            return runner.run(tokens, bt, ctx)[: len(seqs)]
+        return self.model.decode_step(tokens, self.cache,
+                                      self._block_table(seqs), ctx)
 
     def _sample_and_append(self, seqs, logits, params, results):
         dev = self.device
@@ -318,8 +446,7 @@ class LLMEngine:
                 if tok in params.stop_token_ids:
                     out = out[:-1]
                 results[s.seq_id] = out
-                self.blockman.release(s.blocks)
-                s.blocks = []
+                self.release(s)
 
     def warm_graphs(self, batch_sizes: list[int] | None = None) -> None:
         """Pre-capture decode graphs for the given batch buckets."""
@@ -400,15 +527,14 @@ class _GraphRunner:
         side.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(side):
             for _ in range(2):  # warmup allocations/paths
-                engine.model.decode_step(self.tokens, engine.kcaches,
-                                         engine.vcaches, self.bt, self.ctx)
+                engine.model.decode_step(self.tokens, engine.cache,
+                                         self.bt, self.ctx)
         torch.cuda.current_stream().wait_stream(side)
         torch.cuda.synchronize()
         self.graph = torch.cuda.CUDAGraph()
         with torch.cuda.graph(self.graph):
             self.logits = engine.model.decode_step(
-                self.tokens, engine.kcaches, engine.vcaches, self.bt,
-                self.ctx)
+                self.tokens, engine.cache, self.bt, self.ctx)
 
     def run(self, tokens: torch.Tensor, bt: torch.Tensor,
             ctx: torch.Tensor) -> torch.Tensor:

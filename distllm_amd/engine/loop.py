@@ -116,7 +116,7 @@ class EngineLoop:
             if admitted:
                 try:
                     seqs = [r.seq for r in admitted]
-                    eng._run_prefill(seqs, params, results)
+                    eng._start(seqs, params, results)
                 except Exception as e:
                     for r in admitted:
                         eng.blockman.release(r.seq.blocks)
@@ -145,8 +145,8 @@ class EngineLoop:
                         self._cv.wait(0.05)
                 continue
             try:
-                eng._run_decode([r.seq for r in self._running], params,
-                                results)
+                eng._advance([r.seq for r in self._running], params,
+                             results)
             except Exception as e:
                 for r in self._running:
                     eng.blockman.release(r.seq.blocks)

@@ -1,0 +1,133 @@
+"""Ragged step batches: what a model that runs them gets for one step.
+
+A step holds, for each of its sequences, the next tokens of that
+sequence — a portion of a prompt or one decoded token — and where its
+cache pages are. Rows (tokens) of all sequences are packed without
+padding between them. Sequences with few new tokens come first ("folded"
+rows, attended one by one against the paged cache); longer portions
+follow and are attended by the packed flash kernel. The row count is
+rounded up so that products see few distinct shapes; padding rows have
+ctx 0 and touch nothing.
+"""
+
+from __future__ import annotations
+
+from dataclasses import dataclass, field
+
+import numpy as np
+import torch
+
+from .. import ops
+
+
+def row_bucket(n: int) -> int:
+    """Rows a step of n tokens runs with: powers of two, then multiples
+    of 256 (which also lets the large MFMA GEMMs compete)."""
+    b = 8
+    while b < n and b < 256:
+        b <<= 1
+    return b if n <= b else (n + 255) // 256 * 256
+
+
+@dataclass
+class Expansion:
+    """Visible cached tokens of the expanded portions for one window."""
+
+    key_seq: torch.Tensor    # [Tk] block-table row of each packed key
+    key_pos: torch.Tensor    # [Tk] its position
+    cu_q: torch.Tensor       # [P + 1]
+    cu_k: torch.Tensor       # [P + 1]
+    block_map: tuple[torch.Tensor, torch.Tensor]
+
+
+@dataclass
+class StepBatch:
+    tokens: torch.Tensor       # [M] int64
+    ctx: torch.Tensor          # [M] int32, position + 1; 0 = padding
+    row_seq: torch.Tensor      # [M] int32, block-table row
+    block_table: torch.Tensor  # [S, max_blocks] int32
+    n_folded: int              # leading rows attended one by one
+    # rows of each entry, in the order in which entries were given
+    rows: list[np.ndarray] = field(default_factory=list)
+    # expanded portions: (block-table row, first position, new tokens)
+    portions: list[tuple[int, int, int]] = field(default_factory=list)
+    _expansions: dict[int, Expansion] = field(default_factory=dict)
+
+    @classmethod
+    def decode(cls, tokens, block_table, ctx) -> "StepBatch":
+        """One token per sequence, everything already on the device."""
+        n = tokens.shape[0]
+        return cls(tokens=tokens.long(), ctx=ctx.int(),
+                   row_seq=torch.arange(n, dtype=torch.int32,
+                                        device=tokens.device),
+                   block_table=block_table.int(), n_folded=n)
+
+    @classmethod
+    def build(cls, entries, blk: int, device,
+              expand_min: int = 32) -> "StepBatch":
+        """entries: (new tokens, tokens already cached, cache blocks).
+        Portions of at least expand_min tokens are expanded."""
+        order = sorted(range(len(entries)),
+                       key=lambda i: len(entries[i][0]) >= expand_min)
+        total = sum(len(t) for t, _, _ in entries)
+        n_folded = sum(len(t) for t, _, _ in entries
+                       if len(t) < expand_min)
+        M = row_bucket(total)
+        tokens = np.zeros(M, np.int64)
+        ctx = np.zeros(M, np.int32)
+        row_seq = np.zeros(M, np.int32)
+        width = max(1, max((len(b) for _, _, b in entries), default=1))
+        table = np.zeros((max(1, len(entries)), width), np.int32)
+        rows: list = [None] * len(entries)
+        portions = []
+        at = 0
+        for i in order:
+            toks, start, blocks = entries[i]
+            n = len(toks)
+            if start + n > len(blocks) * blk:
+                raise ValueError("step entry exceeds its cache blocks")
+            table[i, : len(blocks)] = blocks
+            tokens[at: at + n] = toks
+            ctx[at: at + n] = np.arange(start + 1, start + n + 1)
+            row_seq[at: at + n] = i
+            rows[i] = np.arange(at, at + n)
+            if n >= expand_min:
+                portions.append((i, start, n))
+            at += n
+
+        def up(a):
+            return torch.from_numpy(a).to(device)
+
+        return cls(tokens=up(tokens), ctx=up(ctx), row_seq=up(row_seq),
+                   block_table=up(table),
+                   n_folded=n_folded if portions else M, rows=rows,
+                   portions=portions)
+
+    def expansion(self, window: int) -> Expansion:
+        """Key map of the expanded portions under a window: each
+        portion's own tokens and the window - 1 cached before them."""
+        e = self._expansions.get(window)
+        if e is not None:
+            return e
+        dev = self.tokens.device
+        seqs, poss, nq, nk = [], [], [0], [0]
+        for s, start, n in self.portions:
+            lo = max(0, start - (window - 1))
+            poss.append(np.arange(lo, start + n, dtype=np.int32))
+            seqs.append(np.full(start + n - lo, s, np.int32))
+            nq.append(n)
+            nk.append(start + n - lo)
+        cu_q = torch.from_numpy(np.cumsum(nq).astype(np.int32))
+        cu_k = torch.from_numpy(np.cumsum(nk).astype(np.int32))
+        b_seq, b_qb = ops.varlen_block_map(cu_q)
+        # packed keys get the same rounding as rows: few product shapes
+        T = row_bucket(int(cu_k[-1]))
+        key_seq = np.zeros(T, np.int32)
+        key_pos = np.zeros(T, np.int32)
+        key_seq[: cu_k[-1]] = np.concatenate(seqs)
+        key_pos[: cu_k[-1]] = np.concatenate(poss)
+        e = Expansion(torch.from_numpy(key_seq).to(dev),
+                      torch.from_numpy(key_pos).to(dev), cu_q.to(dev),
+                      cu_k.to(dev), (b_seq.to(dev), b_qb.to(dev)))
+        self._expansions[window] = e
+        return e

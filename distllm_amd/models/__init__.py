@@ -5,8 +5,10 @@ from __future__ import annotations
 import torch
 
 from .bert import BertEncoder
-from .config import PRESETS, ModelDims, get_dims
+from .config import (PRESETS, LayeredDims, ModelDims, dims_from_checkpoint,
+                     get_dims)
 from .esm import Esm2Encoder, EsmCEncoder
+from .kanotar import KanotarModel
 from .mistral import DecoderModel
 
 __all__ = [
@@ -14,14 +16,18 @@ __all__ = [
     "DecoderModel",
     "Esm2Encoder",
     "EsmCEncoder",
+    "KanotarModel",
+    "LayeredDims",
     "ModelDims",
     "PRESETS",
     "build_model",
+    "dims_from_checkpoint",
     "get_dims",
+    "load_pretrained",
 ]
 
 
-def build_model(name_or_dims: str | ModelDims, device: str | None = None,
+def build_model(name_or_dims: str | ModelDims | LayeredDims, device: str | None = None,
                 dtype=torch.bfloat16, **kw):
     dims = (
         get_dims(name_or_dims)
@@ -36,9 +42,27 @@ def build_model(name_or_dims: str | ModelDims, device: str | None = None,
         m = EsmCEncoder(dims, dtype=dtype, **kw)
     elif dims.arch in ("mistral", "llama", "qwen2"):
         m = DecoderModel(dims, dtype=dtype, **kw)
+    elif dims.arch == "kanotar":
+        # parameters are made where they stay: no host copy of the model
+        with torch.device(device or "cpu"):
+            m = KanotarModel(dims, dtype=dtype, **kw)
     else:
         raise ValueError(f"unknown arch {dims.arch}")
     if device is not None:
         m = m.to(device)
     m.eval()
     return m
+
+
+def load_pretrained(path, device: str | None = None, dtype=torch.bfloat16,
+                    **kw):
+    """Model of a checkpoint folder whose config.json describes it in
+    full (the file's architecture names the model class)."""
+    from .loader import load_weights
+
+    dims = dims_from_checkpoint(path)
+    if dims is None:
+        raise ValueError(f"{path}/config.json names no known architecture")
+    model = build_model(dims, device=device, dtype=dtype, **kw)
+    load_weights(model, path)
+    return model

@@ -1,0 +1,198 @@
+"""Mixers and feed-forwards of decoders that are described layer by layer.
+
+A mixer maps the normed rows of a ragged step batch (engine/step.py) to
+the sublayer's output and owns what it keeps in the cache. Sizes of the
+parameters are rounded up to multiples of 64 with zeros, so that the
+16-byte loads and MFMA tiles of the kernels never see a partial row; the
+zeros leave every product and (with the true sizes passed along) every
+norm unchanged. `load` takes the checkpoint's unpadded tensors.
+"""
+
+from __future__ import annotations
+
+import torch
+from torch import nn
+
+from .. import ops
+from .config import ClampedGluDims, LatentAttentionDims
+
+
+def pad64(n: int) -> int:
+    return (n + 63) // 64 * 64
+
+
+def head_pad(n: int) -> int:
+    """Head sizes of the packed-prompt attention kernel: 64, 128, 256."""
+    for p in (64, 128, 256):
+        if n <= p:
+            return p
+    return pad64(n)
+
+
+def padded(w: torch.Tensor, *shape: int) -> torch.Tensor:
+    out = w.new_zeros(shape)
+    out[tuple(slice(0, n) for n in w.shape)] = w
+    return out
+
+
+def padded_heads(w: torch.Tensor, heads: int, d: int, dp: int,
+                 cols: int) -> torch.Tensor:
+    """[heads * d, c] -> [heads * dp, cols]."""
+    out = w.new_zeros(heads, dp, cols)
+    out[:, :d, : w.shape[1]] = w.view(heads, d, -1)
+    return out.view(heads * dp, cols)
+
+
+def expect(name: str, w: torch.Tensor, *shape: int) -> torch.Tensor:
+    if tuple(w.shape) != shape:
+        raise ValueError(f"checkpoint weight {name} has shape "
+                         f"{tuple(w.shape)}, the configuration says {shape}")
+    return w
+
+
+def _weight(rows: int, cols: int, dtype) -> nn.Parameter:
+    return nn.Parameter(torch.empty(rows, cols, dtype=dtype))
+
+
+def norm_weight(n: int) -> nn.Parameter:
+    # norms are computed in fp32 whatever the model's dtype
+    return nn.Parameter(torch.empty(n, dtype=torch.float32))
+
+
+class LatentAttention(nn.Module):
+    """Latent attention with a sliding window, on paged latents.
+
+    Two forms of the same function:
+      folded   queries are taken into the latent space (q' = Uk^T q) and
+               every head reads the cached latent itself — single tokens
+               and short portions, where reading the cache is the cost;
+      expanded keys and values of the visible latents are formed by one
+               product and attended by the flash kernel — long portions,
+               where the score products are the cost.
+    """
+
+    def __init__(self, d: LatentAttentionDims, width: int, eps: float,
+                 dtype):
+        super().__init__()
+        self.d, self.width, self.eps = d, width, eps
+        self.wp = pad64(width)
+        self.dp, self.vp = head_pad(d.dim), head_pad(d.vdim)
+        self.qp, self.rp = pad64(d.q_rank), pad64(d.kv_rank)
+        self.own = d.kv_from is None
+        H = d.heads
+        # one product for both down-projections of a layer
+        self.wdown = _weight(self.qp + (self.rp if self.own else 0),
+                             self.wp, dtype)
+        self.q_norm = norm_weight(self.qp)
+        self.kv_norm = norm_weight(self.rp) if self.own else None
+        self.wuq = _weight(H * self.dp, self.qp, dtype)
+        # all heads' key rows, then all heads' value rows
+        self.wukv = _weight(H * (self.dp + self.vp), self.rp, dtype)
+        self.wo = _weight(self.wp, H * self.vp, dtype)
+        self._fold: tuple | None = None
+
+    def checkpoint(self, src: dict, pre: str) -> dict[str, torch.Tensor]:
+        """Own parameter name -> padded tensor, from a raw checkpoint."""
+        d, H = self.d, self.d.heads
+
+        def get(name, *shape):
+            return expect(pre + name, src[pre + name], *shape)
+
+        down = [padded(get("dq", d.q_rank, self.width), self.qp, self.wp)]
+        out = {"q_norm": padded(get("dq.norm", d.q_rank), self.qp)}
+        if self.own:
+            down.append(padded(get("dkv", d.kv_rank, self.width),
+                               self.rp, self.wp))
+            out["kv_norm"] = padded(get("dkv.norm", d.kv_rank), self.rp)
+        out["wdown"] = torch.cat(down)
+        out["wuq"] = padded_heads(get("uq", H * d.dim, d.q_rank), H, d.dim,
+                                  self.dp, self.qp)
+        out["wukv"] = torch.cat([
+            padded_heads(get("uk", H * d.dim, d.kv_rank), H, d.dim,
+                         self.dp, self.rp),
+            padded_heads(get("uv", H * d.vdim, d.kv_rank), H, d.vdim,
+                         self.vp, self.rp)])
+        out["wo"] = padded_heads(
+            get("o", self.width, H * d.vdim).t(), H, d.vdim, self.vp,
+            self.wp).t()
+        return out
+
+    def _folded(self) -> tuple[torch.Tensor, torch.Tensor]:
+        """(Uk^T [H, R, dim], Uv [H, vdim, R]); Uk^T is a copy, renewed
+        when the weights change."""
+        w, H = self.wukv, self.d.heads
+        key = (w.data_ptr(), w._version)
+        if self._fold is None or self._fold[0] != key:
+            uk = w[: H * self.dp].view(H, self.dp, self.rp)
+            self._fold = (key, uk.detach().transpose(1, 2).contiguous())
+        return self._fold[1], w[H * self.dp:].view(H, self.vp, self.rp)
+
+    def expands(self) -> bool:
+        """Whether the flash kernel covers this layer's dtype and sizes."""
+        w = self.wuq
+        return (max(self.dp, self.vp) <= 256
+                and (w.dtype == torch.bfloat16 or not w.is_cuda))
+
+    def forward(self, h, batch, latents):
+        """h [M, width]; latents: the paged cache [blocks, BLK, rank] of
+        the layer that owns it."""
+        d, H = self.d, self.d.heads
+        M = h.shape[0]
+        bt, ctx = batch.block_table, batch.ctx
+        ab = ops.linear(h, self.wdown)
+        cq = ops.latent_prep(ab, self.qp, d.q_rank, d.kv_rank, self.q_norm,
+                             self.kv_norm, self.eps,
+                             latents if self.own else None, bt,
+                             batch.row_seq, ctx)
+        q = ops.linear(cq, self.wuq).view(M, H, self.dp)
+        # leading rows folded, then the rows of expanded portions; padding
+        # rows trail and count as folded ones that see nothing
+        n = batch.n_folded if self.expands() else M
+        if n == M:
+            o = h.new_empty(M, H, self.vp)
+        else:
+            o = h.new_zeros(M, H, self.vp)
+        if n > 0:
+            uk_t, uv = self._folded()
+            ql = ops.head_gemm(q[:n], uk_t)
+            ol = ops.latent_attn(ql, latents, bt, batch.row_seq[:n],
+                                 ctx[:n], d.window, d.scale)
+            ops.head_gemm(ol, uv, out=o[:n])
+        if n < M:
+            e = batch.expansion(d.window)
+            c = ops.latent_gather(latents, bt, e.key_seq, e.key_pos)
+            kv = ops.linear(c, self.wukv)
+            ops.attn_window(q[n:], kv, o[n:], e.cu_q, e.cu_k, e.block_map,
+                            d.window, d.scale)
+        return ops.linear(o.view(M, H * self.vp), self.wo)
+
+
+class ClampedGlu(nn.Module):
+    def __init__(self, d: ClampedGluDims, width: int, dtype):
+        super().__init__()
+        self.d, self.width = d, width
+        self.wp, self.fp = pad64(width), pad64(d.ff)
+        self.wgup = _weight(2 * self.fp, self.wp, dtype)
+        self.wdown = _weight(self.wp, self.fp, dtype)
+
+    def checkpoint(self, src: dict, pre: str) -> dict[str, torch.Tensor]:
+        ff, W = self.d.ff, self.width
+
+        def get(name, *shape):
+            return expect(pre + name, src[pre + name], *shape)
+
+        return {
+            "wgup": torch.cat([padded(get("gate", ff, W), self.fp, self.wp),
+                               padded(get("up", ff, W), self.fp, self.wp)]),
+            "wdown": padded(get("down", W, ff), self.wp, self.fp),
+        }
+
+    def forward(self, h):
+        d = self.d
+        return ops.linear(
+            ops.gateup_clamped_glu(h, self.wgup, d.limit, d.alpha, d.shift),
+            self.wdown)
+
+
+MIXERS = {"latent_attention": LatentAttention}
+MLPS = {"dense": ClampedGlu}

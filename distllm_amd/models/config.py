@@ -9,15 +9,18 @@ decoder family used for generation (K15):
   - Mistral-class decoder embedders (SFR-Embedding-Mistral)
   - Llama-class causal LMs for generation
   - Qwen2-class causal LMs (llama family + qkv bias)
+  - Kanotar causal LMs: every layer has its own description (LayeredDims)
 Dims are from the public model cards; weights are random-init here
 (no network) or loadable from local safetensors.
 """
 
 from __future__ import annotations
 
+import json
+from pathlib import Path
 from typing import Literal
 
-from pydantic import BaseModel
+from pydantic import BaseModel, ConfigDict, PositiveInt, model_validator
 
 
 class ModelDims(BaseModel):
@@ -50,7 +53,133 @@ class ModelDims(BaseModel):
         return self.num_kv_heads or self.num_heads
 
 
-PRESETS: dict[str, ModelDims] = {
+class _Strict(BaseModel):
+    model_config = ConfigDict(extra="forbid")
+
+
+class LatentAttentionDims(_Strict):
+    """Attention whose keys and values are linear in one cached latent of
+    kv_rank numbers per token; queries come from a latent of q_rank."""
+
+    type: Literal["latent_attention"] = "latent_attention"
+    heads: PositiveInt
+    dim: PositiveInt           # query/key size per head
+    vdim: PositiveInt          # value size per head
+    q_rank: PositiveInt
+    kv_rank: PositiveInt
+    scale: float
+    window: PositiveInt        # a token sees itself and window - 1 before
+    kv_from: int | None = None  # layer whose latents this one reads
+
+
+class ClampedGluDims(_Strict):
+    """Feed-forward g * sigmoid(alpha g) * (u + shift), gate g clamped
+    from above and up-projection u from both sides at `limit`."""
+
+    kind: Literal["dense"] = "dense"
+    ff: PositiveInt
+    limit: float
+    alpha: float = 1.702
+    shift: float = 1.0
+
+
+class LayerDims(_Strict):
+    mixer: LatentAttentionDims
+    mlp: ClampedGluDims | None = None
+
+
+class LayeredDims(BaseModel):
+    """A decoder whose layers are described one by one."""
+
+    arch: Literal["kanotar"]
+    vocab_size: PositiveInt
+    hidden_size: PositiveInt
+    layers: list[LayerDims]
+    norm_eps: float
+    logit_scale: float = 1.0
+    # no rotation and no position table: nothing in the design bounds it
+    max_position_embeddings: int = 1 << 20
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @model_validator(mode="after")
+    def _check_sharing(self):
+        if not self.layers:
+            raise ValueError("a model needs at least one layer")
+        for i, layer in enumerate(self.layers):
+            j = layer.mixer.kv_from
+            if j is None:
+                continue
+            if not 0 <= j < i:
+                raise ValueError(f"layer {i}: kv_from {j} is not an "
+                                 "earlier layer")
+            src = self.layers[j].mixer
+            if src.kv_from is not None:
+                raise ValueError(f"layer {i}: kv_from {j} has no latent "
+                                 "of its own")
+            if src.kv_rank != layer.mixer.kv_rank:
+                raise ValueError(f"layer {i}: kv_rank differs from that "
+                                 f"of layer {j}")
+        return self
+
+
+def _kanotar_dims(cfg: dict) -> LayeredDims:
+    layers = []
+    for i, entry in enumerate(cfg["layers"]):
+        if entry["type"] != "latent_attention":
+            raise ValueError(f"layer {i}: unknown mixer {entry['type']!r}")
+        mixer = dict(entry["mixer"])
+        mask = dict(mixer.pop("mask"))
+        mixer["window"] = mask.pop("size")
+        if mask:
+            raise ValueError(f"layer {i}: unknown mask keys {sorted(mask)}")
+        layers.append(LayerDims(mixer=LatentAttentionDims(**mixer),
+                                mlp=entry.get("mlp")))
+    return LayeredDims(arch="kanotar", vocab_size=cfg["vocab"],
+                       hidden_size=cfg["width"], layers=layers,
+                       norm_eps=cfg["norm"]["eps"],
+                       logit_scale=cfg["logit_scale"])
+
+
+# config.json "architecture" -> reader of the rest of the file
+CONFIG_READERS = {"Kanotar": _kanotar_dims}
+
+
+def dims_from_checkpoint(path: str | Path) -> LayeredDims | None:
+    """Dims from a checkpoint folder's config.json; None when there is no
+    such file or it names no architecture that is described in full."""
+    f = Path(path) / "config.json"
+    if not f.is_file():
+        return None
+    cfg = json.loads(f.read_text())
+    reader = CONFIG_READERS.get(cfg.get("architecture"))
+    return reader(cfg) if reader else None
+
+
+def layered_preset(num_layers: int, hidden: int, vocab: int, heads: int,
+                   dim: int, vdim: int, q_rank: int, kv_rank: int, ff: int,
+                   windows: list[int], share_from: int | None = None,
+                   limit: float = 7.0, logit_scale: float = 1.0,
+                   eps: float = 1e-5) -> LayeredDims:
+    """Kanotar dims of repeated layers: window i is windows[i % len]; from
+    layer share_from on, layers read the latents of layer share_from - 1."""
+    layers = []
+    for i in range(num_layers):
+        shared = share_from is not None and i >= share_from
+        layers.append(LayerDims(
+            mixer=LatentAttentionDims(
+                heads=heads, dim=dim, vdim=vdim, q_rank=q_rank,
+                kv_rank=kv_rank, scale=dim ** -0.5,
+                window=windows[i % len(windows)],
+                kv_from=share_from - 1 if shared else None),
+            mlp=ClampedGluDims(ff=ff, limit=limit)))
+    return LayeredDims(arch="kanotar", vocab_size=vocab, hidden_size=hidden,
+                       layers=layers, norm_eps=eps, logit_scale=logit_scale)
+
+
+PRESETS: dict[str, ModelDims | LayeredDims] = {
     # S-PubMedBERT / PubMedBERT-base: the reference's headline embed
     # encoder (examples/embed/AMP.nougat.pubmedbert.yaml)
     "pubmedbert-base": ModelDims(
@@ -135,10 +264,19 @@ PRESETS: dict[str, ModelDims] = {
         max_position_embeddings=512, rms_norm_eps=1e-6,
         attention_bias=True,
     ),
+    # layers of the llama3-8b size, for like-for-like measurements
+    "kanotar-8b": layered_preset(
+        32, 4096, 128256, heads=32, dim=128, vdim=128, q_rank=1536,
+        kv_rank=512, ff=14336, windows=[4096],
+    ),
+    "kanotar-tiny": layered_preset(
+        3, 256, 1024, heads=4, dim=32, vdim=32, q_rank=64, kv_rank=64,
+        ff=512, windows=[48, 32], share_from=2,
+    ),
 }
 
 
-def get_dims(name: str) -> ModelDims:
+def get_dims(name: str) -> ModelDims | LayeredDims:
     if name not in PRESETS:
         raise KeyError(
             f"unknown model preset {name!r}; available: {sorted(PRESETS)}"

@@ -174,6 +174,14 @@ def load_weights(model, path: str | Path) -> None:
             mapped = _map_llama(src, model)
         elif arch == "esm2":
             mapped = _map_esm2(src, model)
+        elif arch == "kanotar":
+            missing = sorted(model.checkpoint_names() - set(src))
+            if missing:
+                raise ValueError(f"checkpoint lacks {missing}")
+            extra = sorted(set(src) - model.checkpoint_names())
+            if extra:
+                raise ValueError(f"checkpoint has unknown weights {extra}")
+            mapped = model.checkpoint(src)
         else:
             raise ValueError(
                 f"no HF mapping for arch {arch}; provide a native checkpoint"

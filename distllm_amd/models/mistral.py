@@ -72,8 +72,25 @@ class DecoderLayer(nn.Module):
         return self.wgup[self._inter:]
 
 
+class KVCache:
+    """Paged keys and values, one [blocks, HKV, BLK, D] pair per layer."""
+
+    def __init__(self, model: "DecoderModel", num_blocks: int, blk: int,
+                 dtype):
+        d = model.dims
+        self.k = [
+            torch.zeros(num_blocks, model.local_kv_heads, blk, d.head_dim,
+                        dtype=dtype, device=model.device)
+            for _ in range(d.num_layers)
+        ]
+        self.v = [torch.zeros_like(k) for k in self.k]
+
+
 class DecoderModel(nn.Module):
     """forward() -> last_hidden_state; generation via prefill()/decode()."""
+
+    # the engine prefills whole padded prompts and decodes in lockstep
+    ragged = False
 
     def __init__(self, dims: ModelDims, dtype=torch.bfloat16,
                  with_lm_head: bool | None = None,
@@ -239,6 +256,17 @@ class DecoderModel(nn.Module):
         return ops.linear(hidden, w).float()
 
     # ---- generation-engine entry points --------------------------------
+    def cache_bytes_per_block(self, blk: int, kv_cache_dtype: str) -> int:
+        el = 1 if kv_cache_dtype == "fp8_e4m3" else 2
+        d = self.dims
+        return self.local_kv_heads * blk * d.head_dim * el * 2 * d.num_layers
+
+    def make_cache(self, num_blocks: int, blk: int,
+                   kv_cache_dtype: str) -> KVCache:
+        fp8 = kv_cache_dtype == "fp8_e4m3"
+        return KVCache(self, num_blocks, blk,
+                       torch.uint8 if fp8 else self.dtype)
+
     @torch.no_grad()
     def prefill(self, input_ids, attention_mask):
         """Full prefill; returns (last_hidden [B,S,H], kv list per layer
@@ -248,15 +276,16 @@ class DecoderModel(nn.Module):
         return hidden, kv
 
     @torch.no_grad()
-    def decode_step(self, tokens, kcaches, vcaches, block_tables, ctx_lens):
+    def decode_step(self, tokens, cache: KVCache, block_tables, ctx_lens):
         """One decode step for B sequences.
 
-        tokens: [B] int; caches: per-layer paged [nblk, HKV, BLK, D];
+        tokens: [B] int; cache: per-layer paged [nblk, HKV, BLK, D];
         ctx_lens: [B] int32 length INCLUDING the new token (the new
         token's kv is written at position ctx_lens-1 by this call).
         Returns logits [B, V] f32.
         """
         d = self.dims
+        kcaches, vcaches = cache.k, cache.v
         B = tokens.shape[0]
         nh, kvh, hd = self.local_heads, self.local_kv_heads, d.head_dim
         cs, sn = self._rope(tokens.device)
