@@ -34,11 +34,14 @@ def main() -> None:
     ap.add_argument("--seq-len", type=int, default=512)
     ap.add_argument("--model", type=str, default="pubmedbert-base")
     ap.add_argument("--mode", type=str, default="embed",
-                    choices=["embed", "generate", "pipeline"],
+                    choices=["embed", "generate", "pipeline", "decoders"],
                     help="embed = flagship seqs/s; generate = decode "
                          "tokens/s (Llama-class, paged KV); pipeline = "
                          "full jsonl_chunk -> semantic_chunk embed -> "
-                         "write (tokenizer + staging included)")
+                         "write (tokenizer + staging included); "
+                         "decoders = prefill and decode of latent-"
+                         "attention layers beside llama layers of equal "
+                         "size")
     ap.add_argument("--docs-per-file", type=int, default=128)
     ap.add_argument("--pooler", type=str, default="mean",
                     choices=["mean", "last_token"])
@@ -46,8 +49,15 @@ def main() -> None:
     ap.add_argument("--weight-dtype", type=str, default="bf16",
                     choices=["bf16", "fp8_e4m3"],
                     help="generate mode: W8A16 fp8 decode weights")
+    ap.add_argument("--layers", type=int, default=8,
+                    help="decoders mode: layers per model")
+    ap.add_argument("--only", type=str, default="",
+                    help="decoders mode: sizes to run, with commas")
     args = ap.parse_args()
 
+    if args.mode == "decoders":
+        bench_decoders(args)
+        return
     if args.mode == "generate":
         bench_generate(args)
         return
@@ -233,6 +243,113 @@ def bench_generate(args) -> None:
                 "parallelism": f"dp{world}",
             },
         }))
+
+
+def bench_decoders(args) -> None:
+    """Kanotar layers beside llama layers of the same width, heads and
+    feed-forward, through the same engine: tokens/s of prefilling a batch
+    of prompts and of decoding at a given context, both models in turn.
+    Random weights, synthetic tokens, one GPU."""
+    from distllm_amd.engine import LLMEngine, SamplingParams
+    from distllm_amd.engine.engine import _Seq
+    from distllm_amd.models import ModelDims, build_model
+    from distllm_amd.models.config import layered_preset
+
+    dev = "cuda:0"
+    torch.manual_seed(5)
+    V = 32768
+
+    def llama(hidden, heads, kv, ff):
+        return ModelDims(arch="llama", vocab_size=V, hidden_size=hidden,
+                         num_layers=args.layers, num_heads=heads,
+                         num_kv_heads=kv, intermediate_size=ff,
+                         max_position_embeddings=16384)
+
+    def kanotar(hidden, heads, q_rank, kv_rank, ff, window, share=None):
+        return layered_preset(args.layers, hidden, V, heads, 128, 128,
+                              q_rank, kv_rank, ff, [window], share)
+
+    # name: (kanotar, llama, [(prompts, prompt len)], [(batch, context)])
+    sizes = {
+        "4096x32h full": (
+            kanotar(4096, 32, 1536, 512, 14336, 8192),
+            llama(4096, 32, 8, 14336),
+            [(16, 2048), (2, 8000)], [(1, 2048), (32, 2048), (128, 2048),
+                                      (32, 8000)]),
+        "4096x32h window 1024": (
+            kanotar(4096, 32, 1536, 512, 14336, 1024),
+            llama(4096, 32, 8, 14336), [(2, 8000)], [(32, 8000)]),
+        "2048x16h full": (
+            kanotar(2048, 16, 768, 256, 8192, 8192),
+            llama(2048, 16, 4, 8192),
+            [(16, 2048)], [(1, 2048), (128, 2048)]),
+        "7168x64h shared latents": (
+            kanotar(7168, 64, 1536, 512, 18432, 8192, args.layers // 2),
+            llama(7168, 56, 8, 18432), [(8, 2048)], [(32, 2048)]),
+    }
+    params = SamplingParams(temperature=0.0, min_p=0.0, max_tokens=10 ** 6)
+    rows = []
+    for name, (kd, ld, prefills, decodes) in sizes.items():
+        if args.only and name.split()[0] not in args.only.split(",") \
+                and name not in args.only.split(","):
+            continue
+        models = {"kanotar": build_model(kd, device=dev),
+                  "llama": build_model(ld, device=dev)}
+
+        def run(kind, model, batch, ctx):
+            eng = LLMEngine(model, max_batch_size=batch,
+                            max_model_len=ctx + 64,
+                            num_blocks=batch * ((ctx + 64) // 16 + 2))
+            ids = torch.randint(4, V, (batch, ctx)).tolist()
+
+            def start():
+                seqs = [_Seq(seq_id=i, prompt_ids=p)
+                        for i, p in enumerate(ids)]
+                for s in seqs:
+                    s.blocks = eng.blockman.alloc((ctx + 64) // 16 + 1)
+                return seqs
+
+            times = []
+            if kind == "prefill":
+                for i in range(args.warmup + args.steps):
+                    seqs = start()
+                    torch.cuda.synchronize()
+                    t0 = time.perf_counter()
+                    eng._run_prefill(seqs, params, {})
+                    torch.cuda.synchronize()
+                    times.append(time.perf_counter() - t0)
+                    for s in seqs:
+                        eng.release(s)
+                n = batch * ctx
+            else:
+                seqs = start()
+                eng._run_prefill(seqs, params, {})
+                for i in range(args.warmup + args.steps):
+                    torch.cuda.synchronize()
+                    t0 = time.perf_counter()
+                    eng._run_decode(seqs, params, {})
+                    torch.cuda.synchronize()
+                    times.append(time.perf_counter() - t0)
+                n = batch
+            times = sorted(times[args.warmup:])
+            return n, times[len(times) // 2]
+
+        for kind, todo in (("prefill", prefills), ("decode", decodes)):
+            for batch, ctx in todo:
+                row = {"size": name, "kind": kind, "batch": batch,
+                       "context": ctx}
+                for which, model in models.items():
+                    n, t = run(kind, model, batch, ctx)
+                    row[which + "_ms"] = round(t * 1e3, 3)
+                    row[which + "_tok_s"] = round(n / t, 1)
+                rows.append(row)
+                print(json.dumps(row), flush=True)
+        del models
+        torch.cuda.empty_cache()
+    print(json.dumps({"metric": "decoder layers, tokens/s",
+                      "layers": args.layers, "steps": args.steps,
+                      "warmup": args.warmup, "dtype": "bf16",
+                      "data": "synthetic", "rows": rows}))
 
 
 def bench_pipeline(args) -> None:

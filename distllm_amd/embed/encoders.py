@@ -15,8 +15,8 @@ from typing import Any, Literal, Union
 import torch
 from pydantic import Field, model_validator
 
-from ..models import build_model, get_dims
-from ..models.config import PRESETS, ModelDims
+from ..models import build_model, dims_from_checkpoint, get_dims
+from ..models.config import PRESETS, LayeredDims, ModelDims
 from ..registry import registry
 from ..utils import BaseConfig
 from .tokenizers import load_tokenizer
@@ -54,6 +54,16 @@ def resolve_preset(name_or_path: str) -> str:
     if "qwen" in low:
         return "qwen2-7b"
     raise ValueError(f"cannot resolve model preset for {name_or_path!r}")
+
+
+def resolve_model(name_or_path: str) -> tuple[ModelDims | LayeredDims, str]:
+    """Dims of a preset, a known model id or a checkpoint folder, and the
+    folder to load weights from: a folder whose config.json describes its
+    model in full stands for itself."""
+    dims = dims_from_checkpoint(name_or_path)
+    if dims is not None:
+        return dims, str(name_or_path)
+    return get_dims(resolve_preset(name_or_path)), ""
 
 
 class _NativeEncoder:
@@ -150,8 +160,7 @@ class EsmCambrianEncoderConfig(BaseConfig):
 
 
 def _build(cfg) -> _NativeEncoder:
-    preset = resolve_preset(cfg.pretrained_model_name_or_path)
-    dims = get_dims(preset)
+    dims, folder = resolve_model(cfg.pretrained_model_name_or_path)
     device = _default_device()
     if device != "cpu" and not cfg.half_precision:
         # The MFMA kernel path is bf16-I/O by design (fp32 accumulate);
@@ -167,7 +176,7 @@ def _build(cfg) -> _NativeEncoder:
         model_max_length=dims.max_position_embeddings,
     )
     return _NativeEncoder(dims, device, dtype, tok,
-                          weights_path=cfg.weights_path or None)
+                          weights_path=cfg.weights_path or folder or None)
 
 
 EncoderConfigs = Union[

@@ -148,7 +148,11 @@ def load_tokenizer(name_or_path: str, arch: str = "bert",
     import warnings
 
     p = Path(name_or_path) if name_or_path else None
-    if p is not None and p.exists():
+    # a checkpoint folder may come without a tokenizer
+    bare = (p is not None and p.is_dir() and (p / "config.json").exists()
+            and not any(f for pat in ("*token*", "vocab*", "*.model")
+                        for f in p.glob(pat)))
+    if p is not None and p.exists() and not bare:
         from transformers import AutoTokenizer
 
         tok = AutoTokenizer.from_pretrained(str(p))

@@ -18,6 +18,7 @@ Architecture (MI355X-first):
 
 from __future__ import annotations
 
+import gc
 import math
 from dataclasses import dataclass, field
 
@@ -271,8 +272,8 @@ class LLMEngine:
             pick = [i for i, w in enumerate(want) for _ in w]
             out = None
             if pick:
-                out = (logits if pick == list(range(len(work)))
-                       else logits[pick])
+                # a copy: the next replay overwrites the graph's output
+                out = logits[torch.tensor(pick, device=self.device)]
         else:
             batch = StepBatch.build(
                 [(t, s.cached, s.blocks) for s, t in work], self.BLK,
@@ -516,7 +517,8 @@ class _GraphRunner:
 
     def __init__(self, engine: LLMEngine, batch: int):
         dev = engine.device
-        self.engine = engine
+        # no reference to the engine is kept: the pair would be a cycle,
+        # freed only by a garbage collection at some arbitrary moment
         self.batch = batch
         self.tokens = torch.zeros(batch, dtype=torch.long, device=dev)
         self.bt = torch.zeros(batch, engine.max_blocks_per_seq,
@@ -532,9 +534,19 @@ class _GraphRunner:
         torch.cuda.current_stream().wait_stream(side)
         torch.cuda.synchronize()
         self.graph = torch.cuda.CUDAGraph()
-        with torch.cuda.graph(self.graph):
-            self.logits = engine.model.decode_step(
-                self.tokens, engine.cache, self.bt, self.ctx)
+        # A collection during capture may destroy graphs of a dead engine
+        # or synchronize (see __del__); neither is allowed while a stream
+        # is capturing, and the failed destructor ends the process.
+        gc.collect()
+        enabled = gc.isenabled()
+        gc.disable()
+        try:
+            with torch.cuda.graph(self.graph):
+                self.logits = engine.model.decode_step(
+                    self.tokens, engine.cache, self.bt, self.ctx)
+        finally:
+            if enabled:
+                gc.enable()
 
     def run(self, tokens: torch.Tensor, bt: torch.Tensor,
             ctx: torch.Tensor) -> torch.Tensor:

@@ -88,16 +88,17 @@ class NativeGenerator:
     def __init__(self, config: NativeGeneratorConfig):
         import torch
 
-        from ..embed.encoders import resolve_preset
+        from ..embed.encoders import resolve_model
         from ..embed.tokenizers import load_tokenizer
         from ..engine import LLMEngine, SamplingParams
-        from ..models import build_model, get_dims
+        from ..models import build_model
 
         self.config = config
-        preset = resolve_preset(config.model)
-        dims = get_dims(preset)
+        dims, folder = resolve_model(config.model)
         device = "cuda" if torch.cuda.is_available() else "cpu"
         dtype = torch.bfloat16 if device != "cpu" else torch.float32
+        if config.dtype == "float32" and dims.arch == "kanotar":
+            dtype = torch.float32  # its kernels run in 32-bit as well
         kw = {}
         if config.tensor_parallel_size > 1:
             import torch.distributed as dist
@@ -113,11 +114,11 @@ class NativeGenerator:
                     "(TP subgroups are not split out in this round)"
                 )
             kw["tp_group"] = dist.group.WORLD
-        self.model = build_model(preset, device=device, dtype=dtype, **kw)
-        if config.weights_path:
+        self.model = build_model(dims, device=device, dtype=dtype, **kw)
+        if config.weights_path or folder:
             from ..models.loader import load_weights
 
-            load_weights(self.model, config.weights_path)
+            load_weights(self.model, config.weights_path or folder)
         self.tokenizer = load_tokenizer(
             config.tokenizer_path or config.model,
             arch=dims.arch, vocab_size=dims.vocab_size,

@@ -29,6 +29,14 @@ def head_pad(n: int) -> int:
     return pad64(n)
 
 
+def rank_pad(n: int) -> int:
+    """Latent sizes of the MFMA decode kernel, or any multiple of 64."""
+    for p in (64, 128, 192, 256, 384, 512):
+        if n <= p:
+            return p
+    return pad64(n)
+
+
 def padded(w: torch.Tensor, *shape: int) -> torch.Tensor:
     out = w.new_zeros(shape)
     out[tuple(slice(0, n) for n in w.shape)] = w
@@ -77,7 +85,7 @@ class LatentAttention(nn.Module):
         self.d, self.width, self.eps = d, width, eps
         self.wp = pad64(width)
         self.dp, self.vp = head_pad(d.dim), head_pad(d.vdim)
-        self.qp, self.rp = pad64(d.q_rank), pad64(d.kv_rank)
+        self.qp, self.rp = pad64(d.q_rank), rank_pad(d.kv_rank)
         self.own = d.kv_from is None
         H = d.heads
         # one product for both down-projections of a layer

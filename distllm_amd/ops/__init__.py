@@ -583,14 +583,16 @@ def head_gemm(x, w, out=None):
     return out.copy_(res)
 
 
-def latent_attn(q, cache, block_table, row_seq, ctx, window, scale):
+def latent_attn(q, cache, block_table, row_seq, ctx, window, scale,
+                nsplit=0):
     """Attention of single-token rows over paged latents, queries folded
     into the latent space: q [M, H, R] -> [M, H, R]. A row sees the last
-    `window` positions of its sequence up to its own (ctx - 1)."""
+    `window` positions of its sequence up to its own (ctx - 1). nsplit:
+    workgroups that share a row's keys (0: chosen from the sizes)."""
     if q.is_cuda:
         _require_hip("_hip_latent")
         return _hip_ops.latent_attn(q, cache, block_table, row_seq, ctx,
-                                    window, scale)
+                                    window, scale, nsplit)
     return torch_ref.latent_attn(q, cache, block_table, row_seq, ctx,
                                  window, scale)
 

@@ -17,6 +17,11 @@ void launch_head_gemm(const void*, const void*, void*, int, int, int, int,
 void launch_latent_attn_rows(const void*, const void*, const int*,
                              const int*, const int*, void*, int, int, int,
                              int, int, float, bool, hipStream_t);
+int latent_decode_waves(int);
+bool latent_decode_covers(int);
+void launch_latent_decode(const void*, const void*, const int*, const int*,
+                          const int*, void*, void*, void*, int, int, int, int,
+                          int, int, float, hipStream_t);
 void launch_attn_window(const void*, const void*, const void*, void*,
                         const int*, const int*, const int*, const int*, int,
                         int, int, int, int, long, int, float, hipStream_t);
@@ -150,7 +155,9 @@ void head_gemm(torch::Tensor x, torch::Tensor W, torch::Tensor out) {
 
 torch::Tensor latent_attn(torch::Tensor q, torch::Tensor cache,
                           torch::Tensor bt, torch::Tensor row_seq,
-                          torch::Tensor ctx, int64_t window, double scale) {
+                          torch::Tensor ctx, int64_t window, double scale,
+                          int64_t nsplit) {
+  // nsplit: workgroups that share a row's keys; 0 = choose
   CHECK_DEV(q); CHECK_CONT(q); CHECK_T(q);
   const int M = q.size(0), H = q.size(1), R = q.size(2);
   check_pages(cache, bt, row_seq, ctx, M);
@@ -160,12 +167,40 @@ torch::Tensor latent_attn(torch::Tensor q, torch::Tensor cache,
   TORCH_CHECK(window > 0, "window must be positive");
   const int win = (int)std::min<int64_t>(window, 1 << 30);
   auto out = torch::empty_like(q);
-  if (M > 0)
+  if (M == 0) return out;
+  if (is_f32(q) || !latent_decode_covers(R)) {
     launch_latent_attn_rows(q.data_ptr(), cache.data_ptr(),
                             bt.data_ptr<int>(), row_seq.data_ptr<int>(),
                             ctx.data_ptr<int>(), out.data_ptr(), M, H, R,
                             bt.size(1), win, (float)scale, is_f32(q),
                             cur_stream());
+    return out;
+  }
+  // Split each row's keys until there are two workgroups per CU, as long
+  // as a split keeps two tiles. All sizes are known on the host, so a
+  // captured graph stays valid as contexts grow.
+  long NS = nsplit;
+  if (NS <= 0) {
+    const long per_wg = 16L * latent_decode_waves(H);
+    const long wgs = (long)M * ((H + per_wg - 1) / per_wg);
+    const long keys = std::min<long>(win, bt.size(1) * 16L);
+    const long tiles = keys / 32 + 1;
+    NS = std::min<long>({(512 + wgs - 1) / wgs, (tiles + 1) / 2, 64L});
+  }
+  NS = std::max<long>(NS, 1);
+  torch::Tensor pacc, pml;
+  void *pa = nullptr, *pm = nullptr;
+  if (NS > 1) {
+    auto f32 = q.options().dtype(at::kFloat);
+    pacc = torch::empty({(long)M * H * NS, R}, f32);
+    pml = torch::empty({(long)M * H * NS, 2}, f32);
+    pa = pacc.data_ptr();
+    pm = pml.data_ptr();
+  }
+  launch_latent_decode(q.data_ptr(), cache.data_ptr(), bt.data_ptr<int>(),
+                       row_seq.data_ptr<int>(), ctx.data_ptr<int>(),
+                       out.data_ptr(), pa, pm, M, H, R, (int)NS, bt.size(1),
+                       win, (float)scale, cur_stream());
   return out;
 }
 
@@ -219,7 +254,9 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("latent_prep", &latent_prep);
   m.def("latent_gather", &latent_gather);
   m.def("head_gemm", &head_gemm);
-  m.def("latent_attn", &latent_attn);
+  m.def("latent_attn", &latent_attn, py::arg("q"), py::arg("cache"),
+        py::arg("block_table"), py::arg("row_seq"), py::arg("ctx"),
+        py::arg("window"), py::arg("scale"), py::arg("nsplit") = 0);
   m.def("attn_window", &attn_window);
   m.def("clamped_glu", &clamped_glu);
 }

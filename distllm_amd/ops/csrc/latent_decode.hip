@@ -1,0 +1,302 @@
+// MFMA attention of single-token rows over paged bf16 latents (see
+// latent_attention.hip for the mechanism, the cache layout and the row
+// arguments; that file's one-head kernel covers the other types and ranks).
+//
+// A wave owns 16 heads of one row and keeps their folded queries and output
+// accumulators in registers; a workgroup of NW waves covers 16 * NW heads,
+// so a latent is read from HBM once for all of them. The visible keys of a
+// row are split over NS workgroups whose partial results a second kernel
+// joins.
+//
+// Tiles of 32 keys go global -> registers -> LDS, where each tile is kept
+// twice: row-major (key operand of the score product) and transposed (the
+// same numbers as value operand). The next tile's loads are in flight while
+// the current one is used.
+//
+// Both products use mfma_f32_16x16x32_bf16 with keys (then latent columns)
+// as rows and heads as columns, so a lane holds scores of ONE head: softmax
+// state is lane-local, and the score fragment is the weight fragment of the
+// second product as it stands, given that the transposed copy orders the 32
+// keys the way the score tiles leave them: slot g*8 + i is key g*4 + i for
+// i < 4 and key 16 + g*4 + (i - 4) above.
+#include "common.h"
+
+#define PBLK 16
+#define KT 32
+#define LOG2E 1.4426950408889634f
+
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+
+extern __shared__ __attribute__((aligned(16))) char smem[];
+
+// byte address of the 16-byte slot (4 per row: 32 keys) of latent column r;
+// 64 bytes of padding per 8 rows and the slot swizzle spread the banks
+__device__ __forceinline__ int ct_slot(int r, int slot) {
+  return r * 64 + (r >> 3) * 64 + ((slot ^ ((r >> 2) & 3)) * 16);
+}
+
+template <int R, int NW>
+__global__ void __launch_bounds__(64 * NW, NW == 4 ? 2 : 1)
+latent_decode_kernel(const unsigned short* __restrict__ q,
+                     const unsigned short* __restrict__ cache,
+                     const int* __restrict__ block_table,
+                     const int* __restrict__ row_seq,
+                     const int* __restrict__ ctx,
+                     unsigned short* __restrict__ out,
+                     float* __restrict__ pacc, float* __restrict__ pml,
+                     int H, int HG, int NS, int max_blocks, int window,
+                     float scale) {
+  constexpr int NT = 64 * NW;
+  constexpr int UNITS = R;  // a unit: 4 keys x 8 latent columns
+  constexpr int UPT = (UNITS + NT - 1) / NT;
+  constexpr int SW = R % 128 == 0 ? 15 : 7;
+  constexpr int CT = KT * R * 2;  // LDS offset of the transposed copy
+
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int i16 = lane & 15, g = lane >> 4;
+  const int split = blockIdx.x % NS;
+  const int hg = blockIdx.x / NS % HG;
+  const int row = blockIdx.x / NS / HG;
+  const int head = (hg * NW + wid) * 16 + i16;
+  const bool live = head < H;
+
+  const int L = min(ctx[row], max_blocks * PBLK);
+  const int lo = L > window ? L - window : 0;
+  const int T0 = lo / KT, T1 = L > 0 ? (L + KT - 1) / KT : T0;
+  const int per = (T1 - T0 + NS - 1) / NS;
+  const int ts = T0 + split * per, te = min(T1, ts + per);
+  const int last_page = L > 0 ? (L - 1) / PBLK : 0;
+  const int* bt = block_table + (long)row_seq[row] * max_blocks;
+
+  bf16x8 qf[R / 32];
+  {
+    const unsigned short* qr =
+        q + ((long)row * H + (live ? head : 0)) * R + g * 8;
+#pragma unroll
+    for (int s = 0; s < R / 32; ++s) {
+      s16x8 v = *reinterpret_cast<const s16x8*>(qr + s * 32);
+      if (!live) v = (s16x8)(short)0;
+      qf[s] = __builtin_bit_cast(bf16x8, v);
+    }
+  }
+
+  const int kg = (threadIdx.x >> 3) & 7;  // key group of all my units
+  auto page_of = [&](int t) {
+    return bt[min(t * (KT / PBLK) + (kg >> 2), last_page)];
+  };
+  i32x4 kv[UPT][4];
+  auto issue = [&](int page) {
+    const unsigned short* base =
+        cache + ((long)page * PBLK + (kg & 3) * 4) * R;
+#pragma unroll
+    for (int i = 0; i < UPT; ++i) {
+      const int u = threadIdx.x + i * NT;
+      if (UNITS % NT == 0 || u < UNITS) {
+        const int c = (u >> 6) * 8 + (u & 7);
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          kv[i][j] =
+              *reinterpret_cast<const i32x4*>(base + (long)j * R + c * 8);
+      }
+    }
+  };
+  auto stage = [&]() {
+#pragma unroll
+    for (int i = 0; i < UPT; ++i) {
+      const int u = threadIdx.x + i * NT;
+      if (UNITS % NT == 0 || u < UNITS) {
+        const int c = (u >> 6) * 8 + (u & 7);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+          const int key = kg * 4 + j;
+          *reinterpret_cast<i32x4*>(smem + key * (R * 2) +
+                                    ((c ^ (key & SW)) * 16)) = kv[i][j];
+        }
+#pragma unroll
+        for (int w = 0; w < 4; ++w) {
+          i32x2 even, odd;
+          even[0] = __builtin_amdgcn_perm(kv[i][1][w], kv[i][0][w],
+                                          0x05040100);
+          even[1] = __builtin_amdgcn_perm(kv[i][3][w], kv[i][2][w],
+                                          0x05040100);
+          odd[0] = __builtin_amdgcn_perm(kv[i][1][w], kv[i][0][w],
+                                         0x07060302);
+          odd[1] = __builtin_amdgcn_perm(kv[i][3][w], kv[i][2][w],
+                                         0x07060302);
+          const int r = c * 8 + w * 2;
+          char* dst = smem + CT + (kg >> 2) * 8;
+          *reinterpret_cast<i32x2*>(dst + ct_slot(r, kg & 3)) = even;
+          *reinterpret_cast<i32x2*>(dst + ct_slot(r + 1, kg & 3)) = odd;
+        }
+      }
+    }
+  };
+
+  float m = -1e30f, l = 0.f;
+  f32x4 acc[R / 16];
+#pragma unroll
+  for (int i = 0; i < R / 16; ++i) acc[i] = {0.f, 0.f, 0.f, 0.f};
+  const float scale2 = scale * LOG2E;
+
+  int page = 0;
+  if (ts < te) {
+    issue(page_of(ts));
+    page = page_of(min(ts + 1, te - 1));
+  }
+  for (int t = ts; t < te; ++t) {
+    __syncthreads();  // every wave is done with the previous tile
+    stage();
+    if (t + 1 < te) {
+      issue(page);
+      page = page_of(min(t + 2, te - 1));
+    }
+    __syncthreads();
+
+    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int s = 0; s < R / 32; ++s) {
+      const char* a =
+          smem + i16 * (R * 2) + (((s * 4 + g) ^ (i16 & SW)) * 16);
+      const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(a);
+      const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(a + 16 * R * 2);
+      s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, qf[s], s0, 0, 0, 0);
+      s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, qf[s], s1, 0, 0, 0);
+    }
+    float p[8];
+    float pmax = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const int key = t * KT + (i >> 2) * 16 + g * 4 + (i & 3);
+      const float s = (i < 4 ? s0[i & 3] : s1[i & 3]) * scale2;
+      p[i] = key >= lo && key < L ? s : -INFINITY;
+      pmax = fmaxf(pmax, p[i]);
+    }
+    pmax = fmaxf(pmax, __shfl_xor(pmax, 16, 64));
+    pmax = fmaxf(pmax, __shfl_xor(pmax, 32, 64));
+    if (!__all(pmax <= m)) {
+      const float mn = fmaxf(m, pmax);
+      const float alpha = __builtin_amdgcn_exp2f(m - mn);
+      m = mn;
+      l *= alpha;
+#pragma unroll
+      for (int i = 0; i < R / 16; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) acc[i][r] *= alpha;
+    }
+    s16x8 pb;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      const float e = __builtin_amdgcn_exp2f(p[i] - m);
+      l += e;  // this lane's keys only; lanes are joined at the end
+      pb[i] = (short)f2bf(e);
+    }
+    const bf16x8 pf = __builtin_bit_cast(bf16x8, pb);
+#pragma unroll
+    for (int i = 0; i < R / 16; ++i) {
+      const bf16x8 v = *reinterpret_cast<const bf16x8*>(
+          smem + CT + ct_slot(i * 16 + i16, g));
+      acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pf, acc[i], 0, 0,
+                                                       0);
+    }
+  }
+  l += __shfl_xor(l, 16, 64);
+  l += __shfl_xor(l, 32, 64);
+  if (!live) return;
+  const long rh = (long)row * H + head;
+  if (NS == 1) {
+    const float inv = l > 0.f ? 1.f / l : 0.f;
+#pragma unroll
+    for (int i = 0; i < R / 16; ++i) {
+      s16x4 o;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[r] = (short)f2bf(acc[i][r] * inv);
+      *reinterpret_cast<s16x4*>(out + rh * R + i * 16 + g * 4) = o;
+    }
+  } else {
+    const long part = rh * NS + split;
+#pragma unroll
+    for (int i = 0; i < R / 16; ++i)
+      *reinterpret_cast<f32x4*>(pacc + part * R + i * 16 + g * 4) = acc[i];
+    if (g == 0) {
+      pml[part * 2] = m;
+      pml[part * 2 + 1] = l;
+    }
+  }
+}
+
+// one wave per (row, head): join NS partial results
+__global__ void __launch_bounds__(256)
+latent_combine_kernel(const float* __restrict__ pacc,
+                      const float* __restrict__ pml,
+                      unsigned short* __restrict__ out, int RH, int R,
+                      int NS) {
+  const int lane = threadIdx.x & 63;
+  const long rh = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (rh >= RH) return;
+  float M = -1e30f;
+  for (int s = 0; s < NS; ++s) M = fmaxf(M, pml[(rh * NS + s) * 2]);
+  float l = 0.f;
+  for (int s = 0; s < NS; ++s)
+    l += pml[(rh * NS + s) * 2 + 1] *
+         __builtin_amdgcn_exp2f(pml[(rh * NS + s) * 2] - M);
+  const float inv = l > 0.f ? 1.f / l : 0.f;
+  for (int c = lane * 4; c < R; c += 256) {
+    f32x4 o = {0.f, 0.f, 0.f, 0.f};
+    for (int s = 0; s < NS; ++s) {
+      const float a =
+          __builtin_amdgcn_exp2f(pml[(rh * NS + s) * 2] - M) * inv;
+      const f32x4 v =
+          *reinterpret_cast<const f32x4*>(pacc + (rh * NS + s) * R + c);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) o[i] += a * v[i];
+    }
+    s16x4 ov;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) ov[i] = (short)f2bf(o[i]);
+    *reinterpret_cast<s16x4*>(out + rh * R + c) = ov;
+  }
+}
+
+extern "C" int latent_decode_waves(int H) {
+  return H <= 16 ? 1 : H <= 32 ? 2 : 4;
+}
+
+extern "C" bool latent_decode_covers(int R) {
+  return R == 64 || R == 128 || R == 192 || R == 256 || R == 384 || R == 512;
+}
+
+extern "C" void launch_latent_decode(
+    const void* q, const void* cache, const int* block_table,
+    const int* row_seq, const int* ctx, void* out, void* pacc, void* pml,
+    int M, int H, int R, int NS, int max_blocks, int window, float scale,
+    hipStream_t stream) {
+  const int nw = latent_decode_waves(H);
+  const int hg = (H + 16 * nw - 1) / (16 * nw);
+  const int lds = KT * R * 2 + R * 72;
+#define LD(RR, NW)                                                            \
+  hipLaunchKernelGGL((latent_decode_kernel<RR, NW>), dim3(M * hg * NS),       \
+                     dim3(64 * NW), lds, stream, (const unsigned short*)q,    \
+                     (const unsigned short*)cache, block_table, row_seq, ctx, \
+                     (unsigned short*)out, (float*)pacc, (float*)pml, H, hg,  \
+                     NS, max_blocks, window, scale)
+#define LD_R(RR)                   \
+  do {                             \
+    if (nw == 1) LD(RR, 1);        \
+    else if (nw == 2) LD(RR, 2);   \
+    else LD(RR, 4);                \
+  } while (0)
+  switch (R) {
+    case 64: LD_R(64); break;
+    case 128: LD_R(128); break;
+    case 192: LD_R(192); break;
+    case 256: LD_R(256); break;
+    case 384: LD_R(384); break;
+    default: LD_R(512); break;
+  }
+#undef LD_R
+#undef LD
+  if (NS > 1)
+    hipLaunchKernelGGL(latent_combine_kernel, dim3((M * H + 3) / 4),
+                       dim3(256), 0, stream, (const float*)pacc,
+                       (const float*)pml, (unsigned short*)out, M * H, R, NS);
+}

@@ -26,8 +26,8 @@ GROUPS = {
     "_hip_gemm": ["ext_gemm.cpp", "blt_gemm.cpp", "gemm.hip", "gemm8.hip",
                   "gemm16.hip", "decode_gemm.hip"],
     "_hip_latent": ["ext_latent.cpp", "latent_attention.hip",
-                    "window_attention.hip", "sandwich_norm.hip",
-                    "clamped_glu.hip"],
+                    "latent_decode.hip", "window_attention.hip",
+                    "sandwich_norm.hip", "clamped_glu.hip"],
 }
 _taken = {s for group in GROUPS.values() for s in group}
 # *_hip.hip files are torch-hipify build artifacts — exclude them.
