@@ -94,7 +94,7 @@ class BlockManager:
 class LLMEngine:
     BLK = 16
     # prompt tokens that a ragged step takes on at most
-    STEP_TOKENS = 8192
+    STEP_TOKENS = 16384
 
     def __init__(self, model: DecoderModel, max_batch_size: int = 64,
                  max_model_len: int = 4096,

@@ -120,6 +120,13 @@ class StepBatch:
         cu_q = torch.from_numpy(np.cumsum(nq).astype(np.int32))
         cu_k = torch.from_numpy(np.cumsum(nk).astype(np.int32))
         b_seq, b_qb = ops.varlen_block_map(cu_q)
+        # workgroups with the most keys start first: they would otherwise
+        # be the tail of the launch
+        start = torch.tensor([s for _, s, _ in self.portions])
+        last = start[b_seq.long()] + (b_qb + 1) * 128
+        order = torch.argsort(last.clamp(max=window + 127),
+                              descending=True, stable=True)
+        b_seq, b_qb = b_seq[order], b_qb[order]
         # packed keys get the same rounding as rows: few product shapes
         T = row_bucket(int(cu_k[-1]))
         key_seq = np.zeros(T, np.int32)

@@ -36,6 +36,7 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 #define QWAVE 32
 #define LOG2E 1.4426950408889634f
 #define VROW 68   // padded V^T row length in bf16 elems (136 B)
+#define VROW4 72  // the same for 4-key units (144 B: aligned 16-byte reads)
 
 extern __shared__ __attribute__((aligned(16))) char smem[];
 
@@ -54,10 +55,12 @@ union frag_u {
 // last ones of its packed keys (cu for queries, cu_k for keys), as when a
 // prompt is continued from a cache, and a query sees only the `window`
 // latest keys up to its own position. Keys and values may have different
-// head sizes (DV) and interleave in one row (tstr_k counts both).
+// head sizes (DV) and interleave in one row (tstr_k counts both). V is
+// staged in units of 4 keys x 8 columns, transposed in registers, so that
+// the V^T image is written 8 bytes at a time.
 template <int D, bool CAUSAL, bool HAS_MASK, bool VDIRECT,
           bool VARLEN = false, int DV = D, bool WINDOW = false>
-__global__ void __launch_bounds__(256, 1)
+__global__ void __launch_bounds__(256, WINDOW && D + DV <= 256 ? 2 : 1)
 attn_fwd_kernel(const unsigned short* __restrict__ Q,
                 const unsigned short* __restrict__ Kt,
                 const unsigned short* __restrict__ Vt,
@@ -76,8 +79,12 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
   constexpr int NCHV = DV / 8;           // 16B chunks per V row
   constexpr int DBLK = DV / 32;          // 32-wide d blocks of V
   constexpr int KTILE_B = KVBLK * D * 2; // K tile bytes
-  constexpr int VTILE_B = DV * VROW * 2; // V^T tile bytes
-  constexpr int VCH = KVBLK * NCHV / NTHR;  // V chunks per thread
+  constexpr int VR = WINDOW ? VROW4 : VROW; // V^T row length
+  constexpr int VTILE_B = DV * VR * 2;   // V^T tile bytes
+  // V chunks per thread; 4-key units with WINDOW
+  constexpr int VUNITS = KVBLK / 4 * NCHV;
+  constexpr int VCH =
+      WINDOW ? (VUNITS + NTHR - 1) / NTHR * 4 : KVBLK * NCHV / NTHR;
 
   const int lane = threadIdx.x & 63;
   const int wid = threadIdx.x >> 6;
@@ -197,6 +204,21 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
 
   // T14 split: issue V loads into regs (no wait) ...
   auto v_issue = [&](int k0, s16x8* vreg) {
+    if constexpr (WINDOW) {
+#pragma unroll
+      for (int c = 0; c < VCH / 4; ++c) {
+        const int u = threadIdx.x + c * NTHR;
+        if (VUNITS % NTHR == 0 || u < VUNITS) {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const int key = min(k0 + u / NCHV * 4 + j, SKV - 1);
+            vreg[c * 4 + j] = *reinterpret_cast<const s16x8*>(
+                Vb + (long)key * tstr_k + u % NCHV * 8);
+          }
+        }
+      }
+      return;
+    }
     const long koff = (long)k0 * tstr_k;
 #pragma unroll
     for (int c = 0; c < VCH; ++c) {
@@ -210,6 +232,30 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
   // ... and transpose-write them into the padded V^T image later.
   auto v_write = [&](int buf, const s16x8* vreg) {
     unsigned short* vt = reinterpret_cast<unsigned short*>(smem + offV[buf]);
+    if constexpr (WINDOW) {
+#pragma unroll
+      for (int c = 0; c < VCH / 4; ++c) {
+        const int u = threadIdx.x + c * NTHR;
+        if (VUNITS % NTHR == 0 || u < VUNITS) {
+          i32x4 k[4];
+#pragma unroll
+          for (int j = 0; j < 4; ++j)
+            k[j] = __builtin_bit_cast(i32x4, vreg[c * 4 + j]);
+          unsigned short* dst = vt + u % NCHV * 8 * VR + u / NCHV * 4;
+#pragma unroll
+          for (int w = 0; w < 4; ++w) {
+            i32x2 even, odd;
+            even[0] = __builtin_amdgcn_perm(k[1][w], k[0][w], 0x05040100);
+            even[1] = __builtin_amdgcn_perm(k[3][w], k[2][w], 0x05040100);
+            odd[0] = __builtin_amdgcn_perm(k[1][w], k[0][w], 0x07060302);
+            odd[1] = __builtin_amdgcn_perm(k[3][w], k[2][w], 0x07060302);
+            *reinterpret_cast<i32x2*>(dst + w * 2 * VR) = even;
+            *reinterpret_cast<i32x2*>(dst + (w * 2 + 1) * VR) = odd;
+          }
+        }
+      }
+      return;
+    }
 #pragma unroll
     for (int c = 0; c < VCH; ++c) {
 #pragma unroll
@@ -262,13 +308,16 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
     const bool wave_active =
         q0w < SQ && (!CAUSAL || k0 <= q0w + shift + QWAVE - 1) &&
         (!WINDOW || k0 + KVBLK - 1 > q0w + shift - window);
-    // a tile that every row of the wave sees in full needs no compares
-    const bool tile_edge = !WINDOW || k0 + KVBLK - 1 > q0w + shift ||
-                           k0 <= q0w + shift + QWAVE - 1 - window;
     // mask values are only needed when a real mask exists or the tile
     // hangs over the end of the sequence (padded keys); skipping the 32
     // LDS reads otherwise removes a large per-tile VALU cost.
-    const bool tile_masked = HAS_MASK || (k0 + KVBLK > SKV);
+    // (WINDOW needs neither: padded keys are past every query.)
+    const bool tile_masked = HAS_MASK || (!WINDOW && k0 + KVBLK > SKV);
+    // WINDOW: key k is visible when 0 <= k - qlo <= qpos - qlo, one
+    // unsigned compare; kept free of branches, which cost the unrolled
+    // score loop far more than the compares
+    const unsigned int wspan = WINDOW ? qpos - qlo : 0;
+    const int woff = WINDOW ? k0 + 4 * h - qlo : 0;
 
     if (wave_active) {
       // ---- QK^T: two 32-key blocks, ONE live accumulator ----------
@@ -300,8 +349,8 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
           float s2 = accP[r] * scale2;
           if (tile_masked) s2 += mrow[key_loc];
           if (WINDOW) {
-            if (tile_edge && (k0 + key_loc > qpos || k0 + key_loc < qlo))
-              s2 = -INFINITY;
+            const int e = woff + kb * 32 + (r & 3) + 8 * (r >> 2);
+            s2 = (unsigned int)e <= wspan ? s2 : -INFINITY;
           } else if (CAUSAL && (k0 + key_loc > qrow_abs)) {
             s2 = -INFINITY;
           }
@@ -374,7 +423,7 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
             }
           } else {
             vf = *reinterpret_cast<const bf16x8*>(
-                vimg + (d * 32 + (lane & 31)) * VROW + kh * 16 + h * 8);
+                vimg + (d * 32 + (lane & 31)) * VR + kh * 16 + h * 8);
           }
           accO[d] = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
               vf, pa.v, accO[d], 0, 0, 0);

@@ -17,7 +17,7 @@ void launch_head_gemm(const void*, const void*, void*, int, int, int, int,
 void launch_latent_attn_rows(const void*, const void*, const int*,
                              const int*, const int*, void*, int, int, int,
                              int, int, float, bool, hipStream_t);
-int latent_decode_waves(int);
+int latent_decode_heads(int);
 bool latent_decode_covers(int);
 void launch_latent_decode(const void*, const void*, const int*, const int*,
                           const int*, void*, void*, void*, int, int, int, int,
@@ -100,6 +100,8 @@ torch::Tensor latent_prep(torch::Tensor ab, int64_t QP, int64_t qn,
   const int M = ab.size(0), ld = ab.size(1);
   const int R = ld - (int)QP;
   TORCH_CHECK(R >= 0 && wq.numel() == QP && qn > 0 && qn <= QP, "q sizes");
+  TORCH_CHECK(QP % 8 == 0 && QP <= 8192 && R <= 8192,
+              "latent sizes must be multiples of 8, at most 8192");
   void* cp = nullptr;
   const float* wcp = nullptr;
   int nblk = 0;
@@ -147,7 +149,7 @@ void head_gemm(torch::Tensor x, torch::Tensor W, torch::Tensor out) {
   TORCH_CHECK(W.size(0) == H && W.size(2) == K && out.size(0) == M &&
                   out.size(1) == H && out.size(2) == N,
               "head_gemm: shape mismatch");
-  TORCH_CHECK(N % 64 == 0 && K % 32 == 0, "N % 64, K % 32");
+  TORCH_CHECK(N % 64 == 0 && K % 64 == 0, "N % 64, K % 64");
   if (M > 0)
     launch_head_gemm(x.data_ptr(), W.data_ptr(), out.data_ptr(), M, H, N, K,
                      cur_stream());
@@ -176,16 +178,17 @@ torch::Tensor latent_attn(torch::Tensor q, torch::Tensor cache,
                             cur_stream());
     return out;
   }
-  // Split each row's keys until there are two workgroups per CU, as long
-  // as a split keeps two tiles. All sizes are known on the host, so a
-  // captured graph stays valid as contexts grow.
+  // Split each row's keys until the CUs are full (two workgroups each, one
+  // of the largest), as long as a split keeps four tiles. All sizes are
+  // known on the host, so a captured graph stays valid as contexts grow.
   long NS = nsplit;
   if (NS <= 0) {
-    const long per_wg = 16L * latent_decode_waves(H);
+    const long per_wg = latent_decode_heads(H);
     const long wgs = (long)M * ((H + per_wg - 1) / per_wg);
     const long keys = std::min<long>(win, bt.size(1) * 16L);
     const long tiles = keys / 32 + 1;
-    NS = std::min<long>({(512 + wgs - 1) / wgs, (tiles + 1) / 2, 64L});
+    const long fill = per_wg > 32 ? 256 : 512;
+    NS = std::min<long>({(fill + wgs - 1) / wgs, (tiles + 3) / 4, 64L});
   }
   NS = std::max<long>(NS, 1);
   torch::Tensor pacc, pml;

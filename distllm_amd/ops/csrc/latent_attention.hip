@@ -33,7 +33,8 @@ __device__ __forceinline__ void from_f(float* p, float v) { *p = v; }
 // columns, true size qn), wave 1 the cached latent (next R columns, true
 // size rn) and writes it to its cache slot. cache == nullptr: the layer
 // reads another layer's cache and has no latent of its own.
-template <typename T>
+// Rows of up to 8192 columns stay in registers between the two passes.
+template <typename T, int NC>
 __global__ void __launch_bounds__(128)
 latent_prep_kernel(const T* __restrict__ ab, int ld, int QP, int qn, int R,
                    int rn, const float* __restrict__ wq,
@@ -57,15 +58,34 @@ latent_prep_kernel(const T* __restrict__ ab, int ld, int QP, int qn, int R,
     if (blk < 0 || blk >= num_blocks) return;
     dst = cache + ((long)blk * PBLK + pos % PBLK) * R;
   }
+  float v[NC][8];
   float ss = 0.f;
-  for (int c = lane; c < np; c += 64) {
-    const float v = to_f(src[c]);
-    ss += v * v;
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = (k * 64 + lane) * 8;
+    if (c < np) {
+      load8<T>(src + c, v[k]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss += v[k][i] * v[k][i];
+    }
+  }
+  float wv[NC][8];  // in flight while the sum is reduced
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = (k * 64 + lane) * 8;
+    if (c < np) load8<float>(w + c, wv[k]);
   }
   ss = wave_reduce_sum(ss);
   const float inv = 1.f / sqrtf(ss / n + eps);
-  for (int c = lane; c < np; c += 64)
-    from_f(dst + c, to_f(src[c]) * inv * w[c]);
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = (k * 64 + lane) * 8;
+    if (c < np) {
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] *= inv * wv[k][i];
+      store8(dst + c, v[k]);
+    }
+  }
 }
 
 extern "C" void launch_latent_prep(
@@ -74,13 +94,23 @@ extern "C" void launch_latent_prep(
     const int* block_table, int max_blocks, int num_blocks,
     const int* row_seq, const int* ctx, bool fp32, hipStream_t stream) {
   const dim3 grid(M), block(cache != nullptr ? 128 : 64);
-#define LP(T)                                                               \
-  hipLaunchKernelGGL((latent_prep_kernel<T>), grid, block, 0, stream,       \
+  const int nc = ((QP > R ? QP : R) + 511) / 512;
+#define LP(T, NC)                                                           \
+  hipLaunchKernelGGL((latent_prep_kernel<T, NC>), grid, block, 0, stream,   \
                      (const T*)ab, ld, QP, qn, R, rn, wq, wc, eps, (T*)cq,  \
                      (T*)cache, block_table, max_blocks, num_blocks,        \
                      row_seq, ctx)
-  if (fp32) LP(float);
-  else LP(unsigned short);
+#define LP_N(T)                \
+  do {                         \
+    if (nc == 1) LP(T, 1);     \
+    else if (nc == 2) LP(T, 2); \
+    else if (nc <= 4) LP(T, 4); \
+    else if (nc <= 8) LP(T, 8); \
+    else LP(T, 16);            \
+  } while (0)
+  if (fp32) LP_N(float);
+  else LP_N(unsigned short);
+#undef LP_N
 #undef LP
 }
 
@@ -125,7 +155,7 @@ extern "C" void launch_latent_gather(const void* cache,
 // out[m, h, :] = W[h] x[m, h, :], W [H, N, K] bf16, for the few rows of a
 // decode step (weight-streaming bound). A wave owns 16 output columns; the
 // weight fragment is read once and used for MT tiles of 16 rows.
-template <int MT>
+template <int MT, int KU>
 __global__ void __launch_bounds__(256)
 head_gemm_kernel(const unsigned short* __restrict__ x,
                  const unsigned short* __restrict__ W,
@@ -148,15 +178,22 @@ head_gemm_kernel(const unsigned short* __restrict__ x,
   f32x4 acc[MT];
 #pragma unroll
   for (int t = 0; t < MT; ++t) acc[t] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-  for (int k = 0; k < K; k += 32) {
-    const bf16x8 wf = *reinterpret_cast<const bf16x8*>(wrow + k);
+  // KU steps of loads are in flight together
+  for (int k0 = 0; k0 < K; k0 += 32 * KU) {
+    bf16x8 wf[KU], xf[KU][MT];
 #pragma unroll
-    for (int t = 0; t < MT; ++t) {
-      const bf16x8 xf = *reinterpret_cast<const bf16x8*>(xrow[t] + k);
-      acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf, xf, acc[t], 0, 0,
-                                                       0);
+    for (int s = 0; s < KU; ++s) {
+      wf[s] = *reinterpret_cast<const bf16x8*>(wrow + k0 + s * 32);
+#pragma unroll
+      for (int t = 0; t < MT; ++t)
+        xf[s][t] = *reinterpret_cast<const bf16x8*>(xrow[t] + k0 + s * 32);
     }
+#pragma unroll
+    for (int s = 0; s < KU; ++s)
+#pragma unroll
+      for (int t = 0; t < MT; ++t)
+        acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(wf[s], xf[s][t],
+                                                         acc[t], 0, 0, 0);
   }
 #pragma unroll
   for (int t = 0; t < MT; ++t) {
@@ -174,16 +211,28 @@ head_gemm_kernel(const unsigned short* __restrict__ x,
 extern "C" void launch_head_gemm(const void* x, const void* W, void* out,
                                  int M, int H, int N, int K,
                                  hipStream_t stream) {
-#define HG(MT)                                                            \
-  hipLaunchKernelGGL((head_gemm_kernel<MT>),                              \
-                     dim3(H*(N / 64), (M + 16 * MT - 1) / (16 * MT)),     \
+  // row tiles per workgroup: as many as leave two workgroups per CU
+  const int tiles = (M + 15) / 16;
+  const long cols = (long)H * (N / 64);
+  int mt = 1;
+  while (mt < 4 && mt < tiles && cols * ((tiles + 2 * mt - 1) / (2 * mt)) >= 512)
+    mt *= 2;
+#define HG(MT, KU)                                                        \
+  hipLaunchKernelGGL((head_gemm_kernel<MT, KU>),                          \
+                     dim3(cols, (M + 16 * MT - 1) / (16 * MT)),           \
                      dim3(256), 0, stream, (const unsigned short*)x,      \
                      (const unsigned short*)W, (unsigned short*)out, M, H, \
                      N, K)
-  if (M <= 16) HG(1);
-  else if (M <= 32) HG(2);
-  else if (M <= 64) HG(4);
-  else HG(8);
+#define HG_K(MT)                     \
+  do {                               \
+    if (K % 256 == 0) HG(MT, 8);     \
+    else if (K % 128 == 0) HG(MT, 4); \
+    else HG(MT, 2);                  \
+  } while (0)
+  if (mt == 1) HG_K(1);
+  else if (mt == 2) HG_K(2);
+  else HG_K(4);
+#undef HG_K
 #undef HG
 }
 

@@ -2,23 +2,21 @@
 // latent_attention.hip for the mechanism, the cache layout and the row
 // arguments; that file's one-head kernel covers the other types and ranks).
 //
-// A wave owns 16 heads of one row and keeps their folded queries and output
-// accumulators in registers; a workgroup of NW waves covers 16 * NW heads,
-// so a latent is read from HBM once for all of them. The visible keys of a
-// row are split over NS workgroups whose partial results a second kernel
-// joins.
+// A workgroup serves HG groups of 16 heads of one row, so a latent is read
+// from HBM once for all of them; the visible keys of a row are split over NS
+// workgroups whose partial results a second kernel joins.
 //
 // Tiles of 32 keys go global -> registers -> LDS, where each tile is kept
 // twice: row-major (key operand of the score product) and transposed (the
 // same numbers as value operand). The next tile's loads are in flight while
 // the current one is used.
 //
-// Both products use mfma_f32_16x16x32_bf16 with keys (then latent columns)
-// as rows and heads as columns, so a lane holds scores of ONE head: softmax
-// state is lane-local, and the score fragment is the weight fragment of the
-// second product as it stands, given that the transposed copy orders the 32
-// keys the way the score tiles leave them: slot g*8 + i is key g*4 + i for
-// i < 4 and key 16 + g*4 + (i - 4) above.
+// KS waves work on each head group. For the scores they split the keys of
+// the tile (and, when KS is 4, the latent columns, whose partial sums meet
+// in LDS); for the output each owns R / KS latent columns, which keeps the
+// accumulators of a wave small. Both products use
+// mfma_f32_16x16x32_bf16 with keys (then latent columns) as rows and heads
+// as columns, so softmax state and rescaling are lane-local.
 #include "common.h"
 
 #define PBLK 16
@@ -29,14 +27,16 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 
 extern __shared__ __attribute__((aligned(16))) char smem[];
 
+#define SROW 36  // padded row of 32 scores
+
 // byte address of the 16-byte slot (4 per row: 32 keys) of latent column r;
 // 64 bytes of padding per 8 rows and the slot swizzle spread the banks
 __device__ __forceinline__ int ct_slot(int r, int slot) {
   return r * 64 + (r >> 3) * 64 + ((slot ^ ((r >> 2) & 3)) * 16);
 }
 
-template <int R, int NW>
-__global__ void __launch_bounds__(64 * NW, NW == 4 ? 2 : 1)
+template <int R, int HG, int KS>
+__global__ void __launch_bounds__(64 * HG * KS, 2)
 latent_decode_kernel(const unsigned short* __restrict__ q,
                      const unsigned short* __restrict__ cache,
                      const int* __restrict__ block_table,
@@ -44,20 +44,27 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
                      const int* __restrict__ ctx,
                      unsigned short* __restrict__ out,
                      float* __restrict__ pacc, float* __restrict__ pml,
-                     int H, int HG, int NS, int max_blocks, int window,
+                     int H, int NG, int NS, int max_blocks, int window,
                      float scale) {
-  constexpr int NT = 64 * NW;
+  constexpr int NT = 64 * HG * KS;
   constexpr int UNITS = R;  // a unit: 4 keys x 8 latent columns
   constexpr int UPT = (UNITS + NT - 1) / NT;
   constexpr int SW = R % 128 == 0 ? 15 : 7;
-  constexpr int CT = KT * R * 2;  // LDS offset of the transposed copy
+  constexpr int CT = KT * R * 2;        // LDS offset of the transposed copy
+  constexpr int SC = CT + R * 72;       // LDS offset of the scores
+  constexpr int RSPLIT = KS / 2;       // column parts, besides key halves
+  constexpr int QS = R / 32 / RSPLIT;  // score steps of a wave
+  constexpr int OB = R / 16 / KS;      // output blocks of a wave
+  static_assert(KS == 2 || KS == 4, "two key halves");
 
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int i16 = lane & 15, g = lane >> 4;
+  const int hgrp = wid / KS, ks = wid % KS;
+  const int khalf = ks % 2, rhalf = ks / 2;
   const int split = blockIdx.x % NS;
-  const int hg = blockIdx.x / NS % HG;
-  const int row = blockIdx.x / NS / HG;
-  const int head = (hg * NW + wid) * 16 + i16;
+  const int grp = blockIdx.x / NS % NG;
+  const int row = blockIdx.x / NS / NG;
+  const int head = (grp * HG + hgrp) * 16 + i16;
   const bool live = head < H;
 
   const int L = min(ctx[row], max_blocks * PBLK);
@@ -67,18 +74,6 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
   const int ts = T0 + split * per, te = min(T1, ts + per);
   const int last_page = L > 0 ? (L - 1) / PBLK : 0;
   const int* bt = block_table + (long)row_seq[row] * max_blocks;
-
-  bf16x8 qf[R / 32];
-  {
-    const unsigned short* qr =
-        q + ((long)row * H + (live ? head : 0)) * R + g * 8;
-#pragma unroll
-    for (int s = 0; s < R / 32; ++s) {
-      s16x8 v = *reinterpret_cast<const s16x8*>(qr + s * 32);
-      if (!live) v = (s16x8)(short)0;
-      qf[s] = __builtin_bit_cast(bf16x8, v);
-    }
-  }
 
   const int kg = (threadIdx.x >> 3) & 7;  // key group of all my units
   auto page_of = [&](int t) {
@@ -124,25 +119,39 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
           odd[1] = __builtin_amdgcn_perm(kv[i][3][w], kv[i][2][w],
                                          0x07060302);
           const int r = c * 8 + w * 2;
-          char* dst = smem + CT + (kg >> 2) * 8;
-          *reinterpret_cast<i32x2*>(dst + ct_slot(r, kg & 3)) = even;
-          *reinterpret_cast<i32x2*>(dst + ct_slot(r + 1, kg & 3)) = odd;
+          char* dst = smem + CT + (kg & 1) * 8;
+          *reinterpret_cast<i32x2*>(dst + ct_slot(r, kg >> 1)) = even;
+          *reinterpret_cast<i32x2*>(dst + ct_slot(r + 1, kg >> 1)) = odd;
         }
       }
     }
   };
-
-  float m = -1e30f, l = 0.f;
-  f32x4 acc[R / 16];
-#pragma unroll
-  for (int i = 0; i < R / 16; ++i) acc[i] = {0.f, 0.f, 0.f, 0.f};
-  const float scale2 = scale * LOG2E;
 
   int page = 0;
   if (ts < te) {
     issue(page_of(ts));
     page = page_of(min(ts + 1, te - 1));
   }
+  bf16x8 qf[QS];
+  {
+    const unsigned short* qr = q + ((long)row * H + (live ? head : 0)) * R +
+                               rhalf * (QS * 32) + g * 8;
+#pragma unroll
+    for (int s = 0; s < QS; ++s) {
+      s16x8 v = *reinterpret_cast<const s16x8*>(qr + s * 32);
+      if (!live) v = (s16x8)(short)0;
+      qf[s] = __builtin_bit_cast(bf16x8, v);
+    }
+  }
+
+  float m = -1e30f, l = 0.f;
+  f32x4 acc[OB];
+#pragma unroll
+  for (int i = 0; i < OB; ++i) acc[i] = {0.f, 0.f, 0.f, 0.f};
+  const float scale2 = scale * LOG2E;
+  float* scores = reinterpret_cast<float*>(smem + SC) +
+                  hgrp * (RSPLIT * 16 * SROW) + i16 * SROW;
+
   for (int t = ts; t < te; ++t) {
     __syncthreads();  // every wave is done with the previous tile
     stage();
@@ -152,24 +161,43 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
     }
     __syncthreads();
 
-    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
+    // scores of my keys over my columns, in two chains
+    f32x4 sa[2];
+    sa[0] = {0.f, 0.f, 0.f, 0.f};
+    sa[1] = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int s = 0; s < R / 32; ++s) {
-      const char* a =
-          smem + i16 * (R * 2) + (((s * 4 + g) ^ (i16 & SW)) * 16);
+    for (int s = 0; s < QS; ++s) {
+      const int chunk = (rhalf * QS + s) * 4 + g;
+      const char* a = smem + (khalf * 16 + i16) * (R * 2) +
+                      ((chunk ^ (i16 & SW)) * 16);
       const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(a);
-      const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(a + 16 * R * 2);
-      s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, qf[s], s0, 0, 0, 0);
-      s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, qf[s], s1, 0, 0, 0);
+      sa[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+          k0, qf[s], sa[s & 1], 0, 0, 0);
     }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) sa[0][r] += sa[1][r];
+    *reinterpret_cast<f32x4*>(scores + rhalf * (16 * SROW) + khalf * 16 +
+                              g * 4) = sa[0];
+    __syncthreads();
+
+    // weights of all 32 keys for my head: lane group g has keys g*8 .. + 7
     float p[8];
     float pmax = -INFINITY;
 #pragma unroll
-    for (int i = 0; i < 8; ++i) {
-      const int key = t * KT + (i >> 2) * 16 + g * 4 + (i & 3);
-      const float s = (i < 4 ? s0[i & 3] : s1[i & 3]) * scale2;
-      p[i] = key >= lo && key < L ? s : -INFINITY;
-      pmax = fmaxf(pmax, p[i]);
+    for (int h = 0; h < 2; ++h) {
+      f32x4 v = *reinterpret_cast<const f32x4*>(scores + g * 8 + h * 4);
+      if (RSPLIT == 2) {
+        const f32x4 v2 = *reinterpret_cast<const f32x4*>(
+            scores + 16 * SROW + g * 8 + h * 4);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] += v2[r];
+      }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = t * KT + g * 8 + h * 4 + r;
+        p[h * 4 + r] = key >= lo && key < L ? v[r] * scale2 : -INFINITY;
+        pmax = fmaxf(pmax, p[h * 4 + r]);
+      }
     }
     pmax = fmaxf(pmax, __shfl_xor(pmax, 16, 64));
     pmax = fmaxf(pmax, __shfl_xor(pmax, 32, 64));
@@ -179,7 +207,7 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
       m = mn;
       l *= alpha;
 #pragma unroll
-      for (int i = 0; i < R / 16; ++i)
+      for (int i = 0; i < OB; ++i)
 #pragma unroll
         for (int r = 0; r < 4; ++r) acc[i][r] *= alpha;
     }
@@ -192,9 +220,9 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
     }
     const bf16x8 pf = __builtin_bit_cast(bf16x8, pb);
 #pragma unroll
-    for (int i = 0; i < R / 16; ++i) {
+    for (int i = 0; i < OB; ++i) {
       const bf16x8 v = *reinterpret_cast<const bf16x8*>(
-          smem + CT + ct_slot(i * 16 + i16, g));
+          smem + CT + ct_slot((ks * OB + i) * 16 + i16, g));
       acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(v, pf, acc[i], 0, 0,
                                                        0);
     }
@@ -203,21 +231,22 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
   l += __shfl_xor(l, 32, 64);
   if (!live) return;
   const long rh = (long)row * H + head;
+  const int col = ks * (OB * 16) + g * 4;
   if (NS == 1) {
     const float inv = l > 0.f ? 1.f / l : 0.f;
 #pragma unroll
-    for (int i = 0; i < R / 16; ++i) {
+    for (int i = 0; i < OB; ++i) {
       s16x4 o;
 #pragma unroll
       for (int r = 0; r < 4; ++r) o[r] = (short)f2bf(acc[i][r] * inv);
-      *reinterpret_cast<s16x4*>(out + rh * R + i * 16 + g * 4) = o;
+      *reinterpret_cast<s16x4*>(out + rh * R + col + i * 16) = o;
     }
   } else {
     const long part = rh * NS + split;
 #pragma unroll
-    for (int i = 0; i < R / 16; ++i)
-      *reinterpret_cast<f32x4*>(pacc + part * R + i * 16 + g * 4) = acc[i];
-    if (g == 0) {
+    for (int i = 0; i < OB; ++i)
+      *reinterpret_cast<f32x4*>(pacc + part * R + col + i * 16) = acc[i];
+    if (g == 0 && ks == 0) {
       pml[part * 2] = m;
       pml[part * 2 + 1] = l;
     }
@@ -257,8 +286,9 @@ latent_combine_kernel(const float* __restrict__ pacc,
   }
 }
 
-extern "C" int latent_decode_waves(int H) {
-  return H <= 16 ? 1 : H <= 32 ? 2 : 4;
+// heads that one workgroup serves
+extern "C" int latent_decode_heads(int H) {
+  return H <= 16 ? 16 : H <= 32 ? 32 : 64;
 }
 
 extern "C" bool latent_decode_covers(int R) {
@@ -270,20 +300,22 @@ extern "C" void launch_latent_decode(
     const int* row_seq, const int* ctx, void* out, void* pacc, void* pml,
     int M, int H, int R, int NS, int max_blocks, int window, float scale,
     hipStream_t stream) {
-  const int nw = latent_decode_waves(H);
-  const int hg = (H + 16 * nw - 1) / (16 * nw);
-  const int lds = KT * R * 2 + R * 72;
-#define LD(RR, NW)                                                            \
-  hipLaunchKernelGGL((latent_decode_kernel<RR, NW>), dim3(M * hg * NS),       \
-                     dim3(64 * NW), lds, stream, (const unsigned short*)q,    \
+  const int heads = latent_decode_heads(H);
+  const int ng = (H + heads - 1) / heads;
+#define LD(RR, HG, KS)                                                        \
+  hipLaunchKernelGGL((latent_decode_kernel<RR, HG, KS>), dim3(M * ng * NS),   \
+                     dim3(64 * HG * KS),                                      \
+                     KT * RR * 2 + RR * 72 +                                  \
+                         HG * (KS == 4 ? 2 : 1) * 16 * SROW * 4,              \
+                     stream, (const unsigned short*)q,                        \
                      (const unsigned short*)cache, block_table, row_seq, ctx, \
-                     (unsigned short*)out, (float*)pacc, (float*)pml, H, hg,  \
+                     (unsigned short*)out, (float*)pacc, (float*)pml, H, ng,  \
                      NS, max_blocks, window, scale)
-#define LD_R(RR)                   \
-  do {                             \
-    if (nw == 1) LD(RR, 1);        \
-    else if (nw == 2) LD(RR, 2);   \
-    else LD(RR, 4);                \
+#define LD_R(RR)                      \
+  do {                                \
+    if (heads == 16) LD(RR, 1, 4);    \
+    else if (heads == 32) LD(RR, 2, 2); \
+    else LD(RR, 4, 2);                \
   } while (0)
   switch (R) {
     case 64: LD_R(64); break;

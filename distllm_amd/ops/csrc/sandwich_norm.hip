@@ -10,40 +10,6 @@
 // with zeros to W columns. T is the type of y, h and E (bf16 or fp32).
 #include "common.h"
 
-template <typename T>
-__device__ __forceinline__ void load8(const T* p, float* f);
-template <>
-__device__ __forceinline__ void load8<unsigned short>(const unsigned short* p,
-                                                      float* f) {
-  bf8_to_f32(*reinterpret_cast<const s16x8*>(p), f);
-}
-template <>
-__device__ __forceinline__ void load8<float>(const float* p, float* f) {
-  const f32x4 a = *reinterpret_cast<const f32x4*>(p);
-  const f32x4 b = *reinterpret_cast<const f32x4*>(p + 4);
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    f[i] = a[i];
-    f[4 + i] = b[i];
-  }
-}
-__device__ __forceinline__ void store8(unsigned short* p, const float* f) {
-  s16x8 v;
-#pragma unroll
-  for (int i = 0; i < 8; ++i) v[i] = (short)f2bf(f[i]);
-  *reinterpret_cast<s16x8*>(p) = v;
-}
-__device__ __forceinline__ void store8(float* p, const float* f) {
-  f32x4 a, b;
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    a[i] = f[i];
-    b[i] = f[4 + i];
-  }
-  *reinterpret_cast<f32x4*>(p) = a;
-  *reinterpret_cast<f32x4*>(p + 4) = b;
-}
-
 // sum over the TPR threads (one or four waves) that share a row
 template <int TPR>
 __device__ __forceinline__ float row_sum(float v, float* scratch) {

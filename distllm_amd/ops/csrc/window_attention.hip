@@ -11,14 +11,14 @@ extern "C" void launch_attn_window(const void* Q, const void* K,
                                    int window, float scale,
                                    hipStream_t stream) {
   const int nwave = 4;
-  const int ktile = KVBLK * DK * 2, vtile = DV * VROW * 2;
+  const int ktile = KVBLK * DK * 2, vtile = DV * VROW4 * 2;
   const int stage_b = 2 * ktile + 2 * vtile + 2 * KVBLK * 4;
   const int epi_b = nwave * QWAVE * (DV + 1) * 4;
   const int lds = stage_b > epi_b ? stage_b : epi_b;
   const long tq = (long)H * DK;
 #define AWN(KK, VV)                                                           \
   hipLaunchKernelGGL(                                                         \
-      (attn_fwd_kernel<KK, true, false, (VV >= 128), true, VV, true>),        \
+      (attn_fwd_kernel<KK, true, false, false, true, VV, true>),        \
       dim3(nblocks * H), dim3(nwave * 64), lds, stream,                       \
       (const unsigned short*)Q, (const unsigned short*)K,                     \
       (const unsigned short*)V, (const float*)nullptr, (unsigned short*)O, B, \
