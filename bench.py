@@ -7,7 +7,7 @@ rank per GPU (RCCL over xGMI). One timed step = embed one batch of
 native HIP-kernel encoder forward + fused mean-pool + L2 normalize +
 async D2H into a pinned host buffer — the hot loop of the reference's
 headline config (examples/embed/AMP.nougat.pubmedbert.yaml:
-batch_size=512, maxlen 512, mean pool; BASELINE.md).
+batch_size=512, maxlen 512, mean pool).
 
 Rank 0 prints ONE JSON line with the whole-job aggregate.
 """
@@ -353,11 +353,11 @@ def bench_decoders(args) -> None:
 
 
 def bench_pipeline(args) -> None:
-    """End-to-end semantic-chunk pipeline throughput (VERDICT.md #8):
+    """End-to-end semantic-chunk pipeline throughput:
     one step = one synthetic jsonl file through
     tokenize/split/buffer -> embed buffers -> GPU distance ->
     percentile chunking -> re-embed chunks -> write shard — the
-    BASELINE config #2 wording ("semantic_chunk embedder") measured as
+    reference's wording ("semantic_chunk embedder") measured as
     a whole, host staging included. Reports docs/s and seqs/s plus a
     tokenize-vs-GPU breakdown. Single-rank (the DP story is covered by
     --mode embed)."""

@@ -142,7 +142,9 @@ def generate(
         "native", "--generator-name", "--generator_name", "-gn",
         help="native|vllm|openai_http"),
     llm_name: str = typer.Option(
-        "llama3-8b", "--llm-name", "--llm_name", "-vmn"),
+        "llama3-8b", "--llm-name", "--llm_name", "-vmn",
+        help="preset, model id, or checkpoint folder whose config.json "
+             "describes its model"),
     temperature: float = typer.Option(
         0.5, "--temperature", "-t"),
     min_p: float = typer.Option(0.1, "--min-p", "--min_p", "-mp"),

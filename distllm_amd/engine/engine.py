@@ -1,6 +1,6 @@
 """Native generation engine: paged KV cache + continuous batching +
 fused HIP sampling. Replaces the reference's vLLM dependency
-(reference generate/generators/vllm_backend.py; SURVEY.md K15).
+(reference generate/generators/vllm_backend.py).
 
 Architecture (MI355X-first):
   - a paged cache sized for the 288 GB HBM budget, in the model's own
@@ -151,7 +151,7 @@ class LLMEngine:
         # the decode step is ~300 small launches per step for a 32-layer
         # model — graph replay removes the launch overhead. ROCm 7
         # supports RCCL collectives inside graph capture, so tp>1
-        # captures the per-layer all-reduces too (VERDICT.md #6); if
+        # captures the per-layer all-reduces too; if
         # capture fails on a given stack, _graph_for falls back to
         # eager decode with a warning.
         self.use_graphs = (use_graphs if use_graphs is not None

@@ -154,7 +154,7 @@ class BertEncoder(nn.Module):
         """Varlen path for padded text batches (jsonl_chunk buffers are
         length-dispersed): valid tokens packed to [T, H], GEMMs/norms on
         packed rows, attention through the cu_seqlens flash kernel
-        (SURVEY.md §5.7; same design as the ESM packed path). Returns
+        (same design as the ESM packed path). Returns
         padded [B, S, H] with zeros at padding."""
         d = self.dims
         B, S = ids.shape

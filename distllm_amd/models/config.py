@@ -1,6 +1,6 @@
 """Model architecture configs for the native MI355X model family.
 
-Covers the reference's encoder zoo (SURVEY.md §2.3 / K1-K4) plus the
+Covers the reference's encoder zoo plus the
 decoder family used for generation (K15):
   - BERT-class bidirectional encoders (S-PubMedBERT, pubmedbert,
     bert-base) and RoBERTa-class (offset position ids)
@@ -232,7 +232,7 @@ PRESETS: dict[str, ModelDims | LayeredDims] = {
         num_heads=4, num_kv_heads=2, intermediate_size=512,
         max_position_embeddings=512,
     ),
-    # Llama-3-8B for the generate/RAG path (BASELINE config #5)
+    # Llama-3-8B for the generate/RAG path
     "llama3-8b": ModelDims(
         arch="llama", vocab_size=128256, hidden_size=4096, num_layers=32,
         num_heads=32, num_kv_heads=8, intermediate_size=14336,

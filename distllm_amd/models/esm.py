@@ -1,6 +1,6 @@
 """ESM protein-language-model encoders on the distllm-amd HIP ops.
 
-Covers the reference's protein path (SURVEY.md K3/K4; reference:
+Covers the reference's protein path (reference:
 distllm/embed/encoders/esm2.py, esmc.py — which delegated to HF
 EsmForMaskedLM / faesm flash-attn / EvolutionaryScale ESMC):
 
@@ -166,7 +166,7 @@ class Esm2Encoder(nn.Module, _RotaryMixin):
         """Varlen path for mixed-length protein batches: pack the valid
         tokens ([T, H]), run every GEMM/norm on packed rows (zero padded
         FLOPs) and attention through the cu_seqlens flash kernel
-        (SURVEY.md K3 / §5.7; reference used faesm flash-attn varlen,
+        (reference used faesm flash-attn varlen,
         distllm/embed/encoders/esm2.py:41-55). Returns padded [B,S,H]
         with zeros at padding (poolers mask them out)."""
         d = self.dims

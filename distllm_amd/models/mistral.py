@@ -6,7 +6,7 @@ One implementation serves both reference roles:
     examples/embed/leonardo-scaling/sfr-mistral.*.yaml), and
   - Llama/Mistral *causal LM* for the generate path (reference delegated
     to vLLM, generate/generators/vllm_backend.py; here: HIP paged-KV
-    decode + fused sampling, SURVEY.md K15).
+    decode + fused sampling).
 
 Pre-RMSNorm, RoPE (half-split), GQA, SwiGLU; bf16 weights, fp32 accum.
 """
@@ -28,7 +28,7 @@ class DecoderLayer(nn.Module):
     (Megatron-style sharding; all-reduce after wo and wdown). The q/k/v
     and gate/up projections live in ONE parameter each so the decode
     step issues ONE GEMM for qkv and ONE for the MLP up-path
-    (VERDICT.md #5: 7 -> 4 weight streams per layer); wq/wk/... remain
+    (7 -> 4 weight streams per layer); wq/wk/... remain
     available as row-slice views for checkpoint export and tests."""
 
     def __init__(self, d: ModelDims, tp: int = 1):

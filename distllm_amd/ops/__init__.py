@@ -577,7 +577,11 @@ def head_gemm(x, w, out=None):
             out = x.new_empty(x.shape[0], x.shape[1], w.shape[1])
         _hip_ops.head_gemm(x.contiguous(), w, out)
         return out
-    res = torch_ref.head_gemm(x, w)
+    if x.is_cuda:  # true 32-bit product
+        res = torch.bmm(x.transpose(0, 1), w.transpose(1, 2))
+        res = res.transpose(0, 1).contiguous()
+    else:
+        res = torch_ref.head_gemm(x, w)
     if out is None:
         return res
     return out.copy_(res)

@@ -1,8 +1,8 @@
 // Fused elementwise activation kernels (bf16, vectorized s16x8 loads).
 //
 // bias_gelu: y = gelu(x + bias)   (BERT/ESM FFN; reference delegated to
-//   HF transformers — SURVEY.md K1/K3 rows)
-// swiglu:    y = silu(gate) * up  (Mistral/Llama FFN; SURVEY.md K2 row)
+//   HF transformers)
+// swiglu:    y = silu(gate) * up  (Mistral/Llama FFN)
 //
 // Guide Appendix B: memory-bound; the only job is full-width vectorized
 // HBM streaming. Grid-stride, <= 2048 blocks.

@@ -1,7 +1,7 @@
 // Fused flash-attention forward for CDNA4 (gfx950), bf16 I/O, fp32 accum.
 //
-// One kernel family covers the reference's four encoder geometries
-// (SURVEY.md K1-K4/K15-prefill): bidirectional + additive key-pad mask
+// One kernel family covers the reference's four encoder geometries:
+// bidirectional + additive key-pad mask
 // (BERT/PubMedBERT, ESM2/ESMC), causal (+GQA) for Mistral/Llama prefill.
 // The reference delegated all of this to HF transformers / faesm /
 // flash-attn (reference: distllm/embed/encoders/*.py).
@@ -49,7 +49,7 @@ union frag_u {
 // [B+1]); one workgroup per (sequence, q-block, head) via the
 // host-built blk_seq/blk_qb map — the protein/fasta path with zero
 // padded FLOPs (reference: the faesm flash-attn varlen role,
-// distllm/embed/encoders/esm2.py:41-55; SURVEY.md K3, §5.7).
+// distllm/embed/encoders/esm2.py:41-55).
 //
 // WINDOW (with VARLEN and CAUSAL): the packed queries of a sequence are the
 // last ones of its packed keys (cu for queries, cu_k for keys), as when a

@@ -1,8 +1,8 @@
 // Hand-written CDNA4 MFMA GEMM: C[M,N] = A[M,K] @ B[N,K]^T (+bias, +act).
 //
 // This is the fused-epilogue GEMM for encoder FFN/projection layers
-// (reference delegated all GEMMs to HF transformers / vLLM; SURVEY.md
-// K1/K2). Plain unfused GEMMs may still go through hipBLASLt; this
+// (reference delegated all GEMMs to HF transformers / vLLM).
+// Plain unfused GEMMs may still go through hipBLASLt; this
 // kernel exists for the fused bias+GELU/SiLU paths and as the
 // MFMA/LDS-tiled evidence path.
 //

@@ -3,7 +3,7 @@
 // K-shallow flagship encoder shapes (M=262144, N in {768,2304,3072},
 // K in {768,3072}) where hipBLASLt previously owned ~52% of the
 // flagship step (reference anchor: the delegated projection GEMMs of
-// distllm/embed/encoders/auto.py:116-138; SURVEY.md K1/K2).
+// distllm/embed/encoders/auto.py:116-138).
 //
 // Structure per the guide's 256^2 8-phase template
 // (cdna_hip_programming.md §5 "The 256² 8-phase template"), own

@@ -10,7 +10,7 @@
 // and applied after the fp32 dot: dot(w_q*s, x) == s * dot(w_q, x), so
 // quantization only rounds the weights, never the accumulation.
 // Reference anchor: the vLLM latency role the reference delegated
-// (distllm/generate/generators/vllm_backend.py:62-93); VERDICT.md #5.
+// (distllm/generate/generators/vllm_backend.py:62-93).
 #include <hip/hip_fp8.h>
 
 #include "common.h"

@@ -2,7 +2,7 @@
 //
 // Replaces the LayerNorm/RMSNorm work the reference delegated to HF
 // transformers model forwards (reference: distllm/embed/encoders/auto.py
-// encode() running AutoModel; SURVEY.md K1/K2 rows).
+// encode() running AutoModel).
 //
 // Design (guide: Appendix B element-wise/reduction rules):
 //  - one WAVE per row (row = hidden vector of size H), 4 rows per 256-thread
@@ -105,8 +105,7 @@ norm_fwd_kernel(const unsigned short* __restrict__ x,
 // chunks, LDS cross-wave combine). At decode B<=8 the wave-per-row
 // kernel is a single wave doing NCL dependent 16-B load rounds
 // (~9.5us/call measured at B=1 H=4096); spreading the row across the
-// block quarters the rounds on the per-token critical path
-//
+// block quarters the rounds on the per-token critical path.
 template <int NCL, bool HAS_RES, bool WRITE_SUM, bool RMS>
 __global__ void __launch_bounds__(256)
 norm_fwd_small_kernel(const unsigned short* __restrict__ x,

@@ -1,6 +1,6 @@
 // Paged-KV decode attention (single new token per sequence), bf16.
 // Replaces vLLM's paged attention (reference delegated generation to
-// vLLM, generate/generators/vllm_backend.py; SURVEY.md K15).
+// vLLM, generate/generators/vllm_backend.py).
 //
 // Cache layout: kcache/vcache [nblocks, HKV, BLK, D] bf16, BLK=16.
 // block_table [B, max_blocks] int32 ; ctx_len [B] int32.

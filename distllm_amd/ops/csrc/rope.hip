@@ -1,6 +1,6 @@
 // RoPE (rotary position embedding) application, half-split (NeoX) style:
 //   out[..., :D/2] = x1*cos - x2*sin ; out[..., D/2:] = x2*cos + x1*sin
-// used by Mistral/Llama (SURVEY.md K2/K15) and ESM2 (K3).
+// used by Mistral/Llama and ESM2 (K3).
 //
 // cos/sin tables are HOST-precomputed f32 [S, D/2] (guide Appendix B:
 // on-device trig turns memory-bound into VALU-bound).
@@ -19,7 +19,7 @@ rope_kernel(const unsigned short* __restrict__ x,
             int Hx, int D, int rope_heads) {
   // heads >= rope_heads pass through unchanged: lets ONE launch rope
   // the q|k part of a fused qkv tensor while copying v (decode-path
-  // launch fusion, VERDICT.md #5)
+  // launch fusion)
   const int half = D / 2;
   const long stride = (long)gridDim.x * blockDim.x;
   const long total = n_rows * half;

@@ -1,4 +1,4 @@
-// Fused sampling kernel for the generation engine (SURVEY.md K15):
+// Fused sampling kernel for the generation engine:
 // temperature + min-p filter + categorical draw in one pass family,
 // plus greedy argmax. Replaces vLLM's sampler (reference
 // generate/generators/vllm_backend.py:46-60 defaults: temp=.5, min_p=.1).

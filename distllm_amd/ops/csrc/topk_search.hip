@@ -1,5 +1,5 @@
-// kNN search kernels replacing faiss-gpu (reference rag/search.py:231-399,
-// SURVEY.md K11/K12/K14): chunked radix-select top-k over a score matrix,
+// kNN search kernels replacing faiss-gpu (reference rag/search.py:231-399):
+// chunked radix-select top-k over a score matrix,
 // and packed-binary Hamming scoring for the ubinary precision path.
 //
 // Pipeline (python side, rag/search.py here):
@@ -179,7 +179,7 @@ extern "C" void launch_hamming_score(const void* qcodes, const void* codes_t,
                      (const unsigned long long*)codes_t, out, N, W);
 }
 
-// ---- batched IVF chunk scoring (approximate search) --------
+// ---- batched IVF chunk scoring (approximate search) --------------------
 // slabs: [nchunks, cap, H] f32 padded chunk slabs; probes: [Q*nprobe]
 // int32 chunk ids; qv: [Q, H] f32; out: [Q*nprobe*cap] f32 (-inf at
 // pad rows). One block per (query, probe): the query vector is staged

@@ -1,6 +1,5 @@
 """Semantic search: GPU-resident flat index + retriever, replacing
-faiss-gpu entirely (reference distllm/rag/search.py:59-928; SURVEY.md
-K11/K12/K14).
+faiss-gpu entirely (reference distllm/rag/search.py:59-928).
 
 Design (MI355X-first): the corpus embedding matrix lives in HBM
 (288 GB/GPU holds ~17B fp32x4 dims); exact inner-product search is a
@@ -204,7 +203,7 @@ class HipFlatIndex:
         per-query host loop) and top-ks over the padded candidate
         matrix. Replaces the reference's faiss HNSW approximate option
         (rag/search.py:237,245) with a design sized for 10M+ corpora
-        resident in 288 GB HBM (VERDICT.md #7)."""
+        resident in 288 GB HBM."""
         C = self.nlist or max(int(self.n ** 0.5), 1)
         C = min(C, self.n)
         dev = self.corpus.device
@@ -268,7 +267,7 @@ class HipFlatIndex:
     def _topk_ivf(self, q: torch.Tensor, k: int):
         """Batched IVF search: score ALL (query, probe) chunks in one
         kernel launch (GPU: ivf_score HIP kernel; CPU: one bmm), then a
-        single padded top-k. No per-query host loop (VERDICT.md #7)."""
+        single padded top-k. No per-query host loop."""
         Q = q.shape[0]
         nprobe = min(self.nprobe, self.ivf_nchunks)
         cscores = q @ self.ivf_centroids.t()

@@ -2,7 +2,7 @@
 with the HIP encoder, merge the shards, then run the native generate
 pass over the merged dataset — the reference's primary pipeline
 (distributed_embedding -> merge -> distributed_generation) end-to-end
-via `distllm` commands (reference: distllm/cli.py + SURVEY.md §3.1/3.2).
+via `distllm` commands (reference: distllm/cli.py).
 Small models (bert-tiny / llama-tiny, random weights) keep it fast; the
 point is that the CLI surface drives the HIP compute path."""
 

@@ -1,5 +1,4 @@
-"""CPU end-to-end tests of the embed pipeline (reference call stack
-SURVEY.md §3.1) on tiny fixtures — no GPU required."""
+"""CPU end-to-end tests of the embed pipeline on tiny fixtures — no GPU required."""
 
 import json
 

@@ -1,4 +1,4 @@
-"""Defaults-hygiene and ADVICE-fix regression tests (round 2).
+"""Defaults-hygiene regression tests.
 
 Covers: HashWordTokenizer opt-in gating, ubinary recall warning,
 huggingface-alias decoding defaults, IVF -1 index filtering, beam

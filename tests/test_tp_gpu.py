@@ -1,7 +1,7 @@
 """tp=2 on real GPUs over RCCL, with hipGraph-captured decode
 (collectives in-graph). Runs whenever >=2 GPUs are visible; skipped on
 1-GPU boxes (the driver's round-end tier is 1-GPU — the 8-GPU scaling
-tier exercises this). VERDICT.md #6."""
+tier exercises this)."""
 
 import os
 import subprocess

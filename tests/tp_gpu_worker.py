@@ -2,7 +2,7 @@
 Run under torchrun by tests/test_tp_gpu.py when >=2 GPUs are visible.
 
 Verifies: (1) tp=2 greedy decode THROUGH THE ENGINE (hipGraph capture
-with the per-layer RCCL all-reduces IN-GRAPH, VERDICT.md #6) produces
+with the per-layer RCCL all-reduces IN-GRAPH) produces
 the same tokens as a single-GPU tp=1 engine with the same weights;
 (2) both ranks agree.
 """
