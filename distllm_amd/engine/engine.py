@@ -4,7 +4,8 @@ fused HIP sampling. Replaces the reference's vLLM dependency
 
 Architecture (MI355X-first):
   - a paged cache sized for the 288 GB HBM budget, in the model's own
-    layout (per-layer K/V pages, or pages of latents);
+    layout (per-layer K/V pages, or pages of latents), and state slots,
+    one per running sequence, for models with recurrent layers;
   - prefill: batched padded forward through the flash-attention prefill
     kernel, K/V scattered into the paged cache; models that run ragged
     step batches (engine/step.py) take prompts in portions instead, in
@@ -51,6 +52,7 @@ class _Seq:
     # per-sequence token budget; None -> the batch SamplingParams cap
     max_tokens: int | None = None
     cached: int = 0  # leading tokens whose cache entries are written
+    slot: int | None = None  # recurrent state, where the model has one
 
     @property
     def length(self) -> int:
@@ -91,6 +93,22 @@ class BlockManager:
         return (n_tokens + self.blk - 1) // self.blk
 
 
+class SlotManager:
+    """State slots of the running sequences. Slot 0 is reserved as the
+    target of padded graph rows."""
+
+    def __init__(self, num_slots: int):
+        self.free: list[int] = list(range(1, num_slots))
+
+    def alloc(self) -> int:
+        if not self.free:
+            raise RuntimeError("state slots exhausted")
+        return self.free.pop(0)
+
+    def release(self, slot: int) -> None:
+        self.free.append(slot)
+
+
 class LLMEngine:
     BLK = 16
     # prompt tokens that a ragged step takes on at most
@@ -128,14 +146,20 @@ class LLMEngine:
         if kv_cache_dtype not in ("bf16", "fp8_e4m3"):
             raise ValueError(f"kv_cache_dtype {kv_cache_dtype!r}")
         self.kv_cache_dtype = kv_cache_dtype
+        # recurrent state: a slot per running sequence and the reserved one
+        slot_bytes = model.state_bytes_per_slot()
+        self.slotman = (SlotManager(max_batch_size + 1) if slot_bytes
+                        else None)
+        num_slots = max_batch_size + 1 if slot_bytes else 0
         if num_blocks is None:
             if str(dev).startswith("cuda"):
                 free, _total = torch.cuda.mem_get_info(dev)
                 budget = int(free * kv_memory_fraction)
             else:
                 budget = 64 << 20  # CPU tests: 64 MiB
-            num_blocks = max(budget // model.cache_bytes_per_block(
-                self.BLK, kv_cache_dtype), 16)
+            budget = max(budget - num_slots * slot_bytes, 0)
+            per_block = model.cache_bytes_per_block(self.BLK, kv_cache_dtype)
+            num_blocks = max(budget // max(per_block, 1), 16)
             # cap: enough for max_batch_size * max_model_len
             need = (self.max_model_len // self.BLK + 1) * max_batch_size
             num_blocks = min(num_blocks, need)
@@ -143,7 +167,8 @@ class LLMEngine:
         self.num_blocks = num_blocks
         if kv_cache_dtype == "fp8_e4m3" and not str(dev).startswith("cuda"):
             raise ValueError("fp8_e4m3 KV cache requires a GPU")
-        self.cache = model.make_cache(num_blocks, self.BLK, kv_cache_dtype)
+        self.cache = model.make_cache(num_blocks, self.BLK, kv_cache_dtype,
+                                      num_slots)
         self.ragged = model.ragged
         self.blockman = BlockManager(num_blocks, self.BLK)
         self._next_id = 0
@@ -277,7 +302,8 @@ class LLMEngine:
         else:
             batch = StepBatch.build(
                 [(t, s.cached, s.blocks) for s, t in work], self.BLK,
-                self.device, self.model.expand_min)
+                self.device, self.model.expand_min,
+                self._slots([s for s, _ in work]))
             hidden = self.model.forward_step(batch, self.cache)
             pick = [int(batch.rows[i][k]) for i, w in enumerate(want)
                     for k in w]
@@ -301,13 +327,27 @@ class LLMEngine:
                             - len(s.blocks)))
         if not self.blockman.can_alloc(sum(need)):
             raise RuntimeError("KV blocks exhausted")
+        if self.slotman is not None:
+            new = [s for s, _ in work if s.slot is None]
+            if len(new) > len(self.slotman.free):
+                raise RuntimeError("state slots exhausted")
+            for s in new:
+                s.slot = self.slotman.alloc()
         for (s, _), n in zip(work, need):
             if n:
                 s.blocks = s.blocks + self.blockman.alloc(n)
 
+    def _slots(self, seqs: list[_Seq]) -> list[int] | None:
+        if self.slotman is None:
+            return None
+        return [s.slot for s in seqs]
+
     def release(self, s: _Seq) -> None:
         """Give back everything a finished sequence holds."""
         self.blockman.release(s.blocks)
+        if s.slot is not None:
+            self.slotman.release(s.slot)
+            s.slot = None
         s.blocks = []
         s.cached = 0
 
@@ -415,11 +455,15 @@ class LLMEngine:
         runner = None
         if self.use_graphs:
             runner = self._graph_for_or_eager(len(seqs))
+        state = ()
+        if self.slotman is not None:
+            state = (torch.tensor(self._slots(seqs), dtype=torch.int32,
+                                  device=self.device),)
         if runner is not None:
             bt = self._block_table(seqs, width=self.max_blocks_per_seq)
-            return runner.run(tokens, bt, ctx)[: len(seqs)]
+            return runner.run(tokens, bt, ctx, *state)[: len(seqs)]
         return self.model.decode_step(tokens, self.cache,
-                                      self._block_table(seqs), ctx)
+                                      self._block_table(seqs), ctx, *state)
 
     def _sample_and_append(self, seqs, logits, params, results):
         dev = self.device
@@ -495,9 +539,9 @@ class LLMEngine:
 class _GraphRunner:
     """One hipGraph-captured decode step at a fixed batch size.
 
-    Static input/output tensors; padded slots point at the reserved
-    dummy KV block 0 with ctx_len=1, so their cache writes and reads are
-    harmless. Capture follows the torch.cuda.graph protocol (side-stream
+    Static input/output tensors; padded rows point at the reserved
+    dummy KV block 0 (and state slot 0) with ctx_len=1, so their cache
+    writes and reads are harmless. Capture follows the torch.cuda.graph protocol (side-stream
     warmup, then capture); replay removes the ~10 launches/layer CPU
     overhead that dominates small-batch decode.
     """
@@ -524,13 +568,16 @@ class _GraphRunner:
         self.bt = torch.zeros(batch, engine.max_blocks_per_seq,
                               dtype=torch.int32, device=dev)
         self.ctx = torch.ones(batch, dtype=torch.int32, device=dev)
+        self.state = ()
+        if engine.slotman is not None:
+            self.state = (torch.zeros(batch, dtype=torch.int32, device=dev),)
         torch.cuda.synchronize()
         side = torch.cuda.Stream()
         side.wait_stream(torch.cuda.current_stream())
         with torch.cuda.stream(side):
             for _ in range(2):  # warmup allocations/paths
                 engine.model.decode_step(self.tokens, engine.cache,
-                                         self.bt, self.ctx)
+                                         self.bt, self.ctx, *self.state)
         torch.cuda.current_stream().wait_stream(side)
         torch.cuda.synchronize()
         self.graph = torch.cuda.CUDAGraph()
@@ -543,13 +590,14 @@ class _GraphRunner:
         try:
             with torch.cuda.graph(self.graph):
                 self.logits = engine.model.decode_step(
-                    self.tokens, engine.cache, self.bt, self.ctx)
+                    self.tokens, engine.cache, self.bt, self.ctx,
+                    *self.state)
         finally:
             if enabled:
                 gc.enable()
 
     def run(self, tokens: torch.Tensor, bt: torch.Tensor,
-            ctx: torch.Tensor) -> torch.Tensor:
+            ctx: torch.Tensor, *state: torch.Tensor) -> torch.Tensor:
         n = tokens.shape[0]
         self.tokens[:n] = tokens
         if n < self.batch:
@@ -560,5 +608,8 @@ class _GraphRunner:
         self.ctx[:n] = ctx
         if n < self.batch:
             self.ctx[n:] = 1
+        for own, new in zip(self.state, state):
+            own[:n] = new
+            own[n:] = 0
         self.graph.replay()
         return self.logits

@@ -119,7 +119,7 @@ class EngineLoop:
                     eng._start(seqs, params, results)
                 except Exception as e:
                     for r in admitted:
-                        eng.blockman.release(r.seq.blocks)
+                        eng.release(r.seq)
                         self._finish(r, None, e)
                     admitted = []
                 self._running.extend(r for r in admitted)
@@ -131,8 +131,7 @@ class EngineLoop:
                 if done:
                     out = results.pop(r.seq.seq_id, r.seq.out_ids)
                     if not r.seq.done:  # hit per-request cap
-                        eng.blockman.release(r.seq.blocks)
-                        r.seq.blocks = []
+                        eng.release(r.seq)
                     self._finish(r, out)
                 else:
                     still.append(r)
@@ -149,7 +148,7 @@ class EngineLoop:
                              results)
             except Exception as e:
                 for r in self._running:
-                    eng.blockman.release(r.seq.blocks)
+                    eng.release(r.seq)
                     self._finish(r, None, e)
                 self._running = []
 

@@ -8,6 +8,11 @@ rows, attended one by one against the paged cache); longer portions
 follow and are attended by the packed flash kernel. The row count is
 rounded up so that products see few distinct shapes; padding rows have
 ctx 0 and touch nothing.
+
+Models with a recurrent state also get each sequence's state slot and
+where its rows are: the rows of a sequence are consecutive and in order.
+A sequence that starts in the step (ctx 1) starts from a zero state,
+whatever its slot holds.
 """
 
 from __future__ import annotations
@@ -41,6 +46,27 @@ class Expansion:
 
 
 @dataclass
+class PromptBlocks:
+    """Query blocks of the expanded portions for attention over paged keys
+    and values: blocks[i] = (portion, block of QBLK queries)."""
+
+    portions: torch.Tensor   # [P, 4] table row, first row, first pos, rows
+    blocks: torch.Tensor     # [N, 2]
+
+    QBLK = 128
+
+
+@dataclass
+class Segments:
+    """Rows of each block-table row, and its state slot."""
+
+    row0: torch.Tensor       # [S] int32
+    rows: torch.Tensor       # [S] int32
+    slot: torch.Tensor       # [S] int32
+    longest: int
+
+
+@dataclass
 class StepBatch:
     tokens: torch.Tensor       # [M] int64
     ctx: torch.Tensor          # [M] int32, position + 1; 0 = padding
@@ -51,22 +77,27 @@ class StepBatch:
     rows: list[np.ndarray] = field(default_factory=list)
     # expanded portions: (block-table row, first position, new tokens)
     portions: list[tuple[int, int, int]] = field(default_factory=list)
+    segments: Segments | None = None  # with state slots
     _expansions: dict[int, Expansion] = field(default_factory=dict)
+    _prompts: dict[int, PromptBlocks] = field(default_factory=dict)
 
     @classmethod
-    def decode(cls, tokens, block_table, ctx) -> "StepBatch":
+    def decode(cls, tokens, block_table, ctx, slots=None) -> "StepBatch":
         """One token per sequence, everything already on the device."""
         n = tokens.shape[0]
-        return cls(tokens=tokens.long(), ctx=ctx.int(),
-                   row_seq=torch.arange(n, dtype=torch.int32,
-                                        device=tokens.device),
-                   block_table=block_table.int(), n_folded=n)
+        each = torch.arange(n, dtype=torch.int32, device=tokens.device)
+        seg = None
+        if slots is not None:
+            seg = Segments(each, torch.ones_like(each), slots.int(), 1)
+        return cls(tokens=tokens.long(), ctx=ctx.int(), row_seq=each,
+                   block_table=block_table.int(), n_folded=n, segments=seg)
 
     @classmethod
     def build(cls, entries, blk: int, device,
-              expand_min: int = 32) -> "StepBatch":
+              expand_min: int = 32, slots=None) -> "StepBatch":
         """entries: (new tokens, tokens already cached, cache blocks).
-        Portions of at least expand_min tokens are expanded."""
+        Portions of at least expand_min tokens are expanded. slots: the
+        entries' state slots, for models that have a state."""
         order = sorted(range(len(entries)),
                        key=lambda i: len(entries[i][0]) >= expand_min)
         total = sum(len(t) for t, _, _ in entries)
@@ -98,10 +129,43 @@ class StepBatch:
         def up(a):
             return torch.from_numpy(a).to(device)
 
+        seg = None
+        if slots is not None:
+            seg = Segments(up(np.array([r[0] if len(r) else 0 for r in rows],
+                                       np.int32)),
+                           up(np.array([len(r) for r in rows], np.int32)),
+                           up(np.array(slots, np.int32)),
+                           max((len(r) for r in rows), default=0))
+
         return cls(tokens=up(tokens), ctx=up(ctx), row_seq=up(row_seq),
                    block_table=up(table),
                    n_folded=n_folded if portions else M, rows=rows,
-                   portions=portions)
+                   portions=portions, segments=seg)
+
+    def prompt_blocks(self, chunk: int) -> PromptBlocks:
+        """Query blocks of the expanded portions, those that see most keys
+        (in chunks of `chunk` positions) first: they would otherwise be
+        the tail of the launch."""
+        p = self._prompts.get(chunk)
+        if p is not None:
+            return p
+        dev, Q = self.tokens.device, PromptBlocks.QBLK
+        meta, blocks, keys = [], [], []
+        at = self.n_folded
+        for i, (s, start, n) in enumerate(self.portions):
+            meta.append((s, at, start, n))
+            at += n
+            for b in range((n + Q - 1) // Q):
+                blocks.append((i, b))
+                first = start + b * Q
+                keys.append(min(first + Q, start + n)
+                            - first // chunk * chunk)
+        order = np.argsort(-np.array(keys), kind="stable")
+        p = PromptBlocks(
+            torch.tensor(meta, dtype=torch.int32).to(dev),
+            torch.from_numpy(np.array(blocks, np.int32)[order]).to(dev))
+        self._prompts[chunk] = p
+        return p
 
     def expansion(self, window: int) -> Expansion:
         """Key map of the expanded portions under a window: each

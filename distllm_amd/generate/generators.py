@@ -91,14 +91,14 @@ class NativeGenerator:
         from ..embed.encoders import resolve_model
         from ..embed.tokenizers import load_tokenizer
         from ..engine import LLMEngine, SamplingParams
-        from ..models import build_model
+        from ..models import LayeredDims, build_model
 
         self.config = config
         dims, folder = resolve_model(config.model)
         device = "cuda" if torch.cuda.is_available() else "cpu"
         dtype = torch.bfloat16 if device != "cpu" else torch.float32
-        if config.dtype == "float32" and dims.arch == "kanotar":
-            dtype = torch.float32  # its kernels run in 32-bit as well
+        if config.dtype == "float32" and isinstance(dims, LayeredDims):
+            dtype = torch.float32  # their kernels run in 32-bit as well
         kw = {}
         if config.tensor_parallel_size > 1:
             import torch.distributed as dist

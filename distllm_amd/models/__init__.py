@@ -5,6 +5,7 @@ from __future__ import annotations
 import torch
 
 from .bert import BertEncoder
+from .bufulorn import BufulornModel
 from .config import (PRESETS, LayeredDims, ModelDims, dims_from_checkpoint,
                      get_dims)
 from .esm import Esm2Encoder, EsmCEncoder
@@ -13,6 +14,7 @@ from .mistral import DecoderModel
 
 __all__ = [
     "BertEncoder",
+    "BufulornModel",
     "DecoderModel",
     "Esm2Encoder",
     "EsmCEncoder",
@@ -25,6 +27,10 @@ __all__ = [
     "get_dims",
     "load_pretrained",
 ]
+
+
+# decoders that are described layer by layer
+LAYERED = {"kanotar": KanotarModel, "bufulorn": BufulornModel}
 
 
 def build_model(name_or_dims: str | ModelDims | LayeredDims, device: str | None = None,
@@ -42,10 +48,10 @@ def build_model(name_or_dims: str | ModelDims | LayeredDims, device: str | None 
         m = EsmCEncoder(dims, dtype=dtype, **kw)
     elif dims.arch in ("mistral", "llama", "qwen2"):
         m = DecoderModel(dims, dtype=dtype, **kw)
-    elif dims.arch == "kanotar":
+    elif dims.arch in LAYERED:
         # parameters are made where they stay: no host copy of the model
         with torch.device(device or "cpu"):
-            m = KanotarModel(dims, dtype=dtype, **kw)
+            m = LAYERED[dims.arch](dims, dtype=dtype, **kw)
     else:
         raise ValueError(f"unknown arch {dims.arch}")
     if device is not None:

@@ -1,11 +1,15 @@
-"""Mixers and feed-forwards of decoders that are described layer by layer.
+"""Parts of decoders that are described layer by layer: what mixers and
+feed-forwards have in common, and the latent-attention family.
 
-A mixer maps the normed rows of a ragged step batch (engine/step.py) to
-the sublayer's output and owns what it keeps in the cache. Sizes of the
+A mixer maps the rows of a ragged step batch (engine/step.py) to the
+sublayer's output and says what it keeps in the cache. Sizes of the
 parameters are rounded up to multiples of 64 with zeros, so that the
 16-byte loads and MFMA tiles of the kernels never see a partial row; the
 zeros leave every product and (with the true sizes passed along) every
-norm unchanged. `load` takes the checkpoint's unpadded tensors.
+norm unchanged.
+
+`tensors` names a part's checkpoint tensors with their (unpadded) shapes,
+`checkpoint` maps them to the padded parameters.
 """
 
 from __future__ import annotations
@@ -58,7 +62,7 @@ def expect(name: str, w: torch.Tensor, *shape: int) -> torch.Tensor:
     return w
 
 
-def _weight(rows: int, cols: int, dtype) -> nn.Parameter:
+def weight(rows: int, cols: int, dtype) -> nn.Parameter:
     return nn.Parameter(torch.empty(rows, cols, dtype=dtype))
 
 
@@ -67,7 +71,41 @@ def norm_weight(n: int) -> nn.Parameter:
     return nn.Parameter(torch.empty(n, dtype=torch.float32))
 
 
-class LatentAttention(nn.Module):
+class Part(nn.Module):
+    """A mixer or feed-forward."""
+
+    # a mixer that reads another layer's cache has none of its own
+    own = True
+    kv_from: int | None = None
+
+    def tensors(self) -> dict[str, tuple[int, ...]]:
+        """Checkpoint tensor name (within the part) -> its shape."""
+        raise NotImplementedError
+
+    def checkpoint(self, src: dict, pre: str) -> dict[str, torch.Tensor]:
+        """Own parameter name -> padded tensor, from a raw checkpoint
+        (`checked` has seen to the shapes)."""
+        raise NotImplementedError
+
+    def checked(self, src: dict, pre: str) -> dict[str, torch.Tensor]:
+        return {n: expect(pre + n, src[pre + n], *shape)
+                for n, shape in self.tensors().items()}
+
+    def cache_numel(self) -> int:
+        """Numbers that a token keeps in the paged cache."""
+        return 0
+
+    def state_numel(self) -> tuple[int, int]:
+        """Numbers of a state slot: in fp32, in the model's dtype."""
+        return 0, 0
+
+    def make_cache(self, num_blocks: int, blk: int, num_slots: int, dtype,
+                   device):
+        """What the layer keeps between steps."""
+        return None
+
+
+class LatentAttention(Part):
     """Latent attention with a sliding window, on paged latents.
 
     Two forms of the same function:
@@ -89,41 +127,52 @@ class LatentAttention(nn.Module):
         self.own = d.kv_from is None
         H = d.heads
         # one product for both down-projections of a layer
-        self.wdown = _weight(self.qp + (self.rp if self.own else 0),
+        self.wdown = weight(self.qp + (self.rp if self.own else 0),
                              self.wp, dtype)
         self.q_norm = norm_weight(self.qp)
         self.kv_norm = norm_weight(self.rp) if self.own else None
-        self.wuq = _weight(H * self.dp, self.qp, dtype)
+        self.wuq = weight(H * self.dp, self.qp, dtype)
         # all heads' key rows, then all heads' value rows
-        self.wukv = _weight(H * (self.dp + self.vp), self.rp, dtype)
-        self.wo = _weight(self.wp, H * self.vp, dtype)
+        self.wukv = weight(H * (self.dp + self.vp), self.rp, dtype)
+        self.wo = weight(self.wp, H * self.vp, dtype)
         self._fold: tuple | None = None
 
-    def checkpoint(self, src: dict, pre: str) -> dict[str, torch.Tensor]:
-        """Own parameter name -> padded tensor, from a raw checkpoint."""
-        d, H = self.d, self.d.heads
+    @property
+    def kv_from(self):
+        return self.d.kv_from
 
-        def get(name, *shape):
-            return expect(pre + name, src[pre + name], *shape)
-
-        down = [padded(get("dq", d.q_rank, self.width), self.qp, self.wp)]
-        out = {"q_norm": padded(get("dq.norm", d.q_rank), self.qp)}
+    def tensors(self):
+        d, H, W = self.d, self.d.heads, self.width
+        t = {"dq": (d.q_rank, W), "dq.norm": (d.q_rank,),
+             "uq": (H * d.dim, d.q_rank)}
         if self.own:
-            down.append(padded(get("dkv", d.kv_rank, self.width),
-                               self.rp, self.wp))
-            out["kv_norm"] = padded(get("dkv.norm", d.kv_rank), self.rp)
+            t |= {"dkv": (d.kv_rank, W), "dkv.norm": (d.kv_rank,)}
+        return t | {"uk": (H * d.dim, d.kv_rank),
+                    "uv": (H * d.vdim, d.kv_rank), "o": (W, H * d.vdim)}
+
+    def checkpoint(self, src, pre):
+        d, H = self.d, self.d.heads
+        t = self.checked(src, pre)
+        down = [padded(t["dq"], self.qp, self.wp)]
+        out = {"q_norm": padded(t["dq.norm"], self.qp)}
+        if self.own:
+            down.append(padded(t["dkv"], self.rp, self.wp))
+            out["kv_norm"] = padded(t["dkv.norm"], self.rp)
         out["wdown"] = torch.cat(down)
-        out["wuq"] = padded_heads(get("uq", H * d.dim, d.q_rank), H, d.dim,
-                                  self.dp, self.qp)
+        out["wuq"] = padded_heads(t["uq"], H, d.dim, self.dp, self.qp)
         out["wukv"] = torch.cat([
-            padded_heads(get("uk", H * d.dim, d.kv_rank), H, d.dim,
-                         self.dp, self.rp),
-            padded_heads(get("uv", H * d.vdim, d.kv_rank), H, d.vdim,
-                         self.vp, self.rp)])
-        out["wo"] = padded_heads(
-            get("o", self.width, H * d.vdim).t(), H, d.vdim, self.vp,
-            self.wp).t()
+            padded_heads(t["uk"], H, d.dim, self.dp, self.rp),
+            padded_heads(t["uv"], H, d.vdim, self.vp, self.rp)])
+        out["wo"] = padded_heads(t["o"].t(), H, d.vdim, self.vp, self.wp).t()
         return out
+
+    def cache_numel(self):
+        return self.rp if self.own else 0
+
+    def make_cache(self, num_blocks, blk, num_slots, dtype, device):
+        """Paged latents [blocks, BLK, rank]."""
+        return torch.zeros(num_blocks, blk, self.rp, dtype=dtype,
+                           device=device)
 
     def _folded(self) -> tuple[torch.Tensor, torch.Tensor]:
         """(Uk^T [H, R, dim], Uv [H, vdim, R]); Uk^T is a copy, renewed
@@ -175,24 +224,24 @@ class LatentAttention(nn.Module):
         return ops.linear(o.view(M, H * self.vp), self.wo)
 
 
-class ClampedGlu(nn.Module):
+class ClampedGlu(Part):
     def __init__(self, d: ClampedGluDims, width: int, dtype):
         super().__init__()
         self.d, self.width = d, width
         self.wp, self.fp = pad64(width), pad64(d.ff)
-        self.wgup = _weight(2 * self.fp, self.wp, dtype)
-        self.wdown = _weight(self.wp, self.fp, dtype)
+        self.wgup = weight(2 * self.fp, self.wp, dtype)
+        self.wdown = weight(self.wp, self.fp, dtype)
 
-    def checkpoint(self, src: dict, pre: str) -> dict[str, torch.Tensor]:
+    def tensors(self):
         ff, W = self.d.ff, self.width
+        return {"gate": (ff, W), "up": (ff, W), "down": (W, ff)}
 
-        def get(name, *shape):
-            return expect(pre + name, src[pre + name], *shape)
-
+    def checkpoint(self, src, pre):
+        t = self.checked(src, pre)
         return {
-            "wgup": torch.cat([padded(get("gate", ff, W), self.fp, self.wp),
-                               padded(get("up", ff, W), self.fp, self.wp)]),
-            "wdown": padded(get("down", W, ff), self.wp, self.fp),
+            "wgup": torch.cat([padded(t["gate"], self.fp, self.wp),
+                               padded(t["up"], self.fp, self.wp)]),
+            "wdown": padded(t["down"], self.wp, self.fp),
         }
 
     def forward(self, h):
@@ -200,7 +249,3 @@ class ClampedGlu(nn.Module):
         return ops.linear(
             ops.gateup_clamped_glu(h, self.wgup, d.limit, d.alpha, d.shift),
             self.wdown)
-
-
-MIXERS = {"latent_attention": LatentAttention}
-MLPS = {"dense": ClampedGlu}

@@ -9,7 +9,8 @@ decoder family used for generation (K15):
   - Mistral-class decoder embedders (SFR-Embedding-Mistral)
   - Llama-class causal LMs for generation
   - Qwen2-class causal LMs (llama family + qkv bias)
-  - Kanotar causal LMs: every layer has its own description (LayeredDims)
+  - Kanotar and Bufulorn causal LMs: every layer has its own description
+    (LayeredDims)
 Dims are from the public model cards; weights are random-init here
 (no network) or loadable from local safetensors.
 """
@@ -20,7 +21,8 @@ import json
 from pathlib import Path
 from typing import Literal
 
-from pydantic import BaseModel, ConfigDict, PositiveInt, model_validator
+from pydantic import (BaseModel, ConfigDict, NonNegativeInt, PositiveFloat,
+                      PositiveInt, model_validator)
 
 
 class ModelDims(BaseModel):
@@ -72,6 +74,47 @@ class LatentAttentionDims(_Strict):
     kv_from: int | None = None  # layer whose latents this one reads
 
 
+    def shared_sizes(self) -> dict[str, int]:
+        """What a layer and the layer whose cache it reads agree on."""
+        return {"kv_rank": self.kv_rank}
+
+
+class AttentionDims(_Strict):
+    """Softmax attention on cached keys and values. Queries and keys are
+    normed per head; scores are capped at softcap * tanh and lose
+    r1 * ln(1 + r2 * distance), r1 and r2 being weights of the head; the
+    heads' outputs are gated. A token sees the earlier tokens of its own
+    chunk: positions are cut into chunks of `chunk` from position 0."""
+
+    type: Literal["attention"] = "attention"
+    heads: PositiveInt
+    kv_heads: PositiveInt
+    dim: PositiveInt           # query/key size per head
+    vdim: PositiveInt          # value size per head
+    scale: float
+    softcap: PositiveFloat
+    chunk: PositiveInt
+    kv_from: NonNegativeInt | None = None  # layer whose keys and values
+
+    def shared_sizes(self) -> dict[str, int]:
+        return {k: getattr(self, k)
+                for k in ("heads", "kv_heads", "dim", "vdim")}
+
+
+class DeltaDims(_Strict):
+    """Gated delta rule: a recurrent [dim, vdim] state per head, behind
+    short causal convolutions of `conv` taps; kv_heads queries and keys,
+    heads values."""
+
+    type: Literal["delta"] = "delta"
+    heads: PositiveInt
+    kv_heads: PositiveInt
+    dim: PositiveInt
+    vdim: PositiveInt
+    conv: PositiveInt
+    unit_eps: float = 1e-6     # of the unit queries and keys
+
+
 class ClampedGluDims(_Strict):
     """Feed-forward g * sigmoid(alpha g) * (u + shift), gate g clamped
     from above and up-projection u from both sides at `limit`."""
@@ -83,22 +126,55 @@ class ClampedGluDims(_Strict):
     shift: float = 1.0
 
 
+class XieluDims(_Strict):
+    """Feed-forward down(xielu(up)), the activation's two numbers being
+    weights of the layer."""
+
+    kind: Literal["xielu"] = "xielu"
+    ff: PositiveInt
+
+
+class ExpertsDims(_Strict):
+    """Routed gated-unit experts. Experts form `groups` equal groups of
+    neighbours; the `top` experts of the `keep` best groups serve a token,
+    weighted by their softmax scores over all experts."""
+
+    kind: Literal["experts"] = "experts"
+    ff: PositiveInt
+    experts: PositiveInt
+    top: PositiveInt
+    groups: PositiveInt = 1
+    keep: PositiveInt = 1
+
+    @model_validator(mode="after")
+    def _check_groups(self):
+        if self.experts % self.groups:
+            raise ValueError(f"{self.experts} experts do not form "
+                             f"{self.groups} equal groups")
+        if self.keep > self.groups:
+            raise ValueError(f"keep {self.keep} of {self.groups} groups")
+        if self.top > self.experts // self.groups * self.keep:
+            raise ValueError(f"top {self.top} is more than the experts of "
+                             f"{self.keep} groups")
+        return self
+
+
 class LayerDims(_Strict):
-    mixer: LatentAttentionDims
-    mlp: ClampedGluDims | None = None
+    mixer: LatentAttentionDims | AttentionDims | DeltaDims
+    mlp: ClampedGluDims | XieluDims | ExpertsDims | None = None
 
 
 class LayeredDims(BaseModel):
     """A decoder whose layers are described one by one."""
 
-    arch: Literal["kanotar"]
+    arch: Literal["kanotar", "bufulorn"]
     vocab_size: PositiveInt
     hidden_size: PositiveInt
     layers: list[LayerDims]
     norm_eps: float
     logit_scale: float = 1.0
-    # no rotation and no position table: nothing in the design bounds it
-    max_position_embeddings: int = 1 << 20
+    # bounded only by a position table, where the design has one
+    max_position_embeddings: PositiveInt = 1 << 20
 
     @property
     def num_layers(self) -> int:
@@ -109,20 +185,33 @@ class LayeredDims(BaseModel):
         if not self.layers:
             raise ValueError("a model needs at least one layer")
         for i, layer in enumerate(self.layers):
-            j = layer.mixer.kv_from
+            m = layer.mixer
+            if not isinstance(m, LatentAttentionDims) \
+                    and m.heads % m.kv_heads:
+                raise ValueError(f"layer {i}: {m.heads} heads are not a "
+                                 f"multiple of {m.kv_heads} kv_heads")
+            j = getattr(m, "kv_from", None)
             if j is None:
                 continue
             if not 0 <= j < i:
                 raise ValueError(f"layer {i}: kv_from {j} is not an "
                                  "earlier layer")
             src = self.layers[j].mixer
-            if src.kv_from is not None:
-                raise ValueError(f"layer {i}: kv_from {j} has no latent "
-                                 "of its own")
-            if src.kv_rank != layer.mixer.kv_rank:
-                raise ValueError(f"layer {i}: kv_rank differs from that "
-                                 f"of layer {j}")
+            if type(src) is not type(m) or src.kv_from is not None:
+                raise ValueError(f"layer {i}: kv_from {j} has no keys and "
+                                 "values of its own")
+            for k, v in m.shared_sizes().items():
+                if src.shared_sizes()[k] != v:
+                    raise ValueError(f"layer {i}: {k} differs from that "
+                                     f"of layer {j}")
         return self
+
+
+def _take(d: dict, name: str, where: str):
+    """The only entry of a nested description."""
+    if name not in d or len(d) != 1:
+        raise ValueError(f"{where} has keys {sorted(d)}, expected {name}")
+    return d[name]
 
 
 def _kanotar_dims(cfg: dict) -> LayeredDims:
@@ -131,20 +220,59 @@ def _kanotar_dims(cfg: dict) -> LayeredDims:
         if entry["type"] != "latent_attention":
             raise ValueError(f"layer {i}: unknown mixer {entry['type']!r}")
         mixer = dict(entry["mixer"])
-        mask = dict(mixer.pop("mask"))
-        mixer["window"] = mask.pop("size")
-        if mask:
-            raise ValueError(f"layer {i}: unknown mask keys {sorted(mask)}")
-        layers.append(LayerDims(mixer=LatentAttentionDims(**mixer),
-                                mlp=entry.get("mlp")))
+        mixer["window"] = _take(mixer.pop("mask"), "size", f"layer {i}: mask")
+        mlp = entry.get("mlp")
+        layers.append(LayerDims(
+            mixer=LatentAttentionDims(**mixer),
+            mlp=None if mlp is None else ClampedGluDims(**mlp)))
     return LayeredDims(arch="kanotar", vocab_size=cfg["vocab"],
                        hidden_size=cfg["width"], layers=layers,
                        norm_eps=cfg["norm"]["eps"],
                        logit_scale=cfg["logit_scale"])
 
 
+def _bufulorn_mlp(mlp: dict, where: str):
+    mlp = dict(mlp)
+    kind = mlp.pop("kind", None)
+    if kind == "dense":
+        return XieluDims(**mlp)
+    if kind != "moe":
+        raise ValueError(f"{where}: unknown feed-forward kind {kind!r}")
+    router = dict(mlp.pop("router"))
+    groups = dict(router.pop("groups"))
+    dims = ExpertsDims(ff=_take(mlp.pop("expert"), "ff", f"{where}: expert"),
+                       groups=groups.pop("count"), keep=groups.pop("keep"),
+                       **router)
+    if mlp or groups:
+        raise ValueError(f"{where}: unknown feed-forward keys "
+                         f"{sorted({**mlp, **groups})}")
+    return dims
+
+
+def _bufulorn_dims(cfg: dict) -> LayeredDims:
+    layers = []
+    for i, entry in enumerate(cfg["layers"]):
+        mixer = dict(entry["mixer"])
+        if entry["type"] == "attention":
+            mixer["chunk"] = _take(mixer.pop("mask"), "size",
+                                   f"layer {i}: mask")
+            mixer = AttentionDims(**mixer)
+        elif entry["type"] == "delta":
+            mixer = DeltaDims(**mixer)
+        else:
+            raise ValueError(f"layer {i}: unknown mixer {entry['type']!r}")
+        mlp = entry.get("mlp")
+        layers.append(LayerDims(
+            mixer=mixer,
+            mlp=None if mlp is None else _bufulorn_mlp(mlp, f"layer {i}")))
+    return LayeredDims(arch="bufulorn", vocab_size=cfg["vocab"],
+                       hidden_size=cfg["width"], layers=layers,
+                       norm_eps=cfg["norm"]["eps"],
+                       max_position_embeddings=cfg["max_positions"])
+
+
 # config.json "architecture" -> reader of the rest of the file
-CONFIG_READERS = {"Kanotar": _kanotar_dims}
+CONFIG_READERS = {"Kanotar": _kanotar_dims, "Bufulorn": _bufulorn_dims}
 
 
 def dims_from_checkpoint(path: str | Path) -> LayeredDims | None:
@@ -177,6 +305,36 @@ def layered_preset(num_layers: int, hidden: int, vocab: int, heads: int,
             mlp=ClampedGluDims(ff=ff, limit=limit)))
     return LayeredDims(arch="kanotar", vocab_size=vocab, hidden_size=hidden,
                        layers=layers, norm_eps=eps, logit_scale=logit_scale)
+
+
+def hybrid_preset(num_layers: int, hidden: int, vocab: int, heads: int,
+                  kv_heads: int, dim: int, ff: int, chunk: int,
+                  experts: ExpertsDims | None = None,
+                  order: str = "AD", share: bool = False,
+                  delta_dim: int | None = None, conv: int = 4,
+                  max_positions: int = 16384,
+                  eps: float = 1e-5) -> LayeredDims:
+    """Bufulorn dims of repeated layers: mixers follow `order` (A attention,
+    D delta rule), every other feed-forward is `experts` where given. With
+    `share`, every other attention layer reads the keys and values of the
+    one before."""
+    layers, owner = [], None
+    for i in range(num_layers):
+        if order[i % len(order)] == "A":
+            mixer = AttentionDims(
+                heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim,
+                scale=dim ** -0.5, softcap=30.0, chunk=chunk,
+                kv_from=owner if share else None)
+            owner = i if owner is None else None
+        else:
+            mixer = DeltaDims(heads=heads, kv_heads=kv_heads,
+                              dim=delta_dim or dim, vdim=dim, conv=conv)
+        dense = experts is None or i % 2 == 0
+        layers.append(LayerDims(
+            mixer=mixer, mlp=XieluDims(ff=ff) if dense else experts))
+    return LayeredDims(arch="bufulorn", vocab_size=vocab, hidden_size=hidden,
+                       layers=layers, norm_eps=eps,
+                       max_position_embeddings=max_positions)
 
 
 PRESETS: dict[str, ModelDims | LayeredDims] = {
@@ -272,6 +430,18 @@ PRESETS: dict[str, ModelDims | LayeredDims] = {
     "kanotar-tiny": layered_preset(
         3, 256, 1024, heads=4, dim=32, vdim=32, q_rank=64, kv_rank=64,
         ff=512, windows=[48, 32], share_from=2,
+    ),
+    # attention and delta-rule layers of the llama3-8b size, every other
+    # feed-forward routed
+    "bufulorn-8b": hybrid_preset(
+        32, 4096, 128256, heads=32, kv_heads=8, dim=128, ff=14336,
+        chunk=8192, experts=ExpertsDims(ff=1792, experts=32, top=4,
+                                        groups=4, keep=2),
+    ),
+    "bufulorn-tiny": hybrid_preset(
+        4, 256, 1024, heads=4, kv_heads=2, dim=32, ff=512, chunk=48,
+        experts=ExpertsDims(ff=64, experts=6, top=2, groups=3, keep=2),
+        order="AAD", share=True, max_positions=512,
     ),
 }
 

@@ -1,0 +1,86 @@
+"""Feed-forwards: xIELU and routed gated-unit experts."""
+
+from __future__ import annotations
+
+import torch
+from torch import nn
+
+from .. import ops
+from .blocks import Part, pad64, padded, weight
+from .config import ExpertsDims, XieluDims
+
+
+class XieluMlp(Part):
+    """down(xielu(up h)); the activation's two numbers stay on the device,
+    where the kernels read them."""
+
+    def __init__(self, d: XieluDims, width: int, dtype):
+        super().__init__()
+        self.d, self.width = d, width
+        self.wp, self.fp = pad64(width), pad64(d.ff)
+        self.wup = weight(self.fp, self.wp, dtype)
+        self.wdown = weight(self.wp, self.fp, dtype)
+        self.act = nn.Parameter(torch.empty(2, dtype=torch.float32))
+
+    def tensors(self):
+        ff, W = self.d.ff, self.width
+        return {"up": (ff, W), "down": (W, ff), "act": (2,)}
+
+    def checkpoint(self, src, pre):
+        t = self.checked(src, pre)
+        return {"wup": padded(t["up"], self.fp, self.wp),
+                "wdown": padded(t["down"], self.wp, self.fp),
+                "act": t["act"]}
+
+    def forward(self, h):
+        return ops.linear(ops.up_xielu(h, self.wup, self.act), self.wdown)
+
+
+class RoutedExperts(Part):
+    """Routed experts (ExpertsDims): rows are sorted by expert and every
+    expert's products run on its rows only. Gate and up rows of an expert
+    alternate in groups of 16, so that one tile of the product holds both
+    halves of the unit."""
+
+    UNIT = 16
+
+    def __init__(self, d: ExpertsDims, width: int, dtype):
+        super().__init__()
+        self.d, self.width = d, width
+        self.wp, self.fp = pad64(width), pad64(d.ff)
+        self.router = weight(d.experts, self.wp, dtype)
+        self.wgup = nn.Parameter(torch.empty(d.experts, 2 * self.fp, self.wp,
+                                             dtype=dtype))
+        self.wdown = nn.Parameter(torch.empty(d.experts, self.wp, self.fp,
+                                              dtype=dtype))
+
+    def tensors(self):
+        ff, W = self.d.ff, self.width
+        t = {}
+        for e in range(self.d.experts):
+            t |= {f"e{e}.gate": (ff, W), f"e{e}.up": (ff, W),
+                  f"e{e}.down": (W, ff)}
+        return t | {"router": (self.d.experts, W)}
+
+    def checkpoint(self, src, pre):
+        t = self.checked(src, pre)
+        U = self.UNIT
+
+        def gup(e):
+            halves = [padded(t[f"e{e}.{n}"], self.fp, self.wp)
+                      .view(-1, U, self.wp) for n in ("gate", "up")]
+            return torch.stack(halves, 1).view(2 * self.fp, self.wp)
+
+        return {"router": padded(t["router"], self.d.experts, self.wp),
+                "wgup": torch.stack([gup(e) for e in range(self.d.experts)]),
+                "wdown": torch.stack([padded(t[f"e{e}.down"], self.wp,
+                                             self.fp)
+                                      for e in range(self.d.experts)])}
+
+    def forward(self, h, ctx):
+        """-> outputs [rows * top, width] of the chosen experts, row by
+        row, and their weights [rows, top]; rows with ctx 0 have none."""
+        d = self.d
+        ids, weights = ops.route(h, self.router, ctx, d.top, d.groups,
+                                 d.keep)
+        return ops.experts(h, ids, self.wgup, self.wdown), weights

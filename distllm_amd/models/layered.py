@@ -1,0 +1,259 @@
+"""Decoders that are described layer by layer (LayeredDims).
+
+A layer is a mixer and, mostly, a feed-forward, each with sizes of its
+own; how they are joined to the fp32 residual stream is the design's and
+left to a subclass (`forward_step`). The model runs on ragged step
+batches only (engine/step.py): rows of any mix of prompt portions and
+single decoded tokens, against one cache entry per layer that owns one
+and, where there are recurrent layers, one state slot per sequence.
+"""
+
+from __future__ import annotations
+
+import torch
+from torch import nn
+
+from .. import ops
+from .attention import PagedAttention
+from .blocks import (ClampedGlu, LatentAttention, expect, norm_weight, pad64,
+                     padded, weight)
+from .config import (AttentionDims, ClampedGluDims, DeltaDims, ExpertsDims,
+                     LatentAttentionDims, LayeredDims, XieluDims)
+from .delta import GatedDelta
+from .feedforward import RoutedExperts, XieluMlp
+
+MIXERS = {LatentAttentionDims: LatentAttention,
+          AttentionDims: PagedAttention, DeltaDims: GatedDelta}
+MLPS = {ClampedGluDims: ClampedGlu, XieluDims: XieluMlp,
+        ExpertsDims: RoutedExperts}
+
+
+class LayeredCache:
+    """What every layer keeps between steps. A layer that shares another
+    layer's cache holds the same object."""
+
+    def __init__(self, model: "LayeredModel", num_blocks: int, blk: int,
+                 num_slots: int = 0):
+        self.layers: list = []
+        for layer in model.layers:
+            m = layer.mixer
+            self.layers.append(
+                m.make_cache(num_blocks, blk, num_slots, model.dtype,
+                             model.device)
+                if m.own else self.layers[m.kv_from])
+
+
+class Layer(nn.Module):
+    def __init__(self, d, width: int, eps: float, dtype,
+                 norms: tuple[str, ...], mlp_norms: tuple[str, ...]):
+        super().__init__()
+        wp = pad64(width)
+        self.mixer = MIXERS[type(d.mixer)](d.mixer, width, eps, dtype)
+        self.mlp = None
+        if d.mlp is not None:
+            self.mlp = MLPS[type(d.mlp)](d.mlp, width, dtype)
+        self.norm_names = norms + (mlp_norms if self.mlp is not None else ())
+        for n in norms + mlp_norms:
+            present = n in self.norm_names
+            setattr(self, n.replace(".", "_"),
+                    norm_weight(wp) if present else None)
+
+
+class LayeredModel(nn.Module):
+    # the engine feeds ragged step batches and grows sequences as they go
+    ragged = True
+    # portions of at least this many tokens take the attention form that
+    # is made for prompts
+    expand_min = 32
+    # norm tensors of a layer, of a layer with a feed-forward, of the model
+    layer_norms: tuple[str, ...] = ()
+    mlp_norms: tuple[str, ...] = ()
+    final_norms: tuple[str, ...] = ("final.norm",)
+    has_positions = False  # a table of position vectors
+
+    def __init__(self, dims: LayeredDims, dtype=torch.bfloat16,
+                 tp_group=None):
+        super().__init__()
+        if tp_group is not None:
+            raise ValueError(f"{dims.arch} models run on one GPU per engine "
+                             "(tensor_parallel_size 1)")
+        self.dims = dims
+        W, wp = dims.hidden_size, pad64(dims.hidden_size)
+        self.vp = pad64(dims.vocab_size)
+        self.tok_emb = weight(dims.vocab_size, wp, dtype)
+        self.pos_emb = (weight(dims.max_position_embeddings, wp, dtype)
+                        if self.has_positions else None)
+        self.layers = nn.ModuleList(
+            Layer(d, W, dims.norm_eps, dtype, self.layer_norms,
+                  self.mlp_norms) for d in dims.layers)
+        for n in self.final_norms:
+            setattr(self, n.replace(".", "_"), norm_weight(wp))
+        self.lm_head = weight(self.vp, wp, dtype)
+        self.reset_parameters()
+
+    # ---- weights --------------------------------------------------------
+    def _end_shapes(self) -> dict[str, tuple[int, ...]]:
+        d = self.dims
+        t = {"embed": (d.vocab_size, d.hidden_size),
+             "head": (d.vocab_size, d.hidden_size)}
+        if self.has_positions:
+            t["pos"] = (d.max_position_embeddings, d.hidden_size)
+        return t | {n: (d.hidden_size,) for n in self.final_norms}
+
+    def _layer_shapes(self, i: int) -> dict[str, tuple[int, ...]]:
+        layer, p = self.layers[i], f"l{i}."
+        t = {p + n: (self.dims.hidden_size,) for n in layer.norm_names}
+        for pre, part in (("mix.", layer.mixer), ("mlp.", layer.mlp)):
+            if part is not None:
+                t |= {p + pre + n: s for n, s in part.tensors().items()}
+        return t
+
+    def checkpoint_names(self) -> set[str]:
+        """Every tensor name that a checkpoint of these dims holds."""
+        names = set(self._end_shapes())
+        for i in range(len(self.layers)):
+            names |= set(self._layer_shapes(i))
+        return names
+
+    def _end_tensors(self, src: dict) -> dict[str, torch.Tensor]:
+        wp = self.tok_emb.shape[1]
+        t = {n: expect(n, src[n], *s) for n, s in self._end_shapes().items()}
+        out = {"tok_emb": padded(t["embed"], self.dims.vocab_size, wp),
+               "lm_head": padded(t["head"], self.vp, wp)}
+        if self.has_positions:
+            out["pos_emb"] = padded(t["pos"], t["pos"].shape[0], wp)
+        for n in self.final_norms:
+            out[n.replace(".", "_")] = padded(t[n], wp)
+        return out
+
+    def _layer_tensors(self, src: dict, i: int) -> dict[str, torch.Tensor]:
+        layer, p = self.layers[i], f"l{i}."
+        W, wp = self.dims.hidden_size, self.tok_emb.shape[1]
+        out = {n.replace(".", "_"): padded(expect(p + n, src[p + n], W), wp)
+               for n in layer.norm_names}
+        for name, pre, part in (("mixer.", "mix.", layer.mixer),
+                                ("mlp.", "mlp.", layer.mlp)):
+            if part is not None:
+                for k, v in part.checkpoint(src, p + pre).items():
+                    out[name + k] = v
+        return {f"layers.{i}.{k}": v for k, v in out.items()}
+
+    def checkpoint(self, src: dict) -> dict[str, torch.Tensor]:
+        """Parameter name -> tensor, from a checkpoint's raw tensors."""
+        out = self._end_tensors(src)
+        for i in range(len(self.layers)):
+            out.update(self._layer_tensors(src, i))
+        return out
+
+    @torch.no_grad()
+    def reset_parameters(self):
+        """Random weights, through the loader so that padding stays 0;
+        layer by layer, so that a large model is not held twice."""
+        own = dict(self.named_parameters())
+
+        def fill(shapes, to_own):
+            src = {}
+            for n, s in shapes.items():
+                if n.endswith(".b") and len(s) == 1:
+                    src[n] = torch.zeros(s, device=self.device)
+                elif len(s) == 1:
+                    src[n] = torch.ones(s, device=self.device)
+                else:
+                    src[n] = torch.randn(s, device=self.device,
+                                         dtype=self.dtype) * 0.02
+            for k, v in to_own(src).items():
+                own[k].copy_(v.to(own[k].dtype))
+
+        for i in range(len(self.layers)):
+            fill(self._layer_shapes(i), lambda src: self._layer_tensors(
+                src, i))
+        fill(self._end_shapes(), self._end_tensors)
+
+    # ---- cache ----------------------------------------------------------
+    def cache_bytes_per_block(self, blk: int, kv_cache_dtype: str) -> int:
+        el = self.tok_emb.element_size()
+        return sum(layer.mixer.cache_numel() * blk * el
+                   for layer in self.layers if layer.mixer.own)
+
+    def state_bytes_per_slot(self) -> int:
+        el = self.tok_emb.element_size()
+        return sum(f32 * 4 + own * el for f32, own in
+                   (layer.mixer.state_numel() for layer in self.layers))
+
+    def make_cache(self, num_blocks: int, blk: int, kv_cache_dtype: str,
+                   num_slots: int = 0) -> LayeredCache:
+        if kv_cache_dtype != "bf16":
+            raise ValueError(f"the cache of {self.dims.arch} models is kept "
+                             f"in the model's dtype, not {kv_cache_dtype}")
+        return LayeredCache(self, num_blocks, blk, num_slots)
+
+    # ---- step -----------------------------------------------------------
+    def forward_step(self, batch, cache: LayeredCache,
+                     trace: list | None = None) -> torch.Tensor:
+        """Final normed hidden state [M, padded width] of every row.
+        trace, when given, collects the residual after every layer."""
+        raise NotImplementedError
+
+    @torch.no_grad()
+    def logits(self, hidden: torch.Tensor) -> torch.Tensor:
+        """hidden [..., width or padded width] -> [..., vocab] f32."""
+        wp = self.lm_head.shape[1]
+        if hidden.shape[-1] != wp:
+            hidden = nn.functional.pad(hidden, (0, wp - hidden.shape[-1]))
+        out = ops.linear(hidden.contiguous(), self.lm_head)
+        out = out[..., : self.dims.vocab_size].float()
+        scale = self.dims.logit_scale
+        return out if scale == 1.0 else out * scale
+
+    @torch.no_grad()
+    def decode_step(self, tokens, cache: LayeredCache, block_tables,
+                    ctx_lens, slots=None) -> torch.Tensor:
+        """One token for each of B sequences (ctx_lens counts it)."""
+        from ..engine.step import StepBatch
+
+        batch = StepBatch.decode(tokens, block_tables, ctx_lens, slots)
+        return self.logits(self.forward_step(batch, cache))
+
+    @torch.no_grad()
+    def forward(self, input_ids: torch.Tensor,
+                attention_mask: torch.Tensor) -> torch.Tensor:
+        """Whole padded sequences without an engine: [B, S] ->
+        hidden [B, S, width], zeros at padding."""
+        from ..engine.step import StepBatch
+
+        blk = 16
+        mask = attention_mask.bool()
+        rows = [input_ids[b][mask[b]].tolist()
+                for b in range(input_ids.shape[0])]
+        need = [(len(r) + blk - 1) // blk for r in rows]
+        slots = None
+        if self.state_bytes_per_slot():
+            slots = list(range(1, sum(1 for r in rows if r) + 1))
+        cache = LayeredCache(self, sum(need) + 1, blk,
+                             len(slots) + 1 if slots else 0)
+        entries, at = [], 1
+        for b, r in enumerate(rows):
+            if r:
+                entries.append((r, 0, list(range(at, at + need[b]))))
+            at += need[b]
+        out = torch.zeros(*input_ids.shape, self.dims.hidden_size,
+                          dtype=self.dtype, device=self.device)
+        if entries:
+            batch = StepBatch.build(entries, blk, self.device, slots=slots)
+            h = self.forward_step(batch, cache)
+            order = torch.cat([torch.as_tensor(r) for r in batch.rows])
+            out[mask] = h[order.to(self.device),
+                          : self.dims.hidden_size]
+        return out
+
+    @property
+    def device(self):
+        return self.tok_emb.device
+
+    @property
+    def dtype(self):
+        return self.tok_emb.dtype
+
+    @property
+    def embedding_size(self) -> int:
+        return self.dims.hidden_size

@@ -18,6 +18,8 @@ from pathlib import Path
 
 import torch
 
+from .config import LayeredDims
+
 
 def _load_safetensors_dir(path: Path) -> dict[str, torch.Tensor]:
     from safetensors.torch import load_file
@@ -174,7 +176,7 @@ def load_weights(model, path: str | Path) -> None:
             mapped = _map_llama(src, model)
         elif arch == "esm2":
             mapped = _map_esm2(src, model)
-        elif arch == "kanotar":
+        elif isinstance(model.dims, LayeredDims):
             missing = sorted(model.checkpoint_names() - set(src))
             if missing:
                 raise ValueError(f"checkpoint lacks {missing}")

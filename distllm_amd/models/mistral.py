@@ -261,8 +261,11 @@ class DecoderModel(nn.Module):
         d = self.dims
         return self.local_kv_heads * blk * d.head_dim * el * 2 * d.num_layers
 
-    def make_cache(self, num_blocks: int, blk: int,
-                   kv_cache_dtype: str) -> KVCache:
+    def state_bytes_per_slot(self) -> int:
+        return 0  # no recurrent layers
+
+    def make_cache(self, num_blocks: int, blk: int, kv_cache_dtype: str,
+                   num_slots: int = 0) -> KVCache:
         fp8 = kv_cache_dtype == "fp8_e4m3"
         return KVCache(self, num_blocks, blk,
                        torch.uint8 if fp8 else self.dtype)

@@ -613,3 +613,77 @@ def attn_window(q, kv, out, cu_q, cu_k, block_map, window, scale):
         return out
     return out.copy_(torch_ref.attn_window(q, kv, out.shape[2], cu_q, cu_k,
                                            window, scale))
+
+
+# ---- chunked attention / delta rule / experts decoder -----------------------
+
+def embed_positions(tokens, ctx, table, pos):
+    """Start of a residual stream with position vectors: x = table[token]
+    + pos[ctx - 1] in fp32. -> (x in the table's dtype, x)"""
+    return torch_ref.embed_positions(tokens, ctx, table, pos)
+
+
+def layer_norm_add(y, x, w, b, n, eps, final=None, mix=None):
+    """End of a sublayer whose output is layer-normed: x += norm(y) (x
+    fp32, in place; statistics over n columns). Returns x in y's dtype,
+    normed by final = (weight, bias) if given. With mix [M, top] the
+    sublayer output is sum_k mix[m, k] * y[m * top + k]."""
+    return torch_ref.layer_norm_add(y, x, w, b, n, eps, final, mix)
+
+
+def attn_prep(ab, heads, kv_heads, dp, vp, dim, wq, wk, eps, pages,
+              block_table, row_seq, ctx):
+    """Norm the query heads of a fused projection (returned, [M, heads,
+    dp]) and its key heads, and write keys and values to their pages
+    (position ctx - 1; ctx 0 writes nothing). pages None: the layer has
+    no keys and values of its own."""
+    return torch_ref.attn_prep(ab, heads, kv_heads, dp, vp, dim, wq, wk, eps,
+                               pages, block_table, row_seq, ctx)
+
+
+def paged_attn_rows(q, kpages, vpages, ab, gate_at, out, block_table,
+                    row_seq, ctx, chunk, scale, softcap, dist, nsplit=0):
+    """Attention of single-token rows over paged keys and values. A row
+    sees the positions of its chunk up to its own. The output is gated by
+    the sigmoid of ab's columns from gate_at on."""
+    return torch_ref.paged_attn_rows(q, kpages, vpages, ab, gate_at, out,
+                                     block_table, row_seq, ctx, chunk, scale,
+                                     softcap, dist)
+
+
+def paged_attn_prompts(q, kpages, vpages, ab, gate_at, out, block_table,
+                       prompts, chunk, scale, softcap, dist):
+    """The same for the rows of prompt portions (step.PromptBlocks)."""
+    return torch_ref.paged_attn_prompts(q, kpages, vpages, ab, gate_at, out,
+                                        block_table, prompts, chunk, scale,
+                                        softcap, dist)
+
+
+def gated_delta(ab, heads, kv_heads, dp, vp, dim, vdim, conv_w, decay,
+                o_norm, unit_eps, eps, state, conv, segments, row_seq, ctx):
+    """Gated delta rule of a ragged step on the fused projection ab
+    [M, queries | keys | values | gates | b | a]: short convolutions, unit
+    queries and keys, recurrence in fp32, gated output norm.
+    -> [M, heads * vp]; state and convolution slots are updated."""
+    return torch_ref.gated_delta(
+        ab, heads, kv_heads, dp, vp, dim, vdim, conv_w, decay, o_norm,
+        unit_eps, eps, state, conv, segments, row_seq, ctx)
+
+
+def up_xielu(x, wup, act):
+    """xielu(x @ wup^T); act: the activation's two raw numbers."""
+    return torch_ref.xielu(linear(x, wup), act)
+
+
+def route(h, router, ctx, top, groups, keep):
+    """Experts of every row: ids [M, top] int32 and their softmax scores.
+    Only experts of the `keep` groups with the largest scores count; rows
+    with ctx 0 get ids -1 and weights 0."""
+    return torch_ref.route(h, router, ctx, top, groups, keep)
+
+
+def experts(h, ids, wgup, wdown):
+    """Gated-unit experts: row m * top + k of the result is expert
+    ids[m, k] of row m (undefined for id -1). wgup [E, 2F, W]: gate and up
+    rows alternate in groups of 16."""
+    return torch_ref.experts(h, ids, wgup, wdown)

@@ -368,3 +368,174 @@ def clamped_glu(gu, limit, alpha, shift):
     g = gu[..., :F_].float().clamp(max=limit)
     u = gu[..., F_:].float().clamp(-limit, limit)
     return (g * torch.sigmoid(alpha * g) * (u + shift)).to(gu.dtype)
+
+
+# ---- chunked attention / delta rule / experts decoder -----------------------
+
+def embed_positions(tokens, ctx, table, pos):
+    p = (ctx.long() - 1).clamp(min=0)
+    x = table[tokens.long()].float() + pos[p].float()
+    return x.to(table.dtype), x
+
+
+def _layer_norm_n(v, w, b, n, eps):
+    """Layer norm over the first n columns; w and b are 0 beyond."""
+    mean = v[:, :n].mean(-1, keepdim=True)
+    var = (v[:, :n] - mean).pow(2).mean(-1, keepdim=True)
+    return (v - mean) / torch.sqrt(var + eps) * w + b
+
+
+def layer_norm_add(y, x, w, b, n, eps, final=None, mix=None):
+    """x += layer_norm(y) in place; returns x (normed by final's weight
+    and bias, if given) in y's dtype. With mix [M, top], y [M * top, W]
+    is first summed with these weights."""
+    yf = y.float()
+    if mix is not None:
+        yf = yf.view(*mix.shape, -1).masked_fill(mix[..., None] == 0, 0)
+        yf = (yf * mix[..., None]).sum(1)
+    x += _layer_norm_n(yf, w, b, n, eps)
+    if final is None:
+        return x.to(y.dtype)
+    return _layer_norm_n(x, final[0], final[1], n, eps).to(y.dtype)
+
+
+def attn_prep(ab, heads, kv_heads, dp, vp, dim, wq, wk, eps, pages,
+              block_table, row_seq, ctx):
+    """Per-head norm of the queries (returned) and keys; keys and values
+    go to their pages."""
+
+    def norm(v, w):
+        v = v.float()
+        ms = v.pow(2).sum(-1, keepdim=True) / dim
+        return (v / torch.sqrt(ms + eps) * w).to(ab.dtype)
+
+    M = ab.shape[0]
+    if pages is not None:
+        kp, vpg = pages
+        blk = kp.shape[2]
+        live = ctx > 0
+        rows = _cache_rows(block_table, row_seq[live], ctx[live] - 1, blk)
+        at = heads * dp
+        k = ab[live, at: at + kv_heads * dp].view(-1, kv_heads, dp)
+        v = ab[live, at + kv_heads * dp:][:, : kv_heads * vp]
+        kp[rows // blk, :, rows % blk] = norm(k, wk)
+        vpg[rows // blk, :, :, rows % blk] = v.reshape(-1, kv_heads, vp)
+    return norm(ab[:, : heads * dp].reshape(M, heads, dp), wq)
+
+
+def paged_attn_rows(q, kpages, vpages, ab, gate_at, out, block_table,
+                    row_seq, ctx, chunk, scale, softcap, dist):
+    """Attention of single-token rows over the visible part of the pages:
+    the positions of the row's chunk up to its own."""
+    M, H, _ = q.shape
+    G, blk, dv = kpages.shape[1], kpages.shape[2], vpages.shape[2]
+    gate = torch.sigmoid(ab[:, gate_at: gate_at + H * dv].float()
+                         .reshape(M, H, dv))
+    for r in range(M):
+        p = int(ctx[r]) - 1
+        if p < 0:
+            out[r] = 0
+            continue
+        pos = torch.arange(p // chunk * chunk, p + 1)
+        rows = _cache_rows(block_table, row_seq[r].expand(len(pos)), pos,
+                           blk)
+        k = kpages[rows // blk, :, rows % blk].float()
+        v = vpages[rows // blk, :, :, rows % blk].float()
+        k = k.repeat_interleave(H // G, 1).transpose(0, 1)   # [H, n, d]
+        v = v.repeat_interleave(H // G, 1).transpose(0, 1)
+        s = (k * q[r].float()[:, None]).sum(-1) * scale
+        s = softcap * torch.tanh(s / softcap)
+        s = s - dist[0][:, None] * torch.log1p(
+            dist[1][:, None] * (p - pos)[None].float())
+        w = torch.softmax(s, -1)
+        out[r] = ((w[..., None] * v).sum(1) * gate[r]).to(q.dtype)
+    return out
+
+
+def paged_attn_prompts(q, kpages, vpages, ab, gate_at, out, block_table,
+                       prompts, chunk, scale, softcap, dist):
+    for seq, row0, start, n in prompts.portions.tolist():
+        r = slice(row0, row0 + n)
+        paged_attn_rows(q[r], kpages, vpages, ab[r], gate_at, out[r],
+                        block_table,
+                        torch.full((n,), seq, dtype=torch.int32),
+                        torch.arange(start + 1, start + n + 1), chunk, scale,
+                        softcap, dist)
+    return out
+
+
+def gated_delta(ab, heads, kv_heads, dp, vp, dim, vdim, conv_w, decay,
+                o_norm, unit_eps, eps, state, conv, segments, row_seq, ctx):
+    """Convolutions, recurrence and gated output norm of every segment;
+    state and conv slots are read and written."""
+    M, C, taps = ab.shape[0], conv_w.shape[1], conv_w.shape[0]
+    G, H = kv_heads, heads
+    out = torch.zeros(M, H * vp, dtype=ab.dtype)
+    own = torch.arange(H) // (H // G)
+    for row0, n, slot in zip(segments.row0.tolist(), segments.rows.tolist(),
+                             segments.slot.tolist()):
+        if n == 0:
+            continue
+        start = int(ctx[row0]) - 1
+        S = state[slot] * (start > 0)                  # [H, vp, dp]
+        past = conv[slot] * (start > 0)
+        x = torch.cat([past, ab[row0: row0 + n, :C]])
+        conv[slot] = x[n:]
+        z = sum(x[a: a + n].float() * conv_w[a] for a in range(taps))
+        z = torch.nn.functional.silu(z)
+        qk = z[:, : 2 * G * dp].view(n, 2, G, dp)
+        qk = qk / torch.sqrt(qk.pow(2).sum(-1, keepdim=True) + unit_eps)
+        q, k = qk[:, 0, own] * dim ** -0.5, qk[:, 1, own]
+        v = z[:, 2 * G * dp:].to(ab.dtype).float().view(n, H, vp)
+        gate = ab[row0: row0 + n, C: C + H * vp].float().view(n, H, vp)
+        ba = ab[row0: row0 + n, C + H * vp:][:, : 2 * H].float()
+        beta = torch.sigmoid(ba[:, :H])
+        g = torch.exp(-torch.exp(decay[0]) * torch.nn.functional.softplus(
+            ba[:, H:] + decay[1]))
+        for i in range(n):
+            S = S * g[i, :, None, None]
+            u = beta[i, :, None] * (v[i] - (S * k[i, :, None]).sum(-1))
+            S = S + u[..., None] * k[i, :, None]
+            o = (S * q[i, :, None]).sum(-1)            # [H, vp]
+            ms = o.pow(2).sum(-1, keepdim=True) / vdim
+            y = o / torch.sqrt(ms + eps) * o_norm
+            y = y * torch.nn.functional.silu(gate[i])
+            out[row0 + i] = y.reshape(-1).to(ab.dtype)
+        state[slot] = S
+    return out
+
+
+def xielu(z, act):
+    p, q = torch.nn.functional.softplus(act.float())
+    f = z.float()
+    pos = p * f * f + 0.5 * f
+    neg = (0.5 + q) * (torch.expm1(f.clamp(max=0)) - f) + 0.5 * f
+    return torch.where(f > 0, pos, neg).to(z.dtype)
+
+
+def route(h, router, ctx, top, groups, keep):
+    """-> expert ids [M, top] int32 (-1: none) and weights [M, top]."""
+    s = torch.softmax(h.float() @ router.float().t(), -1)
+    M, E = s.shape
+    best = s.view(M, groups, -1).amax(-1).topk(keep, -1).indices
+    allowed = torch.zeros(M, groups, dtype=torch.bool).scatter(1, best, True)
+    allowed = allowed.repeat_interleave(E // groups, 1)
+    w, ids = s.masked_fill(~allowed, -1).topk(top, -1)
+    dead = (ctx <= 0)[:, None]
+    return ids.int().masked_fill(dead, -1), w.masked_fill(dead, 0)
+
+
+def experts(h, ids, wgup, wdown, unit=16):
+    M, top = ids.shape
+    out = torch.zeros(M * top, wdown.shape[1], dtype=h.dtype)
+    flat = ids.reshape(-1)
+    for e in flat.unique().tolist():
+        if e < 0:
+            continue
+        rows = (flat == e).nonzero()[:, 0]
+        gu = h[rows // top].float() @ wgup[e].float().t()
+        gu = gu.view(len(rows), -1, 2, unit)
+        a = torch.nn.functional.silu(gu[:, :, 0]) * gu[:, :, 1]
+        a = a.reshape(len(rows), -1).to(h.dtype)
+        out[rows] = (a.float() @ wdown[e].float().t()).to(h.dtype)
+    return out

@@ -104,12 +104,12 @@ def check_whole(c: Case, n=90):
 def check_residuals(c: Case, n=40):
     """The residual stream after every layer."""
     from distllm_amd.engine.step import StepBatch
-    from distllm_amd.models.kanotar import LatentCache
+    from distllm_amd.models.layered import LayeredCache
 
     toks = c.tokens(n, 2)
     want, got = [], []
     oracle.forward(c.config, c.tensors, toks, want)
-    cache = LatentCache(c.model, n // 16 + 2, 16)
+    cache = LayeredCache(c.model, n // 16 + 2, 16)
     batch = StepBatch.build([(toks, 0, list(range(1, n // 16 + 2)))], 16,
                             c.model.device)
     c.model.forward_step(batch, cache, trace=got)

@@ -118,7 +118,7 @@ def test_latent_attention_forms():
     c = oracle.latent(h, t, "l0.mix.", 1e-5)
     want = oracle.latent_attention(h, c, t, "l0.mix.", m, 1e-5)
     from distllm_amd.engine.step import StepBatch
-    from distllm_amd.models.kanotar import LatentCache
+    from distllm_amd.models.layered import LayeredCache
 
     model = build_model(CONFIG_READERS["Kanotar"](cfg), dtype=F32)
     own = dict(model.named_parameters())
@@ -129,7 +129,7 @@ def test_latent_attention_forms():
         hp = torch.zeros(64, 64)
         hp[:40, :48] = h
         for expand_min in (1000, 2):
-            cache = LatentCache(model, 4, 16)
+            cache = LayeredCache(model, 4, 16)
             b = StepBatch.build([(list(range(40)), 0, [3, 1, 2])], 16,
                                 "cpu", expand_min)
             assert bool(b.portions) == (expand_min == 2)
