@@ -5,12 +5,27 @@ Imports neither torch nor the ops package, so it can run before them.
 
 from __future__ import annotations
 
+import json
 import os
 import subprocess
 import sys
 from pathlib import Path
 
 ROOT = Path(__file__).resolve().parents[1]
+
+
+# config.json "architecture" -> the extensions that the model's steps use
+NEEDED = {"Kanotar": ("_hip_gemm", "_hip_residual", "_hip_latent"),
+          "Bufulorn": ("_hip_gemm", "_hip_residual", "_hip_hybrid")}
+
+
+def needed_for(model_dir: str) -> tuple[str, ...]:
+    """Extensions for a checkpoint folder; none if it names no
+    architecture that is described in full."""
+    f = Path(model_dir) / "config.json"
+    if not f.is_file():
+        return ()
+    return NEEDED.get(json.loads(f.read_text()).get("architecture"), ())
 
 
 def is_built(name: str) -> bool:

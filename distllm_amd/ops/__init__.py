@@ -529,7 +529,7 @@ def embed_norm(tokens, table, w_next, n, eps):
     """Start of the residual stream: x = table[token] in fp32 and h =
     rms(x) * w_next, statistics over the first n columns. -> (h, x)"""
     if table.is_cuda:
-        _require_hip("_hip_latent")
+        _require_hip("_hip_residual")
         x = torch.empty(tokens.shape[0], table.shape[1],
                         dtype=torch.float32, device=table.device)
         h = _hip_ops.sandwich_norm(table, tokens, x, None, w_next, n, eps)
@@ -541,7 +541,7 @@ def post_norm_add(y, x, w_post, w_next, n, eps):
     """End of a sandwich-normed sublayer: x += rms(y) * w_post (x fp32,
     in place), returns the next sublayer's input rms(x) * w_next."""
     if y.is_cuda:
-        _require_hip("_hip_latent")
+        _require_hip("_hip_residual")
         return _hip_ops.sandwich_norm(y, None, x, w_post, w_next, n, eps)
     return torch_ref.post_norm_add(y, x, w_post, w_next, n, eps)
 
@@ -620,6 +620,11 @@ def attn_window(q, kv, out, cu_q, cu_k, block_map, window, scale):
 def embed_positions(tokens, ctx, table, pos):
     """Start of a residual stream with position vectors: x = table[token]
     + pos[ctx - 1] in fp32. -> (x in the table's dtype, x)"""
+    if table.is_cuda:
+        _require_hip("_hip_residual")
+        x = torch.empty(tokens.shape[0], table.shape[1],
+                        dtype=torch.float32, device=table.device)
+        return _hip_ops.embed_positions(tokens, ctx, table, pos, x), x
     return torch_ref.embed_positions(tokens, ctx, table, pos)
 
 
@@ -628,6 +633,10 @@ def layer_norm_add(y, x, w, b, n, eps, final=None, mix=None):
     fp32, in place; statistics over n columns). Returns x in y's dtype,
     normed by final = (weight, bias) if given. With mix [M, top] the
     sublayer output is sum_k mix[m, k] * y[m * top + k]."""
+    if y.is_cuda:
+        _require_hip("_hip_residual")
+        wf, bf = final if final is not None else (None, None)
+        return _hip_ops.layer_norm_add(y, x, w, b, n, eps, wf, bf, mix)
     return torch_ref.layer_norm_add(y, x, w, b, n, eps, final, mix)
 
 
@@ -637,6 +646,11 @@ def attn_prep(ab, heads, kv_heads, dp, vp, dim, wq, wk, eps, pages,
     dp]) and its key heads, and write keys and values to their pages
     (position ctx - 1; ctx 0 writes nothing). pages None: the layer has
     no keys and values of its own."""
+    if ab.is_cuda:
+        _require_hip("_hip_hybrid")
+        kp, vpg = pages if pages is not None else (None, None)
+        return _hip_ops.attn_prep(ab, heads, kv_heads, dp, vp, dim, wq, wk,
+                                  eps, kp, vpg, block_table, row_seq, ctx)
     return torch_ref.attn_prep(ab, heads, kv_heads, dp, vp, dim, wq, wk, eps,
                                pages, block_table, row_seq, ctx)
 
@@ -646,6 +660,12 @@ def paged_attn_rows(q, kpages, vpages, ab, gate_at, out, block_table,
     """Attention of single-token rows over paged keys and values. A row
     sees the positions of its chunk up to its own. The output is gated by
     the sigmoid of ab's columns from gate_at on."""
+    if q.is_cuda:
+        _require_hip("_hip_hybrid")
+        _hip_ops.paged_attn_rows(q, kpages, vpages, ab, gate_at, out,
+                                 block_table, row_seq, ctx, chunk, scale,
+                                 softcap, dist, nsplit)
+        return out
     return torch_ref.paged_attn_rows(q, kpages, vpages, ab, gate_at, out,
                                      block_table, row_seq, ctx, chunk, scale,
                                      softcap, dist)
@@ -654,6 +674,13 @@ def paged_attn_rows(q, kpages, vpages, ab, gate_at, out, block_table,
 def paged_attn_prompts(q, kpages, vpages, ab, gate_at, out, block_table,
                        prompts, chunk, scale, softcap, dist):
     """The same for the rows of prompt portions (step.PromptBlocks)."""
+    if q.is_cuda:
+        _require_hip("_hip_hybrid")
+        _hip_ops.paged_attn_prompts(q, kpages, vpages, ab, gate_at, out,
+                                    block_table, prompts.portions,
+                                    prompts.blocks, chunk, scale, softcap,
+                                    dist)
+        return out
     return torch_ref.paged_attn_prompts(q, kpages, vpages, ab, gate_at, out,
                                         block_table, prompts, chunk, scale,
                                         softcap, dist)
@@ -665,6 +692,12 @@ def gated_delta(ab, heads, kv_heads, dp, vp, dim, vdim, conv_w, decay,
     [M, queries | keys | values | gates | b | a]: short convolutions, unit
     queries and keys, recurrence in fp32, gated output norm.
     -> [M, heads * vp]; state and convolution slots are updated."""
+    if ab.is_cuda:
+        _require_hip("_hip_hybrid")
+        return _hip_ops.gated_delta(
+            ab, heads, kv_heads, dp, vp, dim, vdim, conv_w, decay, o_norm,
+            unit_eps, eps, state, conv, segments.row0, segments.rows,
+            segments.slot, segments.longest, row_seq, ctx)
     return torch_ref.gated_delta(
         ab, heads, kv_heads, dp, vp, dim, vdim, conv_w, decay, o_norm,
         unit_eps, eps, state, conv, segments, row_seq, ctx)
@@ -672,6 +705,17 @@ def gated_delta(ab, heads, kv_heads, dp, vp, dim, vdim, conv_w, decay,
 
 def up_xielu(x, wup, act):
     """xielu(x @ wup^T); act: the activation's two raw numbers."""
+    M, K = x.shape
+    if x.is_cuda:
+        _require_hip("_hip_gemm")
+        _require_hip("_hip_hybrid")
+        if (M <= 256 and x.dtype == torch.bfloat16 and K % 64 == 0
+                and wup.shape[0] % 64 == 0):
+            sk = _decode_splitk(M, wup.shape[0], K)
+            if sk > 1:
+                return _hip_ops.decode_gemm(x, wup, None, sk, 3,
+                                            act_nums=act)
+        return _hip_ops.xielu(linear(x, wup), act)
     return torch_ref.xielu(linear(x, wup), act)
 
 
@@ -679,6 +723,12 @@ def route(h, router, ctx, top, groups, keep):
     """Experts of every row: ids [M, top] int32 and their softmax scores.
     Only experts of the `keep` groups with the largest scores count; rows
     with ctx 0 get ids -1 and weights 0."""
+    if h.is_cuda:
+        _require_hip("_hip_hybrid")
+        if h.dtype == torch.bfloat16 and router.shape[0] <= 256:
+            return _hip_ops.route(h, router, ctx, top, groups, keep)
+        logits = torch.nn.functional.linear(h.float(), router.float())
+        return _hip_ops.route(logits, None, ctx, top, groups, keep)
     return torch_ref.route(h, router, ctx, top, groups, keep)
 
 
@@ -686,4 +736,7 @@ def experts(h, ids, wgup, wdown):
     """Gated-unit experts: row m * top + k of the result is expert
     ids[m, k] of row m (undefined for id -1). wgup [E, 2F, W]: gate and up
     rows alternate in groups of 16."""
+    if h.is_cuda:
+        _require_hip("_hip_hybrid")
+        return _hip_ops.experts(h, ids, wgup, wdown)
     return torch_ref.experts(h, ids, wgup, wdown)

@@ -132,6 +132,31 @@ __device__ __forceinline__ float clamped_glu_exact(float gate, float up,
   return g / (1.f + expf(-alpha * g)) * (u + shift);
 }
 
+// xIELU with ap = softplus(p), an = softplus(q): the fast form for 16-bit
+// outputs and the form on library functions for 32-bit ones.
+__device__ __forceinline__ float softplus_exact(float z) {
+  return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z)));
+}
+__device__ __forceinline__ float xielu(float z, float ap, float an) {
+  const float neg = (0.5f + an) * (fast_exp(fminf(z, 0.f)) - 1.f - z);
+  return 0.5f * z + (z > 0.f ? ap * z * z : neg);
+}
+__device__ __forceinline__ float xielu_exact(float z, float ap, float an) {
+  const float neg = (0.5f + an) * (expm1f(fminf(z, 0.f)) - z);
+  return 0.5f * z + (z > 0.f ? ap * z * z : neg);
+}
+__device__ __forceinline__ float sigmoid_exact(float z) {
+  return 1.f / (1.f + expf(-z));
+}
+
+// Scalars of the two tensor types as fp32.
+__device__ __forceinline__ float to_f(unsigned short v) { return bf2f(v); }
+__device__ __forceinline__ float to_f(float v) { return v; }
+__device__ __forceinline__ void from_f(unsigned short* p, float v) {
+  *p = f2bf(v);
+}
+__device__ __forceinline__ void from_f(float* p, float v) { *p = v; }
+
 // Eight consecutive numbers of a bf16 or fp32 array, as fp32.
 template <typename T>
 __device__ __forceinline__ void load8(const T* p, float* f);

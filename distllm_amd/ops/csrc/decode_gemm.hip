@@ -141,13 +141,20 @@ decode_gemm_kernel(const unsigned short* __restrict__ X,
     }
 }
 
-// reduce fp32 slabs [SPLITK, MP, N] -> bf16 [M, N] (+bias)
+// reduce fp32 slabs [SPLITK, MP, N] -> bf16 [M, N] (+bias); XIELU: with
+// the activation of numbers act[0..1] applied
+template <bool XIELU>
 __global__ void __launch_bounds__(256)
 dg_reduce_kernel(const float* __restrict__ slabs,
                  const unsigned short* __restrict__ bias,
                  unsigned short* __restrict__ out, int M, int MP, int N,
-                 int splitk) {
+                 int splitk, const float* __restrict__ act) {
   const long total = (long)M * N;
+  float ap = 0.f, an = 0.f;
+  if (XIELU) {
+    ap = softplus_exact(act[0]);
+    an = softplus_exact(act[1]);
+  }
   const long stride = (long)gridDim.x * blockDim.x;
   for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
        i += stride) {
@@ -157,7 +164,7 @@ dg_reduce_kernel(const float* __restrict__ slabs,
     for (int s = 0; s < splitk; ++s)
       v += slabs[((long)s * MP + row) * N + col];
     if (bias != nullptr) v += bf2f(bias[col]);
-    out[i] = f2bf(v);
+    out[i] = f2bf(XIELU ? xielu(v, ap, an) : v);
   }
 }
 
@@ -197,6 +204,7 @@ extern "C" void launch_decode_gemm(const void* X, const void* W,
                                    const void* bias, void* out, void* slabs,
                                    int M, int N, int K, int splitk, int act,
                                    float limit, float alpha, float shift,
+                                   const float* act_nums,
                                    hipStream_t stream) {
   const int MP = M <= 128 ? 128 : 256;
   const int ncb = N / DG_BN;
@@ -212,7 +220,8 @@ extern "C" void launch_decode_gemm(const void* X, const void* W,
   else { if (slab) DG(256, true); else DG(256, false); }
 #undef DG
   if (slab) {
-    const long total = (long)M * (act != 0 ? N / 2 : N);
+    const bool glu = act == 1 || act == 2;
+    const long total = (long)M * (glu ? N / 2 : N);
     int blocks = (int)min((total / 256) + 1, (long)2048);
 #define DGR(A)                                                                 \
   hipLaunchKernelGGL((dg_reduce_glu_kernel<A>), dim3(blocks), dim3(256), 0,    \
@@ -221,11 +230,16 @@ extern "C" void launch_decode_gemm(const void* X, const void* W,
                      N, splitk, limit, alpha, shift)
     if (act == 1) DGR(1);
     else if (act == 2) DGR(2);
-    else
-      hipLaunchKernelGGL(dg_reduce_kernel, dim3(blocks), dim3(256), 0,
+    else if (act == 3)
+      hipLaunchKernelGGL(dg_reduce_kernel<true>, dim3(blocks), dim3(256), 0,
                          stream, (const float*)slabs,
                          (const unsigned short*)bias, (unsigned short*)out,
-                         M, MP, N, splitk);
+                         M, MP, N, splitk, act_nums);
+    else
+      hipLaunchKernelGGL(dg_reduce_kernel<false>, dim3(blocks), dim3(256), 0,
+                         stream, (const float*)slabs,
+                         (const unsigned short*)bias, (unsigned short*)out,
+                         M, MP, N, splitk, act_nums);
 #undef DGR
   }
 }

@@ -1,0 +1,545 @@
+// Routed gated-unit experts.
+//
+//   route:   softmax scores of a row over all experts, the best groups, the
+//            best experts in them                    -> ids, weights [M, top]
+//   plan:    (row, choice) pairs sorted by expert, cut into tiles of rows
+//   product: one grouped product per tile; the first one gathers the rows
+//            and applies silu(gate) * up, the second scatters its rows to
+//            row * top + choice
+//
+// wgup [E, 2F, K]: gate and up rows alternate in groups of 16, so that a
+// tile of columns holds both halves of the unit. The number of tiles is
+// known on the device only: grids have the most there can be and surplus
+// workgroups leave at once.
+#include "common.h"
+
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+
+extern __shared__ __attribute__((aligned(16))) char smem[];
+
+__device__ __forceinline__ void wave_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
+// ---- routing ----------------------------------------------------------------
+// One wave chooses for one row. z [E]: logits, overwritten; gm, ok [groups].
+__device__ void select_row(float* z, float* gm, int* ok, int E, int groups,
+                           int keep, int top, int* __restrict__ ids,
+                           float* __restrict__ weights, int lane) {
+  float mx = -INFINITY;
+  for (int e = lane; e < E; e += 64) mx = fmaxf(mx, z[e]);
+  mx = wave_reduce_max(mx);
+  float sum = 0.f;
+  for (int e = lane; e < E; e += 64) {
+    const float s = expf(z[e] - mx);
+    z[e] = s;
+    sum += s;
+  }
+  sum = wave_reduce_sum(sum);
+  wave_sync();
+  const int per = E / groups;
+  for (int c = lane; c < groups; c += 64) {
+    float b = -1.f;
+    for (int i = 0; i < per; ++i) b = fmaxf(b, z[c * per + i]);
+    gm[c] = b;
+  }
+  wave_sync();
+  for (int c = lane; c < groups; c += 64) {
+    int rank = 0;
+    for (int i = 0; i < groups; ++i)
+      rank += gm[i] > gm[c] || (gm[i] == gm[c] && i < c);
+    ok[c] = rank < keep;
+  }
+  wave_sync();
+  for (int e = lane; e < E; e += 64)
+    if (!ok[e / per]) z[e] = -1.f;
+  wave_sync();
+  for (int t = 0; t < top; ++t) {
+    float best = -2.f;
+    int at = E;
+    for (int e = lane; e < E; e += 64)
+      if (z[e] > best) {
+        best = z[e];
+        at = e;
+      }
+#pragma unroll
+    for (int off = 32; off > 0; off >>= 1) {
+      const float b = __shfl_xor(best, off, 64);
+      const int a = __shfl_xor(at, off, 64);
+      if (b > best || (b == best && a < at)) {
+        best = b;
+        at = a;
+      }
+    }
+    if (lane == 0) {
+      ids[t] = at;
+      weights[t] = best / sum;
+      z[at] = -3.f;
+    }
+    wave_sync();
+  }
+}
+
+__device__ __forceinline__ void no_choice(int top, int* ids, float* weights,
+                                          int lane) {
+  for (int t = lane; t < top; t += 64) {
+    ids[t] = -1;
+    weights[t] = 0.f;
+  }
+}
+
+// from given logits [M, E]; one wave per row
+__global__ void __launch_bounds__(256)
+select_kernel(const float* __restrict__ logits, const int* __restrict__ ctx,
+              int M, int E, int groups, int keep, int top,
+              int* __restrict__ ids, float* __restrict__ weights) {
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  float* z = reinterpret_cast<float*>(smem) + wid * (E + 2 * groups);
+  float* gm = z + E;
+  int* ok = reinterpret_cast<int*>(gm + groups);
+  const int row = blockIdx.x * 4 + wid;
+  if (row >= M) return;
+  int* id = ids + (long)row * top;
+  float* w = weights + (long)row * top;
+  if (ctx[row] <= 0) {
+    no_choice(top, id, w, lane);
+    return;
+  }
+  for (int e = lane; e < E; e += 64) z[e] = logits[(long)row * E + e];
+  wave_sync();
+  select_row(z, gm, ok, E, groups, keep, top, id, w, lane);
+}
+
+// bf16 rows against the router's weights [E, K], fp32 sums, then the
+// choice: 16 rows per workgroup, the four waves split K. NE tiles of 16
+// experts.
+template <int NE>
+__global__ void __launch_bounds__(256)
+route_kernel(const unsigned short* __restrict__ h,
+             const unsigned short* __restrict__ W,
+             const int* __restrict__ ctx, int M, int E, int K, int groups,
+             int keep, int top, int* __restrict__ ids,
+             float* __restrict__ weights) {
+  constexpr int EP = NE * 16;
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int i16 = lane & 15, g = lane >> 4;
+  const int m0 = blockIdx.x * 16;
+  const unsigned short* hr =
+      h + (long)min(m0 + i16, M - 1) * K + g * 8;
+  const unsigned short* wr[NE];
+#pragma unroll
+  for (int j = 0; j < NE; ++j)
+    wr[j] = W + (long)min(j * 16 + i16, E - 1) * K + g * 8;
+  f32x4 acc[NE];
+#pragma unroll
+  for (int j = 0; j < NE; ++j) acc[j] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 2
+  for (int k = wid * 32; k < K; k += 128) {
+    const bf16x8 a = *reinterpret_cast<const bf16x8*>(hr + k);
+#pragma unroll
+    for (int j = 0; j < NE; ++j)
+      acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+          *reinterpret_cast<const bf16x8*>(wr[j] + k), a, acc[j], 0, 0, 0);
+  }
+  // rows of the sum: experts (g * 4 + r); columns: rows of h (i16)
+  float* part = reinterpret_cast<float*>(smem);  // [4][16][EP + 4]
+#pragma unroll
+  for (int j = 0; j < NE; ++j)
+    *reinterpret_cast<f32x4*>(part + (wid * 16 + i16) * (EP + 4) + j * 16 +
+                              g * 4) = acc[j];
+  __syncthreads();
+  float* gm = part + 64 * (EP + 4) + wid * 2 * groups;
+  int* ok = reinterpret_cast<int*>(gm + groups);
+  for (int i = wid * 4; i < wid * 4 + 4; ++i) {
+    const int row = m0 + i;
+    if (row >= M) break;
+    int* id = ids + (long)row * top;
+    float* w = weights + (long)row * top;
+    if (ctx[row] <= 0) {
+      no_choice(top, id, w, lane);
+      continue;
+    }
+    float* z = part + i * (EP + 4);
+    for (int e = lane; e < E; e += 64)
+      z[e] = (z[e] + z[e + 16 * (EP + 4)]) +
+             (z[e + 32 * (EP + 4)] + z[e + 48 * (EP + 4)]);
+    wave_sync();
+    select_row(z, gm, ok, E, groups, keep, top, id, w, lane);
+  }
+}
+
+extern "C" bool route_covers(int E) { return E <= 256; }
+
+extern "C" void launch_select(const float* logits, const int* ctx, int M,
+                              int E, int groups, int keep, int top, int* ids,
+                              float* weights, hipStream_t stream) {
+  hipLaunchKernelGGL(select_kernel, dim3((M + 3) / 4), dim3(256),
+                     4 * (E + 2 * groups) * 4, stream, logits, ctx, M, E,
+                     groups, keep, top, ids, weights);
+}
+
+extern "C" void launch_route(const void* h, const void* W, const int* ctx,
+                             int M, int E, int K, int groups, int keep,
+                             int top, int* ids, float* weights,
+                             hipStream_t stream) {
+#define RT(NE)                                                               \
+  hipLaunchKernelGGL((route_kernel<NE>), dim3((M + 15) / 16), dim3(256),     \
+                     (64 * (NE * 16 + 4) + 8 * groups) * 4, stream,          \
+                     (const unsigned short*)h, (const unsigned short*)W, ctx, \
+                     M, E, K, groups, keep, top, ids, weights)
+  if (E <= 16) RT(1);
+  else if (E <= 32) RT(2);
+  else if (E <= 64) RT(4);
+  else if (E <= 128) RT(8);
+  else RT(16);
+#undef RT
+}
+
+// ---- plan ---------------------------------------------------------------------
+// perm [A]: pair (row * top + choice) of each sorted place; tiles
+// [max_tiles, 4]: expert, first place, places; ntiles. One workgroup.
+__global__ void __launch_bounds__(1024)
+expert_plan_kernel(const int* __restrict__ ids, int A, int E, int TM,
+                   int max_tiles, int* __restrict__ perm,
+                   int* __restrict__ tiles, int* __restrict__ ntiles) {
+  __shared__ int count[1024], first[1024], tile0[1024];
+  const int tid = threadIdx.x;
+  count[tid] = 0;
+  __syncthreads();
+  for (int a = tid; a < A; a += 1024) {
+    const int e = ids[a];
+    if (e >= 0 && e < E) atomicAdd(&count[e], 1);
+  }
+  __syncthreads();
+  const int c = count[tid], nt = (c + TM - 1) / TM;
+  first[tid] = c;
+  tile0[tid] = nt;
+  __syncthreads();
+  for (int off = 1; off < 1024; off <<= 1) {  // inclusive sums
+    const int x = tid >= off ? first[tid - off] : 0;
+    const int y = tid >= off ? tile0[tid - off] : 0;
+    __syncthreads();
+    first[tid] += x;
+    tile0[tid] += y;
+    __syncthreads();
+  }
+  const int f = first[tid] - c, t0 = tile0[tid] - nt;
+  if (tid == 1023) *ntiles = min(tile0[tid], max_tiles);
+  for (int i = 0; i < nt; ++i)
+    if (t0 + i < max_tiles) {
+      int* t = tiles + (long)(t0 + i) * 4;
+      t[0] = tid;
+      t[1] = f + i * TM;
+      t[2] = min(TM, c - i * TM);
+    }
+  __syncthreads();
+  count[tid] = f;
+  __syncthreads();
+  for (int a = tid; a < A; a += 1024) {
+    const int e = ids[a];
+    if (e >= 0 && e < E) perm[atomicAdd(&count[e], 1)] = a;
+  }
+}
+
+extern "C" void launch_expert_plan(const int* ids, int A, int E, int TM,
+                                   int max_tiles, int* perm, int* tiles,
+                                   int* ntiles, hipStream_t stream) {
+  hipLaunchKernelGGL(expert_plan_kernel, dim3(1), dim3(1024), 0, stream, ids,
+                     A, E, TM, max_tiles, perm, tiles, ntiles);
+}
+
+// ---- product, few rows per expert ----------------------------------------------
+// Weight-streaming bound: a workgroup takes 64 weight rows and up to 16 MT
+// places; its waves split K and read the weights straight into registers.
+// GLU: rows are gathered (place -> perm / top) and the output is F wide;
+// else rows are places and the output row is perm[place].
+template <int MT, bool GLU>
+__global__ void __launch_bounds__(256)
+expert_rows_kernel(const unsigned short* __restrict__ x,
+                   const unsigned short* __restrict__ W,
+                   unsigned short* __restrict__ out,
+                   const int* __restrict__ perm,
+                   const int* __restrict__ tiles,
+                   const int* __restrict__ ntiles, int N, int K, int top) {
+  constexpr int RROW = 68;  // padded row of 64 sums
+  if ((int)blockIdx.y >= *ntiles) return;
+  const int* tile = tiles + (long)blockIdx.y * 4;
+  const int e = tile[0], s0 = tile[1], cnt = tile[2];
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+  const int i16 = lane & 15, g = lane >> 4;
+  const int n0 = blockIdx.x * 64;
+  const unsigned short* wr =
+      W + ((long)e * N + n0 + i16) * K + g * 8;
+  const unsigned short* xr[MT];
+#pragma unroll
+  for (int t = 0; t < MT; ++t) {
+    const int s = s0 + min(t * 16 + i16, cnt - 1);
+    xr[t] = x + (long)(GLU ? perm[s] / top : s) * K + g * 8;
+  }
+  f32x4 acc[MT][4];
+#pragma unroll
+  for (int t = 0; t < MT; ++t)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[t][j] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 4
+  for (int k = wid * 32; k < K; k += 128) {
+    bf16x8 wf[4], xf[MT];
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      wf[j] = *reinterpret_cast<const bf16x8*>(wr + (long)j * 16 * K + k);
+#pragma unroll
+    for (int t = 0; t < MT; ++t)
+      xf[t] = *reinterpret_cast<const bf16x8*>(xr[t] + k);
+#pragma unroll
+    for (int t = 0; t < MT; ++t)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        acc[t][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            wf[j], xf[t], acc[t][j], 0, 0, 0);
+  }
+  // sums: rows are weight rows, columns places -> [wave][place][column]
+  float* part = reinterpret_cast<float*>(smem);
+#pragma unroll
+  for (int t = 0; t < MT; ++t)
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+      *reinterpret_cast<f32x4*>(
+          part + ((wid * MT + t) * 16 + i16) * RROW + j * 16 + g * 4) =
+          acc[t][j];
+  __syncthreads();
+  constexpr int WS = MT * 16 * RROW;  // per wave
+  constexpr int OC = GLU ? 32 : 64;   // output columns
+  for (int i = threadIdx.x; i < cnt * (OC / 4); i += 256) {
+    const int m = i / (OC / 4), c = i % (OC / 4) * 4;
+    const float* p = part + m * RROW + (GLU ? c / 16 * 32 + c % 16 : c);
+    s16x4 o;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      float v = (p[r] + p[WS + r]) + (p[2 * WS + r] + p[3 * WS + r]);
+      if (GLU) {
+        const float* u = p + 16;
+        v = silu(v) *
+            ((u[r] + u[WS + r]) + (u[2 * WS + r] + u[3 * WS + r]));
+      }
+      o[r] = (short)f2bf(v);
+    }
+    const long row = GLU ? s0 + m : perm[s0 + m];
+    *reinterpret_cast<s16x4*>(out + row * (GLU ? N / 2 : N) +
+                              blockIdx.x * OC + c) = o;
+  }
+}
+
+// ---- product, many rows per expert ----------------------------------------------
+// 128 x 128 x 64 tiles, four waves of 64 x 64, both operands through LDS in
+// two buffers by global_load_lds with the bank swizzle on the source address
+// (the structure of gemm.hip, with gathered and scattered rows).
+#define ET_M 128
+#define ET_N 128
+#define ET_K 64
+#define ET_TILE (128 * ET_K * 2)
+#define ET_LDS (68 * 1024)
+
+template <bool GLU>
+__global__ void __launch_bounds__(256, 2)
+expert_tile_kernel(const unsigned short* __restrict__ x,
+                   const unsigned short* __restrict__ W,
+                   unsigned short* __restrict__ out,
+                   const int* __restrict__ perm,
+                   const int* __restrict__ tiles,
+                   const int* __restrict__ ntiles, int N, int K, int top) {
+  const int nt_all = *ntiles;
+  const int ncol = (N + ET_N - 1) / ET_N;
+  // contiguous runs of (tile, column block) per XCD, columns fastest: they
+  // share the rows of x
+  const int total = nt_all * ncol;
+  const int per = (total + 7) / 8;
+  const int xcd = blockIdx.x % 8, j8 = blockIdx.x / 8;
+  const int bid = xcd * per + j8;
+  if (j8 >= per || bid >= total) return;
+  const int* tile = tiles + (long)(bid / ncol) * 4;
+  const int e = tile[0], s0 = tile[1], cnt = tile[2];
+  const int n0 = bid % ncol * ET_N;
+  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+
+  // rows of this thread's four pieces of each operand
+  const int r_in = lane >> 3, c_src = ((lane & 7) ^ r_in) * 8;
+  const unsigned short *xs[4], *ws[4];
+#pragma unroll
+  for (int p = 0; p < 4; ++p) {
+    const int r = wid * 32 + p * 8 + r_in;
+    const int s = s0 + min(r, cnt - 1);
+    xs[p] = x + (long)(GLU ? perm[s] / top : s) * K + c_src;
+    ws[p] = W + ((long)e * N + min(n0 + r, N - 1)) * K + c_src;
+  }
+  auto stage = [&](int k0, int buf) {
+#pragma unroll
+    for (int p = 0; p < 4; ++p) {
+      char* dst = smem + buf * 2 * ET_TILE + (wid * 32 + p * 8) * 128 +
+                  lane * 16;
+      __builtin_amdgcn_global_load_lds(
+          (const __attribute__((address_space(1))) unsigned int*)(xs[p] + k0),
+          (__attribute__((address_space(3))) unsigned int*)dst, 16, 0, 0);
+      __builtin_amdgcn_global_load_lds(
+          (const __attribute__((address_space(1))) unsigned int*)(ws[p] + k0),
+          (__attribute__((address_space(3))) unsigned int*)(dst + ET_TILE),
+          16, 0, 0);
+    }
+  };
+  auto frag = [&](int off, int row, int chunk) {
+    return *reinterpret_cast<const bf16x8*>(
+        smem + off + row * 128 + ((chunk ^ (row & 7)) * 16));
+  };
+
+  f32x4 acc[4][4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = {0.f, 0.f, 0.f, 0.f};
+  const int wrow = (wid >> 1) * 64, wcol = (wid & 1) * 64;
+
+  stage(0, 0);
+  asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+  __syncthreads();
+  const int nk = K / ET_K;
+  for (int t = 0; t < nk; ++t) {
+    const int buf = t & 1;
+    if (t + 1 < nk) stage((t + 1) * ET_K, buf ^ 1);
+    const int offX = buf * 2 * ET_TILE, offW = offX + ET_TILE;
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) {
+      bf16x8 af[4], bf[4];
+      const int chunk = kk * 4 + (lane >> 4);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        af[i] = frag(offX, wrow + i * 16 + (lane & 15), chunk);
+        bf[i] = frag(offW, wcol + i * 16 + (lane & 15), chunk);
+      }
+      __builtin_amdgcn_s_setprio(1);
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          acc[i][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              af[i], bf[j], acc[i][j], 0, 0, 0);
+      __builtin_amdgcn_s_setprio(0);
+    }
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+  }
+
+  // sums -> padded LDS (a wave's own 64 x 64) -> rows
+  float* ep = reinterpret_cast<float*>(smem) + wid * 64 * 65;
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        ep[(i * 16 + (lane >> 4) * 4 + r) * 65 + j * 16 + (lane & 15)] =
+            acc[i][j][r];
+  __syncthreads();
+  if (GLU) {
+    const int F = N / 2;
+    const int c = lane & 31;
+    const int col = (n0 + wcol) / 2 + c;
+    const float* p = ep + c / 16 * 32 + c % 16;
+    for (int r = lane >> 5; r < 64; r += 2) {
+      if (wrow + r >= cnt) break;
+      if (col < F)
+        out[(long)(s0 + wrow + r) * F + col] =
+            f2bf(silu(p[r * 65]) * p[r * 65 + 16]);
+    }
+  } else {
+    const int col = n0 + wcol + lane;
+    for (int r = 0; r < 64; ++r) {
+      if (wrow + r >= cnt) break;
+      if (col < N)
+        out[(long)perm[s0 + wrow + r] * N + col] = f2bf(ep[r * 65 + lane]);
+    }
+  }
+}
+
+// ---- product in 32-bit: 16 places x 64 columns, one sum in four per thread ---
+template <bool GLU>
+__global__ void __launch_bounds__(256)
+expert_f32_kernel(const float* __restrict__ x, const float* __restrict__ W,
+                  float* __restrict__ out, const int* __restrict__ perm,
+                  const int* __restrict__ tiles,
+                  const int* __restrict__ ntiles, int N, int K, int top) {
+  __shared__ float xl[16][33], wl[64][33], sum[16][65];
+  if ((int)blockIdx.y >= *ntiles) return;
+  const int* tile = tiles + (long)blockIdx.y * 4;
+  const int e = tile[0], s0 = tile[1], cnt = tile[2];
+  const int n0 = blockIdx.x * 64, tid = threadIdx.x;
+  const int m = tid / 16, c = tid % 16;
+  float acc[4] = {0.f, 0.f, 0.f, 0.f};
+  for (int k0 = 0; k0 < K; k0 += 32) {
+    __syncthreads();
+    for (int i = tid; i < 16 * 32; i += 256) {
+      const int s = s0 + min(i / 32, cnt - 1);
+      xl[i / 32][i % 32] =
+          x[(long)(GLU ? perm[s] / top : s) * K + k0 + i % 32];
+    }
+    for (int i = tid; i < 64 * 32; i += 256)
+      wl[i / 32][i % 32] = W[((long)e * N + n0 + i / 32) * K + k0 + i % 32];
+    __syncthreads();
+    for (int k = 0; k < 32; ++k)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[j] += xl[m][k] * wl[c + j * 16][k];
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) sum[m][c + j * 16] = acc[j];
+  __syncthreads();
+  constexpr int OC = GLU ? 32 : 64;
+  for (int i = tid; i < cnt * OC; i += 256) {
+    const int r = i / OC, o = i % OC;
+    float v = sum[r][GLU ? o / 16 * 32 + o % 16 : o];
+    if (GLU) v = v * sigmoid_exact(v) * sum[r][o / 16 * 32 + o % 16 + 16];
+    const long row = GLU ? s0 + r : perm[s0 + r];
+    out[row * (GLU ? N / 2 : N) + blockIdx.x * OC + o] = v;
+  }
+}
+
+// TM: rows per tile of the plan (16, 32, 64, or 128 for the large tiles)
+extern "C" void launch_expert_gemm(const void* x, const void* W, void* out,
+                                   const int* perm, const int* tiles,
+                                   const int* ntiles, int max_tiles, int N,
+                                   int K, int top, int TM, bool glu,
+                                   bool fp32, hipStream_t stream) {
+  typedef unsigned short u16;
+  const dim3 grid(N / 64, max_tiles);
+  if (fp32) {
+#define EF(GL)                                                              \
+  hipLaunchKernelGGL((expert_f32_kernel<GL>), grid, dim3(256), 0, stream,   \
+                     (const float*)x, (const float*)W, (float*)out, perm,   \
+                     tiles, ntiles, N, K, top)
+    if (glu) EF(true);
+    else EF(false);
+#undef EF
+    return;
+  }
+#define ER(MT, GL)                                                          \
+  hipLaunchKernelGGL((expert_rows_kernel<MT, GL>), grid, dim3(256),         \
+                     4 * MT * 16 * 68 * 4, stream, (const u16*)x,           \
+                     (const u16*)W, (u16*)out, perm, tiles, ntiles, N, K, top)
+#define ET(GL)                                                              \
+  hipLaunchKernelGGL((expert_tile_kernel<GL>),                              \
+                     dim3(((long)max_tiles * ((N + ET_N - 1) / ET_N) + 7) /  \
+                          8 * 8),                                           \
+                     dim3(256), ET_LDS, stream, (const u16*)x,              \
+                     (const u16*)W, (u16*)out, perm, tiles, ntiles, N, K, top)
+#define EX(GL)                   \
+  do {                           \
+    if (TM == 16) ER(1, GL);     \
+    else if (TM == 32) ER(2, GL); \
+    else if (TM == 64) ER(4, GL); \
+    else ET(GL);                 \
+  } while (0)
+  if (glu) EX(true);
+  else EX(false);
+#undef EX
+#undef ET
+#undef ER
+}

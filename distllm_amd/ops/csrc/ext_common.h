@@ -14,6 +14,17 @@
   TORCH_CHECK(x.scalar_type() == at::kFloat, #x " must be f32")
 #define CHECK_I32(x) TORCH_CHECK(x.scalar_type() == at::kInt, #x " must be i32")
 
+#define CHECK_T(x)                                              \
+  TORCH_CHECK(x.scalar_type() == at::kBFloat16 ||               \
+                  x.scalar_type() == at::kFloat,                \
+              #x " must be bf16 or f32")
+#define CHECK_SAME(x, y) \
+  TORCH_CHECK(x.scalar_type() == y.scalar_type(), #x " and " #y " differ")
+
+static inline bool is_f32(const torch::Tensor& t) {
+  return t.scalar_type() == at::kFloat;
+}
+
 static inline hipStream_t cur_stream() {
   return c10::hip::getCurrentHIPStream().stream();
 }

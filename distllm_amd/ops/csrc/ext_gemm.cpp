@@ -12,7 +12,7 @@ void launch_gemm16_bf16(const void*, const void*, const void*, void*, int,
                         int, int, int, hipStream_t);
 void launch_decode_gemm(const void*, const void*, const void*, void*, void*,
                         int, int, int, int, int, float, float, float,
-                        hipStream_t);
+                        const float*, hipStream_t);
 }
 
 // ---- GEMM ------------------------------------------------------------------
@@ -65,10 +65,12 @@ torch::Tensor decode_gemm(torch::Tensor X, torch::Tensor W,
                           c10::optional<torch::Tensor> bias,
                           int64_t splitk, int64_t act = 0,
                           double limit = 0.0, double alpha = 0.0,
-                          double shift = 0.0) {
-  // act != 0 = packed gated unit in the reduce (1 swiglu, 2 clamped with
-  // the given constants): W is [2I, K] (gate rows then up rows), output
-  // is [M, I]; requires splitk > 1.
+                          double shift = 0.0,
+                          c10::optional<torch::Tensor> act_nums = {}) {
+  // act 1, 2 = packed gated unit in the reduce (swiglu, clamped with the
+  // given constants): W is [2I, K] (gate rows then up rows), output is
+  // [M, I]. act 3 = xIELU with the raw numbers act_nums [2]. All require
+  // splitk > 1.
   CHECK_DEV(X); CHECK_CONT(X); CHECK_BF16(X);
   CHECK_DEV(W); CHECK_CONT(W); CHECK_BF16(W);
   const int M = X.size(0), K = X.size(1), N = W.size(0);
@@ -76,10 +78,17 @@ torch::Tensor decode_gemm(torch::Tensor X, torch::Tensor W,
   TORCH_CHECK(M <= 256, "decode_gemm is for M <= 256");
   TORCH_CHECK(N % 64 == 0, "N % 64");
   TORCH_CHECK(K % (64 * splitk) == 0, "K % (64*splitk)");
-  TORCH_CHECK(act == 0 || (splitk > 1 && N % 128 == 0),
-              "gated-unit fusion needs splitk > 1 and even I");
+  const bool glu = act == 1 || act == 2;
+  TORCH_CHECK(act == 0 || splitk > 1, "a fused activation needs splitk > 1");
+  TORCH_CHECK(!glu || N % 128 == 0, "gated-unit fusion needs N % 128 == 0");
+  const float* nums = nullptr;
+  if (act == 3) {
+    TORCH_CHECK(act_nums.has_value() && act_nums->numel() == 2, "act_nums");
+    CHECK_DEV(act_nums.value()); CHECK_F32(act_nums.value());
+    nums = act_nums->data_ptr<float>();
+  }
   const int MP = M <= 128 ? 128 : 256;
-  auto out = torch::empty({M, act != 0 ? N / 2 : N}, X.options());
+  auto out = torch::empty({M, glu ? N / 2 : N}, X.options());
   torch::Tensor slabs;
   void* slabp = nullptr;
   if (splitk > 1) {
@@ -90,7 +99,7 @@ torch::Tensor decode_gemm(torch::Tensor X, torch::Tensor W,
   launch_decode_gemm(X.data_ptr(), W.data_ptr(),
                      bias ? bias->data_ptr() : nullptr, out.data_ptr(),
                      slabp, M, N, K, (int)splitk, (int)act, (float)limit,
-                     (float)alpha, (float)shift, cur_stream());
+                     (float)alpha, (float)shift, nums, cur_stream());
   return out;
 }
 
@@ -107,5 +116,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("decode_gemm", &decode_gemm, py::arg("X"), py::arg("W"),
         py::arg("bias"), py::arg("splitk"), py::arg("act") = 0,
         py::arg("limit") = 0.0, py::arg("alpha") = 0.0,
-        py::arg("shift") = 0.0);
+        py::arg("shift") = 0.0, py::arg("act_nums") = py::none());
 }

@@ -1,11 +1,8 @@
-// Torch bindings of the latent-attention decoder kernels: sandwich norms,
-// latent preparation and attention, the clamped gated unit.
+// Torch bindings of the latent-attention decoder kernels: latent
+// preparation and attention, the clamped gated unit.
 #include "ext_common.h"
 
 extern "C" {
-void launch_sandwich_norm(const void*, const long*, float*, const float*,
-                          const float*, void*, int, int, int, float, bool,
-                          hipStream_t);
 void launch_latent_prep(const void*, int, int, int, int, int, int,
                         const float*, const float*, float, void*, void*,
                         const int*, int, int, const int*, const int*, bool,
@@ -29,17 +26,6 @@ void launch_clamped_glu(const void*, void*, long, int, float, float, float,
                         bool, hipStream_t);
 }
 
-#define CHECK_T(x)                                              \
-  TORCH_CHECK(x.scalar_type() == at::kBFloat16 ||               \
-                  x.scalar_type() == at::kFloat,                \
-              #x " must be bf16 or f32")
-#define CHECK_SAME(x, y) \
-  TORCH_CHECK(x.scalar_type() == y.scalar_type(), #x " and " #y " differ")
-
-static bool is_f32(const torch::Tensor& t) {
-  return t.scalar_type() == at::kFloat;
-}
-
 static void check_pages(const torch::Tensor& cache, const torch::Tensor& bt,
                         const torch::Tensor& row_seq,
                         const torch::Tensor& ctx, long M) {
@@ -52,41 +38,6 @@ static void check_pages(const torch::Tensor& cache, const torch::Tensor& bt,
   CHECK_DEV(ctx); CHECK_CONT(ctx); CHECK_I32(ctx);
   TORCH_CHECK(bt.dim() == 2 && row_seq.numel() == M && ctx.numel() == M,
               "one row_seq and ctx entry per row");
-}
-
-// y == embedding table when tokens are given
-torch::Tensor sandwich_norm(torch::Tensor y,
-                            c10::optional<torch::Tensor> tokens,
-                            torch::Tensor x,
-                            c10::optional<torch::Tensor> w_post,
-                            torch::Tensor w_next, int64_t n, double eps) {
-  CHECK_DEV(y); CHECK_CONT(y); CHECK_T(y);
-  CHECK_DEV(x); CHECK_CONT(x); CHECK_F32(x);
-  CHECK_DEV(w_next); CHECK_CONT(w_next); CHECK_F32(w_next);
-  const int M = x.size(0), W = x.size(1);
-  TORCH_CHECK(x.dim() == 2 && y.dim() == 2 && y.size(1) == W, "row sizes");
-  TORCH_CHECK(W % 8 == 0 && W <= 16384 && n > 0 && n <= W,
-              "width must be a multiple of 8, at most 16384");
-  TORCH_CHECK(w_next.numel() == W, "w_next size");
-  const long* tok = nullptr;
-  if (tokens) {
-    CHECK_DEV(tokens.value()); CHECK_CONT(tokens.value());
-    TORCH_CHECK(tokens->scalar_type() == at::kLong && tokens->numel() == M,
-                "tokens must be int64, one per row");
-    tok = (const long*)tokens->data_ptr<int64_t>();
-  } else {
-    TORCH_CHECK(y.size(0) == M, "y rows");
-    TORCH_CHECK(w_post.has_value() && w_post->numel() == W, "w_post size");
-    CHECK_DEV(w_post.value()); CHECK_CONT(w_post.value());
-    CHECK_F32(w_post.value());
-  }
-  auto h = torch::empty({M, W}, y.options());
-  if (M > 0)
-    launch_sandwich_norm(y.data_ptr(), tok, x.data_ptr<float>(),
-                         tok ? nullptr : w_post->data_ptr<float>(),
-                         w_next.data_ptr<float>(), h.data_ptr(), M, W,
-                         (int)n, (float)eps, is_f32(y), cur_stream());
-  return h;
 }
 
 torch::Tensor latent_prep(torch::Tensor ab, int64_t QP, int64_t qn,
@@ -253,7 +204,6 @@ torch::Tensor clamped_glu(torch::Tensor gu, double limit, double alpha,
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
-  m.def("sandwich_norm", &sandwich_norm);
   m.def("latent_prep", &latent_prep);
   m.def("latent_gather", &latent_gather);
   m.def("head_gemm", &head_gemm);

@@ -1,0 +1,115 @@
+// Torch bindings of the fp32 residual stream's norms.
+#include "ext_common.h"
+
+extern "C" {
+void launch_sandwich_norm(const void*, const long*, float*, const float*,
+                          const float*, void*, int, int, int, float, bool,
+                          hipStream_t);
+void launch_embed_positions(const void*, const void*, const long*, const int*,
+                            float*, void*, int, int, int, bool, hipStream_t);
+void launch_layer_norm_add(const void*, const float*, int, float*,
+                           const float*, const float*, const float*,
+                           const float*, void*, int, int, int, float, bool,
+                           hipStream_t);
+}
+
+// y == embedding table when tokens are given
+torch::Tensor sandwich_norm(torch::Tensor y,
+                            c10::optional<torch::Tensor> tokens,
+                            torch::Tensor x,
+                            c10::optional<torch::Tensor> w_post,
+                            torch::Tensor w_next, int64_t n, double eps) {
+  CHECK_DEV(y); CHECK_CONT(y); CHECK_T(y);
+  CHECK_DEV(x); CHECK_CONT(x); CHECK_F32(x);
+  CHECK_DEV(w_next); CHECK_CONT(w_next); CHECK_F32(w_next);
+  const int M = x.size(0), W = x.size(1);
+  TORCH_CHECK(x.dim() == 2 && y.dim() == 2 && y.size(1) == W, "row sizes");
+  TORCH_CHECK(W % 8 == 0 && W <= 16384 && n > 0 && n <= W,
+              "width must be a multiple of 8, at most 16384");
+  TORCH_CHECK(w_next.numel() == W, "w_next size");
+  const long* tok = nullptr;
+  if (tokens) {
+    CHECK_DEV(tokens.value()); CHECK_CONT(tokens.value());
+    TORCH_CHECK(tokens->scalar_type() == at::kLong && tokens->numel() == M,
+                "tokens must be int64, one per row");
+    tok = (const long*)tokens->data_ptr<int64_t>();
+  } else {
+    TORCH_CHECK(y.size(0) == M, "y rows");
+    TORCH_CHECK(w_post.has_value() && w_post->numel() == W, "w_post size");
+    CHECK_DEV(w_post.value()); CHECK_CONT(w_post.value());
+    CHECK_F32(w_post.value());
+  }
+  auto h = torch::empty({M, W}, y.options());
+  if (M > 0)
+    launch_sandwich_norm(y.data_ptr(), tok, x.data_ptr<float>(),
+                         tok ? nullptr : w_post->data_ptr<float>(),
+                         w_next.data_ptr<float>(), h.data_ptr(), M, W,
+                         (int)n, (float)eps, is_f32(y), cur_stream());
+  return h;
+}
+
+torch::Tensor embed_positions(torch::Tensor tokens, torch::Tensor ctx,
+                              torch::Tensor table, torch::Tensor pos,
+                              torch::Tensor x) {
+  CHECK_DEV(table); CHECK_CONT(table); CHECK_T(table);
+  CHECK_DEV(pos); CHECK_CONT(pos); CHECK_SAME(pos, table);
+  CHECK_DEV(tokens); CHECK_CONT(tokens);
+  CHECK_DEV(ctx); CHECK_CONT(ctx); CHECK_I32(ctx);
+  CHECK_DEV(x); CHECK_CONT(x); CHECK_F32(x);
+  const int M = x.size(0), W = x.size(1);
+  TORCH_CHECK(tokens.scalar_type() == at::kLong && tokens.numel() == M &&
+                  ctx.numel() == M,
+              "tokens (int64) and ctx: one per row");
+  TORCH_CHECK(W % 8 == 0 && table.size(1) == W && pos.size(1) == W &&
+                  pos.size(0) > 0,
+              "row sizes");
+  auto h = torch::empty({M, W}, table.options());
+  if (M > 0)
+    launch_embed_positions(table.data_ptr(), pos.data_ptr(),
+                           (const long*)tokens.data_ptr<int64_t>(),
+                           ctx.data_ptr<int>(), x.data_ptr<float>(),
+                           h.data_ptr(), M, W, pos.size(0), is_f32(table),
+                           cur_stream());
+  return h;
+}
+
+static const float* norm_vec(const torch::Tensor& t, long W) {
+  CHECK_DEV(t); CHECK_CONT(t); CHECK_F32(t);
+  TORCH_CHECK(t.numel() == W, "norm size");
+  return t.data_ptr<float>();
+}
+
+torch::Tensor layer_norm_add(torch::Tensor y, torch::Tensor x,
+                             torch::Tensor w, torch::Tensor b, int64_t n,
+                             double eps, c10::optional<torch::Tensor> wf,
+                             c10::optional<torch::Tensor> bf,
+                             c10::optional<torch::Tensor> mix) {
+  CHECK_DEV(y); CHECK_CONT(y); CHECK_T(y);
+  CHECK_DEV(x); CHECK_CONT(x); CHECK_F32(x);
+  const int M = x.size(0), W = x.size(1);
+  TORCH_CHECK(x.dim() == 2 && y.dim() == 2 && y.size(1) == W, "row sizes");
+  TORCH_CHECK(W % 8 == 0 && W <= 16384 && n > 0 && n <= W,
+              "width must be a multiple of 8, at most 16384");
+  TORCH_CHECK(wf.has_value() == bf.has_value(), "final weight and bias");
+  int top = 1;
+  if (mix) {
+    CHECK_DEV(mix.value()); CHECK_CONT(mix.value()); CHECK_F32(mix.value());
+    TORCH_CHECK(mix->dim() == 2 && mix->size(0) == M, "mix rows");
+    top = mix->size(1);
+  }
+  TORCH_CHECK(y.size(0) == (long)M * top, "y rows");
+  auto h = torch::empty({M, W}, y.options());
+  if (M > 0)
+    launch_layer_norm_add(y.data_ptr(), mix ? mix->data_ptr<float>() : nullptr,
+                          top, x.data_ptr<float>(), norm_vec(w, W),
+                          norm_vec(b, W), wf ? norm_vec(*wf, W) : nullptr,
+                          bf ? norm_vec(*bf, W) : nullptr, h.data_ptr(), M, W,
+                          (int)n, (float)eps, is_f32(y), cur_stream());
+  return h;
+}
+
+PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
+  m.def("sandwich_norm", &sandwich_norm);
+  m.def("embed_positions", &embed_positions);
+  m.def("layer_norm_add", &layer_norm_add);
+}

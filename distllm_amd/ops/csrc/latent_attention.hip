@@ -21,13 +21,6 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 
 extern __shared__ __attribute__((aligned(16))) char smem[];
 
-__device__ __forceinline__ float to_f(unsigned short v) { return bf2f(v); }
-__device__ __forceinline__ float to_f(float v) { return v; }
-__device__ __forceinline__ void from_f(unsigned short* p, float v) {
-  *p = f2bf(v);
-}
-__device__ __forceinline__ void from_f(float* p, float v) { *p = v; }
-
 // ---- norm of the two down-projections + cache write ----------------------
 // ab [M, QP (+ R)]: wave 0 of a workgroup norms the query latent (first QP
 // columns, true size qn), wave 1 the cached latent (next R columns, true

@@ -10,7 +10,8 @@ from __future__ import annotations
 
 import importlib
 
-EXTENSIONS = ("_hip_gemm", "_hip_latent", "_hip_ops")
+EXTENSIONS = ("_hip_gemm", "_hip_residual", "_hip_latent", "_hip_hybrid",
+              "_hip_ops")
 
 
 class Native:

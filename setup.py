@@ -5,9 +5,11 @@
 The kernels are grouped into a few extensions, so that a process which
 needs one group does not have to compile the others:
 
-    _hip_gemm    matrix products (every model)
-    _hip_latent  latent attention, sandwich norms, clamped GLU
-    _hip_ops     everything else
+    _hip_gemm      matrix products (every model)
+    _hip_residual  norms around an fp32 residual stream
+    _hip_latent    latent attention, clamped GLU
+    _hip_hybrid    chunked attention, delta rule, xIELU, routed experts
+    _hip_ops       everything else
 
 DISTLLM_EXT=_hip_gemm,_hip_latent restricts a build to the named ones.
 The resulting distllm_amd/ops/_hip_*.so are git-ignored.
@@ -27,7 +29,11 @@ GROUPS = {
                   "gemm16.hip", "decode_gemm.hip"],
     "_hip_latent": ["ext_latent.cpp", "latent_attention.hip",
                     "latent_decode.hip", "window_attention.hip",
-                    "sandwich_norm.hip", "clamped_glu.hip"],
+                    "clamped_glu.hip"],
+    "_hip_residual": ["ext_residual.cpp", "residual_norms.hip"],
+    "_hip_hybrid": ["ext_hybrid.cpp", "chunk_attention.hip",
+                    "chunk_flash.hip", "delta_rule.hip", "experts.hip",
+                    "xielu.hip"],
 }
 _taken = {s for group in GROUPS.values() for s in group}
 # *_hip.hip files are torch-hipify build artifacts — exclude them.
