@@ -191,3 +191,98 @@ def forward(config, tensors, tokens, trace=None):
             trace.append(x)
     x = layer_norm(x, t["final.norm"], t["final.norm.b"], eps)
     return x @ t["head"].T
+
+
+# ---- random models ---------------------------------------------------------
+
+def make_config(layers, width=48, vocab=97, eps=1e-5, max_positions=512):
+    return {"architecture": "Bufulorn", "width": width, "vocab": vocab,
+            "norm": {"eps": eps}, "max_positions": max_positions,
+            "layers": layers}
+
+
+def dense_mlp(ff=56):
+    return {"kind": "dense", "ff": ff}
+
+
+def moe_mlp(ff=40, experts=6, top=2, count=3, keep=2):
+    return {"kind": "moe", "expert": {"ff": ff},
+            "router": {"experts": experts, "top": top,
+                       "groups": {"count": count, "keep": keep}}}
+
+
+def attention_layer(mlp, heads=4, kv_heads=2, dim=16, vdim=24, size=20,
+                    scale=0.25, softcap=20.0, kv_from=None):
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim,
+         "mask": {"size": size}, "scale": scale, "softcap": softcap}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "attention", "mixer": m, "mlp": mlp}
+
+
+def delta_layer(mlp, heads=4, kv_heads=2, dim=16, vdim=24, conv=4):
+    return {"type": "delta", "mlp": mlp,
+            "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim,
+                      "vdim": vdim, "conv": conv}}
+
+
+def make_tensors(config, seed=0, gain=1.0, router=5.0):
+    """Random weights of a config, rounded to bfloat16 so that every dtype
+    under test starts from the same numbers. `gain` scales the queries:
+    larger values make attention peaky, so that a wrong key shows. So does
+    `router` with the routers' choices."""
+    g = torch.Generator().manual_seed(seed)
+    W, V = config["width"], config["vocab"]
+    t = {}
+
+    def lin(name, out, inp, s=1.0):
+        t[name] = torch.randn(out, inp, generator=g) * (s / math.sqrt(inp))
+
+    def vec(name, n, mid=1.0, spread=0.3):
+        t[name] = mid + spread * torch.randn(n, generator=g)
+
+    def bias(name, n):
+        vec(name + ".b", n, 0.0, 0.3)
+
+    t["embed"] = torch.randn(V, W, generator=g)
+    t["pos"] = 0.7 * torch.randn(config["max_positions"], W, generator=g)
+    for i, layer in enumerate(config["layers"]):
+        p, m = f"l{i}.mix.", layer["mixer"]
+        H, G, d, e = m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        if layer["type"] == "attention":
+            lin(p + "q", H * d, W), bias(p + "q", H * d)
+            vec(p + "q.norm", d, gain)
+            if m.get("kv_from") is None:
+                lin(p + "k", G * d, W), bias(p + "k", G * d)
+                lin(p + "v", G * e, W), bias(p + "v", G * e)
+                vec(p + "k.norm", d)
+            t[p + "r1"] = torch.rand(H, generator=g) * 2
+            t[p + "r2"] = torch.rand(H, generator=g)
+        else:
+            for n, c in (("q", G * d), ("k", G * d), ("v", H * e)):
+                lin(p + n, c, W)
+                t[p + n + ".conv"] = torch.randn(c, m["conv"], generator=g) \
+                    / math.sqrt(m["conv"])
+            lin(p + "b", H, W), lin(p + "a", H, W)
+            vec(p + "A_log", H, -1.5), vec(p + "dt_bias", H, -1.0)
+            vec(p + "norm", e)
+        lin(p + "g", H * e, W)
+        lin(p + "o", W, H * e)
+        vec(f"l{i}.norm1", W), bias(f"l{i}.norm1", W)
+        f, p = layer["mlp"], f"l{i}.mlp."
+        if f is None:
+            continue
+        vec(f"l{i}.norm2", W), bias(f"l{i}.norm2", W)
+        if f["kind"] == "dense":
+            lin(p + "up", f["ff"], W, 2.0)
+            lin(p + "down", W, f["ff"])
+            vec(p + "act", 2, 0.2, 0.5)
+        else:
+            for n in range(f["router"]["experts"]):
+                lin(f"{p}e{n}.gate", f["expert"]["ff"], W, 2.0)
+                lin(f"{p}e{n}.up", f["expert"]["ff"], W)
+                lin(f"{p}e{n}.down", W, f["expert"]["ff"])
+            lin(p + "router", f["router"]["experts"], W, router)
+    vec("final.norm", W), bias("final.norm", W)
+    lin("head", V, W)
+    return {k: v.to(torch.bfloat16) for k, v in t.items()}
