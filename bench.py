@@ -39,8 +39,8 @@ def main() -> None:
                          "tokens/s (Llama-class, paged KV); pipeline = "
                          "full jsonl_chunk -> semantic_chunk embed -> "
                          "write (tokenizer + staging included); "
-                         "decoders = prefill and decode of latent-"
-                         "attention layers beside llama layers of equal "
+                         "decoders = prefill and decode of Kanotar "
+                         "and Bufulorn layers beside llama layers of equal "
                          "size")
     ap.add_argument("--docs-per-file", type=int, default=128)
     ap.add_argument("--pooler", type=str, default="mean",
@@ -246,14 +246,16 @@ def bench_generate(args) -> None:
 
 
 def bench_decoders(args) -> None:
-    """Kanotar layers beside llama layers of the same width, heads and
-    feed-forward, through the same engine: tokens/s of prefilling a batch
-    of prompts and of decoding at a given context, both models in turn.
-    Random weights, synthetic tokens, one GPU."""
+    """Kanotar and Bufulorn layers beside llama layers of the same width,
+    heads and (active) feed-forward weights, through the same engine:
+    tokens/s of prefilling a batch of prompts and of decoding at a given
+    context, both models in turn. Random weights, synthetic tokens, one
+    GPU."""
     from distllm_amd.engine import LLMEngine, SamplingParams
     from distllm_amd.engine.engine import _Seq
     from distllm_amd.models import ModelDims, build_model
-    from distllm_amd.models.config import layered_preset
+    from distllm_amd.models.config import (ExpertsDims, hybrid_preset,
+                                           layered_preset)
 
     dev = "cuda:0"
     torch.manual_seed(5)
@@ -269,7 +271,13 @@ def bench_decoders(args) -> None:
         return layered_preset(args.layers, hidden, V, heads, 128, 128,
                               q_rank, kv_rank, ff, [window], share)
 
-    # name: (kanotar, llama, [(prompts, prompt len)], [(batch, context)])
+    def bufulorn(hidden, heads, kv, ff, chunk, order="A", **kw):
+        # two matrices per dense feed-forward where llama has three
+        return hybrid_preset(args.layers, hidden, V, heads, kv, 128,
+                             ff * 3 // 2, chunk, order=order, **kw)
+
+    # name: (model, llama, [(prompts, prompt len)], [(batch, context)])
+    some = [(16, 2048)], [(1, 2048), (32, 2048), (128, 2048)]
     sizes = {
         "4096x32h full": (
             kanotar(4096, 32, 1536, 512, 14336, 8192),
@@ -286,14 +294,27 @@ def bench_decoders(args) -> None:
         "7168x64h shared latents": (
             kanotar(7168, 64, 1536, 512, 18432, 8192, args.layers // 2),
             llama(7168, 56, 8, 18432), [(8, 2048)], [(32, 2048)]),
+        "4096x32h attention": (
+            bufulorn(4096, 32, 8, 14336, 8192), llama(4096, 32, 8, 14336),
+            [(16, 2048), (2, 8000)], [(1, 2048), (32, 2048), (128, 2048),
+                                      (32, 8000)]),
+        "4096x32h attention and delta": (
+            bufulorn(4096, 32, 8, 14336, 1024, "AD"),
+            llama(4096, 32, 8, 14336), some[0] + [(2, 8000)], some[1]),
+        # 8 of 64 experts of 1024: the active weights of one of 8192
+        "2048x16h experts": (
+            bufulorn(2048, 16, 4, 8192, 4096, "AAD", share=True,
+                     experts=ExpertsDims(ff=1024, experts=64, top=8,
+                                         groups=8, keep=4)),
+            llama(2048, 16, 4, 8192), *some),
     }
     params = SamplingParams(temperature=0.0, min_p=0.0, max_tokens=10 ** 6)
     rows = []
-    for name, (kd, ld, prefills, decodes) in sizes.items():
+    for name, (md, ld, prefills, decodes) in sizes.items():
         if args.only and name.split()[0] not in args.only.split(",") \
                 and name not in args.only.split(","):
             continue
-        models = {"kanotar": build_model(kd, device=dev),
+        models = {md.arch: build_model(md, device=dev),
                   "llama": build_model(ld, device=dev)}
 
         def run(kind, model, batch, ctx):
