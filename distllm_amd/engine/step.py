@@ -58,12 +58,35 @@ class PromptBlocks:
 
 @dataclass
 class Segments:
-    """Rows of each block-table row, and its state slot."""
+    """Rows of each block-table row, and its state slot. Segments of more
+    than SHORT rows are also described in chunks of CHUNK rows, for
+    kernels that work chunk by chunk."""
 
     row0: torch.Tensor       # [S] int32
     rows: torch.Tensor       # [S] int32
     slot: torch.Tensor       # [S] int32
     longest: int
+    longs: torch.Tensor | None = None   # [P, 2] segment, its first chunk
+    chunks: torch.Tensor | None = None  # [N, 2] segment, chunk in it
+
+    SHORT = 16
+    CHUNK = 32
+
+    @classmethod
+    def build(cls, row0, rows, slots, device) -> "Segments":
+        def up(a, *shape):
+            return torch.from_numpy(
+                np.array(a, np.int32).reshape(*shape)).to(device)
+
+        longs, chunks = [], []
+        for i, n in enumerate(rows):
+            if n > cls.SHORT:
+                longs.append((i, len(chunks)))
+                chunks += [(i, c) for c in range(-(-n // cls.CHUNK))]
+        return cls(up(row0, -1), up(rows, -1), up(slots, -1),
+                   max(rows, default=0),
+                   up(longs, -1, 2) if longs else None,
+                   up(chunks, -1, 2) if longs else None)
 
 
 @dataclass
@@ -131,11 +154,8 @@ class StepBatch:
 
         seg = None
         if slots is not None:
-            seg = Segments(up(np.array([r[0] if len(r) else 0 for r in rows],
-                                       np.int32)),
-                           up(np.array([len(r) for r in rows], np.int32)),
-                           up(np.array(slots, np.int32)),
-                           max((len(r) for r in rows), default=0))
+            seg = Segments.build([r[0] if len(r) else 0 for r in rows],
+                                 [len(r) for r in rows], slots, device)
 
         return cls(tokens=up(tokens), ctx=up(ctx), row_seq=up(row_seq),
                    block_table=up(table),

@@ -697,7 +697,8 @@ def gated_delta(ab, heads, kv_heads, dp, vp, dim, vdim, conv_w, decay,
         return _hip_ops.gated_delta(
             ab, heads, kv_heads, dp, vp, dim, vdim, conv_w, decay, o_norm,
             unit_eps, eps, state, conv, segments.row0, segments.rows,
-            segments.slot, segments.longest, row_seq, ctx)
+            segments.slot, segments.longest, row_seq, ctx, segments.longs,
+            segments.chunks, segments.SHORT)
     return torch_ref.gated_delta(
         ab, heads, kv_heads, dp, vp, dim, vdim, conv_w, decay, o_norm,
         unit_eps, eps, state, conv, segments, row_seq, ctx)

@@ -7,36 +7,11 @@ extern __shared__ __attribute__((aligned(16))) char smem[];
 
 // ---- norm of query and key heads, cache write -----------------------------
 // ab row: H query heads of dp, then (own keys) G key heads of dp and G value
-// heads of vp. LPH lanes share a query or key head. Values: the first row of
-// a run of consecutive positions in one page writes the run, whole 32-byte
-// page rows where the run covers the page.
-template <typename T, int LPH>
-__device__ __forceinline__ void norm_head(const T* __restrict__ src,
-                                          const float* __restrict__ w,
-                                          T* __restrict__ dst, int dp, int n,
-                                          float eps, int sub) {
-  float ss = 0.f;
-  for (int c = sub * 8; c < dp; c += LPH * 8) {
-    float v[8];
-    load8<T>(src + c, v);
-#pragma unroll
-    for (int i = 0; i < 8; ++i) ss += v[i] * v[i];
-  }
-#pragma unroll
-  for (int off = LPH / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
-  const float inv = 1.f / sqrtf(ss / n + eps);
-  if (dst == nullptr) return;
-  for (int c = sub * 8; c < dp; c += LPH * 8) {
-    float v[8], wv[8];
-    load8<T>(src + c, v);
-    load8<float>(w + c, wv);
-#pragma unroll
-    for (int i = 0; i < 8; ++i) v[i] *= inv * wv[i];
-    store8(dst + c, v);
-  }
-}
-
-template <typename T, int LPH>
+// heads of vp. LPH lanes share a query or key head, a workgroup norms UN
+// times 256 / LPH of them. Values: the first row of a run of consecutive
+// positions in one page writes the run, whole 32-byte page rows where the
+// run covers the page; a wave looks at VR rows of one head.
+template <typename T, int LPH, int UN>
 __global__ void __launch_bounds__(256)
 attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
                  int dp, int vp, int n, const float* __restrict__ wq,
@@ -44,7 +19,7 @@ attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
                  T* __restrict__ kpages, T* __restrict__ vpages,
                  const int* __restrict__ block_table, int max_blocks,
                  int num_blocks, const int* __restrict__ row_seq,
-                 const int* __restrict__ ctx, int norm_wgs) {
+                 const int* __restrict__ ctx, int norm_wgs, int VR) {
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   // page of a position, or -1
   auto page_of = [&](int row, int pos) {
@@ -53,52 +28,110 @@ attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
     return b >= 0 && b < num_blocks ? b : -1;
   };
   if ((int)blockIdx.x < norm_wgs) {
+    constexpr int UPI = 256 / LPH;
     const int units = H + (kpages != nullptr ? G : 0);
-    const long u = (long)blockIdx.x * (256 / LPH) + threadIdx.x / LPH;
-    if (u >= (long)M * units) return;  // whole LPH groups
-    const int row = (int)(u / units), hd = (int)(u % units);
-    const bool key = hd >= H;
-    T* dst = q + ((long)row * H + hd) * dp;
-    if (key) {
-      const int pos = ctx[row] - 1, page = page_of(row, pos);
-      dst = page < 0 ? nullptr
-                     : kpages + (((long)page * G + hd - H) * PBLK +
-                                 pos % PBLK) * dp;
+    const int total = M * units;  // the host checks that it fits
+    const int c0 = threadIdx.x % LPH * 8;
+    const int u0 = blockIdx.x * UPI * UN + threadIdx.x / LPH;
+    // a unit's head starts at (row, hd); its lanes' first eight columns
+    // stay in registers, heads of more than 512 read the others twice
+    float v[UN][8];
+#pragma unroll
+    for (int k = 0; k < UN; ++k) {
+      const int u = min(u0 + k * UPI, total - 1);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] = 0.f;
+      if (c0 < dp)
+        load8<T>(ab + (long)(u / units) * ld + (long)(u % units) * dp + c0,
+                 v[k]);
     }
-    norm_head<T, LPH>(ab + (long)row * ld + (long)hd * dp, key ? wk : wq,
-                      dst, dp, n, eps, threadIdx.x % LPH);
+#pragma unroll
+    for (int k = 0; k < UN; ++k) {
+      const int u = u0 + k * UPI;
+      if (u >= total) return;  // whole LPH groups
+      const int row = u / units, hd = u % units;
+      const T* src = ab + (long)row * ld + (long)hd * dp;
+      const float* w = hd >= H ? wk : wq;
+      float ss = 0.f;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss += v[k][i] * v[k][i];
+      for (int c = c0 + LPH * 8; c < dp; c += LPH * 8) {
+        float x[8];
+        load8<T>(src + c, x);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
+      }
+#pragma unroll
+      for (int off = LPH / 2; off > 0; off >>= 1)
+        ss += __shfl_xor(ss, off, 64);
+      const float inv = 1.f / sqrtf(ss / n + eps);
+      T* dst = q + ((long)row * H + hd) * dp;
+      if (hd >= H) {
+        const int pos = ctx[row] - 1, page = page_of(row, pos);
+        if (page < 0) continue;
+        dst = kpages +
+              (((long)page * G + hd - H) * PBLK + pos % PBLK) * dp;
+      }
+      for (int c = c0; c < dp; c += LPH * 8) {
+        float x[8], wv[8];
+        if (c != c0) load8<T>(src + c, v[k]);
+        load8<float>(w + c, wv);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) x[i] = v[k][i] * inv * wv[i];
+        store8(dst + c, x);
+      }
+    }
     return;
   }
-  // values: one wave per (row, head)
   const long u = ((long)blockIdx.x - norm_wgs) * 4 + wid;
-  if (u >= (long)M * G) return;
-  const int row = (int)(u / G), g = (int)(u % G);
-  const int pos = ctx[row] - 1;
-  if (pos < 0) return;
-  const int seq = row_seq[row];
-  const bool first = pos % PBLK == 0 || row == 0 ||
-                     row_seq[row - 1] != seq || ctx[row - 1] != ctx[row] - 1;
-  if (!first) return;
-  const int page = page_of(row, pos);
-  if (page < 0) return;
-  int run = 1;
-  while (pos % PBLK + run < PBLK && row + run < M &&
-         row_seq[row + run] == seq && ctx[row + run] == ctx[row] + run)
-    ++run;
-  const T* src = ab + (long)row * ld + (long)(H + G) * dp + (long)g * vp;
-  T* dst = vpages + ((long)page * G + g) * vp * PBLK;
-  for (int c = lane; c < vp; c += 64) {
-    if (run == PBLK) {
-      T v[PBLK];
+  const int r0 = (int)(u / G) * VR, g = (int)(u % G);
+  if (r0 >= M) return;
+  bool first = false;
+  if (lane < VR && r0 + lane < M) {
+    const int row = r0 + lane, pos = ctx[row] - 1;
+    first = pos >= 0 && (pos % PBLK == 0 || row == 0 ||
+                         row_seq[row - 1] != row_seq[row] ||
+                         ctx[row - 1] != pos);
+  }
+  for (unsigned long long todo = __ballot(first); todo != 0;
+       todo &= todo - 1) {
+    const int row = r0 + __builtin_ctzll(todo);
+    const int pos = ctx[row] - 1, seq = row_seq[row];
+    const int page = page_of(row, pos);
+    if (page < 0) continue;
+    int run = 1;
+    while (pos % PBLK + run < PBLK && row + run < M &&
+           row_seq[row + run] == seq && ctx[row + run] == ctx[row] + run)
+      ++run;
+    const T* src = ab + (long)row * ld + (long)(H + G) * dp + (long)g * vp;
+    T* dst = vpages + ((long)page * G + g) * vp * PBLK;
+    for (int c = lane * 2; c < vp; c += 128) {
+      typedef __attribute__((ext_vector_type(2))) T pair;
+      if (run == PBLK) {
+        pair v[PBLK];
 #pragma unroll
-      for (int j = 0; j < PBLK; ++j) v[j] = src[(long)j * ld + c];
-      T* d = dst + (long)c * PBLK;
+        for (int j = 0; j < PBLK; ++j)
+          v[j] = *reinterpret_cast<const pair*>(src + (long)j * ld + c);
 #pragma unroll
-      for (int j = 0; j < PBLK * (int)sizeof(T) / 16; ++j)
-        reinterpret_cast<i32x4*>(d)[j] = reinterpret_cast<const i32x4*>(v)[j];
-    } else {
-      for (int j = 0; j < run; ++j)
-        dst[(long)c * PBLK + pos % PBLK + j] = src[(long)j * ld + c];
+        for (int h = 0; h < 2; ++h) {
+          T t[PBLK];
+#pragma unroll
+          for (int j = 0; j < PBLK; ++j) t[j] = v[j][h];
+          T* d = dst + (long)(c + h) * PBLK;
+#pragma unroll
+          for (int j = 0; j < PBLK * (int)sizeof(T) / 16; ++j)
+            reinterpret_cast<i32x4*>(d)[j] =
+                reinterpret_cast<const i32x4*>(t)[j];
+        }
+      } else {
+        for (int j = 0; j < run; ++j) {
+          const pair v =
+              *reinterpret_cast<const pair*>(src + (long)j * ld + c);
+          T* d = dst + (long)c * PBLK + pos % PBLK + j;
+          d[0] = v[0];
+          d[PBLK] = v[1];
+        }
+      }
     }
   }
 }
@@ -111,24 +144,32 @@ extern "C" void launch_attn_prep(
   const int lph = dp <= 64 ? 8 : dp <= 128 ? 16 : dp <= 256 ? 32 : 64;
   const bool own = kpages != nullptr;
   const long units = (long)M * (H + (own ? G : 0));
-  const int norm_wgs = (int)((units + 256 / lph - 1) / (256 / lph));
-  const int v_wgs = own ? (int)(((long)M * G + 3) / 4) : 0;
-#define APK(T, L)                                                             \
-  hipLaunchKernelGGL((attn_prep_kernel<T, L>), dim3(norm_wgs + v_wgs),        \
+  const int un = units >= 65536 ? 4 : 1, vr = M >= 2048 ? 16 : 1;
+  const int per = 256 / lph * un;
+  const int norm_wgs = (int)((units + per - 1) / per);
+  const int v_wgs = own ? (int)(((long)(M + vr - 1) / vr * G + 3) / 4) : 0;
+#define APK(T, L, U)                                                          \
+  hipLaunchKernelGGL((attn_prep_kernel<T, L, U>), dim3(norm_wgs + v_wgs),     \
                      dim3(256), 0, stream, (const T*)ab, ld, M, H, G, dp, vp, \
                      n, wq, wk, eps, (T*)q, (T*)kpages, (T*)vpages,           \
                      block_table, max_blocks, num_blocks, row_seq, ctx,       \
-                     norm_wgs)
+                     norm_wgs, vr)
+#define APK_U(T, L)           \
+  do {                        \
+    if (un == 1) APK(T, L, 1); \
+    else APK(T, L, 4);        \
+  } while (0)
 #define APK_L(T)                 \
   do {                           \
-    if (lph == 8) APK(T, 8);     \
-    else if (lph == 16) APK(T, 16); \
-    else if (lph == 32) APK(T, 32); \
-    else APK(T, 64);             \
+    if (lph == 8) APK_U(T, 8);   \
+    else if (lph == 16) APK_U(T, 16); \
+    else if (lph == 32) APK_U(T, 32); \
+    else APK_U(T, 64);           \
   } while (0)
   if (fp32) APK_L(float);
   else APK_L(unsigned short);
 #undef APK_L
+#undef APK_U
 #undef APK
 }
 

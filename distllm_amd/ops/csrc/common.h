@@ -51,6 +51,13 @@ __device__ __forceinline__ float wave_reduce_max(float v) {
   return v;
 }
 
+// Order one wave's LDS accesses across its lanes.
+__device__ __forceinline__ void wave_sync() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+  __builtin_amdgcn_wave_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+}
+
 // Block-level reduce across NW waves using LDS scratch (NW <= 16).
 template <int NW>
 __device__ __forceinline__ float block_reduce_sum(float v, float* lds_scratch) {

@@ -18,113 +18,150 @@ __device__ __forceinline__ float act_silu(float z) {
 }
 
 // ---- convolutions, unit queries and keys, decays ---------------------------
-// One wave per (run of `rb` rows, unit); units: 2G query/key heads, H value
-// heads, one for all scalars. A lane owns CPL channels of its head. shift:
-// every segment has one row, and the wave renews its channels of the
-// convolution slot itself (else conv_state_kernel does).
-template <typename T, int CPL>
-__device__ __forceinline__ void conv_unit(
-    const T* __restrict__ ab, int ld, int M, int C, int ch0, int unit_kind,
-    int unit, int G, int dp, int vp, const float* __restrict__ conv_w,
-    int taps, float q_scale, float unit_eps, float* __restrict__ qk,
-    T* __restrict__ v, int H, T* __restrict__ conv,
-    const int* __restrict__ seg_row0, const int* __restrict__ seg_slot,
-    const int* __restrict__ row_seq, const int* __restrict__ ctx, int r0,
-    int rb, bool shift, int lane) {
-  const int ch = ch0 + lane * CPL;
-  for (int row = r0; row < min(r0 + rb, M); ++row) {
-    const int pos = ctx[row] - 1;
-    if (pos < 0) continue;
-    const int seg = row_seq[row];
-    const int o = row - seg_row0[seg];  // offset in its segment
-    T* slot = conv + (long)seg_slot[seg] * (taps - 1) * C + ch;
-    float z[CPL];
+// A unit is a query, key or value head over a run of `rb` rows; LPH lanes of
+// eight channels each share it. The window of inputs stays in registers
+// from row to row. TAPS: 0 for any number, at the price of reading every
+// input of every row. shift: every segment has one row, and the unit renews
+// its channels of the convolution slot itself (else conv_state_kernel does).
+template <typename T>
+struct ConvArgs {
+  const T* ab;
+  int ld, M, C, taps, rb;
+  const float* w;
+  T* conv;
+  const int *seg_row0, *seg_slot, *row_seq, *ctx;
+  bool shift;
+};
+
+// input j rows before `row`, as fp32; zeros before the start
+template <typename T>
+__device__ __forceinline__ void conv_input(const ConvArgs<T>& a, int row,
+                                           int pos, int o, const T* slot,
+                                           int ch, int j, float* x) {
 #pragma unroll
-    for (int i = 0; i < CPL; ++i) z[i] = 0.f;
-    // tap `taps - 1 - j` meets the input j rows back
-    for (int j = taps - 1; j >= 0; --j) {
-      if (pos - j < 0) continue;  // before the start
-      const T* src = o >= j ? ab + (long)(row - j) * ld + ch
-                            : slot + (long)(taps - 1 + o - j) * C;
-      const float* w = conv_w + (long)(taps - 1 - j) * C + ch;
+  for (int i = 0; i < 8; ++i) x[i] = 0.f;
+  if (pos < j) return;
+  load8<T>(o >= j ? a.ab + (long)(row - j) * a.ld + ch
+                  : slot + (long)(a.taps - 1 + o - j) * a.C,
+           x);
+}
+
+template <typename T, int LPH, int TAPS, bool QK>
+__device__ __forceinline__ void conv_unit(const ConvArgs<T>& a, int unit,
+                                          int r0, int sub, int ch0, int G,
+                                          int H, float q_scale,
+                                          float unit_eps, float* qk, T* v) {
+  constexpr int D = LPH * 8;
+  constexpr int NT = TAPS > 0 ? TAPS : 1;
+  const int ch = ch0 + sub * 8;
+  float w[NT][8], x[NT][8];  // x[j]: the input j rows back
+  if (TAPS > 0)
 #pragma unroll
-      for (int i = 0; i < CPL; ++i) z[i] += to_f(src[i]) * w[i];
+    for (int j = 0; j < NT; ++j)
+      load8<float>(a.w + (long)(NT - 1 - j) * a.C + ch, w[j]);
+  int before = -1;  // sequence of the previous row
+  for (int row = r0; row < min(r0 + a.rb, a.M); ++row) {
+    const int pos = a.ctx[row] - 1;
+    if (pos < 0) {
+      before = -1;
+      continue;
     }
-    if (shift) {
-      for (int j = 0; j < taps - 2; ++j)
+    const int seg = a.row_seq[row];
+    const int o = row - a.seg_row0[seg];  // offset in its segment
+    T* slot = a.conv + (long)a.seg_slot[seg] * (a.taps - 1) * a.C + ch;
+    float z[8];
 #pragma unroll
-        for (int i = 0; i < CPL; ++i)
-          slot[(long)j * C + i] = slot[(long)(j + 1) * C + i];
-      if (taps > 1)
+    for (int i = 0; i < 8; ++i) z[i] = 0.f;
+    if (TAPS > 0) {
 #pragma unroll
-        for (int i = 0; i < CPL; ++i)
-          slot[(long)(taps - 2) * C + i] = ab[(long)row * ld + ch + i];
+      for (int j = NT - 1; j > 0; --j) {
+        if (seg == before)
+#pragma unroll
+          for (int i = 0; i < 8; ++i) x[j][i] = x[j - 1][i];
+        else
+          conv_input(a, row, pos, o, slot, ch, j, x[j]);
+      }
+      load8<T>(a.ab + (long)row * a.ld + ch, x[0]);
+#pragma unroll
+      for (int j = NT - 1; j >= 0; --j)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) z[i] += x[j][i] * w[j][i];
+    } else {
+      for (int j = a.taps - 1; j >= 0; --j) {
+        conv_input(a, row, pos, o, slot, ch, j, x[0]);
+        load8<float>(a.w + (long)(a.taps - 1 - j) * a.C + ch, w[0]);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) z[i] += x[0][i] * w[0][i];
+      }
+    }
+    before = seg;
+    if (a.shift && a.taps > 1) {
+      float t[8];
+      for (int j = 0; j < a.taps - 2; ++j) {
+        load8<T>(slot + (long)(j + 1) * a.C, t);
+        store8(slot + (long)j * a.C, t);
+      }
+      load8<T>(a.ab + (long)row * a.ld + ch, t);
+      store8(slot + (long)(a.taps - 2) * a.C, t);
     }
 #pragma unroll
-    for (int i = 0; i < CPL; ++i) z[i] = act_silu<T>(z[i]);
-    if (unit_kind == 0) {  // query or key head
+    for (int i = 0; i < 8; ++i) z[i] = act_silu<T>(z[i]);
+    if (QK) {
       float ss = 0.f;
 #pragma unroll
-      for (int i = 0; i < CPL; ++i) ss += z[i] * z[i];
-      ss = wave_reduce_sum(ss);
-      const float inv =
-          (unit < G ? q_scale : 1.f) / sqrtf(ss + unit_eps);
-      float* dst = qk + ((long)row * 2 * G + unit) * dp + lane * CPL;
+      for (int i = 0; i < 8; ++i) ss += z[i] * z[i];
 #pragma unroll
-      for (int i = 0; i < CPL; ++i) dst[i] = z[i] * inv;
+      for (int off = LPH / 2; off > 0; off >>= 1)
+        ss += __shfl_xor(ss, off, 64);
+      const float inv = (unit < G ? q_scale : 1.f) / sqrtf(ss + unit_eps);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) z[i] *= inv;
+      store8(qk + ((long)row * 2 * G + unit) * D + sub * 8, z);
     } else {
-      T* dst = v + ((long)row * H + unit) * vp + lane * CPL;
-#pragma unroll
-      for (int i = 0; i < CPL; ++i) from_f(dst + i, z[i]);
+      store8(v + ((long)row * H + unit) * D + sub * 8, z);
     }
   }
 }
 
-template <typename T>
+// workgroups: first those of query and key heads, then of value heads, then
+// one thread per (row, head) for decays and step sizes
+template <typename T, int LQ, int LV, int TAPS>
 __global__ void __launch_bounds__(256)
-delta_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
-                  int dp, int vp, const float* __restrict__ conv_w, int taps,
-                  const float* __restrict__ decay, float q_scale,
-                  float unit_eps, float* __restrict__ qk, T* __restrict__ v,
-                  float* __restrict__ gb, T* __restrict__ conv,
-                  const int* __restrict__ seg_row0,
-                  const int* __restrict__ seg_slot,
-                  const int* __restrict__ row_seq,
-                  const int* __restrict__ ctx, int rb, bool shift) {
-  const int lane = threadIdx.x & 63;
-  const int units = 2 * G + H + 1;
-  const long w = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
-  const int unit = (int)(w % units);
-  const int r0 = (int)(w / units) * rb;
-  if (r0 >= M) return;
-  const int C = 2 * G * dp + H * vp;
-  if (unit == units - 1) {
-    const int ba = C + H * vp;
-    for (int row = r0; row < min(r0 + rb, M); ++row) {
-      if (ctx[row] <= 0) continue;
-      for (int h = lane; h < H; h += 64) {
-        const float b = to_f(ab[(long)row * ld + ba + h]);
-        const float a = to_f(ab[(long)row * ld + ba + H + h]);
-        // log of the decay, and the step size
-        gb[((long)row * H + h) * 2] =
-            -expf(decay[h]) * softplus_exact(a + decay[H + h]);
-        gb[((long)row * H + h) * 2 + 1] = sigmoid_exact(b);
-      }
-    }
+delta_prep_kernel(ConvArgs<T> a, int H, int G, const float* __restrict__ decay,
+                  float q_scale, float unit_eps, float* __restrict__ qk,
+                  T* __restrict__ v, float* __restrict__ gb, int wg_qk,
+                  int wg_v) {
+  const int runs = (a.M + a.rb - 1) / a.rb;
+  int wg = blockIdx.x;
+  if (wg < wg_qk) {
+    const long u = (long)wg * (256 / LQ) + threadIdx.x / LQ;
+    if (u >= (long)runs * 2 * G) return;  // whole units
+    const int unit = (int)(u % (2 * G));
+    conv_unit<T, LQ, TAPS, true>(a, unit, (int)(u / (2 * G)) * a.rb,
+                                 threadIdx.x % LQ, unit * LQ * 8, G, H,
+                                 q_scale, unit_eps, qk, v);
     return;
   }
-  const bool head_qk = unit < 2 * G;
-  const int u = head_qk ? unit : unit - 2 * G;
-  const int ch0 = head_qk ? u * dp : 2 * G * dp + u * vp;
-  const int cpl = (head_qk ? dp : vp) / 64;
-#define CONV(N)                                                              \
-  conv_unit<T, N>(ab, ld, M, C, ch0, head_qk ? 0 : 1, u, G, dp, vp, conv_w,  \
-                  taps, q_scale, unit_eps, qk, v, H, conv, seg_row0,         \
-                  seg_slot, row_seq, ctx, r0, rb, shift, lane)
-  if (cpl == 1) CONV(1);
-  else if (cpl == 2) CONV(2);
-  else CONV(4);
-#undef CONV
+  wg -= wg_qk;
+  if (wg < wg_v) {
+    const long u = (long)wg * (256 / LV) + threadIdx.x / LV;
+    if (u >= (long)runs * H) return;
+    const int unit = (int)(u % H);
+    conv_unit<T, LV, TAPS, false>(
+        a, unit, (int)(u / H) * a.rb, threadIdx.x % LV,
+        2 * G * LQ * 8 + unit * LV * 8, G, H, q_scale, unit_eps, qk, v);
+    return;
+  }
+  wg -= wg_v;
+  const long i = (long)wg * 256 + threadIdx.x;
+  if (i >= (long)a.M * H) return;
+  const int row = (int)(i / H), h = (int)(i % H);
+  if (a.ctx[row] <= 0) return;
+  const T* ba = a.ab + (long)row * a.ld + a.C + H * LV * 8;
+  // log of the decay, and the step size
+  gb[i * 2] =
+      -expf(decay[h]) * softplus_exact(to_f(ba[H + h]) + decay[H + h]);
+  gb[i * 2 + 1] = sigmoid_exact(to_f(ba[h]));
 }
 
 // last taps - 1 inputs of every segment -> its slot; a thread owns a channel
@@ -159,24 +196,49 @@ extern "C" void launch_delta_prep(
     int longest, const int* row_seq, const int* ctx, bool fp32,
     hipStream_t stream) {
   const bool shift = longest <= 1;
-  const int rb = M > 2048 ? 8 : 1;
+  const int rb = M >= 8192 ? 8 : M >= 2048 ? 4 : 1;
   const int C = 2 * G * dp + H * vp;
-  const long waves = (long)((M + rb - 1) / rb) * (2 * G + H + 1);
-#define DP(T)                                                                 \
-  do {                                                                        \
-    hipLaunchKernelGGL((delta_prep_kernel<T>), dim3((waves + 3) / 4),         \
-                       dim3(256), 0, stream, (const T*)ab, ld, M, H, G, dp,   \
-                       vp, conv_w, taps, decay, q_scale, unit_eps, qk, (T*)v, \
-                       gb, (T*)conv, seg_row0, seg_slot, row_seq, ctx, rb,    \
-                       shift);                                                \
-    if (!shift && taps > 1)                                                   \
-      hipLaunchKernelGGL((conv_state_kernel<T>),                              \
-                         dim3((C + 255) / 256, nseg), dim3(256), 0, stream,   \
-                         (const T*)ab, ld, C, taps, (T*)conv, seg_row0,       \
-                         seg_rows, seg_slot, ctx);                            \
+  const long runs = (M + rb - 1) / rb;
+  const int lq = dp / 8, lv = vp / 8;
+  const long wg_qk = (runs * 2 * G + 256 / lq - 1) / (256 / lq);
+  const long wg_v = (runs * H + 256 / lv - 1) / (256 / lv);
+  const long wg_s = ((long)M * H + 255) / 256;
+#define DP(T, LQ, LV, TAPS)                                                  \
+  do {                                                                       \
+    const ConvArgs<T> a{(const T*)ab, ld, M, C, taps, rb, conv_w,            \
+                        (T*)conv, seg_row0, seg_slot, row_seq, ctx, shift};  \
+    hipLaunchKernelGGL((delta_prep_kernel<T, LQ, LV, TAPS>),                 \
+                       dim3(wg_qk + wg_v + wg_s), dim3(256), 0, stream, a,   \
+                       H, G, decay, q_scale, unit_eps, qk, (T*)v, gb,        \
+                       (int)wg_qk, (int)wg_v);                               \
+    if (!shift && taps > 1)                                                  \
+      hipLaunchKernelGGL((conv_state_kernel<T>),                             \
+                         dim3((C + 255) / 256, nseg), dim3(256), 0, stream,  \
+                         (const T*)ab, ld, C, taps, (T*)conv, seg_row0,      \
+                         seg_rows, seg_slot, ctx);                           \
   } while (0)
-  if (fp32) DP(float);
-  else DP(unsigned short);
+#define DP_T(T, LQ, LV)              \
+  do {                               \
+    if (taps == 4) DP(T, LQ, LV, 4); \
+    else DP(T, LQ, LV, 0);           \
+  } while (0)
+#define DP_V(T, LQ)              \
+  do {                           \
+    if (lv == 8) DP_T(T, LQ, 8); \
+    else if (lv == 16) DP_T(T, LQ, 16); \
+    else DP_T(T, LQ, 32);        \
+  } while (0)
+#define DP_Q(T)                  \
+  do {                           \
+    if (lq == 8) DP_V(T, 8);     \
+    else if (lq == 16) DP_V(T, 16); \
+    else DP_V(T, 32);            \
+  } while (0)
+  if (fp32) DP_Q(float);
+  else DP_Q(unsigned short);
+#undef DP_Q
+#undef DP_V
+#undef DP_T
 #undef DP
 }
 
@@ -184,7 +246,8 @@ extern "C" void launch_delta_prep(
 // One workgroup per (segment, head). LPC lanes share a value column, each
 // with 16 entries of the state's column in registers (float4 number i of
 // lane `part` is float4 i * LPC + part of the column); a thread has NCOL
-// columns. The output is normed over vdim and gated in place.
+// columns. The output is normed over vdim and gated in place. Segments of
+// more than max_rows rows are left to the chunked form (delta_chunk.hip).
 template <typename T, int LPC, int NCOL>
 __global__ void __launch_bounds__(1024)
 delta_scan_kernel(const float* __restrict__ qk, const T* __restrict__ v,
@@ -195,12 +258,12 @@ delta_scan_kernel(const float* __restrict__ qk, const T* __restrict__ v,
                   const int* __restrict__ seg_row0,
                   const int* __restrict__ seg_rows,
                   const int* __restrict__ seg_slot,
-                  const int* __restrict__ ctx) {
+                  const int* __restrict__ ctx, int max_rows) {
   constexpr int dp = LPC * 16;
   __shared__ float red[2][16];
   const int seg = blockIdx.x / H, head = blockIdx.x % H;
   const int n = seg_rows[seg];
-  if (n == 0) return;
+  if (n == 0 || n > max_rows) return;
   const int row0 = seg_row0[seg];
   const int part = threadIdx.x % LPC;
   const int col0 = threadIdx.x / LPC, cstep = blockDim.x / LPC;
@@ -304,7 +367,7 @@ extern "C" void launch_delta_scan(
     int ld_gate, const float* o_norm, float* state, void* y, int H, int G,
     int dp, int vp, int vdim, float eps, const int* seg_row0,
     const int* seg_rows, const int* seg_slot, int nseg, const int* ctx,
-    bool fp32, hipStream_t stream) {
+    int max_rows, bool fp32, hipStream_t stream) {
   const int lpc = dp / 16;
   const int threads = min(1024, lpc * vp);
   const int ncol = lpc * vp / threads;
@@ -312,7 +375,8 @@ extern "C" void launch_delta_scan(
   hipLaunchKernelGGL((delta_scan_kernel<T, L, N>), dim3(nseg * H),           \
                      dim3(threads), 0, stream, qk, (const T*)v, gb,          \
                      (const T*)gate, ld_gate, o_norm, state, (T*)y, H, G,    \
-                     vp, vdim, eps, seg_row0, seg_rows, seg_slot, ctx)
+                     vp, vdim, eps, seg_row0, seg_rows, seg_slot, ctx,       \
+                     max_rows)
 #define DS_N(T)                                \
   do {                                         \
     if (lpc == 4) DS(T, 4, 1);                 \

@@ -17,68 +17,83 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 
 extern __shared__ __attribute__((aligned(16))) char smem[];
 
-__device__ __forceinline__ void wave_sync() {
-  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
-  __builtin_amdgcn_wave_barrier();
-  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-}
-
 // ---- routing ----------------------------------------------------------------
 // One wave chooses for one row. z [E]: logits, overwritten; gm, ok [groups].
+// A lane holds the scores of experts lane + 64 i, i < PER.
+template <int PER>
 __device__ void select_row(float* z, float* gm, int* ok, int E, int groups,
                            int keep, int top, int* __restrict__ ids,
                            float* __restrict__ weights, int lane) {
+  float s[PER];
   float mx = -INFINITY;
-  for (int e = lane; e < E; e += 64) mx = fmaxf(mx, z[e]);
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int e = lane + 64 * i;
+    s[i] = e < E ? z[e] : -INFINITY;
+    mx = fmaxf(mx, s[i]);
+  }
   mx = wave_reduce_max(mx);
   float sum = 0.f;
-  for (int e = lane; e < E; e += 64) {
-    const float s = expf(z[e] - mx);
-    z[e] = s;
-    sum += s;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    s[i] = expf(s[i] - mx);
+    sum += s[i];
   }
   sum = wave_reduce_sum(sum);
-  wave_sync();
-  const int per = E / groups;
-  for (int c = lane; c < groups; c += 64) {
-    float b = -1.f;
-    for (int i = 0; i < per; ++i) b = fmaxf(b, z[c * per + i]);
-    gm[c] = b;
-  }
-  wave_sync();
-  for (int c = lane; c < groups; c += 64) {
-    int rank = 0;
-    for (int i = 0; i < groups; ++i)
-      rank += gm[i] > gm[c] || (gm[i] == gm[c] && i < c);
-    ok[c] = rank < keep;
-  }
-  wave_sync();
-  for (int e = lane; e < E; e += 64)
-    if (!ok[e / per]) z[e] = -1.f;
-  wave_sync();
-  for (int t = 0; t < top; ++t) {
-    float best = -2.f;
-    int at = E;
-    for (int e = lane; e < E; e += 64)
-      if (z[e] > best) {
-        best = z[e];
-        at = e;
-      }
+  if (groups > 1) {
 #pragma unroll
-    for (int off = 32; off > 0; off >>= 1) {
-      const float b = __shfl_xor(best, off, 64);
-      const int a = __shfl_xor(at, off, 64);
-      if (b > best || (b == best && a < at)) {
-        best = b;
-        at = a;
-      }
-    }
-    if (lane == 0) {
-      ids[t] = at;
-      weights[t] = best / sum;
-      z[at] = -3.f;
+    for (int i = 0; i < PER; ++i)
+      if (lane + 64 * i < E) z[lane + 64 * i] = s[i];
+    wave_sync();
+    const int per = E / groups;
+    for (int c = lane; c < groups; c += 64) {
+      float b = -1.f;
+      for (int i = 0; i < per; ++i) b = fmaxf(b, z[c * per + i]);
+      gm[c] = b;
     }
     wave_sync();
+    for (int c = lane; c < groups; c += 64) {
+      int rank = 0;
+      for (int i = 0; i < groups; ++i)
+        rank += gm[i] > gm[c] || (gm[i] == gm[c] && i < c);
+      ok[c] = rank < keep;
+    }
+    wave_sync();
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int e = lane + 64 * i;
+      if (e < E && !ok[e / per]) s[i] = -1.f;
+    }
+  }
+#pragma unroll
+  for (int i = 0; i < PER; ++i)
+    if (lane + 64 * i >= E) s[i] = -2.f;
+  float own = -3.f;  // the lane's best, and which it is
+  int at = 0;
+  auto best = [&]() {
+    own = -3.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i)
+      if (s[i] > own) {
+        own = s[i];
+        at = i;
+      }
+  };
+  best();
+  for (int t = 0; t < top; ++t) {
+    const float m = wave_reduce_max(own);
+    const unsigned long long who = __ballot(own == m);
+    if (who != 0 && lane == __builtin_ctzll(who)) {
+      ids[t] = lane + 64 * at;
+      weights[t] = m / sum;
+#pragma unroll
+      for (int i = 0; i < PER; ++i)
+        if (i == at) s[i] = -2.f;
+      best();
+    } else if (who == 0 && lane == 0) {  // not a number: no expert
+      ids[t] = -1;
+      weights[t] = 0.f;
+    }
   }
 }
 
@@ -109,20 +124,21 @@ select_kernel(const float* __restrict__ logits, const int* __restrict__ ctx,
   }
   for (int e = lane; e < E; e += 64) z[e] = logits[(long)row * E + e];
   wave_sync();
-  select_row(z, gm, ok, E, groups, keep, top, id, w, lane);
+  select_row<16>(z, gm, ok, E, groups, keep, top, id, w, lane);
 }
 
 // bf16 rows against the router's weights [E, K], fp32 sums, then the
-// choice: 16 rows per workgroup, the four waves split K. NE tiles of 16
-// experts.
-template <int NE>
-__global__ void __launch_bounds__(256)
+// choice: 16 rows per workgroup, its NW waves split K and then the rows. NE
+// tiles of 16 experts.
+template <int NE, int NW>
+__global__ void __launch_bounds__(NW * 64)
 route_kernel(const unsigned short* __restrict__ h,
              const unsigned short* __restrict__ W,
              const int* __restrict__ ctx, int M, int E, int K, int groups,
              int keep, int top, int* __restrict__ ids,
              float* __restrict__ weights) {
   constexpr int EP = NE * 16;
+  constexpr int WS = 16 * (EP + 4);  // sums of a wave
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int i16 = lane & 15, g = lane >> 4;
   const int m0 = blockIdx.x * 16;
@@ -135,8 +151,8 @@ route_kernel(const unsigned short* __restrict__ h,
   f32x4 acc[NE];
 #pragma unroll
   for (int j = 0; j < NE; ++j) acc[j] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 2
-  for (int k = wid * 32; k < K; k += 128) {
+#pragma unroll 4
+  for (int k = wid * 32; k < K; k += NW * 32) {
     const bf16x8 a = *reinterpret_cast<const bf16x8*>(hr + k);
 #pragma unroll
     for (int j = 0; j < NE; ++j)
@@ -144,15 +160,15 @@ route_kernel(const unsigned short* __restrict__ h,
           *reinterpret_cast<const bf16x8*>(wr[j] + k), a, acc[j], 0, 0, 0);
   }
   // rows of the sum: experts (g * 4 + r); columns: rows of h (i16)
-  float* part = reinterpret_cast<float*>(smem);  // [4][16][EP + 4]
+  float* part = reinterpret_cast<float*>(smem);  // [NW][16][EP + 4]
 #pragma unroll
   for (int j = 0; j < NE; ++j)
-    *reinterpret_cast<f32x4*>(part + (wid * 16 + i16) * (EP + 4) + j * 16 +
+    *reinterpret_cast<f32x4*>(part + wid * WS + i16 * (EP + 4) + j * 16 +
                               g * 4) = acc[j];
   __syncthreads();
-  float* gm = part + 64 * (EP + 4) + wid * 2 * groups;
+  float* gm = part + NW * WS + wid * 2 * groups;
   int* ok = reinterpret_cast<int*>(gm + groups);
-  for (int i = wid * 4; i < wid * 4 + 4; ++i) {
+  for (int i = wid; i < 16; i += NW) {
     const int row = m0 + i;
     if (row >= M) break;
     int* id = ids + (long)row * top;
@@ -162,11 +178,15 @@ route_kernel(const unsigned short* __restrict__ h,
       continue;
     }
     float* z = part + i * (EP + 4);
-    for (int e = lane; e < E; e += 64)
-      z[e] = (z[e] + z[e + 16 * (EP + 4)]) +
-             (z[e + 32 * (EP + 4)] + z[e + 48 * (EP + 4)]);
+    for (int e = lane; e < E; e += 64) {
+      float v = z[e];
+#pragma unroll
+      for (int p = 1; p < NW; ++p) v += z[e + p * WS];
+      z[e] = v;
+    }
     wave_sync();
-    select_row(z, gm, ok, E, groups, keep, top, id, w, lane);
+    select_row<(EP + 63) / 64>(z, gm, ok, E, groups, keep, top, id, w, lane);
+    wave_sync();
   }
 }
 
@@ -184,16 +204,17 @@ extern "C" void launch_route(const void* h, const void* W, const int* ctx,
                              int M, int E, int K, int groups, int keep,
                              int top, int* ids, float* weights,
                              hipStream_t stream) {
-#define RT(NE)                                                               \
-  hipLaunchKernelGGL((route_kernel<NE>), dim3((M + 15) / 16), dim3(256),     \
-                     (64 * (NE * 16 + 4) + 8 * groups) * 4, stream,          \
+#define RT(NE, NW)                                                           \
+  hipLaunchKernelGGL((route_kernel<NE, NW>), dim3((M + 15) / 16),            \
+                     dim3(NW * 64),                                          \
+                     (NW * (16 * (NE * 16 + 4) + 2 * groups)) * 4, stream,   \
                      (const unsigned short*)h, (const unsigned short*)W, ctx, \
                      M, E, K, groups, keep, top, ids, weights)
-  if (E <= 16) RT(1);
-  else if (E <= 32) RT(2);
-  else if (E <= 64) RT(4);
-  else if (E <= 128) RT(8);
-  else RT(16);
+  if (E <= 16) RT(1, 16);
+  else if (E <= 32) RT(2, 16);
+  else if (E <= 64) RT(4, 16);
+  else if (E <= 128) RT(8, 8);
+  else RT(16, 4);
 #undef RT
 }
 
@@ -204,13 +225,20 @@ __global__ void __launch_bounds__(1024)
 expert_plan_kernel(const int* __restrict__ ids, int A, int E, int TM,
                    int max_tiles, int* __restrict__ perm,
                    int* __restrict__ tiles, int* __restrict__ ntiles) {
+  constexpr int PU = 8;
   __shared__ int count[1024], first[1024], tile0[1024];
   const int tid = threadIdx.x;
   count[tid] = 0;
   __syncthreads();
-  for (int a = tid; a < A; a += 1024) {
-    const int e = ids[a];
-    if (e >= 0 && e < E) atomicAdd(&count[e], 1);
+  // several at a time: their round trips to memory and LDS overlap
+  for (int a0 = tid; a0 < A; a0 += 1024 * PU) {
+    int e[PU];
+#pragma unroll
+    for (int i = 0; i < PU; ++i)
+      e[i] = a0 + i * 1024 < A ? ids[a0 + i * 1024] : -1;
+#pragma unroll
+    for (int i = 0; i < PU; ++i)
+      if (e[i] >= 0 && e[i] < E) atomicAdd(&count[e[i]], 1);
   }
   __syncthreads();
   const int c = count[tid], nt = (c + TM - 1) / TM;
@@ -237,9 +265,17 @@ expert_plan_kernel(const int* __restrict__ ids, int A, int E, int TM,
   __syncthreads();
   count[tid] = f;
   __syncthreads();
-  for (int a = tid; a < A; a += 1024) {
-    const int e = ids[a];
-    if (e >= 0 && e < E) perm[atomicAdd(&count[e], 1)] = a;
+  for (int a0 = tid; a0 < A; a0 += 1024 * PU) {
+    int e[PU], at[PU];
+#pragma unroll
+    for (int i = 0; i < PU; ++i)
+      e[i] = a0 + i * 1024 < A ? ids[a0 + i * 1024] : -1;
+#pragma unroll
+    for (int i = 0; i < PU; ++i)
+      at[i] = e[i] >= 0 && e[i] < E ? atomicAdd(&count[e[i]], 1) : -1;
+#pragma unroll
+    for (int i = 0; i < PU; ++i)
+      if (at[i] >= 0) perm[at[i]] = a0 + i * 1024;
   }
 }
 
@@ -430,33 +466,35 @@ expert_tile_kernel(const unsigned short* __restrict__ x,
   }
 
   // sums -> padded LDS (a wave's own 64 x 64) -> rows
-  float* ep = reinterpret_cast<float*>(smem) + wid * 64 * 65;
+  float* ep = reinterpret_cast<float*>(smem) + wid * 64 * 68;
 #pragma unroll
   for (int i = 0; i < 4; ++i)
 #pragma unroll
     for (int j = 0; j < 4; ++j)
 #pragma unroll
       for (int r = 0; r < 4; ++r)
-        ep[(i * 16 + (lane >> 4) * 4 + r) * 65 + j * 16 + (lane & 15)] =
+        ep[(i * 16 + (lane >> 4) * 4 + r) * 68 + j * 16 + (lane & 15)] =
             acc[i][j][r];
   __syncthreads();
   if (GLU) {
     const int F = N / 2;
-    const int c = lane & 31;
-    const int col = (n0 + wcol) / 2 + c;
-    const float* p = ep + c / 16 * 32 + c % 16;
-    for (int r = lane >> 5; r < 64; r += 2) {
-      if (wrow + r >= cnt) break;
-      if (col < F)
-        out[(long)(s0 + wrow + r) * F + col] =
-            f2bf(silu(p[r * 65]) * p[r * 65 + 16]);
+    const int c8 = lane & 3, col = (n0 + wcol) / 2 + c8 * 8;
+    for (int r = lane >> 2; r < 64; r += 16) {
+      if (wrow + r >= cnt || col >= F) break;
+      const float* p = ep + r * 68 + (c8 >> 1) * 32 + (c8 & 1) * 8;
+      float o[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) o[i] = silu(p[i]) * p[16 + i];
+      store8(out + (long)(s0 + wrow + r) * F + col, o);
     }
   } else {
-    const int col = n0 + wcol + lane;
-    for (int r = 0; r < 64; ++r) {
-      if (wrow + r >= cnt) break;
-      if (col < N)
-        out[(long)perm[s0 + wrow + r] * N + col] = f2bf(ep[r * 65 + lane]);
+    const int c8 = lane & 7, col = n0 + wcol + c8 * 8;
+    for (int r = lane >> 3; r < 64; r += 8) {
+      if (wrow + r >= cnt || col >= N) break;
+      float o[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) o[i] = ep[r * 68 + c8 * 8 + i];
+      store8(out + (long)perm[s0 + wrow + r] * N + col, o);
     }
   }
 }
@@ -502,7 +540,12 @@ expert_f32_kernel(const float* __restrict__ x, const float* __restrict__ W,
   }
 }
 
-// TM: rows per tile of the plan (16, 32, 64, or 128 for the large tiles)
+// TM: rows per tile of the plan (16, 32, 64, 128, or 256 for the tiles of
+// expert_gemm16.hip)
+extern "C" void launch_expert_gemm16(const void*, const void*, void*,
+                                     const int*, const int*, const int*, int,
+                                     int, int, int, bool, hipStream_t);
+
 extern "C" void launch_expert_gemm(const void* x, const void* W, void* out,
                                    const int* perm, const int* tiles,
                                    const int* ntiles, int max_tiles, int N,
@@ -518,6 +561,11 @@ extern "C" void launch_expert_gemm(const void* x, const void* W, void* out,
     if (glu) EF(true);
     else EF(false);
 #undef EF
+    return;
+  }
+  if (TM == 256) {
+    launch_expert_gemm16(x, W, out, perm, tiles, ntiles, max_tiles, N, K, top,
+                         glu, stream);
     return;
   }
 #define ER(MT, GL)                                                          \

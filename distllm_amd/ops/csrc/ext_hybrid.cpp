@@ -27,9 +27,16 @@ void launch_delta_prep(const void*, int, int, int, int, int, int,
 void launch_delta_scan(const float*, const void*, const float*, const void*,
                        int, const float*, float*, void*, int, int, int, int,
                        int, float, const int*, const int*, const int*, int,
-                       const int*, bool, hipStream_t);
+                       const int*, int, bool, hipStream_t);
+void launch_delta_chunks(const float*, const void*, const float*, const void*,
+                         int, const float*, float*, void*, float*, float*,
+                         float*, float*, int, int, int, int, int, int, float,
+                         const int*, int, const int*, int, int, const int*,
+                         const int*, const int*, const int*, const int*,
+                         hipStream_t);
 void launch_xielu(const void*, const float*, void*, long, bool, hipStream_t);
 bool route_covers(int);
+bool expert_gemm16_covers(int, int);
 void launch_select(const float*, const int*, int, int, int, int, int, int*,
                    float*, hipStream_t);
 void launch_route(const void*, const void*, const int*, int, int, int, int,
@@ -113,6 +120,7 @@ torch::Tensor attn_prep(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
     cols += G * (dp + vp);
   }
   TORCH_CHECK(ab.size(1) >= cols, "projection columns");
+  TORCH_CHECK((long)M * (H + G) < (1L << 30), "too many rows");
   auto q = torch::empty({M, H, dp}, ab.options());
   if (M > 0)
     launch_attn_prep(ab.data_ptr(), ld, M, H, G, dp, vp, (int)n,
@@ -227,6 +235,8 @@ void paged_attn_prompts(torch::Tensor q, torch::Tensor k, torch::Tensor v,
                      (float)softcap, dist.data_ptr<float>(), cur_stream());
 }
 
+// longs [P, 2]: segments of more than max_rows rows and their first chunk,
+// chunks [N, 2]: segment and number of every chunk of 32 rows; bf16 only
 torch::Tensor gated_delta(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
                           int64_t vp, int64_t dim, int64_t vdim,
                           torch::Tensor conv_w, torch::Tensor decay,
@@ -234,7 +244,10 @@ torch::Tensor gated_delta(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
                           torch::Tensor state, torch::Tensor conv,
                           torch::Tensor seg_row0, torch::Tensor seg_rows,
                           torch::Tensor seg_slot, int64_t longest,
-                          torch::Tensor row_seq, torch::Tensor ctx) {
+                          torch::Tensor row_seq, torch::Tensor ctx,
+                          c10::optional<torch::Tensor> longs,
+                          c10::optional<torch::Tensor> chunks,
+                          int64_t max_rows) {
   CHECK_DEV(ab); CHECK_CONT(ab); CHECK_T(ab);
   const int M = ab.size(0), ld = ab.size(1);
   auto size_ok = [](int64_t d) { return d == 64 || d == 128 || d == 256; };
@@ -269,7 +282,8 @@ torch::Tensor gated_delta(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
   auto qk = torch::empty({M, 2 * G, dp}, f32);
   auto v = torch::empty({M, H * vp}, ab.options());
   auto gb = torch::empty({M, H, 2}, f32);
-  const int es = ab.element_size();
+  const void* gate =
+      (const char*)ab.data_ptr() + C * (long)ab.element_size();
   launch_delta_prep(ab.data_ptr(), ld, M, H, G, dp, vp,
                     conv_w.data_ptr<float>(), taps, decay.data_ptr<float>(),
                     1.f / sqrtf((float)dim), (float)unit_eps,
@@ -278,13 +292,35 @@ torch::Tensor gated_delta(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
                     seg_rows.data_ptr<int>(), seg_slot.data_ptr<int>(), S,
                     (int)longest, row_seq.data_ptr<int>(),
                     ctx.data_ptr<int>(), is_f32(ab), cur_stream());
+  const bool chunked = longs && !is_f32(ab) && longs->size(0) > 0;
+  const int limit = chunked ? (int)max_rows : INT_MAX;
   launch_delta_scan(qk.data_ptr<float>(), v.data_ptr(), gb.data_ptr<float>(),
-                    (const char*)ab.data_ptr() + C * es, ld,
-                    o_norm.data_ptr<float>(), state.data_ptr<float>(),
+                    gate, ld, o_norm.data_ptr<float>(), state.data_ptr<float>(),
                     y.data_ptr(), H, G, dp, vp, vdim, (float)eps,
                     seg_row0.data_ptr<int>(), seg_rows.data_ptr<int>(),
-                    seg_slot.data_ptr<int>(), S, ctx.data_ptr<int>(),
+                    seg_slot.data_ptr<int>(), S, ctx.data_ptr<int>(), limit,
                     is_f32(ab), cur_stream());
+  if (chunked) {
+    TORCH_CHECK(chunks.has_value(), "chunks");
+    CHECK_INTS(longs.value()); CHECK_INTS(chunks.value());
+    TORCH_CHECK(longs->dim() == 2 && longs->size(1) == 2 &&
+                    chunks->dim() == 2 && chunks->size(1) == 2 &&
+                    chunks->size(0) >= longs->size(0),
+                "chunk maps");
+    const int N = chunks->size(0);
+    auto tp = torch::empty({2, N, H, 32 * 32}, f32);
+    auto bsum = torch::empty({M, H}, f32);
+    auto o = torch::empty({M, H * vp}, f32);
+    launch_delta_chunks(
+        qk.data_ptr<float>(), v.data_ptr(), gb.data_ptr<float>(), gate, ld,
+        o_norm.data_ptr<float>(), state.data_ptr<float>(), y.data_ptr(),
+        tp.data_ptr<float>(), tp.data_ptr<float>() + tp.numel() / 2,
+        bsum.data_ptr<float>(), o.data_ptr<float>(), M, H, G, dp, vp, vdim,
+        (float)eps, longs->data_ptr<int>(), longs->size(0),
+        chunks->data_ptr<int>(), N, limit, seg_row0.data_ptr<int>(),
+        seg_rows.data_ptr<int>(), seg_slot.data_ptr<int>(),
+        row_seq.data_ptr<int>(), ctx.data_ptr<int>(), cur_stream());
+  }
   return y;
 }
 
@@ -360,8 +396,10 @@ torch::Tensor experts(torch::Tensor h, torch::Tensor ids, torch::Tensor wgup,
   // about 48 rows on
   const bool f32 = is_f32(h);
   const long mean = (A + E - 1) / E;
-  const int TM = f32 || mean <= 8 ? 16 : mean <= 16 ? 32 : mean <= 48 ? 64
-                                                                      : 128;
+  int TM = f32 || mean <= 8 ? 16 : mean <= 16 ? 32 : mean <= 48 ? 64 : 128;
+  if (!f32 && mean >= 512 && expert_gemm16_covers(2 * F, K) &&
+      expert_gemm16_covers(K, F))
+    TM = 256;
   const int max_tiles = (int)std::min<long>(A, A / TM + E);
   auto i32 = ids.options();
   auto plan = torch::empty({A + 4L * max_tiles + 1}, i32);

@@ -32,8 +32,8 @@ GROUPS = {
                     "clamped_glu.hip"],
     "_hip_residual": ["ext_residual.cpp", "residual_norms.hip"],
     "_hip_hybrid": ["ext_hybrid.cpp", "chunk_attention.hip",
-                    "chunk_flash.hip", "delta_rule.hip", "experts.hip",
-                    "xielu.hip"],
+                    "chunk_flash.hip", "delta_rule.hip", "delta_chunk.hip",
+                    "experts.hip", "expert_gemm16.hip", "xielu.hip"],
 }
 _taken = {s for group in GROUPS.values() for s in group}
 # *_hip.hip files are torch-hipify build artifacts — exclude them.
