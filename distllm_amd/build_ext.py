@@ -16,7 +16,10 @@ ROOT = Path(__file__).resolve().parents[1]
 
 # config.json "architecture" -> the extensions that the model's steps use
 NEEDED = {"Kanotar": ("_hip_gemm", "_hip_residual", "_hip_latent"),
-          "Bufulorn": ("_hip_gemm", "_hip_residual", "_hip_hybrid")}
+          "Bufulorn": ("_hip_gemm", "_hip_residual", "_hip_hybrid",
+                       "_hip_experts"),
+          "Tebasun": ("_hip_gemm", "_hip_residual", "_hip_hybrid",
+                      "_hip_lru")}
 
 
 def needed_for(model_dir: str) -> tuple[str, ...]:

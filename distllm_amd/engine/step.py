@@ -68,6 +68,8 @@ class Segments:
     longest: int
     longs: torch.Tensor | None = None   # [P, 2] segment, its first chunk
     chunks: torch.Tensor | None = None  # [N, 2] segment, chunk in it
+    sizes: list[int] = field(default_factory=list)  # rows, on the host
+    _lists: dict[int, tuple] = field(default_factory=dict)
 
     SHORT = 16
     CHUNK = 32
@@ -78,15 +80,24 @@ class Segments:
             return torch.from_numpy(
                 np.array(a, np.int32).reshape(*shape)).to(device)
 
-        longs, chunks = [], []
-        for i, n in enumerate(rows):
-            if n > cls.SHORT:
-                longs.append((i, len(chunks)))
-                chunks += [(i, c) for c in range(-(-n // cls.CHUNK))]
-        return cls(up(row0, -1), up(rows, -1), up(slots, -1),
-                   max(rows, default=0),
-                   up(longs, -1, 2) if longs else None,
-                   up(chunks, -1, 2) if longs else None)
+        seg = cls(up(row0, -1), up(rows, -1), up(slots, -1),
+                  max(rows, default=0), sizes=list(rows))
+        seg.longs, seg.chunks = seg.chunk_lists(cls.CHUNK)
+        return seg
+
+    def chunk_lists(self, size: int) -> tuple:
+        """(longs, chunks) in chunks of `size` rows; None where no segment
+        is long."""
+        if size not in self._lists:
+            longs, chunks = [], []
+            for i, n in enumerate(self.sizes):
+                if n > self.SHORT:
+                    longs.append((i, len(chunks)))
+                    chunks += [(i, c) for c in range(-(-n // size))]
+            self._lists[size] = (None, None) if not longs else tuple(
+                torch.tensor(a, dtype=torch.int32).to(self.row0.device)
+                for a in (longs, chunks))
+        return self._lists[size]
 
 
 @dataclass
@@ -103,6 +114,14 @@ class StepBatch:
     segments: Segments | None = None  # with state slots
     _expansions: dict[int, Expansion] = field(default_factory=dict)
     _prompts: dict[int, PromptBlocks] = field(default_factory=dict)
+    _rotations: dict = field(default_factory=dict)
+
+    def rotation(self, key, freq: torch.Tensor, mult: float):
+        """cos and sin of every row's position, [M, pairs, 2] fp32; layers
+        with the same rotation (`key`) share them."""
+        if key not in self._rotations:
+            self._rotations[key] = ops.rotation_table(self.ctx, freq, mult)
+        return self._rotations[key]
 
     @classmethod
     def decode(cls, tokens, block_table, ctx, slots=None) -> "StepBatch":

@@ -11,6 +11,7 @@ from .config import (PRESETS, LayeredDims, ModelDims, dims_from_checkpoint,
 from .esm import Esm2Encoder, EsmCEncoder
 from .kanotar import KanotarModel
 from .mistral import DecoderModel
+from .tebasun import TebasunModel
 
 __all__ = [
     "BertEncoder",
@@ -22,6 +23,7 @@ __all__ = [
     "LayeredDims",
     "ModelDims",
     "PRESETS",
+    "TebasunModel",
     "build_model",
     "dims_from_checkpoint",
     "get_dims",
@@ -30,7 +32,8 @@ __all__ = [
 
 
 # decoders that are described layer by layer
-LAYERED = {"kanotar": KanotarModel, "bufulorn": BufulornModel}
+LAYERED = {"kanotar": KanotarModel, "bufulorn": BufulornModel,
+           "tebasun": TebasunModel}
 
 
 def build_model(name_or_dims: str | ModelDims | LayeredDims, device: str | None = None,

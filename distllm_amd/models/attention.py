@@ -1,4 +1,4 @@
-"""Softmax attention on paged keys and values, visible chunk by chunk."""
+"""Softmax attention on paged keys and values."""
 
 from __future__ import annotations
 
@@ -6,9 +6,9 @@ import torch
 from torch import nn
 
 from .. import ops
-from .blocks import (Part, head_pad, norm_weight, pad64, padded,
+from .blocks import (Branch, Part, head_pad, norm_weight, pad64, padded,
                      padded_heads, weight)
-from .config import AttentionDims
+from .config import AttentionDims, RotaryAttentionDims
 
 
 class PagedAttention(Part):
@@ -118,3 +118,87 @@ class PagedAttention(Part):
                 batch.prompt_blocks(d.chunk), d.chunk, d.scale, d.softcap,
                 self.dist)
         return ops.linear(o.view(M, d.heads * self.vp), self.wo)
+
+
+class RotaryAttention(Branch):
+    """Causal attention with normed and rotated queries and keys, keys as
+    projected for values and a sink per head (RotaryAttentionDims), on the
+    pages of PagedAttention. One launch norms, rotates and writes the
+    cache."""
+
+    EVERYTHING = 1 << 30  # chunk size of plain causal attention
+
+    def __init__(self, d: RotaryAttentionDims, width: int, eps: float,
+                 dtype):
+        super().__init__()
+        self.d, self.width, self.eps = d, width, eps
+        self.wp, self.dp = pad64(width), head_pad(d.dim)
+        self.in_rows = (d.heads + d.kv_heads) * self.dp
+        self.out_cols = d.heads * self.dp
+        self.q_norm = norm_weight(self.dp)
+        self.k_norm = norm_weight(self.dp)
+        self.sink = norm_weight(d.heads)
+        freq, self.rot_mult = d.rot.frequencies()
+        self.rot_key = d.rot.model_dump_json()
+        self.register_buffer("freq", torch.tensor(freq, dtype=torch.float64),
+                             persistent=False)
+        self.bf16 = dtype == torch.bfloat16
+
+    def tensors(self):
+        d, W = self.d, self.width
+        q, k = d.heads * d.dim, d.kv_heads * d.dim
+        return {"q": (q, W), "q.b": (q,), "q.norm": (d.dim,),
+                "k": (k, W), "k.b": (k,), "k.norm": (d.dim,),
+                "sink": (d.heads,), "o": (W, q), "o.b": (W,)}
+
+    def _heads(self):
+        return (("q", self.d.heads), ("k", self.d.kv_heads))
+
+    def in_weight(self, t):
+        return torch.cat([padded_heads(t[n], h, self.d.dim, self.dp, self.wp)
+                          for n, h in self._heads()])
+
+    def in_bias(self, t):
+        return torch.cat([padded_heads(t[n + ".b"][:, None], h, self.d.dim,
+                                       self.dp, 1)[:, 0]
+                          for n, h in self._heads()])
+
+    def out_weight(self, t):
+        return padded_heads(t["o"].t(), self.d.heads, self.d.dim, self.dp,
+                            self.wp).t()
+
+    def out_bias(self, t):
+        return t["o.b"]
+
+    def extra(self, t):
+        return {"q_norm": padded(t["q.norm"], self.dp),
+                "k_norm": padded(t["k.norm"], self.dp), "sink": t["sink"]}
+
+    def cache_numel(self):
+        return 2 * self.d.kv_heads * self.dp
+
+    def make_cache(self, num_blocks, blk, num_slots, dtype, device):
+        G = self.d.kv_heads
+        return (torch.zeros(num_blocks, G, blk, self.dp, dtype=dtype,
+                            device=device),
+                torch.zeros(num_blocks, G, self.dp, blk, dtype=dtype,
+                            device=device))
+
+    def run(self, ab, batch, pages, out, scale):
+        d, M = self.d, ab.shape[0]
+        kpages, vpages = pages
+        table = batch.rotation(self.rot_key, self.freq, self.rot_mult)
+        q = ops.rotary_prep(ab, d.heads, d.kv_heads, self.dp, d.dim,
+                            self.q_norm, self.k_norm, self.eps, table, pages,
+                            batch.block_table, batch.row_seq, batch.ctx)
+        flash = self.dp <= 256 and (self.bf16 or not ab.is_cuda)
+        n = batch.n_folded if flash else M
+        if n > 0:
+            ops.sink_attn_rows(q[:n], kpages, vpages, out[:n],
+                               batch.block_table, batch.row_seq[:n],
+                               batch.ctx[:n], d.scale, self.sink, scale)
+        if n < M:
+            ops.sink_attn_prompts(
+                q, kpages, vpages, out, batch.block_table,
+                batch.prompt_blocks(self.EVERYTHING), d.scale, self.sink,
+                scale)

@@ -105,6 +105,39 @@ class Part(nn.Module):
         return None
 
 
+class Branch(Part):
+    """A mechanism between an input and an output product, both of which
+    may be shared with other branches (branches.py). It says which rows of
+    the input product it wants and what its output columns are multiplied
+    with, and fills its columns of the output product's input."""
+
+    in_rows: int   # columns of the input product, padded
+    out_cols: int  # columns given to the output product, padded
+
+    def in_weight(self, t: dict) -> torch.Tensor:
+        """[in_rows, padded width], from the branch's checked tensors."""
+        raise NotImplementedError
+
+    def in_bias(self, t: dict) -> torch.Tensor | None:
+        return None
+
+    def out_weight(self, t: dict) -> torch.Tensor:
+        """[padded width, out_cols]"""
+        raise NotImplementedError
+
+    def out_bias(self, t: dict) -> torch.Tensor | None:
+        return None
+
+    def extra(self, t: dict) -> dict[str, torch.Tensor]:
+        """The branch's own parameters."""
+        raise NotImplementedError
+
+    def run(self, ab, batch, cache, out, scale: float) -> None:
+        """ab [M, in_rows]: the branch's columns of the input product;
+        out [M, out_cols] takes its result, times `scale`."""
+        raise NotImplementedError
+
+
 class LatentAttention(Part):
     """Latent attention with a sliding window, on paged latents.
 

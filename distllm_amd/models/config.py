@@ -9,8 +9,8 @@ decoder family used for generation (K15):
   - Mistral-class decoder embedders (SFR-Embedding-Mistral)
   - Llama-class causal LMs for generation
   - Qwen2-class causal LMs (llama family + qkv bias)
-  - Kanotar and Bufulorn causal LMs: every layer has its own description
-    (LayeredDims)
+  - Kanotar, Bufulorn and Tebasun causal LMs: every layer has its own
+    description (LayeredDims)
 Dims are from the public model cards; weights are random-init here
 (no network) or loadable from local safetensors.
 """
@@ -18,6 +18,7 @@ Dims are from the public model cards; weights are random-init here
 from __future__ import annotations
 
 import json
+import math
 from pathlib import Path
 from typing import Literal
 
@@ -57,6 +58,13 @@ class ModelDims(BaseModel):
 
 class _Strict(BaseModel):
     model_config = ConfigDict(extra="forbid")
+
+
+def _check_groups(m):
+    if m.heads % m.kv_heads:
+        raise ValueError(f"{m.heads} heads are not a multiple of "
+                         f"{m.kv_heads} kv_heads")
+    return m
 
 
 class LatentAttentionDims(_Strict):
@@ -115,6 +123,125 @@ class DeltaDims(_Strict):
     unit_eps: float = 1e-6     # of the unit queries and keys
 
 
+class YarnDims(_Strict):
+    """YaRN: frequencies are divided by `factor`, by degrees between the
+    pairs that turn `fast` and `slow` times over `original` positions."""
+
+    factor: PositiveFloat
+    original: PositiveFloat
+    fast: PositiveFloat
+    slow: PositiveFloat
+
+
+class RotaryDims(_Strict):
+    """Rotation of the first `dims` numbers of a head: number i pairs with
+    number i + dims / 2 and turns by base^(-2i / dims) per position."""
+
+    base: PositiveFloat
+    dims: PositiveInt
+    scaling: YarnDims | None = None
+
+    @model_validator(mode="after")
+    def _check_even(self):
+        if self.dims % 2:
+            raise ValueError(f"{self.dims} rotated numbers form no pairs")
+        return self
+
+    def frequencies(self) -> tuple[list[float], float]:
+        """-> frequency of every pair, and the factor on cos and sin."""
+        n, half = self.dims, self.dims // 2
+        freq = [self.base ** (-2.0 * i / n) for i in range(half)]
+        y = self.scaling
+        if y is None:
+            return freq, 1.0
+
+        def pair_of(turns: float) -> float:
+            return (n * math.log(y.original / (2 * math.pi * turns))
+                    / (2 * math.log(self.base)))
+
+        lo = max(math.floor(pair_of(y.fast)), 0)
+        hi = min(math.ceil(pair_of(y.slow)), n - 1)
+        for i in range(half):
+            ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+            freq[i] *= ramp / y.factor + 1.0 - ramp
+        return freq, 0.1 * math.log(y.factor) + 1.0
+
+
+class RotaryAttentionDims(_Strict):
+    """Causal softmax attention whose values are the keys as projected,
+    before norm and rotation. Queries and keys are normed per head, then
+    rotated; a learned sink per head takes part in the softmax."""
+
+    type: Literal["rotary_attention"] = "rotary_attention"
+    heads: PositiveInt
+    kv_heads: PositiveInt
+    dim: PositiveInt
+    vdim: PositiveInt          # dim, as the values are keys
+    rot: RotaryDims
+    scale: float
+
+    @model_validator(mode="after")
+    def _check_sizes(self):
+        if self.vdim != self.dim:
+            raise ValueError(f"values are keys: vdim {self.vdim} must be "
+                             f"dim {self.dim}")
+        if self.rot.dims > self.dim:
+            raise ValueError(f"{self.rot.dims} rotated numbers in heads of "
+                             f"{self.dim}")
+        return _check_groups(self)
+
+
+class ChannelDeltaDims(_Strict):
+    """Gated delta rule with a decay per head and key channel, which
+    comes from a pair of products through `decay_rank` numbers; the output
+    gate comes from a pair through `gate_rank`."""
+
+    type: Literal["channel_delta"] = "channel_delta"
+    heads: PositiveInt
+    kv_heads: PositiveInt
+    dim: PositiveInt
+    vdim: PositiveInt
+    conv: PositiveInt
+    decay_rank: PositiveInt
+    gate_rank: PositiveInt
+    unit_eps: float = 1e-6
+
+    @model_validator(mode="after")
+    def _check_sizes(self):
+        return _check_groups(self)
+
+
+class ParallelDims(_Strict):
+    """Two mixers side by side on the same input:
+    left_scale * left + right_scale * right."""
+
+    type: Literal["parallel"] = "parallel"
+    left: RotaryAttentionDims
+    right: ChannelDeltaDims
+    left_scale: float
+    right_scale: float
+
+
+class LruDims(_Strict):
+    """Real-gated linear recurrent unit on one branch of `width`, behind a
+    causal convolution of `conv` taps, times a GELU branch. Its gates are
+    block-diagonal products of `blocks` blocks; decays are
+    exp(-decay_scale * gate * softplus(lam))."""
+
+    type: Literal["rglru"] = "rglru"
+    width: PositiveInt
+    blocks: PositiveInt
+    conv: PositiveInt
+    decay_scale: float = 8.0
+
+    @model_validator(mode="after")
+    def _check_blocks(self):
+        if self.width % self.blocks:
+            raise ValueError(f"width {self.width} does not split into "
+                             f"{self.blocks} equal blocks")
+        return self
+
+
 class ClampedGluDims(_Strict):
     """Feed-forward g * sigmoid(alpha g) * (u + shift), gate g clamped
     from above and up-projection u from both sides at `limit`."""
@@ -124,6 +251,13 @@ class ClampedGluDims(_Strict):
     limit: float
     alpha: float = 1.702
     shift: float = 1.0
+
+
+class SwigluDims(_Strict):
+    """Feed-forward down(silu(gate) * up)."""
+
+    kind: Literal["swiglu"] = "swiglu"
+    ff: PositiveInt
 
 
 class XieluDims(_Strict):
@@ -160,19 +294,32 @@ class ExpertsDims(_Strict):
 
 
 class LayerDims(_Strict):
-    mixer: LatentAttentionDims | AttentionDims | DeltaDims
-    mlp: ClampedGluDims | XieluDims | ExpertsDims | None = None
+    mixer: (LatentAttentionDims | AttentionDims | DeltaDims | ParallelDims
+            | LruDims)
+    mlp: ClampedGluDims | SwigluDims | XieluDims | ExpertsDims | None = None
+
+
+class LoopDims(_Strict):
+    """Layers start .. stop - 1 run `times` times in a row with the same
+    weights; each pass has its own cache and state."""
+
+    start: NonNegativeInt
+    stop: PositiveInt
+    times: PositiveInt
 
 
 class LayeredDims(BaseModel):
     """A decoder whose layers are described one by one."""
 
-    arch: Literal["kanotar", "bufulorn"]
+    arch: Literal["kanotar", "bufulorn", "tebasun"]
     vocab_size: PositiveInt
     hidden_size: PositiveInt
     layers: list[LayerDims]
     norm_eps: float
     logit_scale: float = 1.0
+    embed_scale: float = 1.0
+    loop: LoopDims | None = None
+    side_dim: PositiveInt | None = None  # per-layer token inputs
     # bounded only by a position table, where the design has one
     max_position_embeddings: PositiveInt = 1 << 20
 
@@ -180,13 +327,34 @@ class LayeredDims(BaseModel):
     def num_layers(self) -> int:
         return len(self.layers)
 
+    def layer_runs(self) -> list[tuple[int, int | None]]:
+        """Layers in running order, each with the number of the loop's
+        pass that begins with it, or None."""
+        n = len(self.layers)
+        if self.loop is None:
+            return [(i, None) for i in range(n)]
+        lp, runs = self.loop, []
+        for t in range(lp.times):
+            runs += [(i, t if i == lp.start else None)
+                     for i in range(lp.start, lp.stop)]
+        return ([(i, None) for i in range(lp.start)] + runs
+                + [(i, None) for i in range(lp.stop, n)])
+
+    @model_validator(mode="after")
+    def _check_loop(self):
+        lp = self.loop
+        if lp is not None and not lp.start < lp.stop <= len(self.layers):
+            raise ValueError(f"loop over layers {lp.start} to {lp.stop} of "
+                             f"{len(self.layers)}")
+        return self
+
     @model_validator(mode="after")
     def _check_sharing(self):
         if not self.layers:
             raise ValueError("a model needs at least one layer")
         for i, layer in enumerate(self.layers):
             m = layer.mixer
-            if not isinstance(m, LatentAttentionDims) \
+            if isinstance(m, (AttentionDims, DeltaDims)) \
                     and m.heads % m.kv_heads:
                 raise ValueError(f"layer {i}: {m.heads} heads are not a "
                                  f"multiple of {m.kv_heads} kv_heads")
@@ -214,7 +382,7 @@ def _take(d: dict, name: str, where: str):
     return d[name]
 
 
-def _kanotar_dims(cfg: dict) -> LayeredDims:
+def _kanotar_dims(cfg: dict, shapes=None) -> LayeredDims:
     layers = []
     for i, entry in enumerate(cfg["layers"]):
         if entry["type"] != "latent_attention":
@@ -249,7 +417,7 @@ def _bufulorn_mlp(mlp: dict, where: str):
     return dims
 
 
-def _bufulorn_dims(cfg: dict) -> LayeredDims:
+def _bufulorn_dims(cfg: dict, shapes=None) -> LayeredDims:
     layers = []
     for i, entry in enumerate(cfg["layers"]):
         mixer = dict(entry["mixer"])
@@ -271,8 +439,56 @@ def _bufulorn_dims(cfg: dict) -> LayeredDims:
                        max_position_embeddings=cfg["max_positions"])
 
 
-# config.json "architecture" -> reader of the rest of the file
-CONFIG_READERS = {"Kanotar": _kanotar_dims, "Bufulorn": _bufulorn_dims}
+def _tebasun_dims(cfg: dict, shapes=None) -> LayeredDims:
+    layers, sizes = [], shapes()
+    for i, entry in enumerate(cfg["layers"]):
+        mixer = dict(entry["mixer"])
+        if entry["type"] == "parallel":
+            # the inner sizes of the two pairs of products are told by
+            # their tensors alone
+            pre = f"l{i}.mix.right."
+            mixer["right"] = dict(mixer["right"],
+                                  decay_rank=sizes[pre + "a1"][0],
+                                  gate_rank=sizes[pre + "g1"][0])
+            mixer = ParallelDims(**mixer)
+        elif entry["type"] == "rglru":
+            mixer = LruDims(**mixer)
+        else:
+            raise ValueError(f"layer {i}: unknown mixer {entry['type']!r}")
+        mlp = entry.get("mlp")
+        if mlp is not None:
+            mlp = dict(mlp)
+            kind = mlp.pop("kind", None)
+            if kind != "dense":
+                raise ValueError(f"layer {i}: unknown feed-forward kind "
+                                 f"{kind!r}")
+            mlp = SwigluDims(**mlp)
+        layers.append(LayerDims(mixer=mixer, mlp=mlp))
+    loop, side = cfg.get("loop"), cfg.get("token_side")
+    return LayeredDims(arch="tebasun", vocab_size=cfg["vocab"],
+                       hidden_size=cfg["width"], layers=layers,
+                       norm_eps=cfg["norm"]["eps"],
+                       embed_scale=cfg["embedding"]["scale"],
+                       loop=None if loop is None else LoopDims(**loop),
+                       side_dim=None if side is None else side["dim"])
+
+
+# config.json "architecture" -> reader of the rest of the file; `shapes`
+# returns the checkpoint's tensor shapes
+CONFIG_READERS = {"Kanotar": _kanotar_dims, "Bufulorn": _bufulorn_dims,
+                  "Tebasun": _tebasun_dims}
+
+
+def checkpoint_shapes(path: str | Path) -> dict[str, tuple[int, ...]]:
+    """Tensor name -> shape, from the headers of a folder's safetensors."""
+    from safetensors import safe_open
+
+    shapes = {}
+    for f in sorted(Path(path).glob("*.safetensors")):
+        with safe_open(str(f), "pt") as src:
+            for name in src.keys():
+                shapes[name] = tuple(src.get_slice(name).get_shape())
+    return shapes
 
 
 def dims_from_checkpoint(path: str | Path) -> LayeredDims | None:
@@ -283,7 +499,7 @@ def dims_from_checkpoint(path: str | Path) -> LayeredDims | None:
         return None
     cfg = json.loads(f.read_text())
     reader = CONFIG_READERS.get(cfg.get("architecture"))
-    return reader(cfg) if reader else None
+    return reader(cfg, lambda: checkpoint_shapes(path)) if reader else None
 
 
 def layered_preset(num_layers: int, hidden: int, vocab: int, heads: int,
@@ -335,6 +551,40 @@ def hybrid_preset(num_layers: int, hidden: int, vocab: int, heads: int,
     return LayeredDims(arch="bufulorn", vocab_size=vocab, hidden_size=hidden,
                        layers=layers, norm_eps=eps,
                        max_position_embeddings=max_positions)
+
+
+def looped_preset(num_layers: int, hidden: int, vocab: int, heads: int,
+                  kv_heads: int, dim: int, ff: int, order: str = "PPR",
+                  lru_width: int | None = None, blocks: int = 16,
+                  rank: int | None = None, side: int = 256,
+                  loop: tuple[int, int, int] | None = None,
+                  original: int = 8192, eps: float = 1e-5) -> LayeredDims:
+    """Tebasun dims of repeated layers: mixers follow `order` (P attention
+    beside the delta rule, with half of the heads each; R linear recurrent
+    unit)."""
+    layers = []
+    for i in range(num_layers):
+        if order[i % len(order)] == "P":
+            mixer = ParallelDims(
+                left=RotaryAttentionDims(
+                    heads=heads // 2, kv_heads=kv_heads // 2, dim=dim,
+                    vdim=dim, scale=dim ** -0.5, rot=RotaryDims(
+                        base=500000.0, dims=dim // 2, scaling=YarnDims(
+                            factor=4.0, original=original, fast=32.0,
+                            slow=1.0))),
+                right=ChannelDeltaDims(
+                    heads=heads // 2, kv_heads=heads // 2, dim=dim,
+                    vdim=dim, conv=4, decay_rank=rank or dim,
+                    gate_rank=rank or dim),
+                left_scale=0.7, right_scale=0.7)
+        else:
+            mixer = LruDims(width=lru_width or hidden, blocks=blocks, conv=4)
+        layers.append(LayerDims(mixer=mixer, mlp=SwigluDims(ff=ff)))
+    lp = loop or (0, num_layers, 1)
+    return LayeredDims(arch="tebasun", vocab_size=vocab, hidden_size=hidden,
+                       layers=layers, norm_eps=eps,
+                       embed_scale=hidden ** 0.5, side_dim=side,
+                       loop=LoopDims(start=lp[0], stop=lp[1], times=lp[2]))
 
 
 PRESETS: dict[str, ModelDims | LayeredDims] = {
@@ -442,6 +692,16 @@ PRESETS: dict[str, ModelDims | LayeredDims] = {
         4, 256, 1024, heads=4, kv_heads=2, dim=32, ff=512, chunk=48,
         experts=ExpertsDims(ff=64, experts=6, top=2, groups=3, keep=2),
         order="AAD", share=True, max_positions=512,
+    ),
+    # attention beside the delta rule, and linear recurrent layers, of the
+    # llama3-8b size; the middle layers run twice
+    "tebasun-8b": looped_preset(
+        24, 4096, 128256, heads=32, kv_heads=16, dim=128, ff=14336,
+        loop=(8, 16, 2),
+    ),
+    "tebasun-tiny": looped_preset(
+        4, 256, 1024, heads=8, kv_heads=4, dim=32, ff=512, order="PR",
+        blocks=4, rank=16, side=32, loop=(1, 3, 2), original=64,
     ),
 }
 

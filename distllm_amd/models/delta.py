@@ -1,4 +1,4 @@
-"""Gated delta rule with short convolutions."""
+"""Gated delta rules with short convolutions."""
 
 from __future__ import annotations
 
@@ -6,8 +6,9 @@ import torch
 from torch import nn
 
 from .. import ops
-from .blocks import Part, norm_weight, pad64, padded, padded_heads, weight
-from .config import DeltaDims
+from .blocks import (Branch, Part, norm_weight, pad64, padded, padded_heads,
+                     weight)
+from .config import ChannelDeltaDims, DeltaDims
 
 
 def state_pad(n: int) -> int:
@@ -23,7 +24,7 @@ class DeltaState:
     vdim, dim] so that what one value column needs is contiguous, and the
     convolutions' last inputs [slots, taps - 1, channels]."""
 
-    def __init__(self, m: "GatedDelta", num_slots: int, dtype, device):
+    def __init__(self, m: "GatedDelta | ChannelDelta", num_slots: int, dtype, device):
         self.s = torch.zeros(num_slots, m.d.heads, m.vp, m.dp,
                              dtype=torch.float32, device=device)
         self.conv = torch.zeros(num_slots, m.d.conv - 1, m.channels,
@@ -96,3 +97,90 @@ class GatedDelta(Part):
             self.conv, self.decay, self.o_norm, d.unit_eps, self.eps,
             state.s, state.conv, batch.segments, batch.row_seq, batch.ctx)
         return ops.linear(y, self.wo)
+
+
+class ChannelDelta(Branch):
+    """The delta rule with a decay per head and key channel
+    (ChannelDeltaDims). The inner numbers of decays and output gates are
+    columns of the input product; one second product, block-diagonal, turns
+    them into both."""
+
+    def __init__(self, d: ChannelDeltaDims, width: int, eps: float, dtype):
+        super().__init__()
+        self.d, self.width, self.eps = d, width, eps
+        self.wp = pad64(width)
+        self.dp, self.vp = state_pad(d.dim), state_pad(d.vdim)
+        H, G = d.heads, d.kv_heads
+        # columns: queries, keys, values (these pass the convolutions),
+        # the numbers behind step sizes, then the inner numbers
+        self.channels = 2 * G * self.dp + H * self.vp
+        self.inner_at = self.channels + pad64(H)
+        self.inner = pad64(d.decay_rank + d.gate_rank)
+        self.in_rows = self.inner_at + self.inner
+        self.out_cols = H * self.vp
+        # decays of all heads, then gates of all heads
+        self.w2 = weight(H * (self.dp + self.vp), self.inner, dtype)
+        self.conv = nn.Parameter(torch.empty(d.conv, self.channels,
+                                             dtype=torch.float32))
+        self.a_log = norm_weight(H)
+        self.dt_bias = norm_weight(H * self.dp)
+        self.o_norm = norm_weight(self.vp)
+
+    def tensors(self):
+        d, W = self.d, self.width
+        qk, k, v = d.kv_heads * d.dim, d.heads * d.dim, d.heads * d.vdim
+        return {"q": (qk, W), "q.conv": (qk, d.conv), "k": (qk, W),
+                "k.conv": (qk, d.conv), "v": (v, W), "v.conv": (v, d.conv),
+                "b": (d.heads, W), "A_log": (d.heads,), "norm": (d.vdim,),
+                "a1": (d.decay_rank, W), "a2": (k, d.decay_rank),
+                "dt_bias": (k,), "g1": (d.gate_rank, W),
+                "g2": (v, d.gate_rank), "o": (W, v)}
+
+    def _heads(self):
+        d = self.d
+        return (("q", d.kv_heads, d.dim, self.dp),
+                ("k", d.kv_heads, d.dim, self.dp),
+                ("v", d.heads, d.vdim, self.vp))
+
+    def in_weight(self, t):
+        w = [padded_heads(t[n], h, a, b, self.wp)
+             for n, h, a, b in self._heads()]
+        w.append(padded(t["b"], pad64(self.d.heads), self.wp))
+        w.append(padded(torch.cat([t["a1"], t["g1"]]), self.inner, self.wp))
+        return torch.cat(w)
+
+    def out_weight(self, t):
+        d = self.d
+        return padded_heads(t["o"].t(), d.heads, d.vdim, self.vp,
+                            self.wp).t()
+
+    def extra(self, t):
+        d, r = self.d, self.d.decay_rank
+        a2 = padded_heads(t["a2"], d.heads, d.dim, self.dp, self.inner)
+        g2 = padded_heads(t["g2"], d.heads, d.vdim, self.vp, d.gate_rank)
+        low = a2.new_zeros(d.heads * self.vp, self.inner)
+        low[:, r: r + d.gate_rank] = g2
+        return {"w2": torch.cat([a2, low]),
+                "conv": torch.cat([padded_heads(t[n + ".conv"], h, a, b,
+                                                d.conv)
+                                   for n, h, a, b in self._heads()]).t(),
+                "a_log": t["A_log"],
+                "dt_bias": padded_heads(t["dt_bias"][:, None], d.heads,
+                                        d.dim, self.dp, 1)[:, 0],
+                "o_norm": padded(t["norm"], self.vp)}
+
+    def state_numel(self):
+        return (self.d.heads * self.vp * self.dp,
+                (self.d.conv - 1) * self.channels)
+
+    def make_cache(self, num_blocks, blk, num_slots, dtype, device):
+        return DeltaState(self, num_slots, dtype, device)
+
+    def run(self, ab, batch, state, out, scale):
+        d = self.d
+        ag = ops.linear(ab[:, self.inner_at:], self.w2)
+        ops.channel_delta(
+            ab, ag, d.heads, d.kv_heads, self.dp, self.vp, d.dim, d.vdim,
+            self.conv, self.a_log, self.dt_bias, self.o_norm, d.unit_eps,
+            self.eps, scale, state.s, state.conv, batch.segments,
+            batch.row_seq, batch.ctx, out)

@@ -1,4 +1,4 @@
-"""Feed-forwards: xIELU and routed gated-unit experts."""
+"""Feed-forwards: SwiGLU, xIELU and routed gated-unit experts."""
 
 from __future__ import annotations
 
@@ -7,7 +7,32 @@ from torch import nn
 
 from .. import ops
 from .blocks import Part, pad64, padded, weight
-from .config import ExpertsDims, XieluDims
+from .config import ExpertsDims, SwigluDims, XieluDims
+
+
+class SwigluMlp(Part):
+    """down(silu(gate h) * (up h)): the clamped unit without a limit."""
+
+    def __init__(self, d: SwigluDims, width: int, dtype):
+        super().__init__()
+        self.d, self.width = d, width
+        self.wp, self.fp = pad64(width), pad64(d.ff)
+        self.wgup = weight(2 * self.fp, self.wp, dtype)
+        self.wdown = weight(self.wp, self.fp, dtype)
+
+    def tensors(self):
+        ff, W = self.d.ff, self.width
+        return {"gate": (ff, W), "up": (ff, W), "down": (W, ff)}
+
+    def checkpoint(self, src, pre):
+        t = self.checked(src, pre)
+        return {"wgup": torch.cat([padded(t[n], self.fp, self.wp)
+                                   for n in ("gate", "up")]),
+                "wdown": padded(t["down"], self.wp, self.fp)}
+
+    def forward(self, h):
+        y = ops.gateup_clamped_glu(h, self.wgup, float("inf"), 1.0, 0.0)
+        return ops.linear(y, self.wdown)
 
 
 class XieluMlp(Part):

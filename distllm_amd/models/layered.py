@@ -5,7 +5,8 @@ own; how they are joined to the fp32 residual stream is the design's and
 left to a subclass (`forward_step`). The model runs on ragged step
 batches only (engine/step.py): rows of any mix of prompt portions and
 single decoded tokens, against one cache entry per layer that owns one
-and, where there are recurrent layers, one state slot per sequence.
+and, where there are recurrent layers, one state slot per sequence. Layers
+of a loop run several times; every run has a cache entry of its own.
 """
 
 from __future__ import annotations
@@ -17,46 +18,67 @@ from .. import ops
 from .attention import PagedAttention
 from .blocks import (ClampedGlu, LatentAttention, expect, norm_weight, pad64,
                      padded, weight)
+from .branches import parallel_mixer
 from .config import (AttentionDims, ClampedGluDims, DeltaDims, ExpertsDims,
-                     LatentAttentionDims, LayeredDims, XieluDims)
+                     LatentAttentionDims, LayeredDims, LruDims, ParallelDims,
+                     SwigluDims, XieluDims)
 from .delta import GatedDelta
-from .feedforward import RoutedExperts, XieluMlp
+from .feedforward import RoutedExperts, SwigluMlp, XieluMlp
+from .recurrent import GatedLru
+from .side import SideInput
 
 MIXERS = {LatentAttentionDims: LatentAttention,
-          AttentionDims: PagedAttention, DeltaDims: GatedDelta}
-MLPS = {ClampedGluDims: ClampedGlu, XieluDims: XieluMlp,
-        ExpertsDims: RoutedExperts}
+          AttentionDims: PagedAttention, DeltaDims: GatedDelta,
+          ParallelDims: parallel_mixer, LruDims: GatedLru}
+MLPS = {ClampedGluDims: ClampedGlu, SwigluDims: SwigluMlp,
+        XieluDims: XieluMlp, ExpertsDims: RoutedExperts}
 
 
 class LayeredCache:
-    """What every layer keeps between steps. A layer that shares another
-    layer's cache holds the same object."""
+    """What every layer run keeps between steps. A layer that shares
+    another layer's cache holds the same object."""
 
     def __init__(self, model: "LayeredModel", num_blocks: int, blk: int,
                  num_slots: int = 0):
         self.layers: list = []
-        for layer in model.layers:
-            m = layer.mixer
-            self.layers.append(
-                m.make_cache(num_blocks, blk, num_slots, model.dtype,
-                             model.device)
-                if m.own else self.layers[m.kv_from])
+        latest: dict[int, object] = {}  # of the layer's runs so far
+        for i, _ in model.runs:
+            m = model.layers[i].mixer
+            latest[i] = (m.make_cache(num_blocks, blk, num_slots,
+                                      model.dtype, model.device)
+                         if m.own else latest[m.kv_from])
+            self.layers.append(latest[i])
 
 
 class Layer(nn.Module):
     def __init__(self, d, width: int, eps: float, dtype,
-                 norms: tuple[str, ...], mlp_norms: tuple[str, ...]):
+                 norms: tuple[str, ...], mlp_norms: tuple[str, ...],
+                 side: int | None = None):
         super().__init__()
         wp = pad64(width)
         self.mixer = MIXERS[type(d.mixer)](d.mixer, width, eps, dtype)
         self.mlp = None
         if d.mlp is not None:
             self.mlp = MLPS[type(d.mlp)](d.mlp, width, dtype)
+        self.side = (SideInput(side, width, dtype) if side is not None
+                     else None)
         self.norm_names = norms + (mlp_norms if self.mlp is not None else ())
         for n in norms + mlp_norms:
             present = n in self.norm_names
             setattr(self, n.replace(".", "_"),
-                    norm_weight(wp) if present else None)
+                    norm_weight(norm_size(n, wp)) if present else None)
+
+    def parts(self) -> list[tuple[str, str, nn.Module]]:
+        """(parameter prefix, checkpoint prefix, part)"""
+        return [(a, b, m) for a, b, m in
+                (("mixer.", "mix.", self.mixer), ("mlp.", "mlp.", self.mlp),
+                 ("side.", "side.", self.side)) if m is not None]
+
+
+def norm_size(name: str, wp: int) -> int:
+    """Numbers of a norm's tensor: one scale before the activation, or a
+    vector."""
+    return 1 if name.endswith(".alpha") else wp
 
 
 class LayeredModel(nn.Module):
@@ -70,6 +92,7 @@ class LayeredModel(nn.Module):
     mlp_norms: tuple[str, ...] = ()
     final_norms: tuple[str, ...] = ("final.norm",)
     has_positions = False  # a table of position vectors
+    tied_head = False      # the output product uses the embedding table
 
     def __init__(self, dims: LayeredDims, dtype=torch.bfloat16,
                  tp_group=None):
@@ -80,32 +103,51 @@ class LayeredModel(nn.Module):
         self.dims = dims
         W, wp = dims.hidden_size, pad64(dims.hidden_size)
         self.vp = pad64(dims.vocab_size)
-        self.tok_emb = weight(dims.vocab_size, wp, dtype)
+        # layer runs in order: (layer, loop pass that begins with it)
+        self.runs = dims.layer_runs()
+        self.tok_emb = weight(self.vp if self.tied_head else dims.vocab_size,
+                              wp, dtype)
         self.pos_emb = (weight(dims.max_position_embeddings, wp, dtype)
                         if self.has_positions else None)
         self.layers = nn.ModuleList(
             Layer(d, W, dims.norm_eps, dtype, self.layer_norms,
-                  self.mlp_norms) for d in dims.layers)
+                  self.mlp_norms, dims.side_dim) for d in dims.layers)
         for n in self.final_norms:
-            setattr(self, n.replace(".", "_"), norm_weight(wp))
-        self.lm_head = weight(self.vp, wp, dtype)
+            setattr(self, n.replace(".", "_"),
+                    norm_weight(norm_size(n, wp)))
+        self.side_emb = self.loop_step = None
+        if dims.side_dim is not None:
+            self.side_emb = weight(dims.vocab_size,
+                                   len(dims.layers) * dims.side_dim, dtype)
+        if dims.loop is not None:
+            self.loop_step = nn.Parameter(torch.empty(
+                dims.loop.times, wp, dtype=torch.float32))
+        if not self.tied_head:
+            self.lm_head = weight(self.vp, wp, dtype)
         self.reset_parameters()
 
     # ---- weights --------------------------------------------------------
     def _end_shapes(self) -> dict[str, tuple[int, ...]]:
         d = self.dims
-        t = {"embed": (d.vocab_size, d.hidden_size),
-             "head": (d.vocab_size, d.hidden_size)}
+        t = {"embed": (d.vocab_size, d.hidden_size)}
+        if not self.tied_head:
+            t["head"] = (d.vocab_size, d.hidden_size)
         if self.has_positions:
             t["pos"] = (d.max_position_embeddings, d.hidden_size)
-        return t | {n: (d.hidden_size,) for n in self.final_norms}
+        if d.side_dim is not None:
+            t["side.embed"] = (d.vocab_size, len(d.layers) * d.side_dim)
+        if d.loop is not None:
+            t["loop.step"] = (d.loop.times, d.hidden_size)
+        return t | {n: self._norm_shape(n) for n in self.final_norms}
+
+    def _norm_shape(self, name: str) -> tuple[int, ...]:
+        return () if name.endswith(".alpha") else (self.dims.hidden_size,)
 
     def _layer_shapes(self, i: int) -> dict[str, tuple[int, ...]]:
         layer, p = self.layers[i], f"l{i}."
-        t = {p + n: (self.dims.hidden_size,) for n in layer.norm_names}
-        for pre, part in (("mix.", layer.mixer), ("mlp.", layer.mlp)):
-            if part is not None:
-                t |= {p + pre + n: s for n, s in part.tensors().items()}
+        t = {p + n: self._norm_shape(n) for n in layer.norm_names}
+        for _, pre, part in layer.parts():
+            t |= {p + pre + n: s for n, s in part.tensors().items()}
         return t
 
     def checkpoint_names(self) -> set[str]:
@@ -118,24 +160,32 @@ class LayeredModel(nn.Module):
     def _end_tensors(self, src: dict) -> dict[str, torch.Tensor]:
         wp = self.tok_emb.shape[1]
         t = {n: expect(n, src[n], *s) for n, s in self._end_shapes().items()}
-        out = {"tok_emb": padded(t["embed"], self.dims.vocab_size, wp),
-               "lm_head": padded(t["head"], self.vp, wp)}
+        out = {"tok_emb": padded(t["embed"], *self.tok_emb.shape)}
+        if not self.tied_head:
+            out["lm_head"] = padded(t["head"], self.vp, wp)
         if self.has_positions:
             out["pos_emb"] = padded(t["pos"], t["pos"].shape[0], wp)
+        if self.side_emb is not None:
+            out["side_emb"] = t["side.embed"]
+        if self.loop_step is not None:
+            out["loop_step"] = padded(t["loop.step"], *self.loop_step.shape)
         for n in self.final_norms:
-            out[n.replace(".", "_")] = padded(t[n], wp)
+            out[n.replace(".", "_")] = self._norm_tensor(n, t[n])
         return out
+
+    def _norm_tensor(self, name: str, w: torch.Tensor) -> torch.Tensor:
+        w = expect(name, w, *self._norm_shape(name))
+        if w.dim() == 0:
+            return w.reshape(1)
+        return padded(w, self.tok_emb.shape[1])
 
     def _layer_tensors(self, src: dict, i: int) -> dict[str, torch.Tensor]:
         layer, p = self.layers[i], f"l{i}."
-        W, wp = self.dims.hidden_size, self.tok_emb.shape[1]
-        out = {n.replace(".", "_"): padded(expect(p + n, src[p + n], W), wp)
+        out = {n.replace(".", "_"): self._norm_tensor(p + n, src[p + n])
                for n in layer.norm_names}
-        for name, pre, part in (("mixer.", "mix.", layer.mixer),
-                                ("mlp.", "mlp.", layer.mlp)):
-            if part is not None:
-                for k, v in part.checkpoint(src, p + pre).items():
-                    out[name + k] = v
+        for name, pre, part in layer.parts():
+            for k, v in part.checkpoint(src, p + pre).items():
+                out[name + k] = v
         return {f"layers.{i}.{k}": v for k, v in out.items()}
 
     def checkpoint(self, src: dict) -> dict[str, torch.Tensor]:
@@ -156,7 +206,7 @@ class LayeredModel(nn.Module):
             for n, s in shapes.items():
                 if n.endswith(".b") and len(s) == 1:
                     src[n] = torch.zeros(s, device=self.device)
-                elif len(s) == 1:
+                elif len(s) <= 1:
                     src[n] = torch.ones(s, device=self.device)
                 else:
                     src[n] = torch.randn(s, device=self.device,
@@ -172,13 +222,14 @@ class LayeredModel(nn.Module):
     # ---- cache ----------------------------------------------------------
     def cache_bytes_per_block(self, blk: int, kv_cache_dtype: str) -> int:
         el = self.tok_emb.element_size()
-        return sum(layer.mixer.cache_numel() * blk * el
-                   for layer in self.layers if layer.mixer.own)
+        mixers = [self.layers[i].mixer for i, _ in self.runs]
+        return sum(m.cache_numel() * blk * el for m in mixers if m.own)
 
     def state_bytes_per_slot(self) -> int:
         el = self.tok_emb.element_size()
         return sum(f32 * 4 + own * el for f32, own in
-                   (layer.mixer.state_numel() for layer in self.layers))
+                   (self.layers[i].mixer.state_numel()
+                    for i, _ in self.runs))
 
     def make_cache(self, num_blocks: int, blk: int, kv_cache_dtype: str,
                    num_slots: int = 0) -> LayeredCache:
@@ -191,16 +242,17 @@ class LayeredModel(nn.Module):
     def forward_step(self, batch, cache: LayeredCache,
                      trace: list | None = None) -> torch.Tensor:
         """Final normed hidden state [M, padded width] of every row.
-        trace, when given, collects the residual after every layer."""
+        trace, when given, collects the residual after every layer run."""
         raise NotImplementedError
 
     @torch.no_grad()
     def logits(self, hidden: torch.Tensor) -> torch.Tensor:
         """hidden [..., width or padded width] -> [..., vocab] f32."""
-        wp = self.lm_head.shape[1]
+        head = self.tok_emb if self.tied_head else self.lm_head
+        wp = head.shape[1]
         if hidden.shape[-1] != wp:
             hidden = nn.functional.pad(hidden, (0, wp - hidden.shape[-1]))
-        out = ops.linear(hidden.contiguous(), self.lm_head)
+        out = ops.linear(hidden.contiguous(), head)
         out = out[..., : self.dims.vocab_size].float()
         scale = self.dims.logit_scale
         return out if scale == 1.0 else out * scale

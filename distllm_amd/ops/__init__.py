@@ -418,7 +418,6 @@ def gateup_clamped_glu(x, wgup, limit, alpha, shift):
     M, K = x.shape
     if x.is_cuda:
         _require_hip("_hip_gemm")
-        _require_hip("_hip_latent")
         if (M <= 256 and x.dtype == torch.bfloat16 and K % 64 == 0
                 and wgup.shape[0] % 128 == 0):
             sk = _decode_splitk(M, wgup.shape[0], K)
@@ -709,7 +708,7 @@ def up_xielu(x, wup, act):
     M, K = x.shape
     if x.is_cuda:
         _require_hip("_hip_gemm")
-        _require_hip("_hip_hybrid")
+        _require_hip("_hip_experts")
         if (M <= 256 and x.dtype == torch.bfloat16 and K % 64 == 0
                 and wup.shape[0] % 64 == 0):
             sk = _decode_splitk(M, wup.shape[0], K)
@@ -725,7 +724,7 @@ def route(h, router, ctx, top, groups, keep):
     Only experts of the `keep` groups with the largest scores count; rows
     with ctx 0 get ids -1 and weights 0."""
     if h.is_cuda:
-        _require_hip("_hip_hybrid")
+        _require_hip("_hip_experts")
         if h.dtype == torch.bfloat16 and router.shape[0] <= 256:
             return _hip_ops.route(h, router, ctx, top, groups, keep)
         logits = torch.nn.functional.linear(h.float(), router.float())
@@ -738,6 +737,143 @@ def experts(h, ids, wgup, wdown):
     ids[m, k] of row m (undefined for id -1). wgup [E, 2F, W]: gate and up
     rows alternate in groups of 16."""
     if h.is_cuda:
-        _require_hip("_hip_hybrid")
+        _require_hip("_hip_experts")
         return _hip_ops.experts(h, ids, wgup, wdown)
     return torch_ref.experts(h, ids, wgup, wdown)
+
+
+# ---- parallel attention and delta rule / linear recurrent decoder -----------
+
+def residual_step(x, y=None, bias=None, rms=None, embed=None, vec=None,
+                  act=None, fresh=False, dtype=None):
+    """One boundary of an fp32 residual stream x [M, W], in place:
+      x += y + bias (fp32 vector), or rms(y) * w with rms = (w, n, eps),
+           statistics over n columns
+      x += scale * table[token] with embed = (tokens, table, scale)
+      x += vec (fp32 vector)
+    all of them optional; with `fresh` x starts from zeros. Returns x, or
+    tanh(alpha x) * w + b with act = (w, b, alpha), in `dtype` (default:
+    that of y, of the table without y)."""
+    if dtype is None:
+        dtype = y.dtype if y is not None else embed[1].dtype
+    if x.is_cuda:
+        _require_hip("_hip_residual")
+        tokens, table, scale = embed if embed is not None else (None, None,
+                                                                1.0)
+        w_rms, n, eps = rms if rms is not None else (None, x.shape[1], 0.0)
+        w, b, alpha = act if act is not None else (None, None, None)
+        h = torch.empty(x.shape, dtype=dtype, device=x.device)
+        _hip_ops.residual_step(x, y, bias, w_rms, n, eps, tokens, table,
+                               scale, vec, w, b, alpha, fresh, h)
+        return h
+    return torch_ref.residual_step(x, y, bias, rms, embed, vec, act, fresh,
+                                   dtype)
+
+
+def gated_rows(x, wgate, tokens, table, col0, n):
+    """gelu_tanh(x @ wgate^T) * table[token, col0: col0 + n], zeros in the
+    columns of wgate behind n."""
+    if x.is_cuda:
+        _require_hip("_hip_gemm")
+        M, K = x.shape
+        if (M <= 256 and x.dtype == torch.bfloat16 and K % 64 == 0):
+            sk = _decode_splitk(M, wgate.shape[0], K)
+            if sk > 1:
+                return _hip_ops.decode_gemm_rows(x, wgate, sk, tokens, table,
+                                                 col0, n)
+        return _hip_ops.gelu_rows(linear(x, wgate), tokens, table, col0, n)
+    return torch_ref.gelu_rows(linear(x, wgate), tokens, table, col0, n)
+
+
+def rotation_table(ctx, freq, mult):
+    """mult * (cos, sin) of freq (fp64) times the position ctx - 1 of every
+    row: [M, pairs, 2] fp32."""
+    if ctx.is_cuda:
+        _require_hip("_hip_hybrid")
+        return _hip_ops.rotation_table(ctx, freq, mult)
+    return torch_ref.rotation_table(ctx, freq, mult)
+
+
+def rotary_prep(ab, heads, kv_heads, dp, dim, wq, wk, eps, table, pages,
+                block_table, row_seq, ctx):
+    """Norm and rotate the query heads of a projection ab [M, queries |
+    keys] (returned, [M, heads, dp]) and its key heads; those go to the key
+    pages, keys as projected to the value pages (position ctx - 1; ctx 0
+    writes nothing). The first 2 * pairs numbers of a head rotate."""
+    if ab.is_cuda:
+        _require_hip("_hip_hybrid")
+        return _hip_ops.rotary_prep(ab, heads, kv_heads, dp, dim, wq, wk,
+                                    eps, table, pages[0], pages[1],
+                                    block_table, row_seq, ctx)
+    return torch_ref.rotary_prep(ab, heads, kv_heads, dp, dim, wq, wk, eps,
+                                 table, pages, block_table, row_seq, ctx)
+
+
+def sink_attn_rows(q, kpages, vpages, out, block_table, row_seq, ctx, scale,
+                   sink, out_scale, nsplit=0):
+    """Causal attention of single-token rows over paged keys and values;
+    exp(sink) of the head is part of the softmax's denominator. out
+    [M, heads * vdim] (rows may be strided) takes the result times
+    out_scale."""
+    if q.is_cuda:
+        _require_hip("_hip_hybrid")
+        _hip_ops.sink_attn_rows(q, kpages, vpages, out, block_table, row_seq,
+                                ctx, scale, sink, out_scale, nsplit)
+        return out
+    return torch_ref.sink_attn_rows(q, kpages, vpages, out, block_table,
+                                    row_seq, ctx, scale, sink, out_scale)
+
+
+def sink_attn_prompts(q, kpages, vpages, out, block_table, prompts, scale,
+                      sink, out_scale):
+    """The same for the rows of prompt portions (step.PromptBlocks)."""
+    if q.is_cuda:
+        _require_hip("_hip_hybrid")
+        _hip_ops.sink_attn_prompts(q, kpages, vpages, out, block_table,
+                                   prompts.portions, prompts.blocks, scale,
+                                   sink, out_scale)
+        return out
+    return torch_ref.sink_attn_prompts(q, kpages, vpages, out, block_table,
+                                       prompts, scale, sink, out_scale)
+
+
+def channel_delta(ab, ag, heads, kv_heads, dp, vp, dim, vdim, conv_w, a_log,
+                  dt_bias, o_norm, unit_eps, eps, out_scale, state, conv,
+                  segments, row_seq, ctx, out):
+    """Delta rule with a decay per key channel of a ragged step, on the
+    projection ab [M, queries | keys | values | b] and the second product
+    ag [M, decays | gates]: short convolutions, unit queries and keys,
+    recurrence in fp32, output norm, sigmoid gate, out_scale. out
+    [M, heads * vp] (rows may be strided); state and convolution slots are
+    updated."""
+    if ab.is_cuda:
+        _require_hip("_hip_hybrid")
+        _hip_ops.channel_delta(
+            ab, ag, heads, kv_heads, dp, vp, dim, vdim, conv_w, a_log,
+            dt_bias, o_norm, unit_eps, eps, out_scale, state, conv,
+            segments.row0, segments.rows, segments.slot, segments.longest,
+            row_seq, ctx, segments.longs, segments.chunks, segments.SHORT,
+            out)
+        return out
+    return torch_ref.channel_delta(
+        ab, ag, heads, kv_heads, dp, vp, dim, vdim, conv_w, a_log, dt_bias,
+        o_norm, unit_eps, eps, out_scale, state, conv, segments, row_seq,
+        ctx, out)
+
+
+def gated_lru(ab, conv_w, conv_b, gates, gates_b, decay, state, conv,
+              segments, row_seq, ctx, chunk):
+    """Linear recurrent unit of a ragged step on the projection ab [M,
+    GELU branch | recurrent branch]: convolution, block-diagonal gates,
+    recurrence in fp32, times the GELU branch. -> [M, width]; state and
+    convolution slots are updated. Long segments run in chunks of `chunk`
+    rows."""
+    if ab.is_cuda:
+        _require_hip("_hip_lru")
+        longs, chunks = segments.chunk_lists(chunk)
+        return _hip_ops.gated_lru(
+            ab, conv_w, conv_b, gates, gates_b, decay, state, conv,
+            segments.row0, segments.rows, segments.slot, segments.longest,
+            row_seq, ctx, longs, chunks, chunk, segments.SHORT)
+    return torch_ref.gated_lru(ab, conv_w, conv_b, gates, gates_b, decay,
+                               state, conv, segments, row_seq, ctx)

@@ -539,3 +539,169 @@ def experts(h, ids, wgup, wdown, unit=16):
         a = a.reshape(len(rows), -1).to(h.dtype)
         out[rows] = (a.float() @ wdown[e].float().t()).to(h.dtype)
     return out
+
+
+# ---- parallel attention and delta rule / linear recurrent decoder -----------
+
+def residual_step(x, y, bias, rms, embed, vec, act, fresh, dtype):
+    if fresh:
+        x.zero_()
+    if y is not None:
+        v = y.float()
+        if rms is not None:
+            w, n, eps = rms
+            ms = v.pow(2).sum(-1, keepdim=True) / n
+            v = v / torch.sqrt(ms + eps) * w
+        x += v if bias is None else v + bias
+    if embed is not None:
+        tokens, table, scale = embed
+        x += table[tokens.long()].float() * scale
+    if vec is not None:
+        x += vec
+    if act is None:
+        return x.to(dtype)
+    w, b, alpha = act
+    return (torch.tanh(alpha * x) * w + b).to(dtype)
+
+
+def gelu_rows(z, tokens, table, col0, n):
+    e = table[tokens.long(), col0: col0 + n].float()
+    out = torch.zeros_like(z)
+    out[:, :n] = (F.gelu(z[:, :n].float(), approximate="tanh") * e).to(
+        z.dtype)
+    return out
+
+
+def rotation_table(ctx, freq, mult):
+    a = (ctx.double() - 1).clamp(min=0)[:, None] * freq
+    return (torch.stack([a.cos(), a.sin()], -1) * mult).float()
+
+
+def rotary_prep(ab, heads, kv_heads, dp, dim, wq, wk, eps, table, pages,
+                block_table, row_seq, ctx):
+    M, half = ab.shape[0], table.shape[1]
+    cos, sin = table[:, None, :, 0], table[:, None, :, 1]
+
+    def prep(v, w):
+        v = v.reshape(M, -1, dp).float()
+        ms = v.pow(2).sum(-1, keepdim=True) / dim
+        v = v / torch.sqrt(ms + eps) * w
+        a, b = v[..., :half], v[..., half: 2 * half]
+        return torch.cat([a * cos - b * sin, b * cos + a * sin,
+                          v[..., 2 * half:]], -1).to(ab.dtype)
+
+    kp, vpg = pages
+    blk = kp.shape[2]
+    live = ctx > 0
+    rows = _cache_rows(block_table, row_seq[live], ctx[live] - 1, blk)
+    k = ab[:, heads * dp: (heads + kv_heads) * dp]
+    kp[rows // blk, :, rows % blk] = prep(k, wk)[live]
+    vpg[rows // blk, :, :, rows % blk] = k[live].reshape(-1, kv_heads, dp)
+    return prep(ab[:, : heads * dp], wq)
+
+
+def sink_attn_rows(q, kpages, vpages, out, block_table, row_seq, ctx, scale,
+                   sink, out_scale):
+    M, H, _ = q.shape
+    G, blk = kpages.shape[1], kpages.shape[2]
+    for r in range(M):
+        n = int(ctx[r])
+        if n <= 0:
+            out[r] = 0
+            continue
+        rows = _cache_rows(block_table, row_seq[r].expand(n),
+                           torch.arange(n), blk)
+        k = kpages[rows // blk, :, rows % blk].float()
+        v = vpages[rows // blk, :, :, rows % blk].float()
+        k = k.repeat_interleave(H // G, 1).transpose(0, 1)   # [H, n, d]
+        v = v.repeat_interleave(H // G, 1).transpose(0, 1)
+        s = (k * q[r].float()[:, None]).sum(-1) * scale
+        w = torch.softmax(torch.cat([s, sink.float()[:, None]], 1), -1)
+        o = (w[:, :n, None] * v).sum(1) * out_scale
+        out[r] = o.reshape(-1).to(q.dtype)
+    return out
+
+
+def sink_attn_prompts(q, kpages, vpages, out, block_table, prompts, scale,
+                      sink, out_scale):
+    for seq, row0, start, n in prompts.portions.tolist():
+        r = slice(row0, row0 + n)
+        sink_attn_rows(q[r], kpages, vpages, out[r], block_table,
+                       torch.full((n,), seq, dtype=torch.int32),
+                       torch.arange(start + 1, start + n + 1), scale, sink,
+                       out_scale)
+    return out
+
+
+def _short_conv(x, conv_w, slot, conv, start):
+    """Causal convolution of one segment's rows x [n, C] (fp32 result); its
+    slot of last inputs is read and renewed."""
+    n, taps = x.shape[0], conv_w.shape[0]
+    x = torch.cat([conv[slot] * (start > 0), x])
+    conv[slot] = x[n:]
+    return sum(x[a: a + n].float() * conv_w[a] for a in range(taps))
+
+
+def channel_delta(ab, ag, heads, kv_heads, dp, vp, dim, vdim, conv_w, a_log,
+                  dt_bias, o_norm, unit_eps, eps, out_scale, state, conv,
+                  segments, row_seq, ctx, out):
+    C = conv_w.shape[1]
+    G, H = kv_heads, heads
+    own = torch.arange(H) // (H // G)
+    for row0, n, slot in zip(segments.row0.tolist(), segments.rows.tolist(),
+                             segments.slot.tolist()):
+        if n == 0:
+            continue
+        r = slice(row0, row0 + n)
+        start = int(ctx[row0]) - 1
+        S = state[slot] * (start > 0)                  # [H, vp, dp]
+        z = F.silu(_short_conv(ab[r, :C], conv_w, slot, conv, start))
+        qk = z[:, : 2 * G * dp].view(n, 2, G, dp)
+        qk = qk / torch.sqrt(qk.pow(2).sum(-1, keepdim=True) + unit_eps)
+        q, k = qk[:, 0, own] * dim ** -0.5, qk[:, 1, own]
+        v = z[:, 2 * G * dp:].to(ab.dtype).float().view(n, H, vp)
+        beta = torch.sigmoid(ab[r, C: C + H].float())
+        a = F.softplus(ag[r, : H * dp].float() + dt_bias).view(n, H, dp)
+        g = torch.exp(-torch.exp(a_log)[:, None] * a)
+        gate = torch.sigmoid(ag[r, H * dp:].float()).view(n, H, vp)
+        for i in range(n):
+            S = S * g[i, :, None]
+            u = beta[i, :, None] * (v[i] - (S * k[i, :, None]).sum(-1))
+            S = S + u[..., None] * k[i, :, None]
+            o = (S * q[i, :, None]).sum(-1)            # [H, vp]
+            ms = o.pow(2).sum(-1, keepdim=True) / vdim
+            y = o / torch.sqrt(ms + eps) * o_norm * gate[i] * out_scale
+            out[row0 + i] = y.reshape(-1).to(ab.dtype)
+        state[slot] = S
+    return out
+
+
+def gated_lru(ab, conv_w, conv_b, gates, gates_b, decay, state, conv,
+              segments, row_seq, ctx):
+    M, C = ab.shape[0], conv_w.shape[1]
+    B, bs = gates.shape[1], gates.shape[2]
+    out = torch.zeros(M, C, dtype=ab.dtype)
+    for row0, n, slot in zip(segments.row0.tolist(), segments.rows.tolist(),
+                             segments.slot.tolist()):
+        if n == 0:
+            continue
+        r = slice(row0, row0 + n)
+        start = int(ctx[row0]) - 1
+        S = state[slot] * (start > 0)
+        u = _short_conv(ab[r, C:], conv_w, slot, conv, start) + conv_b
+        u = u.to(ab.dtype).float()
+        z = torch.zeros(2, n, C)
+        z[..., : B * bs] = torch.matmul(
+            u[:, : B * bs].view(n, B, bs).transpose(0, 1),
+            gates.float().transpose(2, 3).contiguous()
+        ).transpose(1, 2).reshape(2, n, B * bs)
+        z = torch.sigmoid(z + gates_b[:, None])
+        log_a = decay * z[0]
+        drive = torch.sqrt(-torch.expm1(2 * log_a)) * z[1] * u
+        a = torch.exp(log_a)
+        y = F.gelu(ab[r, :C].float(), approximate="tanh")
+        for i in range(n):
+            S = a[i] * S + drive[i]
+            out[row0 + i] = (S * y[i]).to(ab.dtype)
+        state[slot] = S
+    return out

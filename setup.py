@@ -5,10 +5,12 @@
 The kernels are grouped into a few extensions, so that a process which
 needs one group does not have to compile the others:
 
-    _hip_gemm      matrix products (every model)
+    _hip_gemm      matrix products and gated units (every model)
     _hip_residual  norms around an fp32 residual stream
-    _hip_latent    latent attention, clamped GLU
-    _hip_hybrid    chunked attention, delta rule, xIELU, routed experts
+    _hip_latent    latent attention
+    _hip_hybrid    attention over pages of keys and values, delta rules
+    _hip_experts   xIELU, routed experts
+    _hip_lru       linear recurrent unit
     _hip_ops       everything else
 
 DISTLLM_EXT=_hip_gemm,_hip_latent restricts a build to the named ones.
@@ -26,14 +28,17 @@ from torch.utils.cpp_extension import BuildExtension, CUDAExtension
 CSRC = Path(__file__).parent / "distllm_amd" / "ops" / "csrc"
 GROUPS = {
     "_hip_gemm": ["ext_gemm.cpp", "blt_gemm.cpp", "gemm.hip", "gemm8.hip",
-                  "gemm16.hip", "decode_gemm.hip"],
+                  "gemm16.hip", "decode_gemm.hip", "clamped_glu.hip"],
     "_hip_latent": ["ext_latent.cpp", "latent_attention.hip",
-                    "latent_decode.hip", "window_attention.hip",
-                    "clamped_glu.hip"],
+                    "latent_decode.hip", "window_attention.hip"],
     "_hip_residual": ["ext_residual.cpp", "residual_norms.hip"],
     "_hip_hybrid": ["ext_hybrid.cpp", "chunk_attention.hip",
-                    "chunk_flash.hip", "delta_rule.hip", "delta_chunk.hip",
-                    "experts.hip", "expert_gemm16.hip", "xielu.hip"],
+                    "chunk_rows.hip", "chunk_flash.hip", "sink_rows.hip",
+                    "sink_flash.hip", "delta_rule.hip", "delta_chunk.hip",
+                    "delta_channel.hip"],
+    "_hip_experts": ["ext_experts.cpp", "experts.hip", "expert_gemm16.hip",
+                     "xielu.hip"],
+    "_hip_lru": ["ext_lru.cpp", "lru.hip"],
 }
 _taken = {s for group in GROUPS.values() for s in group}
 # *_hip.hip files are torch-hipify build artifacts — exclude them.
