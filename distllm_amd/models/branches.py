@@ -44,15 +44,14 @@ class BranchMixer(Part):
         biases = [b.in_bias(t) for b, t, _ in each]
         out = {"win": torch.cat([b.in_weight(t) for b, t, _ in each]),
                "bias": torch.cat([
-                   x if x is not None else self.win.new_zeros(b.in_rows)
-                   for x, b in zip(biases, self.branches)]),
+                   x if x is not None else next(iter(t.values())).new_zeros(
+                       b.in_rows)
+                   for x, (b, t, _) in zip(biases, each)]),
                "wo": torch.cat([b.out_weight(t) for b, t, _ in each], 1)}
-        total = torch.zeros_like(self.out_bias)
-        for b, t, scale in each:
-            x = b.out_bias(t)
-            if x is not None:
-                total += scale * padded(x.float(), self.wp).to(total.device)
-        out["out_bias"] = total
+        total = [scale * padded(b.out_bias(t).float(), self.wp)
+                 for b, t, scale in each if b.out_bias(t) is not None]
+        out["out_bias"] = sum(total, out["win"].new_zeros(
+            self.wp, dtype=torch.float32))
         for i, (b, t, _) in enumerate(each):
             out |= {f"branches.{i}.{k}": v for k, v in b.extra(t).items()}
         return out

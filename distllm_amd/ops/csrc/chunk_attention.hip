@@ -1,17 +1,56 @@
-// Attention of single-token rows (see chunk_attention.h): norm and cache
-// write, a generic kernel for any size and type, and the MFMA kernel of
-// bf16 decode steps.
+// What precedes attention over pages (see chunk_attention.h): norm and
+// rotation of query and key heads, cache write.
 #include "chunk_attention.h"
 
-extern __shared__ __attribute__((aligned(16))) char smem[];
+// ---- cos and sin of every row's position ------------------------------------
+__global__ void __launch_bounds__(256)
+rotation_table_kernel(const int* __restrict__ ctx,
+                      const double* __restrict__ freq, float mult,
+                      float* __restrict__ table, int M, int pairs) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= (long)M * pairs) return;
+  const double a = (double)max(ctx[i / pairs] - 1, 0) * freq[i % pairs];
+  // to [-pi, pi] before the angle becomes 32 bits wide
+  const double turns = a * 0.15915494309189535;
+  float s, c;
+  sincosf((float)((turns - rint(turns)) * 6.283185307179586), &s, &c);
+  table[i * 2] = c * mult;
+  table[i * 2 + 1] = s * mult;
+}
+
+extern "C" void launch_rotation_table(const int* ctx, const double* freq,
+                                      float mult, float* table, int M,
+                                      int pairs, hipStream_t stream) {
+  hipLaunchKernelGGL(rotation_table_kernel,
+                     dim3(((long)M * pairs + 255) / 256), dim3(256), 0,
+                     stream, ctx, freq, mult, table, M, pairs);
+}
+
+// Rotation of the numbers c .. c + 7 of a normed head, in place; x_of(i)
+// yields number i of the head. cs: cos, sin of the row's pairs.
+template <typename F>
+__device__ __forceinline__ void rotate8(float* x, int c, int half,
+                                        const float* cs, F x_of) {
+#pragma unroll
+  for (int i = 0; i < 8; ++i) {
+    const int col = c + i;
+    if (col >= 2 * half) return;
+    const bool low = col < half;
+    const int pair = low ? col : col - half;
+    const float other = x_of(low ? col + half : pair);
+    x[i] = x[i] * cs[pair * 2] +
+           (low ? -other : other) * cs[pair * 2 + 1];
+  }
+}
 
 // ---- norm of query and key heads, cache write -----------------------------
 // ab row: H query heads of dp, then (own keys) G key heads of dp and G value
-// heads of vp. LPH lanes share a query or key head, a workgroup norms UN
-// times 256 / LPH of them. Values: the first row of a run of consecutive
-// positions in one page writes the run, whole 32-byte page rows where the
-// run covers the page; a wave looks at VR rows of one head.
-template <typename T, int LPH, int UN>
+// heads of vp, from column v_at on. With a table, the first 2 * half numbers
+// of a normed head are rotated. LPH lanes share a query or key head, a
+// workgroup norms UN times 256 / LPH of them. Values: the first row of a run
+// of consecutive positions in one page writes the run, whole 32-byte page
+// rows where the run covers the page; a wave looks at VR rows of one head.
+template <typename T, int LPH, int UN, bool ROT>
 __global__ void __launch_bounds__(256)
 attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
                  int dp, int vp, int n, const float* __restrict__ wq,
@@ -19,7 +58,8 @@ attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
                  T* __restrict__ kpages, T* __restrict__ vpages,
                  const int* __restrict__ block_table, int max_blocks,
                  int num_blocks, const int* __restrict__ row_seq,
-                 const int* __restrict__ ctx, int norm_wgs, int VR) {
+                 const int* __restrict__ ctx, int norm_wgs, int VR, int v_at,
+                 const float* __restrict__ table, int half) {
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   // page of a position, or -1
   auto page_of = [&](int row, int pos) {
@@ -78,6 +118,22 @@ attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
         load8<float>(w + c, wv);
 #pragma unroll
         for (int i = 0; i < 8; ++i) x[i] = v[k][i] * inv * wv[i];
+        if (ROT && c < 2 * half) {
+          const float* cs = table + (long)row * 2 * half;
+          if (half % 8 == 0) {  // the other numbers are eight in a row too
+            const int o = c < half ? c + half : c - half;
+            float y[8], yw[8];
+            load8<T>(src + o, y);
+            load8<float>(w + o, yw);
+            rotate8(x, c, half, cs, [&](int j) {
+              return y[j - o] * inv * yw[j - o];
+            });
+          } else {
+            rotate8(x, c, half, cs, [&](int j) {
+              return to_f(src[j]) * inv * w[j];
+            });
+          }
+        }
         store8(dst + c, x);
       }
     }
@@ -103,7 +159,7 @@ attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
     while (pos % PBLK + run < PBLK && row + run < M &&
            row_seq[row + run] == seq && ctx[row + run] == ctx[row] + run)
       ++run;
-    const T* src = ab + (long)row * ld + (long)(H + G) * dp + (long)g * vp;
+    const T* src = ab + (long)row * ld + v_at + (long)g * vp;
     T* dst = vpages + ((long)page * G + g) * vp * PBLK;
     for (int c = lane * 2; c < vp; c += 128) {
       typedef __attribute__((ext_vector_type(2))) T pair;
@@ -136,11 +192,13 @@ attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
   }
 }
 
+// table [M, half, 2] or null
 extern "C" void launch_attn_prep(
     const void* ab, int ld, int M, int H, int G, int dp, int vp, int n,
     const float* wq, const float* wk, float eps, void* q, void* kpages,
     void* vpages, const int* block_table, int max_blocks, int num_blocks,
-    const int* row_seq, const int* ctx, bool fp32, hipStream_t stream) {
+    const int* row_seq, const int* ctx, int v_at, const float* table,
+    int half, bool fp32, hipStream_t stream) {
   const int lph = dp <= 64 ? 8 : dp <= 128 ? 16 : dp <= 256 ? 32 : 64;
   const bool own = kpages != nullptr;
   const long units = (long)M * (H + (own ? G : 0));
@@ -148,12 +206,17 @@ extern "C" void launch_attn_prep(
   const int per = 256 / lph * un;
   const int norm_wgs = (int)((units + per - 1) / per);
   const int v_wgs = own ? (int)(((long)(M + vr - 1) / vr * G + 3) / 4) : 0;
-#define APK(T, L, U)                                                          \
-  hipLaunchKernelGGL((attn_prep_kernel<T, L, U>), dim3(norm_wgs + v_wgs),     \
+#define APK_R(T, L, U, R)                                                     \
+  hipLaunchKernelGGL((attn_prep_kernel<T, L, U, R>), dim3(norm_wgs + v_wgs),  \
                      dim3(256), 0, stream, (const T*)ab, ld, M, H, G, dp, vp, \
                      n, wq, wk, eps, (T*)q, (T*)kpages, (T*)vpages,           \
                      block_table, max_blocks, num_blocks, row_seq, ctx,       \
-                     norm_wgs, vr)
+                     norm_wgs, vr, v_at, table, half)
+#define APK(T, L, U)                             \
+  do {                                           \
+    if (table != nullptr) APK_R(T, L, U, true);  \
+    else APK_R(T, L, U, false);                  \
+  } while (0)
 #define APK_U(T, L)           \
   do {                        \
     if (un == 1) APK(T, L, 1); \
@@ -171,373 +234,5 @@ extern "C" void launch_attn_prep(
 #undef APK_L
 #undef APK_U
 #undef APK
-}
-
-// ---- one workgroup per (row, head), any size and type ---------------------
-// NV: value columns per thread (DV <= 256 * NV). Library functions
-// throughout: this is also the kernel of the 32-bit mode.
-template <typename T, int NV>
-__global__ void __launch_bounds__(256)
-chunk_rows_kernel(const T* __restrict__ q, const T* __restrict__ kpages,
-                  const T* __restrict__ vpages, const T* __restrict__ gate,
-                  int ld_gate, const int* __restrict__ block_table,
-                  const int* __restrict__ row_seq,
-                  const int* __restrict__ ctx, T* __restrict__ out, int H,
-                  int G, int DK, int DV, int max_blocks, int chunk,
-                  float scale, float softcap,
-                  const float* __restrict__ dist) {
-  constexpr int V = 16 / sizeof(T);
-  typedef __attribute__((ext_vector_type(V))) T vec;
-  float* q_lds = reinterpret_cast<float*>(smem);         // DK
-  float* p_lds = q_lds + DK;                             // 256
-  int* page_lds = reinterpret_cast<int*>(p_lds + 256);   // 256
-  float* red = reinterpret_cast<float*>(page_lds + 256);  // 8
-  const int row = blockIdx.x / H, head = blockIdx.x % H;
-  const int g = head / (H / G);
-  const int tid = threadIdx.x, wid = tid >> 6, lane = tid & 63;
-  const int L = min(ctx[row], max_blocks * PBLK);
-  const int lo = L > 0 ? (L - 1) / chunk * chunk : 0;
-  const int* bt = block_table + (long)row_seq[row] * max_blocks;
-  const T* qr = q + ((long)row * H + head) * DK;
-  for (int c = tid; c < DK; c += 256) q_lds[c] = to_f(qr[c]);
-  const float r1 = dist[head], r2 = dist[H + head];
-
-  float m = -INFINITY, l = 0.f, acc[NV];
-#pragma unroll
-  for (int i = 0; i < NV; ++i) acc[i] = 0.f;
-  for (int t0 = lo; t0 < L; t0 += 256) {
-    const int key = t0 + tid;
-    const bool live = key < L;
-    __syncthreads();  // q is staged; the previous tile is consumed
-    float s = -INFINITY;
-    if (live) {
-      const long page = (long)bt[key / PBLK] * G + g;
-      page_lds[tid] = (int)page;
-      const T* k = kpages + (page * PBLK + key % PBLK) * DK;
-      float dot = 0.f;
-      for (int c = 0; c < DK; c += V) {
-        const vec kv = *reinterpret_cast<const vec*>(k + c);
-#pragma unroll
-        for (int i = 0; i < V; ++i) dot += to_f((T)kv[i]) * q_lds[c + i];
-      }
-      s = softcap * tanhf(dot * scale / softcap) -
-          r1 * log1pf(r2 * (float)(L - 1 - key));
-    }
-    const float wmax = wave_reduce_max(s);
-    if (lane == 0) red[wid] = wmax;
-    __syncthreads();
-    const float mn =
-        fmaxf(m, fmaxf(fmaxf(red[0], red[1]), fmaxf(red[2], red[3])));
-    const float p = live ? expf(s - mn) : 0.f;
-    p_lds[tid] = p;
-    const float wsum = wave_reduce_sum(p);
-    if (lane == 0) red[4 + wid] = wsum;
-    __syncthreads();
-    const float alpha = expf(m - mn);  // 0 on the first tile
-    l = l * alpha + (red[4] + red[5]) + (red[6] + red[7]);
-    m = mn;
-    const int nk = min(256, L - t0);
-#pragma unroll
-    for (int i = 0; i < NV; ++i) {
-      const int c = tid + i * 256;
-      if (c < DV) {
-        float a = acc[i] * alpha;
-        for (int j = 0; j < nk; ++j)
-          a += p_lds[j] * to_f(vpages[((long)page_lds[j] * DV + c) * PBLK +
-                                      (t0 + j) % PBLK]);
-        acc[i] = a;
-      }
-    }
-  }
-  const float inv = l > 0.f ? 1.f / l : 0.f;
-  T* o = out + ((long)row * H + head) * DV;
-  const T* gr = gate + (long)row * ld_gate + (long)head * DV;
-#pragma unroll
-  for (int i = 0; i < NV; ++i) {
-    const int c = tid + i * 256;
-    if (c < DV) from_f(o + c, acc[i] * inv * sigmoid_exact(to_f(gr[c])));
-  }
-}
-
-extern "C" void launch_chunk_rows(const void* q, const void* kpages,
-                                  const void* vpages, const void* gate,
-                                  int ld_gate, const int* block_table,
-                                  const int* row_seq, const int* ctx,
-                                  void* out, int M, int H, int G, int DK,
-                                  int DV, int max_blocks, int chunk,
-                                  float scale, float softcap,
-                                  const float* dist, bool fp32,
-                                  hipStream_t stream) {
-  const int lds = (DK + 256 + 256 + 8) * 4;
-#define CR(T, NV)                                                             \
-  hipLaunchKernelGGL((chunk_rows_kernel<T, NV>), dim3(M * H), dim3(256), lds, \
-                     stream, (const T*)q, (const T*)kpages, (const T*)vpages, \
-                     (const T*)gate, ld_gate, block_table, row_seq, ctx,      \
-                     (T*)out, H, G, DK, DV, max_blocks, chunk, scale,         \
-                     softcap, dist)
-#define CR_N(T)                  \
-  do {                           \
-    if (DV <= 256) CR(T, 1);     \
-    else if (DV <= 1024) CR(T, 4); \
-    else CR(T, 16);              \
-  } while (0)
-  if (fp32) CR_N(float);
-  else CR_N(unsigned short);
-#undef CR_N
-#undef CR
-}
-
-// ---- MFMA kernel of decode rows --------------------------------------------
-// A workgroup serves up to 16 query heads of one key/value head of one row;
-// NS workgroups share a row's keys. A wave takes every fourth tile of 32
-// keys (two pages), both operands straight from the pages: for the scores
-// (keys x heads) the 16 x DK key page is the A operand, for the output
-// (value columns x heads) the DV x 16 value pages are. Key tile position
-// t * 16 + g * 4 + r sits in lane group g of both products' operands, so the
-// weights need no exchange between lanes.
-template <int DK, int DV>
-__global__ void __launch_bounds__(256, 2)
-chunk_decode_kernel(const unsigned short* __restrict__ q,
-                    const unsigned short* __restrict__ kpages,
-                    const unsigned short* __restrict__ vpages,
-                    const unsigned short* __restrict__ gate, int ld_gate,
-                    const int* __restrict__ block_table,
-                    const int* __restrict__ row_seq,
-                    const int* __restrict__ ctx,
-                    unsigned short* __restrict__ out,
-                    float* __restrict__ pacc, float* __restrict__ pml, int H,
-                    int G, int NG, int NS, int max_blocks, int chunk,
-                    float c_in, float c_out,
-                    const float* __restrict__ dist) {
-  constexpr int OROW = DV + 4;  // padded row of the joining buffer
-  const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
-  const int i16 = lane & 15, g = lane >> 4;
-  const int split = blockIdx.x % NS;
-  const int grp = blockIdx.x / NS % NG;
-  const int kvh = blockIdx.x / NS / NG % G;
-  const int row = blockIdx.x / NS / NG / G;
-  const int GR = H / G;
-  const int nlive = min(16, GR - grp * 16);
-  const bool live = i16 < nlive;
-  const int head = kvh * GR + grp * 16 + (live ? i16 : 0);
-
-  const int L = min(ctx[row], max_blocks * PBLK);
-  const int lo = L > 0 ? (L - 1) / chunk * chunk : 0;
-  const int T0 = lo / 32, T1 = L > 0 ? (L + 31) / 32 : T0;
-  const int per = (T1 - T0 + NS - 1) / NS;
-  const int ts = T0 + split * per, te = min(T1, ts + per);
-  const int last_page = L > 0 ? (L - 1) / PBLK : 0;
-  const int* bt = block_table + (long)row_seq[row] * max_blocks;
-
-  bf16x8 qf[DK / 32];
-  {
-    const unsigned short* qr = q + ((long)row * H + head) * DK + g * 8;
-#pragma unroll
-    for (int s = 0; s < DK / 32; ++s) {
-      s16x8 v = *reinterpret_cast<const s16x8*>(qr + s * 32);
-      if (!live) v = (s16x8)(short)0;
-      qf[s] = __builtin_bit_cast(bf16x8, v);
-    }
-  }
-  const float r1 = dist[head], r2 = dist[H + head];
-
-  float m = -1e30f, l = 0.f;
-  f32x4 acc[DV / 16];
-#pragma unroll
-  for (int i = 0; i < DV / 16; ++i) acc[i] = {0.f, 0.f, 0.f, 0.f};
-
-  for (int t = ts + wid; t < te; t += 4) {
-    long page[2];
-#pragma unroll
-    for (int h = 0; h < 2; ++h)
-      page[h] = (long)bt[min(t * 2 + h, last_page)] * G + kvh;
-    bf16x8 kf[2][DK / 32];
-    i32x2 vf[2][DV / 16];
-#pragma unroll
-    for (int h = 0; h < 2; ++h)
-#pragma unroll
-      for (int s = 0; s < DK / 32; ++s)
-        kf[h][s] = *reinterpret_cast<const bf16x8*>(
-            kpages + (page[h] * PBLK + i16) * DK + s * 32 + g * 8);
-#pragma unroll
-    for (int h = 0; h < 2; ++h)
-#pragma unroll
-      for (int b = 0; b < DV / 16; ++b)
-        vf[h][b] = *reinterpret_cast<const i32x2*>(
-            vpages + (page[h] * DV + b * 16 + i16) * PBLK + g * 4);
-    float p[2][4];
-    float pmax = -INFINITY;
-#pragma unroll
-    for (int h = 0; h < 2; ++h) {
-      f32x4 s = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int k = 0; k < DK / 32; ++k)
-        s = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[h][k], qf[k], s, 0, 0,
-                                                    0);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int key = t * 32 + h * 16 + g * 4 + r;
-        const float v = capped_score(s[r], c_in, c_out, r1, r2,
-                                     (float)(L - 1 - key));
-        p[h][r] = key >= lo && key < L ? v : -INFINITY;
-        pmax = fmaxf(pmax, p[h][r]);
-      }
-    }
-    pmax = fmaxf(pmax, __shfl_xor(pmax, 16, 64));
-    pmax = fmaxf(pmax, __shfl_xor(pmax, 32, 64));
-    if (!__all(pmax <= m)) {
-      const float mn = fmaxf(m, pmax);
-      const float alpha = __builtin_amdgcn_exp2f(m - mn);
-      m = mn;
-      l *= alpha;
-#pragma unroll
-      for (int i = 0; i < DV / 16; ++i)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) acc[i][r] *= alpha;
-    }
-    s16x8 pb;
-#pragma unroll
-    for (int h = 0; h < 2; ++h)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const float e = __builtin_amdgcn_exp2f(p[h][r] - m);
-        l += e;  // this lane's keys only; lanes are joined at the end
-        pb[h * 4 + r] = (short)f2bf(e);
-      }
-    const bf16x8 pf = __builtin_bit_cast(bf16x8, pb);
-#pragma unroll
-    for (int b = 0; b < DV / 16; ++b) {
-      i32x4 v;
-      v[0] = vf[0][b][0];
-      v[1] = vf[0][b][1];
-      v[2] = vf[1][b][0];
-      v[3] = vf[1][b][1];
-      acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-          __builtin_bit_cast(bf16x8, v), pf, acc[b], 0, 0, 0);
-    }
-  }
-  l += __shfl_xor(l, 16, 64);
-  l += __shfl_xor(l, 32, 64);
-
-  // join the four waves
-  float* wm = reinterpret_cast<float*>(smem);  // [4][16]
-  float* wl = wm + 64;                         // [4][16]
-  float* wo = wl + 64;                         // [4][16][OROW]
-  if (g == 0) {
-    wm[wid * 16 + i16] = m;
-    wl[wid * 16 + i16] = l;
-  }
-#pragma unroll
-  for (int b = 0; b < DV / 16; ++b)
-    *reinterpret_cast<f32x4*>(wo + (wid * 16 + i16) * OROW + b * 16 + g * 4) =
-        acc[b];
-  __syncthreads();
-  for (int i = threadIdx.x; i < nlive * (DV / 4); i += 256) {
-    const int hl = i / (DV / 4), c = i % (DV / 4) * 4;
-    float M = -1e30f, lsum = 0.f;
-#pragma unroll
-    for (int w = 0; w < 4; ++w) M = fmaxf(M, wm[w * 16 + hl]);
-    f32x4 o = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-    for (int w = 0; w < 4; ++w) {
-      const float a = __builtin_amdgcn_exp2f(wm[w * 16 + hl] - M);
-      lsum += a * wl[w * 16 + hl];
-      const f32x4 v =
-          *reinterpret_cast<const f32x4*>(wo + (w * 16 + hl) * OROW + c);
-#pragma unroll
-      for (int r = 0; r < 4; ++r) o[r] += a * v[r];
-    }
-    const int hd = kvh * GR + grp * 16 + hl;
-    const long rh = (long)row * H + hd;
-    if (NS == 1) {
-      const float inv = lsum > 0.f ? 1.f / lsum : 0.f;
-      const s16x4 gv = *reinterpret_cast<const s16x4*>(
-          gate + (long)row * ld_gate + (long)hd * DV + c);
-      s16x4 ov;
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        ov[r] = (short)f2bf(
-            o[r] * inv *
-            fast_rcp(1.f + fast_exp(-bf2f((unsigned short)gv[r]))));
-      *reinterpret_cast<s16x4*>(out + rh * DV + c) = ov;
-    } else {
-      *reinterpret_cast<f32x4*>(pacc + (rh * NS + split) * DV + c) = o;
-      if (c == 0) {
-        pml[(rh * NS + split) * 2] = M;
-        pml[(rh * NS + split) * 2 + 1] = lsum;
-      }
-    }
-  }
-}
-
-// one wave per (row, head): join NS partial results and gate
-__global__ void __launch_bounds__(256)
-chunk_combine_kernel(const float* __restrict__ pacc,
-                     const float* __restrict__ pml,
-                     const unsigned short* __restrict__ gate, int ld_gate,
-                     unsigned short* __restrict__ out, int RH, int H, int DV,
-                     int NS) {
-  const int lane = threadIdx.x & 63;
-  const long rh = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (rh >= RH) return;
-  float M = -1e30f;
-  for (int s = 0; s < NS; ++s) M = fmaxf(M, pml[(rh * NS + s) * 2]);
-  float l = 0.f;
-  for (int s = 0; s < NS; ++s)
-    l += pml[(rh * NS + s) * 2 + 1] *
-         __builtin_amdgcn_exp2f(pml[(rh * NS + s) * 2] - M);
-  const float inv = l > 0.f ? 1.f / l : 0.f;
-  for (int c = lane * 4; c < DV; c += 256) {
-    f32x4 o = {0.f, 0.f, 0.f, 0.f};
-    for (int s = 0; s < NS; ++s) {
-      const float a =
-          __builtin_amdgcn_exp2f(pml[(rh * NS + s) * 2] - M) * inv;
-      const f32x4 v =
-          *reinterpret_cast<const f32x4*>(pacc + (rh * NS + s) * DV + c);
-#pragma unroll
-      for (int i = 0; i < 4; ++i) o[i] += a * v[i];
-    }
-    const s16x4 gv = *reinterpret_cast<const s16x4*>(
-        gate + rh / H * ld_gate + rh % H * DV + c);
-    s16x4 ov;
-#pragma unroll
-    for (int i = 0; i < 4; ++i)
-      ov[i] = (short)f2bf(
-          o[i] * fast_rcp(1.f + fast_exp(-bf2f((unsigned short)gv[i]))));
-    *reinterpret_cast<s16x4*>(out + rh * DV + c) = ov;
-  }
-}
-
-extern "C" void launch_chunk_decode(
-    const void* q, const void* kpages, const void* vpages, const void* gate,
-    int ld_gate, const int* block_table, const int* row_seq, const int* ctx,
-    void* out, void* pacc, void* pml, int M, int H, int G, int DK, int DV,
-    int NS, int max_blocks, int chunk, float scale, float softcap,
-    const float* dist, hipStream_t stream) {
-  const int ng = (H / G + 15) / 16;
-  const float c_in = 2.f * scale / softcap * LOG2E, c_out = softcap * LOG2E;
-#define CD(KK, VV)                                                           \
-  hipLaunchKernelGGL(                                                        \
-      (chunk_decode_kernel<KK, VV>), dim3((long)M * G * ng * NS), dim3(256), \
-      (128 + 64 * (VV + 4)) * 4, stream, (const unsigned short*)q,           \
-      (const unsigned short*)kpages, (const unsigned short*)vpages,          \
-      (const unsigned short*)gate, ld_gate, block_table, row_seq, ctx,       \
-      (unsigned short*)out, (float*)pacc, (float*)pml, H, G, ng, NS,         \
-      max_blocks, chunk, c_in, c_out, dist)
-#define CD_V(KK)               \
-  do {                         \
-    if (DV == 64) CD(KK, 64);  \
-    else if (DV == 128) CD(KK, 128); \
-    else CD(KK, 256);          \
-  } while (0)
-  if (DK == 64) CD_V(64);
-  else if (DK == 128) CD_V(128);
-  else CD_V(256);
-#undef CD_V
-#undef CD
-  if (NS > 1)
-    hipLaunchKernelGGL(chunk_combine_kernel, dim3((M * H + 3) / 4), dim3(256),
-                       0, stream, (const float*)pacc, (const float*)pml,
-                       (const unsigned short*)gate, ld_gate,
-                       (unsigned short*)out, M * H, H, DV, NS);
+#undef APK_R
 }

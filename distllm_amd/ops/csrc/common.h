@@ -116,6 +116,11 @@ __device__ __forceinline__ float fast_gelu(float x) {
   const float k1 = 0.044715f;
   return 0.5f * x * (1.f + fast_tanh(k0 * (x + k1 * x * x * x)));
 }
+// the same on library functions
+__device__ __forceinline__ float gelu_exact(float x) {
+  return 0.5f * x *
+         (1.f + tanhf(0.7978845608028654f * (x + 0.044715f * x * x * x)));
+}
 __device__ __forceinline__ float gelu_erf(float x) {
   return 0.5f * x * (1.f + fast_erf(x * 0.70710678118654752f));
 }

@@ -17,6 +17,7 @@
 //  - SPLITK > 1 writes fp32 partial slabs; a tiny reduce kernel sums
 //    them with fused bias (separate launch: simple and graph-safe).
 #include "common.h"
+#include "gelu_rows.h"
 
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 
@@ -200,11 +201,34 @@ dg_reduce_glu_kernel(const float* __restrict__ slabs,
   }
 }
 
+// the same with gelu(.) * a part of a table's row
+__global__ void __launch_bounds__(256)
+dg_reduce_rows_kernel(const float* __restrict__ slabs,
+                      unsigned short* __restrict__ out, int M, int MP, int N,
+                      int splitk, const RowsArgs r) {
+  const long total = (long)M * N;
+  const long stride = (long)gridDim.x * blockDim.x;
+  for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
+       i += stride) {
+    const int row = (int)(i / N);
+    const int col = (int)(i % N);
+    float v = 0.f;
+    if (col < r.n) {
+      for (int s = 0; s < splitk; ++s)
+        v += slabs[((long)s * MP + row) * N + col];
+      v = fast_gelu(v) * bf2f(((const unsigned short*)r.table)
+                                  [r.tokens[row] * r.ld + r.col0 + col]);
+    }
+    out[i] = f2bf(v);
+  }
+}
+
 extern "C" void launch_decode_gemm(const void* X, const void* W,
                                    const void* bias, void* out, void* slabs,
                                    int M, int N, int K, int splitk, int act,
                                    float limit, float alpha, float shift,
                                    const float* act_nums,
+                                   const RowsArgs* rows,
                                    hipStream_t stream) {
   const int MP = M <= 128 ? 128 : 256;
   const int ncb = N / DG_BN;
@@ -230,6 +254,10 @@ extern "C" void launch_decode_gemm(const void* X, const void* W,
                      N, splitk, limit, alpha, shift)
     if (act == 1) DGR(1);
     else if (act == 2) DGR(2);
+    else if (act == 4)
+      hipLaunchKernelGGL(dg_reduce_rows_kernel, dim3(blocks), dim3(256), 0,
+                         stream, (const float*)slabs, (unsigned short*)out,
+                         M, MP, N, splitk, *rows);
     else if (act == 3)
       hipLaunchKernelGGL(dg_reduce_kernel<true>, dim3(blocks), dim3(256), 0,
                          stream, (const float*)slabs,

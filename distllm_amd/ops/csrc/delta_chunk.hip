@@ -12,22 +12,7 @@
 //                       columns
 //   delta_norm_kernel   gated output norm
 // All of it in fp32, the products on the fp32 MFMA.
-#include "common.h"
-
-#define CH 32        // rows of a chunk
-#define TROW 36      // padded LDS row of a chunk x chunk matrix
-
-extern __shared__ __attribute__((aligned(16))) char smem[];
-
-__device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
-}
-
-// Operands of the 16 x 16 x 4 product: lane group g = lane / 16 holds inner
-// index 4 j + g for step j as the instruction has it; here step r of a block
-// of 16 takes inner indices g * 4 + r instead, which lets a lane read both
-// operands as float4 and lets an accumulator (rows g * 4 + r) be the right
-// operand of the next product as it is.
+#include "delta_chunk.h"
 
 // ---- T and P: one wave per (chunk, key head) -------------------------------
 template <int DP>
@@ -115,20 +100,8 @@ delta_chunk_kernel(const float* __restrict__ qk, const float* __restrict__ gb,
       }
     }
     wave_sync();
-    // a lane solves for one column of the inverse
     float x[CH];
-#pragma unroll
-    for (int i = 0; i < CH; ++i) {
-      float v = i == j ? 1.f : 0.f;
-#pragma unroll
-      for (int s4 = 0; s4 < i; s4 += 4) {
-        const f32x4 a = *reinterpret_cast<const f32x4*>(A + i * TROW + s4);
-#pragma unroll
-        for (int e = 0; e < 4; ++e)
-          if (s4 + e < i) v -= a[e] * x[s4 + e];
-      }
-      x[i] = v;
-    }
+    inverse_column(A, j, x);
     if (lane < CH) {
       float* Tg = T + ((long)ch * H + head) * CH * CH + j;
 #pragma unroll
@@ -336,14 +309,15 @@ delta_carry_kernel(const float* __restrict__ qk,
   for (int k = 0; k < KT; ++k) *reinterpret_cast<f32x4*>(st + k * 16) = S[k];
 }
 
-// ---- output norm and gate; LV lanes share a head of a row -------------------
-template <int LV>
+// ---- output norm and gate, silu(gate) or sigmoid(gate) * out_scale; LV lanes
+// share a head of a row ---------------------------------------------------------
+template <int LV, bool SIGMOID>
 __global__ void __launch_bounds__(256)
 delta_norm_kernel(const float* __restrict__ o,
                   const unsigned short* __restrict__ gate, int ld_gate,
                   const float* __restrict__ o_norm,
-                  unsigned short* __restrict__ y, int M, int H, int vdim,
-                  float eps, int max_rows, const int* __restrict__ seg_rows,
+                  float out_scale, unsigned short* __restrict__ y, long ld_y,
+                  int M, int H, int vdim, float eps, int max_rows, const int* __restrict__ seg_rows,
                   const int* __restrict__ row_seq,
                   const int* __restrict__ ctx) {
   constexpr int VP = LV * 8;
@@ -361,10 +335,39 @@ delta_norm_kernel(const float* __restrict__ o,
   for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
 #pragma unroll
   for (int off = LV / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, 64);
-  const float inv = 1.f / sqrtf(ss / vdim + eps);
+  const float inv =
+      1.f / sqrtf(ss / vdim + eps) * (SIGMOID ? out_scale : 1.f);
 #pragma unroll
-  for (int i = 0; i < 8; ++i) x[i] *= inv * w[i] * silu(gt[i]);
-  store8(y + u * VP + sub * 8, x);
+  for (int i = 0; i < 8; ++i)
+    x[i] *= inv * w[i] *
+            (SIGMOID ? fast_rcp(1.f + fast_exp(-gt[i])) : silu(gt[i]));
+  store8(y + row * ld_y + head * VP + sub * 8, x);
+}
+
+// rows of y are ld_y apart; segments of more than max_rows rows only
+extern "C" void launch_delta_norm(const float* o, const void* gate,
+                                  int ld_gate, const float* o_norm,
+                                  float out_scale, void* y, long ld_y, int M,
+                                  int H, int vp, int vdim, float eps,
+                                  int max_rows, const int* seg_rows,
+                                  const int* row_seq, const int* ctx,
+                                  bool sigmoid, hipStream_t stream) {
+#define DN_G(L, S)                                                          \
+  hipLaunchKernelGGL((delta_norm_kernel<L, S>),                             \
+                     dim3(((long)M * H + 256 / L - 1) / (256 / L)),         \
+                     dim3(256), 0, stream, o, (const unsigned short*)gate,  \
+                     ld_gate, o_norm, out_scale, (unsigned short*)y, ld_y,  \
+                     M, H, vdim, eps, max_rows, seg_rows, row_seq, ctx)
+#define DN(L)                      \
+  do {                             \
+    if (sigmoid) DN_G(L, true);    \
+    else DN_G(L, false);           \
+  } while (0)
+  if (vp == 64) DN(8);
+  else if (vp == 128) DN(16);
+  else DN(32);
+#undef DN
+#undef DN_G
 }
 
 // T, P [nchunks, H, 32, 32], bsum [M, H], o [M, H * vp]: scratch. longs
@@ -407,14 +410,7 @@ extern "C" void launch_delta_chunks(
   else DY_N(256);
 #undef DY_N
 #undef DY
-#define DN(L)                                                               \
-  hipLaunchKernelGGL((delta_norm_kernel<L>),                                \
-                     dim3(((long)M * H + 256 / L - 1) / (256 / L)),         \
-                     dim3(256), 0, stream, o, (const unsigned short*)gate,  \
-                     ld_gate, o_norm, (unsigned short*)y, M, H, vdim, eps,  \
-                     max_rows, seg_rows, row_seq, ctx)
-  if (vp == 64) DN(8);
-  else if (vp == 128) DN(16);
-  else DN(32);
-#undef DN
+  launch_delta_norm(o, gate, ld_gate, o_norm, 1.f, y, (long)H * vp, M, H, vp,
+                    vdim, eps, max_rows, seg_rows, row_seq, ctx, false,
+                    stream);
 }

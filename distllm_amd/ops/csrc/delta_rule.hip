@@ -2,12 +2,14 @@
 //   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
 //
 // The fused projection ab of a row holds G query heads, G key heads (dp
-// numbers each), H value heads, H gate heads (vp each), then b and a of
-// every head. delta_prep runs the short convolutions and makes what enters
+// numbers each) and H value heads (vp each). Decays are one number per head,
+// g = exp(-exp(A) softplus(a + dt)) with the step sizes' b and the a of every
+// head side by side and an output gate silu(.), or (CHAN) one per head and
+// key channel, with an output gate sigmoid(.) times a constant. delta_prep runs the short convolutions and makes what enters
 // the recurrence, in fp32; a scan kernel runs the recurrence. A segment is
 // the consecutive rows of one sequence; a sequence that starts in the step
 // (ctx 1 in its first row) starts from zeros, whatever its slot holds.
-#include "common.h"
+#include "short_conv.h"
 
 extern __shared__ __attribute__((aligned(16))) char smem[];
 
@@ -21,31 +23,7 @@ __device__ __forceinline__ float act_silu(float z) {
 // A unit is a query, key or value head over a run of `rb` rows; LPH lanes of
 // eight channels each share it. The window of inputs stays in registers
 // from row to row. TAPS: 0 for any number, at the price of reading every
-// input of every row. shift: every segment has one row, and the unit renews
-// its channels of the convolution slot itself (else conv_state_kernel does).
-template <typename T>
-struct ConvArgs {
-  const T* ab;
-  int ld, M, C, taps, rb;
-  const float* w;
-  T* conv;
-  const int *seg_row0, *seg_slot, *row_seq, *ctx;
-  bool shift;
-};
-
-// input j rows before `row`, as fp32; zeros before the start
-template <typename T>
-__device__ __forceinline__ void conv_input(const ConvArgs<T>& a, int row,
-                                           int pos, int o, const T* slot,
-                                           int ch, int j, float* x) {
-#pragma unroll
-  for (int i = 0; i < 8; ++i) x[i] = 0.f;
-  if (pos < j) return;
-  load8<T>(o >= j ? a.ab + (long)(row - j) * a.ld + ch
-                  : slot + (long)(a.taps - 1 + o - j) * a.C,
-           x);
-}
-
+// input of every row.
 template <typename T, int LPH, int TAPS, bool QK>
 __device__ __forceinline__ void conv_unit(const ConvArgs<T>& a, int unit,
                                           int r0, int sub, int ch0, int G,
@@ -95,15 +73,7 @@ __device__ __forceinline__ void conv_unit(const ConvArgs<T>& a, int unit,
       }
     }
     before = seg;
-    if (a.shift && a.taps > 1) {
-      float t[8];
-      for (int j = 0; j < a.taps - 2; ++j) {
-        load8<T>(slot + (long)(j + 1) * a.C, t);
-        store8(slot + (long)j * a.C, t);
-      }
-      load8<T>(a.ab + (long)row * a.ld + ch, t);
-      store8(slot + (long)(a.taps - 2) * a.C, t);
-    }
+    if (a.shift && a.taps > 1) conv_shift(a, row, slot, ch);
 #pragma unroll
     for (int i = 0; i < 8; ++i) z[i] = act_silu<T>(z[i]);
     if (QK) {
@@ -123,13 +93,27 @@ __device__ __forceinline__ void conv_unit(const ConvArgs<T>& a, int unit,
   }
 }
 
+// What decays and step sizes come from.
+template <typename T>
+struct DecayArgs {
+  const T* ba;         // b of every head (CHAN false: then a), rows a.ld apart
+  const float* a_log;  // [H]
+  const float* dt;     // [H], CHAN: [H * dp]
+  const T* ag;         // CHAN: a [H * dp], rows ld_ag apart
+  int ld_ag;
+  const int* seg_rows;
+  int max_rows;        // CHAN: decays are for segments of up to this many
+};
+
 // workgroups: first those of query and key heads, then of value heads, then
-// one thread per (row, head) for decays and step sizes
-template <typename T, int LQ, int LV, int TAPS>
+// one thread per (row, head) for decays and step sizes -> gb [M, H, 2]: log
+// of the decay, step size. CHAN: one thread per (row, head, 8 channels) ->
+// gb [M, H]: step size, gc [M, H, dp]: decay.
+template <typename T, int LQ, int LV, int TAPS, bool CHAN>
 __global__ void __launch_bounds__(256)
-delta_prep_kernel(ConvArgs<T> a, int H, int G, const float* __restrict__ decay,
-                  float q_scale, float unit_eps, float* __restrict__ qk,
-                  T* __restrict__ v, float* __restrict__ gb, int wg_qk,
+delta_prep_kernel(ConvArgs<T> a, DecayArgs<T> d, int H, int G, float q_scale,
+                  float unit_eps, float* __restrict__ qk, T* __restrict__ v,
+                  float* __restrict__ gb, float* __restrict__ gc, int wg_qk,
                   int wg_v) {
   const int runs = (a.M + a.rb - 1) / a.rb;
   int wg = blockIdx.x;
@@ -153,47 +137,39 @@ delta_prep_kernel(ConvArgs<T> a, int H, int G, const float* __restrict__ decay,
     return;
   }
   wg -= wg_v;
-  const long i = (long)wg * 256 + threadIdx.x;
+  const long u = (long)wg * 256 + threadIdx.x;
+  const long i = CHAN ? u / LQ : u;
   if (i >= (long)a.M * H) return;
   const int row = (int)(i / H), h = (int)(i % H);
   if (a.ctx[row] <= 0) return;
-  const T* ba = a.ab + (long)row * a.ld + a.C + H * LV * 8;
-  // log of the decay, and the step size
-  gb[i * 2] =
-      -expf(decay[h]) * softplus_exact(to_f(ba[H + h]) + decay[H + h]);
-  gb[i * 2 + 1] = sigmoid_exact(to_f(ba[h]));
-}
-
-// last taps - 1 inputs of every segment -> its slot; a thread owns a channel
-template <typename T>
-__global__ void __launch_bounds__(256)
-conv_state_kernel(const T* __restrict__ ab, int ld, int C, int taps,
-                  T* __restrict__ conv, const int* __restrict__ seg_row0,
-                  const int* __restrict__ seg_rows,
-                  const int* __restrict__ seg_slot,
-                  const int* __restrict__ ctx) {
-  const int seg = blockIdx.y;
-  const int ch = blockIdx.x * 256 + threadIdx.x;
-  const int n = seg_rows[seg];
-  if (ch >= C || n == 0) return;
-  const int row0 = seg_row0[seg];
-  const bool fresh = ctx[row0] <= 1;
-  T* slot = conv + (long)seg_slot[seg] * (taps - 1) * C + ch;
-  for (int i = 0; i < taps - 1; ++i) {  // ascending: old entries move down
-    const int o = n - (taps - 1) + i;   // offset in the segment
-    T x = (T)0;
-    if (o >= 0) x = ab[(long)(row0 + o) * ld + ch];
-    else if (!fresh) x = slot[(long)(i + n) * C];
-    slot[(long)i * C] = x;
+  const T* ba = d.ba + (long)row * a.ld;
+  if constexpr (CHAN) {
+    const int c = (int)(u % LQ) * 8;
+    if (c == 0) gb[i] = sigmoid_exact(to_f(ba[h]));
+    if (d.seg_rows[a.row_seq[row]] > d.max_rows) return;
+    float x[8], t[8];
+    load8<T>(d.ag + (long)row * d.ld_ag + h * LQ * 8 + c, x);
+    load8<float>(d.dt + h * LQ * 8 + c, t);
+    const float rate = -expf(d.a_log[h]);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) x[k] = expf(rate * softplus_exact(x[k] + t[k]));
+    store8(gc + i * LQ * 8 + c, x);
+  } else {
+    gb[i * 2] =
+        -expf(d.a_log[h]) * softplus_exact(to_f(ba[H + h]) + d.dt[h]);
+    gb[i * 2 + 1] = sigmoid_exact(to_f(ba[h]));
   }
 }
 
+// chan: decays per channel from ag, a_log [H] and dt [H * dp]; else from the
+// columns behind H gates of vp numbers in ab, a_log [H] and dt [H]
 extern "C" void launch_delta_prep(
-    const void* ab, int ld, int M, int H, int G, int dp, int vp,
-    const float* conv_w, int taps, const float* decay, float q_scale,
-    float unit_eps, float* qk, void* v, float* gb, void* conv,
-    const int* seg_row0, const int* seg_rows, const int* seg_slot, int nseg,
-    int longest, const int* row_seq, const int* ctx, bool fp32,
+    const void* ab, int ld, const void* ag, int ld_ag, int M, int H, int G,
+    int dp, int vp, const float* conv_w, int taps, const float* a_log,
+    const float* dt, float q_scale, float unit_eps, float* qk, void* v,
+    float* gb, float* gc, void* conv, const int* seg_row0,
+    const int* seg_rows, const int* seg_slot, int nseg, int longest,
+    int max_rows, const int* row_seq, const int* ctx, bool chan, bool fp32,
     hipStream_t stream) {
   const bool shift = longest <= 1;
   const int rb = M >= 8192 ? 8 : M >= 2048 ? 4 : 1;
@@ -202,20 +178,28 @@ extern "C" void launch_delta_prep(
   const int lq = dp / 8, lv = vp / 8;
   const long wg_qk = (runs * 2 * G + 256 / lq - 1) / (256 / lq);
   const long wg_v = (runs * H + 256 / lv - 1) / (256 / lv);
-  const long wg_s = ((long)M * H + 255) / 256;
-#define DP(T, LQ, LV, TAPS)                                                  \
+  const long wg_s = ((long)M * H * (chan ? lq : 1) + 255) / 256;
+  const int ba_at = chan ? C : C + H * vp;
+#define DP_C(T, LQ, LV, TAPS, CH)                                            \
   do {                                                                       \
     const ConvArgs<T> a{(const T*)ab, ld, M, C, taps, rb, conv_w,            \
                         (T*)conv, seg_row0, seg_slot, row_seq, ctx, shift};  \
-    hipLaunchKernelGGL((delta_prep_kernel<T, LQ, LV, TAPS>),                 \
+    const DecayArgs<T> d{(const T*)ab + ba_at, a_log, dt, (const T*)ag,      \
+                         ld_ag, seg_rows, max_rows};                         \
+    hipLaunchKernelGGL((delta_prep_kernel<T, LQ, LV, TAPS, CH>),             \
                        dim3(wg_qk + wg_v + wg_s), dim3(256), 0, stream, a,   \
-                       H, G, decay, q_scale, unit_eps, qk, (T*)v, gb,        \
+                       d, H, G, q_scale, unit_eps, qk, (T*)v, gb, gc,        \
                        (int)wg_qk, (int)wg_v);                               \
     if (!shift && taps > 1)                                                  \
       hipLaunchKernelGGL((conv_state_kernel<T>),                             \
                          dim3((C + 255) / 256, nseg), dim3(256), 0, stream,  \
                          (const T*)ab, ld, C, taps, (T*)conv, seg_row0,      \
                          seg_rows, seg_slot, ctx);                           \
+  } while (0)
+#define DP(T, LQ, LV, TAPS)                 \
+  do {                                      \
+    if (chan) DP_C(T, LQ, LV, TAPS, true);  \
+    else DP_C(T, LQ, LV, TAPS, false);      \
   } while (0)
 #define DP_T(T, LQ, LV)              \
   do {                               \
@@ -240,21 +224,24 @@ extern "C" void launch_delta_prep(
 #undef DP_V
 #undef DP_T
 #undef DP
+#undef DP_C
 }
 
 // ---- recurrence, token by token ---------------------------------------------
 // One workgroup per (segment, head). LPC lanes share a value column, each
 // with 16 entries of the state's column in registers (float4 number i of
 // lane `part` is float4 i * LPC + part of the column); a thread has NCOL
-// columns. The output is normed over vdim and gated in place. Segments of
-// more than max_rows rows are left to the chunked form (delta_chunk.hip).
-template <typename T, int LPC, int NCOL>
+// columns. The output is normed over vdim and gated in place; rows of y are
+// ld_y apart. Segments of more than max_rows rows are left to the chunked
+// forms (delta_chunk.hip, delta_channel.hip).
+template <typename T, int LPC, int NCOL, bool CHAN>
 __global__ void __launch_bounds__(1024)
 delta_scan_kernel(const float* __restrict__ qk, const T* __restrict__ v,
-                  const float* __restrict__ gb, const T* __restrict__ gate,
-                  int ld_gate, const float* __restrict__ o_norm,
-                  float* __restrict__ state, T* __restrict__ y, int H, int G,
-                  int vp, int vdim, float eps,
+                  const float* __restrict__ gb, const float* __restrict__ gc,
+                  const T* __restrict__ gate, int ld_gate,
+                  const float* __restrict__ o_norm, float out_scale,
+                  float* __restrict__ state, T* __restrict__ y, long ld_y,
+                  int H, int G, int vp, int vdim, float eps,
                   const int* __restrict__ seg_row0,
                   const int* __restrict__ seg_rows,
                   const int* __restrict__ seg_slot,
@@ -304,8 +291,20 @@ delta_scan_kernel(const float* __restrict__ qk, const T* __restrict__ v,
         k[i * 4 + e] = b[e];
       }
     }
-    const float g = expf(gb[(row * H + head) * 2]);
-    const float beta = gb[(row * H + head) * 2 + 1];
+    float g[CHAN ? 16 : 1], beta;
+    if constexpr (CHAN) {
+      beta = gb[row * H + head];
+      const float* gr = gc + (row * H + head) * dp + part * 4;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const f32x4 a = *reinterpret_cast<const f32x4*>(gr + i * LPC * 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) g[i * 4 + e] = a[e];
+      }
+    } else {
+      g[0] = expf(gb[(row * H + head) * 2]);
+      beta = gb[(row * H + head) * 2 + 1];
+    }
     float o[NCOL];
     float ss = 0.f;
 #pragma unroll
@@ -313,7 +312,7 @@ delta_scan_kernel(const float* __restrict__ qk, const T* __restrict__ v,
       float dot = 0.f;
 #pragma unroll
       for (int e = 0; e < 16; ++e) {
-        S[c][e] *= g;
+        S[c][e] *= g[CHAN ? e : 0];
         dot += S[c][e] * k[e];
       }
 #pragma unroll
@@ -339,14 +338,15 @@ delta_scan_kernel(const float* __restrict__ qk, const T* __restrict__ v,
     __syncthreads();
     float tot = 0.f;
     for (int i = 0; i < nwave; ++i) tot += red[t & 1][i];
-    const float inv = 1.f / sqrtf(tot / vdim + eps);
+    const float inv = 1.f / sqrtf(tot / vdim + eps) * (CHAN ? out_scale : 1.f);
     if (part == 0) {
 #pragma unroll
       for (int c = 0; c < NCOL; ++c) {
         const int j = col0 + c * cstep;
         const float gt = to_f(gate[row * ld_gate + (long)head * vp + j]);
-        from_f(y + (row * H + head) * vp + j,
-               o[c] * inv * w[c] * act_silu<T>(gt));
+        from_f(y + row * ld_y + (long)head * vp + j,
+               o[c] * inv * w[c] *
+                   (CHAN ? sigmoid_exact(gt) : act_silu<T>(gt)));
       }
     }
   }
@@ -363,20 +363,26 @@ delta_scan_kernel(const float* __restrict__ qk, const T* __restrict__ v,
 }
 
 extern "C" void launch_delta_scan(
-    const float* qk, const void* v, const float* gb, const void* gate,
-    int ld_gate, const float* o_norm, float* state, void* y, int H, int G,
-    int dp, int vp, int vdim, float eps, const int* seg_row0,
-    const int* seg_rows, const int* seg_slot, int nseg, const int* ctx,
-    int max_rows, bool fp32, hipStream_t stream) {
+    const float* qk, const void* v, const float* gb, const float* gc,
+    const void* gate, int ld_gate, const float* o_norm, float out_scale,
+    float* state, void* y, long ld_y, int H, int G, int dp, int vp, int vdim,
+    float eps, const int* seg_row0, const int* seg_rows, const int* seg_slot,
+    int nseg, const int* ctx, int max_rows, bool chan, bool fp32,
+    hipStream_t stream) {
   const int lpc = dp / 16;
   const int threads = min(1024, lpc * vp);
   const int ncol = lpc * vp / threads;
-#define DS(T, L, N)                                                          \
-  hipLaunchKernelGGL((delta_scan_kernel<T, L, N>), dim3(nseg * H),           \
-                     dim3(threads), 0, stream, qk, (const T*)v, gb,          \
-                     (const T*)gate, ld_gate, o_norm, state, (T*)y, H, G,    \
-                     vp, vdim, eps, seg_row0, seg_rows, seg_slot, ctx,       \
-                     max_rows)
+#define DS_C(T, L, N, CH)                                                    \
+  hipLaunchKernelGGL((delta_scan_kernel<T, L, N, CH>), dim3(nseg * H),       \
+                     dim3(threads), 0, stream, qk, (const T*)v, gb, gc,      \
+                     (const T*)gate, ld_gate, o_norm, out_scale, state,      \
+                     (T*)y, ld_y, H, G, vp, vdim, eps, seg_row0, seg_rows,   \
+                     seg_slot, ctx, max_rows)
+#define DS(T, L, N)                  \
+  do {                               \
+    if (chan) DS_C(T, L, N, true);   \
+    else DS_C(T, L, N, false);       \
+  } while (0)
 #define DS_N(T)                                \
   do {                                         \
     if (lpc == 4) DS(T, 4, 1);                 \
@@ -390,4 +396,5 @@ extern "C" void launch_delta_scan(
   else DS_N(unsigned short);
 #undef DS_N
 #undef DS
+#undef DS_C
 }

@@ -28,3 +28,19 @@ static inline bool is_f32(const torch::Tensor& t) {
 static inline hipStream_t cur_stream() {
   return c10::hip::getCurrentHIPStream().stream();
 }
+
+#define CHECK_INTS(x)                          \
+  do {                                         \
+    CHECK_DEV(x); CHECK_CONT(x); CHECK_I32(x); \
+  } while (0)
+#define CHECK_FLOATS(x)                        \
+  do {                                         \
+    CHECK_DEV(x); CHECK_CONT(x); CHECK_F32(x); \
+  } while (0)
+
+// stride of the rows of a matrix whose columns are contiguous
+static inline int row_stride(const torch::Tensor& t) {
+  CHECK_DEV(t);
+  TORCH_CHECK(t.dim() == 2 && t.stride(1) == 1, "rows must be contiguous");
+  return (int)t.stride(0);
+}

@@ -1,12 +1,14 @@
-// Torch bindings of chunked attention over paged keys and values, the gated
-// delta rule, xIELU and routed experts.
+// Torch bindings of attention over paged keys and values and of the gated
+// delta rules.
 #include "ext_common.h"
 
 extern "C" {
+void launch_rotation_table(const int*, const double*, float, float*, int, int,
+                           hipStream_t);
 void launch_attn_prep(const void*, int, int, int, int, int, int, int,
                       const float*, const float*, float, void*, void*, void*,
-                      const int*, int, int, const int*, const int*, bool,
-                      hipStream_t);
+                      const int*, int, int, const int*, const int*, int,
+                      const float*, int, bool, hipStream_t);
 void launch_chunk_rows(const void*, const void*, const void*, const void*,
                        int, const int*, const int*, const int*, void*, int,
                        int, int, int, int, int, int, float, float,
@@ -19,49 +21,40 @@ void launch_chunk_flash(const void*, const void*, const void*, const void*,
                         int, void*, const int*, int, const int*, const int*,
                         int, int, int, int, int, int, float, float,
                         const float*, hipStream_t);
-void launch_delta_prep(const void*, int, int, int, int, int, int,
-                       const float*, int, const float*, float, float, float*,
-                       void*, float*, void*, const int*, const int*,
-                       const int*, int, int, const int*, const int*, bool,
-                       hipStream_t);
-void launch_delta_scan(const float*, const void*, const float*, const void*,
-                       int, const float*, float*, void*, int, int, int, int,
-                       int, float, const int*, const int*, const int*, int,
-                       const int*, int, bool, hipStream_t);
+void launch_sink_rows(const void*, const void*, const void*, const int*,
+                      const int*, const int*, void*, long, int, int, int, int,
+                      int, int, float, const float*, float, bool,
+                      hipStream_t);
+void launch_sink_decode(const void*, const void*, const void*, const int*,
+                        const int*, const int*, void*, long, void*, void*,
+                        int, int, int, int, int, int, int, float,
+                        const float*, float, hipStream_t);
+void launch_sink_flash(const void*, const void*, const void*, void*, long,
+                       const int*, int, const int*, const int*, int, int, int,
+                       int, int, float, const float*, float, hipStream_t);
+void launch_delta_prep(const void*, int, const void*, int, int, int, int, int,
+                       int, const float*, int, const float*, const float*,
+                       float, float, float*, void*, float*, float*, void*,
+                       const int*, const int*, const int*, int, int, int,
+                       const int*, const int*, bool, bool, hipStream_t);
+void launch_delta_scan(const float*, const void*, const float*, const float*,
+                       const void*, int, const float*, float, float*, void*,
+                       long, int, int, int, int, int, float, const int*,
+                       const int*, const int*, int, const int*, int, bool,
+                       bool, hipStream_t);
 void launch_delta_chunks(const float*, const void*, const float*, const void*,
                          int, const float*, float*, void*, float*, float*,
                          float*, float*, int, int, int, int, int, int, float,
                          const int*, int, const int*, int, int, const int*,
                          const int*, const int*, const int*, const int*,
                          hipStream_t);
-void launch_xielu(const void*, const float*, void*, long, bool, hipStream_t);
-bool route_covers(int);
-bool expert_gemm16_covers(int, int);
-void launch_select(const float*, const int*, int, int, int, int, int, int*,
-                   float*, hipStream_t);
-void launch_route(const void*, const void*, const int*, int, int, int, int,
-                  int, int, int*, float*, hipStream_t);
-void launch_expert_plan(const int*, int, int, int, int, int*, int*, int*,
-                        hipStream_t);
-void launch_expert_gemm(const void*, const void*, void*, const int*,
-                        const int*, const int*, int, int, int, int, int, bool,
-                        bool, hipStream_t);
-}
-
-#define CHECK_INTS(x)                       \
-  do {                                      \
-    CHECK_DEV(x); CHECK_CONT(x); CHECK_I32(x); \
-  } while (0)
-#define CHECK_FLOATS(x)                     \
-  do {                                      \
-    CHECK_DEV(x); CHECK_CONT(x); CHECK_F32(x); \
-  } while (0)
-
-// rows of a matrix whose columns are contiguous
-static int row_stride(const torch::Tensor& t) {
-  CHECK_DEV(t);
-  TORCH_CHECK(t.dim() == 2 && t.stride(1) == 1, "rows must be contiguous");
-  return (int)t.stride(0);
+void launch_channel_chunks(const float*, const void*, const float*,
+                           const void*, int, const float*, const float*,
+                           const float*, float, float*, void*, long, float*,
+                           float*, float*, float*, int, int, int, int, int,
+                           int, float, const int*, int, const int*, int, int,
+                           const int*, const int*, const int*, const int*,
+                           const int*, hipStream_t);
 }
 
 struct Pages {
@@ -127,6 +120,56 @@ torch::Tensor attn_prep(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
                      wq.data_ptr<float>(), wkp, (float)eps, q.data_ptr(), kp,
                      vpg, bt.data_ptr<int>(), bt.size(1), nblk,
                      row_seq.data_ptr<int>(), ctx.data_ptr<int>(),
+                     (int)((H + G) * dp), nullptr, 0, is_f32(ab),
+                     cur_stream());
+  return q;
+}
+
+torch::Tensor rotation_table(torch::Tensor ctx, torch::Tensor freq,
+                             double mult) {
+  CHECK_INTS(ctx);
+  CHECK_DEV(freq); CHECK_CONT(freq);
+  TORCH_CHECK(freq.scalar_type() == at::kDouble, "freq must be f64");
+  const long M = ctx.numel(), P = freq.numel();
+  auto t = torch::empty({M, P, 2}, ctx.options().dtype(at::kFloat));
+  if (M * P > 0)
+    launch_rotation_table(ctx.data_ptr<int>(), freq.data_ptr<double>(),
+                          (float)mult, t.data_ptr<float>(), M, P,
+                          cur_stream());
+  return t;
+}
+
+// ab: H query heads, G key heads of dp columns; keys as projected are the
+// values. table [M, pairs, 2] of rotation_table.
+torch::Tensor rotary_prep(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
+                          int64_t n, torch::Tensor wq, torch::Tensor wk,
+                          double eps, torch::Tensor table,
+                          torch::Tensor kpages, torch::Tensor vpages,
+                          torch::Tensor bt, torch::Tensor row_seq,
+                          torch::Tensor ctx) {
+  CHECK_T(ab); CHECK_SAME(ab, kpages);
+  const int M = ab.size(0), ld = row_stride(ab);
+  check_rows(bt, row_seq, ctx, M);
+  CHECK_FLOATS(wq); CHECK_FLOATS(wk); CHECK_FLOATS(table);
+  const Pages p = check_pages(kpages, vpages);
+  TORCH_CHECK(dp % 64 == 0 && ld % 8 == 0 && n > 0 && n <= dp &&
+                  wq.numel() == dp && wk.numel() == dp,
+              "head sizes");
+  TORCH_CHECK(p.G == G && p.DK == dp && p.DV == dp, "page sizes");
+  TORCH_CHECK(ab.size(1) >= (H + G) * dp, "projection columns");
+  TORCH_CHECK(table.dim() == 3 && table.size(0) == M && table.size(1) > 0 &&
+                  2 * table.size(1) <= n && table.size(2) == 2,
+              "rotation table");
+  TORCH_CHECK((uintptr_t)ab.data_ptr() % 16 == 0, "alignment");
+  TORCH_CHECK((long)M * (H + G) < (1L << 30), "too many rows");
+  auto q = torch::empty({M, H, dp}, ab.options());
+  if (M > 0)
+    launch_attn_prep(ab.data_ptr(), ld, M, H, G, dp, dp, (int)n,
+                     wq.data_ptr<float>(), wk.data_ptr<float>(), (float)eps,
+                     q.data_ptr(), kpages.data_ptr(), vpages.data_ptr(),
+                     bt.data_ptr<int>(), bt.size(1), p.nblk,
+                     row_seq.data_ptr<int>(), ctx.data_ptr<int>(),
+                     (int)(H * dp), table.data_ptr<float>(), table.size(1),
                      is_f32(ab), cur_stream());
   return q;
 }
@@ -160,6 +203,19 @@ static AttnArgs check_attn(const torch::Tensor& q, const torch::Tensor& k,
           (const char*)ab.data_ptr() + gate_at * ab.element_size()};
 }
 
+// Split each row's keys until the CUs are full (four workgroups each), as
+// long as a wave keeps two tiles. All sizes are known on the host, so a
+// captured graph stays valid as contexts grow.
+static long key_splits(long nsplit, long M, long H, long G, long chunk,
+                       long max_blocks) {
+  if (nsplit <= 0) {
+    const long wgs = M * G * ((H / G + 15) / 16);
+    const long tiles = std::min<long>(chunk, max_blocks * 16L) / 32 + 1;
+    nsplit = std::min<long>({(1024 + wgs - 1) / wgs, tiles / 8, 64L});
+  }
+  return std::max<long>(nsplit, 1);
+}
+
 static bool mfma_size(int d) { return d == 64 || d == 128 || d == 256; }
 
 void paged_attn_rows(torch::Tensor q, torch::Tensor k, torch::Tensor v,
@@ -183,17 +239,7 @@ void paged_attn_rows(torch::Tensor q, torch::Tensor k, torch::Tensor v,
                       cur_stream());
     return;
   }
-  // Split each row's keys until the CUs are full (four workgroups each), as
-  // long as a wave keeps two tiles. All sizes are known on the host, so a
-  // captured graph stays valid as contexts grow.
-  long NS = nsplit;
-  if (NS <= 0) {
-    const long wgs = (long)a.M * p.G * ((a.H / p.G + 15) / 16);
-    const long keys = std::min<long>(ch, bt.size(1) * 16L);
-    const long tiles = keys / 32 + 1;
-    NS = std::min<long>({(1024 + wgs - 1) / wgs, tiles / 8, 64L});
-  }
-  NS = std::max<long>(NS, 1);
+  const long NS = key_splits(nsplit, a.M, a.H, p.G, ch, bt.size(1));
   torch::Tensor pacc, pml;
   void *pa = nullptr, *pm = nullptr;
   if (NS > 1) {
@@ -233,6 +279,86 @@ void paged_attn_prompts(torch::Tensor q, torch::Tensor k, torch::Tensor v,
                      blocks.size(0), a.H, a.p.G, a.p.DK, a.p.DV,
                      (int)std::min<int64_t>(chunk, 1 << 30), (float)scale,
                      (float)softcap, dist.data_ptr<float>(), cur_stream());
+}
+
+struct SinkArgs {
+  Pages p;
+  int M, H;
+  long ld_out;
+};
+
+// out [M, H * DV], rows may be strided
+static SinkArgs check_sink(const torch::Tensor& q, const torch::Tensor& k,
+                           const torch::Tensor& v, const torch::Tensor& out,
+                           const torch::Tensor& sink) {
+  const Pages p = check_pages(k, v);
+  CHECK_DEV(q); CHECK_CONT(q); CHECK_SAME(q, k);
+  CHECK_SAME(out, k);
+  CHECK_FLOATS(sink);
+  TORCH_CHECK(q.dim() == 3, "rank");
+  const int M = q.size(0), H = q.size(1), ld = row_stride(out);
+  TORCH_CHECK(q.size(2) == p.DK && out.size(0) == M &&
+                  out.size(1) == (long)H * p.DV && H % p.G == 0 &&
+                  ld % 8 == 0 && (uintptr_t)out.data_ptr() % 16 == 0,
+              "attention shapes");
+  TORCH_CHECK(sink.numel() == H, "one sink per head");
+  return {p, M, H, ld};
+}
+
+void sink_attn_rows(torch::Tensor q, torch::Tensor k, torch::Tensor v,
+                    torch::Tensor out, torch::Tensor bt,
+                    torch::Tensor row_seq, torch::Tensor ctx, double scale,
+                    torch::Tensor sink, double out_scale, int64_t nsplit) {
+  const SinkArgs a = check_sink(q, k, v, out, sink);
+  check_rows(bt, row_seq, ctx, a.M);
+  if (a.M == 0) return;
+  const Pages& p = a.p;
+  if (is_f32(q) || !mfma_size(p.DK) || !mfma_size(p.DV)) {
+    TORCH_CHECK(p.DK <= 8192 && p.DV <= 4096, "head sizes");
+    launch_sink_rows(q.data_ptr(), k.data_ptr(), v.data_ptr(),
+                     bt.data_ptr<int>(), row_seq.data_ptr<int>(),
+                     ctx.data_ptr<int>(), out.data_ptr(), a.ld_out, a.M, a.H,
+                     p.G, p.DK, p.DV, bt.size(1), (float)scale,
+                     sink.data_ptr<float>(), (float)out_scale, is_f32(q),
+                     cur_stream());
+    return;
+  }
+  const long NS = key_splits(nsplit, a.M, a.H, p.G, 1L << 30, bt.size(1));
+  torch::Tensor pacc, pml;
+  void *pa = nullptr, *pm = nullptr;
+  if (NS > 1) {
+    auto f32 = q.options().dtype(at::kFloat);
+    pacc = torch::empty({(long)a.M * a.H * NS, p.DV}, f32);
+    pml = torch::empty({(long)a.M * a.H * NS, 2}, f32);
+    pa = pacc.data_ptr();
+    pm = pml.data_ptr();
+  }
+  launch_sink_decode(q.data_ptr(), k.data_ptr(), v.data_ptr(),
+                     bt.data_ptr<int>(), row_seq.data_ptr<int>(),
+                     ctx.data_ptr<int>(), out.data_ptr(), a.ld_out, pa, pm,
+                     a.M, a.H, p.G, p.DK, p.DV, (int)NS, bt.size(1),
+                     (float)scale, sink.data_ptr<float>(), (float)out_scale,
+                     cur_stream());
+}
+
+void sink_attn_prompts(torch::Tensor q, torch::Tensor k, torch::Tensor v,
+                       torch::Tensor out, torch::Tensor bt,
+                       torch::Tensor portions, torch::Tensor blocks,
+                       double scale, torch::Tensor sink, double out_scale) {
+  const SinkArgs a = check_sink(q, k, v, out, sink);
+  CHECK_BF16(q);
+  CHECK_INTS(bt); CHECK_INTS(portions); CHECK_INTS(blocks);
+  TORCH_CHECK(bt.dim() == 2 && portions.dim() == 2 && portions.size(1) == 4 &&
+                  blocks.dim() == 2 && blocks.size(1) == 2,
+              "portion maps");
+  TORCH_CHECK(mfma_size(a.p.DK) && mfma_size(a.p.DV),
+              "head sizes must be 64, 128 or 256");
+  if (blocks.size(0) == 0) return;
+  launch_sink_flash(q.data_ptr(), k.data_ptr(), v.data_ptr(), out.data_ptr(),
+                    a.ld_out, bt.data_ptr<int>(), bt.size(1),
+                    portions.data_ptr<int>(), blocks.data_ptr<int>(),
+                    blocks.size(0), a.H, a.p.G, a.p.DK, a.p.DV, (float)scale,
+                    sink.data_ptr<float>(), (float)out_scale, cur_stream());
 }
 
 // longs [P, 2]: segments of more than max_rows rows and their first chunk,
@@ -284,22 +410,24 @@ torch::Tensor gated_delta(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
   auto gb = torch::empty({M, H, 2}, f32);
   const void* gate =
       (const char*)ab.data_ptr() + C * (long)ab.element_size();
-  launch_delta_prep(ab.data_ptr(), ld, M, H, G, dp, vp,
+  launch_delta_prep(ab.data_ptr(), ld, nullptr, 0, M, H, G, dp, vp,
                     conv_w.data_ptr<float>(), taps, decay.data_ptr<float>(),
-                    1.f / sqrtf((float)dim), (float)unit_eps,
-                    qk.data_ptr<float>(), v.data_ptr(), gb.data_ptr<float>(),
-                    conv.data_ptr(), seg_row0.data_ptr<int>(),
-                    seg_rows.data_ptr<int>(), seg_slot.data_ptr<int>(), S,
-                    (int)longest, row_seq.data_ptr<int>(),
-                    ctx.data_ptr<int>(), is_f32(ab), cur_stream());
+                    decay.data_ptr<float>() + H, 1.f / sqrtf((float)dim),
+                    (float)unit_eps, qk.data_ptr<float>(), v.data_ptr(),
+                    gb.data_ptr<float>(), nullptr, conv.data_ptr(),
+                    seg_row0.data_ptr<int>(), seg_rows.data_ptr<int>(),
+                    seg_slot.data_ptr<int>(), S, (int)longest, INT_MAX,
+                    row_seq.data_ptr<int>(), ctx.data_ptr<int>(), false,
+                    is_f32(ab), cur_stream());
   const bool chunked = longs && !is_f32(ab) && longs->size(0) > 0;
   const int limit = chunked ? (int)max_rows : INT_MAX;
   launch_delta_scan(qk.data_ptr<float>(), v.data_ptr(), gb.data_ptr<float>(),
-                    gate, ld, o_norm.data_ptr<float>(), state.data_ptr<float>(),
-                    y.data_ptr(), H, G, dp, vp, vdim, (float)eps,
-                    seg_row0.data_ptr<int>(), seg_rows.data_ptr<int>(),
-                    seg_slot.data_ptr<int>(), S, ctx.data_ptr<int>(), limit,
-                    is_f32(ab), cur_stream());
+                    nullptr, gate, ld, o_norm.data_ptr<float>(), 1.f,
+                    state.data_ptr<float>(), y.data_ptr(), H * vp, H, G, dp,
+                    vp, vdim, (float)eps, seg_row0.data_ptr<int>(),
+                    seg_rows.data_ptr<int>(), seg_slot.data_ptr<int>(), S,
+                    ctx.data_ptr<int>(), limit, false, is_f32(ab),
+                    cur_stream());
   if (chunked) {
     TORCH_CHECK(chunks.has_value(), "chunks");
     CHECK_INTS(longs.value()); CHECK_INTS(chunks.value());
@@ -324,106 +452,118 @@ torch::Tensor gated_delta(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
   return y;
 }
 
-torch::Tensor xielu(torch::Tensor z, torch::Tensor act) {
-  CHECK_DEV(z); CHECK_CONT(z); CHECK_T(z);
-  CHECK_FLOATS(act);
-  TORCH_CHECK(act.numel() == 2 && z.numel() % 8 == 0, "xielu sizes");
-  auto out = torch::empty_like(z);
-  if (z.numel() > 0)
-    launch_xielu(z.data_ptr(), act.data_ptr<float>(), out.data_ptr(),
-                 z.numel(), is_f32(z), cur_stream());
-  return out;
-}
-
-static void check_route(int64_t E, int64_t top, int64_t groups,
-                        int64_t keep) {
-  TORCH_CHECK(E > 0 && E <= 1024, "1 to 1024 experts");
-  TORCH_CHECK(groups > 0 && E % groups == 0 && keep > 0 && keep <= groups &&
-                  top > 0 && top <= E / groups * keep,
-              "experts, groups and choices");
-}
-
-// h: bf16 rows with the router's weights, or fp32 logits (W absent)
-std::tuple<torch::Tensor, torch::Tensor> route(
-    torch::Tensor h, c10::optional<torch::Tensor> W, torch::Tensor ctx,
-    int64_t top, int64_t groups, int64_t keep) {
-  CHECK_DEV(h); CHECK_CONT(h);
-  CHECK_INTS(ctx);
-  const int M = h.size(0);
-  const int E = W ? W->size(0) : h.size(1);
-  check_route(E, top, groups, keep);
-  TORCH_CHECK(h.dim() == 2 && ctx.numel() == M, "one ctx entry per row");
-  auto ids = torch::empty({M, top}, h.options().dtype(at::kInt));
-  auto w = torch::empty({M, top}, h.options().dtype(at::kFloat));
-  if (M == 0) return {ids, w};
-  if (W) {
-    CHECK_BF16(h);
-    CHECK_DEV(W.value()); CHECK_CONT(W.value()); CHECK_BF16(W.value());
-    const int K = h.size(1);
-    TORCH_CHECK(W->size(1) == K && K % 32 == 0 && route_covers(E),
-                "router shape");
-    launch_route(h.data_ptr(), W->data_ptr(), ctx.data_ptr<int>(), M, E, K,
-                 groups, keep, top, ids.data_ptr<int>(),
-                 w.data_ptr<float>(), cur_stream());
-  } else {
-    CHECK_F32(h);
-    launch_select(h.data_ptr<float>(), ctx.data_ptr<int>(), M, E, groups,
-                  keep, top, ids.data_ptr<int>(), w.data_ptr<float>(),
-                  cur_stream());
-  }
-  return {ids, w};
-}
-
-torch::Tensor experts(torch::Tensor h, torch::Tensor ids, torch::Tensor wgup,
-                      torch::Tensor wdown) {
-  CHECK_DEV(h); CHECK_CONT(h); CHECK_T(h);
-  CHECK_INTS(ids);
-  CHECK_DEV(wgup); CHECK_CONT(wgup); CHECK_SAME(wgup, h);
-  CHECK_DEV(wdown); CHECK_CONT(wdown); CHECK_SAME(wdown, h);
-  const int M = h.size(0), K = h.size(1), top = ids.size(1);
-  const int E = wgup.size(0), F = wdown.size(2);
-  TORCH_CHECK(ids.size(0) == M && wgup.dim() == 3 && wdown.dim() == 3 &&
-                  wgup.size(1) == 2L * F && wgup.size(2) == K &&
-                  wdown.size(0) == E && wdown.size(1) == K,
-              "expert shapes");
-  TORCH_CHECK(K % 64 == 0 && F % 64 == 0 && E <= 1024,
-              "sizes % 64, at most 1024 experts");
-  const long A = (long)M * top;
-  TORCH_CHECK(A < (1L << 31), "too many rows");
-  auto y = torch::empty({A, K}, h.options());
-  if (A == 0) return y;
-  // rows of a tile: twice what an expert gets on average, large tiles from
-  // about 48 rows on
-  const bool f32 = is_f32(h);
-  const long mean = (A + E - 1) / E;
-  int TM = f32 || mean <= 8 ? 16 : mean <= 16 ? 32 : mean <= 48 ? 64 : 128;
-  if (!f32 && mean >= 512 && expert_gemm16_covers(2 * F, K) &&
-      expert_gemm16_covers(K, F))
-    TM = 256;
-  const int max_tiles = (int)std::min<long>(A, A / TM + E);
-  auto i32 = ids.options();
-  auto plan = torch::empty({A + 4L * max_tiles + 1}, i32);
-  int* perm = plan.data_ptr<int>();
-  int* tiles = perm + A;
-  int* ntiles = tiles + 4L * max_tiles;
-  launch_expert_plan(ids.data_ptr<int>(), (int)A, E, TM, max_tiles, perm,
-                     tiles, ntiles, cur_stream());
-  auto inter = torch::empty({A, F}, h.options());
-  launch_expert_gemm(h.data_ptr(), wgup.data_ptr(), inter.data_ptr(), perm,
-                     tiles, ntiles, max_tiles, 2 * F, K, top, TM, true, f32,
-                     cur_stream());
-  launch_expert_gemm(inter.data_ptr(), wdown.data_ptr(), y.data_ptr(), perm,
-                     tiles, ntiles, max_tiles, K, F, top, TM, false, f32,
-                     cur_stream());
-  return y;
+// ab: queries, keys, values and b of every head; ag: decays [H * dp] and
+// output gates [H * vp]; out [M, H * vp], rows may be strided. longs and
+// chunks as for gated_delta.
+void channel_delta(torch::Tensor ab, torch::Tensor ag, int64_t H, int64_t G,
+                   int64_t dp, int64_t vp, int64_t dim, int64_t vdim,
+                   torch::Tensor conv_w, torch::Tensor a_log,
+                   torch::Tensor dt_bias, torch::Tensor o_norm,
+                   double unit_eps, double eps, double out_scale,
+                   torch::Tensor state, torch::Tensor conv,
+                   torch::Tensor seg_row0, torch::Tensor seg_rows,
+                   torch::Tensor seg_slot, int64_t longest,
+                   torch::Tensor row_seq, torch::Tensor ctx,
+                   c10::optional<torch::Tensor> longs,
+                   c10::optional<torch::Tensor> chunks, int64_t max_rows,
+                   torch::Tensor out) {
+  CHECK_T(ab); CHECK_SAME(ag, ab); CHECK_SAME(out, ab);
+  const int M = ab.size(0), ld = row_stride(ab), ld_ag = row_stride(ag);
+  const int ld_y = row_stride(out);
+  auto size_ok = [](int64_t d) { return d == 64 || d == 128 || d == 256; };
+  TORCH_CHECK(size_ok(dp) && size_ok(vp), "head sizes must be 64, 128, 256");
+  TORCH_CHECK(dim > 0 && dim <= dp && vdim > 0 && vdim <= vp && G > 0 &&
+                  H % G == 0,
+              "head counts");
+  const long C = 2 * G * dp + H * vp;
+  auto aligned = [](const torch::Tensor& t) {
+    return (uintptr_t)t.data_ptr() % 16 == 0 && t.stride(0) % 8 == 0;
+  };
+  TORCH_CHECK(ab.size(1) >= C + H && ag.size(0) == M &&
+                  ag.size(1) == H * (dp + vp) && out.size(0) == M &&
+                  out.size(1) == H * vp && aligned(ab) && aligned(ag) &&
+                  aligned(out),
+              "projection columns");
+  CHECK_FLOATS(conv_w); CHECK_FLOATS(a_log); CHECK_FLOATS(dt_bias);
+  CHECK_FLOATS(o_norm); CHECK_FLOATS(state);
+  CHECK_DEV(conv); CHECK_CONT(conv); CHECK_SAME(conv, ab);
+  const int taps = conv_w.size(0);
+  TORCH_CHECK(conv_w.dim() == 2 && conv_w.size(1) == C && taps >= 1,
+              "convolution weights");
+  TORCH_CHECK(a_log.numel() == H && dt_bias.numel() == H * dp &&
+                  o_norm.numel() == vp,
+              "weights");
+  TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == vp &&
+                  state.size(3) == dp,
+              "state must be [slots, heads, vdim, dim]");
+  TORCH_CHECK(conv.dim() == 3 && conv.size(0) == state.size(0) &&
+                  conv.size(1) == taps - 1 && conv.size(2) == C,
+              "conv state must be [slots, taps - 1, channels]");
+  CHECK_INTS(seg_row0); CHECK_INTS(seg_rows); CHECK_INTS(seg_slot);
+  CHECK_INTS(row_seq); CHECK_INTS(ctx);
+  const int S = seg_row0.numel();
+  TORCH_CHECK(seg_rows.numel() == S && seg_slot.numel() == S &&
+                  row_seq.numel() == M && ctx.numel() == M,
+              "segments");
+  if (M == 0 || S == 0) return;
+  const bool chunked = longs && !is_f32(ab) && longs->size(0) > 0;
+  const int limit = chunked ? (int)max_rows : INT_MAX;
+  auto f32 = ab.options().dtype(at::kFloat);
+  auto qk = torch::empty({M, 2 * G, dp}, f32);
+  auto v = torch::empty({M, H * vp}, ab.options());
+  auto beta = torch::empty({M, H}, f32);
+  // decays of short segments, sums of logarithms in chunks of long ones
+  auto gc = torch::empty({M, H, dp}, f32);
+  const void* gate =
+      (const char*)ag.data_ptr() + H * dp * (long)ag.element_size();
+  launch_delta_prep(ab.data_ptr(), ld, ag.data_ptr(), ld_ag, M, H, G, dp, vp,
+                    conv_w.data_ptr<float>(), taps, a_log.data_ptr<float>(),
+                    dt_bias.data_ptr<float>(), 1.f / sqrtf((float)dim),
+                    (float)unit_eps, qk.data_ptr<float>(), v.data_ptr(),
+                    beta.data_ptr<float>(), gc.data_ptr<float>(),
+                    conv.data_ptr(), seg_row0.data_ptr<int>(),
+                    seg_rows.data_ptr<int>(), seg_slot.data_ptr<int>(), S,
+                    (int)longest, limit, row_seq.data_ptr<int>(),
+                    ctx.data_ptr<int>(), true, is_f32(ab), cur_stream());
+  launch_delta_scan(qk.data_ptr<float>(), v.data_ptr(),
+                    beta.data_ptr<float>(), gc.data_ptr<float>(), gate, ld_ag,
+                    o_norm.data_ptr<float>(), (float)out_scale,
+                    state.data_ptr<float>(), out.data_ptr(), ld_y, H, G, dp,
+                    vp, vdim, (float)eps, seg_row0.data_ptr<int>(),
+                    seg_rows.data_ptr<int>(), seg_slot.data_ptr<int>(), S,
+                    ctx.data_ptr<int>(), limit, true, is_f32(ab),
+                    cur_stream());
+  if (!chunked) return;
+  TORCH_CHECK(chunks.has_value(), "chunks");
+  CHECK_INTS(longs.value()); CHECK_INTS(chunks.value());
+  TORCH_CHECK(longs->dim() == 2 && longs->size(1) == 2 &&
+                  chunks->dim() == 2 && chunks->size(1) == 2 &&
+                  chunks->size(0) >= longs->size(0),
+              "chunk maps");
+  const int N = chunks->size(0);
+  auto tp = torch::empty({2, N, H, 32 * 32}, f32);
+  auto o = torch::empty({M, H * vp}, f32);
+  launch_channel_chunks(
+      qk.data_ptr<float>(), v.data_ptr(), beta.data_ptr<float>(),
+      ag.data_ptr(), ld_ag, a_log.data_ptr<float>(),
+      dt_bias.data_ptr<float>(), o_norm.data_ptr<float>(), (float)out_scale,
+      state.data_ptr<float>(), out.data_ptr(), ld_y, tp.data_ptr<float>(),
+      tp.data_ptr<float>() + tp.numel() / 2, gc.data_ptr<float>(),
+      o.data_ptr<float>(), M, H, G, dp, vp, vdim, (float)eps,
+      longs->data_ptr<int>(), longs->size(0), chunks->data_ptr<int>(), N,
+      limit, seg_row0.data_ptr<int>(), seg_rows.data_ptr<int>(),
+      seg_slot.data_ptr<int>(), row_seq.data_ptr<int>(),
+      ctx.data_ptr<int>(), cur_stream());
 }
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("attn_prep", &attn_prep);
   m.def("paged_attn_rows", &paged_attn_rows);
   m.def("paged_attn_prompts", &paged_attn_prompts);
+  m.def("rotation_table", &rotation_table);
+  m.def("rotary_prep", &rotary_prep);
+  m.def("sink_attn_rows", &sink_attn_rows);
+  m.def("sink_attn_prompts", &sink_attn_prompts);
   m.def("gated_delta", &gated_delta);
-  m.def("xielu", &xielu);
-  m.def("route", &route);
-  m.def("experts", &experts);
+  m.def("channel_delta", &channel_delta);
 }

@@ -1,5 +1,5 @@
 // Torch bindings of the latent-attention decoder kernels: latent
-// preparation and attention, the clamped gated unit.
+// preparation and attention.
 #include "ext_common.h"
 
 extern "C" {
@@ -22,8 +22,6 @@ void launch_latent_decode(const void*, const void*, const int*, const int*,
 void launch_attn_window(const void*, const void*, const void*, void*,
                         const int*, const int*, const int*, const int*, int,
                         int, int, int, int, long, int, float, hipStream_t);
-void launch_clamped_glu(const void*, void*, long, int, float, float, float,
-                        bool, hipStream_t);
 }
 
 static void check_pages(const torch::Tensor& cache, const torch::Tensor& bt,
@@ -190,19 +188,6 @@ void attn_window(torch::Tensor q, torch::Tensor kv, torch::Tensor out,
         cur_stream());
 }
 
-torch::Tensor clamped_glu(torch::Tensor gu, double limit, double alpha,
-                          double shift) {
-  CHECK_DEV(gu); CHECK_CONT(gu); CHECK_T(gu);
-  const long R = gu.size(0);
-  const int F = gu.size(1) / 2;
-  TORCH_CHECK(gu.dim() == 2 && F % 8 == 0, "halves must be % 8");
-  auto out = torch::empty({R, F}, gu.options());
-  if (R > 0)
-    launch_clamped_glu(gu.data_ptr(), out.data_ptr(), R, F, (float)limit,
-                       (float)alpha, (float)shift, is_f32(gu), cur_stream());
-  return out;
-}
-
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("latent_prep", &latent_prep);
   m.def("latent_gather", &latent_gather);
@@ -211,5 +196,4 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
         py::arg("block_table"), py::arg("row_seq"), py::arg("ctx"),
         py::arg("window"), py::arg("scale"), py::arg("nsplit") = 0);
   m.def("attn_window", &attn_window);
-  m.def("clamped_glu", &clamped_glu);
 }

@@ -11,6 +11,11 @@ void launch_layer_norm_add(const void*, const float*, int, float*,
                            const float*, const float*, const float*,
                            const float*, void*, int, int, int, float, bool,
                            hipStream_t);
+void launch_residual_step(const void*, const void*, float*, const float*,
+                          const float*, int, float, const long*, float,
+                          const float*, const float*, const float*,
+                          const float*, bool, void*, int, int, bool,
+                          hipStream_t);
 }
 
 // y == embedding table when tokens are given
@@ -108,8 +113,53 @@ torch::Tensor layer_norm_add(torch::Tensor y, torch::Tensor x,
   return h;
 }
 
+typedef c10::optional<torch::Tensor> Maybe;
+
+void residual_step(torch::Tensor x, Maybe y, Maybe bias, Maybe w_rms,
+                   int64_t n, double eps, Maybe tokens, Maybe table,
+                   double scale, Maybe vec, Maybe w, Maybe b, Maybe alpha,
+                   bool fresh, torch::Tensor h) {
+  CHECK_DEV(x); CHECK_CONT(x); CHECK_F32(x);
+  CHECK_DEV(h); CHECK_CONT(h); CHECK_T(h);
+  TORCH_CHECK(x.dim() == 2 && h.sizes() == x.sizes(), "row sizes");
+  const int M = x.size(0), W = x.size(1);
+  TORCH_CHECK(W % 8 == 0 && W <= 16384 && n > 0 && n <= W,
+              "width must be a multiple of 8, at most 16384");
+  const void *yp = nullptr, *tab = nullptr;
+  const long* tok = nullptr;
+  if (y) {
+    CHECK_DEV(y.value()); CHECK_CONT(y.value()); CHECK_SAME(y.value(), h);
+    TORCH_CHECK(y->sizes() == x.sizes(), "y rows");
+    yp = y->data_ptr();
+  }
+  TORCH_CHECK(y.has_value() || (!bias && !w_rms), "bias or norm without y");
+  if (tokens) {
+    TORCH_CHECK(table.has_value(), "tokens without a table");
+    CHECK_DEV(tokens.value()); CHECK_CONT(tokens.value());
+    CHECK_DEV(table.value()); CHECK_CONT(table.value());
+    CHECK_SAME(table.value(), h);
+    TORCH_CHECK(tokens->scalar_type() == at::kLong && tokens->numel() == M &&
+                    table->dim() == 2 && table->size(1) == W,
+                "tokens (int64, one per row) and table");
+    tok = (const long*)tokens->data_ptr<int64_t>();
+    tab = table->data_ptr();
+  }
+  auto opt = [&](const Maybe& t) {
+    return t ? norm_vec(*t, W) : (const float*)nullptr;
+  };
+  TORCH_CHECK(w.has_value() == b.has_value() &&
+                  w.has_value() == alpha.has_value(),
+              "weight, bias and alpha");
+  if (M > 0)
+    launch_residual_step(yp, tab, x.data_ptr<float>(), opt(bias), opt(w_rms),
+                         (int)n, (float)eps, tok, (float)scale, opt(vec),
+                         opt(w), opt(b), alpha ? norm_vec(*alpha, 1) : nullptr,
+                         fresh, h.data_ptr(), M, W, is_f32(h), cur_stream());
+}
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("sandwich_norm", &sandwich_norm);
   m.def("embed_positions", &embed_positions);
   m.def("layer_norm_add", &layer_norm_add);
+  m.def("residual_step", &residual_step);
 }

@@ -7,6 +7,9 @@
 //   embed_positions: x = E[token] + P[pos];   h = x
 //   layer_norm_add:  x += ln(y) * w + b;      h = x, or ln(x) * wf + bf
 // where y may be a weighted sum of several rows (routed experts).
+// Pre-norm streams with an elementwise activation in the norm's place:
+//   residual_step:   x += y + bias, or x += rms(y) * w;  x += scale E[token];
+//                    x += vec;  h = x, or tanh(alpha x) * w + b
 //
 // One launch per boundary: the sublayer output y is normed and added and
 // the next sublayer's input is produced while the row is still in
@@ -290,4 +293,133 @@ extern "C" void launch_layer_norm_add(const void* y, const float* mix,
   else LN_N(unsigned short);
 #undef LN_N
 #undef LN
+}
+
+// tanh to a relative error of about 1e-6, also near 0
+__device__ __forceinline__ float tanh_near(float u) {
+  const float s = u * u;
+  const float p =
+      u + u * s *
+              (-0.33333333f +
+               s * (0.13333333f + s * (-0.05396825f + s * 0.02186949f)));
+  return fabsf(u) < 0.3f ? p : fast_tanh(u);
+}
+
+struct ResidualArgs {
+  const float* bias;
+  const float* w_rms;   // null: y is added as it is
+  int n;                // columns of the rms statistics
+  float eps;
+  const long* tokens;   // null: no table row
+  float scale;
+  const float* vec;
+  const float *w, *b, *alpha;  // w null: h = x
+  bool fresh, store;    // x starts from zeros; x changes
+};
+
+template <typename T, int NC, int TPR>
+__global__ void __launch_bounds__(256)
+residual_step_kernel(const T* __restrict__ y, const T* __restrict__ table,
+                     float* __restrict__ x, const ResidualArgs a,
+                     T* __restrict__ h, int M, int W) {
+  __shared__ float scratch[4];
+  const int sub = threadIdx.x % TPR;
+  const int row = blockIdx.x * (256 / TPR) + threadIdx.x / TPR;
+  if (row >= M) return;  // whole waves; whole blocks when TPR == 256
+  float* xr = x + (long)row * W;
+
+  float v[NC][8];
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = (sub + k * TPR) * 8;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[k][i] = 0.f;
+    if (y != nullptr && c < W) load8<T>(y + (long)row * W + c, v[k]);
+  }
+  float inv = 1.f;
+  if (a.w_rms != nullptr) {
+    float ss = 0.f;
+#pragma unroll
+    for (int k = 0; k < NC; ++k)
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss += v[k][i] * v[k][i];
+    inv = 1.f / sqrtf(row_sum<TPR>(ss, scratch) / a.n + a.eps);
+  }
+  const T* er =
+      a.tokens != nullptr ? table + a.tokens[row] * (long)W : nullptr;
+  const float alpha = a.w != nullptr ? *a.alpha : 0.f;
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = (sub + k * TPR) * 8;
+    if (c >= W) continue;
+    float t[8];
+    if (a.w_rms != nullptr) {
+      load8<float>(a.w_rms + c, t);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] *= inv * t[i];
+    }
+    if (a.bias != nullptr) {
+      load8<float>(a.bias + c, t);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] += t[i];
+    }
+    if (!a.fresh) {
+      load8<float>(xr + c, t);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] += t[i];
+    }
+    if (er != nullptr) {
+      load8<T>(er + c, t);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] += t[i] * a.scale;
+    }
+    if (a.vec != nullptr) {
+      load8<float>(a.vec + c, t);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] += t[i];
+    }
+    if (a.store) store8(xr + c, v[k]);
+    if (a.w != nullptr) {
+      float w[8];
+      load8<float>(a.w + c, w);
+      load8<float>(a.b + c, t);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        const float u = alpha * v[k][i];
+        v[k][i] = (sizeof(T) == 2 ? tanh_near(u) : tanhf(u)) * w[i] + t[i];
+      }
+    }
+    store8(h + (long)row * W + c, v[k]);
+  }
+}
+
+extern "C" void launch_residual_step(
+    const void* y, const void* table, float* x, const float* bias,
+    const float* w_rms, int n, float eps, const long* tokens, float scale,
+    const float* vec, const float* w, const float* b, const float* alpha,
+    bool fresh, void* h, int M, int W, bool fp32, hipStream_t stream) {
+  const ResidualArgs a{bias, w_rms, n, eps, tokens, scale, vec, w, b, alpha,
+                       fresh,
+                       y != nullptr || tokens != nullptr || vec != nullptr ||
+                           fresh};
+  const int tpr = W <= 1024 ? 64 : 256;
+  const int rows = 256 / tpr;
+  const dim3 grid((M + rows - 1) / rows);
+  const int nc = (W / 8 + tpr - 1) / tpr;
+#define RS(T, NC, TPR)                                                      \
+  hipLaunchKernelGGL((residual_step_kernel<T, NC, TPR>), grid, dim3(256), 0, \
+                     stream, (const T*)y, (const T*)table, x, a, (T*)h, M, W)
+#define RS_N(T)                            \
+  do {                                     \
+    if (tpr == 64 && nc == 1) RS(T, 1, 64); \
+    else if (tpr == 64) RS(T, 2, 64);      \
+    else if (nc == 1) RS(T, 1, 256);       \
+    else if (nc == 2) RS(T, 2, 256);       \
+    else if (nc <= 4) RS(T, 4, 256);       \
+    else RS(T, 8, 256);                    \
+  } while (0)
+  if (fp32) RS_N(float);
+  else RS_N(unsigned short);
+#undef RS_N
+#undef RS
 }

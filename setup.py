@@ -28,7 +28,8 @@ from torch.utils.cpp_extension import BuildExtension, CUDAExtension
 CSRC = Path(__file__).parent / "distllm_amd" / "ops" / "csrc"
 GROUPS = {
     "_hip_gemm": ["ext_gemm.cpp", "blt_gemm.cpp", "gemm.hip", "gemm8.hip",
-                  "gemm16.hip", "decode_gemm.hip", "clamped_glu.hip"],
+                  "gemm16.hip", "decode_gemm.hip", "clamped_glu.hip",
+                  "gelu_rows.hip"],
     "_hip_latent": ["ext_latent.cpp", "latent_attention.hip",
                     "latent_decode.hip", "window_attention.hip"],
     "_hip_residual": ["ext_residual.cpp", "residual_norms.hip"],
