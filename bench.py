@@ -41,7 +41,7 @@ def main() -> None:
                          "write (tokenizer + staging included); "
                          "decoders = prefill and decode of Kanotar "
                          "and Bufulorn layers beside llama layers of equal "
-                         "size")
+                         "size, and of Tebasun beside Bufulorn layers")
     ap.add_argument("--docs-per-file", type=int, default=128)
     ap.add_argument("--pooler", type=str, default="mean",
                     choices=["mean", "last_token"])
@@ -247,15 +247,15 @@ def bench_generate(args) -> None:
 
 def bench_decoders(args) -> None:
     """Kanotar and Bufulorn layers beside llama layers of the same width,
-    heads and (active) feed-forward weights, through the same engine:
-    tokens/s of prefilling a batch of prompts and of decoding at a given
-    context, both models in turn. Random weights, synthetic tokens, one
-    GPU."""
+    heads and (active) feed-forward weights, and Tebasun layers beside
+    Bufulorn layers, through the same engine: tokens/s of prefilling a batch
+    of prompts and of decoding at a given context, both models in turn.
+    Random weights, synthetic tokens, one GPU."""
     from distllm_amd.engine import LLMEngine, SamplingParams
     from distllm_amd.engine.engine import _Seq
     from distllm_amd.models import ModelDims, build_model
     from distllm_amd.models.config import (ExpertsDims, hybrid_preset,
-                                           layered_preset)
+                                           layered_preset, looped_preset)
 
     dev = "cuda:0"
     torch.manual_seed(5)
@@ -276,7 +276,13 @@ def bench_decoders(args) -> None:
         return hybrid_preset(args.layers, hidden, V, heads, kv, 128,
                              ff * 3 // 2, chunk, order=order, **kw)
 
-    # name: (model, llama, [(prompts, prompt len)], [(batch, context)])
+    def tebasun(hidden, heads, kv, ff, order, **kw):
+        # half of the heads in each of two mixers side by side
+        return looped_preset(kw.pop("layers", args.layers), hidden, V, heads,
+                             kv, 128, ff, order, **kw)
+
+    # name: (model, the other one, [(prompts, prompt len)],
+    #        [(batch, context)])
     some = [(16, 2048)], [(1, 2048), (32, 2048), (128, 2048)]
     sizes = {
         "4096x32h full": (
@@ -307,6 +313,19 @@ def bench_decoders(args) -> None:
                      experts=ExpertsDims(ff=1024, experts=64, top=8,
                                          groups=8, keep=4)),
             llama(2048, 16, 4, 8192), *some),
+        "4096x32h parallel": (
+            tebasun(4096, 32, 16, 14336, "P"),
+            bufulorn(4096, 32, 8, 14336, 8192, "AD"),
+            some[0] + [(2, 8000)], some[1] + [(32, 8000)]),
+        "4096x32h recurrent": (
+            tebasun(4096, 32, 16, 14336, "R"),
+            bufulorn(4096, 32, 8, 14336, 8192, "D"),
+            some[0] + [(2, 8000)], some[1]),
+        # two thirds of the layers, the first half of them twice
+        "2048x16h looped": (
+            tebasun(2048, 16, 8, 8192, "PPR", layers=args.layers * 2 // 3,
+                    loop=(0, args.layers - args.layers * 2 // 3, 2)),
+            bufulorn(2048, 16, 4, 8192, 8192, "AD"), *some),
     }
     params = SamplingParams(temperature=0.0, min_p=0.0, max_tokens=10 ** 6)
     rows = []
@@ -314,8 +333,7 @@ def bench_decoders(args) -> None:
         if args.only and name.split()[0] not in args.only.split(",") \
                 and name not in args.only.split(","):
             continue
-        models = {md.arch: build_model(md, device=dev),
-                  "llama": build_model(ld, device=dev)}
+        models = {d.arch: build_model(d, device=dev) for d in (md, ld)}
 
         def run(kind, model, batch, ctx):
             eng = LLMEngine(model, max_batch_size=batch,
