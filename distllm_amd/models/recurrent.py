@@ -40,7 +40,8 @@ class GatedLru(Part):
         self.conv = nn.Parameter(torch.empty(d.conv, self.cols,
                                              dtype=torch.float32))
         self.conv_b = norm_weight(self.cols)
-        # decay and input gates: [gate, block, out, in]
+        # decay and input gates: [gate, block, out, in], stored in the order
+        # of ops.lru_gate_order
         self.gates = nn.Parameter(torch.empty(2, d.blocks, self.bs, self.bs,
                                               dtype=dtype))
         self.gates_b = nn.Parameter(torch.empty(2, self.cols,
@@ -76,7 +77,8 @@ class GatedLru(Part):
                 "bias": torch.cat([self._blocks(t[n + ".b"]) for n in "yx"]),
                 "conv": self._blocks(t["conv"]).t(),
                 "conv_b": self._blocks(t["conv.b"]),
-                "gates": torch.stack([gate("ra"), gate("ri")]),
+                "gates": ops.lru_gate_order(
+                    torch.stack([gate("ra"), gate("ri")])),
                 "gates_b": torch.stack([self._blocks(t[n].reshape(-1))
                                         for n in ("ra.b", "ri.b")]),
                 "decay": self._blocks(-self.d.decay_scale * soft),

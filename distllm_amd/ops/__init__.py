@@ -861,6 +861,14 @@ def channel_delta(ab, ag, heads, kv_heads, dp, vp, dim, vdim, conv_w, a_log,
         ctx, out)
 
 
+def lru_gate_order(w):
+    """Gate weights [.., out, in] in the order in which the MFMA takes them
+    (32 outputs by 32 inputs at a time), in the same shape; sizes % 32."""
+    n = w.shape[-1]
+    t = w.reshape(-1, n // 32, 16, 2, n // 32, 4, 8)
+    return t.permute(0, 1, 4, 3, 5, 2, 6).reshape(w.shape)
+
+
 def gated_lru(ab, conv_w, conv_b, gates, gates_b, decay, state, conv,
               segments, row_seq, ctx, chunk):
     """Linear recurrent unit of a ragged step on the projection ab [M,

@@ -52,12 +52,7 @@ attention_flash_kernel(const unsigned short* __restrict__ Q,
 
   // neighbouring query blocks of a head share most of their keys: give
   // each XCD a contiguous run of them
-  const int nwg = gridDim.x;
-  const int per = nwg / 8, rem = nwg % 8;
-  const int xcd = blockIdx.x % 8, j8 = blockIdx.x / 8;
-  const int bid =
-      (xcd < rem ? xcd * (per + 1) : rem * (per + 1) + (xcd - rem) * per) +
-      j8;
+  const int bid = xcd_run(blockIdx.x, gridDim.x);
   const int head = bid / nblocks;
   const int* pm = portions + blocks[(bid % nblocks) * 2] * 4;
   const int qb = blocks[(bid % nblocks) * 2 + 1];

@@ -26,21 +26,17 @@ extern "C" void launch_rotation_table(const int* ctx, const double* freq,
                      stream, ctx, freq, mult, table, M, pairs);
 }
 
-// Rotation of the numbers c .. c + 7 of a normed head, in place; x_of(i)
-// yields number i of the head. cs: cos, sin of the row's pairs.
-template <typename F>
-__device__ __forceinline__ void rotate8(float* x, int c, int half,
-                                        const float* cs, F x_of) {
+// Eight numbers x of a normed head from number c on, rotated with their
+// partners y (normed, too). cs: cos, sin of the row's pairs.
+__device__ __forceinline__ void rotate8(float* x, const float* y, int c,
+                                        int half, const float* cs) {
+  float t[16];
+  const bool low = c < half;
+  load8<float>(cs + (low ? c : c - half) * 2, t);
+  load8<float>(cs + (low ? c : c - half) * 2 + 8, t + 8);
 #pragma unroll
-  for (int i = 0; i < 8; ++i) {
-    const int col = c + i;
-    if (col >= 2 * half) return;
-    const bool low = col < half;
-    const int pair = low ? col : col - half;
-    const float other = x_of(low ? col + half : pair);
-    x[i] = x[i] * cs[pair * 2] +
-           (low ? -other : other) * cs[pair * 2 + 1];
-  }
+  for (int i = 0; i < 8; ++i)
+    x[i] = x[i] * t[2 * i] + (low ? -y[i] : y[i]) * t[2 * i + 1];
 }
 
 // ---- norm of query and key heads, cache write -----------------------------
@@ -50,7 +46,9 @@ __device__ __forceinline__ void rotate8(float* x, int c, int half,
 // workgroup norms UN times 256 / LPH of them. Values: the first row of a run
 // of consecutive positions in one page writes the run, whole 32-byte page
 // rows where the run covers the page; a wave looks at VR rows of one head.
-template <typename T, int LPH, int UN, bool ROT>
+// ROT 1: half is a multiple of 8, so that partners are eight in a row, too;
+// 2: any half.
+template <typename T, int LPH, int UN, int ROT>
 __global__ void __launch_bounds__(256)
 attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
                  int dp, int vp, int n, const float* __restrict__ wq,
@@ -75,15 +73,22 @@ attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
     const int u0 = blockIdx.x * UPI * UN + threadIdx.x / LPH;
     // a unit's head starts at (row, hd); its lanes' first eight columns
     // stay in registers, heads of more than 512 read the others twice
-    float v[UN][8];
+    float v[UN][8], y[ROT == 1 ? UN : 1][8];
+    // where the partners of eight columns start
+    auto partner = [&](int c) {
+      return c < half ? c + half : c < 2 * half ? c - half : c;
+    };
 #pragma unroll
     for (int k = 0; k < UN; ++k) {
       const int u = min(u0 + k * UPI, total - 1);
 #pragma unroll
       for (int i = 0; i < 8; ++i) v[k][i] = 0.f;
-      if (c0 < dp)
-        load8<T>(ab + (long)(u / units) * ld + (long)(u % units) * dp + c0,
-                 v[k]);
+      if (c0 < dp) {
+        const T* src =
+            ab + (long)(u / units) * ld + (long)(u % units) * dp;
+        load8<T>(src + c0, v[k]);
+        if (ROT == 1) load8<T>(src + partner(c0), y[k]);
+      }
     }
 #pragma unroll
     for (int k = 0; k < UN; ++k) {
@@ -118,20 +123,24 @@ attn_prep_kernel(const T* __restrict__ ab, int ld, int M, int H, int G,
         load8<float>(w + c, wv);
 #pragma unroll
         for (int i = 0; i < 8; ++i) x[i] = v[k][i] * inv * wv[i];
-        if (ROT && c < 2 * half) {
-          const float* cs = table + (long)row * 2 * half;
-          if (half % 8 == 0) {  // the other numbers are eight in a row too
-            const int o = c < half ? c + half : c - half;
-            float y[8], yw[8];
-            load8<T>(src + o, y);
-            load8<float>(w + o, yw);
-            rotate8(x, c, half, cs, [&](int j) {
-              return y[j - o] * inv * yw[j - o];
-            });
-          } else {
-            rotate8(x, c, half, cs, [&](int j) {
-              return to_f(src[j]) * inv * w[j];
-            });
+        const float* cs = table + (long)row * 2 * half;
+        if (ROT == 1 && c < 2 * half) {
+          if (c != c0) load8<T>(src + partner(c), y[k]);
+          load8<float>(w + partner(c), wv);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) y[k][i] *= inv * wv[i];
+          rotate8(x, y[k], c, half, cs);
+        }
+        if (ROT == 2) {
+#pragma unroll
+          for (int i = 0; i < 8; ++i) {
+            const int o = partner(c + i);
+            const bool low = c + i < half, in = c + i < 2 * half;
+            const int pair = in ? min(o, c + i) : 0;
+            const float z = to_f(src[o]) * inv * w[o];
+            const float r = x[i] * cs[pair * 2] +
+                            (low ? -z : z) * cs[pair * 2 + 1];
+            x[i] = in ? r : x[i];
           }
         }
         store8(dst + c, x);
@@ -212,10 +221,11 @@ extern "C" void launch_attn_prep(
                      n, wq, wk, eps, (T*)q, (T*)kpages, (T*)vpages,           \
                      block_table, max_blocks, num_blocks, row_seq, ctx,       \
                      norm_wgs, vr, v_at, table, half)
-#define APK(T, L, U)                             \
-  do {                                           \
-    if (table != nullptr) APK_R(T, L, U, true);  \
-    else APK_R(T, L, U, false);                  \
+#define APK(T, L, U)                          \
+  do {                                        \
+    if (table == nullptr) APK_R(T, L, U, 0);  \
+    else if (half % 8 == 0) APK_R(T, L, U, 1); \
+    else APK_R(T, L, U, 2);                   \
   } while (0)
 #define APK_U(T, L)           \
   do {                        \

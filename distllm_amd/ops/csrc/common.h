@@ -58,6 +58,14 @@ __device__ __forceinline__ void wave_sync() {
   __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 }
 
+// Workgroups go round the eight XCDs one by one: number b of n such that
+// each XCD (an L2 cache of its own) gets a contiguous run of numbers.
+__device__ __forceinline__ int xcd_run(int b, int n) {
+  const int per = n / 8, rem = n % 8, xcd = b % 8;
+  return (xcd < rem ? xcd * (per + 1) : rem * (per + 1) + (xcd - rem) * per) +
+         b / 8;
+}
+
 // Block-level reduce across NW waves using LDS scratch (NW <= 16).
 template <int NW>
 __device__ __forceinline__ float block_reduce_sum(float v, float* lds_scratch) {

@@ -147,7 +147,7 @@ torch::Tensor decode_gemm_rows(torch::Tensor X, torch::Tensor W,
 torch::Tensor gelu_rows(torch::Tensor z, torch::Tensor tokens,
                         torch::Tensor table, int64_t col0, int64_t n) {
   CHECK_DEV(z); CHECK_CONT(z); CHECK_T(z); CHECK_SAME(z, table);
-  TORCH_CHECK(z.dim() == 2, "rank");
+  TORCH_CHECK(z.dim() == 2 && z.size(1) % 8 == 0, "columns % 8");
   const long M = z.size(0);
   const int N = z.size(1);
   const RowsArgs r = rows_args(tokens, table, M, col0, n, N);

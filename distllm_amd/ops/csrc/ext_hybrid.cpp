@@ -525,14 +525,14 @@ void channel_delta(torch::Tensor ab, torch::Tensor ag, int64_t H, int64_t G,
                     seg_rows.data_ptr<int>(), seg_slot.data_ptr<int>(), S,
                     (int)longest, limit, row_seq.data_ptr<int>(),
                     ctx.data_ptr<int>(), true, is_f32(ab), cur_stream());
-  launch_delta_scan(qk.data_ptr<float>(), v.data_ptr(),
-                    beta.data_ptr<float>(), gc.data_ptr<float>(), gate, ld_ag,
-                    o_norm.data_ptr<float>(), (float)out_scale,
-                    state.data_ptr<float>(), out.data_ptr(), ld_y, H, G, dp,
-                    vp, vdim, (float)eps, seg_row0.data_ptr<int>(),
-                    seg_rows.data_ptr<int>(), seg_slot.data_ptr<int>(), S,
-                    ctx.data_ptr<int>(), limit, true, is_f32(ab),
-                    cur_stream());
+  if (!chunked || longs->size(0) < S)
+    launch_delta_scan(
+        qk.data_ptr<float>(), v.data_ptr(), beta.data_ptr<float>(),
+        gc.data_ptr<float>(), gate, ld_ag, o_norm.data_ptr<float>(),
+        (float)out_scale, state.data_ptr<float>(), out.data_ptr(), ld_y, H, G,
+        dp, vp, vdim, (float)eps, seg_row0.data_ptr<int>(),
+        seg_rows.data_ptr<int>(), seg_slot.data_ptr<int>(), S,
+        ctx.data_ptr<int>(), limit, true, is_f32(ab), cur_stream());
   if (!chunked) return;
   TORCH_CHECK(chunks.has_value(), "chunks");
   CHECK_INTS(longs.value()); CHECK_INTS(chunks.value());

@@ -5,10 +5,10 @@
 //
 //   lru_conv_kernel   u
 //   lru_gates_kernel  both gate products on the MFMA and everything up to
-//                     the recurrence; rows of short segments: log a and the
+//                     the recurrence; rows of short segments: a and the
 //                     drive; chunks of long ones: their recurrence from
-//                     zeros and the summed log a, so that a state S before
-//                     the chunk adds exp(sum) S
+//                     zeros and the product of the decays so far, times
+//                     which a state before the chunk is added
 //   lru_scan_kernel   short segments, row by row
 //   lru_carry_kernel  long segments: state before every chunk
 //   lru_emit_kernel   long segments: output
@@ -19,6 +19,7 @@
 typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 
 #define LCH 64  // rows of a chunk
+#define LOG2E 1.4426950408889634f
 
 template <typename T>
 __device__ __forceinline__ float gelu_of(float x) {
@@ -85,14 +86,11 @@ lru_conv_kernel(ConvArgs<T> a, const float* __restrict__ bias,
   }
 }
 
-// sqrt(1 - exp(2 la)) for la <= 0, also where la is tiny
-__device__ __forceinline__ float drive_factor(float la) {
-  const float z = 2.f * la;
-  const float near =
-      -z * (1.f +
-            z * 0.5f *
-                (1.f + z * 0.33333333f * (1.f + z * 0.25f * (1.f + z * 0.2f))));
-  return __builtin_amdgcn_sqrtf(z > -0.1f ? near : 1.f - fast_exp(z));
+// sqrt(1 - a^2) of a = exp2(la2) <= 1, also where la2 is tiny
+__device__ __forceinline__ float drive_factor(float la2, float a) {
+  const float z = la2 * 1.3862943611198906f;
+  const float near = -z * (1.f + z * (0.5f + z * 0.16666667f));
+  return __builtin_amdgcn_sqrtf(z > -0.03f ? near : 1.f - a * a);
 }
 
 struct LruGates {
@@ -101,20 +99,44 @@ struct LruGates {
   int M, C, blocks, bs, max_rows;
 };
 
+// Weights of both gates lie in the order in which the MFMA takes them:
+// [gate, block, 32 outputs, 32 inputs, j, g, i, e], output i * 2 + j of the
+// 32 and input g * 8 + e of the 32: a lane gets two neighbouring channels.
+__device__ __forceinline__ long gate_at(const LruGates& a, int z, int blk,
+                                        int n, int k) {
+  const long tile =
+      (((long)z * a.blocks + blk) * (a.bs / 32) + n / 32) * (a.bs / 32) +
+      k / 32;
+  return tile * 1024 + n % 2 * 512 + (k % 32 / 8 * 16 + n % 32 / 2) * 8 +
+         k % 8;
+}
+
+#define PIECE 256        // inner indices that are staged in LDS at once
+#define UROW (PIECE + 8)  // padded LDS row
+
 // A wave: MT * 16 rows and 32 channels of both gates; a workgroup: four
 // neighbouring groups of 32 channels. LONG: the rows are a chunk; else they
-// are 16 consecutive rows, of which those of short segments count.
-template <int MT, bool LONG>
-__global__ void __launch_bounds__(256)
+// are 16 consecutive rows, of which those of short segments count. SHARED:
+// the workgroup's channels are of one block, and its u passes through LDS.
+template <int MT, bool LONG, bool SHARED>
+__global__ void __launch_bounds__(256, 3)
 lru_gates_kernel(const unsigned short* __restrict__ u,
                  const unsigned short* __restrict__ w, const LruGates a,
                  const int* __restrict__ chunks, int groups,
-                 float* __restrict__ sum, float* __restrict__ hs) {
+                 float* __restrict__ prod, float* __restrict__ hs) {
+  __shared__ __attribute__((aligned(16)))
+  unsigned short ul[SHARED ? MT * 16 * UROW : 1];
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int i16 = lane & 15, g = lane >> 4;
-  const int tile = blockIdx.x / groups;
-  const int c0 = (blockIdx.x % groups * 4 + wid) * 32;
-  if (c0 >= a.C) return;
+  // an XCD keeps to neighbouring groups, whose weights stay in its L2
+  int tile = blockIdx.x / groups, group = blockIdx.x % groups;
+  if (groups % 8 == 0) {
+    const int own = groups / 8, i = blockIdx.x / 8;
+    tile = i / own;
+    group = blockIdx.x % 8 * own + i % own;
+  }
+  const int c0 = (group * 4 + wid) * 32;
+  if (!SHARED && c0 >= a.C) return;
   long row0;
   int cnt;
   if (LONG) {
@@ -133,10 +155,10 @@ lru_gates_kernel(const unsigned short* __restrict__ u,
       mine = a.ctx[row0 + i16] > 0 &&
              a.seg_rows[a.row_seq[row0 + i16]] <= a.max_rows;
     live = __ballot(mine);
-    if (live == 0) return;
+    if (live == 0) return;  // the same in every wave
   }
 
-  f32x4 acc[2][2][MT];  // gate, group of 16 channels, row tile
+  f32x4 acc[2][2][MT];  // gate, channel i16 * 2 + j, row tile
 #pragma unroll
   for (int z = 0; z < 2; ++z)
 #pragma unroll
@@ -144,108 +166,168 @@ lru_gates_kernel(const unsigned short* __restrict__ u,
 #pragma unroll
       for (int m = 0; m < MT; ++m) acc[z][j][m] = (f32x4)0.f;
   const bool real = c0 < a.blocks * a.bs;  // else a column of padding
-  if (real) {
+  if (SHARED || real) {
     const int blk = c0 / a.bs, n0 = c0 % a.bs;
-    const unsigned short* ur[MT];
-#pragma unroll
-    for (int m = 0; m < MT; ++m)
-      ur[m] = u + (row0 + min(m * 16 + i16, cnt - 1)) * a.C + blk * a.bs +
-              g * 8;
     const unsigned short* wr[2][2];
 #pragma unroll
     for (int z = 0; z < 2; ++z)
 #pragma unroll
       for (int j = 0; j < 2; ++j)
-        wr[z][j] = w +
-                   (((long)z * a.blocks + blk) * a.bs + n0 + j * 16 + i16) *
-                       a.bs +
-                   g * 8;
+        wr[z][j] = w + gate_at(a, z, blk, n0 + j, 0) + lane * 8;
+    for (int p0 = 0; p0 < a.bs; p0 += PIECE) {
+      const int len = SHARED ? min(PIECE, a.bs - p0) : PIECE;
+      if (SHARED) {
+        __syncthreads();  // the previous piece is consumed
+        for (int i = threadIdx.x; i < MT * 16 * (PIECE / 8); i += 256) {
+          const int row = i / (PIECE / 8), c = i % (PIECE / 8) * 8;
+          if (c < len)
+            *reinterpret_cast<i32x4*>(ul + row * UROW + c) =
+                *reinterpret_cast<const i32x4*>(
+                    u + (row0 + min(row, cnt - 1)) * a.C + blk * a.bs + p0 +
+                    c);
+        }
+        __syncthreads();
+      }
 #pragma unroll 2
-    for (int k = 0; k < a.bs; k += 32) {
-      bf16x8 uf[MT], wf[2][2];
+      for (int k = p0; k < min(p0 + PIECE, a.bs); k += 32) {
+        bf16x8 uf[MT], wf[2][2];
 #pragma unroll
-      for (int m = 0; m < MT; ++m)
-        uf[m] = *reinterpret_cast<const bf16x8*>(ur[m] + k);
+        for (int z = 0; z < 2; ++z)
 #pragma unroll
-      for (int z = 0; z < 2; ++z)
+          for (int j = 0; j < 2; ++j)
+            wf[z][j] =
+                *reinterpret_cast<const bf16x8*>(wr[z][j] + (long)k * 32);
 #pragma unroll
-        for (int j = 0; j < 2; ++j)
-          wf[z][j] = *reinterpret_cast<const bf16x8*>(wr[z][j] + k);
+        for (int m = 0; m < MT; ++m) {
+          const int t = m * 16 + i16;
+          uf[m] = *reinterpret_cast<const bf16x8*>(
+              SHARED ? ul + t * UROW + k - p0 + g * 8
+                     : u + (row0 + min(t, cnt - 1)) * a.C + blk * a.bs + k +
+                           g * 8);
+        }
 #pragma unroll
-      for (int z = 0; z < 2; ++z)
+        for (int z = 0; z < 2; ++z)
 #pragma unroll
-        for (int j = 0; j < 2; ++j)
+          for (int j = 0; j < 2; ++j)
 #pragma unroll
-          for (int m = 0; m < MT; ++m)
-            acc[z][j][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-                uf[m], wf[z][j], acc[z][j][m], 0, 0, 0);
+            for (int m = 0; m < MT; ++m)
+              acc[z][j][m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+                  uf[m], wf[z][j], acc[z][j][m], 0, 0, 0);
+      }
     }
   }
 
+  // Offsets from the first row, in 32 bits; a lane has rows g * 4 + r of
+  // every row tile and channels c, c + 1.
+  const int c = c0 + i16 * 2;
+  const unsigned short* ub = u + row0 * a.C + c;
+  float *pb = prod + row0 * a.C + c, *hb = hs + row0 * a.C + c;
+  const bool full = real && cnt == MT * 16;
+  unsigned uv[MT][4];  // two bf16
+#pragma unroll
+  for (int m = 0; m < MT; ++m)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const unsigned t = m * 16 + g * 4 + r;
+      uv[m][r] = *reinterpret_cast<const unsigned*>(
+          ub + (full ? t : min(t, (unsigned)cnt - 1)) * (unsigned)a.C);
+    }
+  // decays and drives; rows behind the end keep the state as it is
+  f32x4 ea[2][MT], x[2][MT];
 #pragma unroll
   for (int j = 0; j < 2; ++j) {
-    const int c = c0 + j * 16 + i16;
-    const float br = a.br[c], bi = a.bi[c], decay = a.decay[c];
-    float la0 = 0.f, h0 = 0.f;  // sum and state before the row tile
+    const float br = -LOG2E * a.br[c + j], bi = -LOG2E * a.bi[c + j];
+    const float decay = LOG2E * a.decay[c + j];
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float zr = fmaf(acc[0][j][m][r], -LOG2E, br);
+        const float zi = fmaf(acc[1][j][m][r], -LOG2E, bi);
+        const float la =
+            decay * fast_rcp(1.f + __builtin_amdgcn_exp2f(zr));
+        const float e = __builtin_amdgcn_exp2f(la);
+        const float d =
+            drive_factor(la, e) *
+            bf2f((unsigned short)(j ? uv[m][r] >> 16 : uv[m][r])) *
+            fast_rcp(1.f + __builtin_amdgcn_exp2f(zi));
+        const bool ok = full || (real && m * 16 + g * 4 + r < cnt);
+        ea[j][m][r] = ok ? e : 1.f;
+        x[j][m][r] = ok ? d : 0.f;
+      }
+  }
+  if (!LONG) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = g * 4 + r;
+      if (live >> t & 1) {
+        const f32x2 e = {ea[0][0][r], ea[1][0][r]};
+        const f32x2 d = {x[0][0][r], x[1][0][r]};
+        *reinterpret_cast<f32x2*>(pb + (unsigned)(t * a.C)) = e;
+        *reinterpret_cast<f32x2*>(hb + (unsigned)(t * a.C)) = d;
+      }
+    }
+    return;
+  }
+  // a lane's four rows, then the lanes before it in the tile
+  float A[2][MT], h[2][MT], endA[2][MT], endH[2][MT];
+#pragma unroll
+  for (int j = 0; j < 2; ++j)
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
-      // a lane holds rows g * 4 + r of the tile
-      float la[4], x[4];
+      A[j][m] = 1.f;
+      h[j][m] = 0.f;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int t = m * 16 + g * 4 + r;
-        la[r] = x[r] = 0.f;
-        if (t < cnt && real) {
-          const float uv = bf2f(u[(row0 + t) * a.C + c]);
-          la[r] = decay * fast_rcp(1.f + fast_exp(-acc[0][j][m][r] - br));
-          x[r] = drive_factor(la[r]) *
-                 fast_rcp(1.f + fast_exp(-acc[1][j][m][r] - bi)) * uv;
-        }
+        h[j][m] = ea[j][m][r] * h[j][m] + x[j][m][r];
+        A[j][m] *= ea[j][m][r];
       }
-      if (!LONG) {
+    }
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int t = g * 4 + r;
-          if (live >> t & 1) {
-            sum[(row0 + t) * a.C + c] = la[r];
-            hs[(row0 + t) * a.C + c] = x[r];
-          }
-        }
-        continue;
-      }
-      float ea[4], A = 0.f, h = 0.f;
+  for (int off = 16; off <= 32; off <<= 1)
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        ea[r] = fast_exp(la[r]);
-        A += la[r];
-        h = ea[r] * h + x[r];
-      }
-      // lanes g before this one, then the tiles before
+    for (int j = 0; j < 2; ++j)
 #pragma unroll
-      for (int off = 16; off <= 32; off <<= 1) {
-        const float pa = __shfl_up(A, off, 64), ph = __shfl_up(h, off, 64);
-        if (lane >= off) {
-          h += fast_exp(A) * ph;
-          A += pa;
-        }
+      for (int m = 0; m < MT; ++m) {
+        const float fa = __shfl_up(A[j][m], off, 64);
+        const float fh = __shfl_up(h[j][m], off, 64);
+        h[j][m] = lane >= off ? h[j][m] + A[j][m] * fh : h[j][m];
+        A[j][m] = lane >= off ? A[j][m] * fa : A[j][m];
       }
-      const float endA = __shfl(A, 48 + i16, 64);
-      const float endH = __shfl(h, 48 + i16, 64);
-      float pa = __shfl_up(A, 16, 64), ph = __shfl_up(h, 16, 64);
-      if (g == 0) pa = ph = 0.f;
-      float s = fast_exp(pa) * h0 + ph, l = la0 + pa;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int t = m * 16 + g * 4 + r;
-        s = ea[r] * s + x[r];
-        l += la[r];
-        if (t < cnt) {
-          sum[(row0 + t) * a.C + c] = l;
-          hs[(row0 + t) * a.C + c] = s;
-        }
+  for (int j = 0; j < 2; ++j)
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+      endA[j][m] = __shfl(A[j][m], 48 + i16, 64);
+      endH[j][m] = __shfl(h[j][m], 48 + i16, 64);
+      const float pa = __shfl_up(A[j][m], 16, 64);
+      const float ph = __shfl_up(h[j][m], 16, 64);
+      A[j][m] = g == 0 ? 1.f : pa;
+      h[j][m] = g == 0 ? 0.f : ph;
+    }
+  f32x2 A0 = {1.f, 1.f}, h0 = {0.f, 0.f};  // of the tiles before
+#pragma unroll
+  for (int m = 0; m < MT; ++m) {
+    f32x2 s, l;
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+      s[j] = A[j][m] * h0[j] + h[j][m];
+      l[j] = A0[j] * A[j][m];
+      h0[j] = endA[j][m] * h0[j] + endH[j][m];
+      A0[j] *= endA[j][m];
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int t = m * 16 + g * 4 + r;
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        s[j] = ea[j][m][r] * s[j] + x[j][m][r];
+        l[j] *= ea[j][m][r];
       }
-      h0 = fast_exp(endA) * h0 + endH;
-      la0 += endA;
+      if (full || t < cnt) {
+        *reinterpret_cast<f32x2*>(pb + (unsigned)(t * a.C)) = l;
+        *reinterpret_cast<f32x2*>(hb + (unsigned)(t * a.C)) = s;
+      }
     }
   }
 }
@@ -253,7 +335,7 @@ lru_gates_kernel(const unsigned short* __restrict__ u,
 // 32-bit mode: a thread per (row, channel)
 __global__ void __launch_bounds__(256)
 lru_gates32_kernel(const float* __restrict__ u, const float* __restrict__ w,
-                   const LruGates a, float* __restrict__ sum,
+                   const LruGates a, float* __restrict__ prod,
                    float* __restrict__ hs) {
   const long id = (long)blockIdx.x * 256 + threadIdx.x;
   const long row = id / a.C;
@@ -263,13 +345,13 @@ lru_gates32_kernel(const float* __restrict__ u, const float* __restrict__ w,
   if (c < a.blocks * a.bs) {
     const int blk = c / a.bs, n = c % a.bs;
     const float* ur = u + row * a.C + blk * a.bs;
-    const float* wr = w + ((long)blk * a.bs + n) * a.bs;
-    const float* wi = wr + (long)a.blocks * a.bs * a.bs;
     float zr = 0.f, zi = 0.f;
     for (int k = 0; k < a.bs; k += 4) {
       const f32x4 uv = *reinterpret_cast<const f32x4*>(ur + k);
-      const f32x4 rv = *reinterpret_cast<const f32x4*>(wr + k);
-      const f32x4 iv = *reinterpret_cast<const f32x4*>(wi + k);
+      const f32x4 rv =
+          *reinterpret_cast<const f32x4*>(w + gate_at(a, 0, blk, n, k));
+      const f32x4 iv =
+          *reinterpret_cast<const f32x4*>(w + gate_at(a, 1, blk, n, k));
 #pragma unroll
       for (int e = 0; e < 4; ++e) {
         zr += uv[e] * rv[e];
@@ -280,7 +362,7 @@ lru_gates32_kernel(const float* __restrict__ u, const float* __restrict__ w,
     x = sqrtf(-expm1f(2.f * la)) * sigmoid_exact(zi + a.bi[c]) *
         u[row * a.C + c];
   }
-  sum[id] = la;
+  prod[id] = expf(la);
   hs[id] = x;
 }
 
@@ -288,7 +370,7 @@ lru_gates32_kernel(const float* __restrict__ u, const float* __restrict__ w,
 template <typename T>
 __global__ void __launch_bounds__(256)
 lru_scan_kernel(const T* __restrict__ ab, int ld,
-                const float* __restrict__ la, const float* __restrict__ x,
+                const float* __restrict__ a, const float* __restrict__ x,
                 float* __restrict__ state, T* __restrict__ out, int C,
                 const int* __restrict__ seg_row0,
                 const int* __restrict__ seg_rows,
@@ -303,14 +385,14 @@ lru_scan_kernel(const T* __restrict__ ab, int ld,
 #pragma unroll 4
   for (int t = 0; t < n; ++t) {
     const long row = row0 + t;
-    s = expf(la[row * C + c]) * s + x[row * C + c];
+    s = a[row * C + c] * s + x[row * C + c];
     from_f(out + row * C + c, s * gelu_of<T>(to_f(ab[row * ld + c])));
   }
   *st = s;
 }
 
 __global__ void __launch_bounds__(256)
-lru_carry_kernel(const float* __restrict__ sum, const float* __restrict__ hs,
+lru_carry_kernel(const float* __restrict__ prod, const float* __restrict__ hs,
                  float* __restrict__ state, float* __restrict__ start, int C,
                  const int* __restrict__ longs,
                  const int* __restrict__ seg_row0,
@@ -330,14 +412,14 @@ lru_carry_kernel(const float* __restrict__ sum, const float* __restrict__ hs,
 #pragma unroll
     for (int k = 0; k < U; ++k) {  // loads first
       const long row = row0 + min((min(k0 + k, nch - 1) + 1) * LCH, n) - 1;
-      A[k] = sum[row * C + c];
+      A[k] = prod[row * C + c];
       h[k] = hs[row * C + c];
     }
 #pragma unroll
     for (int k = 0; k < U; ++k)
       if (k0 + k < nch) {
         start[(chunk0 + k0 + k) * C + c] = s;
-        s = fast_exp(A[k]) * s + h[k];
+        s = A[k] * s + h[k];
       }
   }
   *st = s;
@@ -346,7 +428,7 @@ lru_carry_kernel(const float* __restrict__ sum, const float* __restrict__ hs,
 // a thread: eight channels of eight rows of a chunk
 __global__ void __launch_bounds__(256)
 lru_emit_kernel(const unsigned short* __restrict__ ab, int ld,
-                const float* __restrict__ sum, const float* __restrict__ hs,
+                const float* __restrict__ prod, const float* __restrict__ hs,
                 const float* __restrict__ start,
                 unsigned short* __restrict__ out, int C,
                 const int* __restrict__ chunks, int nchunks,
@@ -366,23 +448,23 @@ lru_emit_kernel(const unsigned short* __restrict__ ab, int ld,
   for (int t = 0; t < n; ++t) {
     const long row = seg_row0[seg] + t0 + t;
     float A[8], h[8], y[8];
-    load8<float>(sum + row * C + ch, A);
+    load8<float>(prod + row * C + ch, A);
     load8<float>(hs + row * C + ch, h);
     load8<unsigned short>(ab + row * ld + ch, y);
 #pragma unroll
     for (int i = 0; i < 8; ++i)
-      h[i] = (h[i] + fast_exp(A[i]) * s[i]) * fast_gelu(y[i]);
+      h[i] = (h[i] + A[i] * s[i]) * fast_gelu(y[i]);
     store8(out + row * C + ch, h);
   }
 }
 
-// ab [M, y | x] of C columns each; u [M, C], sum and hs [M, C] fp32, start
+// ab [M, y | x] of C columns each; u [M, C], prod and hs [M, C] fp32, start
 // [nchunks, C] fp32: scratch. nlong 0: no long segments.
 extern "C" void launch_gated_lru(
     const void* ab, int ld, int M, int C, const float* conv_w,
     const float* conv_b, int taps, const void* gates, const float* gates_b,
     int blocks, int bs, const float* decay, float* state, void* conv, void* u,
-    float* sum, float* hs, float* start, void* out, const int* seg_row0,
+    float* prod, float* hs, float* start, void* out, const int* seg_row0,
     const int* seg_rows, const int* seg_slot, int nseg, int longest,
     const int* row_seq, const int* ctx, const int* longs, int nlong,
     const int* chunks, int nchunks, int max_rows, bool fp32,
@@ -413,32 +495,34 @@ extern "C" void launch_gated_lru(
   if (fp32) {
     hipLaunchKernelGGL(lru_gates32_kernel, dim3(((long)M * C + 255) / 256),
                        dim3(256), 0, stream, (const float*)u,
-                       (const float*)gates, a, sum, hs);
+                       (const float*)gates, a, prod, hs);
     hipLaunchKernelGGL(lru_scan_kernel<float>, scan_grid, dim3(256), 0,
-                       stream, (const float*)ab, ld, sum, hs, state,
+                       stream, (const float*)ab, ld, prod, hs, state,
                        (float*)out, C, seg_row0, seg_rows, seg_slot, ctx,
                        INT_MAX);
     return;
   }
   typedef unsigned short bf;
   const int groups = (C + 127) / 128;
-  hipLaunchKernelGGL((lru_gates_kernel<1, false>),
-                     dim3((long)(M + 15) / 16 * groups), dim3(256), 0, stream,
-                     (const bf*)u, (const bf*)gates, a, chunks, groups, sum,
-                     hs);
-  hipLaunchKernelGGL(lru_scan_kernel<bf>, scan_grid, dim3(256), 0, stream,
-                     (const bf*)ab, ld, sum, hs, state, (bf*)out, C, seg_row0,
-                     seg_rows, seg_slot, ctx, max_rows);
+  const bool shared = bs % 128 == 0 && blocks * bs == C;
+#define LG(MT, L, S, N)                                                      \
+  hipLaunchKernelGGL((lru_gates_kernel<MT, L, S>), dim3((long)(N) * groups), \
+                     dim3(256), 0, stream, (const bf*)u, (const bf*)gates,   \
+                     a, chunks, groups, prod, hs)
+  if (nlong < nseg) LG(1, false, false, (M + 15) / 16);
+  if (nlong < nseg)
+    hipLaunchKernelGGL(lru_scan_kernel<bf>, scan_grid, dim3(256), 0, stream,
+                       (const bf*)ab, ld, prod, hs, state, (bf*)out, C,
+                       seg_row0, seg_rows, seg_slot, ctx, max_rows);
   if (nlong == 0) return;
-  hipLaunchKernelGGL((lru_gates_kernel<LCH / 16, true>),
-                     dim3((long)nchunks * groups), dim3(256), 0, stream,
-                     (const bf*)u, (const bf*)gates, a, chunks, groups, sum,
-                     hs);
+  if (shared) LG(LCH / 16, true, true, nchunks);
+  else LG(LCH / 16, true, false, nchunks);
+#undef LG
   hipLaunchKernelGGL(lru_carry_kernel, dim3((C + 255) / 256, nlong),
-                     dim3(256), 0, stream, sum, hs, state, start, C, longs,
+                     dim3(256), 0, stream, prod, hs, state, start, C, longs,
                      seg_row0, seg_rows, seg_slot, ctx);
   hipLaunchKernelGGL(lru_emit_kernel,
                      dim3(((long)nchunks * (LCH / 8) * (C / 8) + 255) / 256),
-                     dim3(256), 0, stream, (const bf*)ab, ld, sum, hs, start,
+                     dim3(256), 0, stream, (const bf*)ab, ld, prod, hs, start,
                      (bf*)out, C, chunks, nchunks, seg_row0, seg_rows);
 }

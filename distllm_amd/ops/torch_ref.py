@@ -680,6 +680,9 @@ def gated_lru(ab, conv_w, conv_b, gates, gates_b, decay, state, conv,
               segments, row_seq, ctx):
     M, C = ab.shape[0], conv_w.shape[1]
     B, bs = gates.shape[1], gates.shape[2]
+    # [gate, block, in, out] from the stored order (ops.lru_gate_order)
+    w = gates.float().view(2, B, bs // 32, bs // 32, 2, 4, 16, 8)
+    w = w.permute(0, 1, 3, 5, 7, 2, 6, 4).reshape(2, B, bs, bs)
     out = torch.zeros(M, C, dtype=ab.dtype)
     for row0, n, slot in zip(segments.row0.tolist(), segments.rows.tolist(),
                              segments.slot.tolist()):
@@ -692,8 +695,7 @@ def gated_lru(ab, conv_w, conv_b, gates, gates_b, decay, state, conv,
         u = u.to(ab.dtype).float()
         z = torch.zeros(2, n, C)
         z[..., : B * bs] = torch.matmul(
-            u[:, : B * bs].view(n, B, bs).transpose(0, 1),
-            gates.float().transpose(2, 3).contiguous()
+            u[:, : B * bs].view(n, B, bs).transpose(0, 1), w
         ).transpose(1, 2).reshape(2, n, B * bs)
         z = torch.sigmoid(z + gates_b[:, None])
         log_a = decay * z[0]
