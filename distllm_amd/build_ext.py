@@ -17,7 +17,7 @@ ROOT = Path(__file__).resolve().parents[1]
 # config.json "architecture" -> the extensions that the model's steps use
 NEEDED = {"Kanotar": ("_hip_gemm", "_hip_residual", "_hip_latent"),
           "Bufulorn": ("_hip_gemm", "_hip_residual", "_hip_hybrid",
-                       "_hip_experts"),
+                       "_hip_chunked", "_hip_experts"),
           "Tebasun": ("_hip_gemm", "_hip_residual", "_hip_hybrid",
                       "_hip_lru")}
 

@@ -660,7 +660,7 @@ def paged_attn_rows(q, kpages, vpages, ab, gate_at, out, block_table,
     sees the positions of its chunk up to its own. The output is gated by
     the sigmoid of ab's columns from gate_at on."""
     if q.is_cuda:
-        _require_hip("_hip_hybrid")
+        _require_hip("_hip_chunked")
         _hip_ops.paged_attn_rows(q, kpages, vpages, ab, gate_at, out,
                                  block_table, row_seq, ctx, chunk, scale,
                                  softcap, dist, nsplit)
@@ -674,7 +674,7 @@ def paged_attn_prompts(q, kpages, vpages, ab, gate_at, out, block_table,
                        prompts, chunk, scale, softcap, dist):
     """The same for the rows of prompt portions (step.PromptBlocks)."""
     if q.is_cuda:
-        _require_hip("_hip_hybrid")
+        _require_hip("_hip_chunked")
         _hip_ops.paged_attn_prompts(q, kpages, vpages, ab, gate_at, out,
                                     block_table, prompts.portions,
                                     prompts.blocks, chunk, scale, softcap,

@@ -1,6 +1,6 @@
-// Torch bindings of attention over paged keys and values and of the gated
-// delta rules.
-#include "ext_common.h"
+// Torch bindings of attention with sinks over paged keys and values, of what
+// precedes attention over pages, and of the gated delta rules.
+#include "ext_attention.h"
 
 extern "C" {
 void launch_rotation_table(const int*, const double*, float, float*, int, int,
@@ -9,18 +9,6 @@ void launch_attn_prep(const void*, int, int, int, int, int, int, int,
                       const float*, const float*, float, void*, void*, void*,
                       const int*, int, int, const int*, const int*, int,
                       const float*, int, bool, hipStream_t);
-void launch_chunk_rows(const void*, const void*, const void*, const void*,
-                       int, const int*, const int*, const int*, void*, int,
-                       int, int, int, int, int, int, float, float,
-                       const float*, bool, hipStream_t);
-void launch_chunk_decode(const void*, const void*, const void*, const void*,
-                         int, const int*, const int*, const int*, void*,
-                         void*, void*, int, int, int, int, int, int, int, int,
-                         float, float, const float*, hipStream_t);
-void launch_chunk_flash(const void*, const void*, const void*, const void*,
-                        int, void*, const int*, int, const int*, const int*,
-                        int, int, int, int, int, int, float, float,
-                        const float*, hipStream_t);
 void launch_sink_rows(const void*, const void*, const void*, const int*,
                       const int*, const int*, void*, long, int, int, int, int,
                       int, int, float, const float*, float, bool,
@@ -55,30 +43,6 @@ void launch_channel_chunks(const float*, const void*, const float*,
                            int, float, const int*, int, const int*, int, int,
                            const int*, const int*, const int*, const int*,
                            const int*, hipStream_t);
-}
-
-struct Pages {
-  int nblk, G, DK, DV;
-};
-
-static Pages check_pages(const torch::Tensor& k, const torch::Tensor& v) {
-  CHECK_DEV(k); CHECK_CONT(k); CHECK_T(k);
-  CHECK_DEV(v); CHECK_CONT(v); CHECK_SAME(k, v);
-  TORCH_CHECK(k.dim() == 4 && v.dim() == 4 && k.size(2) == 16 &&
-                  v.size(3) == 16 && k.size(0) == v.size(0) &&
-                  k.size(1) == v.size(1),
-              "pages must be [blocks, heads, 16, dim], [blocks, heads, "
-              "vdim, 16]");
-  TORCH_CHECK(k.size(3) % 64 == 0 && v.size(2) % 64 == 0,
-              "head sizes % 64");
-  return {(int)k.size(0), (int)k.size(1), (int)k.size(3), (int)v.size(2)};
-}
-
-static void check_rows(const torch::Tensor& bt, const torch::Tensor& row_seq,
-                       const torch::Tensor& ctx, long M) {
-  CHECK_INTS(bt); CHECK_INTS(row_seq); CHECK_INTS(ctx);
-  TORCH_CHECK(bt.dim() == 2 && row_seq.numel() == M && ctx.numel() == M,
-              "one row_seq and ctx entry per row");
 }
 
 torch::Tensor attn_prep(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
@@ -172,113 +136,6 @@ torch::Tensor rotary_prep(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
                      (int)(H * dp), table.data_ptr<float>(), table.size(1),
                      is_f32(ab), cur_stream());
   return q;
-}
-
-struct AttnArgs {
-  Pages p;
-  int M, H, ld;
-  const void* gate;
-};
-
-static AttnArgs check_attn(const torch::Tensor& q, const torch::Tensor& k,
-                           const torch::Tensor& v, const torch::Tensor& ab,
-                           int64_t gate_at, const torch::Tensor& out,
-                           int64_t chunk, double softcap,
-                           const torch::Tensor& dist) {
-  const Pages p = check_pages(k, v);
-  CHECK_DEV(q); CHECK_CONT(q); CHECK_SAME(q, k);
-  CHECK_DEV(out); CHECK_CONT(out); CHECK_SAME(out, k);
-  CHECK_SAME(ab, k);
-  CHECK_FLOATS(dist);
-  TORCH_CHECK(q.dim() == 3 && out.dim() == 3, "ranks");
-  const int M = q.size(0), H = q.size(1), ld = row_stride(ab);
-  TORCH_CHECK(q.size(2) == p.DK && out.size(0) == M && out.size(1) == H &&
-                  out.size(2) == p.DV && H % p.G == 0 && ab.size(0) == M,
-              "attention shapes");
-  TORCH_CHECK(gate_at >= 0 && gate_at % 8 == 0 && ld % 8 == 0 &&
-                  ab.size(1) >= gate_at + (long)H * p.DV,
-              "gate columns");
-  TORCH_CHECK(dist.numel() == 2 * H && chunk > 0 && softcap > 0, "constants");
-  return {p, M, H, ld,
-          (const char*)ab.data_ptr() + gate_at * ab.element_size()};
-}
-
-// Split each row's keys until the CUs are full (four workgroups each), as
-// long as a wave keeps two tiles. All sizes are known on the host, so a
-// captured graph stays valid as contexts grow.
-static long key_splits(long nsplit, long M, long H, long G, long chunk,
-                       long max_blocks) {
-  if (nsplit <= 0) {
-    const long wgs = M * G * ((H / G + 15) / 16);
-    const long tiles = std::min<long>(chunk, max_blocks * 16L) / 32 + 1;
-    nsplit = std::min<long>({(1024 + wgs - 1) / wgs, tiles / 8, 64L});
-  }
-  return std::max<long>(nsplit, 1);
-}
-
-static bool mfma_size(int d) { return d == 64 || d == 128 || d == 256; }
-
-void paged_attn_rows(torch::Tensor q, torch::Tensor k, torch::Tensor v,
-                     torch::Tensor ab, int64_t gate_at, torch::Tensor out,
-                     torch::Tensor bt, torch::Tensor row_seq,
-                     torch::Tensor ctx, int64_t chunk, double scale,
-                     double softcap, torch::Tensor dist, int64_t nsplit) {
-  const AttnArgs a = check_attn(q, k, v, ab, gate_at, out, chunk, softcap,
-                                dist);
-  check_rows(bt, row_seq, ctx, a.M);
-  if (a.M == 0) return;
-  const int ch = (int)std::min<int64_t>(chunk, 1 << 30);
-  const Pages& p = a.p;
-  if (is_f32(q) || !mfma_size(p.DK) || !mfma_size(p.DV)) {
-    TORCH_CHECK(p.DK <= 8192 && p.DV <= 4096, "head sizes");
-    launch_chunk_rows(q.data_ptr(), k.data_ptr(), v.data_ptr(), a.gate, a.ld,
-                      bt.data_ptr<int>(), row_seq.data_ptr<int>(),
-                      ctx.data_ptr<int>(), out.data_ptr(), a.M, a.H, p.G,
-                      p.DK, p.DV, bt.size(1), ch, (float)scale,
-                      (float)softcap, dist.data_ptr<float>(), is_f32(q),
-                      cur_stream());
-    return;
-  }
-  const long NS = key_splits(nsplit, a.M, a.H, p.G, ch, bt.size(1));
-  torch::Tensor pacc, pml;
-  void *pa = nullptr, *pm = nullptr;
-  if (NS > 1) {
-    auto f32 = q.options().dtype(at::kFloat);
-    pacc = torch::empty({(long)a.M * a.H * NS, p.DV}, f32);
-    pml = torch::empty({(long)a.M * a.H * NS, 2}, f32);
-    pa = pacc.data_ptr();
-    pm = pml.data_ptr();
-  }
-  launch_chunk_decode(q.data_ptr(), k.data_ptr(), v.data_ptr(), a.gate, a.ld,
-                      bt.data_ptr<int>(), row_seq.data_ptr<int>(),
-                      ctx.data_ptr<int>(), out.data_ptr(), pa, pm, a.M, a.H,
-                      p.G, p.DK, p.DV, (int)NS, bt.size(1), ch, (float)scale,
-                      (float)softcap, dist.data_ptr<float>(), cur_stream());
-}
-
-// portions [P, 4]: block-table row, first row, first position, rows;
-// blocks [N, 2]: portion, block of 128 queries
-void paged_attn_prompts(torch::Tensor q, torch::Tensor k, torch::Tensor v,
-                        torch::Tensor ab, int64_t gate_at, torch::Tensor out,
-                        torch::Tensor bt, torch::Tensor portions,
-                        torch::Tensor blocks, int64_t chunk, double scale,
-                        double softcap, torch::Tensor dist) {
-  const AttnArgs a = check_attn(q, k, v, ab, gate_at, out, chunk, softcap,
-                                dist);
-  CHECK_BF16(q);
-  CHECK_INTS(bt); CHECK_INTS(portions); CHECK_INTS(blocks);
-  TORCH_CHECK(bt.dim() == 2 && portions.dim() == 2 && portions.size(1) == 4 &&
-                  blocks.dim() == 2 && blocks.size(1) == 2,
-              "portion maps");
-  TORCH_CHECK(mfma_size(a.p.DK) && mfma_size(a.p.DV),
-              "head sizes must be 64, 128 or 256");
-  if (blocks.size(0) == 0) return;
-  launch_chunk_flash(q.data_ptr(), k.data_ptr(), v.data_ptr(), a.gate, a.ld,
-                     out.data_ptr(), bt.data_ptr<int>(), bt.size(1),
-                     portions.data_ptr<int>(), blocks.data_ptr<int>(),
-                     blocks.size(0), a.H, a.p.G, a.p.DK, a.p.DV,
-                     (int)std::min<int64_t>(chunk, 1 << 30), (float)scale,
-                     (float)softcap, dist.data_ptr<float>(), cur_stream());
 }
 
 struct SinkArgs {
@@ -558,8 +415,6 @@ void channel_delta(torch::Tensor ab, torch::Tensor ag, int64_t H, int64_t G,
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("attn_prep", &attn_prep);
-  m.def("paged_attn_rows", &paged_attn_rows);
-  m.def("paged_attn_prompts", &paged_attn_prompts);
   m.def("rotation_table", &rotation_table);
   m.def("rotary_prep", &rotary_prep);
   m.def("sink_attn_rows", &sink_attn_rows);

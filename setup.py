@@ -9,6 +9,7 @@ needs one group does not have to compile the others:
     _hip_residual  norms around an fp32 residual stream
     _hip_latent    latent attention
     _hip_hybrid    attention over pages of keys and values, delta rules
+    _hip_chunked   the same attention with capped scores, chunk by chunk
     _hip_experts   xIELU, routed experts
     _hip_lru       linear recurrent unit
     _hip_ops       everything else
@@ -34,9 +35,9 @@ GROUPS = {
                     "latent_decode.hip", "window_attention.hip"],
     "_hip_residual": ["ext_residual.cpp", "residual_norms.hip"],
     "_hip_hybrid": ["ext_hybrid.cpp", "chunk_attention.hip",
-                    "chunk_rows.hip", "chunk_flash.hip", "sink_rows.hip",
-                    "sink_flash.hip", "delta_rule.hip", "delta_chunk.hip",
-                    "delta_channel.hip"],
+                    "sink_rows.hip", "sink_flash.hip", "delta_rule.hip",
+                    "delta_chunk.hip", "delta_channel.hip"],
+    "_hip_chunked": ["ext_chunked.cpp", "chunk_rows.hip", "chunk_flash.hip"],
     "_hip_experts": ["ext_experts.cpp", "experts.hip", "expert_gemm16.hip",
                      "xielu.hip"],
     "_hip_lru": ["ext_lru.cpp", "lru.hip"],

@@ -457,7 +457,8 @@ def test_needed_extensions(case):
 
     need = needed_for(str(case.path))
     assert "_hip_lru" in need and "_hip_hybrid" in need
-    assert not {"_hip_ops", "_hip_latent", "_hip_experts"} & set(need)
+    assert not {"_hip_ops", "_hip_latent", "_hip_chunked",
+                "_hip_experts"} & set(need)
 
 
 def test_cli_generate_from_folder(tmp_path):

@@ -346,7 +346,8 @@ def _lru_inputs(blocks, bs, taps, M, slots, dtype, seed=0):
     (2, 32, 4, [1, 1, 1]), (3, 32, 4, [3, 150, 1, 2]), (1, 64, 1, [70, 5]),
     (2, 96, 2, [64, 65, 63]), (5, 64, 7, [33, 200]), (1, 256, 3, [40, 129]),
     (4, 256, 4, [66, 2, 17]), (16, 64, 4, [16, 17, 64, 31, 1, 400]),
-    (2, 160, 5, [1] * 40)])
+    (2, 160, 5, [1] * 40), (2, 384, 4, [70, 3]), (1, 320, 2, [65, 1]),
+    (1, 512, 4, [130, 16]), (3, 128, 4, [64, 40])])
 def test_gated_lru(device, dtype, blocks, bs, taps, rows):
     """Segments of one row to several chunks, from the start or going on,
     with padding rows behind; the sequence's slots and no others change."""
