@@ -19,7 +19,9 @@ NEEDED = {"Kanotar": ("_hip_gemm", "_hip_residual", "_hip_latent"),
           "Bufulorn": ("_hip_gemm", "_hip_residual", "_hip_hybrid",
                        "_hip_chunked", "_hip_experts"),
           "Tebasun": ("_hip_gemm", "_hip_residual", "_hip_hybrid",
-                      "_hip_lru")}
+                      "_hip_lru"),
+          "Kedelorn": ("_hip_gemm", "_hip_residual", "_hip_latent",
+                       "_hip_experts", "_hip_retention")}
 
 
 def needed_for(model_dir: str) -> tuple[str, ...]:

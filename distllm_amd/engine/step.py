@@ -60,7 +60,8 @@ class PromptBlocks:
 class Segments:
     """Rows of each block-table row, and its state slot. Segments of more
     than SHORT rows are also described in chunks of CHUNK rows, for
-    kernels that work chunk by chunk."""
+    kernels that work chunk by chunk, and in pieces for kernels that run
+    parts of a segment side by side."""
 
     row0: torch.Tensor       # [S] int32
     rows: torch.Tensor       # [S] int32
@@ -69,10 +70,12 @@ class Segments:
     longs: torch.Tensor | None = None   # [P, 2] segment, its first chunk
     chunks: torch.Tensor | None = None  # [N, 2] segment, chunk in it
     sizes: list[int] = field(default_factory=list)  # rows, on the host
-    _lists: dict[int, tuple] = field(default_factory=dict)
+    _lists: dict = field(default_factory=dict)
 
     SHORT = 16
     CHUNK = 32
+    PIECE = 256      # rows of a piece, at least
+    PIECE_WGS = 512
 
     @classmethod
     def build(cls, row0, rows, slots, device) -> "Segments":
@@ -98,6 +101,33 @@ class Segments:
                 torch.tensor(a, dtype=torch.int32).to(self.row0.device)
                 for a in (longs, chunks))
         return self._lists[size]
+
+    def pieces(self, heads: int) -> tuple:
+        """Long segments cut into pieces of about equal size that can run
+        side by side, as many as fill the GPU with a workgroup per piece
+        and head: (longs [L, 2]: segment, its first piece; pieces [P, 5]:
+        segment, first row, rows, number, pieces of the segment; whether
+        there are several of any). None, None, False without a long
+        segment."""
+        key = ("pieces", heads)
+        if key not in self._lists:
+            total = sum(n for n in self.sizes if n > self.SHORT)
+            most = max(self.PIECE, -(-total * heads // self.PIECE_WGS))
+            longs, pieces, several = [], [], False
+            for i, n in enumerate(self.sizes):
+                if n <= self.SHORT:
+                    continue
+                each = -(-n // -(-n // most))
+                each = -(-each // self.CHUNK) * self.CHUNK
+                count = -(-n // each)
+                longs.append((i, len(pieces)))
+                pieces += [(i, p * each, min(each, n - p * each), p, count)
+                           for p in range(count)]
+                several |= count > 1
+            self._lists[key] = (None, None, False) if not longs else (
+                *(torch.tensor(a, dtype=torch.int32).to(self.row0.device)
+                  for a in (longs, pieces)), several)
+        return self._lists[key]
 
 
 @dataclass

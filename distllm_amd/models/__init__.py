@@ -10,6 +10,7 @@ from .config import (PRESETS, LayeredDims, ModelDims, dims_from_checkpoint,
                      get_dims)
 from .esm import Esm2Encoder, EsmCEncoder
 from .kanotar import KanotarModel
+from .kedelorn import KedelornModel
 from .mistral import DecoderModel
 from .tebasun import TebasunModel
 
@@ -20,6 +21,7 @@ __all__ = [
     "Esm2Encoder",
     "EsmCEncoder",
     "KanotarModel",
+    "KedelornModel",
     "LayeredDims",
     "ModelDims",
     "PRESETS",
@@ -33,7 +35,7 @@ __all__ = [
 
 # decoders that are described layer by layer
 LAYERED = {"kanotar": KanotarModel, "bufulorn": BufulornModel,
-           "tebasun": TebasunModel}
+           "tebasun": TebasunModel, "kedelorn": KedelornModel}
 
 
 def build_model(name_or_dims: str | ModelDims | LayeredDims, device: str | None = None,

@@ -91,6 +91,11 @@ class Part(nn.Module):
         return {n: expect(pre + n, src[pre + n], *shape)
                 for n, shape in self.tensors().items()}
 
+    def initial(self) -> dict[str, torch.Tensor]:
+        """Checkpoint tensors whose values before training are not the
+        usual ones."""
+        return {}
+
     def cache_numel(self) -> int:
         """Numbers that a token keeps in the paged cache."""
         return 0

@@ -9,8 +9,8 @@ decoder family used for generation (K15):
   - Mistral-class decoder embedders (SFR-Embedding-Mistral)
   - Llama-class causal LMs for generation
   - Qwen2-class causal LMs (llama family + qkv bias)
-  - Kanotar, Bufulorn and Tebasun causal LMs: every layer has its own
-    description (LayeredDims)
+  - Kanotar, Bufulorn, Tebasun and Kedelorn causal LMs: every layer has
+    its own description (LayeredDims)
 Dims are from the public model cards; weights are random-init here
 (no network) or loadable from local safetensors.
 """
@@ -211,6 +211,59 @@ class ChannelDeltaDims(_Strict):
         return _check_groups(self)
 
 
+class RotaryLatentDims(_Strict):
+    """Causal attention on a cached latent of kv_rank numbers per token and
+    rot_dim rotated key numbers that all heads share; queries have `dim`
+    numbers for the keys made from the latent and rot_dim rotated ones. A
+    learned sink per head takes part in the softmax; head outputs are
+    multiplied by a gate each."""
+
+    type: Literal["rotary_latent"] = "rotary_latent"
+    heads: PositiveInt
+    dim: PositiveInt           # unrotated query/key size per head
+    rot_dim: PositiveInt       # rotated query/key size
+    vdim: PositiveInt          # value size per head
+    kv_rank: PositiveInt
+    rot: RotaryDims
+    scale: float
+    kv_from: NonNegativeInt | None = None  # layer whose cache this one reads
+
+    @model_validator(mode="after")
+    def _check_sizes(self):
+        if self.rot.dims != self.rot_dim:
+            raise ValueError(f"{self.rot.dims} rotated numbers, but rot_dim "
+                             f"{self.rot_dim}")
+        return self
+
+    def shared_sizes(self) -> dict:
+        return {"kv_rank": self.kv_rank, "rot_dim": self.rot_dim,
+                "rot": self.rot}
+
+
+class RetentionDims(_Strict):
+    """Linear attention with a fixed decay per head: a recurrent [dim,
+    vdim] state, rotated queries and keys."""
+
+    type: Literal["retention"] = "retention"
+    heads: PositiveInt
+    dim: PositiveInt
+    vdim: PositiveInt
+    rot: RotaryDims
+    decay: list[float]
+
+    @model_validator(mode="after")
+    def _check_sizes(self):
+        if len(self.decay) != self.heads:
+            raise ValueError(f"{len(self.decay)} decays for {self.heads} "
+                             "heads")
+        if not all(0.0 < x <= 1.0 for x in self.decay):
+            raise ValueError("decays must be above 0 and at most 1")
+        if self.rot.dims > self.dim:
+            raise ValueError(f"{self.rot.dims} rotated numbers in heads of "
+                             f"{self.dim}")
+        return self
+
+
 class ParallelDims(_Strict):
     """Two mixers side by side on the same input:
     left_scale * left + right_scale * right."""
@@ -293,10 +346,31 @@ class ExpertsDims(_Strict):
         return self
 
 
+class GatedExpertsDims(_Strict):
+    """Routed squared-ReLU experts. The `top` experts with the largest
+    sigmoid scores plus corrections serve a token, weighted by `scale`
+    times their scores without them. A shared expert of `shared` columns,
+    where there is one, serves every token through a gate of its own."""
+
+    kind: Literal["gated_experts"] = "gated_experts"
+    ff: PositiveInt
+    experts: PositiveInt
+    top: PositiveInt
+    scale: float = 1.0
+    shared: PositiveInt | None = None
+
+    @model_validator(mode="after")
+    def _check_top(self):
+        if self.top > self.experts:
+            raise ValueError(f"top {self.top} of {self.experts} experts")
+        return self
+
+
 class LayerDims(_Strict):
     mixer: (LatentAttentionDims | AttentionDims | DeltaDims | ParallelDims
-            | LruDims)
-    mlp: ClampedGluDims | SwigluDims | XieluDims | ExpertsDims | None = None
+            | LruDims | RotaryLatentDims | RetentionDims)
+    mlp: (ClampedGluDims | SwigluDims | XieluDims | ExpertsDims
+          | GatedExpertsDims | None) = None
 
 
 class LoopDims(_Strict):
@@ -311,7 +385,7 @@ class LoopDims(_Strict):
 class LayeredDims(BaseModel):
     """A decoder whose layers are described one by one."""
 
-    arch: Literal["kanotar", "bufulorn", "tebasun"]
+    arch: Literal["kanotar", "bufulorn", "tebasun", "kedelorn"]
     vocab_size: PositiveInt
     hidden_size: PositiveInt
     layers: list[LayerDims]
@@ -320,6 +394,7 @@ class LayeredDims(BaseModel):
     embed_scale: float = 1.0
     loop: LoopDims | None = None
     side_dim: PositiveInt | None = None  # per-layer token inputs
+    streams: PositiveInt | None = None   # copies of the residual stream
     # bounded only by a position table, where the design has one
     max_position_embeddings: PositiveInt = 1 << 20
 
@@ -473,10 +548,47 @@ def _tebasun_dims(cfg: dict, shapes=None) -> LayeredDims:
                        side_dim=None if side is None else side["dim"])
 
 
+def _kedelorn_mlp(mlp: dict, where: str) -> GatedExpertsDims:
+    mlp = dict(mlp)
+    kind = mlp.pop("kind", None)
+    if kind != "moe":
+        raise ValueError(f"{where}: unknown feed-forward kind {kind!r}")
+    shared = mlp.pop("shared", None)
+    if shared is not None:
+        shared = _take(shared, "ff", f"{where}: shared")
+    router = dict(mlp.pop("router"))
+    dims = GatedExpertsDims(
+        ff=_take(mlp.pop("expert"), "ff", f"{where}: expert"), shared=shared,
+        experts=router.pop("experts"), top=router.pop("top"),
+        scale=router.pop("scale"))
+    if mlp or router:
+        raise ValueError(f"{where}: unknown feed-forward keys "
+                         f"{sorted({**mlp, **router})}")
+    return dims
+
+
+def _kedelorn_dims(cfg: dict, shapes=None) -> LayeredDims:
+    layers = []
+    for i, entry in enumerate(cfg["layers"]):
+        if entry["type"] == "retention":
+            mixer = RetentionDims(**entry["mixer"])
+        elif entry["type"] == "latent_attention":
+            mixer = RotaryLatentDims(**entry["mixer"])
+        else:
+            raise ValueError(f"layer {i}: unknown mixer {entry['type']!r}")
+        mlp = entry.get("mlp")
+        layers.append(LayerDims(
+            mixer=mixer,
+            mlp=None if mlp is None else _kedelorn_mlp(mlp, f"layer {i}")))
+    return LayeredDims(arch="kedelorn", vocab_size=cfg["vocab"],
+                       hidden_size=cfg["width"], layers=layers,
+                       norm_eps=cfg["norm"]["eps"], streams=cfg["streams"])
+
+
 # config.json "architecture" -> reader of the rest of the file; `shapes`
 # returns the checkpoint's tensor shapes
 CONFIG_READERS = {"Kanotar": _kanotar_dims, "Bufulorn": _bufulorn_dims,
-                  "Tebasun": _tebasun_dims}
+                  "Tebasun": _tebasun_dims, "Kedelorn": _kedelorn_dims}
 
 
 def checkpoint_shapes(path: str | Path) -> dict[str, tuple[int, ...]]:
@@ -585,6 +697,36 @@ def looped_preset(num_layers: int, hidden: int, vocab: int, heads: int,
                        layers=layers, norm_eps=eps,
                        embed_scale=hidden ** 0.5, side_dim=side,
                        loop=LoopDims(start=lp[0], stop=lp[1], times=lp[2]))
+
+
+def streamed_preset(num_layers: int, hidden: int, vocab: int, heads: int,
+                    dim: int, kv_rank: int, mlp: GatedExpertsDims | None,
+                    order: str = "RL", rot_dim: int = 64,
+                    vdim: int | None = None, streams: int = 4,
+                    share: bool = False, original: int = 4096,
+                    eps: float = 1e-5) -> LayeredDims:
+    """Kedelorn dims of repeated layers: mixers follow `order` (R
+    retention, L latent attention). With `share`, every other attention
+    layer reads the latents of the one before."""
+    layers, owner = [], None
+    for i in range(num_layers):
+        if order[i % len(order)] == "R":
+            mixer = RetentionDims(
+                heads=heads, dim=dim, vdim=vdim or dim,
+                rot=RotaryDims(base=1e6, dims=dim),
+                decay=[1 - 2.0 ** (-5 - 5 * h / heads)
+                       for h in range(heads)])
+        else:
+            mixer = RotaryLatentDims(
+                heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim or dim,
+                kv_rank=kv_rank, scale=(dim + rot_dim) ** -0.5,
+                rot=RotaryDims(base=10000.0, dims=rot_dim, scaling=YarnDims(
+                    factor=4.0, original=original, fast=32.0, slow=1.0)),
+                kv_from=owner if share else None)
+            owner = i if owner is None else None
+        layers.append(LayerDims(mixer=mixer, mlp=mlp))
+    return LayeredDims(arch="kedelorn", vocab_size=vocab, hidden_size=hidden,
+                       layers=layers, norm_eps=eps, streams=streams)
 
 
 PRESETS: dict[str, ModelDims | LayeredDims] = {
@@ -702,6 +844,18 @@ PRESETS: dict[str, ModelDims | LayeredDims] = {
     "tebasun-tiny": looped_preset(
         4, 256, 1024, heads=8, kv_heads=4, dim=32, ff=512, order="PR",
         blocks=4, rank=16, side=32, loop=(1, 3, 2), original=64,
+    ),
+    # retention and latent attention of the llama3-8b size on four
+    # streams, every feed-forward routed
+    "kedelorn-8b": streamed_preset(
+        32, 4096, 128256, heads=32, dim=128, kv_rank=512,
+        mlp=GatedExpertsDims(ff=1792, experts=32, top=4, scale=2.0,
+                             shared=3584), order="RRLL", share=True,
+    ),
+    "kedelorn-tiny": streamed_preset(
+        4, 256, 1024, heads=4, dim=32, kv_rank=64,
+        mlp=GatedExpertsDims(ff=64, experts=6, top=2, shared=128),
+        order="RLL", rot_dim=16, share=True, streams=2, original=64,
     ),
 }
 

@@ -1,4 +1,5 @@
-"""Feed-forwards: SwiGLU, xIELU and routed gated-unit experts."""
+"""Feed-forwards: SwiGLU, xIELU, routed gated-unit and squared-ReLU
+experts."""
 
 from __future__ import annotations
 
@@ -6,8 +7,8 @@ import torch
 from torch import nn
 
 from .. import ops
-from .blocks import Part, pad64, padded, weight
-from .config import ExpertsDims, SwigluDims, XieluDims
+from .blocks import Part, norm_weight, pad64, padded, weight
+from .config import ExpertsDims, GatedExpertsDims, SwigluDims, XieluDims
 
 
 class SwigluMlp(Part):
@@ -109,3 +110,66 @@ class RoutedExperts(Part):
         ids, weights = ops.route(h, self.router, ctx, d.top, d.groups,
                                  d.keep)
         return ops.experts(h, ids, self.wgup, self.wdown), weights
+
+
+class GatedExperts(Part):
+    """Squared-ReLU experts chosen by corrected sigmoid scores, beside a
+    shared one with a gate per token (GatedExpertsDims). The shared
+    expert's gate is a row behind the router's and its weight one behind
+    those of the chosen experts."""
+
+    def __init__(self, d: GatedExpertsDims, width: int, dtype):
+        super().__init__()
+        self.d, self.width = d, width
+        self.wp, self.fp = pad64(width), pad64(d.ff)
+        n = d.experts
+        self.router = weight(n + (d.shared is not None), self.wp, dtype)
+        self.correction = norm_weight(n)
+        self.wup = nn.Parameter(torch.empty(n, self.fp, self.wp,
+                                            dtype=dtype))
+        self.wdown = nn.Parameter(torch.empty(n, self.wp, self.fp,
+                                              dtype=dtype))
+        if d.shared is not None:
+            self.sp = pad64(d.shared)
+            self.shared_up = weight(self.sp, self.wp, dtype)
+            self.shared_down = weight(self.wp, self.sp, dtype)
+
+    def tensors(self):
+        d, W = self.d, self.width
+        t = {}
+        for e in range(d.experts):
+            t |= {f"e{e}.up": (d.ff, W), f"e{e}.down": (W, d.ff)}
+        t |= {"router": (d.experts, W), "correction": (d.experts,)}
+        if d.shared is not None:
+            t |= {"shared.up": (d.shared, W), "shared.down": (W, d.shared),
+                  "shared.sg": (1, W)}
+        return t
+
+    def checkpoint(self, src, pre):
+        t, n = self.checked(src, pre), self.d.experts
+        router, out = t["router"], {}
+        if self.d.shared is not None:
+            router = torch.cat([router, t["shared.sg"]])
+            out = {"shared_up": padded(t["shared.up"], self.sp, self.wp),
+                   "shared_down": padded(t["shared.down"], self.wp, self.sp)}
+        return out | {
+            "router": padded(router, *self.router.shape),
+            "correction": t["correction"],
+            "wup": torch.stack([padded(t[f"e{e}.up"], self.fp, self.wp)
+                                for e in range(n)]),
+            "wdown": torch.stack([padded(t[f"e{e}.down"], self.wp, self.fp)
+                                  for e in range(n)])}
+
+    def forward(self, h, ctx):
+        """-> outputs [rows * top, width] of the chosen experts, row by
+        row, the shared expert's [rows, width] or None, and the weights of
+        both [rows, top (+ 1)]; rows with ctx 0 have none."""
+        d = self.d
+        ids, weights = ops.route_sigmoid(h, self.router, self.correction,
+                                         ctx, d.top, d.scale)
+        y = ops.experts(h, ids, self.wup, self.wdown, gated=False)
+        shared = None
+        if d.shared is not None:
+            shared = ops.linear(ops.up_relu2(h, self.shared_up),
+                                self.shared_down)
+        return y, shared, weights

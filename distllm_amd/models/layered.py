@@ -20,18 +20,24 @@ from .blocks import (ClampedGlu, LatentAttention, expect, norm_weight, pad64,
                      padded, weight)
 from .branches import parallel_mixer
 from .config import (AttentionDims, ClampedGluDims, DeltaDims, ExpertsDims,
-                     LatentAttentionDims, LayeredDims, LruDims, ParallelDims,
+                     GatedExpertsDims, LatentAttentionDims, LayeredDims,
+                     LruDims, ParallelDims, RetentionDims, RotaryLatentDims,
                      SwigluDims, XieluDims)
 from .delta import GatedDelta
-from .feedforward import RoutedExperts, SwigluMlp, XieluMlp
+from .feedforward import GatedExperts, RoutedExperts, SwigluMlp, XieluMlp
+from .latent import RotaryLatentAttention
 from .recurrent import GatedLru
+from .retention import Retention
 from .side import SideInput
+from .streams import StreamMix
 
 MIXERS = {LatentAttentionDims: LatentAttention,
           AttentionDims: PagedAttention, DeltaDims: GatedDelta,
-          ParallelDims: parallel_mixer, LruDims: GatedLru}
+          ParallelDims: parallel_mixer, LruDims: GatedLru,
+          RotaryLatentDims: RotaryLatentAttention, RetentionDims: Retention}
 MLPS = {ClampedGluDims: ClampedGlu, SwigluDims: SwigluMlp,
-        XieluDims: XieluMlp, ExpertsDims: RoutedExperts}
+        XieluDims: XieluMlp, ExpertsDims: RoutedExperts,
+        GatedExpertsDims: GatedExperts}
 
 
 class LayeredCache:
@@ -53,7 +59,7 @@ class LayeredCache:
 class Layer(nn.Module):
     def __init__(self, d, width: int, eps: float, dtype,
                  norms: tuple[str, ...], mlp_norms: tuple[str, ...],
-                 side: int | None = None):
+                 side: int | None = None, streams: int | None = None):
         super().__init__()
         wp = pad64(width)
         self.mixer = MIXERS[type(d.mixer)](d.mixer, width, eps, dtype)
@@ -62,6 +68,11 @@ class Layer(nn.Module):
             self.mlp = MLPS[type(d.mlp)](d.mlp, width, dtype)
         self.side = (SideInput(side, width, dtype) if side is not None
                      else None)
+        # how either sublayer sits between several residual streams
+        self.hc1 = self.hc2 = None
+        if streams is not None:
+            self.hc1 = StreamMix(streams)
+            self.hc2 = StreamMix(streams) if self.mlp is not None else None
         self.norm_names = norms + (mlp_norms if self.mlp is not None else ())
         for n in norms + mlp_norms:
             present = n in self.norm_names
@@ -72,7 +83,8 @@ class Layer(nn.Module):
         """(parameter prefix, checkpoint prefix, part)"""
         return [(a, b, m) for a, b, m in
                 (("mixer.", "mix.", self.mixer), ("mlp.", "mlp.", self.mlp),
-                 ("side.", "side.", self.side)) if m is not None]
+                 ("side.", "side.", self.side), ("hc1.", "hc1.", self.hc1),
+                 ("hc2.", "hc2.", self.hc2)) if m is not None]
 
 
 def norm_size(name: str, wp: int) -> int:
@@ -93,6 +105,7 @@ class LayeredModel(nn.Module):
     final_norms: tuple[str, ...] = ("final.norm",)
     has_positions = False  # a table of position vectors
     tied_head = False      # the output product uses the embedding table
+    norm_offset = 0.0      # what is added to stored norm weights
 
     def __init__(self, dims: LayeredDims, dtype=torch.bfloat16,
                  tp_group=None):
@@ -111,7 +124,8 @@ class LayeredModel(nn.Module):
                         if self.has_positions else None)
         self.layers = nn.ModuleList(
             Layer(d, W, dims.norm_eps, dtype, self.layer_norms,
-                  self.mlp_norms, dims.side_dim) for d in dims.layers)
+                  self.mlp_norms, dims.side_dim, dims.streams)
+            for d in dims.layers)
         for n in self.final_norms:
             setattr(self, n.replace(".", "_"),
                     norm_weight(norm_size(n, wp)))
@@ -177,6 +191,8 @@ class LayeredModel(nn.Module):
         w = expect(name, w, *self._norm_shape(name))
         if w.dim() == 0:
             return w.reshape(1)
+        if self.norm_offset:
+            w = w.float() + self.norm_offset
         return padded(w, self.tok_emb.shape[1])
 
     def _layer_tensors(self, src: dict, i: int) -> dict[str, torch.Tensor]:
@@ -201,10 +217,12 @@ class LayeredModel(nn.Module):
         layer by layer, so that a large model is not held twice."""
         own = dict(self.named_parameters())
 
-        def fill(shapes, to_own):
+        def fill(shapes, to_own, initial={}):
             src = {}
             for n, s in shapes.items():
-                if n.endswith(".b") and len(s) == 1:
+                if n in initial:
+                    src[n] = initial[n].to(self.device)
+                elif n.endswith(".b") and len(s) == 1:
                     src[n] = torch.zeros(s, device=self.device)
                 elif len(s) <= 1:
                     src[n] = torch.ones(s, device=self.device)
@@ -214,10 +232,22 @@ class LayeredModel(nn.Module):
             for k, v in to_own(src).items():
                 own[k].copy_(v.to(own[k].dtype))
 
+        def unit_norms(pre, names):
+            if not self.norm_offset:
+                return {}
+            return {pre + n: torch.full(self._norm_shape(n),
+                                        1.0 - self.norm_offset)
+                    for n in names}
+
         for i in range(len(self.layers)):
+            initial = {f"l{i}.{pre}{n}": v
+                       for _, pre, part in self.layers[i].parts()
+                       for n, v in part.initial().items()}
+            initial |= unit_norms(f"l{i}.", self.layers[i].norm_names)
             fill(self._layer_shapes(i), lambda src: self._layer_tensors(
-                src, i))
-        fill(self._end_shapes(), self._end_tensors)
+                src, i), initial)
+        fill(self._end_shapes(), self._end_tensors,
+             unit_norms("", self.final_norms))
 
     # ---- cache ----------------------------------------------------------
     def cache_bytes_per_block(self, blk: int, kv_cache_dtype: str) -> int:

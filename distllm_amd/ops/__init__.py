@@ -560,21 +560,46 @@ def latent_prep(ab, q_cols, q_rank, rank, wq, wc, eps, cache, block_table,
                                  cache, block_table, row_seq, ctx)
 
 
-def latent_gather(cache, block_table, key_seq, key_pos):
-    """Cached latents of (sequence, position) pairs, packed."""
+def rotary_latent_prep(ab, heads, dp, tp, rank, wc, eps, table, cache,
+                       block_table, row_seq, ctx, ql):
+    """What precedes latent attention with rotated parts, on a projection
+    ab [M, heads * (dp unrotated, tp rotated numbers) | latent | key part |
+    ...], in one launch: the rotated numbers of the queries of the first
+    len(ql) rows go to the last tp columns of ql [n, heads, latent + tp],
+    those of the others back to ab; normed latents (statistics over rank
+    numbers) and rotated key parts go to their cache rows (position ctx - 1;
+    ctx 0 writes nothing). cache None: the layer has none of its own."""
+    if ab.is_cuda:
+        _require_hip("_hip_latent")
+        _hip_ops.rotary_latent_prep(ab, heads, dp, tp, rank, wc, eps, table,
+                                    cache, block_table, row_seq, ctx, ql)
+        return
+    torch_ref.rotary_latent_prep(ab, heads, dp, tp, rank, wc, eps, table,
+                                 cache, block_table, row_seq, ctx, ql)
+
+
+def latent_gather(cache, block_table, key_seq, key_pos, rank=None):
+    """Cached latents of (sequence, position) pairs, packed. With rank
+    (fewer columns than a cache row has): the first rank columns and the
+    others, as two tensors."""
     if cache.is_cuda:
         _require_hip("_hip_latent")
-        return _hip_ops.latent_gather(cache, block_table, key_seq, key_pos)
-    return torch_ref.latent_gather(cache, block_table, key_seq, key_pos)
+        c, rest = _hip_ops.latent_gather(cache, block_table, key_seq,
+                                         key_pos, rank or cache.shape[2])
+        return c if rank is None else (c, rest)
+    c = torch_ref.latent_gather(cache, block_table, key_seq, key_pos)
+    return c if rank is None else (c[:, :rank].contiguous(),
+                                   c[:, rank:].contiguous())
 
 
 def head_gemm(x, w, out=None):
-    """One product per head: x [M, H, K], w [H, N, K] -> [M, H, N]."""
+    """One product per head: x [M, H, K], w [H, N, K] -> [M, H, N]. Rows
+    and heads of x and out may be strided."""
     if x.is_cuda and x.dtype == torch.bfloat16:
         _require_hip("_hip_latent")
         if out is None:
             out = x.new_empty(x.shape[0], x.shape[1], w.shape[1])
-        _hip_ops.head_gemm(x.contiguous(), w, out)
+        _hip_ops.head_gemm(x, w, out)
         return out
     if x.is_cuda:  # true 32-bit product
         res = torch.bmm(x.transpose(0, 1), w.transpose(1, 2))
@@ -587,31 +612,38 @@ def head_gemm(x, w, out=None):
 
 
 def latent_attn(q, cache, block_table, row_seq, ctx, window, scale,
-                nsplit=0):
+                nsplit=0, rank=None, sink=None, gate=None):
     """Attention of single-token rows over paged latents, queries folded
     into the latent space: q [M, H, R] -> [M, H, R]. A row sees the last
     `window` positions of its sequence up to its own (ctx - 1). nsplit:
-    workgroups that share a row's keys (0: chosen from the sizes)."""
+    workgroups that share a row's keys (0: chosen from the sizes). With
+    rank, only the first rank columns of a cache row are the value. sink
+    [H]: exp(sink) is part of the softmax's denominator; gate [M, H]: head
+    outputs are multiplied by its sigmoid."""
+    rank = rank or cache.shape[2]
     if q.is_cuda:
         _require_hip("_hip_latent")
         return _hip_ops.latent_attn(q, cache, block_table, row_seq, ctx,
-                                    window, scale, nsplit)
+                                    window, scale, nsplit, rank, sink, gate)
     return torch_ref.latent_attn(q, cache, block_table, row_seq, ctx,
-                                 window, scale)
+                                 window, scale, rank, sink, gate)
 
 
-def attn_window(q, kv, out, cu_q, cu_k, block_map, window, scale):
+def attn_window(q, kv, out, cu_q, cu_k, block_map, window, scale, kr=None,
+                sink=None, gate=None):
     """Sliding-window causal attention of packed queries that are the
     last ones of their packed keys (a prompt portion after its cached
-    part). q [Tq, H, DK], kv [Tk, H*DK + H*DV], out [Tq, H, DV]."""
+    part). q [Tq, H, DK], kv [Tk, H*DK + H*DV], out [Tq, H, DV]. With kr
+    [Tk, DR], key numbers that all heads share, queries have DK + DR
+    numbers. sink, gate: as for latent_attn."""
     if q.is_cuda:
         _require_hip("_hip_latent")
         blk_seq, blk_qb = block_map
         _hip_ops.attn_window(q, kv, out, cu_q, cu_k, blk_seq, blk_qb,
-                             window, scale)
+                             window, scale, kr, sink, gate)
         return out
     return out.copy_(torch_ref.attn_window(q, kv, out.shape[2], cu_q, cu_k,
-                                           window, scale))
+                                           window, scale, kr, sink, gate))
 
 
 # ---- chunked attention / delta rule / experts decoder -----------------------
@@ -732,14 +764,45 @@ def route(h, router, ctx, top, groups, keep):
     return torch_ref.route(h, router, ctx, top, groups, keep)
 
 
-def experts(h, ids, wgup, wdown):
-    """Gated-unit experts: row m * top + k of the result is expert
-    ids[m, k] of row m (undefined for id -1). wgup [E, 2F, W]: gate and up
-    rows alternate in groups of 16."""
+def experts(h, ids, wup, wdown, gated=True):
+    """Experts: row m * top + k of the result is expert ids[m, k] of row m
+    (undefined for id -1). Gated units, wup [E, 2F, W]: gate and up rows
+    alternate in groups of 16; else squared ReLU, wup [E, F, W]."""
     if h.is_cuda:
         _require_hip("_hip_experts")
-        return _hip_ops.experts(h, ids, wgup, wdown)
-    return torch_ref.experts(h, ids, wgup, wdown)
+        return _hip_ops.experts(h, ids, wup, wdown, gated)
+    return torch_ref.experts(h, ids, wup, wdown, gated)
+
+
+def route_sigmoid(h, router, correction, ctx, top, scale):
+    """Experts of every row by sigmoid scores: ids [M, top] int32 of the
+    largest sums of score and correction, and scale times their scores
+    without it. Rows of the router behind the experts (one per correction)
+    are gates of their own: their sigmoids are further columns of the
+    weights. Rows with ctx 0 get ids -1 and weights 0."""
+    if h.is_cuda:
+        _require_hip("_hip_experts")
+        if h.dtype == torch.bfloat16 and router.shape[0] <= 256:
+            return _hip_ops.route_sigmoid(h, router, correction, ctx, top,
+                                          scale)
+        logits = torch.nn.functional.linear(h.float(), router.float())
+        return _hip_ops.route_sigmoid(logits, None, correction, ctx, top,
+                                      scale)
+    return torch_ref.route_sigmoid(h, router, correction, ctx, top, scale)
+
+
+def up_relu2(x, wup):
+    """The square of relu(x @ wup^T)."""
+    M, K = x.shape
+    if x.is_cuda:
+        _require_hip("_hip_gemm")
+        if (M <= 256 and x.dtype == torch.bfloat16 and K % 64 == 0
+                and wup.shape[0] % 64 == 0):
+            sk = _decode_splitk(M, wup.shape[0], K)
+            if sk > 1:
+                return _hip_ops.decode_gemm(x, wup, None, sk, 5)
+        return _hip_ops.relu2(linear(x, wup))
+    return torch_ref.relu2(linear(x, wup))
 
 
 # ---- parallel attention and delta rule / linear recurrent decoder -----------
@@ -885,3 +948,46 @@ def gated_lru(ab, conv_w, conv_b, gates, gates_b, decay, state, conv,
             row_seq, ctx, longs, chunks, chunk, segments.SHORT)
     return torch_ref.gated_lru(ab, conv_w, conv_b, gates, gates_b, decay,
                                state, conv, segments, row_seq, ctx)
+
+
+# ---- retention / rotary latent attention decoder on several streams ---------
+
+def stream_step(x, y=None, writes=None, mix=None, shared=None, embed=None,
+                read=None, norm=None, store=True, dtype=None):
+    """One boundary of fp32 residual streams x [M, S, W], in place. With a
+    sublayer's output y [M, W] and writes = (out [S], then the matrix mix,
+    from-major), x_t becomes sum_s mix[s, t] x_s + out[t] y. With mix
+    [M, top] (+ 1 column with shared [M, W]), y [M * top, W] is summed with
+    these weights first. With embed = (tokens, table) every old stream is
+    the token's row and x is not read; without `store` x is not written.
+    Returns rms(sum_s read[s] x_s) * w (read None: the plain sum) with norm
+    = (w, n, eps), statistics over n columns, in `dtype` (default: y's)."""
+    w, n, eps = norm
+    if dtype is None:
+        dtype = y.dtype
+    if x.is_cuda:
+        _require_hip("_hip_residual")
+        tokens, table = embed if embed is not None else (None, None)
+        h = torch.empty(x.shape[0], x.shape[2], dtype=dtype, device=x.device)
+        _hip_ops.stream_step(x, y, writes, mix, shared, tokens, table, read,
+                             w, n, eps, store, h)
+        return h
+    return torch_ref.stream_step(x, y, writes, mix, shared, embed, read,
+                                 norm, store, dtype)
+
+
+def retention(ab, heads, dp, vp, dim, vdim, decay, table, eps, state,
+              segments, ctx):
+    """Linear attention with a fixed decay per head (decay [2, heads]: the
+    decays, their base-2 logarithms) of a ragged step, on the projection
+    ab [M, queries | keys | values | gates]: rotation by table, recurrence
+    in fp32, heads normed over vdim and gated by silu. -> [M, heads * vp];
+    the sequences' slots of state [slots, heads, vp, dp] are updated."""
+    if ab.is_cuda:
+        _require_hip("_hip_retention")
+        return _hip_ops.retention(
+            ab, heads, dp, vp, dim, vdim, decay, table, eps, state,
+            segments.row0, segments.rows, segments.slot, ctx,
+            *segments.pieces(heads), segments.SHORT)
+    return torch_ref.retention(ab, heads, dp, vp, dim, vdim, decay, table,
+                               eps, state, segments, ctx)

@@ -36,7 +36,6 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 #define QWAVE 32
 #define LOG2E 1.4426950408889634f
 #define VROW 68   // padded V^T row length in bf16 elems (136 B)
-#define VROW4 72  // the same for 4-key units (144 B: aligned 16-byte reads)
 
 extern __shared__ __attribute__((aligned(16))) char smem[];
 
@@ -57,9 +56,14 @@ union frag_u {
 // latest keys up to its own position. Keys and values may have different
 // head sizes (DV) and interleave in one row (tstr_k counts both). V is
 // staged in units of 4 keys x 8 columns, transposed in registers, so that
-// the V^T image is written 8 bytes at a time.
+// the V^T image is written 8 bytes at a time; its 16-byte pieces are swizzled
+// by the row, for both the writes and the reads.
+// With ROT, queries have ROT more numbers per head, against ROT numbers of
+// each key that all heads share (Kr [Tk, ROT]). sink (a number per head, part
+// of the softmax's denominator) and gate (sigmoid of a number per query and
+// head on the output) may be null.
 template <int D, bool CAUSAL, bool HAS_MASK, bool VDIRECT,
-          bool VARLEN = false, int DV = D, bool WINDOW = false>
+          bool VARLEN = false, int DV = D, bool WINDOW = false, int ROT = 0>
 __global__ void __launch_bounds__(256, WINDOW && D + DV <= 256 ? 2 : 1)
 attn_fwd_kernel(const unsigned short* __restrict__ Q,
                 const unsigned short* __restrict__ Kt,
@@ -71,7 +75,11 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
                 const int* __restrict__ cu = nullptr,
                 const int* __restrict__ blk_seq = nullptr,
                 const int* __restrict__ blk_qb = nullptr,
-                const int* __restrict__ cu_k = nullptr, int window = 0) {
+                const int* __restrict__ cu_k = nullptr, int window = 0,
+                const unsigned short* __restrict__ Kr = nullptr,
+                const float* __restrict__ sink = nullptr,
+                const unsigned short* __restrict__ gate = nullptr,
+                int ld_gate = 0) {
   constexpr int NWAVE = 4;  // waves per workgroup (8 measured slower)
   constexpr int NTHR = NWAVE * 64;
   constexpr int QBLK = NWAVE * QWAVE;       // q rows per workgroup
@@ -79,7 +87,8 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
   constexpr int NCHV = DV / 8;           // 16B chunks per V row
   constexpr int DBLK = DV / 32;          // 32-wide d blocks of V
   constexpr int KTILE_B = KVBLK * D * 2; // K tile bytes
-  constexpr int VR = WINDOW ? VROW4 : VROW; // V^T row length
+  constexpr int RTILE_B = KVBLK * ROT * 2; // shared key part of a tile
+  constexpr int VR = WINDOW ? KVBLK : VROW; // V^T row length
   constexpr int VTILE_B = DV * VR * 2;   // V^T tile bytes
   // V chunks per thread; 4-key units with WINDOW
   constexpr int VUNITS = KVBLK / 4 * NCHV;
@@ -136,7 +145,7 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
   const long kbase = WINDOW   ? (long)cu_k[b] * tstr_k
                      : VARLEN ? (long)cu[b] * tstr_k
                               : (long)b * bstr_k;
-  const unsigned short* Qb = Q + qbase + (long)head * D;
+  const unsigned short* Qb = Q + qbase + (long)head * (D + ROT);
   const unsigned short* Kb = Kt + kbase + (long)kvhead * D;
   const unsigned short* Vb = Vt + kbase + (long)kvhead * DV;
   unsigned short* Ob = O + (VARLEN ? (long)cu[b] : (long)b * SQ) * ostride +
@@ -149,16 +158,17 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
   const int qload = qrow_abs < SQ ? qrow_abs : (SQ > 0 ? SQ - 1 : 0);
 
   const int offK[2] = {0, KTILE_B};
-  const int offV[2] = {2 * KTILE_B, 2 * KTILE_B + VTILE_B};
+  constexpr int offR = 2 * KTILE_B;
+  const int offV[2] = {offR + 2 * RTILE_B, offR + 2 * RTILE_B + VTILE_B};
   const int offM[2] = {2 * KTILE_B + 2 * VTILE_B,
                        2 * KTILE_B + 2 * VTILE_B + KVBLK * 4};
 
   const float scale2 = scale * LOG2E;
 
   // ---- Q fragments in registers ---------------------------------------
-  bf16x8 qf[D / 16];
+  bf16x8 qf[(D + ROT) / 16];
 #pragma unroll
-  for (int s = 0; s < D / 16; ++s)
+  for (int s = 0; s < (D + ROT) / 16; ++s)
     qf[s] = *reinterpret_cast<const bf16x8*>(Qb + (long)qload * tstr_q +
                                              s * 16 + h * 8);
 
@@ -186,6 +196,20 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
       __builtin_amdgcn_global_load_lds(
           (const __attribute__((address_space(1))) unsigned int*)src, dst,
           16, 0, 0);
+    }
+    if constexpr (ROT > 0) {
+      static_assert(ROT == 64, "eight 16-byte pieces per row");
+      for (int p = wid; p < KVBLK / 8; p += NWAVE) {
+        const int row = p * 8 + (lane >> 3);
+        const int krow = min(k0 + row, SKV - 1);
+        const unsigned short* src =
+            Kr + (long)(cu_k[b] + krow) * ROT + ((lane & 7) ^ (row & 7)) * 8;
+        auto dst = (__attribute__((address_space(3))) unsigned int*)(
+            smem + offR + buf * RTILE_B + p * 1024 + lane * 16);
+        __builtin_amdgcn_global_load_lds(
+            (const __attribute__((address_space(1))) unsigned int*)src, dst,
+            16, 0, 0);
+      }
     }
   };
   // per-thread V staging geometry, hoisted out of the tile loop
@@ -241,7 +265,9 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
 #pragma unroll
           for (int j = 0; j < 4; ++j)
             k[j] = __builtin_bit_cast(i32x4, vreg[c * 4 + j]);
-          unsigned short* dst = vt + u % NCHV * 8 * VR + u / NCHV * 4;
+          const int d8 = u % NCHV, kq = u / NCHV;
+          unsigned short* dst = vt + d8 * 8 * VR + (kq & 1) * 4;
+          const int piece = (kq >> 1) ^ (d8 & 7);
 #pragma unroll
           for (int w = 0; w < 4; ++w) {
             i32x2 even, odd;
@@ -249,8 +275,10 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
             even[1] = __builtin_amdgcn_perm(k[3][w], k[2][w], 0x05040100);
             odd[0] = __builtin_amdgcn_perm(k[1][w], k[0][w], 0x07060302);
             odd[1] = __builtin_amdgcn_perm(k[3][w], k[2][w], 0x07060302);
-            *reinterpret_cast<i32x2*>(dst + w * 2 * VR) = even;
-            *reinterpret_cast<i32x2*>(dst + (w * 2 + 1) * VR) = odd;
+            *reinterpret_cast<i32x2*>(dst + w * 2 * VR +
+                                      (piece ^ (w * 2)) * 8) = even;
+            *reinterpret_cast<i32x2*>(dst + (w * 2 + 1) * VR +
+                                      (piece ^ (w * 2 + 1)) * 8) = odd;
           }
         }
       }
@@ -264,7 +292,7 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
     }
   };
   auto stage_m = [&](int k0, int buf) {
-    if (threadIdx.x < KVBLK) {
+    if (!WINDOW && threadIdx.x < KVBLK) {
       const int krow = k0 + threadIdx.x;
       float mv;
       if (krow >= SKV) mv = -INFINITY;
@@ -341,6 +369,15 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
               smem + offK[cur] + key * (2 * D) + swz * 16);
           accP = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
               kf, qf[s], accP, 0, 0, 0);
+        }
+#pragma unroll
+        for (int s = 0; s < ROT / 16; ++s) {
+          const int key = kb * 32 + (lane & 31);
+          bf16x8 kf = *reinterpret_cast<const bf16x8*>(
+              smem + offR + cur * RTILE_B + key * (2 * ROT) +
+              (((s * 2 + h) ^ (key & 7)) * 16));
+          accP = __builtin_amdgcn_mfma_f32_32x32x16_bf16(
+              kf, qf[D / 16 + s], accP, 0, 0, 0);
         }
         __builtin_amdgcn_s_setprio(0);
 #pragma unroll
@@ -421,6 +458,11 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
               vf[i] = *reinterpret_cast<const __bf16*>(
                   Vb + (long)key * tstr_k + d * 32 + (lane & 31));
             }
+          } else if (WINDOW) {
+            const int row = d * 32 + (lane & 31);
+            vf = *reinterpret_cast<const bf16x8*>(
+                vimg + row * VR +
+                ((kh * 2 + h) ^ ((row ^ (row >> 3)) & 7)) * 8);
           } else {
             vf = *reinterpret_cast<const bf16x8*>(
                 vimg + (d * 32 + (lane & 31)) * VR + kh * 16 + h * 8);
@@ -442,7 +484,14 @@ attn_fwd_kernel(const unsigned short* __restrict__ Q,
   }
 
   // ---- epilogue: O^T regs -> padded LDS -> coalesced bf16 stores ------
-  const float inv_l = (l > 0.f) ? 1.f / l : 0.f;
+  float inv_l = (l > 0.f) ? 1.f / l : 0.f;
+  if (WINDOW && sink != nullptr && l > 0.f) {
+    const float s = sink[head] * LOG2E, top = fmaxf(m, s);
+    const float a = __builtin_amdgcn_exp2f(m - top);
+    inv_l = a / (l * a + __builtin_amdgcn_exp2f(s - top));
+  }
+  if (WINDOW && gate != nullptr)
+    inv_l *= sigmoid_exact(bf2f(gate[(cu[b] + (long)qload) * ld_gate + head]));
   float* oimg = reinterpret_cast<float*>(smem) + wid * QWAVE * (DV + 1);
 #pragma unroll
   for (int d = 0; d < DBLK; ++d)

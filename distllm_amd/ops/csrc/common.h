@@ -165,6 +165,10 @@ __device__ __forceinline__ float xielu_exact(float z, float ap, float an) {
   const float neg = (0.5f + an) * (expm1f(fminf(z, 0.f)) - z);
   return 0.5f * z + (z > 0.f ? ap * z * z : neg);
 }
+__device__ __forceinline__ float relu2(float z) {
+  const float r = fmaxf(z, 0.f);
+  return r * r;
+}
 __device__ __forceinline__ float sigmoid_exact(float z) {
   return 1.f / (1.f + expf(-z));
 }

@@ -142,9 +142,9 @@ decode_gemm_kernel(const unsigned short* __restrict__ X,
     }
 }
 
-// reduce fp32 slabs [SPLITK, MP, N] -> bf16 [M, N] (+bias); XIELU: with
-// the activation of numbers act[0..1] applied
-template <bool XIELU>
+// reduce fp32 slabs [SPLITK, MP, N] -> bf16 [M, N] (+bias); ACT 3: with
+// xIELU of numbers act[0..1] applied, 5: with relu(.)^2
+template <int ACT>
 __global__ void __launch_bounds__(256)
 dg_reduce_kernel(const float* __restrict__ slabs,
                  const unsigned short* __restrict__ bias,
@@ -152,7 +152,7 @@ dg_reduce_kernel(const float* __restrict__ slabs,
                  int splitk, const float* __restrict__ act) {
   const long total = (long)M * N;
   float ap = 0.f, an = 0.f;
-  if (XIELU) {
+  if (ACT == 3) {
     ap = softplus_exact(act[0]);
     an = softplus_exact(act[1]);
   }
@@ -165,7 +165,7 @@ dg_reduce_kernel(const float* __restrict__ slabs,
     for (int s = 0; s < splitk; ++s)
       v += slabs[((long)s * MP + row) * N + col];
     if (bias != nullptr) v += bf2f(bias[col]);
-    out[i] = f2bf(XIELU ? xielu(v, ap, an) : v);
+    out[i] = f2bf(ACT == 3 ? xielu(v, ap, an) : ACT == 5 ? relu2(v) : v);
   }
 }
 
@@ -258,16 +258,16 @@ extern "C" void launch_decode_gemm(const void* X, const void* W,
       hipLaunchKernelGGL(dg_reduce_rows_kernel, dim3(blocks), dim3(256), 0,
                          stream, (const float*)slabs, (unsigned short*)out,
                          M, MP, N, splitk, *rows);
-    else if (act == 3)
-      hipLaunchKernelGGL(dg_reduce_kernel<true>, dim3(blocks), dim3(256), 0,
-                         stream, (const float*)slabs,
-                         (const unsigned short*)bias, (unsigned short*)out,
-                         M, MP, N, splitk, act_nums);
-    else
-      hipLaunchKernelGGL(dg_reduce_kernel<false>, dim3(blocks), dim3(256), 0,
-                         stream, (const float*)slabs,
-                         (const unsigned short*)bias, (unsigned short*)out,
-                         M, MP, N, splitk, act_nums);
+    else {
+#define DGE(A)                                                                 \
+  hipLaunchKernelGGL(dg_reduce_kernel<A>, dim3(blocks), dim3(256), 0, stream,  \
+                     (const float*)slabs, (const unsigned short*)bias,         \
+                     (unsigned short*)out, M, MP, N, splitk, act_nums)
+      if (act == 3) DGE(3);
+      else if (act == 5) DGE(5);
+      else DGE(0);
+#undef DGE
+    }
 #undef DGR
   }
 }

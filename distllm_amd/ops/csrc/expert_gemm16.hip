@@ -1,10 +1,10 @@
 // Grouped products of routed experts for many rows per expert (see
 // experts.hip for the plan): 256 x 256 x 64 tiles on the deep-pipelined
-// main loop of gemm16.hip, with gathered rows and silu(gate) * up, or
-// scattered rows. N % 256 == 0, K % 128 == 0.
+// main loop of gemm16.hip, with gathered rows and silu(gate) * up or
+// relu(up)^2, or scattered rows. N % 256 == 0, K % 128 == 0.
 #include "gemm16_core.h"
 
-template <bool GLU>
+template <int UNIT>
 __global__ void __launch_bounds__(512, 2)
 expert_gemm16_kernel(const unsigned short* __restrict__ x,
                      const unsigned short* __restrict__ W,
@@ -12,6 +12,7 @@ expert_gemm16_kernel(const unsigned short* __restrict__ x,
                      const int* __restrict__ perm,
                      const int* __restrict__ tiles,
                      const int* __restrict__ ntiles, int N, int K, int top) {
+  constexpr bool GLU = UNIT == 1, UP = UNIT != 0;
   const int ncol = N / G16_BN;
   // contiguous runs of (tile, column block) per XCD, columns fastest: they
   // share the rows of x
@@ -36,7 +37,7 @@ expert_gemm16_kernel(const unsigned short* __restrict__ x,
     for (int pp = 0; pp < 2; ++pp) {
       const int r = half * 128 + (wid * 2 + pp) * 8 + r_in;
       const int s = s0 + min(r, cnt - 1);
-      xs[half][pp] = x + (long)(GLU ? perm[s] / top : s) * K + c_src;
+      xs[half][pp] = x + (long)(UP ? perm[s] / top : s) * K + c_src;
     }
   const unsigned short* wb =
       W + ((long)e * N + n0 + wid * 16 + r_in) * K + c_src;
@@ -86,10 +87,14 @@ expert_gemm16_kernel(const unsigned short* __restrict__ x,
         const int r = p * 8 + (lane >> 3), c8 = lane & 7;
         float o[8];
 #pragma unroll
-        for (int i = 0; i < 8; ++i) o[i] = slab[r * SLAB_W + c8 * 8 + i];
-        if (row0 + r < cnt)
-          store8(out + (long)perm[s0 + row0 + r] * N + n0 + nw * 64 + c8 * 8,
-                 o);
+        for (int i = 0; i < 8; ++i) {
+          o[i] = slab[r * SLAB_W + c8 * 8 + i];
+          if (UNIT == 2) o[i] = relu2(o[i]);
+        }
+        if (row0 + r < cnt) {
+          const long row = UP ? s0 + row0 + r : perm[s0 + row0 + r];
+          store8(out + row * N + n0 + nw * 64 + c8 * 8, o);
+        }
       }
     }
     asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
@@ -103,7 +108,7 @@ extern "C" bool expert_gemm16_covers(int N, int K) {
 extern "C" void launch_expert_gemm16(const void* x, const void* W, void* out,
                                      const int* perm, const int* tiles,
                                      const int* ntiles, int max_tiles, int N,
-                                     int K, int top, bool glu,
+                                     int K, int top, int unit,
                                      hipStream_t stream) {
   typedef unsigned short u16;
   const long wgs = ((long)max_tiles * (N / G16_BN) + 7) / 8 * 8;
@@ -111,7 +116,8 @@ extern "C" void launch_expert_gemm16(const void* x, const void* W, void* out,
   hipLaunchKernelGGL((expert_gemm16_kernel<GL>), dim3(wgs), dim3(512),       \
                      G16_LDS, stream, (const u16*)x, (const u16*)W,          \
                      (u16*)out, perm, tiles, ntiles, N, K, top)
-  if (glu) EG(true);
-  else EG(false);
+  if (unit == 1) EG(1);
+  else if (unit == 2) EG(2);
+  else EG(0);
 #undef EG
 }

@@ -1,14 +1,15 @@
-// Routed gated-unit experts.
+// Routed experts, gated units or squared ReLU.
 //
 //   route:   softmax scores of a row over all experts, the best groups, the
 //            best experts in them                    -> ids, weights [M, top]
+//            or sigmoid scores, the best with a correction added
 //   plan:    (row, choice) pairs sorted by expert, cut into tiles of rows
 //   product: one grouped product per tile; the first one gathers the rows
-//            and applies silu(gate) * up, the second scatters its rows to
-//            row * top + choice
+//            and applies silu(gate) * up or relu(up)^2, the second scatters
+//            its rows to row * top + choice
 //
-// wgup [E, 2F, K]: gate and up rows alternate in groups of 16, so that a
-// tile of columns holds both halves of the unit. The number of tiles is
+// Gated units, [E, 2F, K]: gate and up rows alternate in groups of 16, so
+// that a tile of columns holds both halves of the unit. The number of tiles is
 // known on the device only: grids have the most there can be and surplus
 // workgroups leave at once.
 #include "common.h"
@@ -18,28 +19,55 @@ typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
 extern __shared__ __attribute__((aligned(16))) char smem[];
 
 // ---- routing ----------------------------------------------------------------
-// One wave chooses for one row. z [E]: logits, overwritten; gm, ok [groups].
-// A lane holds the scores of experts lane + 64 i, i < PER.
+// Softmax scores, or (correction not null) sigmoid scores whose sum with the
+// correction [E] makes the choice; weights are the scores times `scale`.
+// `gates` logits behind those of the experts are weights of their own, by
+// their sigmoids.
+struct RouteArgs {
+  int E, groups, keep, top;
+  const float* correction;
+  float scale;
+  int gates;
+
+  __host__ __device__ __forceinline__ int logits() const { return E + gates; }
+  __host__ __device__ __forceinline__ int cols() const { return top + gates; }
+};
+
+// One wave chooses for one row. z [E + gates]: logits, overwritten; gm, ok
+// [groups]. A lane holds the scores of experts lane + 64 i, i < PER.
 template <int PER>
-__device__ void select_row(float* z, float* gm, int* ok, int E, int groups,
-                           int keep, int top, int* __restrict__ ids,
-                           float* __restrict__ weights, int lane) {
-  float s[PER];
-  float mx = -INFINITY;
+__device__ void select_row(float* z, float* gm, int* ok, const RouteArgs& a,
+                           int* __restrict__ ids, float* __restrict__ weights,
+                           int lane) {
+  const int E = a.E, groups = a.groups;
+  float s[PER], w[PER];  // what is compared, what it weighs
+  float scale = a.scale;
+  if (a.correction != nullptr) {
 #pragma unroll
-  for (int i = 0; i < PER; ++i) {
-    const int e = lane + 64 * i;
-    s[i] = e < E ? z[e] : -INFINITY;
-    mx = fmaxf(mx, s[i]);
-  }
-  mx = wave_reduce_max(mx);
-  float sum = 0.f;
+    for (int i = 0; i < PER; ++i) {
+      const int e = lane + 64 * i;
+      w[i] = e < E ? sigmoid_exact(z[e]) : 0.f;
+      s[i] = e < E ? w[i] + a.correction[e] : 0.f;
+    }
+    for (int j = lane; j < a.gates; j += 64)
+      weights[a.top + j] = sigmoid_exact(z[E + j]);
+  } else {
+    float mx = -INFINITY;
 #pragma unroll
-  for (int i = 0; i < PER; ++i) {
-    s[i] = expf(s[i] - mx);
-    sum += s[i];
+    for (int i = 0; i < PER; ++i) {
+      const int e = lane + 64 * i;
+      s[i] = e < E ? z[e] : -INFINITY;
+      mx = fmaxf(mx, s[i]);
+    }
+    mx = wave_reduce_max(mx);
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      w[i] = s[i] = expf(s[i] - mx);
+      sum += s[i];
+    }
+    scale /= wave_reduce_sum(sum);
   }
-  sum = wave_reduce_sum(sum);
   if (groups > 1) {
 #pragma unroll
     for (int i = 0; i < PER; ++i)
@@ -47,7 +75,7 @@ __device__ void select_row(float* z, float* gm, int* ok, int E, int groups,
     wave_sync();
     const int per = E / groups;
     for (int c = lane; c < groups; c += 64) {
-      float b = -1.f;
+      float b = -INFINITY;
       for (int i = 0; i < per; ++i) b = fmaxf(b, z[c * per + i]);
       gm[c] = b;
     }
@@ -56,39 +84,41 @@ __device__ void select_row(float* z, float* gm, int* ok, int E, int groups,
       int rank = 0;
       for (int i = 0; i < groups; ++i)
         rank += gm[i] > gm[c] || (gm[i] == gm[c] && i < c);
-      ok[c] = rank < keep;
+      ok[c] = rank < a.keep;
     }
     wave_sync();
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
       const int e = lane + 64 * i;
-      if (e < E && !ok[e / per]) s[i] = -1.f;
+      if (e < E && !ok[e / per]) s[i] = -INFINITY;
     }
   }
 #pragma unroll
   for (int i = 0; i < PER; ++i)
-    if (lane + 64 * i >= E) s[i] = -2.f;
-  float own = -3.f;  // the lane's best, and which it is
+    if (lane + 64 * i >= E) s[i] = -INFINITY;
+  float own = -INFINITY, weight = 0.f;  // the lane's best, and which it is
   int at = 0;
   auto best = [&]() {
-    own = -3.f;
+    own = -INFINITY;
 #pragma unroll
     for (int i = 0; i < PER; ++i)
       if (s[i] > own) {
         own = s[i];
+        weight = w[i];
         at = i;
       }
   };
   best();
-  for (int t = 0; t < top; ++t) {
+  for (int t = 0; t < a.top; ++t) {
     const float m = wave_reduce_max(own);
-    const unsigned long long who = __ballot(own == m);
+    const unsigned long long who =
+        m > -INFINITY ? __ballot(own == m) : 0ull;
     if (who != 0 && lane == __builtin_ctzll(who)) {
       ids[t] = lane + 64 * at;
-      weights[t] = m / sum;
+      weights[t] = weight * scale;
 #pragma unroll
       for (int i = 0; i < PER; ++i)
-        if (i == at) s[i] = -2.f;
+        if (i == at) s[i] = -INFINITY;
       best();
     } else if (who == 0 && lane == 0) {  // not a number: no expert
       ids[t] = -1;
@@ -97,47 +127,46 @@ __device__ void select_row(float* z, float* gm, int* ok, int E, int groups,
   }
 }
 
-__device__ __forceinline__ void no_choice(int top, int* ids, float* weights,
-                                          int lane) {
-  for (int t = lane; t < top; t += 64) {
-    ids[t] = -1;
-    weights[t] = 0.f;
-  }
+__device__ __forceinline__ void no_choice(const RouteArgs& a, int* ids,
+                                          float* weights, int lane) {
+  for (int t = lane; t < a.top; t += 64) ids[t] = -1;
+  for (int t = lane; t < a.cols(); t += 64) weights[t] = 0.f;
 }
 
-// from given logits [M, E]; one wave per row
+// from given logits [M, E + gates]; one wave per row
 __global__ void __launch_bounds__(256)
 select_kernel(const float* __restrict__ logits, const int* __restrict__ ctx,
-              int M, int E, int groups, int keep, int top,
-              int* __restrict__ ids, float* __restrict__ weights) {
+              int M, const RouteArgs a, int* __restrict__ ids,
+              float* __restrict__ weights) {
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
-  float* z = reinterpret_cast<float*>(smem) + wid * (E + 2 * groups);
-  float* gm = z + E;
-  int* ok = reinterpret_cast<int*>(gm + groups);
+  const int n = a.logits();
+  float* z = reinterpret_cast<float*>(smem) + wid * (n + 2 * a.groups);
+  float* gm = z + n;
+  int* ok = reinterpret_cast<int*>(gm + a.groups);
   const int row = blockIdx.x * 4 + wid;
   if (row >= M) return;
-  int* id = ids + (long)row * top;
-  float* w = weights + (long)row * top;
+  int* id = ids + (long)row * a.top;
+  float* w = weights + (long)row * a.cols();
   if (ctx[row] <= 0) {
-    no_choice(top, id, w, lane);
+    no_choice(a, id, w, lane);
     return;
   }
-  for (int e = lane; e < E; e += 64) z[e] = logits[(long)row * E + e];
+  for (int e = lane; e < n; e += 64) z[e] = logits[(long)row * n + e];
   wave_sync();
-  select_row<16>(z, gm, ok, E, groups, keep, top, id, w, lane);
+  select_row<16>(z, gm, ok, a, id, w, lane);
 }
 
-// bf16 rows against the router's weights [E, K], fp32 sums, then the
+// bf16 rows against the router's weights [E + gates, K], fp32 sums, then the
 // choice: 16 rows per workgroup, its NW waves split K and then the rows. NE
-// tiles of 16 experts.
+// tiles of 16 logits.
 template <int NE, int NW>
 __global__ void __launch_bounds__(NW * 64)
 route_kernel(const unsigned short* __restrict__ h,
              const unsigned short* __restrict__ W,
-             const int* __restrict__ ctx, int M, int E, int K, int groups,
-             int keep, int top, int* __restrict__ ids,
-             float* __restrict__ weights) {
+             const int* __restrict__ ctx, int M, int K, const RouteArgs args,
+             int* __restrict__ ids, float* __restrict__ weights) {
   constexpr int EP = NE * 16;
+  const int E = args.logits(), groups = args.groups;
   constexpr int WS = 16 * (EP + 4);  // sums of a wave
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int i16 = lane & 15, g = lane >> 4;
@@ -171,10 +200,10 @@ route_kernel(const unsigned short* __restrict__ h,
   for (int i = wid; i < 16; i += NW) {
     const int row = m0 + i;
     if (row >= M) break;
-    int* id = ids + (long)row * top;
-    float* w = weights + (long)row * top;
+    int* id = ids + (long)row * args.top;
+    float* w = weights + (long)row * args.cols();
     if (ctx[row] <= 0) {
-      no_choice(top, id, w, lane);
+      no_choice(args, id, w, lane);
       continue;
     }
     float* z = part + i * (EP + 4);
@@ -185,35 +214,43 @@ route_kernel(const unsigned short* __restrict__ h,
       z[e] = v;
     }
     wave_sync();
-    select_row<(EP + 63) / 64>(z, gm, ok, E, groups, keep, top, id, w, lane);
+    select_row<(EP + 63) / 64>(z, gm, ok, args, id, w, lane);
     wave_sync();
   }
 }
 
-extern "C" bool route_covers(int E) { return E <= 256; }
+extern "C" bool route_covers(int logits) { return logits <= 256; }
 
 extern "C" void launch_select(const float* logits, const int* ctx, int M,
-                              int E, int groups, int keep, int top, int* ids,
-                              float* weights, hipStream_t stream) {
+                              int E, int groups, int keep, int top,
+                              const float* correction, float scale, int gates,
+                              int* ids, float* weights, hipStream_t stream) {
+  const RouteArgs a{E, groups, keep, top, correction, scale, gates};
   hipLaunchKernelGGL(select_kernel, dim3((M + 3) / 4), dim3(256),
-                     4 * (E + 2 * groups) * 4, stream, logits, ctx, M, E,
-                     groups, keep, top, ids, weights);
+                     4 * (E + gates + 2 * groups) * 4, stream, logits, ctx, M,
+                     a, ids, weights);
 }
 
 extern "C" void launch_route(const void* h, const void* W, const int* ctx,
                              int M, int E, int K, int groups, int keep,
-                             int top, int* ids, float* weights,
+                             int top, const float* correction, float scale,
+                             int gates, int* ids, float* weights,
                              hipStream_t stream) {
+  const RouteArgs a{E, groups, keep, top, correction, scale, gates};
+  const int n = E + gates;
 #define RT(NE, NW)                                                           \
   hipLaunchKernelGGL((route_kernel<NE, NW>), dim3((M + 15) / 16),            \
                      dim3(NW * 64),                                          \
                      (NW * (16 * (NE * 16 + 4) + 2 * groups)) * 4, stream,   \
                      (const unsigned short*)h, (const unsigned short*)W, ctx, \
-                     M, E, K, groups, keep, top, ids, weights)
-  if (E <= 16) RT(1, 16);
-  else if (E <= 32) RT(2, 16);
-  else if (E <= 64) RT(4, 16);
-  else if (E <= 128) RT(8, 8);
+                     M, K, a, ids, weights)
+  if (n <= 16) RT(1, 16);
+  else if (n <= 32) RT(2, 16);
+  else if (n <= 48) RT(3, 16);
+  else if (n <= 64) RT(4, 16);
+  else if (n <= 80) RT(5, 16);
+  else if (n <= 128) RT(8, 8);
+  else if (n <= 144) RT(9, 8);
   else RT(16, 4);
 #undef RT
 }
@@ -289,9 +326,10 @@ extern "C" void launch_expert_plan(const int* ids, int A, int E, int TM,
 // ---- product, few rows per expert ----------------------------------------------
 // Weight-streaming bound: a workgroup takes 64 weight rows and up to 16 MT
 // places; its waves split K and read the weights straight into registers.
-// GLU: rows are gathered (place -> perm / top) and the output is F wide;
-// else rows are places and the output row is perm[place].
-template <int MT, bool GLU>
+// UNIT: 1, 2: rows are gathered (place -> perm / top), a gated unit halves
+// the columns, or each is relu(.)^2; 0: rows are places and the output row is
+// perm[place].
+template <int MT, int UNIT>
 __global__ void __launch_bounds__(256)
 expert_rows_kernel(const unsigned short* __restrict__ x,
                    const unsigned short* __restrict__ W,
@@ -299,6 +337,7 @@ expert_rows_kernel(const unsigned short* __restrict__ x,
                    const int* __restrict__ perm,
                    const int* __restrict__ tiles,
                    const int* __restrict__ ntiles, int N, int K, int top) {
+  constexpr bool GLU = UNIT == 1, UP = UNIT != 0;
   constexpr int RROW = 68;  // padded row of 64 sums
   if ((int)blockIdx.y >= *ntiles) return;
   const int* tile = tiles + (long)blockIdx.y * 4;
@@ -312,7 +351,7 @@ expert_rows_kernel(const unsigned short* __restrict__ x,
 #pragma unroll
   for (int t = 0; t < MT; ++t) {
     const int s = s0 + min(t * 16 + i16, cnt - 1);
-    xr[t] = x + (long)(GLU ? perm[s] / top : s) * K + g * 8;
+    xr[t] = x + (long)(UP ? perm[s] / top : s) * K + g * 8;
   }
   f32x4 acc[MT][4];
 #pragma unroll
@@ -359,9 +398,10 @@ expert_rows_kernel(const unsigned short* __restrict__ x,
         v = silu(v) *
             ((u[r] + u[WS + r]) + (u[2 * WS + r] + u[3 * WS + r]));
       }
+      if (UNIT == 2) v = relu2(v);
       o[r] = (short)f2bf(v);
     }
-    const long row = GLU ? s0 + m : perm[s0 + m];
+    const long row = UP ? s0 + m : perm[s0 + m];
     *reinterpret_cast<s16x4*>(out + row * (GLU ? N / 2 : N) +
                               blockIdx.x * OC + c) = o;
   }
@@ -377,7 +417,7 @@ expert_rows_kernel(const unsigned short* __restrict__ x,
 #define ET_TILE (128 * ET_K * 2)
 #define ET_LDS (68 * 1024)
 
-template <bool GLU>
+template <int UNIT>
 __global__ void __launch_bounds__(256, 2)
 expert_tile_kernel(const unsigned short* __restrict__ x,
                    const unsigned short* __restrict__ W,
@@ -385,6 +425,7 @@ expert_tile_kernel(const unsigned short* __restrict__ x,
                    const int* __restrict__ perm,
                    const int* __restrict__ tiles,
                    const int* __restrict__ ntiles, int N, int K, int top) {
+  constexpr bool GLU = UNIT == 1, UP = UNIT != 0;
   const int nt_all = *ntiles;
   const int ncol = (N + ET_N - 1) / ET_N;
   // contiguous runs of (tile, column block) per XCD, columns fastest: they
@@ -406,7 +447,7 @@ expert_tile_kernel(const unsigned short* __restrict__ x,
   for (int p = 0; p < 4; ++p) {
     const int r = wid * 32 + p * 8 + r_in;
     const int s = s0 + min(r, cnt - 1);
-    xs[p] = x + (long)(GLU ? perm[s] / top : s) * K + c_src;
+    xs[p] = x + (long)(UP ? perm[s] / top : s) * K + c_src;
     ws[p] = W + ((long)e * N + min(n0 + r, N - 1)) * K + c_src;
   }
   auto stage = [&](int k0, int buf) {
@@ -493,19 +534,24 @@ expert_tile_kernel(const unsigned short* __restrict__ x,
       if (wrow + r >= cnt || col >= N) break;
       float o[8];
 #pragma unroll
-      for (int i = 0; i < 8; ++i) o[i] = ep[r * 68 + c8 * 8 + i];
-      store8(out + (long)perm[s0 + wrow + r] * N + col, o);
+      for (int i = 0; i < 8; ++i) {
+        o[i] = ep[r * 68 + c8 * 8 + i];
+        if (UNIT == 2) o[i] = relu2(o[i]);
+      }
+      const long row = UP ? s0 + wrow + r : perm[s0 + wrow + r];
+      store8(out + row * N + col, o);
     }
   }
 }
 
 // ---- product in 32-bit: 16 places x 64 columns, one sum in four per thread ---
-template <bool GLU>
+template <int UNIT>
 __global__ void __launch_bounds__(256)
 expert_f32_kernel(const float* __restrict__ x, const float* __restrict__ W,
                   float* __restrict__ out, const int* __restrict__ perm,
                   const int* __restrict__ tiles,
                   const int* __restrict__ ntiles, int N, int K, int top) {
+  constexpr bool GLU = UNIT == 1, UP = UNIT != 0;
   __shared__ float xl[16][33], wl[64][33], sum[16][65];
   if ((int)blockIdx.y >= *ntiles) return;
   const int* tile = tiles + (long)blockIdx.y * 4;
@@ -518,7 +564,7 @@ expert_f32_kernel(const float* __restrict__ x, const float* __restrict__ W,
     for (int i = tid; i < 16 * 32; i += 256) {
       const int s = s0 + min(i / 32, cnt - 1);
       xl[i / 32][i % 32] =
-          x[(long)(GLU ? perm[s] / top : s) * K + k0 + i % 32];
+          x[(long)(UP ? perm[s] / top : s) * K + k0 + i % 32];
     }
     for (int i = tid; i < 64 * 32; i += 256)
       wl[i / 32][i % 32] = W[((long)e * N + n0 + i / 32) * K + k0 + i % 32];
@@ -535,7 +581,8 @@ expert_f32_kernel(const float* __restrict__ x, const float* __restrict__ W,
     const int r = i / OC, o = i % OC;
     float v = sum[r][GLU ? o / 16 * 32 + o % 16 : o];
     if (GLU) v = v * sigmoid_exact(v) * sum[r][o / 16 * 32 + o % 16 + 16];
-    const long row = GLU ? s0 + r : perm[s0 + r];
+    if (UNIT == 2) v = relu2(v);
+    const long row = UP ? s0 + r : perm[s0 + r];
     out[row * (GLU ? N / 2 : N) + blockIdx.x * OC + o] = v;
   }
 }
@@ -544,12 +591,13 @@ expert_f32_kernel(const float* __restrict__ x, const float* __restrict__ W,
 // expert_gemm16.hip)
 extern "C" void launch_expert_gemm16(const void*, const void*, void*,
                                      const int*, const int*, const int*, int,
-                                     int, int, int, bool, hipStream_t);
+                                     int, int, int, int, hipStream_t);
 
+// unit: 0 second product, 1 gated units, 2 squared ReLU
 extern "C" void launch_expert_gemm(const void* x, const void* W, void* out,
                                    const int* perm, const int* tiles,
                                    const int* ntiles, int max_tiles, int N,
-                                   int K, int top, int TM, bool glu,
+                                   int K, int top, int TM, int unit,
                                    bool fp32, hipStream_t stream) {
   typedef unsigned short u16;
   const dim3 grid(N / 64, max_tiles);
@@ -558,14 +606,15 @@ extern "C" void launch_expert_gemm(const void* x, const void* W, void* out,
   hipLaunchKernelGGL((expert_f32_kernel<GL>), grid, dim3(256), 0, stream,   \
                      (const float*)x, (const float*)W, (float*)out, perm,   \
                      tiles, ntiles, N, K, top)
-    if (glu) EF(true);
-    else EF(false);
+    if (unit == 1) EF(1);
+    else if (unit == 2) EF(2);
+    else EF(0);
 #undef EF
     return;
   }
   if (TM == 256) {
     launch_expert_gemm16(x, W, out, perm, tiles, ntiles, max_tiles, N, K, top,
-                         glu, stream);
+                         unit, stream);
     return;
   }
 #define ER(MT, GL)                                                          \
@@ -585,8 +634,9 @@ extern "C" void launch_expert_gemm(const void* x, const void* W, void* out,
     else if (TM == 64) ER(4, GL); \
     else ET(GL);                 \
   } while (0)
-  if (glu) EX(true);
-  else EX(false);
+  if (unit == 1) EX(1);
+  else if (unit == 2) EX(2);
+  else EX(0);
 #undef EX
 #undef ET
 #undef ER

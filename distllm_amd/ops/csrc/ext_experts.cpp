@@ -5,14 +5,15 @@ extern "C" {
 void launch_xielu(const void*, const float*, void*, long, bool, hipStream_t);
 bool route_covers(int);
 bool expert_gemm16_covers(int, int);
-void launch_select(const float*, const int*, int, int, int, int, int, int*,
-                   float*, hipStream_t);
+void launch_select(const float*, const int*, int, int, int, int, int,
+                   const float*, float, int, int*, float*, hipStream_t);
 void launch_route(const void*, const void*, const int*, int, int, int, int,
-                  int, int, int*, float*, hipStream_t);
+                  int, int, const float*, float, int, int*, float*,
+                  hipStream_t);
 void launch_expert_plan(const int*, int, int, int, int, int*, int*, int*,
                         hipStream_t);
 void launch_expert_gemm(const void*, const void*, void*, const int*,
-                        const int*, const int*, int, int, int, int, int, bool,
+                        const int*, const int*, int, int, int, int, int, int,
                         bool, hipStream_t);
 }
 
@@ -35,47 +36,68 @@ static void check_route(int64_t E, int64_t top, int64_t groups,
               "experts, groups and choices");
 }
 
-// h: bf16 rows with the router's weights, or fp32 logits (W absent)
-std::tuple<torch::Tensor, torch::Tensor> route(
+// h: bf16 rows with the router's weights, or fp32 logits (W absent). Logits
+// behind those of the experts, `gates` of them, have weights of their own.
+static std::tuple<torch::Tensor, torch::Tensor> choose(
     torch::Tensor h, c10::optional<torch::Tensor> W, torch::Tensor ctx,
-    int64_t top, int64_t groups, int64_t keep) {
+    int64_t top, int64_t groups, int64_t keep, const float* correction,
+    double scale, int gates) {
   CHECK_DEV(h); CHECK_CONT(h);
   CHECK_INTS(ctx);
   const int M = h.size(0);
-  const int E = W ? W->size(0) : h.size(1);
+  const int E = (int)(W ? W->size(0) : h.size(1)) - gates;
   check_route(E, top, groups, keep);
   TORCH_CHECK(h.dim() == 2 && ctx.numel() == M, "one ctx entry per row");
   auto ids = torch::empty({M, top}, h.options().dtype(at::kInt));
-  auto w = torch::empty({M, top}, h.options().dtype(at::kFloat));
+  auto w = torch::empty({M, top + gates}, h.options().dtype(at::kFloat));
   if (M == 0) return {ids, w};
   if (W) {
     CHECK_BF16(h);
     CHECK_DEV(W.value()); CHECK_CONT(W.value()); CHECK_BF16(W.value());
     const int K = h.size(1);
-    TORCH_CHECK(W->size(1) == K && K % 32 == 0 && route_covers(E),
+    TORCH_CHECK(W->size(1) == K && K % 32 == 0 && route_covers(E + gates),
                 "router shape");
     launch_route(h.data_ptr(), W->data_ptr(), ctx.data_ptr<int>(), M, E, K,
-                 groups, keep, top, ids.data_ptr<int>(),
-                 w.data_ptr<float>(), cur_stream());
+                 groups, keep, top, correction, (float)scale, gates,
+                 ids.data_ptr<int>(), w.data_ptr<float>(), cur_stream());
   } else {
     CHECK_F32(h);
     launch_select(h.data_ptr<float>(), ctx.data_ptr<int>(), M, E, groups,
-                  keep, top, ids.data_ptr<int>(), w.data_ptr<float>(),
-                  cur_stream());
+                  keep, top, correction, (float)scale, gates,
+                  ids.data_ptr<int>(), w.data_ptr<float>(), cur_stream());
   }
   return {ids, w};
 }
 
-torch::Tensor experts(torch::Tensor h, torch::Tensor ids, torch::Tensor wgup,
-                      torch::Tensor wdown) {
+std::tuple<torch::Tensor, torch::Tensor> route(
+    torch::Tensor h, c10::optional<torch::Tensor> W, torch::Tensor ctx,
+    int64_t top, int64_t groups, int64_t keep) {
+  return choose(h, W, ctx, top, groups, keep, nullptr, 1.0, 0);
+}
+
+std::tuple<torch::Tensor, torch::Tensor> route_sigmoid(
+    torch::Tensor h, c10::optional<torch::Tensor> W, torch::Tensor correction,
+    torch::Tensor ctx, int64_t top, double scale) {
+  CHECK_FLOATS(correction);
+  const long n = W ? W->size(0) : h.size(1);
+  const long gates = n - correction.numel();
+  TORCH_CHECK(gates >= 0 && gates <= 16, "one correction per expert");
+  return choose(h, W, ctx, top, 1, 1, correction.data_ptr<float>(), scale,
+                (int)gates);
+}
+
+// gated units, wup [E, 2F, K], or squared ReLU, wup [E, F, K]
+torch::Tensor experts(torch::Tensor h, torch::Tensor ids, torch::Tensor wup,
+                      torch::Tensor wdown, bool gated) {
   CHECK_DEV(h); CHECK_CONT(h); CHECK_T(h);
   CHECK_INTS(ids);
-  CHECK_DEV(wgup); CHECK_CONT(wgup); CHECK_SAME(wgup, h);
+  CHECK_DEV(wup); CHECK_CONT(wup); CHECK_SAME(wup, h);
   CHECK_DEV(wdown); CHECK_CONT(wdown); CHECK_SAME(wdown, h);
   const int M = h.size(0), K = h.size(1), top = ids.size(1);
-  const int E = wgup.size(0), F = wdown.size(2);
-  TORCH_CHECK(ids.size(0) == M && wgup.dim() == 3 && wdown.dim() == 3 &&
-                  wgup.size(1) == 2L * F && wgup.size(2) == K &&
+  const int E = wup.size(0), F = wdown.size(2);
+  const int N = gated ? 2 * F : F;  // columns of the first product
+  TORCH_CHECK(ids.size(0) == M && wup.dim() == 3 && wdown.dim() == 3 &&
+                  wup.size(1) == N && wup.size(2) == K &&
                   wdown.size(0) == E && wdown.size(1) == K,
               "expert shapes");
   TORCH_CHECK(K % 64 == 0 && F % 64 == 0 && E <= 1024,
@@ -89,7 +111,7 @@ torch::Tensor experts(torch::Tensor h, torch::Tensor ids, torch::Tensor wgup,
   const bool f32 = is_f32(h);
   const long mean = (A + E - 1) / E;
   int TM = f32 || mean <= 8 ? 16 : mean <= 16 ? 32 : mean <= 48 ? 64 : 128;
-  if (!f32 && mean >= 512 && expert_gemm16_covers(2 * F, K) &&
+  if (!f32 && mean >= 512 && expert_gemm16_covers(N, K) &&
       expert_gemm16_covers(K, F))
     TM = 256;
   const int max_tiles = (int)std::min<long>(A, A / TM + E);
@@ -101,11 +123,11 @@ torch::Tensor experts(torch::Tensor h, torch::Tensor ids, torch::Tensor wgup,
   launch_expert_plan(ids.data_ptr<int>(), (int)A, E, TM, max_tiles, perm,
                      tiles, ntiles, cur_stream());
   auto inter = torch::empty({A, F}, h.options());
-  launch_expert_gemm(h.data_ptr(), wgup.data_ptr(), inter.data_ptr(), perm,
-                     tiles, ntiles, max_tiles, 2 * F, K, top, TM, true, f32,
-                     cur_stream());
+  launch_expert_gemm(h.data_ptr(), wup.data_ptr(), inter.data_ptr(), perm,
+                     tiles, ntiles, max_tiles, N, K, top, TM, gated ? 1 : 2,
+                     f32, cur_stream());
   launch_expert_gemm(inter.data_ptr(), wdown.data_ptr(), y.data_ptr(), perm,
-                     tiles, ntiles, max_tiles, K, F, top, TM, false, f32,
+                     tiles, ntiles, max_tiles, K, F, top, TM, 0, f32,
                      cur_stream());
   return y;
 }
@@ -113,5 +135,6 @@ torch::Tensor experts(torch::Tensor h, torch::Tensor ids, torch::Tensor wgup,
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("xielu", &xielu);
   m.def("route", &route);
+  m.def("route_sigmoid", &route_sigmoid);
   m.def("experts", &experts);
 }

@@ -16,6 +16,7 @@ void launch_decode_gemm(const void*, const void*, const void*, void*, void*,
                         const float*, const RowsArgs*, hipStream_t);
 void launch_clamped_glu(const void*, void*, long, int, float, float, float,
                         bool, hipStream_t);
+void launch_relu2(const void*, void*, long, bool, hipStream_t);
 void launch_gelu_rows(const void*, void*, long, int, const RowsArgs*, bool,
                       hipStream_t);
 }
@@ -76,7 +77,7 @@ static torch::Tensor decode_gemm_act(torch::Tensor X, torch::Tensor W,
   // act 1, 2 = packed gated unit in the reduce (swiglu, clamped with the
   // given constants): W is [2I, K] (gate rows then up rows), output is
   // [M, I]. act 3 = xIELU with the raw numbers act_nums [2]. act 4 = GELU
-  // times a part of a table's row. All require splitk > 1.
+  // times a part of a table's row. act 5 = relu(.)^2. All require splitk > 1.
   CHECK_DEV(X); CHECK_CONT(X); CHECK_BF16(X);
   CHECK_DEV(W); CHECK_CONT(W); CHECK_BF16(W);
   const int M = X.size(0), K = X.size(1), N = W.size(0);
@@ -115,7 +116,7 @@ torch::Tensor decode_gemm(torch::Tensor X, torch::Tensor W,
                           double limit = 0.0, double alpha = 0.0,
                           double shift = 0.0,
                           c10::optional<torch::Tensor> act_nums = {}) {
-  TORCH_CHECK(act >= 0 && act <= 3, "activation");
+  TORCH_CHECK((act >= 0 && act <= 3) || act == 5, "activation");
   return decode_gemm_act(X, W, bias, splitk, act, limit, alpha, shift,
                          act_nums, nullptr);
 }
@@ -171,6 +172,15 @@ torch::Tensor clamped_glu(torch::Tensor gu, double limit, double alpha,
   return out;
 }
 
+torch::Tensor relu2(torch::Tensor z) {
+  CHECK_DEV(z); CHECK_CONT(z); CHECK_T(z);
+  TORCH_CHECK(z.numel() % 8 == 0, "size % 8");
+  auto out = torch::empty_like(z);
+  if (z.numel() > 0)
+    launch_relu2(z.data_ptr(), out.data_ptr(), z.numel(), is_f32(z),
+                 cur_stream());
+  return out;
+}
 
 // blt_gemm.cpp: hipBLASLt GEMM with fused bias/GELU/swish epilogue.
 torch::Tensor blt_linear(torch::Tensor x, torch::Tensor w,
@@ -189,4 +199,5 @@ PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("decode_gemm_rows", &decode_gemm_rows);
   m.def("gelu_rows", &gelu_rows);
   m.def("clamped_glu", &clamped_glu);
+  m.def("relu2", &relu2);
 }

@@ -3,8 +3,6 @@
 #include "ext_attention.h"
 
 extern "C" {
-void launch_rotation_table(const int*, const double*, float, float*, int, int,
-                           hipStream_t);
 void launch_attn_prep(const void*, int, int, int, int, int, int, int,
                       const float*, const float*, float, void*, void*, void*,
                       const int*, int, int, const int*, const int*, int,
@@ -87,20 +85,6 @@ torch::Tensor attn_prep(torch::Tensor ab, int64_t H, int64_t G, int64_t dp,
                      (int)((H + G) * dp), nullptr, 0, is_f32(ab),
                      cur_stream());
   return q;
-}
-
-torch::Tensor rotation_table(torch::Tensor ctx, torch::Tensor freq,
-                             double mult) {
-  CHECK_INTS(ctx);
-  CHECK_DEV(freq); CHECK_CONT(freq);
-  TORCH_CHECK(freq.scalar_type() == at::kDouble, "freq must be f64");
-  const long M = ctx.numel(), P = freq.numel();
-  auto t = torch::empty({M, P, 2}, ctx.options().dtype(at::kFloat));
-  if (M * P > 0)
-    launch_rotation_table(ctx.data_ptr<int>(), freq.data_ptr<double>(),
-                          (float)mult, t.data_ptr<float>(), M, P,
-                          cur_stream());
-  return t;
 }
 
 // ab: H query heads, G key heads of dp columns; keys as projected are the
@@ -415,7 +399,6 @@ void channel_delta(torch::Tensor ab, torch::Tensor ag, int64_t H, int64_t G,
 
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("attn_prep", &attn_prep);
-  m.def("rotation_table", &rotation_table);
   m.def("rotary_prep", &rotary_prep);
   m.def("sink_attn_rows", &sink_attn_rows);
   m.def("sink_attn_prompts", &sink_attn_prompts);

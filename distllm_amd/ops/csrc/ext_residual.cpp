@@ -1,4 +1,5 @@
-// Torch bindings of the fp32 residual stream's norms.
+// Torch bindings of what all layered decoders share: boundaries of fp32
+// residual streams, rotation tables.
 #include "ext_common.h"
 
 extern "C" {
@@ -16,6 +17,12 @@ void launch_residual_step(const void*, const void*, float*, const float*,
                           const float*, const float*, const float*,
                           const float*, bool, void*, int, int, bool,
                           hipStream_t);
+void launch_stream_step(const void*, const void*, const float*, int,
+                        const long*, const void*, float*, const float*,
+                        const float*, const float*, int, float, bool, void*,
+                        int, int, int, bool, hipStream_t);
+void launch_rotation_table(const int*, const double*, float, float*, int, int,
+                           hipStream_t);
 }
 
 // y == embedding table when tokens are given
@@ -157,9 +164,89 @@ void residual_step(torch::Tensor x, Maybe y, Maybe bias, Maybe w_rms,
                          fresh, h.data_ptr(), M, W, is_f32(h), cur_stream());
 }
 
+// x [M, S, W]; y [M, W], or [M * top, W] with weights mix [M, top] (and one
+// more column for `shared` [M, W])
+void stream_step(torch::Tensor x, Maybe y, Maybe writes, Maybe mix,
+                 Maybe shared, Maybe tokens, Maybe table, Maybe read,
+                 torch::Tensor w, int64_t n, double eps, bool store,
+                 torch::Tensor h) {
+  CHECK_FLOATS(x);
+  CHECK_DEV(h); CHECK_CONT(h); CHECK_T(h);
+  TORCH_CHECK(x.dim() == 3 && h.dim() == 2 && h.size(0) == x.size(0) &&
+                  h.size(1) == x.size(2),
+              "row sizes");
+  const int M = x.size(0), S = x.size(1), W = x.size(2);
+  TORCH_CHECK(W % 8 == 0 && W <= 16384 && n > 0 && n <= W,
+              "width must be a multiple of 8, at most 16384");
+  TORCH_CHECK(S >= 1 && S <= 16, "1 to 16 streams");
+  const void *yp = nullptr, *sp = nullptr, *tab = nullptr;
+  const float* mp = nullptr;
+  const long* tok = nullptr;
+  int top = 1;
+  TORCH_CHECK(y.has_value() == writes.has_value() &&
+                  (y.has_value() || (!mix && !shared)) &&
+                  (mix.has_value() || !shared),
+              "output, its weights and the shared output");
+  if (mix) {
+    CHECK_FLOATS(mix.value());
+    top = (int)mix->size(1) - (shared ? 1 : 0);
+    TORCH_CHECK(mix->dim() == 2 && mix->size(0) == M && top > 0, "mix rows");
+    mp = mix->data_ptr<float>();
+  }
+  if (y) {
+    CHECK_DEV(y.value()); CHECK_CONT(y.value()); CHECK_SAME(y.value(), h);
+    TORCH_CHECK(y->dim() == 2 && y->size(0) == (long)M * top &&
+                    y->size(1) == W,
+                "y rows");
+    yp = y->data_ptr();
+  }
+  if (shared) {
+    CHECK_DEV(shared.value()); CHECK_CONT(shared.value());
+    CHECK_SAME(shared.value(), h);
+    TORCH_CHECK(shared->sizes() == h.sizes(), "shared rows");
+    sp = shared->data_ptr();
+  }
+  if (tokens) {
+    TORCH_CHECK(table.has_value(), "tokens without a table");
+    CHECK_DEV(tokens.value()); CHECK_CONT(tokens.value());
+    CHECK_DEV(table.value()); CHECK_CONT(table.value());
+    CHECK_SAME(table.value(), h);
+    TORCH_CHECK(tokens->scalar_type() == at::kLong && tokens->numel() == M &&
+                    table->dim() == 2 && table->size(1) == W,
+                "tokens (int64, one per row) and table");
+    tok = (const long*)tokens->data_ptr<int64_t>();
+    tab = table->data_ptr();
+  }
+  auto opt = [&](const Maybe& t, long k) {
+    return t ? norm_vec(*t, k) : (const float*)nullptr;
+  };
+  if (M > 0)
+    launch_stream_step(yp, sp, mp, top, tok, tab, x.data_ptr<float>(),
+                       opt(writes, (long)S * (S + 1)), opt(read, S),
+                       norm_vec(w, W), (int)n, (float)eps,
+                       store && y.has_value(), h.data_ptr(), M, S, W,
+                       is_f32(h), cur_stream());
+}
+
+torch::Tensor rotation_table(torch::Tensor ctx, torch::Tensor freq,
+                             double mult) {
+  CHECK_INTS(ctx);
+  CHECK_DEV(freq); CHECK_CONT(freq);
+  TORCH_CHECK(freq.scalar_type() == at::kDouble, "freq must be f64");
+  const long M = ctx.numel(), P = freq.numel();
+  auto t = torch::empty({M, P, 2}, ctx.options().dtype(at::kFloat));
+  if (M * P > 0)
+    launch_rotation_table(ctx.data_ptr<int>(), freq.data_ptr<double>(),
+                          (float)mult, t.data_ptr<float>(), M, P,
+                          cur_stream());
+  return t;
+}
+
 PYBIND11_MODULE(TORCH_EXTENSION_NAME, m) {
   m.def("sandwich_norm", &sandwich_norm);
   m.def("embed_positions", &embed_positions);
   m.def("layer_norm_add", &layer_norm_add);
   m.def("residual_step", &residual_step);
+  m.def("stream_step", &stream_step);
+  m.def("rotation_table", &rotation_table);
 }

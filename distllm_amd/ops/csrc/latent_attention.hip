@@ -6,9 +6,11 @@
 // q_h) and Uv into the output leaves one shared "head" whose key and value
 // are both c:
 //     s_hj = scale * q'_h . c_j      o'_h = sum_j softmax(s)_hj c_j
-// so a decode step reads R numbers per cached token for all heads.
+// so a decode step reads R numbers per cached token for all heads. A cache
+// row may go on behind the latent, with a key part that all heads share (and
+// that queries have a part of their own for); RT is the length of a row.
 //
-// Cache layout: [num_blocks, PBLK, R], block_table [S, max_blocks] int32.
+// Cache layout: [num_blocks, PBLK, RT], block_table [S, max_blocks] int32.
 // Every row of a batch is one token: row_seq[row] is its block-table row,
 // ctx[row] its position + 1 (0: padding row, nothing is read or written).
 // A row sees the last `window` positions up to its own.
@@ -107,14 +109,137 @@ extern "C" void launch_latent_prep(
 #undef LP
 }
 
+// ---- norm of the latent, rotation of queries and key part, cache write -------
+// ab row: H heads of dp unrotated and tp rotated numbers, the latent (R, true
+// size rn), the key part (tp). The first 2 * half of tp numbers rotate, those
+// behind are zeros. Rotated query parts go to the end of ql's rows (first n
+// rows; ql_row numbers per head) or back to ab; three waves of a workgroup do
+// that, the fourth makes the cache row.
+
+// pairs i0 .. i0 + 7 of src (number i and i + half) to dst
+template <typename T>
+__device__ __forceinline__ void rotate_pairs(const T* src, T* dst, int i0,
+                                             int half, const float* table) {
+  if ((half & 7) == 0) {
+    float a[8], b[8], t[16], x[8], y[8];
+    load8<T>(src + i0, a);
+    load8<T>(src + half + i0, b);
+    load8<float>(table + i0 * 2, t);
+    load8<float>(table + i0 * 2 + 8, t + 8);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      x[i] = a[i] * t[2 * i] - b[i] * t[2 * i + 1];
+      y[i] = b[i] * t[2 * i] + a[i] * t[2 * i + 1];
+    }
+    store8(dst + i0, x);
+    store8(dst + half + i0, y);
+    return;
+  }
+  for (int i = i0; i < min(i0 + 8, half); ++i) {
+    const float a = to_f(src[i]), b = to_f(src[half + i]);
+    const float c = table[i * 2], s = table[i * 2 + 1];
+    from_f(dst + i, a * c - b * s);
+    from_f(dst + half + i, b * c + a * s);
+  }
+}
+
+template <typename T, int NC>
+__global__ void __launch_bounds__(256)
+rotary_latent_prep_kernel(T* __restrict__ ab, int ld, int H, int dp, int tp,
+                          int R, int rn, const float* __restrict__ wc,
+                          float eps, const float* __restrict__ table,
+                          int half, T* __restrict__ ql, int n, int ql_row,
+                          T* __restrict__ cache,
+                          const int* __restrict__ block_table,
+                          int max_blocks, int num_blocks,
+                          const int* __restrict__ row_seq,
+                          const int* __restrict__ ctx) {
+  const int row = blockIdx.x;
+  T* src = ab + (long)row * ld;
+  const float* cs = table + (long)row * half * 2;
+  const int groups = (half + 7) / 8;
+  if (threadIdx.x < 192) {
+    for (int u = threadIdx.x; u < H * groups; u += 192) {
+      const int head = u / groups, i0 = u % groups * 8;
+      T* q = src + head * (dp + tp) + dp;
+      T* dst = q;
+      if (row < n) {
+        dst = ql + ((long)row * H + head) * ql_row + ql_row - tp;
+        if (i0 == 0)
+          for (int c = 2 * half; c < tp; ++c) from_f(dst + c, 0.f);
+      }
+      rotate_pairs(q, dst, i0, half, cs);
+    }
+    return;
+  }
+  if (cache == nullptr) return;
+  const int lane = threadIdx.x & 63;
+  const int pos = ctx[row] - 1;
+  if (pos < 0 || pos / PBLK >= max_blocks) return;
+  const int blk = block_table[(long)row_seq[row] * max_blocks + pos / PBLK];
+  if (blk < 0 || blk >= num_blocks) return;
+  T* dst = cache + ((long)blk * PBLK + pos % PBLK) * (R + tp);
+  src += H * (dp + tp);
+  for (int g = lane; g < groups; g += 64)
+    rotate_pairs(src + R, dst + R, g * 8, half, cs);
+  float v[NC][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = (k * 64 + lane) * 8;
+    if (c < R) {
+      load8<T>(src + c, v[k]);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) ss += v[k][i] * v[k][i];
+    }
+  }
+  const float inv = 1.f / sqrtf(wave_reduce_sum(ss) / rn + eps);
+#pragma unroll
+  for (int k = 0; k < NC; ++k) {
+    const int c = (k * 64 + lane) * 8;
+    if (c < R) {
+      float w[8];
+      load8<float>(wc + c, w);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[k][i] *= inv * w[i];
+      store8(dst + c, v[k]);
+    }
+  }
+}
+
+extern "C" void launch_rotary_latent_prep(
+    void* ab, int M, int ld, int H, int dp, int tp, int R, int rn,
+    const float* wc, float eps, const float* table, int half, void* ql, int n,
+    int ql_row, void* cache, const int* block_table, int max_blocks,
+    int num_blocks, const int* row_seq, const int* ctx, bool fp32,
+    hipStream_t stream) {
+  const dim3 grid(M), block(cache != nullptr ? 256 : 192);
+#define RP(T, NC)                                                           \
+  hipLaunchKernelGGL((rotary_latent_prep_kernel<T, NC>), grid, block, 0,    \
+                     stream, (T*)ab, ld, H, dp, tp, R, rn, wc, eps, table,  \
+                     half, (T*)ql, n, ql_row, (T*)cache, block_table,       \
+                     max_blocks, num_blocks, row_seq, ctx)
+#define RP_N(T)                   \
+  do {                            \
+    if (R <= 512) RP(T, 1);       \
+    else if (R <= 1024) RP(T, 2); \
+    else RP(T, 8);                \
+  } while (0)
+  if (fp32) RP_N(float);
+  else RP_N(unsigned short);
+#undef RP_N
+#undef RP
+}
+
 // ---- latents of chosen positions, packed ----------------------------------
-// out[i] = cache entry of position key_pos[i] of block-table row key_seq[i]
+// Row i of out is the first vec0 pieces of the cache entry of position
+// key_pos[i] of block-table row key_seq[i], row i of rest the others.
 __global__ void __launch_bounds__(256)
 latent_gather_kernel(const i32x4* __restrict__ cache,
                      const int* __restrict__ block_table, int max_blocks,
                      int num_blocks, const int* __restrict__ key_seq,
                      const int* __restrict__ key_pos, i32x4* __restrict__ out,
-                     int T, int vec) {
+                     i32x4* __restrict__ rest, int T, int vec, int vec0) {
   const long total = (long)T * vec;
   const long stride = (long)gridDim.x * blockDim.x;
   for (long i = (long)blockIdx.x * blockDim.x + threadIdx.x; i < total;
@@ -128,32 +253,37 @@ latent_gather_kernel(const i32x4* __restrict__ cache,
       if (blk >= 0 && blk < num_blocks)
         v = cache[((long)blk * PBLK + pos % PBLK) * vec + c];
     }
-    out[i] = v;
+    if (c < vec0) out[(long)row * vec0 + c] = v;
+    else rest[(long)row * (vec - vec0) + c - vec0] = v;
   }
 }
 
 extern "C" void launch_latent_gather(const void* cache,
                                      const int* block_table, int max_blocks,
                                      int num_blocks, const int* key_seq,
-                                     const int* key_pos, void* out, int T,
-                                     int row_bytes, hipStream_t stream) {
+                                     const int* key_pos, void* out,
+                                     void* rest, int T, int row_bytes,
+                                     int out_bytes, hipStream_t stream) {
   const int vec = row_bytes / 16;
   const int blocks = (int)min(((long)T * vec + 255) / 256, (long)4096);
   hipLaunchKernelGGL(latent_gather_kernel, dim3(blocks), dim3(256), 0, stream,
                      (const i32x4*)cache, block_table, max_blocks, num_blocks,
-                     key_seq, key_pos, (i32x4*)out, T, vec);
+                     key_seq, key_pos, (i32x4*)out, (i32x4*)rest, T, vec,
+                     out_bytes / 16);
 }
 
 // ---- per-head products -----------------------------------------------------
 // out[m, h, :] = W[h] x[m, h, :], W [H, N, K] bf16, for the few rows of a
-// decode step (weight-streaming bound). A wave owns 16 output columns; the
+// decode step (weight-streaming bound); rows and heads of x and out are
+// strided. A wave owns 16 output columns; the
 // weight fragment is read once and used for MT tiles of 16 rows.
 template <int MT, int KU>
 __global__ void __launch_bounds__(256)
 head_gemm_kernel(const unsigned short* __restrict__ x,
                  const unsigned short* __restrict__ W,
                  unsigned short* __restrict__ out, int M, int H, int N,
-                 int K) {
+                 int K, long xrow_s, int xhead_s, long orow_s,
+                 int ohead_s) {
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int nb = N / 64;
   const int head = blockIdx.x / nb;
@@ -166,7 +296,7 @@ head_gemm_kernel(const unsigned short* __restrict__ x,
 #pragma unroll
   for (int t = 0; t < MT; ++t) {
     const int m = min(m0 + t * 16 + i16, M - 1);
-    xrow[t] = x + ((long)m * H + head) * K + g * 8;
+    xrow[t] = x + m * xrow_s + (long)head * xhead_s + g * 8;
   }
   f32x4 acc[MT];
 #pragma unroll
@@ -195,14 +325,15 @@ head_gemm_kernel(const unsigned short* __restrict__ x,
       s16x4 o;
 #pragma unroll
       for (int r = 0; r < 4; ++r) o[r] = (short)f2bf(acc[t][r]);
-      *reinterpret_cast<s16x4*>(out + ((long)m * H + head) * N + n0 + g * 4) =
-          o;
+      *reinterpret_cast<s16x4*>(out + m * orow_s + (long)head * ohead_s +
+                                n0 + g * 4) = o;
     }
   }
 }
 
 extern "C" void launch_head_gemm(const void* x, const void* W, void* out,
-                                 int M, int H, int N, int K,
+                                 int M, int H, int N, int K, long xrow_s,
+                                 int xhead_s, long orow_s, int ohead_s,
                                  hipStream_t stream) {
   // row tiles per workgroup: as many as leave two workgroups per CU
   const int tiles = (M + 15) / 16;
@@ -215,7 +346,7 @@ extern "C" void launch_head_gemm(const void* x, const void* W, void* out,
                      dim3(cols, (M + 16 * MT - 1) / (16 * MT)),           \
                      dim3(256), 0, stream, (const unsigned short*)x,      \
                      (const unsigned short*)W, (unsigned short*)out, M, H, \
-                     N, K)
+                     N, K, xrow_s, xhead_s, orow_s, ohead_s)
 #define HG_K(MT)                     \
   do {                               \
     if (K % 256 == 0) HG(MT, 8);     \
@@ -230,19 +361,21 @@ extern "C" void launch_head_gemm(const void* x, const void* W, void* out,
 }
 
 // ---- attention, one workgroup per (row, head), any rank and type ----------
-// NV: latent columns per thread (R <= 256 * NV).
+// NV: latent columns per thread (R <= 256 * NV). sink, gate: null or the
+// numbers of the heads (gate rows are ld_gate apart).
 template <typename T, int NV>
 __global__ void __launch_bounds__(256)
 latent_attn_rows_kernel(const T* __restrict__ q, const T* __restrict__ cache,
                         const int* __restrict__ block_table,
                         const int* __restrict__ row_seq,
                         const int* __restrict__ ctx, T* __restrict__ out,
-                        int H, int R, int max_blocks, int window,
-                        float scale) {
+                        int H, int R, int RT, int max_blocks, int window,
+                        float scale, const float* __restrict__ sink,
+                        const T* __restrict__ gate, int ld_gate) {
   constexpr int V = 16 / sizeof(T);
   typedef __attribute__((ext_vector_type(V))) T vec;
-  float* q_lds = reinterpret_cast<float*>(smem);  // R
-  float* p_lds = q_lds + R;                       // 256
+  float* q_lds = reinterpret_cast<float*>(smem);  // RT
+  float* p_lds = q_lds + RT;                      // 256
   int* off_lds = reinterpret_cast<int*>(p_lds + 256);  // 256 cache rows
   float* red = reinterpret_cast<float*>(off_lds + 256);  // 8
   const int row = blockIdx.x / H, head = blockIdx.x % H;
@@ -250,8 +383,8 @@ latent_attn_rows_kernel(const T* __restrict__ q, const T* __restrict__ cache,
   const int L = min(ctx[row], max_blocks * PBLK);
   const int lo = L > window ? L - window : 0;
   const int* bt = block_table + (long)row_seq[row] * max_blocks;
-  const T* qr = q + ((long)row * H + head) * R;
-  for (int c = tid; c < R; c += 256) q_lds[c] = to_f(qr[c]) * scale;
+  const T* qr = q + ((long)row * H + head) * RT;
+  for (int c = tid; c < RT; c += 256) q_lds[c] = to_f(qr[c]) * scale;
 
   float m = -INFINITY, l = 0.f, acc[NV];
 #pragma unroll
@@ -264,9 +397,9 @@ latent_attn_rows_kernel(const T* __restrict__ q, const T* __restrict__ cache,
     if (live) {
       const int off = bt[key / PBLK] * PBLK + key % PBLK;
       off_lds[tid] = off;
-      const T* c = cache + (long)off * R;
+      const T* c = cache + (long)off * RT;
       float dot = 0.f;
-      for (int k = 0; k < R; k += V) {
+      for (int k = 0; k < RT; k += V) {
         const vec cv = *reinterpret_cast<const vec*>(c + k);
 #pragma unroll
         for (int i = 0; i < V; ++i) dot += to_f((T)cv[i]) * q_lds[k + i];
@@ -293,12 +426,18 @@ latent_attn_rows_kernel(const T* __restrict__ q, const T* __restrict__ cache,
       if (c < R) {
         float a = acc[i] * alpha;
         for (int j = 0; j < nk; ++j)
-          a += p_lds[j] * to_f(cache[(long)off_lds[j] * R + c]);
+          a += p_lds[j] * to_f(cache[(long)off_lds[j] * RT + c]);
         acc[i] = a;
       }
     }
   }
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  float inv = l > 0.f ? 1.f / l : 0.f;
+  if (sink != nullptr && l > 0.f) {
+    const float top = fmaxf(m, sink[head]), a = expf(m - top);
+    inv = a / (l * a + expf(sink[head] - top));
+  }
+  if (gate != nullptr)
+    inv *= sigmoid_exact(to_f(gate[(long)row * ld_gate + head]));
   T* o = out + ((long)row * H + head) * R;
 #pragma unroll
   for (int i = 0; i < NV; ++i) {
@@ -310,13 +449,14 @@ latent_attn_rows_kernel(const T* __restrict__ q, const T* __restrict__ cache,
 extern "C" void launch_latent_attn_rows(
     const void* q, const void* cache, const int* block_table,
     const int* row_seq, const int* ctx, void* out, int M, int H, int R,
-    int max_blocks, int window, float scale, bool fp32, hipStream_t stream) {
-  const int lds = (R + 256 + 256 + 8) * 4;
+    int RT, int max_blocks, int window, float scale, const float* sink,
+    const void* gate, int ld_gate, bool fp32, hipStream_t stream) {
+  const int lds = (RT + 256 + 256 + 8) * 4;
 #define LA(T, NV)                                                            \
   hipLaunchKernelGGL((latent_attn_rows_kernel<T, NV>), dim3(M * H),          \
                      dim3(256), lds, stream, (const T*)q, (const T*)cache,   \
-                     block_table, row_seq, ctx, (T*)out, H, R, max_blocks,   \
-                     window, scale)
+                     block_table, row_seq, ctx, (T*)out, H, R, RT,           \
+                     max_blocks, window, scale, sink, (const T*)gate, ld_gate)
 #define LA_N(T)                    \
   do {                             \
     if (R <= 256) LA(T, 1);        \

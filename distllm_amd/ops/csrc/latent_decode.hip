@@ -17,6 +17,9 @@
 // accumulators of a wave small. Both products use
 // mfma_f32_16x16x32_bf16 with keys (then latent columns) as rows and heads
 // as columns, so softmax state and rescaling are lane-local.
+//
+// Cache rows and queries have RR = R + ROT numbers, of which all take part in
+// the scores and the first R are the value.
 #include "common.h"
 
 #define PBLK 16
@@ -35,7 +38,23 @@ __device__ __forceinline__ int ct_slot(int r, int slot) {
   return r * 64 + (r >> 3) * 64 + ((slot ^ ((r >> 2) & 3)) * 16);
 }
 
-template <int R, int HG, int KS>
+// Weight of a row's sum: 1 / l with the softmax's state m (log2 units), l and
+// the sink of the head, times its gate.
+__device__ __forceinline__ float row_weight(float m, float l, long row,
+                                            int head, const float* sink,
+                                            const unsigned short* gate,
+                                            int ld_gate) {
+  float inv = l > 0.f ? 1.f / l : 0.f;
+  if (sink != nullptr && l > 0.f) {
+    const float s = sink[head] * LOG2E, top = fmaxf(m, s);
+    const float a = __builtin_amdgcn_exp2f(m - top);
+    inv = a / (l * a + __builtin_amdgcn_exp2f(s - top));
+  }
+  if (gate != nullptr) inv *= sigmoid_exact(bf2f(gate[row * ld_gate + head]));
+  return inv;
+}
+
+template <int R, int ROT, int HG, int KS>
 __global__ void __launch_bounds__(64 * HG * KS, 2)
 latent_decode_kernel(const unsigned short* __restrict__ q,
                      const unsigned short* __restrict__ cache,
@@ -45,15 +64,17 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
                      unsigned short* __restrict__ out,
                      float* __restrict__ pacc, float* __restrict__ pml,
                      int H, int NG, int NS, int max_blocks, int window,
-                     float scale) {
+                     float scale, const float* __restrict__ sink,
+                     const unsigned short* __restrict__ gate, int ld_gate) {
   constexpr int NT = 64 * HG * KS;
-  constexpr int UNITS = R;  // a unit: 4 keys x 8 latent columns
+  constexpr int RR = R + ROT;
+  constexpr int UNITS = RR;  // a unit: 4 keys x 8 columns
   constexpr int UPT = (UNITS + NT - 1) / NT;
-  constexpr int SW = R % 128 == 0 ? 15 : 7;
-  constexpr int CT = KT * R * 2;        // LDS offset of the transposed copy
+  constexpr int SW = RR % 128 == 0 ? 15 : 7;
+  constexpr int CT = KT * RR * 2;       // LDS offset of the transposed copy
   constexpr int SC = CT + R * 72;       // LDS offset of the scores
   constexpr int RSPLIT = KS / 2;       // column parts, besides key halves
-  constexpr int QS = R / 32 / RSPLIT;  // score steps of a wave
+  constexpr int QS = RR / 32 / RSPLIT;  // score steps of a wave
   constexpr int OB = R / 16 / KS;      // output blocks of a wave
   static_assert(KS == 2 || KS == 4, "two key halves");
 
@@ -82,7 +103,7 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
   i32x4 kv[UPT][4];
   auto issue = [&](int page) {
     const unsigned short* base =
-        cache + ((long)page * PBLK + (kg & 3) * 4) * R;
+        cache + ((long)page * PBLK + (kg & 3) * 4) * RR;
 #pragma unroll
     for (int i = 0; i < UPT; ++i) {
       const int u = threadIdx.x + i * NT;
@@ -91,7 +112,7 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
 #pragma unroll
         for (int j = 0; j < 4; ++j)
           kv[i][j] =
-              *reinterpret_cast<const i32x4*>(base + (long)j * R + c * 8);
+              *reinterpret_cast<const i32x4*>(base + (long)j * RR + c * 8);
       }
     }
   };
@@ -104,9 +125,10 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           const int key = kg * 4 + j;
-          *reinterpret_cast<i32x4*>(smem + key * (R * 2) +
+          *reinterpret_cast<i32x4*>(smem + key * (RR * 2) +
                                     ((c ^ (key & SW)) * 16)) = kv[i][j];
         }
+        if (ROT > 0 && c >= R / 8) continue;  // no value
 #pragma unroll
         for (int w = 0; w < 4; ++w) {
           i32x2 even, odd;
@@ -134,7 +156,7 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
   }
   bf16x8 qf[QS];
   {
-    const unsigned short* qr = q + ((long)row * H + (live ? head : 0)) * R +
+    const unsigned short* qr = q + ((long)row * H + (live ? head : 0)) * RR +
                                rhalf * (QS * 32) + g * 8;
 #pragma unroll
     for (int s = 0; s < QS; ++s) {
@@ -168,7 +190,7 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
 #pragma unroll
     for (int s = 0; s < QS; ++s) {
       const int chunk = (rhalf * QS + s) * 4 + g;
-      const char* a = smem + (khalf * 16 + i16) * (R * 2) +
+      const char* a = smem + (khalf * 16 + i16) * (RR * 2) +
                       ((chunk ^ (i16 & SW)) * 16);
       const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(a);
       sa[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
@@ -233,7 +255,7 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
   const long rh = (long)row * H + head;
   const int col = ks * (OB * 16) + g * 4;
   if (NS == 1) {
-    const float inv = l > 0.f ? 1.f / l : 0.f;
+    const float inv = row_weight(m, l, row, head, sink, gate, ld_gate);
 #pragma unroll
     for (int i = 0; i < OB; ++i) {
       s16x4 o;
@@ -258,7 +280,8 @@ __global__ void __launch_bounds__(256)
 latent_combine_kernel(const float* __restrict__ pacc,
                       const float* __restrict__ pml,
                       unsigned short* __restrict__ out, int RH, int R,
-                      int NS) {
+                      int NS, int H, const float* __restrict__ sink,
+                      const unsigned short* __restrict__ gate, int ld_gate) {
   const int lane = threadIdx.x & 63;
   const long rh = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (rh >= RH) return;
@@ -268,7 +291,8 @@ latent_combine_kernel(const float* __restrict__ pacc,
   for (int s = 0; s < NS; ++s)
     l += pml[(rh * NS + s) * 2 + 1] *
          __builtin_amdgcn_exp2f(pml[(rh * NS + s) * 2] - M);
-  const float inv = l > 0.f ? 1.f / l : 0.f;
+  const float inv =
+      row_weight(M, l, rh / H, (int)(rh % H), sink, gate, ld_gate);
   for (int c = lane * 4; c < R; c += 256) {
     f32x4 o = {0.f, 0.f, 0.f, 0.f};
     for (int s = 0; s < NS; ++s) {
@@ -291,31 +315,39 @@ extern "C" int latent_decode_heads(int H) {
   return H <= 16 ? 16 : H <= 32 ? 32 : 64;
 }
 
-extern "C" bool latent_decode_covers(int R) {
+extern "C" bool latent_decode_covers(int R, int rot) {
+  if (rot != 0 && rot != 64) return false;
   return R == 64 || R == 128 || R == 192 || R == 256 || R == 384 || R == 512;
 }
 
 extern "C" void launch_latent_decode(
     const void* q, const void* cache, const int* block_table,
     const int* row_seq, const int* ctx, void* out, void* pacc, void* pml,
-    int M, int H, int R, int NS, int max_blocks, int window, float scale,
+    int M, int H, int R, int rot, int NS, int max_blocks, int window,
+    float scale, const float* sink, const void* gate, int ld_gate,
     hipStream_t stream) {
   const int heads = latent_decode_heads(H);
   const int ng = (H + heads - 1) / heads;
-#define LD(RR, HG, KS)                                                        \
-  hipLaunchKernelGGL((latent_decode_kernel<RR, HG, KS>), dim3(M * ng * NS),   \
-                     dim3(64 * HG * KS),                                      \
-                     KT * RR * 2 + RR * 72 +                                  \
+#define LD(RR, RO, HG, KS)                                                    \
+  hipLaunchKernelGGL((latent_decode_kernel<RR, RO, HG, KS>),                  \
+                     dim3(M * ng * NS), dim3(64 * HG * KS),                   \
+                     KT * (RR + RO) * 2 + RR * 72 +                           \
                          HG * (KS == 4 ? 2 : 1) * 16 * SROW * 4,              \
                      stream, (const unsigned short*)q,                        \
                      (const unsigned short*)cache, block_table, row_seq, ctx, \
                      (unsigned short*)out, (float*)pacc, (float*)pml, H, ng,  \
-                     NS, max_blocks, window, scale)
-#define LD_R(RR)                      \
-  do {                                \
-    if (heads == 16) LD(RR, 1, 4);    \
-    else if (heads == 32) LD(RR, 2, 2); \
-    else LD(RR, 4, 2);                \
+                     NS, max_blocks, window, scale, sink,                     \
+                     (const unsigned short*)gate, ld_gate)
+#define LD_H(RR, RO)                      \
+  do {                                    \
+    if (heads == 16) LD(RR, RO, 1, 4);    \
+    else if (heads == 32) LD(RR, RO, 2, 2); \
+    else LD(RR, RO, 4, 2);                \
+  } while (0)
+#define LD_R(RR)              \
+  do {                        \
+    if (rot == 0) LD_H(RR, 0); \
+    else LD_H(RR, 64);        \
   } while (0)
   switch (R) {
     case 64: LD_R(64); break;
@@ -326,9 +358,11 @@ extern "C" void launch_latent_decode(
     default: LD_R(512); break;
   }
 #undef LD_R
+#undef LD_H
 #undef LD
   if (NS > 1)
     hipLaunchKernelGGL(latent_combine_kernel, dim3((M * H + 3) / 4),
                        dim3(256), 0, stream, (const float*)pacc,
-                       (const float*)pml, (unsigned short*)out, M * H, R, NS);
+                       (const float*)pml, (unsigned short*)out, M * H, R, NS,
+                       H, sink, (const unsigned short*)gate, ld_gate);
 }

@@ -11,7 +11,8 @@ from __future__ import annotations
 import importlib
 
 EXTENSIONS = ("_hip_gemm", "_hip_residual", "_hip_latent", "_hip_hybrid",
-              "_hip_chunked", "_hip_experts", "_hip_lru", "_hip_ops")
+              "_hip_chunked", "_hip_experts", "_hip_lru", "_hip_retention",
+              "_hip_ops")
 
 
 class Native:

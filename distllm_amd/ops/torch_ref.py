@@ -315,6 +315,37 @@ def latent_prep(ab, q_cols, q_rank, rank, wq, wc, eps, cache, block_table,
     return norm(ab[:, :q_cols], q_rank, wq)
 
 
+def _rotate(x, table):
+    """x [M, .., n]: its first 2 * pairs numbers turned by table [M, pairs,
+    2], in fp32."""
+    x, half = x.float(), table.shape[1]
+    cs = table.view(len(x), *[1] * (x.dim() - 2), half, 2)
+    a, b = x[..., :half], x[..., half: 2 * half]
+    cos, sin = cs[..., 0], cs[..., 1]
+    return torch.cat([a * cos - b * sin, b * cos + a * sin,
+                      x[..., 2 * half:]], -1)
+
+
+def rotary_latent_prep(ab, heads, dp, tp, rank, wc, eps, table, cache,
+                       block_table, row_seq, ctx, ql):
+    M, n = ab.shape[0], ql.shape[0]
+    qr = ab[:, : heads * (dp + tp)].view(M, heads, dp + tp)[..., dp:]
+    turned = _rotate(qr, table).to(ab.dtype)
+    ql[..., ql.shape[2] - tp:] = turned[:n]
+    qr[n:] = turned[n:]
+    if cache is None:
+        return
+    live = ctx > 0
+    at, R = heads * (dp + tp), cache.shape[2] - tp
+    c = ab[live, at: at + R].float()
+    ms = c.pow(2).sum(-1, keepdim=True) / rank
+    c = (c / torch.sqrt(ms + eps) * wc).to(ab.dtype)
+    kr = _rotate(ab[live, at + R: at + R + tp], table[live]).to(ab.dtype)
+    rows = _cache_rows(block_table, row_seq[live], ctx[live] - 1,
+                       cache.shape[1])
+    cache.view(-1, R + tp)[rows] = torch.cat([c, kr], 1)
+
+
 def latent_gather(cache, block_table, key_seq, key_pos):
     rows = _cache_rows(block_table, key_seq, key_pos, cache.shape[1])
     return cache.view(-1, cache.shape[2])[rows]
@@ -327,10 +358,21 @@ def head_gemm(x, w):
     return out.transpose(0, 1).to(x.dtype).contiguous()
 
 
-def latent_attn(q, cache, block_table, row_seq, ctx, window, scale):
-    """q [M, H, R] against the cached latents of each row's sequence; key
-    and value are both the latent."""
-    out = torch.zeros_like(q)
+def _softmax_sink(s, sink):
+    """Softmax over the last axis of s [H, .., n], with exp(sink) of the
+    head in the denominator."""
+    if sink is None:
+        return torch.softmax(s, -1)
+    own = sink.float().view(-1, *[1] * (s.dim() - 1)).expand(
+        *s.shape[:-1], 1)
+    return torch.softmax(torch.cat([s, own], -1), -1)[..., :-1]
+
+
+def latent_attn(q, cache, block_table, row_seq, ctx, window, scale, rank,
+                sink=None, gate=None):
+    """q [M, H, R] against the cached latents of each row's sequence; the
+    key is the whole cache row, the value its first rank columns."""
+    out = q.new_zeros(q.shape[0], q.shape[1], rank)
     for r in range(q.shape[0]):
         L = int(ctx[r])
         if L <= 0:
@@ -338,17 +380,25 @@ def latent_attn(q, cache, block_table, row_seq, ctx, window, scale):
         pos = torch.arange(max(0, L - window), L)
         c = latent_gather(cache, block_table,
                           row_seq[r].expand(len(pos)), pos).float()
-        p = torch.softmax(q[r].float() @ c.t() * scale, dim=-1)
-        out[r] = (p @ c).to(q.dtype)
+        p = _softmax_sink(q[r].float() @ c.t() * scale, sink)
+        o = p @ c[:, :rank]
+        if gate is not None:
+            o = o * torch.sigmoid(gate[r].float())[:, None]
+        out[r] = o.to(q.dtype)
     return out
 
 
-def attn_window(q, kv, dv, cu_q, cu_k, window, scale):
+def attn_window(q, kv, dv, cu_q, cu_k, window, scale, kr=None, sink=None,
+                gate=None):
     """Packed continuation attention: the queries of a sequence are the
-    last ones of its keys. q [Tq, H, DK]; kv [Tk, H*DK + H*DV]."""
+    last ones of its keys. q [Tq, H, DK (+ DR)]; kv [Tk, H*DK + H*DV]; kr
+    [Tk, DR]."""
     Tq, H, dk = q.shape
+    dk -= 0 if kr is None else kr.shape[1]
     k = kv[:, : H * dk].view(-1, H, dk).float()
     v = kv[:, H * dk:].view(-1, H, dv).float()
+    if kr is not None:
+        k = torch.cat([k, kr[:, None].float().expand(-1, H, -1)], -1)
     out = torch.zeros(Tq, H, dv, dtype=q.dtype)
     for b in range(len(cu_q) - 1):
         q0, q1 = int(cu_q[b]), int(cu_q[b + 1])
@@ -358,8 +408,10 @@ def attn_window(q, kv, dv, cu_q, cu_k, window, scale):
         s = torch.einsum("qhd,khd->hqk", q[q0:q1].float(),
                          k[k0:k1]) * scale
         s = s.masked_fill((j > i) | (j <= i - window), float("-inf"))
-        out[q0:q1] = torch.einsum("hqk,khd->qhd", torch.softmax(s, -1),
-                                  v[k0:k1]).to(q.dtype)
+        o = torch.einsum("hqk,khd->qhd", _softmax_sink(s, sink), v[k0:k1])
+        if gate is not None:
+            o = o * torch.sigmoid(gate[q0:q1].float())[..., None]
+        out[q0:q1] = o.to(q.dtype)
     return out
 
 
@@ -525,7 +577,21 @@ def route(h, router, ctx, top, groups, keep):
     return ids.int().masked_fill(dead, -1), w.masked_fill(dead, 0)
 
 
-def experts(h, ids, wgup, wdown, unit=16):
+def route_sigmoid(h, router, correction, ctx, top, scale):
+    """-> expert ids [M, top] int32 (-1: none), weights [M, top + gates]."""
+    E = correction.shape[0]
+    s = torch.sigmoid(h.float() @ router.float().t())
+    ids = (s[:, :E] + correction).topk(top, -1).indices
+    w = torch.cat([s.gather(1, ids) * scale, s[:, E:]], 1)
+    dead = (ctx <= 0)[:, None]
+    return ids.int().masked_fill(dead, -1), w.masked_fill(dead, 0)
+
+
+def relu2(z):
+    return z.float().clamp(min=0).square().to(z.dtype)
+
+
+def experts(h, ids, wgup, wdown, gated=True, unit=16):
     M, top = ids.shape
     out = torch.zeros(M * top, wdown.shape[1], dtype=h.dtype)
     flat = ids.reshape(-1)
@@ -534,9 +600,12 @@ def experts(h, ids, wgup, wdown, unit=16):
             continue
         rows = (flat == e).nonzero()[:, 0]
         gu = h[rows // top].float() @ wgup[e].float().t()
-        gu = gu.view(len(rows), -1, 2, unit)
-        a = torch.nn.functional.silu(gu[:, :, 0]) * gu[:, :, 1]
-        a = a.reshape(len(rows), -1).to(h.dtype)
+        if gated:
+            gu = gu.view(len(rows), -1, 2, unit)
+            a = torch.nn.functional.silu(gu[:, :, 0]) * gu[:, :, 1]
+            a = a.reshape(len(rows), -1).to(h.dtype)
+        else:
+            a = relu2(gu).to(h.dtype)
         out[rows] = (a.float() @ wdown[e].float().t()).to(h.dtype)
     return out
 
@@ -705,5 +774,57 @@ def gated_lru(ab, conv_w, conv_b, gates, gates_b, decay, state, conv,
         for i in range(n):
             S = a[i] * S + drive[i]
             out[row0 + i] = (S * y[i]).to(ab.dtype)
+        state[slot] = S
+    return out
+
+
+# ---- retention / rotary latent attention decoder on several streams ---------
+
+def stream_step(x, y, writes, mix, shared, embed, read, norm, store, dtype):
+    S = x.shape[1]
+    old = x
+    if embed is not None:
+        tokens, table = embed
+        old = table[tokens.long()].float()[:, None].expand(-1, S, -1)
+    new = old
+    if y is not None:
+        v = y.float()
+        if mix is not None:
+            top = mix.shape[1] - (shared is not None)
+            w = mix[:, :top, None]
+            v = (v.view(len(x), top, -1).masked_fill(w == 0, 0) * w).sum(1)
+            if shared is not None:
+                v = v + shared.float() * mix[:, top:]
+        out, m = writes[:S], writes[S:].view(S, S)
+        new = (old[:, :, None] * m[None, :, :, None]).sum(1) \
+            + out[None, :, None] * v[:, None]
+        if store:
+            x.copy_(new)
+    u = new.sum(1) if read is None else (new * read[None, :, None]).sum(1)
+    w, n, eps = norm
+    ms = u.pow(2).sum(-1, keepdim=True) / n
+    return (u / torch.sqrt(ms + eps) * w).to(dtype)
+
+
+def retention(ab, heads, dp, vp, dim, vdim, decay, table, eps, state,
+              segments, ctx):
+    M, H = ab.shape[0], heads
+    out = torch.zeros(M, H * vp, dtype=ab.dtype)
+    qk = _rotate(ab[:, : 2 * H * dp].reshape(M, 2 * H, dp), table)
+    q, k = qk[:, :H], qk[:, H:] * dim ** -0.5
+    v = ab[:, 2 * H * dp: 2 * H * dp + H * vp].float().view(M, H, vp)
+    gate = F.silu(ab[:, 2 * H * dp + H * vp:].float()).view(M, H, vp)
+    g = decay[0][:, None, None]
+    for row0, n, slot in zip(segments.row0.tolist(), segments.rows.tolist(),
+                             segments.slot.tolist()):
+        if n == 0:
+            continue
+        S = state[slot] * (int(ctx[row0]) > 1)         # [H, vp, dp]
+        for i in range(row0, row0 + n):
+            S = g * S + v[i, :, :, None] * k[i, :, None]
+            o = (S * q[i, :, None]).sum(-1)            # [H, vp]
+            ms = o.pow(2).sum(-1, keepdim=True) / vdim
+            y = o / torch.sqrt(ms + eps) * gate[i]
+            out[i] = y.reshape(-1).to(ab.dtype)
         state[slot] = S
     return out

@@ -6,12 +6,13 @@ The kernels are grouped into a few extensions, so that a process which
 needs one group does not have to compile the others:
 
     _hip_gemm      matrix products and gated units (every model)
-    _hip_residual  norms around an fp32 residual stream
+    _hip_residual  boundaries of fp32 residual streams, rotation tables
     _hip_latent    latent attention
     _hip_hybrid    attention over pages of keys and values, delta rules
     _hip_chunked   the same attention with capped scores, chunk by chunk
     _hip_experts   xIELU, routed experts
     _hip_lru       linear recurrent unit
+    _hip_retention retention
     _hip_ops       everything else
 
 DISTLLM_EXT=_hip_gemm,_hip_latent restricts a build to the named ones.
@@ -30,10 +31,11 @@ CSRC = Path(__file__).parent / "distllm_amd" / "ops" / "csrc"
 GROUPS = {
     "_hip_gemm": ["ext_gemm.cpp", "blt_gemm.cpp", "gemm.hip", "gemm8.hip",
                   "gemm16.hip", "decode_gemm.hip", "clamped_glu.hip",
-                  "gelu_rows.hip"],
+                  "gelu_rows.hip", "relu2.hip"],
     "_hip_latent": ["ext_latent.cpp", "latent_attention.hip",
                     "latent_decode.hip", "window_attention.hip"],
-    "_hip_residual": ["ext_residual.cpp", "residual_norms.hip"],
+    "_hip_residual": ["ext_residual.cpp", "residual_norms.hip", "streams.hip",
+                      "rotation.hip"],
     "_hip_hybrid": ["ext_hybrid.cpp", "chunk_attention.hip",
                     "sink_rows.hip", "sink_flash.hip", "delta_rule.hip",
                     "delta_chunk.hip", "delta_channel.hip"],
@@ -41,6 +43,7 @@ GROUPS = {
     "_hip_experts": ["ext_experts.cpp", "experts.hip", "expert_gemm16.hip",
                      "xielu.hip"],
     "_hip_lru": ["ext_lru.cpp", "lru.hip"],
+    "_hip_retention": ["ext_retention.cpp", "retention.hip"],
 }
 _taken = {s for group in GROUPS.values() for s in group}
 # *_hip.hip files are torch-hipify build artifacts — exclude them.

@@ -60,13 +60,21 @@ def mixed_config(**kw):
 
 class Case:
     """gain: in 16 bits smaller by default, as a norm of numbers that
-    happen to be small magnifies rounding."""
+    happen to be small magnifies rounding. Models of other designs have
+    their own `oracle` and `default_config`."""
+
+    oracle = oracle
+    TOL = TOL
+
+    @staticmethod
+    def default_config():
+        return mixed_config()
 
     def __init__(self, tmp, device, dtype, config=None, seed=0, gain=None,
                  edit=None):
-        self.config = config or mixed_config()
+        self.config = config or self.default_config()
         gain = gain or (1.0 if dtype == F32 else 0.7)
-        self.tensors = oracle.make_tensors(self.config, seed, gain)
+        self.tensors = self.oracle.make_tensors(self.config, seed, gain)
         if edit is not None:
             edit(self.tensors)
         self.device, self.dtype = device, dtype
@@ -91,8 +99,8 @@ class Case:
     def want(self, toks, config=None):
         key = (tuple(toks), json.dumps(config))
         if key not in self._want:
-            self._want[key] = oracle.forward(config or self.config,
-                                             self.tensors, toks)
+            self._want[key] = self.oracle.forward(config or self.config,
+                                                  self.tensors, toks)
         return self._want[key]
 
     def error(self, got, toks):
@@ -103,7 +111,7 @@ class Case:
 
     def passes(self, got, toks):
         err = self.error(got, toks)
-        assert err < TOL[self.dtype], (len(toks), err)
+        assert err < self.TOL[self.dtype], (len(toks), err)
 
 
 def check_whole(c: Case, n=90):
@@ -282,7 +290,7 @@ def check_greedy(c: Case, use_loop=False):
     for p, o in zip(prompts, outs):
         assert len(o) == 24
         gaps, scale = oracle_greedy(c, p, o)
-        assert max(gaps) < 3 * TOL[c.dtype] * scale, (len(p), gaps)
+        assert max(gaps) < 3 * c.TOL[c.dtype] * scale, (len(p), gaps)
 
 
 def check_long_decode(c: Case, prompt=20, new=200):
