@@ -204,7 +204,7 @@ def check_sink_and_gate(tmp, device, dtype):
 
     def edit(t):
         t["l0.mix.sink"] = torch.tensor([6.0, -30.0, 60.0]).to(BF16)
-        t["l0.mix.g"] *= 4
+        t["l0.mix.g"] *= 8
 
     c = Case(tmp, device, dtype, cfg, seed=75, edit=edit)
     toks = c.tokens(80, 5)
