@@ -41,7 +41,8 @@ def main() -> None:
                          "write (tokenizer + staging included); "
                          "decoders = prefill and decode of Kanotar "
                          "and Bufulorn layers beside llama layers of equal "
-                         "size, and of Tebasun beside Bufulorn layers")
+                         "size, and of Tebasun and Kedelorn beside "
+                         "layers of the closest of these")
     ap.add_argument("--docs-per-file", type=int, default=128)
     ap.add_argument("--pooler", type=str, default="mean",
                     choices=["mean", "last_token"])
@@ -247,15 +248,17 @@ def bench_generate(args) -> None:
 
 def bench_decoders(args) -> None:
     """Kanotar and Bufulorn layers beside llama layers of the same width,
-    heads and (active) feed-forward weights, and Tebasun layers beside
-    Bufulorn layers, through the same engine: tokens/s of prefilling a batch
-    of prompts and of decoding at a given context, both models in turn.
+    heads and (active) feed-forward weights, Tebasun layers beside Bufulorn
+    layers, and Kedelorn layers beside Bufulorn and Kanotar layers, through
+    the same engine: tokens/s of prefilling a batch of prompts and of
+    decoding at a given context, both models in turn.
     Random weights, synthetic tokens, one GPU."""
     from distllm_amd.engine import LLMEngine, SamplingParams
     from distllm_amd.engine.engine import _Seq
     from distllm_amd.models import ModelDims, build_model
-    from distllm_amd.models.config import (ExpertsDims, hybrid_preset,
-                                           layered_preset, looped_preset)
+    from distllm_amd.models.config import (ExpertsDims, GatedExpertsDims,
+                                           hybrid_preset, layered_preset,
+                                           looped_preset, streamed_preset)
 
     dev = "cuda:0"
     torch.manual_seed(5)
@@ -273,13 +276,26 @@ def bench_decoders(args) -> None:
 
     def bufulorn(hidden, heads, kv, ff, chunk, order="A", **kw):
         # two matrices per dense feed-forward where llama has three
-        return hybrid_preset(args.layers, hidden, V, heads, kv, 128,
-                             ff * 3 // 2, chunk, order=order, **kw)
+        routed = kw.pop("routed", False)
+        d = hybrid_preset(args.layers, hidden, V, heads, kv, 128,
+                          max(ff * 3 // 2, 1), chunk, order=order, **kw)
+        for layer in d.layers if routed else ():
+            layer.mlp = kw["experts"]
+        return d
 
     def tebasun(hidden, heads, kv, ff, order, **kw):
         # half of the heads in each of two mixers side by side
         return looped_preset(kw.pop("layers", args.layers), hidden, V, heads,
                              kv, 128, ff, order, **kw)
+
+    def kedelorn(hidden, heads, kv_rank, order, mlp=None, **kw):
+        return streamed_preset(args.layers, hidden, V, heads, 128, kv_rank,
+                               mlp, order, **kw)
+
+    def mixers(dims):
+        for layer in dims.layers:
+            layer.mlp = None
+        return dims
 
     # name: (model, the other one, [(prompts, prompt len)],
     #        [(batch, context)])
@@ -326,6 +342,22 @@ def bench_decoders(args) -> None:
             tebasun(2048, 16, 8, 8192, "PPR", layers=args.layers * 2 // 3,
                     loop=(0, args.layers - args.layers * 2 // 3, 2)),
             bufulorn(2048, 16, 4, 8192, 8192, "AD"), *some),
+        "4096x32h retention": (
+            kedelorn(4096, 32, 512, "R"),
+            mixers(bufulorn(4096, 32, 32, 0, 8192, "D")),
+            some[0] + [(2, 8000)], some[1]),
+        "4096x32h rotary latent": (
+            kedelorn(4096, 32, 512, "L"),
+            mixers(kanotar(4096, 32, 1536, 512, 14336, 8192)),
+            some[0] + [(2, 8000)], some[1] + [(32, 8000)]),
+        # two matrices per expert where Bufulorn has three: the same active
+        # weights, and as many in all
+        "2048x16h streams": (
+            kedelorn(2048, 16, 256, "RL", GatedExpertsDims(
+                ff=1280, experts=76, top=8, shared=2048)),
+            bufulorn(2048, 16, 4, 8192, 8192, "DA", routed=True,
+                     experts=ExpertsDims(ff=1024, experts=64, top=8,
+                                         groups=8, keep=4)), *some),
     }
     params = SamplingParams(temperature=0.0, min_p=0.0, max_tokens=10 ** 6)
     rows = []

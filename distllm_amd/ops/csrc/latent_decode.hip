@@ -19,7 +19,8 @@
 // as columns, so softmax state and rescaling are lane-local.
 //
 // Cache rows and queries have RR = R + ROT numbers, of which all take part in
-// the scores and the first R are the value.
+// the scores and the first R are the value. The others need no transposed
+// copy: they go to LDS directly, while the tile before is weighted.
 #include "common.h"
 
 #define PBLK 16
@@ -68,13 +69,15 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
                      const unsigned short* __restrict__ gate, int ld_gate) {
   constexpr int NT = 64 * HG * KS;
   constexpr int RR = R + ROT;
-  constexpr int UNITS = RR;  // a unit: 4 keys x 8 columns
+  constexpr int UNITS = R;  // a unit: 4 keys x 8 latent columns
   constexpr int UPT = (UNITS + NT - 1) / NT;
-  constexpr int SW = RR % 128 == 0 ? 15 : 7;
-  constexpr int CT = KT * RR * 2;       // LDS offset of the transposed copy
+  constexpr int SW = R % 128 == 0 ? 15 : 7;
+  constexpr int CT = KT * R * 2;        // LDS offset of the transposed copy
   constexpr int SC = CT + R * 72;       // LDS offset of the scores
   constexpr int RSPLIT = KS / 2;       // column parts, besides key halves
-  constexpr int QS = RR / 32 / RSPLIT;  // score steps of a wave
+  constexpr int RO = SC + HG * RSPLIT * 16 * SROW * 4;  // of the key parts
+  constexpr int QS = R / 32 / RSPLIT;  // score steps of a wave
+  constexpr int TS = ROT / 32 / RSPLIT;  // and those behind the latent
   constexpr int OB = R / 16 / KS;      // output blocks of a wave
   static_assert(KS == 2 || KS == 4, "two key halves");
 
@@ -125,10 +128,9 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
 #pragma unroll
         for (int j = 0; j < 4; ++j) {
           const int key = kg * 4 + j;
-          *reinterpret_cast<i32x4*>(smem + key * (RR * 2) +
+          *reinterpret_cast<i32x4*>(smem + key * (R * 2) +
                                     ((c ^ (key & SW)) * 16)) = kv[i][j];
         }
-        if (ROT > 0 && c >= R / 8) continue;  // no value
 #pragma unroll
         for (int w = 0; w < 4; ++w) {
           i32x2 even, odd;
@@ -149,18 +151,42 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
     }
   };
 
-  int page = 0;
+  // key parts: four waves copy eight keys each
+  auto part_page = [&](int t) {
+    return bt[min(t * (KT / PBLK) + (wid >> 1), last_page)];
+  };
+  auto stage_part = [&](int page) {
+    static_assert(ROT == 0 || ROT == 64, "eight 16-byte pieces per key");
+    if (wid >= 4) return;
+    const int key = wid * 8 + (lane >> 3);
+    const unsigned short* src = cache +
+                                ((long)page * PBLK + (key & 15)) * RR + R +
+                                ((lane & 7) ^ (key & 7)) * 8;
+    auto dst = (__attribute__((address_space(3))) unsigned int*)(
+        smem + RO + wid * 1024 + lane * 16);
+    __builtin_amdgcn_global_load_lds(
+        (const __attribute__((address_space(1))) unsigned int*)src, dst, 16,
+        0, 0);
+  };
+
+  int page = 0, ppage = 0;
   if (ts < te) {
     issue(page_of(ts));
     page = page_of(min(ts + 1, te - 1));
+    if (ROT > 0) {
+      stage_part(part_page(ts));
+      ppage = part_page(min(ts + 1, te - 1));
+    }
   }
-  bf16x8 qf[QS];
+  bf16x8 qf[QS + TS];
   {
-    const unsigned short* qr = q + ((long)row * H + (live ? head : 0)) * RR +
-                               rhalf * (QS * 32) + g * 8;
+    const unsigned short* qr =
+        q + ((long)row * H + (live ? head : 0)) * RR + g * 8;
 #pragma unroll
-    for (int s = 0; s < QS; ++s) {
-      s16x8 v = *reinterpret_cast<const s16x8*>(qr + s * 32);
+    for (int s = 0; s < QS + TS; ++s) {
+      s16x8 v = *reinterpret_cast<const s16x8*>(
+          qr + (s < QS ? (rhalf * QS + s) * 32
+                       : R + (rhalf * TS + s - QS) * 32));
       if (!live) v = (s16x8)(short)0;
       qf[s] = __builtin_bit_cast(bf16x8, v);
     }
@@ -176,6 +202,7 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
 
   for (int t = ts; t < te; ++t) {
     __syncthreads();  // every wave is done with the previous tile
+    if (ROT > 0) asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
     stage();
     if (t + 1 < te) {
       issue(page);
@@ -190,17 +217,29 @@ latent_decode_kernel(const unsigned short* __restrict__ q,
 #pragma unroll
     for (int s = 0; s < QS; ++s) {
       const int chunk = (rhalf * QS + s) * 4 + g;
-      const char* a = smem + (khalf * 16 + i16) * (RR * 2) +
+      const char* a = smem + (khalf * 16 + i16) * (R * 2) +
                       ((chunk ^ (i16 & SW)) * 16);
       const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(a);
       sa[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
           k0, qf[s], sa[s & 1], 0, 0, 0);
     }
 #pragma unroll
+    for (int s = 0; s < TS; ++s) {
+      const int chunk = (rhalf * TS + s) * 4 + g;
+      const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(
+          smem + RO + (khalf * 16 + i16) * 128 + ((chunk ^ (i16 & 7)) * 16));
+      sa[s & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+          k0, qf[QS + s], sa[s & 1], 0, 0, 0);
+    }
+#pragma unroll
     for (int r = 0; r < 4; ++r) sa[0][r] += sa[1][r];
     *reinterpret_cast<f32x4*>(scores + rhalf * (16 * SROW) + khalf * 16 +
                               g * 4) = sa[0];
     __syncthreads();
+    if (ROT > 0 && t + 1 < te) {
+      stage_part(ppage);
+      ppage = part_page(min(t + 2, te - 1));
+    }
 
     // weights of all 32 keys for my head: lane group g has keys g*8 .. + 7
     float p[8];

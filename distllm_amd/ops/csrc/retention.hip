@@ -10,7 +10,7 @@
 // kept as [slots, H, vp, dp] in fp32, and everything that enters it is fp32.
 //
 //   retention_scan_kernel   token by token, any type, short segments
-//   retention_chunk_kernel  long segments, 32 rows at a time on the fp32 MFMA
+//   retention_chunk_kernel  long segments, 32 rows at a time on the MFMA
 //   retention_join_kernel   states between the pieces of a long segment
 //
 // With n the rows of a chunk and S the state before it (rows t, s from 0):
@@ -21,7 +21,6 @@
 #include "common.h"
 
 #define CH 32    // rows of a chunk
-#define TROW 36  // padded row of a chunk x chunk matrix
 #define PROW 20  // padded row of a 16 x 16 partial sum
 
 extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -49,12 +48,11 @@ __device__ __forceinline__ float gate_silu(float z) {
 template <typename T>
 __device__ __forceinline__ float rotated(const T* src, int c, int half,
                                          const float* cs) {
-  const float x = to_f(src[c]);
-  if (c >= 2 * half) return x;
-  const bool low = c < half;
-  const int i = low ? c : c - half;
-  const float y = to_f(src[low ? c + half : i]);
-  return x * cs[i * 2] + (low ? -y : y) * cs[i * 2 + 1];
+  const bool turn = c < 2 * half, low = c < half;
+  const int i = !turn ? 0 : low ? c : c - half;  // its pair
+  const float x = to_f(src[c]), y = to_f(src[low ? c + half : i]);
+  const float2 t = reinterpret_cast<const float2*>(cs)[i];
+  return turn ? x * t.x + (low ? -y : y) * t.y : x;
 }
 
 // ---- token by token -----------------------------------------------------------
@@ -66,7 +64,7 @@ __device__ __forceinline__ float rotated(const T* src, int c, int half,
 #define TT 16
 
 template <typename T, int LPC, int NCOL>
-__global__ void __launch_bounds__(1024)
+__global__ void __launch_bounds__(1024, 4)
 retention_scan_kernel(const RetentionArgs<T> a, int max_rows) {
   constexpr int dp = LPC * 16;
   __shared__ float red[2][16];
@@ -83,63 +81,68 @@ retention_scan_kernel(const RetentionArgs<T> a, int max_rows) {
   float* st = a.state + ((long)a.seg_slot[seg] * a.H + head) * a.vp * dp +
               part * 4;
 
+  // number u of the queries and keys of rows t0 ..
+  auto input = [&](int t0, int u) {
+    const long row = row0 + t0 + u / (2 * dp);
+    const int which = u / dp % 2;
+    const float x = rotated(a.ab + row * a.ld + (which * a.H + head) * dp,
+                            u % dp, a.half, a.table + row * a.half * 2);
+    return which == 1 ? x * a.kscale : x;
+  };
+  // the first inputs are on their way before the state
+  const int first = min(TT, n) * 2 * dp;
+  const float x0 = (int)threadIdx.x < first ? input(0, threadIdx.x) : 0.f;
   float S[NCOL][16];
   const bool fresh = a.ctx[row0] <= 1;
 #pragma unroll
   for (int c = 0; c < NCOL; ++c)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      f32x4 x = {0.f, 0.f, 0.f, 0.f};
-      if (!fresh)
-        x = *reinterpret_cast<const f32x4*>(
-            st + (long)(col0 + c * cstep) * dp + i * LPC * 4);
+      const f32x4 x = *reinterpret_cast<const f32x4*>(
+          st + (long)(col0 + c * cstep) * dp + i * LPC * 4);
 #pragma unroll
-      for (int e = 0; e < 4; ++e) S[c][i * 4 + e] = x[e];
+      for (int e = 0; e < 4; ++e) S[c][i * 4 + e] = fresh ? 0.f : x[e];
     }
+  if ((int)threadIdx.x < first) (&qk[0][0][0])[threadIdx.x] = x0;
 
   for (int t0 = 0; t0 < n; t0 += TT) {
     const int cnt = min(TT, n - t0);
     if (t0 > 0) __syncthreads();  // the rows before are consumed
-    for (int u = threadIdx.x; u < cnt * 2 * dp; u += blockDim.x) {
-      const int t = u / (2 * dp), which = u / dp % 2, c = u % dp;
-      const long row = row0 + t0 + t;
-      const float x = rotated(a.ab + row * a.ld + (which * a.H + head) * dp,
-                              c, a.half, a.table + row * a.half * 2);
-      qk[t][which][c] = which == 1 ? x * a.kscale : x;
-    }
+    for (int u = threadIdx.x + (t0 == 0 ? blockDim.x : 0); u < cnt * 2 * dp;
+         u += blockDim.x)
+      (&qk[0][0][0])[u] = input(t0, u);
     __syncthreads();
     for (int t = 0; t < cnt; ++t) {
       const long row = row0 + t0 + t;
       const T* vr = a.ab + row * a.ld + 2 * a.H * dp + head * a.vp;
-      float v[NCOL], o[NCOL];
+      float v[NCOL], o[NCOL], gt[NCOL];
 #pragma unroll
-      for (int c = 0; c < NCOL; ++c) v[c] = to_f(vr[col0 + c * cstep]);
-      float q[16], k[16];
+      for (int c = 0; c < NCOL; ++c) {
+        v[c] = to_f(vr[col0 + c * cstep]);
+        gt[c] = to_f(vr[a.H * a.vp + col0 + c * cstep]);
+        o[c] = 0.f;
+      }
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const int at = (i * LPC + part) * 4;
-        const f32x4 x = *reinterpret_cast<const f32x4*>(&qk[t][0][at]);
-        const f32x4 z = *reinterpret_cast<const f32x4*>(&qk[t][1][at]);
+        const f32x4 q = *reinterpret_cast<const f32x4*>(&qk[t][0][at]);
+        const f32x4 k = *reinterpret_cast<const f32x4*>(&qk[t][1][at]);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) {
-          q[i * 4 + e] = x[e];
-          k[i * 4 + e] = z[e];
-        }
+        for (int c = 0; c < NCOL; ++c)
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            float& s = S[c][i * 4 + e];
+            s = g * s + k[e] * v[c];
+            o[c] += s * q[e];
+          }
       }
       float ss = 0.f;
 #pragma unroll
       for (int c = 0; c < NCOL; ++c) {
-        float r = 0.f;
-#pragma unroll
-        for (int e = 0; e < 16; ++e) {
-          S[c][e] = g * S[c][e] + k[e] * v[c];
-          r += S[c][e] * q[e];
-        }
 #pragma unroll
         for (int off = LPC / 2; off > 0; off >>= 1)
-          r += __shfl_xor(r, off, 64);
-        o[c] = r;
-        ss += part == 0 ? r * r : 0.f;
+          o[c] += __shfl_xor(o[c], off, 64);
+        ss += part == 0 ? o[c] * o[c] : 0.f;
       }
       ss = wave_reduce_sum(ss);
       if (lane == 0) red[t & 1][wid] = ss;
@@ -150,10 +153,8 @@ retention_scan_kernel(const RetentionArgs<T> a, int max_rows) {
       if (part == 0) {
 #pragma unroll
         for (int c = 0; c < NCOL; ++c) {
-          const int j = col0 + c * cstep;
-          const float gt = to_f(vr[a.H * a.vp + j]);
-          from_f(a.y + (row * a.H + head) * a.vp + j,
-                 o[c] * inv * gate_silu<T>(gt));
+          from_f(a.y + (row * a.H + head) * a.vp + col0 + c * cstep,
+                 o[c] * inv * gate_silu<T>(gt[c]));
         }
       }
     }
@@ -171,47 +172,106 @@ retention_scan_kernel(const RetentionArgs<T> a, int max_rows) {
 }
 
 // ---- long segments --------------------------------------------------------------
-// Operands of the 16 x 16 x 4 product: step r of a block of 16 inner indices
-// takes those with number g * 4 + r (g = lane / 16), which lets a lane read
-// operands as float4 and lets an accumulator (rows g * 4 + r) be the right
-// operand of the next product as it is.
-__device__ __forceinline__ f32x4 mfma4(float a, float b, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
+// The products run on the bf16 MFMA without giving up fp32: a number is the
+// sum of three bf16 numbers, its leading bits, the next and the last eight of
+// 24 (values are bf16 already). A product of two such sums takes the six
+// products of parts that reach beyond the last bit.
+typedef __attribute__((ext_vector_type(8))) __bf16 bf16x8;
+
+struct Parts {
+  unsigned int p[3];
+};
+
+// two neighbours; every part is packed like two bf16 in memory
+__device__ __forceinline__ Parts split2(float x0, float x1) {
+  Parts out;
+#pragma unroll
+  for (int i = 0; i < 3; ++i) {
+    const unsigned int u0 = __float_as_uint(x0), u1 = __float_as_uint(x1);
+    out.p[i] = __builtin_amdgcn_perm(u1, u0, 0x07060302);
+    x0 -= __uint_as_float(u0 & 0xffff0000u);
+    x1 -= __uint_as_float(u1 & 0xffff0000u);
+  }
+  return out;
+}
+
+__device__ __forceinline__ f32x4 mfma_bf(bf16x8 a, bf16x8 b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+
+// a . b of two numbers in parts, smallest terms first
+__device__ __forceinline__ f32x4 mfma_parts(const bf16x8 (&a)[3],
+                                            const bf16x8 (&b)[3], f32x4 c) {
+  c = mfma_bf(a[2], b[0], c);
+  c = mfma_bf(a[0], b[2], c);
+  c = mfma_bf(a[1], b[1], c);
+  c = mfma_bf(a[1], b[0], c);
+  c = mfma_bf(a[0], b[1], c);
+  return mfma_bf(a[0], b[0], c);
 }
 
 __device__ __forceinline__ float exp2_of(float x) {
   return __builtin_amdgcn_exp2f(x);
 }
 
+// Place of number d of a row of keys or queries in LDS: within 32 numbers,
+// those that a lane group g finds in two accumulators of the state (4 g ..
+// 4 g + 3 and 16 + 4 g ..) are neighbours, so that the state's accumulators
+// are the right operand of the next product as they are.
+__device__ __forceinline__ int lds_place(int d) {
+  const int w = d & 31, h = w >> 4;
+  return (d & ~31) + ((w & 15) >> 2) * 8 + h * 4 + (w & 3);
+}
+
 // pieces [P, 5]: segment, first row in it, rows, number, pieces of the
-// segment. One workgroup per (piece, head), a wave for each 16 value columns
-// (its part of the state, DP x 16, is DP / 16 accumulators).
+// segment. One workgroup per (piece, head), a wave for each 32 value columns
+// (its part of the state, DP x 32, is DP / 8 accumulators).
 //   LOCAL  the piece's state from zeros, to between[piece]; not for the last
 //          piece of a segment
 //   else   the outputs, from the slot's state or (several pieces) from
 //          between[piece]; the last piece writes the slot
-// Rotated queries and keys of a chunk are staged in LDS, those of the next
-// chunk are on their way in registers meanwhile. For the scores the waves
-// split the inner dimension; their sums meet in LDS. VEC: half is a multiple
-// of 8, so that rotation partners are eight in a row, too.
-template <int DP, int NW, bool LOCAL, bool VEC>
-__global__ void __launch_bounds__(NW * 64, NW >= 8 ? 4 : 2)
+// The rotated queries and keys of a chunk are kept in parts in LDS, by rows
+// and, weighted with their decay to the chunk's end, keys by numbers; the
+// next chunk is on its way in registers meanwhile. For the scores the waves
+// split the inner dimension; their sums meet in LDS.
+//
+// A thread's unit of keys and queries is four rows by four numbers: two
+// neighbours and their rotation partners, or four that do not rotate. VEC:
+// half is even; else units are read number by number.
+template <int DP, int VP>
+struct ChunkLds {
+  static constexpr int NW = VP / 32;
+  static constexpr int KJ = DP / 32;
+  static constexpr int NP = NW < KJ ? NW : KJ;  // waves that form scores
+  static constexpr int ROW_B = DP * 2 + 16;     // a row of one part
+  static constexpr int Q_B = 3 * CH * ROW_B;
+  static constexpr int T_B = 3 * DP * CH * 2;   // by numbers
+  static constexpr int K_B = Q_B > T_B ? Q_B : T_B;
+  static constexpr int P_ROW = CH * 2 + 16;
+  static constexpr int P_B = 3 * CH * P_ROW;
+  static constexpr int O_ROW = VP + 4;          // floats
+  static constexpr int S_B = NP * 3 * 16 * PROW * 4;
+  static constexpr int O_B = CH * O_ROW * 4;
+  static constexpr int BYTES = Q_B + K_B + P_B + (S_B > O_B ? S_B : O_B);
+};
+
+template <int DP, int VP, bool LOCAL, bool VEC>
+__global__ void __launch_bounds__(VP * 2, DP <= 128 && VP > 64 ? 2 : 1)
 retention_chunk_kernel(const RetentionArgs<unsigned short> a,
                        const int* __restrict__ pieces,
                        float* __restrict__ between) {
   typedef unsigned short T;
-  constexpr int VP = NW * 16, NT = NW * 64;
-  constexpr int ROW = DP + 4, OROW = VP + 4;
-  constexpr int KT = DP / 16;
-  constexpr int NP = NW < KT ? NW : KT;       // waves that form scores
-  constexpr int WHICH = LOCAL ? 1 : 2;        // keys, then queries
-  constexpr int SLOTS = CH * WHICH * KT;      // of 16 numbers
-  constexpr int NS = (SLOTS + NT - 1) / NT;
-  float* Kl = reinterpret_cast<float*>(smem);
-  float* Ql = Kl + CH * ROW;
-  float* Pl = Ql + CH * ROW;                  // [CH][TROW]
-  float* part = Pl + CH * TROW;               // [NP][3][16][PROW]
-  float* Ol = part;                           // [CH][OROW], later
+  typedef ChunkLds<DP, VP> L;
+  constexpr int NW = L::NW, NT = NW * 64, KT = DP / 16, KJ = L::KJ;
+  constexpr int NP = L::NP;
+  constexpr int UNITS = CH / 4 * (DP / 4);
+  constexpr int NS = (UNITS + NT - 1) / NT;
+  constexpr int LPR = VP / 16;   // lanes that share an output row
+  char* Kl = smem;               // rows [3][CH], then numbers [3][DP]
+  char* Ql = Kl + (LOCAL ? L::T_B : L::K_B);
+  char* Pl = Ql + L::Q_B;
+  float* part = reinterpret_cast<float*>(Pl + L::P_B);  // [NP][3][16][PROW]
+  float* Ol = part;                                     // later
 
   const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
   const int i16 = lane & 15, g = lane >> 4;
@@ -221,124 +281,184 @@ retention_chunk_kernel(const RetentionArgs<unsigned short> a,
   if (LOCAL && number + 1 == count) return;
   const long row0 = a.seg_row0[seg] + pc[1];
   const int nch = (n + CH - 1) / CH;
-  const int col = wid * 16 + i16;
   const float lg = a.decay[a.H + head];
   const int at_q = head * DP, at_k = (a.H + head) * DP;
   const int at_v = 2 * a.H * DP + head * VP, at_g = at_v + a.H * VP;
 
-  // slot number u: 16 numbers of a row of keys or queries, as two groups of
-  // eight that rotate with each other, or two that do not rotate
-  s16x8 ra[NS], rb[NS];
-  float cs[NS][VEC ? 16 : 1];
-  unsigned short vr[2][4];
-  s16x8 gr;
-  auto fetch = [&](int c) {
-    const int cnt = min(CH, n - c * CH);
-    const long r0 = row0 + c * CH;
+  // numbers d[0], d[0] + 1, d[1], d[1] + 1 of rows t .. t + 3 of the chunk
+  struct Unit {
+    int d[2], t;
+    bool turn, live;
+  };
+  auto unit = [&](int i) {
+    const int u = tid + i * NT, q = u % (DP / 4) * 2;
+    Unit x;
+    x.t = u / (DP / 4) * 4;
+    x.live = UNITS % NT == 0 || u < UNITS;
     if constexpr (VEC) {
+      x.turn = q < a.half;
+      x.d[0] = x.turn ? q : q + a.half;
+      x.d[1] = x.turn ? q + a.half : q + DP / 2;
+    } else {
+      x.turn = true;
+      x.d[0] = q;
+      x.d[1] = q + DP / 2;
+    }
+    return x;
+  };
+  unsigned int rk[NS][4][2], rq[NS][4][2];
+  f32x4 cs[NS][4];
+  auto fetch = [&](int c) {
+    if constexpr (VEC) {
+      const int cnt = min(CH, n - c * CH);
 #pragma unroll
       for (int i = 0; i < NS; ++i) {
-        const int u = tid + i * NT;
-        if (SLOTS % NT != 0 && u >= SLOTS) break;
-        const int j = u % KT, which = u / KT % WHICH;
-        const long row = r0 + min(u / (KT * WHICH), cnt - 1);
-        const T* src = a.ab + row * a.ld + (which == 0 ? at_k : at_q);
-        const bool turn = j * 8 < a.half;
-        const int x = turn ? j * 8 : j * 16;
-        ra[i] = *reinterpret_cast<const s16x8*>(src + x);
-        rb[i] = *reinterpret_cast<const s16x8*>(src + x +
-                                                (turn ? a.half : 8));
-        if (turn) {
-          const float* t = a.table + (row * a.half + j * 8) * 2;
-          load8<float>(t, cs[i]);
-          load8<float>(t + 8, cs[i] + 8);
+        const Unit x = unit(i);
+        if (!x.live) break;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          const long row = row0 + c * CH + min(x.t + e, cnt - 1);
+          const T* src = a.ab + row * a.ld;
+#pragma unroll
+          for (int j = 0; j < 2; ++j) {
+            rk[i][e][j] = *reinterpret_cast<const unsigned int*>(
+                src + at_k + x.d[j]);
+            if (!LOCAL)
+              rq[i][e][j] = *reinterpret_cast<const unsigned int*>(
+                  src + at_q + x.d[j]);
+          }
+          if (x.turn)
+            cs[i][e] = *reinterpret_cast<const f32x4*>(
+                a.table + (row * a.half + x.d[0]) * 2);
         }
       }
     }
-#pragma unroll
-    for (int m = 0; m < 2; ++m)
-#pragma unroll
-      for (int r = 0; r < 4; ++r)
-        vr[m][r] = a.ab[(r0 + min(m * 16 + g * 4 + r, cnt - 1)) * a.ld +
-                        at_v + col];
-    if (!LOCAL)
-      gr = *reinterpret_cast<const s16x8*>(
-          a.ab + (r0 + min(tid / (VP / 8), cnt - 1)) * a.ld + at_g +
-          tid % (VP / 8) * 8);
   };
-  auto stage = [&](int c) {
+  // row e of unit i, rotated; zeros behind the end
+  auto turned = [&](int c, int i, const Unit& x, int e, bool key, float* z) {
     const int cnt = min(CH, n - c * CH);
+    if constexpr (VEC) {
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        const unsigned int r = key ? rk[i][e][j] : rq[i][e][j];
+        z[j * 2] = __uint_as_float(r << 16);
+        z[j * 2 + 1] = __uint_as_float(r & 0xffff0000u);
+      }
+      if (x.turn)
+#pragma unroll
+        for (int j = 0; j < 2; ++j) {
+          const float p = z[j], q = z[2 + j];
+          const float cv = cs[i][e][2 * j], sv = cs[i][e][2 * j + 1];
+          z[j] = p * cv - q * sv;
+          z[2 + j] = q * cv + p * sv;
+        }
+    } else {
+      const long row = row0 + c * CH + min(x.t + e, cnt - 1);
+      const T* src = a.ab + row * a.ld + (key ? at_k : at_q);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        z[j] = rotated(src, x.d[j >> 1] + (j & 1), a.half,
+                       a.table + row * a.half * 2);
+    }
+    const float f = x.t + e >= cnt ? 0.f : key ? a.kscale : 1.f;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) z[j] *= f;
+  };
+  float kz[NS][4][4];  // the chunk's keys
+  auto stage = [&](int c) {
 #pragma unroll
     for (int i = 0; i < NS; ++i) {
-      const int u = tid + i * NT;
-      if (SLOTS % NT != 0 && u >= SLOTS) break;
-      const int j = u % KT, which = u / KT % WHICH, t = u / (KT * WHICH);
-      float* dst = (which == 0 ? Kl : Ql) + t * ROW;
-      float z[16];
-      int x = j * 16, y = j * 16 + 8;
-      if constexpr (VEC) {
-        bf8_to_f32(ra[i], z);
-        bf8_to_f32(rb[i], z + 8);
-        if (j * 8 < a.half) {
-          x = j * 8;
-          y = x + a.half;
+      const Unit x = unit(i);
+      if (!x.live) break;
 #pragma unroll
-          for (int e = 0; e < 8; ++e) {
-            const float p = z[e], q = z[8 + e];
-            z[e] = p * cs[i][2 * e] - q * cs[i][2 * e + 1];
-            z[8 + e] = q * cs[i][2 * e] + p * cs[i][2 * e + 1];
+      for (int e = 0; e < 4; ++e) {
+        turned(c, i, x, e, true, kz[i][e]);
+        if constexpr (!LOCAL) {
+          float z[4];
+          turned(c, i, x, e, false, z);
+#pragma unroll
+          for (int j = 0; j < 2; ++j) {
+            char* dst = Kl + (x.t + e) * L::ROW_B + lds_place(x.d[j]) * 2;
+            const Parts k = split2(kz[i][e][j * 2], kz[i][e][j * 2 + 1]);
+            const Parts q = split2(z[j * 2], z[j * 2 + 1]);
+#pragma unroll
+            for (int p = 0; p < 3; ++p) {
+              const int at = p * CH * L::ROW_B;
+              *reinterpret_cast<unsigned int*>(dst + at) = k.p[p];
+              *reinterpret_cast<unsigned int*>(dst + (Ql - Kl) + at) = q.p[p];
+            }
           }
         }
-      } else {
-        const long row = row0 + c * CH + min(t, cnt - 1);
-        const T* src = a.ab + row * a.ld + (which == 0 ? at_k : at_q);
-#pragma unroll
-        for (int e = 0; e < 16; ++e)
-          z[e] = rotated(src, x + e, a.half, a.table + row * a.half * 2);
-      }
-      // rows behind the end count for nothing
-      const float f = t >= cnt ? 0.f : which == 0 ? a.kscale : 1.f;
-#pragma unroll
-      for (int e = 0; e < 16; ++e) z[e] *= f;
-#pragma unroll
-      for (int e = 0; e < 8; e += 4) {
-        *reinterpret_cast<f32x4*>(dst + x + e) =
-            f32x4{z[e], z[e + 1], z[e + 2], z[e + 3]};
-        *reinterpret_cast<f32x4*>(dst + y + e) =
-            f32x4{z[8 + e], z[9 + e], z[10 + e], z[11 + e]};
       }
     }
   };
+  // keys by numbers, eight rows in a 16-byte piece, weighted with
+  // g^(cnt-1-s)
+  auto stage_numbers = [&](int cnt) {
+#pragma unroll
+    for (int i = 0; i < NS; ++i) {
+      const Unit x = unit(i);
+      if (!x.live) break;
+      float w[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        w[e] = exp2_of(lg * max(cnt - 1 - x.t - e, 0));
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int d = x.d[j >> 1] + (j & 1);
+        const Parts lo = split2(kz[i][0][j] * w[0], kz[i][1][j] * w[1]);
+        const Parts hi = split2(kz[i][2][j] * w[2], kz[i][3][j] * w[3]);
+        char* dst = Kl + d * (CH * 2) +
+                    (((x.t >> 3) ^ ((d >> 2) & 3)) * 16) + (x.t & 4) * 2;
+#pragma unroll
+        for (int p = 0; p < 3; ++p)
+          *reinterpret_cast<i32x2*>(dst + p * DP * (CH * 2)) =
+              i32x2{(int)lo.p[p], (int)hi.p[p]};
+      }
+    }
+  };
+  auto row_frags = [&](const char* base, int t, int j, bf16x8 (&f)[3]) {
+#pragma unroll
+    for (int p = 0; p < 3; ++p)
+      f[p] = *reinterpret_cast<const bf16x8*>(
+          base + (p * CH + t) * L::ROW_B + j * 64 + g * 16);
+  };
 
-  f32x4 S[KT];
-  const long own = ((long)piece * a.H + head) * VP + col;
-  float* slot =
-      a.state + (((long)a.seg_slot[seg] * a.H + head) * VP + col) * DP + g * 4;
+  f32x4 S[KT][2];
+  const long own = ((long)piece * a.H + head) * VP + wid * 32 + i16;
+  float* slot = a.state +
+                (((long)a.seg_slot[seg] * a.H + head) * VP + wid * 32 + i16) *
+                    DP + g * 4;
   const float* from = count > 1 ? between + own * DP + g * 4 : slot;
   const bool zero = LOCAL || (count == 1 && a.ctx[row0] <= 1);
 #pragma unroll
-  for (int k = 0; k < KT; ++k) {
-    S[k] = (f32x4)0.f;
-    if (!zero) S[k] = *reinterpret_cast<const f32x4*>(from + k * 16);
-  }
-  // weights of this lane's rows m * 16 + g * 4 + r (chunks of 32 rows)
-  const float glast = exp2_of(lg * CH);
+  for (int k = 0; k < KT; ++k)
+#pragma unroll
+    for (int ct = 0; ct < 2; ++ct) {
+      S[k][ct] = (f32x4)0.f;
+      if (!zero)
+        S[k][ct] =
+            *reinterpret_cast<const f32x4*>(from + ct * 16 * DP + k * 16);
+    }
 
   fetch(0);
   for (int c = 0; c < nch; ++c) {
     const int cnt = min(CH, n - c * CH);
     if (LOCAL && c > 0) __syncthreads();  // the chunk before is consumed
     stage(c);
-    float v[2][4], gt[8];
-#pragma unroll
-    for (int m = 0; m < 2; ++m)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) v[m][r] = bf2f(vr[m][r]);
-    if (!LOCAL) bf8_to_f32(gr, gt);
+    if (LOCAL) stage_numbers(cnt);
     __syncthreads();
+    T vr[2][8];  // values of my columns, rows g * 8 ..
+#pragma unroll
+    for (int ct = 0; ct < 2; ++ct)
+#pragma unroll
+      for (int e = 0; e < 8; ++e)
+        vr[ct][e] = a.ab[(row0 + c * CH + min(g * 8 + e, cnt - 1)) * a.ld +
+                         at_v + wid * 32 + ct * 16 + i16];
     if (c + 1 < nch) fetch(c + 1);
 
-    f32x4 out[2];
+    s16x8 gr[2];
+    f32x4 out[2][2];
     if constexpr (!LOCAL) {
       // my part of q_t.k_s: tiles (0, 0), (1, 0), (1, 1)
       if (wid < NP) {
@@ -346,20 +466,16 @@ retention_chunk_kernel(const RetentionArgs<unsigned short> a,
 #pragma unroll
         for (int i = 0; i < 3; ++i) p[i] = (f32x4)0.f;
 #pragma unroll
-        for (int kt = 0; kt < KT / NP; ++kt) {
-          f32x4 q[2], k[2];
+        for (int jj = 0; jj < KJ / NP; ++jj) {
+          bf16x8 q[2][3], k[2][3];
 #pragma unroll
           for (int m = 0; m < 2; ++m) {
-            const int at = (m * 16 + i16) * ROW + (kt * NP + wid) * 16 + g * 4;
-            q[m] = *reinterpret_cast<const f32x4*>(Ql + at);
-            k[m] = *reinterpret_cast<const f32x4*>(Kl + at);
+            row_frags(Ql, m * 16 + i16, jj * NP + wid, q[m]);
+            row_frags(Kl, m * 16 + i16, jj * NP + wid, k[m]);
           }
-#pragma unroll
-          for (int r = 0; r < 4; ++r) {
-            p[0] = mfma4(q[0][r], k[0][r], p[0]);
-            p[1] = mfma4(q[1][r], k[0][r], p[1]);
-            p[2] = mfma4(q[1][r], k[1][r], p[2]);
-          }
+          p[0] = mfma_parts(q[0], k[0], p[0]);
+          p[1] = mfma_parts(q[1], k[0], p[1]);
+          p[2] = mfma_parts(q[1], k[1], p[2]);
         }
 #pragma unroll
         for (int i = 0; i < 3; ++i)
@@ -369,85 +485,151 @@ retention_chunk_kernel(const RetentionArgs<unsigned short> a,
       }
       // Q S
 #pragma unroll
-      for (int m = 0; m < 2; ++m) out[m] = (f32x4)0.f;
+      for (int m = 0; m < 2; ++m)
 #pragma unroll
-      for (int k = 0; k < KT; ++k) {
-        f32x4 q[2];
+        for (int ct = 0; ct < 2; ++ct) out[m][ct] = (f32x4)0.f;
 #pragma unroll
-        for (int m = 0; m < 2; ++m)
-          q[m] = *reinterpret_cast<const f32x4*>(
-              Ql + (m * 16 + i16) * ROW + k * 16 + g * 4);
+      for (int j = 0; j < KJ; ++j) {
+        bf16x8 q[2][3], s[2][3];
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
+        for (int m = 0; m < 2; ++m) row_frags(Ql, m * 16 + i16, j, q[m]);
 #pragma unroll
-          for (int m = 0; m < 2; ++m)
-            out[m] = mfma4(q[m][r], S[k][r], out[m]);
-      }
-      __syncthreads();
-      for (int e = tid; e < 3 * 256; e += NT) {
-        const int i = e / 256, x = e / 16 % 16, z = e % 16;
-        const int t = (i > 0) * 16 + x, s = (i > 1) * 16 + z;
-        float p = 0.f;
+        for (int ct = 0; ct < 2; ++ct) {
+          i32x4 x[3];
 #pragma unroll
-        for (int w = 0; w < NP; ++w) p += part[((w * 3 + i) * 16 + x) * PROW + z];
-        Pl[t * TROW + s] = s <= t ? p * exp2_of(lg * (t - s)) : 0.f;
-      }
-      __syncthreads();
+          for (int e = 0; e < 4; ++e) {
+            const f32x4& t = S[2 * j + (e >> 1)][ct];
+            const Parts y = split2(t[(e & 1) * 2], t[(e & 1) * 2 + 1]);
 #pragma unroll
-      for (int m = 0; m < 2; ++m) {
+            for (int p = 0; p < 3; ++p) x[p][e] = (int)y.p[p];
+          }
 #pragma unroll
-        for (int r = 0; r < 4; ++r)
-          out[m][r] *= exp2_of(lg * (m * 16 + g * 4 + r + 1));
-#pragma unroll
-        for (int k = 0; k <= m; ++k) {
-          const f32x4 p = *reinterpret_cast<const f32x4*>(
-              Pl + (m * 16 + i16) * TROW + k * 16 + g * 4);
-#pragma unroll
-          for (int r = 0; r < 4; ++r) out[m] = mfma4(p[r], v[k][r], out[m]);
+          for (int p = 0; p < 3; ++p)
+            s[ct][p] = __builtin_bit_cast(bf16x8, x[p]);
         }
 #pragma unroll
+        for (int m = 0; m < 2; ++m)
+#pragma unroll
+          for (int ct = 0; ct < 2; ++ct)
+            out[m][ct] = mfma_parts(q[m], s[ct], out[m][ct]);
+      }
+      const T* src = a.ab +
+                     (row0 + c * CH + min(tid / LPR, cnt - 1)) * a.ld + at_g +
+                     tid % LPR * 16;
+      gr[0] = *reinterpret_cast<const s16x8*>(src);
+      gr[1] = *reinterpret_cast<const s16x8*>(src + 8);
+      __syncthreads();  // the keys' rows are consumed
+      stage_numbers(cnt);
+#pragma unroll 1
+      for (int e0 = 0; e0 < CH * CH / 2; e0 += NT) {
+        const int t = (e0 + tid) / 16, s = (e0 + tid) % 16 * 2;
+        if (NT > CH * CH / 2 && t >= CH) break;
+        float2 p = {0.f, 0.f};
+        if (s <= t) {
+          const int i = (t >> 4) + (s >> 4);
+          const float* at = part + (i * 16 + (t & 15)) * PROW + (s & 15);
+#pragma unroll
+          for (int w = 0; w < NP; ++w) {
+            const float2 x =
+                *reinterpret_cast<const float2*>(at + w * 3 * 16 * PROW);
+            p.x += x.x;
+            p.y += x.y;
+          }
+          p.x *= exp2_of(lg * (t - s));
+          p.y = s < t ? p.y * exp2_of(lg * (t - s - 1)) : 0.f;
+        }
+        const Parts x = split2(p.x, p.y);
+#pragma unroll
+        for (int i = 0; i < 3; ++i)
+          *reinterpret_cast<unsigned int*>(Pl + (i * CH + t) * L::P_ROW +
+                                           s * 2) = x.p[i];
+      }
+      __syncthreads();
+    }
+    bf16x8 v[2];
+#pragma unroll
+    for (int ct = 0; ct < 2; ++ct) {
+      s16x8 x;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) x[e] = (short)vr[ct][e];
+      v[ct] = __builtin_bit_cast(bf16x8, x);
+    }
+    if constexpr (!LOCAL) {
+#pragma unroll
+      for (int m = 0; m < 2; ++m) {
+        float w[4];
+#pragma unroll
         for (int r = 0; r < 4; ++r)
-          Ol[(m * 16 + g * 4 + r) * OROW + col] = out[m][r];
+          w[r] = exp2_of(lg * (m * 16 + g * 4 + r + 1));
+        bf16x8 p[3];
+#pragma unroll
+        for (int i = 0; i < 3; ++i)
+          p[i] = *reinterpret_cast<const bf16x8*>(
+              Pl + (i * CH + m * 16 + i16) * L::P_ROW + g * 16);
+#pragma unroll
+        for (int ct = 0; ct < 2; ++ct) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) out[m][ct][r] *= w[r];
+#pragma unroll
+          for (int i = 2; i >= 0; --i)
+            out[m][ct] = mfma_bf(p[i], v[ct], out[m][ct]);
+#pragma unroll
+          for (int r = 0; r < 4; ++r)
+            Ol[(m * 16 + g * 4 + r) * L::O_ROW + wid * 32 + ct * 16 + i16] =
+                out[m][ct][r];
+        }
       }
     }
-    // S <- g^n S + K^T (g^(n-1-s) V); rows behind the end have zero keys
-    const float decay = cnt == CH ? glast : exp2_of(lg * cnt);
+    // S <- g^n S + K^T V, keys weighted; rows behind the end have zero keys
+    const float decay = exp2_of(lg * cnt);
 #pragma unroll
-    for (int k = 0; k < KT; ++k)
+    for (int k = 0; k < KT; ++k) {
+      const int d = k * 16 + i16;
+      bf16x8 x[3];
 #pragma unroll
-      for (int e = 0; e < 4; ++e) S[k][e] *= decay;
+      for (int p = 0; p < 3; ++p)
+        x[p] = *reinterpret_cast<const bf16x8*>(
+            Kl + (p * DP + d) * (CH * 2) + ((g ^ ((d >> 2) & 3)) * 16));
 #pragma unroll
-    for (int m = 0; m < 2; ++m)
+      for (int ct = 0; ct < 2; ++ct) {
 #pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int s = m * 16 + g * 4 + r;
-        const float w = v[m][r] * exp2_of(lg * max(cnt - 1 - s, 0));
-        const float* kc = Kl + s * ROW + i16;
+        for (int e = 0; e < 4; ++e) S[k][ct][e] *= decay;
 #pragma unroll
-        for (int k = 0; k < KT; ++k) S[k] = mfma4(kc[k * 16], w, S[k]);
+        for (int p = 2; p >= 0; --p)
+          S[k][ct] = mfma_bf(x[p], v[ct], S[k][ct]);
       }
+    }
     if constexpr (!LOCAL) {
       __syncthreads();
-      const int t = tid / (VP / 8), c8 = tid % (VP / 8) * 8;
-      float x[8];
-      load8<float>(Ol + t * OROW + c8, x);
+      const int t = tid / LPR, c16 = tid % LPR * 16;
+      float x[16], gate[16];
+      load8<float>(Ol + t * L::O_ROW + c16, x);
+      load8<float>(Ol + t * L::O_ROW + c16 + 8, x + 8);
+      bf8_to_f32(gr[0], gate);
+      bf8_to_f32(gr[1], gate + 8);
       float ss = 0.f;
 #pragma unroll
-      for (int i = 0; i < 8; ++i) ss += x[i] * x[i];
+      for (int i = 0; i < 16; ++i) ss += x[i] * x[i];
 #pragma unroll
-      for (int off = VP / 16; off > 0; off >>= 1)
+      for (int off = LPR / 2; off > 0; off >>= 1)
         ss += __shfl_xor(ss, off, 64);
       const float inv = 1.f / sqrtf(ss / a.vdim + a.eps);
 #pragma unroll
-      for (int i = 0; i < 8; ++i) x[i] *= inv * silu(gt[i]);
-      if (t < cnt)
-        store8(a.y + ((row0 + c * CH + t) * a.H + head) * VP + c8, x);
+      for (int i = 0; i < 16; ++i) x[i] *= inv * silu(gate[i]);
+      if (t < cnt) {
+        T* dst = a.y + ((row0 + c * CH + t) * a.H + head) * VP + c16;
+        store8(dst, x);
+        store8(dst + 8, x + 8);
+      }
     }
   }
   if (LOCAL || number + 1 == count) {
     float* to = LOCAL ? between + own * DP + g * 4 : slot;
 #pragma unroll
-    for (int k = 0; k < KT; ++k) *reinterpret_cast<f32x4*>(to + k * 16) = S[k];
+    for (int k = 0; k < KT; ++k)
+#pragma unroll
+      for (int ct = 0; ct < 2; ++ct)
+        *reinterpret_cast<f32x4*>(to + ct * 16 * DP + k * 16) = S[k][ct];
   }
 }
 
@@ -485,8 +667,10 @@ extern "C" void launch_retention_scan(
     float eps, const float* decay, const float* table, int half, float* state,
     void* y, const int* seg_row0, const int* seg_rows, const int* seg_slot,
     const int* ctx, int nseg, int max_rows, bool fp32, hipStream_t stream) {
+  // workgroups of 256 threads where these can hold the state: several on a
+  // CU hide one another's round trips
   const int lpc = dp / 16;
-  const int threads = min(1024, lpc * vp);
+  const int threads = min(1024, max(256, lpc * vp / 2));
   const int ncol = lpc * vp / threads;
 #define RS(T, L, N)                                                          \
   hipLaunchKernelGGL((retention_scan_kernel<T, L, N>), dim3(nseg * H),       \
@@ -496,17 +680,21 @@ extern "C" void launch_retention_scan(
                                        (T*)y, seg_row0, seg_rows, seg_slot,  \
                                        ctx}),                                \
                      max_rows)
-#define RS_N(T)                                \
-  do {                                         \
-    if (lpc == 4) RS(T, 4, 1);                 \
-    else if (lpc == 8 && ncol == 1) RS(T, 8, 1); \
-    else if (lpc == 8) RS(T, 8, 2);            \
-    else if (ncol == 1) RS(T, 16, 1);          \
-    else if (ncol == 2) RS(T, 16, 2);          \
-    else RS(T, 16, 4);                         \
+#define RS_N(T, L)          \
+  do {                      \
+    if (ncol == 1) RS(T, L, 1); \
+    else if (ncol == 2) RS(T, L, 2); \
+    else RS(T, L, 4);       \
   } while (0)
-  if (fp32) RS_N(float);
-  else RS_N(unsigned short);
+#define RS_L(T)                  \
+  do {                           \
+    if (lpc == 4) RS_N(T, 4);    \
+    else if (lpc == 8) RS_N(T, 8); \
+    else RS_N(T, 16);            \
+  } while (0)
+  if (fp32) RS_L(float);
+  else RS_L(unsigned short);
+#undef RS_L
 #undef RS_N
 #undef RS
 }
@@ -525,25 +713,21 @@ extern "C" void launch_retention_chunks(
                            ctx};
 #define RC(D, N, LOC, V)                                                     \
   do {                                                                       \
-    constexpr int np = N < D / 16 ? N : D / 16;                              \
-    constexpr int p = np * 3 * 16 * PROW, o = CH * (N * 16 + 4);             \
-    const int lds =                                                          \
-        (LOC ? CH * (D + 4)                                                  \
-             : 2 * CH * (D + 4) + CH * TROW + (p > o ? p : o)) * 4;          \
+    typedef ChunkLds<D, N> L;                                                \
     hipLaunchKernelGGL((retention_chunk_kernel<D, N, LOC, V>),               \
-                       dim3(npieces * H), dim3(N * 64), lds, stream, a,      \
-                       pieces, between);                                     \
+                       dim3(npieces * H), dim3(N * 2),                       \
+                       LOC ? L::T_B : L::BYTES, stream, a, pieces, between); \
   } while (0)
-#define RC_V(D, N, LOC)              \
-  do {                               \
-    if (half % 8 == 0) RC(D, N, LOC, true); \
-    else RC(D, N, LOC, false);       \
+#define RC_V(D, N, LOC)                     \
+  do {                                      \
+    if (half % 2 == 0) RC(D, N, LOC, true); \
+    else RC(D, N, LOC, false);              \
   } while (0)
-#define RC_N(D, LOC)                   \
-  do {                                 \
-    if (vp == 64) RC_V(D, 4, LOC);     \
-    else if (vp == 128) RC_V(D, 8, LOC); \
-    else RC_V(D, 16, LOC);             \
+#define RC_N(D, LOC)                     \
+  do {                                   \
+    if (vp == 64) RC_V(D, 64, LOC);      \
+    else if (vp == 128) RC_V(D, 128, LOC); \
+    else RC_V(D, 256, LOC);              \
   } while (0)
 #define RC_D(LOC)                 \
   do {                            \
