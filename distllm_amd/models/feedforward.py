@@ -115,23 +115,30 @@ class RoutedExperts(Part):
 class GatedExperts(Part):
     """Squared-ReLU experts chosen by corrected sigmoid scores, beside a
     shared one with a gate per token (GatedExpertsDims). The shared
-    expert's gate is a row behind the router's and its weight one behind
-    those of the chosen experts."""
+    expert's gate is a row behind the router's.
+
+    Its columns are cut into shards of the size of an expert: a sum over
+    columns, it is the sum of experts that serve every token. With few rows
+    the shards are stored behind the experts and run with them, which saves
+    the launches of two more products; with many rows they are the two
+    products, the second on a copy of the weights in its order."""
+
+    FEW = 256  # rows
 
     def __init__(self, d: GatedExpertsDims, width: int, dtype):
         super().__init__()
         self.d, self.width = d, width
         self.wp, self.fp = pad64(width), pad64(d.ff)
         n = d.experts
+        self.shards = -(-(d.shared or 0) // self.fp)
         self.router = weight(n + (d.shared is not None), self.wp, dtype)
         self.correction = norm_weight(n)
-        self.wup = nn.Parameter(torch.empty(n, self.fp, self.wp,
-                                            dtype=dtype))
-        self.wdown = nn.Parameter(torch.empty(n, self.wp, self.fp,
-                                              dtype=dtype))
+        self.wup = nn.Parameter(torch.empty(n + self.shards, self.fp,
+                                            self.wp, dtype=dtype))
+        self.wdown = nn.Parameter(torch.empty(n + self.shards, self.wp,
+                                              self.fp, dtype=dtype))
         if d.shared is not None:
             self.sp = pad64(d.shared)
-            self.shared_up = weight(self.sp, self.wp, dtype)
             self.shared_down = weight(self.wp, self.sp, dtype)
 
     def tensors(self):
@@ -147,29 +154,31 @@ class GatedExperts(Part):
 
     def checkpoint(self, src, pre):
         t, n = self.checked(src, pre), self.d.experts
+        up = [padded(t[f"e{e}.up"], self.fp, self.wp) for e in range(n)]
+        down = [padded(t[f"e{e}.down"], self.wp, self.fp) for e in range(n)]
         router, out = t["router"], {}
         if self.d.shared is not None:
             router = torch.cat([router, t["shared.sg"]])
-            out = {"shared_up": padded(t["shared.up"], self.sp, self.wp),
-                   "shared_down": padded(t["shared.down"], self.wp, self.sp)}
-        return out | {
-            "router": padded(router, *self.router.shape),
-            "correction": t["correction"],
-            "wup": torch.stack([padded(t[f"e{e}.up"], self.fp, self.wp)
-                                for e in range(n)]),
-            "wdown": torch.stack([padded(t[f"e{e}.down"], self.wp, self.fp)
-                                  for e in range(n)])}
+            out = {"shared_down": padded(t["shared.down"], self.wp, self.sp)}
+            m = self.shards * self.fp
+            up += padded(t["shared.up"], m, self.wp).split(self.fp)
+            down += padded(t["shared.down"], self.wp, m).split(self.fp, 1)
+        return out | {"router": padded(router, *self.router.shape),
+                      "correction": t["correction"],
+                      "wup": torch.stack(up), "wdown": torch.stack(down)}
 
     def forward(self, h, ctx):
-        """-> outputs [rows * top, width] of the chosen experts, row by
-        row, the shared expert's [rows, width] or None, and the weights of
-        both [rows, top (+ 1)]; rows with ctx 0 have none."""
+        """-> outputs of the chosen experts, row by row [rows * choices,
+        width], the shared expert's [rows, width] where it is not among
+        them, and the weights of both; rows with ctx 0 have none."""
         d = self.d
-        ids, weights = ops.route_sigmoid(h, self.router, self.correction,
-                                         ctx, d.top, d.scale)
+        few = h.shape[0] <= self.FEW
+        ids, weights = ops.route_sigmoid(
+            h, self.router, self.correction, ctx, d.top, d.scale,
+            self.shards if few else 0)
         y = ops.experts(h, ids, self.wup, self.wdown, gated=False)
         shared = None
-        if d.shared is not None:
-            shared = ops.linear(ops.up_relu2(h, self.shared_up),
-                                self.shared_down)
+        if d.shared is not None and not few:
+            up = self.wup[d.experts:].flatten(0, 1)[: self.sp]
+            shared = ops.linear(ops.up_relu2(h, up), self.shared_down)
         return y, shared, weights

@@ -774,21 +774,23 @@ def experts(h, ids, wup, wdown, gated=True):
     return torch_ref.experts(h, ids, wup, wdown, gated)
 
 
-def route_sigmoid(h, router, correction, ctx, top, scale):
+def route_sigmoid(h, router, correction, ctx, top, scale, shards=0):
     """Experts of every row by sigmoid scores: ids [M, top] int32 of the
     largest sums of score and correction, and scale times their scores
-    without it. Rows of the router behind the experts (one per correction)
-    are gates of their own: their sigmoids are further columns of the
-    weights. Rows with ctx 0 get ids -1 and weights 0."""
+    without it. One more row of the router than corrections is the gate of
+    an expert that serves every row: its sigmoid is a further column of the
+    weights, or, with shards, the weight of that many further choices, the
+    experts behind the others. Rows with ctx 0 get ids -1 and weights 0."""
     if h.is_cuda:
         _require_hip("_hip_experts")
         if h.dtype == torch.bfloat16 and router.shape[0] <= 256:
             return _hip_ops.route_sigmoid(h, router, correction, ctx, top,
-                                          scale)
+                                          scale, shards)
         logits = torch.nn.functional.linear(h.float(), router.float())
         return _hip_ops.route_sigmoid(logits, None, correction, ctx, top,
-                                      scale)
-    return torch_ref.route_sigmoid(h, router, correction, ctx, top, scale)
+                                      scale, shards)
+    return torch_ref.route_sigmoid(h, router, correction, ctx, top, scale,
+                                   shards)
 
 
 def up_relu2(x, wup):

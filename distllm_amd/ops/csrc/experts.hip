@@ -21,19 +21,40 @@ extern __shared__ __attribute__((aligned(16))) char smem[];
 // ---- routing ----------------------------------------------------------------
 // Softmax scores, or (correction not null) sigmoid scores whose sum with the
 // correction [E] makes the choice; weights are the scores times `scale`.
-// `gates` logits behind those of the experts are weights of their own, by
-// their sigmoids.
+// With `gate`, one more logit is the gate of an expert that serves every row;
+// its sigmoid is a weight behind those of the chosen experts, or (shards > 0)
+// the weight of `shards` further choices, experts E, E + 1, ..
 struct RouteArgs {
   int E, groups, keep, top;
   const float* correction;
   float scale;
-  int gates;
+  bool gate;
+  int shards;
 
-  __host__ __device__ __forceinline__ int logits() const { return E + gates; }
-  __host__ __device__ __forceinline__ int cols() const { return top + gates; }
+  __host__ __device__ __forceinline__ int logits() const { return E + gate; }
+  __host__ __device__ __forceinline__ int ids() const { return top + shards; }
+  __host__ __device__ __forceinline__ int cols() const {
+    return shards > 0 ? top + shards : top + gate;
+  }
 };
 
-// One wave chooses for one row. z [E + gates]: logits, overwritten; gm, ok
+// the largest number of a wave, by lane shifts within and between rows of 16
+__device__ __forceinline__ float wave_max(float v) {
+#define WM(ctrl, rows)                                                     \
+  v = fmaxf(v, __int_as_float(__builtin_amdgcn_update_dpp(                 \
+                   __float_as_int(v), __float_as_int(v), ctrl, rows, 0xf,  \
+                   false)))
+  WM(0x111, 0xf);  // row_shr:1, :2, :4, :8
+  WM(0x112, 0xf);
+  WM(0x114, 0xf);
+  WM(0x118, 0xf);
+  WM(0x142, 0xa);  // row_bcast:15 to rows 1 and 3
+  WM(0x143, 0xc);  // row_bcast:31 to rows 2 and 3
+#undef WM
+  return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), 63));
+}
+
+// One wave chooses for one row. z: logits, overwritten; gm, ok
 // [groups]. A lane holds the scores of experts lane + 64 i, i < PER.
 template <int PER>
 __device__ void select_row(float* z, float* gm, int* ok, const RouteArgs& a,
@@ -49,8 +70,10 @@ __device__ void select_row(float* z, float* gm, int* ok, const RouteArgs& a,
       w[i] = e < E ? sigmoid_exact(z[e]) : 0.f;
       s[i] = e < E ? w[i] + a.correction[e] : 0.f;
     }
-    for (int j = lane; j < a.gates; j += 64)
-      weights[a.top + j] = sigmoid_exact(z[E + j]);
+    for (int j = a.top + lane; j < a.cols(); j += 64) {
+      weights[j] = sigmoid_exact(z[E]);
+      if (j < a.ids()) ids[j] = E + j - a.top;
+    }
   } else {
     float mx = -INFINITY;
 #pragma unroll
@@ -109,31 +132,44 @@ __device__ void select_row(float* z, float* gm, int* ok, const RouteArgs& a,
       }
   };
   best();
+  int id = -1;  // lane t keeps choice t until 64 are stored together
+  float wt = 0.f;
   for (int t = 0; t < a.top; ++t) {
-    const float m = wave_reduce_max(own);
-    const unsigned long long who =
-        m > -INFINITY ? __ballot(own == m) : 0ull;
-    if (who != 0 && lane == __builtin_ctzll(who)) {
-      ids[t] = lane + 64 * at;
-      weights[t] = weight * scale;
+    const float m = wave_max(own);
+    int e = -1;  // not a number: no expert
+    float we = 0.f;
+    if (m > -INFINITY) {
+      const int who = __builtin_ctzll(__ballot(own == m));
+      e = who + 64 * __builtin_amdgcn_readlane(at, who);
+      we = __int_as_float(
+          __builtin_amdgcn_readlane(__float_as_int(weight), who));
+      const bool mine = lane == who;
 #pragma unroll
       for (int i = 0; i < PER; ++i)
-        if (i == at) s[i] = -INFINITY;
+        if (mine && i == at) s[i] = -INFINITY;
       best();
-    } else if (who == 0 && lane == 0) {  // not a number: no expert
-      ids[t] = -1;
-      weights[t] = 0.f;
+    }
+    if ((t & 63) == lane) {
+      id = e;
+      wt = we * scale;
+    }
+    if ((t & 63) == 63 || t + 1 == a.top) {
+      const int place = (t & ~63) + lane;
+      if (place <= t) {
+        ids[place] = id;
+        weights[place] = wt;
+      }
     }
   }
 }
 
 __device__ __forceinline__ void no_choice(const RouteArgs& a, int* ids,
                                           float* weights, int lane) {
-  for (int t = lane; t < a.top; t += 64) ids[t] = -1;
+  for (int t = lane; t < a.ids(); t += 64) ids[t] = -1;
   for (int t = lane; t < a.cols(); t += 64) weights[t] = 0.f;
 }
 
-// from given logits [M, E + gates]; one wave per row
+// from given logits; one wave per row
 __global__ void __launch_bounds__(256)
 select_kernel(const float* __restrict__ logits, const int* __restrict__ ctx,
               int M, const RouteArgs a, int* __restrict__ ids,
@@ -145,7 +181,7 @@ select_kernel(const float* __restrict__ logits, const int* __restrict__ ctx,
   int* ok = reinterpret_cast<int*>(gm + a.groups);
   const int row = blockIdx.x * 4 + wid;
   if (row >= M) return;
-  int* id = ids + (long)row * a.top;
+  int* id = ids + (long)row * a.ids();
   float* w = weights + (long)row * a.cols();
   if (ctx[row] <= 0) {
     no_choice(a, id, w, lane);
@@ -156,7 +192,7 @@ select_kernel(const float* __restrict__ logits, const int* __restrict__ ctx,
   select_row<16>(z, gm, ok, a, id, w, lane);
 }
 
-// bf16 rows against the router's weights [E + gates, K], fp32 sums, then the
+// bf16 rows against the router's weights [logits, K], fp32 sums, then the
 // choice: 16 rows per workgroup, its NW waves split K and then the rows. NE
 // tiles of 16 logits.
 template <int NE, int NW>
@@ -166,28 +202,53 @@ route_kernel(const unsigned short* __restrict__ h,
              const int* __restrict__ ctx, int M, int K, const RouteArgs args,
              int* __restrict__ ids, float* __restrict__ weights) {
   constexpr int EP = NE * 16;
-  const int E = args.logits(), groups = args.groups;
   constexpr int WS = 16 * (EP + 4);  // sums of a wave
+  const int E = args.logits(), groups = args.groups;
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int i16 = lane & 15, g = lane >> 4;
   const int m0 = blockIdx.x * 16;
-  const unsigned short* hr =
-      h + (long)min(m0 + i16, M - 1) * K + g * 8;
-  const unsigned short* wr[NE];
+  // An operand's 16 rows of 64 bytes are loaded with four lanes to a row,
+  // whole pieces of memory, and pass LDS to get where the product wants them.
+  const int lrow = lane >> 2, lcol = (lane & 3) * 8;
+  const unsigned short* src[NE + 1];
 #pragma unroll
   for (int j = 0; j < NE; ++j)
-    wr[j] = W + (long)min(j * 16 + i16, E - 1) * K + g * 8;
+    src[j] = W + (long)min(j * 16 + lrow, E - 1) * K + lcol;
+  src[NE] = h + (long)min(m0 + lrow, M - 1) * K + lcol;
+  char* own = smem + wid * (NE + 1) * 1024;
+  const int put = lrow * 64 + (((lane & 3) ^ ((lrow >> 2) & 3)) * 16);
+  const int get = i16 * 64 + ((g ^ ((i16 >> 2) & 3)) * 16);
   f32x4 acc[NE];
 #pragma unroll
   for (int j = 0; j < NE; ++j) acc[j] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int k = wid * 32; k < K; k += NW * 32) {
-    const bf16x8 a = *reinterpret_cast<const bf16x8*>(hr + k);
+  // U steps of loads are in flight together
+  constexpr int U = NE <= 9 ? 2 : 1;
+  for (int k0 = wid * 32; k0 < K; k0 += U * NW * 32) {
+    i32x4 x[U][NE + 1];
 #pragma unroll
-    for (int j = 0; j < NE; ++j)
-      acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-          *reinterpret_cast<const bf16x8*>(wr[j] + k), a, acc[j], 0, 0, 0);
+    for (int s = 0; s < U; ++s)
+#pragma unroll
+      for (int j = 0; j <= NE; ++j)
+        x[s][j] = *reinterpret_cast<const i32x4*>(
+            src[j] + min(k0 + s * NW * 32, K - 32));
+    __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+    for (int s = 0; s < U; ++s) {
+      if (k0 + s * NW * 32 >= K) x[s][NE] = (i32x4)0;
+      wave_sync();
+#pragma unroll
+      for (int j = 0; j <= NE; ++j)
+        *reinterpret_cast<i32x4*>(own + j * 1024 + put) = x[s][j];
+      wave_sync();
+      const bf16x8 a = *reinterpret_cast<const bf16x8*>(own + NE * 1024 + get);
+#pragma unroll
+      for (int j = 0; j < NE; ++j)
+        acc[j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+            *reinterpret_cast<const bf16x8*>(own + j * 1024 + get), a, acc[j],
+            0, 0, 0);
+    }
   }
+  __syncthreads();
   // rows of the sum: experts (g * 4 + r); columns: rows of h (i16)
   float* part = reinterpret_cast<float*>(smem);  // [NW][16][EP + 4]
 #pragma unroll
@@ -200,7 +261,7 @@ route_kernel(const unsigned short* __restrict__ h,
   for (int i = wid; i < 16; i += NW) {
     const int row = m0 + i;
     if (row >= M) break;
-    int* id = ids + (long)row * args.top;
+    int* id = ids + (long)row * args.ids();
     float* w = weights + (long)row * args.cols();
     if (ctx[row] <= 0) {
       no_choice(args, id, w, lane);
@@ -223,25 +284,28 @@ extern "C" bool route_covers(int logits) { return logits <= 256; }
 
 extern "C" void launch_select(const float* logits, const int* ctx, int M,
                               int E, int groups, int keep, int top,
-                              const float* correction, float scale, int gates,
-                              int* ids, float* weights, hipStream_t stream) {
-  const RouteArgs a{E, groups, keep, top, correction, scale, gates};
+                              const float* correction, float scale, bool gate,
+                              int shards, int* ids, float* weights,
+                              hipStream_t stream) {
+  const RouteArgs a{E, groups, keep, top, correction, scale, gate, shards};
   hipLaunchKernelGGL(select_kernel, dim3((M + 3) / 4), dim3(256),
-                     4 * (E + gates + 2 * groups) * 4, stream, logits, ctx, M,
+                     4 * (a.logits() + 2 * groups) * 4, stream, logits, ctx, M,
                      a, ids, weights);
 }
 
 extern "C" void launch_route(const void* h, const void* W, const int* ctx,
                              int M, int E, int K, int groups, int keep,
                              int top, const float* correction, float scale,
-                             int gates, int* ids, float* weights,
+                             bool gate, int shards, int* ids, float* weights,
                              hipStream_t stream) {
-  const RouteArgs a{E, groups, keep, top, correction, scale, gates};
-  const int n = E + gates;
+  const RouteArgs a{E, groups, keep, top, correction, scale, gate, shards};
+  const int n = a.logits();
 #define RT(NE, NW)                                                           \
   hipLaunchKernelGGL((route_kernel<NE, NW>), dim3((M + 15) / 16),            \
                      dim3(NW * 64),                                          \
-                     (NW * (16 * (NE * 16 + 4) + 2 * groups)) * 4, stream,   \
+                     max(NW * (16 * (NE * 16 + 4) + 2 * groups) * 4,         \
+                         NW * (NE + 1) * 1024),                              \
+                     stream,                                                 \
                      (const unsigned short*)h, (const unsigned short*)W, ctx, \
                      M, K, a, ids, weights)
   if (n <= 16) RT(1, 16);
@@ -316,16 +380,132 @@ expert_plan_kernel(const int* __restrict__ ids, int A, int E, int TM,
   }
 }
 
+// The same for many pairs, in blocks of PB pairs: counts of every block
+// [blocks, E], then their sums and the tiles (one workgroup), then the places.
+#define PB 2048
+
+__global__ void __launch_bounds__(256)
+expert_count_kernel(const int* __restrict__ ids, int A, int E,
+                    int* __restrict__ counts) {
+  __shared__ int count[1024];
+  for (int e = threadIdx.x; e < E; e += 256) count[e] = 0;
+  __syncthreads();
+  const int a0 = blockIdx.x * PB;
+#pragma unroll
+  for (int i = 0; i < PB / 256; ++i) {
+    const int a = a0 + i * 256 + threadIdx.x;
+    const int e = a < A ? ids[a] : -1;
+    if (e >= 0 && e < E) atomicAdd(&count[e], 1);
+  }
+  __syncthreads();
+  for (int e = threadIdx.x; e < E; e += 256)
+    counts[(long)blockIdx.x * E + e] = count[e];
+}
+
+// counts become the first place of every block's pairs of an expert
+__global__ void __launch_bounds__(1024)
+expert_offset_kernel(int* __restrict__ counts, int blocks, int E, int TM,
+                     int max_tiles, int* __restrict__ tiles,
+                     int* __restrict__ ntiles) {
+  __shared__ int first[1024], tile0[1024], part[1024];
+  const int tid = threadIdx.x;
+  // S threads share an expert's blocks
+  const int S = E <= 64 ? 16 : E <= 128 ? 8 : E <= 256 ? 4 : E <= 512 ? 2 : 1;
+  const int e = tid / S, sub = tid % S;
+  const int per = (blocks + S - 1) / S;
+  const int b0 = sub * per, b1 = min(blocks, b0 + per);
+  int c = 0;
+  if (e < E) {
+#pragma unroll 4
+    for (int b = b0; b < b1; ++b) c += counts[(long)b * E + e];
+  }
+  part[tid] = c;
+  __syncthreads();
+  int before = 0, total = 0;  // of my expert: in blocks before mine, in all
+  for (int i = 0; i < S; ++i) {
+    const int x = part[tid / S * S + i];
+    before += i < sub ? x : 0;
+    total += x;
+  }
+  const bool lead = sub == 0 && e < E;
+  const int nt = lead ? (total + TM - 1) / TM : 0;
+  first[tid] = lead ? total : 0;
+  tile0[tid] = nt;
+  __syncthreads();
+  for (int off = 1; off < 1024; off <<= 1) {  // inclusive sums
+    const int x = tid >= off ? first[tid - off] : 0;
+    const int y = tid >= off ? tile0[tid - off] : 0;
+    __syncthreads();
+    first[tid] += x;
+    tile0[tid] += y;
+    __syncthreads();
+  }
+  const int f = first[tid] - total, t0 = tile0[tid] - nt;
+  if (tid == 1023) *ntiles = min(tile0[tid], max_tiles);
+  for (int i = 0; i < nt; ++i)
+    if (t0 + i < max_tiles) {
+      int* t = tiles + (long)(t0 + i) * 4;
+      t[0] = e;
+      t[1] = f + i * TM;
+      t[2] = min(TM, total - i * TM);
+    }
+  if (e < E) {  // first[] is the same for the threads of an expert
+    int at = first[tid] - total + before;
+    for (int b = b0; b < b1; ++b) {
+      int* p = counts + (long)b * E + e;
+      const int x = *p;
+      *p = at;
+      at += x;
+    }
+  }
+}
+
+__global__ void __launch_bounds__(256)
+expert_place_kernel(const int* __restrict__ ids, int A, int E,
+                    const int* __restrict__ counts, int* __restrict__ perm) {
+  __shared__ int at[1024];
+  for (int e = threadIdx.x; e < E; e += 256)
+    at[e] = counts[(long)blockIdx.x * E + e];
+  __syncthreads();
+  const int a0 = blockIdx.x * PB;
+#pragma unroll
+  for (int i = 0; i < PB / 256; ++i) {
+    const int a = a0 + i * 256 + threadIdx.x;
+    const int e = a < A ? ids[a] : -1;
+    if (e >= 0 && e < E) perm[atomicAdd(&at[e], 1)] = a;
+  }
+}
+
+// ints of scratch that the plan of A pairs needs
+extern "C" long expert_plan_scratch(long A, int E) {
+  return A >= 16 * PB ? (A + PB - 1) / PB * E : 0;
+}
+
 extern "C" void launch_expert_plan(const int* ids, int A, int E, int TM,
                                    int max_tiles, int* perm, int* tiles,
-                                   int* ntiles, hipStream_t stream) {
+                                   int* ntiles, int* scratch,
+                                   hipStream_t stream) {
+  if (expert_plan_scratch(A, E) > 0) {
+    const int blocks = (A + PB - 1) / PB;
+    hipLaunchKernelGGL(expert_count_kernel, dim3(blocks), dim3(256), 0,
+                       stream, ids, A, E, scratch);
+    hipLaunchKernelGGL(expert_offset_kernel, dim3(1), dim3(1024), 0, stream,
+                       scratch, blocks, E, TM, max_tiles, tiles, ntiles);
+    hipLaunchKernelGGL(expert_place_kernel, dim3(blocks), dim3(256), 0,
+                       stream, ids, A, E, scratch, perm);
+    return;
+  }
   hipLaunchKernelGGL(expert_plan_kernel, dim3(1), dim3(1024), 0, stream, ids,
                      A, E, TM, max_tiles, perm, tiles, ntiles);
 }
 
 // ---- product, few rows per expert ----------------------------------------------
 // Weight-streaming bound: a workgroup takes 64 weight rows and up to 16 MT
-// places; its waves split K and read the weights straight into registers.
+// places; its waves split K, 64 numbers at a time. Eight lanes load a row's 128
+// bytes together (a wave that loaded the product's operands directly would
+// ask for 16 rows at once, a line per lane, and be bound by that); the
+// wave's own part of LDS brings them into operand order, the next step's are
+// on their way in registers meanwhile.
 // UNIT: 1, 2: rows are gathered (place -> perm / top), a gated unit halves
 // the columns, or each is relu(.)^2; 0: rows are places and the output row is
 // perm[place].
@@ -339,41 +519,66 @@ expert_rows_kernel(const unsigned short* __restrict__ x,
                    const int* __restrict__ ntiles, int N, int K, int top) {
   constexpr bool GLU = UNIT == 1, UP = UNIT != 0;
   constexpr int RROW = 68;  // padded row of 64 sums
+  constexpr int NL = 8 + 2 * MT;  // loads of 8 rows: weights, places
   if ((int)blockIdx.y >= *ntiles) return;
   const int* tile = tiles + (long)blockIdx.y * 4;
   const int e = tile[0], s0 = tile[1], cnt = tile[2];
   const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
   const int i16 = lane & 15, g = lane >> 4;
   const int n0 = blockIdx.x * 64;
-  const unsigned short* wr =
-      W + ((long)e * N + n0 + i16) * K + g * 8;
-  const unsigned short* xr[MT];
+  const int r8 = lane >> 3, c8 = (lane & 7) * 8;
+  const unsigned short* wr = W + ((long)e * N + n0 + r8) * K + c8;
+  const unsigned short* xr[2 * MT];
 #pragma unroll
-  for (int t = 0; t < MT; ++t) {
-    const int s = s0 + min(t * 16 + i16, cnt - 1);
-    xr[t] = x + (long)(UP ? perm[s] / top : s) * K + g * 8;
+  for (int t = 0; t < 2 * MT; ++t) {
+    const int s = s0 + min(t * 8 + r8, cnt - 1);
+    xr[t] = x + (long)(UP ? perm[s] / top : s) * K + c8;
   }
+  char* own = smem + wid * NL * 1024;
+  const int put = r8 * 128 + (((lane & 7) ^ r8) * 16);
   f32x4 acc[MT][4];
 #pragma unroll
   for (int t = 0; t < MT; ++t)
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[t][j] = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 4
-  for (int k = wid * 32; k < K; k += 128) {
-    bf16x8 wf[4], xf[MT];
+  i32x4 next[NL];
+  auto load = [&](int k) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j)
-      wf[j] = *reinterpret_cast<const bf16x8*>(wr + (long)j * 16 * K + k);
+    for (int q = 0; q < 8; ++q)
+      next[q] = *reinterpret_cast<const i32x4*>(wr + (long)q * 8 * K + k);
 #pragma unroll
-    for (int t = 0; t < MT; ++t)
-      xf[t] = *reinterpret_cast<const bf16x8*>(xr[t] + k);
+    for (int t = 0; t < 2 * MT; ++t)
+      next[8 + t] = *reinterpret_cast<const i32x4*>(xr[t] + k);
+  };
+  auto frag = [&](int row16, int kk) {
+    return *reinterpret_cast<const bf16x8*>(
+        own + (row16 * 16 + i16) * 128 +
+        (((kk * 4 + g) ^ (i16 & 7)) * 16));
+  };
+  if (wid * 64 < K) load(wid * 64);
+  for (int k = wid * 64; k < K; k += 256) {
+    wave_sync();  // the step before is consumed
 #pragma unroll
-    for (int t = 0; t < MT; ++t)
+    for (int q = 0; q < NL; ++q)
+      *reinterpret_cast<i32x4*>(own + q * 1024 + put) = next[q];
+    load(min(k + 256, K - 64));
+    wave_sync();
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        acc[t][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
-            wf[j], xf[t], acc[t][j], 0, 0, 0);
+    for (int kk = 0; kk < 2; ++kk) {
+      bf16x8 wf[4], xf[MT];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) wf[j] = frag(j, kk);
+#pragma unroll
+      for (int t = 0; t < MT; ++t) xf[t] = frag(4 + t, kk);
+#pragma unroll
+      for (int t = 0; t < MT; ++t)
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          acc[t][j] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(
+              wf[j], xf[t], acc[t][j], 0, 0, 0);
+    }
   }
+  __syncthreads();
   // sums: rows are weight rows, columns places -> [wave][place][column]
   float* part = reinterpret_cast<float*>(smem);
 #pragma unroll
@@ -619,7 +824,8 @@ extern "C" void launch_expert_gemm(const void* x, const void* W, void* out,
   }
 #define ER(MT, GL)                                                          \
   hipLaunchKernelGGL((expert_rows_kernel<MT, GL>), grid, dim3(256),         \
-                     4 * MT * 16 * 68 * 4, stream, (const u16*)x,           \
+                     max(4 * MT * 16 * 68 * 4, 4 * (8 + 2 * MT) * 1024),    \
+                     stream, (const u16*)x,                                 \
                      (const u16*)W, (u16*)out, perm, tiles, ntiles, N, K, top)
 #define ET(GL)                                                              \
   hipLaunchKernelGGL((expert_tile_kernel<GL>),                              \

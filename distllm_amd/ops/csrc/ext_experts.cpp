@@ -6,12 +6,13 @@ void launch_xielu(const void*, const float*, void*, long, bool, hipStream_t);
 bool route_covers(int);
 bool expert_gemm16_covers(int, int);
 void launch_select(const float*, const int*, int, int, int, int, int,
-                   const float*, float, int, int*, float*, hipStream_t);
+                   const float*, float, bool, int, int*, float*, hipStream_t);
 void launch_route(const void*, const void*, const int*, int, int, int, int,
-                  int, int, const float*, float, int, int*, float*,
+                  int, int, const float*, float, bool, int, int*, float*,
                   hipStream_t);
+long expert_plan_scratch(long, int);
 void launch_expert_plan(const int*, int, int, int, int, int*, int*, int*,
-                        hipStream_t);
+                        int*, hipStream_t);
 void launch_expert_gemm(const void*, const void*, void*, const int*,
                         const int*, const int*, int, int, int, int, int, int,
                         bool, hipStream_t);
@@ -36,34 +37,37 @@ static void check_route(int64_t E, int64_t top, int64_t groups,
               "experts, groups and choices");
 }
 
-// h: bf16 rows with the router's weights, or fp32 logits (W absent). Logits
-// behind those of the experts, `gates` of them, have weights of their own.
+// h: bf16 rows with the router's weights, or fp32 logits (W absent). gate:
+// the last logit is that of an expert that serves every row, in `shards`
+// pieces behind the experts, or (0) as a weight only.
 static std::tuple<torch::Tensor, torch::Tensor> choose(
     torch::Tensor h, c10::optional<torch::Tensor> W, torch::Tensor ctx,
     int64_t top, int64_t groups, int64_t keep, const float* correction,
-    double scale, int gates) {
+    double scale, bool gate, int64_t shards) {
   CHECK_DEV(h); CHECK_CONT(h);
   CHECK_INTS(ctx);
   const int M = h.size(0);
-  const int E = (int)(W ? W->size(0) : h.size(1)) - gates;
+  const int logits = W ? W->size(0) : h.size(1), E = logits - gate;
   check_route(E, top, groups, keep);
   TORCH_CHECK(h.dim() == 2 && ctx.numel() == M, "one ctx entry per row");
-  auto ids = torch::empty({M, top}, h.options().dtype(at::kInt));
-  auto w = torch::empty({M, top + gates}, h.options().dtype(at::kFloat));
+  TORCH_CHECK(shards >= 0 && (gate || shards == 0), "shards of no expert");
+  auto ids = torch::empty({M, top + shards}, h.options().dtype(at::kInt));
+  auto w = torch::empty({M, top + (shards > 0 ? shards : (int64_t)gate)},
+                        h.options().dtype(at::kFloat));
   if (M == 0) return {ids, w};
   if (W) {
     CHECK_BF16(h);
     CHECK_DEV(W.value()); CHECK_CONT(W.value()); CHECK_BF16(W.value());
     const int K = h.size(1);
-    TORCH_CHECK(W->size(1) == K && K % 32 == 0 && route_covers(E + gates),
+    TORCH_CHECK(W->size(1) == K && K % 32 == 0 && route_covers(logits),
                 "router shape");
     launch_route(h.data_ptr(), W->data_ptr(), ctx.data_ptr<int>(), M, E, K,
-                 groups, keep, top, correction, (float)scale, gates,
-                 ids.data_ptr<int>(), w.data_ptr<float>(), cur_stream());
+                 groups, keep, top, correction, (float)scale, gate,
+                 (int)shards, ids.data_ptr<int>(), w.data_ptr<float>(), cur_stream());
   } else {
     CHECK_F32(h);
     launch_select(h.data_ptr<float>(), ctx.data_ptr<int>(), M, E, groups,
-                  keep, top, correction, (float)scale, gates,
+                  keep, top, correction, (float)scale, gate, (int)shards,
                   ids.data_ptr<int>(), w.data_ptr<float>(), cur_stream());
   }
   return {ids, w};
@@ -72,18 +76,18 @@ static std::tuple<torch::Tensor, torch::Tensor> choose(
 std::tuple<torch::Tensor, torch::Tensor> route(
     torch::Tensor h, c10::optional<torch::Tensor> W, torch::Tensor ctx,
     int64_t top, int64_t groups, int64_t keep) {
-  return choose(h, W, ctx, top, groups, keep, nullptr, 1.0, 0);
+  return choose(h, W, ctx, top, groups, keep, nullptr, 1.0, false, 0);
 }
 
 std::tuple<torch::Tensor, torch::Tensor> route_sigmoid(
     torch::Tensor h, c10::optional<torch::Tensor> W, torch::Tensor correction,
-    torch::Tensor ctx, int64_t top, double scale) {
+    torch::Tensor ctx, int64_t top, double scale, int64_t shards) {
   CHECK_FLOATS(correction);
   const long n = W ? W->size(0) : h.size(1);
-  const long gates = n - correction.numel();
-  TORCH_CHECK(gates >= 0 && gates <= 16, "one correction per expert");
+  const long gate = n - correction.numel();
+  TORCH_CHECK(gate == 0 || gate == 1, "one correction per expert");
   return choose(h, W, ctx, top, 1, 1, correction.data_ptr<float>(), scale,
-                (int)gates);
+                gate == 1, shards);
 }
 
 // gated units, wup [E, 2F, K], or squared ReLU, wup [E, F, K]
@@ -116,12 +120,13 @@ torch::Tensor experts(torch::Tensor h, torch::Tensor ids, torch::Tensor wup,
     TM = 256;
   const int max_tiles = (int)std::min<long>(A, A / TM + E);
   auto i32 = ids.options();
-  auto plan = torch::empty({A + 4L * max_tiles + 1}, i32);
+  auto plan = torch::empty(
+      {A + 4L * max_tiles + 1 + expert_plan_scratch(A, E)}, i32);
   int* perm = plan.data_ptr<int>();
   int* tiles = perm + A;
   int* ntiles = tiles + 4L * max_tiles;
   launch_expert_plan(ids.data_ptr<int>(), (int)A, E, TM, max_tiles, perm,
-                     tiles, ntiles, cur_stream());
+                     tiles, ntiles, ntiles + 1, cur_stream());
   auto inter = torch::empty({A, F}, h.options());
   launch_expert_gemm(h.data_ptr(), wup.data_ptr(), inter.data_ptr(), perm,
                      tiles, ntiles, max_tiles, N, K, top, TM, gated ? 1 : 2,

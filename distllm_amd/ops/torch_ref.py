@@ -368,10 +368,11 @@ def _softmax_sink(s, sink):
     return torch.softmax(torch.cat([s, own], -1), -1)[..., :-1]
 
 
-def latent_attn(q, cache, block_table, row_seq, ctx, window, scale, rank,
-                sink=None, gate=None):
+def latent_attn(q, cache, block_table, row_seq, ctx, window, scale,
+                rank=None, sink=None, gate=None):
     """q [M, H, R] against the cached latents of each row's sequence; the
-    key is the whole cache row, the value its first rank columns."""
+    key is the whole cache row, the value its first rank (or all) columns."""
+    rank = rank or cache.shape[2]
     out = q.new_zeros(q.shape[0], q.shape[1], rank)
     for r in range(q.shape[0]):
         L = int(ctx[r])
@@ -577,12 +578,15 @@ def route(h, router, ctx, top, groups, keep):
     return ids.int().masked_fill(dead, -1), w.masked_fill(dead, 0)
 
 
-def route_sigmoid(h, router, correction, ctx, top, scale):
-    """-> expert ids [M, top] int32 (-1: none), weights [M, top + gates]."""
+def route_sigmoid(h, router, correction, ctx, top, scale, shards=0):
+    """-> expert ids [M, top + shards] int32 (-1: none) and weights."""
     E = correction.shape[0]
     s = torch.sigmoid(h.float() @ router.float().t())
     ids = (s[:, :E] + correction).topk(top, -1).indices
-    w = torch.cat([s.gather(1, ids) * scale, s[:, E:]], 1)
+    w = torch.cat([s.gather(1, ids) * scale,
+                   s[:, E:].repeat(1, max(shards, 1))], 1)
+    ids = torch.cat([ids, (E + torch.arange(shards)).expand(len(ids), -1)],
+                    1)
     dead = (ctx <= 0)[:, None]
     return ids.int().masked_fill(dead, -1), w.masked_fill(dead, 0)
 

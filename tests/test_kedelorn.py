@@ -163,6 +163,45 @@ def test_route_sigmoid(E, top, gates):
         assert torch.allclose(w[live, top:].double(), oracle.sigmoid(
             h.double() @ W[E:].double().T)[live], atol=1e-6)
     assert (ids[2] == -1).all() and not w[2].any()
+    if gates:  # the shared expert as three more choices
+        ids3, w3 = ops.route_sigmoid(h, W, corr, ctx, top, 1.6, 3)
+        assert torch.equal(ids3[:, :top], ids)
+        assert torch.equal(ids3[live, top:],
+                           (E + torch.arange(3)).expand(5, 3).int())
+        assert torch.equal(w3, torch.cat([w[:, :top], w[:, top:].expand(
+            -1, 3)], 1))
+        assert (ids3[2] == -1).all()
+
+
+@pytest.mark.parametrize("shared, shards", [(None, 0), (9, 1), (64, 1),
+                                            (65, 2), (150, 3)])
+def test_shared_expert_in_shards(shared, shards):
+    """With few rows the shared expert runs among the others, with many
+    beside them."""
+    cfg = oracle.make_config([oracle.retention_layer(oracle.moe_mlp(
+        ff=40, shared=shared))])
+    t = oracle.make_tensors(cfg, 4)
+    model = build_model(CONFIG_READERS["Kedelorn"](cfg), dtype=F32)
+    own = dict(model.named_parameters())
+    with torch.no_grad():
+        for k, v in model.checkpoint(t).items():
+            own[k].copy_(v)
+    mlp = model.layers[0].mlp
+    assert mlp.shards == shards and len(mlp.wup) == 6 + shards
+    h = torch.zeros(20, 64)
+    h[:, :48] = _rand(20, 48, seed=5)
+    d = {k: v.double() for k, v in t.items()}
+    want = oracle.moe(h[:, :48].double(), d, "l0.mlp.",
+                      cfg["layers"][0]["mlp"])
+    for few in (256, 8):
+        mlp.FEW = few
+        y, beside, w = mlp(h, torch.ones(20, dtype=torch.int32))
+        assert (beside is None) == (few == 256 or shared is None)
+        n = w.shape[1] - (beside is not None)
+        got = (y.view(20, n, -1) * w[:, :n, None]).sum(1)
+        if beside is not None:
+            got = got + beside * w[:, n:]
+        assert torch.allclose(got[:, :48].double(), want, atol=1e-4)
 
 
 @pytest.mark.parametrize("rot_dim, tp", [(8, 64), (6, 64), (2, 64),

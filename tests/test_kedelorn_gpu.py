@@ -116,6 +116,14 @@ def test_route_sigmoid(device, dtype, E, top, gates):
                               rtol=1e-4)
         assert torch.allclose(w[m, top:].double().cpu(), s[m, E:], rtol=1e-4)
     assert close < 3
+    if gates:  # the shared expert as two more choices
+        ids2, w2 = ops.route_sigmoid(h, router, corr, ctx.cuda(), top, 1.6, 2)
+        live = (ctx > 0).cuda()
+        assert torch.equal(ids2[:, :top], got)
+        assert (ids2[live, top:] == torch.tensor([E, E + 1]).cuda()).all()
+        assert torch.equal(w2, torch.cat([w[:, :top], w[:, top:].expand(
+            -1, 2)], 1))
+        assert (ids2[7] == -1).all()
 
 
 @dtypes
@@ -139,6 +147,33 @@ def test_squared_relu_experts(device, dtype, M, E, top, W, ff):
                              down.cpu().float(), gated=False)
     live = (chosen >= 0).reshape(-1)
     _close(y[live.cuda()], want[live], dtype, 3e-2 if dtype == BF16 else None)
+
+
+@dtypes
+@pytest.mark.parametrize("M, E, top", [
+    (16384, 3, 2), (16385, 64, 2), (9000, 100, 4), (20000, 200, 2),
+    (8200, 500, 5), (40000, 1000, 1)])
+def test_plan_of_many_rows(device, dtype, M, E, top):
+    """Pairs sorted in blocks; uneven experts, some without a row."""
+    h = _rand(M, 64, dtype=dtype)
+    up, down = _rand(E, 64, 64, seed=1), _rand(E, 64, 64, seed=2)
+    g = torch.Generator().manual_seed(3)
+    p = torch.rand(M, E, generator=g) + torch.linspace(0, 0.8, E)
+    p[:, 1] = -1
+    ids = p.topk(top, -1).indices.int()
+    ids[M // 2], ids[M - 1] = -1, -1
+    y = ops.experts(h, ids.cuda(), (up / 8).to(dtype), (down / 8).to(dtype),
+                    gated=False)
+    few = torch.randperm(M - 1, generator=g)[:200]
+    few = few[few != M // 2]
+    want = torch_ref.experts(h[few.cuda()].cpu().float(), ids[few],
+                             (up / 8).to(dtype).cpu().float(),
+                             (down / 8).to(dtype).cpu().float(), gated=False)
+    got = y.view(M, top, -1)[few.cuda()].flatten(0, 1)
+    _close(got, want, dtype, 3e-2 if dtype == BF16 else None)
+    # every pair has a place: none of its rows is left as it was
+    live = (ids >= 0).reshape(-1).cuda()
+    assert torch.isfinite(y[live]).all() and (y[live].abs().sum(1) > 0).all()
 
 
 @dtypes
