@@ -5,9 +5,8 @@ from __future__ import annotations
 import torch
 
 from .. import ops
-from .blocks import Part, pad64, padded_heads, weight
+from .blocks import Part, head_pad, pad64, padded_heads, weight
 from .config import RetentionDims
-from .delta import state_pad
 
 
 class Retention(Part):
@@ -24,7 +23,7 @@ class Retention(Part):
         super().__init__()
         self.d, self.width, self.eps = d, width, eps
         self.wp = pad64(width)
-        self.dp, self.vp = state_pad(d.dim), state_pad(d.vdim)
+        self.dp, self.vp = head_pad(d.dim), head_pad(d.vdim)
         H = d.heads
         self.win = weight(2 * H * (self.dp + self.vp), self.wp, dtype)
         self.wo = weight(self.wp, H * self.vp, dtype)

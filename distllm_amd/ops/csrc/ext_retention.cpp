@@ -8,6 +8,10 @@ void launch_retention_scan(const void*, int, int, int, int, int, float, float,
                            const float*, const float*, int, float*, void*,
                            const int*, const int*, const int*, const int*,
                            int, int, bool, hipStream_t);
+void launch_retention_wide(const void*, int, int, int, int, int, float, float,
+                           const float*, const float*, int, float*, void*,
+                           const int*, const int*, const int*, const int*,
+                           int, bool, hipStream_t);
 void launch_retention_chunks(const void*, int, int, int, int, int, float,
                              float, const float*, const float*, int, float*,
                              void*, const int*, const int*, const int*,
@@ -15,7 +19,8 @@ void launch_retention_chunks(const void*, int, int, int, int, int, float,
                              bool, float*, hipStream_t);
 }
 
-static bool state_size(int64_t d) { return d == 64 || d == 128 || d == 256; }
+// sizes of which a workgroup holds the state
+static bool held(int64_t d) { return d == 64 || d == 128 || d == 256; }
 
 // Segments with state slots; those of more than max_rows rows are described
 // by longs [L, 2] (segment, first piece) and pieces [P, 5], where there are
@@ -36,9 +41,10 @@ torch::Tensor retention(torch::Tensor ab, int64_t H, int64_t dp, int64_t vp,
   TORCH_CHECK(rows.numel() == nseg && slot.numel() == nseg &&
                   ctx.numel() == M,
               "segments and rows");
-  TORCH_CHECK(H > 0 && state_size(dp) && state_size(vp) && dim > 0 &&
-                  dim <= dp && vdim > 0 && vdim <= vp,
-              "heads of 64, 128 or 256 numbers");
+  TORCH_CHECK(H > 0 && dp % 64 == 0 && vp % 64 == 0 && dp <= 4096 &&
+                  vp <= 4096 && dim > 0 && dim <= dp && vdim > 0 &&
+                  vdim <= vp,
+              "heads of up to 4096 numbers, padded to multiples of 64");
   TORCH_CHECK(ab.size(1) >= 2 * H * (dp + vp) && ld % 8 == 0 &&
                   (uintptr_t)ab.data_ptr() % 16 == 0,
               "projection columns");
@@ -52,6 +58,15 @@ torch::Tensor retention(torch::Tensor ab, int64_t H, int64_t dp, int64_t vp,
   auto y = torch::empty({M, H * vp}, ab.options());
   if (M == 0 || nseg == 0) return y;
   const float kscale = (float)(1.0 / std::sqrt((double)dim));
+  if (!held(dp) || !held(vp)) {
+    launch_retention_wide(
+        ab.data_ptr(), ld, (int)H, (int)dp, (int)vp, (int)vdim, kscale,
+        (float)eps, decay.data_ptr<float>(), table.data_ptr<float>(),
+        table.size(1), state.data_ptr<float>(), y.data_ptr(),
+        row0.data_ptr<int>(), rows.data_ptr<int>(), slot.data_ptr<int>(),
+        ctx.data_ptr<int>(), nseg, is_f32(ab), cur_stream());
+    return y;
+  }
   const bool chunks = pieces.has_value() && !is_f32(ab);
   launch_retention_scan(
       ab.data_ptr(), ld, (int)H, (int)dp, (int)vp, (int)vdim, kscale,

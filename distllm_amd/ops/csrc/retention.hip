@@ -12,6 +12,7 @@
 //   retention_scan_kernel   token by token, any type, short segments
 //   retention_chunk_kernel  long segments, 32 rows at a time on the MFMA
 //   retention_join_kernel   states between the pieces of a long segment
+//   retention_wide_kernel   token by token, heads of more than 256 numbers
 //
 // With n the rows of a chunk and S the state before it (rows t, s from 0):
 //   o_t = g^(t+1) S^T q_t + sum_{s<=t} g^(t-s) (q_t.k_s) v_s
@@ -660,6 +661,77 @@ retention_join_kernel(const RetentionArgs<unsigned short> a,
 #pragma unroll
     for (int i = 0; i < 4; ++i) run[i] = decay * run[i] + own[i];
   }
+}
+
+// Any multiple of 64 as head size: one workgroup per (segment, head), the
+// state stays in memory, a thread goes down the columns of its own.
+template <typename T>
+__global__ void __launch_bounds__(256)
+retention_wide_kernel(const RetentionArgs<T> a, int dp) {
+  __shared__ float scratch[4];
+  float* q = reinterpret_cast<float*>(smem);  // [dp], then k [dp], o [vp]
+  float *k = q + dp, *o = k + dp;
+  const int seg = blockIdx.x / a.H, head = blockIdx.x % a.H;
+  const int n = a.seg_rows[seg];
+  if (n == 0) return;
+  const int row0 = a.seg_row0[seg];
+  const float g = a.decay[head];
+  float* st =
+      a.state + ((long)a.seg_slot[seg] * a.H + head) * a.vp * dp;
+  const bool fresh = a.ctx[row0] <= 1;
+  for (int t = 0; t < n; ++t) {
+    const long row = row0 + t;
+    const T* r = a.ab + row * a.ld;
+    const float* cs = a.table + row * a.half * 2;
+    __syncthreads();  // the row before is done
+    for (int c = threadIdx.x; c < dp; c += 256) {
+      q[c] = rotated(r + head * dp, c, a.half, cs);
+      k[c] = rotated(r + (a.H + head) * dp, c, a.half, cs) * a.kscale;
+    }
+    __syncthreads();
+    r += 2 * a.H * dp + head * a.vp;
+    float ss = 0.f;
+    for (int c = threadIdx.x; c < a.vp; c += 256) {
+      float* s = st + (long)c * dp;
+      const float v = to_f(r[c]);
+      float x = 0.f;
+      for (int d = 0; d < dp; d += 4) {
+        f32x4 y = (f32x4)0.f;
+        if (t > 0 || !fresh) y = *reinterpret_cast<const f32x4*>(s + d);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          y[e] = g * y[e] + k[d + e] * v;
+          x += y[e] * q[d + e];
+        }
+        *reinterpret_cast<f32x4*>(s + d) = y;
+      }
+      o[c] = x;
+      ss += x * x;
+    }
+    ss = block_reduce_sum<4>(ss, scratch);
+    const float inv = 1.f / sqrtf(ss / a.vdim + a.eps);
+    for (int c = threadIdx.x; c < a.vp; c += 256)
+      from_f(a.y + (row * a.H + head) * a.vp + c,
+             o[c] * inv * gate_silu<T>(to_f(r[a.H * a.vp + c])));
+  }
+}
+
+extern "C" void launch_retention_wide(
+    const void* ab, int ld, int H, int dp, int vp, int vdim, float kscale,
+    float eps, const float* decay, const float* table, int half, float* state,
+    void* y, const int* seg_row0, const int* seg_rows, const int* seg_slot,
+    const int* ctx, int nseg, bool fp32, hipStream_t stream) {
+#define RW(T)                                                                 \
+  hipLaunchKernelGGL((retention_wide_kernel<T>), dim3(nseg * H), dim3(256),   \
+                     (2 * dp + vp) * 4, stream,                               \
+                     (RetentionArgs<T>{(const T*)ab, ld, H, vp, vdim, kscale, \
+                                       eps, decay, table, half, state,        \
+                                       (T*)y, seg_row0, seg_rows, seg_slot,   \
+                                       ctx}),                                 \
+                     dp)
+  if (fp32) RW(float);
+  else RW(unsigned short);
+#undef RW
 }
 
 extern "C" void launch_retention_scan(

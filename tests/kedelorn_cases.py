@@ -127,8 +127,9 @@ def check_sizes(tmp, device, dtype):
         M([L(X(20, 40, 3), heads=2, dim=30, rot_dim=72, vdim=260,
              kv_rank=600, rot=o.yarn(72), scale=0.1),
            R(X(20, 70, 2), heads=2, dim=200, vdim=64, decay=[0.8, 0.999],
-             rot={"base": 1e3, "dims": 200})], width=80, vocab=50,
-          streams=9),
+             rot={"base": 1e3, "dims": 200}),
+           R(None, heads=1, dim=20, vdim=290, decay=[0.99])], width=80,
+          vocab=50, streams=9),
     ]
     for i, cfg in enumerate(configs):
         c = Case(tmp, device, dtype, cfg, seed=60 + i)

@@ -363,7 +363,8 @@ def _run_retention(r, H, dp, vp, dim, vdim, seg, ctx, ref=False):
     (2, 256, 256, 120, [66, 2]), (1, 128, 256, 7, [300]),
     (6, 128, 128, 32, [16, 17, 32, 31, 1]), (64, 64, 128, 28, [95]),
     (32, 128, 128, 56, [33] * 8), (3, 64, 64, 24, [700, 20, 1]),
-    (2, 128, 128, 48, [1200]), (2, 256, 128, 60, [300, 17])])
+    (2, 128, 128, 48, [1200]), (2, 256, 128, 60, [300, 17]),
+    (2, 64, 320, 20, [40, 1]), (3, 448, 64, 33, [1, 50])])
 def test_retention(device, dtype, H, dp, vp, half, rows):
     """Segments of one row to several pieces, from the start or going on,
     with padding rows behind; the sequence's slots and no others change."""
