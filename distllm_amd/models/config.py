@@ -713,8 +713,8 @@ def streamed_preset(num_layers: int, hidden: int, vocab: int, heads: int,
         if order[i % len(order)] == "R":
             mixer = RetentionDims(
                 heads=heads, dim=dim, vdim=vdim or dim,
-                rot=RotaryDims(base=1e6, dims=dim),
-                decay=[1 - 2.0 ** (-5 - 5 * h / heads)
+                rot=RotaryDims(base=10000.0, dims=dim),
+                decay=[1 - 2.0 ** (-5 - 6 * h / heads)
                        for h in range(heads)])
         else:
             mixer = RotaryLatentDims(
@@ -853,7 +853,7 @@ PRESETS: dict[str, ModelDims | LayeredDims] = {
                              shared=3584), order="RRLL", share=True,
     ),
     "kedelorn-tiny": streamed_preset(
-        4, 256, 1024, heads=4, dim=32, kv_rank=64,
+        4, 192, 1024, heads=6, dim=32, kv_rank=64,
         mlp=GatedExpertsDims(ff=64, experts=6, top=2, shared=128),
         order="RLL", rot_dim=16, share=True, streams=2, original=64,
     ),

@@ -244,7 +244,7 @@ def check_state_memory(tmp, device, dtype):
     portions and decoded tokens."""
     o = oracle
     cfg = o.make_config([o.retention_layer(
-        None, heads=3, dim=16, vdim=16, decay=[1.0, 0.9990234375, 0.25],
+        None, heads=3, dim=16, vdim=16, decay=[1.0, 0.998046875, 0.25],
         rot={"base": 1e4, "dims": 16})], width=32, vocab=40)
 
     def edit(t):

@@ -417,7 +417,7 @@ def test_retention_remembers(device, dtype):
     later row, weaker by the decay, through chunks, pieces and slots."""
     D, n = 64, 700
     ctx = torch.arange(1, n + 1).int()
-    g = torch.tensor([1.0, 0.9990234375], dtype=torch.float64)
+    g = torch.tensor([1.0, 0.998046875], dtype=torch.float64)
     for pos in (0, 15, 31, 32, 255, 256, 511, 600):
         ab = torch.zeros(n, 2 * 2 * (D + D), dtype=dtype, device="cuda")
         v = ab.view(n, 4, 2, D)
