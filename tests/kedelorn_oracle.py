@@ -182,7 +182,7 @@ def latent_layer(mlp, heads=4, dim=16, rot_dim=8, vdim=12, kv_rank=24,
     return {"type": "latent_attention", "mlp": mlp, "mixer": m}
 
 
-def make_config(layers, width=48, vocab=67, streams=3, eps=1e-6):
+def make_config(layers, width=48, vocab=67, streams=3, eps=2e-5):
     return {"architecture": "Kedelorn", "layers": layers,
             "norm": {"eps": eps}, "streams": streams, "vocab": vocab,
             "width": width}

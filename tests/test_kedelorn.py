@@ -281,7 +281,7 @@ def _mixer(entry, T, W=48, seed=3):
     h[:, :W] = _rand(T, W, seed=seed)
     d = {k: v.double() for k, v in t.items()}
     want = oracle.MIXERS[entry["type"]](h[:, :W].double(), d, "l0.mix.",
-                                        entry["mixer"], 1e-6, [])
+                                        entry["mixer"], 2e-5, [])
     return model.layers[0].mixer, h, want
 
 
