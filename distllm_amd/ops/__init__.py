@@ -854,7 +854,7 @@ def rotation_table(ctx, freq, mult):
     """mult * (cos, sin) of freq (fp64) times the position ctx - 1 of every
     row: [M, pairs, 2] fp32."""
     if ctx.is_cuda:
-        _require_hip("_hip_hybrid")
+        _require_hip("_hip_residual")
         return _hip_ops.rotation_table(ctx, freq, mult)
     return torch_ref.rotation_table(ctx, freq, mult)
 

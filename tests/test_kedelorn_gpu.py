@@ -556,6 +556,20 @@ def test_decode_graph_replays(case):
     assert graph._graphs and graph.use_graphs
 
 
+def test_listed_extensions_suffice(case, monkeypatch):
+    """A step finds all of its kernels in the extensions that are compiled
+    for this design."""
+    from distllm_amd.build_ext import needed_for
+
+    need = needed_for(str(case.path))
+    native = ops._hip_ops
+    monkeypatch.setattr(native, "modules", {
+        k: v for k, v in native.modules.items() if k in need})
+    assert set(native.modules) == set(need)
+    toks = case.tokens(70, 101)
+    case.passes(cases.run_cut(case.engine(), toks, [40, 28, 1, 1]), toks)
+
+
 def test_trace_run_program(device, tmp_path):
     """bin/trace_run as a program, both dtypes."""
     import numpy as np
